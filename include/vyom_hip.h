@@ -33,7 +33,8 @@ typedef enum {
   VY_ERR_LAUNCH = -3     /* hipGetLastError() after the launch */
 } vy_status;
 
-typedef enum { VY_ACT_NONE = 0, VY_ACT_GELU_ERF = 1, VY_ACT_GELU_TANH = 2 } vy_act;
+typedef enum { VY_ACT_NONE = 0, VY_ACT_GELU_ERF = 1, VY_ACT_GELU_TANH = 2,
+               VY_ACT_SILU = 3 /* gated products only (vy_gated_act_fwd, the decode steps) */ } vy_act;
 /* OR-ed into `act` of vy_linear_fwd / vy_linear_dgrad (training): the tensor saved for backward is act'(x W^T + b)
  * instead of the pre-activation -- the forward epilogue has Phi and the Gaussian of the erf GELU at hand anyway, and
  * the dgrad epilogue (dX = (dY W) * act') becomes one multiply per element instead of an erf + exp evaluation.
@@ -151,6 +152,64 @@ int vy_rmsnorm_fwd(const void* x, int64_t ldx, const void* w, void* y, int64_t l
  * [gate; up] projection. */
 int vy_gated_act_fwd(const void* gate_up, int64_t ldg, void* out, int64_t ldo, int64_t M, int64_t I,
                      int act, int dtype, void* stream);
+
+/* ------------------------------------------------------------------------------------------
+ * Decoders with an fp32 residual stream (norm before and after every sublayer), latent attention and decayed linear
+ * attention.  Conventions shared by this group:
+ *   - rows may be padded: N columns are used of NP (NP a multiple of 8), and the padding is zero in weights and operands;
+ *   - norm weights are fp32;
+ *   - the batch of a launch is B sequences of L tokens; sequence b owns cache / state slot slots[b] (slots NULL: slot b) and
+ *     already holds start[slot] tokens; count[b] <= L of its tokens are real (NULL: all L), the rest is padding behind them.
+ *
+ * vy_residual_norm: x (fp32) += norm(y) * w_post ; h = norm(x) * w_pre.  ids given: x = table[ids] instead (an id outside
+ *   [0, V) gives zeros and sets *err_flag); w_post NULL: plain add; y and ids NULL: x is only read; h NULL: no second norm.
+ *   rms = 0: (v - mean) / sqrt(var + eps), rms = 1: v / sqrt(mean(v^2) + eps).
+ * vy_latent_norm: p = packed rows [query latent (npq) | key/value latent (npc) | ...]: q_out = RMSNorm(latent) * w_q,
+ *   c_out (nullable) = RMSNorm(latent) * w_c, also written to cache[slot][start + l] (strides c_ss / c_st, cap rows per slot).
+ * vy_rmsnorm_gate: y = RMSNorm(x) * w * sigmoid(gate).
+ * ------------------------------------------------------------------------------------------ */
+int vy_residual_norm(float* x, int64_t ldx, const void* y, int64_t ldy, const void* table, int64_t ldt, const int64_t* ids,
+                     int64_t V, int32_t* err_flag, const float* w_post, float eps_post, const float* w_pre, float eps_pre,
+                     void* h, int64_t ldh, int64_t M, int64_t N, int64_t NP, int rms, int dtype, void* stream);
+int vy_latent_norm(const void* p, int64_t ldp, const float* w_q, void* q_out, int64_t ldq, int32_t nq, int32_t npq,
+                   const float* w_c, void* c_out, int64_t ldc, int32_t nc, int32_t npc, void* cache, int64_t c_ss,
+                   int64_t c_st, int32_t cap, const int32_t* slots, const int32_t* start, const int32_t* count, int64_t B,
+                   int64_t L, float eps, int dtype, void* stream);
+int vy_rmsnorm_gate(const void* x, int64_t ldx, const float* w, const void* gate, int64_t ldg, void* y, int64_t ldy, int64_t M,
+                    int64_t N, int64_t NP, float eps, int dtype, void* stream);
+
+/* vy_attn_fwd_ex: causal attention whose values may have a width of their own (dv), with a start position per sequence
+ * (key j is visible to query i of sequence b iff j <= start[slot] + i; start NULL: 0) and an optional output gate:
+ * out *= sigmoid(gate), gate laid out as out (strides g_sb, g_sl). */
+int vy_attn_fwd_ex(const void* q, int64_t q_sb, int64_t q_sh, int64_t q_sl, const void* k, int64_t k_sb, int64_t k_sh,
+                   int64_t k_sl, const void* v, int64_t v_sb, int64_t v_sh, int64_t v_sl, void* out, int64_t o_sb,
+                   int64_t o_sl, const void* gate, int64_t g_sb, int64_t g_sl, const int32_t* start, const int32_t* slots,
+                   int64_t B, int h, int hk, int64_t L, int64_t S, int dh, int dv, float scale, int dtype, void* stream);
+
+/* vy_latent_decode: one query token per sequence against a cache of latents c (one row of R per token, shared by all
+ * heads).  Keys and values are never expanded:  q~_h = Wuk_h^T q_h,  s_j = scale * q~_h . c_j over j <= start[slot],
+ * u_h = sum_j softmax(s)_j c_j,  out_h = (Wuv_h u_h) * sigmoid(gate_h)  (gate nullable).
+ *   q [B][h*dh] (row stride ldq), wukt [h][R][dh] (= Wuk_h transposed), wuv [h][dv][R], out / gate rows [h*dv];
+ *   cache rows cache[slot][j] with strides c_ss / c_st; max_keys >= every start + 1 (sizes the grid, cap rows per slot);
+ *   ws: vy_latent_decode_ws_bytes(...) of scratch.  dh, dv, R multiples of 8, R <= 1024. */
+int64_t vy_latent_decode_ws_bytes(int32_t B, int32_t h, int32_t R);
+int vy_latent_decode(const void* q, int64_t ldq, const void* wukt, const void* wuv, const void* cache, int64_t c_ss,
+                     int64_t c_st, const int32_t* slots, const int32_t* start, int64_t max_keys, void* out, int64_t ldo,
+                     const void* gate, int64_t ldg, int32_t B, int32_t h, int32_t dh, int32_t dv, int32_t R, float scale,
+                     void* ws, int64_t ws_bytes, int dtype, void* stream);
+
+/* vy_decay_attn: linear attention with a per-head decay on packed rows p (row stride ldp; q / k / v of head a at columns
+ * oq + a*dk, ok + a*dk, ov + a*dv):  S_t = decay_a S_(t-1) + k_t v_t^T,  o_t = S_t^T q_t  with q, k, v = silu of the
+ * projections (silu = 0: taken as they are).  state: fp32 [slot][h][dk][dv], taken as zero where start[slot] == 0 and left as
+ * S after the sequence's last real token.  decay_pow: fp32 [h][VY_DECAY_CHUNK + 1], decay_a^0 .. decay_a^CHUNK.
+ * out rows [h*dv].  ws: vy_decay_attn_ws_bytes(...) of scratch (chunked prefill: bf16, L > 1, dk <= 128; otherwise the
+ * token-by-token recurrence runs and ws may be NULL).  dk, dv multiples of 8, dk <= 512. */
+#define VY_DECAY_CHUNK 64
+int64_t vy_decay_attn_ws_bytes(int64_t B, int64_t L, int32_t h, int32_t dk, int32_t dv, int dtype);
+int vy_decay_attn(const void* p, int64_t ldp, int64_t oq, int64_t ok, int64_t ov, float* state, const float* decay_pow,
+                  const int32_t* slots, const int32_t* start, const int32_t* count, void* out, int64_t ldo, int64_t B,
+                  int64_t L, int32_t h, int32_t dk, int32_t dv, int silu, void* ws, int64_t ws_bytes, int dtype,
+                  void* stream);
 
 /* vy_rope_fwd: in-place rotary embedding on a (B,heads,L,dh) tensor (strides as above);
  * used when the fused epilogue does not apply.  `inverse` != 0 applies the transpose rotation
@@ -429,6 +488,41 @@ int64_t vy_gemma_ws_bytes(int32_t B, int32_t d, int32_t h, int32_t dh, int32_t f
  * logits: (B, ldv). */
 int vy_gemma_decoder_step(const vy_gemma_plan* plan, const void* x, int64_t pos, void* logits, int64_t ldv,
                           void* stream);
+
+/* ------------------------------------------------------------------------------------------
+ * vy_hybrid_decoder_step: one new token for each of B sequences of a decoder that mixes layer kinds over an fp32 residual
+ * stream.  Per layer: h = norm(x) * norm1; mixer; x += norm(y) * norm1b; h = norm(x) * norm2; gated MLP; x += norm(y) * norm2b
+ * (ff = 0: no MLP).  Mixers, all from ONE packed input projection w_in of h:
+ *   VY_MIX_LATENT  rows [query latent | key/value latent | output gate]: vy_latent_norm, q = w_uq latent, vy_latent_decode
+ *   VY_MIX_DECAY   rows [q | k | v | output gate]: vy_decay_attn, vy_rmsnorm_gate
+ * then y = w_o (.).  Sequence b (ids[b]) lives in slot slots[b] (NULL: b) and holds lengths[slot] tokens, which the step
+ * advances by one on the device; max_keys >= every lengths[slot] + 1.  Widths with _p, dim, vdim, ff and dp are padded to
+ * multiples of 8; d, q_rank, kv_rank and mix_n are the true counts the norms divide by.  logits: (B, ldv).
+ * -------------------------------------------------------------------------------------------- */
+enum { VY_MIX_LATENT = 0, VY_MIX_DECAY = 1 };
+typedef struct vy_hybrid_layer {
+  int32_t mixer, heads, dim, vdim, n_in, ff;
+  int32_t q_rank, q_rank_p, kv_rank, kv_rank_p;   /* VY_MIX_LATENT */
+  int32_t cap, mix_n;                             /* cache rows per slot; VY_MIX_DECAY: width of mix_norm */
+  float scale;
+  const float *norm1, *norm1b, *norm2, *norm2b;
+  const void *w_in, *w_o, *w_gu, *w_down;         /* w_gu: packed [gate; up] */
+  const float *q_norm, *c_norm;
+  const void *w_uq, *w_ukt, *w_uv;
+  void* cache; int64_t c_ss, c_st;
+  float* state; const float *decay_pow, *mix_norm;
+} vy_hybrid_layer;
+typedef struct vy_hybrid_plan {
+  int32_t num_layers, B, d, dp, vocab, dtype, rms, act;
+  float eps;
+  const vy_hybrid_layer* layers;                  /* host array [num_layers] */
+  const void *embed, *head; const float* final_norm;
+  int32_t* err;                                   /* nullable: set when an id is outside the vocabulary */
+  void* ws; int64_t ws_bytes;                     /* >= vy_hybrid_ws_bytes(plan) */
+} vy_hybrid_plan;
+int64_t vy_hybrid_ws_bytes(const vy_hybrid_plan* plan);
+int vy_hybrid_decoder_step(const vy_hybrid_plan* plan, const int64_t* ids, const int32_t* slots, int32_t* lengths,
+                           int64_t max_keys, void* logits, int64_t ldv, void* stream);
 
 #ifdef __cplusplus
 }

@@ -14,7 +14,7 @@ _HERE = os.path.dirname(os.path.abspath(__file__))
 LIB_PATH = os.environ.get("VY_LIB_PATH") or os.path.join(_HERE, "lib", "libvyom_hip.so")
 
 VY_F32, VY_BF16 = 0, 1
-ACT_NONE, ACT_GELU_ERF, ACT_GELU_TANH = 0, 1, 2
+ACT_NONE, ACT_GELU_ERF, ACT_GELU_TANH, ACT_SILU = 0, 1, 2, 3
 ACT_SAVE_DERIV = 0x100   # saved tensor = act'(pre) instead of pre (include/vyom_hip.h)
 MASK_NONE, MASK_CAUSAL, MASK_KEYPAD, MASK_ADDITIVE = 0, 1, 2, 4
 
@@ -60,6 +60,16 @@ PROTOTYPES = {
     "vy_sampling_probs": [_p, _i64, _i64, _i64, _i, _f, _i, _f, _p, _i64, _p],
     "vy_decoder_step": [_p, _p, _i64, _p, _p, _p, _i64, _p],
     "vy_gemma_decoder_step": [_p, _p, _i64, _p, _i64, _p],
+    "vy_residual_norm": [_p, _i64, _p, _i64, _p, _i64, _p, _i64, _p, _p, _f, _p, _f, _p, _i64, _i64, _i64, _i64, _i, _i, _p],
+    "vy_latent_norm": [_p, _i64, _p, _p, _i64, _i, _i, _p, _p, _i64, _i, _i, _p, _i64, _i64, _i, _p, _p, _p, _i64, _i64, _f,
+                       _i, _p],
+    "vy_rmsnorm_gate": [_p, _i64, _p, _p, _i64, _p, _i64, _i64, _i64, _i64, _f, _i, _p],
+    "vy_attn_fwd_ex": [_p, _i64, _i64, _i64, _p, _i64, _i64, _i64, _p, _i64, _i64, _i64, _p, _i64, _i64, _p, _i64, _i64,
+                       _p, _p, _i64, _i, _i, _i64, _i64, _i, _i, _f, _i, _p],
+    "vy_latent_decode": [_p, _i64, _p, _p, _p, _i64, _i64, _p, _p, _i64, _p, _i64, _p, _i64, _i, _i, _i, _i, _i, _f, _p, _i64,
+                         _i, _p],
+    "vy_decay_attn": [_p, _i64, _i64, _i64, _i64, _p, _p, _p, _p, _p, _p, _i64, _i64, _i64, _i, _i, _i, _i, _p, _i64, _i, _p],
+    "vy_hybrid_decoder_step": [_p, _p, _p, _p, _i64, _p, _i64, _p],
     "vy_cast": [_p, _p, _i64, _i, _i, _p],
     "vy_ddp_unique_id": [_p],
     "vy_ddp_init": [_p, _i, _i],
@@ -69,7 +79,9 @@ PROTOTYPES = {
     "vy_workspace_set": [_p, _p, _i64],
 }
 OTHER_SYMBOLS = ["vy_last_error", "vy_abi_version", "vy_layernorm_bwd_ws_rows", "vy_decode_ws_bytes",
-                 "vy_gemma_ws_bytes", "vy_ddp_world", "vy_ddp_rank"]
+                 "vy_gemma_ws_bytes", "vy_ddp_world", "vy_ddp_rank", "vy_latent_decode_ws_bytes", "vy_decay_attn_ws_bytes",
+                 "vy_hybrid_ws_bytes"]
+DECAY_CHUNK = 64   # VY_DECAY_CHUNK
 ALL_SYMBOLS = list(PROTOTYPES) + OTHER_SYMBOLS
 
 
@@ -108,6 +120,10 @@ def load() -> C.CDLL:
     lib.vy_layernorm_bwd_ws_rows.argtypes = [_i64]
     lib.vy_decode_ws_bytes.restype = C.c_int64
     lib.vy_decode_ws_bytes.argtypes = [C.c_int32] * 7
+    for name, argtypes in (("vy_latent_decode_ws_bytes", [_i, _i, _i]),
+                           ("vy_decay_attn_ws_bytes", [_i64, _i64, _i, _i, _i, _i]), ("vy_hybrid_ws_bytes", [_p])):
+        getattr(lib, name).restype = C.c_int64
+        getattr(lib, name).argtypes = argtypes
     _lib = lib
     return lib
 

@@ -40,13 +40,22 @@ struct AttnParams {
   int B, h, hk, L, S;
   float scale;
   const int* pos_dev;  // decode under a hipGraph: S = *pos_dev + 1 (else NULL)
+  // per-sequence start positions (vy_attn_fwd_ex): keys before this launch's tokens in sequence b are
+  // start_dev[slots ? slots[b] : b]; NULL = start_pos for every sequence
+  const int* start_dev; const int* slots;
+  int dv;              // value width (0 = as wide as the keys)
+  const void* gate; int64_t g_sb, g_sl;   // output gate (nullable): out *= sigmoid(gate), laid out as out
   int diag;            // timing experiments only (VY_ATTN_DIAG): 1 = no output store, 2 = no tile loop
 };
 
+__device__ __forceinline__ int attn_start(const AttnParams& p, int b) {
+  return p.start_dev ? p.start_dev[p.slots ? p.slots[b] : b] : p.start_pos;
+}
+
 // ------------------------------------------------------------------------------------------
-// MFMA flash forward (bf16)
+// MFMA flash forward (bf16).  EXT: per-sequence start positions and the sigmoid output gate.
 // ------------------------------------------------------------------------------------------
-template <int DH>
+template <int DH, bool EXT = false>
 __global__ __launch_bounds__(256, DH == 64 ? 3 : 1) void attn_fwd_mfma_kernel(AttnParams p) {
   constexpr int RB = DH * 2;            // bytes per K/V row
   constexpr int TILE = 64 * RB;         // bytes per 64-key tile
@@ -75,6 +84,7 @@ __global__ __launch_bounds__(256, DH == 64 ? 3 : 1) void attn_fwd_mfma_kernel(At
   const int qrow = qi < p.L ? qi : p.L - 1;
 
   const bf16* Q = (const bf16*)p.q + (int64_t)b * p.q_sb + (int64_t)head * p.q_sh + (int64_t)qrow * p.q_sl;
+  const int start = EXT ? attn_start(p, b) : p.start_pos;
   const bf16* Kb = (const bf16*)p.k + (int64_t)b * p.k_sb + (int64_t)kvh * p.k_sh;
   const bf16* Vb = (const bf16*)p.v + (int64_t)b * p.v_sb + (int64_t)kvh * p.v_sh;
 
@@ -161,7 +171,7 @@ __global__ __launch_bounds__(256, DH == 64 ? 3 : 1) void attn_fwd_mfma_kernel(At
   const int nt_all = (p.S + 63) / 64;
   int nt = nt_all;
   if (causal) {
-    const int kv_end = min(p.S, p.start_pos + q0 + 128);
+    const int kv_end = min(p.S, start + q0 + 128);
     nt = (kv_end + 63) / 64;
     if (nt < 1) nt = 1;
   }
@@ -183,7 +193,7 @@ __global__ __launch_bounds__(256, DH == 64 ? 3 : 1) void attn_fwd_mfma_kernel(At
   auto compute = [&](int tile, int buf) {
     const int k0 = tile * 64;
     // wave-uniform skip of tiles wholly above this wave's diagonal
-    if (causal && k0 > p.start_pos + wave_last) return;
+    if (causal && k0 > start + wave_last) return;
     const char* kb_ = smem + buf * TILE;
     const char* vb_ = smem + (NS + buf) * TILE;
     f32x16 st[2];
@@ -227,7 +237,7 @@ __global__ __launch_bounds__(256, DH == 64 ? 3 : 1) void attn_fwd_mfma_kernel(At
     });
     unsigned long long vis = ~0ull;
     if (haskp) vis = kpbits[tile];
-    const bool need_mask = hasadd || (k0 + 64 > p.S) || (causal && k0 + 63 > p.start_pos + wave_first) || vis != ~0ull;
+    const bool need_mask = hasadd || (k0 + 64 > p.S) || (causal && k0 + 63 > start + wave_first) || vis != ~0ull;
     // softmax runs on the RAW scores: max first, then p = exp2(fma(s, c, -m)) -- one FMA and one
     // v_exp_f32 per element (the VALU, not the MFMA pipe, bounds dh=64)
     float tmax = -INFINITY;
@@ -236,7 +246,7 @@ __global__ __launch_bounds__(256, DH == 64 ? 3 : 1) void attn_fwd_mfma_kernel(At
       // the lane's 32 keys as one bit word: padding bits shifted by 4fh, AND kofs <= klim (causal
       // diagonal and end of sequence)
       int klim = p.S - 1 - k0 - 4 * fh;
-      if (causal) klim = min(klim, qi + p.start_pos - k0 - 4 * fh);
+      if (causal) klim = min(klim, qi + start - k0 - 4 * fh);
       unsigned long long lm = klim >= 63 ? ~0ull : (klim < 0 ? 0ull : ((2ull << klim) - 1ull));
       lm &= vis >> (4 * fh);
       const unsigned lmw[2] = {(unsigned)lm, (unsigned)(lm >> 32)};
@@ -400,7 +410,14 @@ __global__ __launch_bounds__(256, DH == 64 ? 3 : 1) void attn_fwd_mfma_kernel(At
   for (int it = 0; it < 32 * LPR / 64; ++it) {
     const int r = (it * 64 + lane) / LPR, ch = (it * 64 + lane) % LPR;
     const int qrow_ = q0 + wave * 32 + r;
-    const bf16x8 vv = *reinterpret_cast<const bf16x8*>(ot + r * OROW + ch * 16);
+    bf16x8 vv = *reinterpret_cast<const bf16x8*>(ot + r * OROW + ch * 16);
+    if constexpr (EXT) {
+      if (p.gate && qrow_ < p.L) {
+        const bf16x8 g8 = *reinterpret_cast<const bf16x8*>((const bf16*)p.gate + (int64_t)b * p.g_sb + (int64_t)qrow_ * p.g_sl + head * DH + ch * 8);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) vv[e] = (bf16)((float)vv[e] * vy_sigmoid((float)g8[e]));
+      }
+    }
     if (qrow_ < p.L)
       *reinterpret_cast<bf16x8*>((bf16*)p.out + (int64_t)b * p.o_sb + (int64_t)qrow_ * p.o_sl + head * DH + ch * 8) = vv;
   }
@@ -424,16 +441,19 @@ __global__ __launch_bounds__(256, DH == 64 ? 3 : 1) void attn_fwd_mfma_kernel(At
 // Masks: causal (+ start_pos) and key padding as in attn_fwd_mfma_kernel, rows without a visible key get the
 // reference's uniform average; a dense additive mask goes to the row-wise kernel.
 // ------------------------------------------------------------------------------------------
-template <int DHP>
+// DHP / DVP: padded widths of the keys and of the values (attention whose values have a width of their own).
+template <int DHP, int DVP = DHP, bool EXT = false>
 __global__ __launch_bounds__(256) void attn_fwd_gen_kernel(AttnParams p, int dh) {
-  constexpr int PITCH = (DHP + 8) * 2;       // bytes per LDS row (16 B of padding: conflict-free fragment reads)
+  constexpr int KPITCH = (DHP + 8) * 2;      // bytes per LDS row (16 B of padding: conflict-free fragment reads)
+  constexpr int VPITCH = (DVP + 8) * 2;
   constexpr int KS = DHP / 32;               // k-steps of QK^T
-  constexpr int NDB = DHP / 16;              // 16-wide d blocks of O^T
-  constexpr int CPRW = DHP / 8;              // 16-byte chunks per row
-  constexpr int CPT = 64 * CPRW / 256;       // chunks per thread and tile
-  __shared__ __attribute__((aligned(16))) char smem[2 * 64 * PITCH];
+  constexpr int NDB = DVP / 16;              // 16-wide d blocks of O^T
+  constexpr int KCPR = DHP / 8, VCPR = DVP / 8;          // 16-byte chunks per row
+  constexpr int KCPT = 64 * KCPR / 256, VCPT = 64 * VCPR / 256;   // chunks per thread and tile
+  __shared__ __attribute__((aligned(16))) char smem[64 * (KPITCH + VPITCH)];
   char* kt = smem;
-  char* vt = smem + 64 * PITCH;
+  char* vt = smem + 64 * KPITCH;
+  const int dv = EXT ? p.dv : dh;
   const int tid = threadIdx.x, lane = tid & 63;
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int r16 = lane & 15, kq = lane >> 4;
@@ -447,6 +467,7 @@ __global__ __launch_bounds__(256) void attn_fwd_gen_kernel(AttnParams p, int dh)
   const bf16* Q = (const bf16*)p.q + (int64_t)b * p.q_sb + (int64_t)head * p.q_sh + (int64_t)qrow * p.q_sl;
   const bf16* Kb = (const bf16*)p.k + (int64_t)b * p.k_sb + (int64_t)kvh * p.k_sh;
   const bf16* Vb = (const bf16*)p.v + (int64_t)b * p.v_sb + (int64_t)kvh * p.v_sh;
+  const int start = EXT ? attn_start(p, b) : p.start_pos;
   const bool causal = p.mask_kind & VY_MASK_CAUSAL;
   const bool haskp = p.mask_kind & VY_MASK_KEYPAD;
   const uint8_t* kp = haskp ? p.keypad + (int64_t)b * p.kp_sb : nullptr;
@@ -465,33 +486,55 @@ __global__ __launch_bounds__(256) void attn_fwd_gen_kernel(AttnParams p, int dh)
   const float c = p.scale * LOG2E;
   int nt = (p.S + 63) / 64;
   if (causal) {
-    const int kv_end = min(p.S, p.start_pos + q0 + 64);
+    const int kv_end = min(p.S, start + q0 + 64);
     nt = max(1, (kv_end + 63) / 64);
   }
   // transposing-read addresses of the V tile: lane j of a 16-lane group supplies row (j >> 2), columns 4 (j & 3) ..
-  const unsigned vtr = vy_lds_addr(vt) + (4 * kq + (r16 >> 2)) * PITCH + (4 * (r16 & 3)) * 2;
+  const unsigned vtr = vy_lds_addr(vt) + (4 * kq + (r16 >> 2)) * VPITCH + (4 * (r16 & 3)) * 2;
 
   for (int t = 0; t < nt; ++t) {
     const int k0 = t * 64;
     // stage the tile: 16-byte chunks, zero beyond the head width and beyond the last key
-    bf16x8 kreg[CPT], vreg[CPT];
+    bf16x8 kreg[KCPT], vreg[VCPT];
+    if constexpr (!EXT && DHP == DVP) {
 #pragma unroll
-    for (int i = 0; i < CPT; ++i) {
-      const int cidx = tid + 256 * i;
-      const int row = cidx / CPRW, ch = cidx - row * CPRW;
-      const int kj = k0 + row;
-      const bool ok = ch * 8 < dh && kj < p.S;
-      const int64_t kjc = kj < p.S ? kj : p.S - 1;
-      kreg[i] = ok ? *reinterpret_cast<const bf16x8*>(Kb + kjc * p.k_sl + (ch * 8 < dh ? ch * 8 : 0)) : zero8;
-      vreg[i] = ok ? *reinterpret_cast<const bf16x8*>(Vb + kjc * p.v_sl + (ch * 8 < dh ? ch * 8 : 0)) : zero8;
+      for (int i = 0; i < KCPT; ++i) {
+        const int cidx = tid + 256 * i;
+        const int row = cidx / KCPR, ch = cidx - row * KCPR;
+        const int kj = k0 + row;
+        const bool ok = ch * 8 < dh && kj < p.S;
+        const int64_t kjc = kj < p.S ? kj : p.S - 1;
+        kreg[i] = ok ? *reinterpret_cast<const bf16x8*>(Kb + kjc * p.k_sl + (ch * 8 < dh ? ch * 8 : 0)) : zero8;
+        vreg[i] = ok ? *reinterpret_cast<const bf16x8*>(Vb + kjc * p.v_sl + (ch * 8 < dh ? ch * 8 : 0)) : zero8;
+      }
+    } else {
+      auto fetch = [&](const bf16* src, int64_t sl, int width, int row, int ch) {
+        const int kj = k0 + row;
+        const bool ok = ch * 8 < width && kj < p.S;
+        const int64_t kjc = kj < p.S ? kj : p.S - 1;
+        return ok ? *reinterpret_cast<const bf16x8*>(src + kjc * sl + (ch * 8 < width ? ch * 8 : 0)) : zero8;
+      };
+#pragma unroll
+      for (int i = 0; i < KCPT; ++i) {
+        const int cidx = tid + 256 * i;
+        kreg[i] = fetch(Kb, p.k_sl, dh, cidx / KCPR, cidx % KCPR);
+      }
+#pragma unroll
+      for (int i = 0; i < VCPT; ++i) {
+        const int cidx = tid + 256 * i;
+        vreg[i] = fetch(Vb, p.v_sl, dv, cidx / VCPR, cidx % VCPR);
+      }
     }
     __syncthreads();   // the previous tile's fragments have been read
 #pragma unroll
-    for (int i = 0; i < CPT; ++i) {
+    for (int i = 0; i < KCPT; ++i) {
       const int cidx = tid + 256 * i;
-      const int row = cidx / CPRW, ch = cidx - row * CPRW;
-      *reinterpret_cast<bf16x8*>(kt + row * PITCH + ch * 16) = kreg[i];
-      *reinterpret_cast<bf16x8*>(vt + row * PITCH + ch * 16) = vreg[i];
+      *reinterpret_cast<bf16x8*>(kt + (cidx / KCPR) * KPITCH + (cidx % KCPR) * 16) = kreg[i];
+    }
+#pragma unroll
+    for (int i = 0; i < VCPT; ++i) {
+      const int cidx = tid + 256 * i;
+      *reinterpret_cast<bf16x8*>(vt + (cidx / VCPR) * VPITCH + (cidx % VCPR) * 16) = vreg[i];
     }
     __syncthreads();
     // S^T = K Q^T: four 16-key blocks
@@ -501,7 +544,7 @@ __global__ __launch_bounds__(256) void attn_fwd_gen_kernel(AttnParams p, int dh)
       sc[blk] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
       for (int ks = 0; ks < KS; ++ks) {
-        const bf16x8 kf = *reinterpret_cast<const bf16x8*>(kt + (16 * blk + r16) * PITCH + (32 * ks + 8 * kq) * 2);
+        const bf16x8 kf = *reinterpret_cast<const bf16x8*>(kt + (16 * blk + r16) * KPITCH + (32 * ks + 8 * kq) * 2);
         sc[blk] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[ks], sc[blk], 0, 0, 0);
       }
     }
@@ -513,7 +556,7 @@ __global__ __launch_bounds__(256) void attn_fwd_gen_kernel(AttnParams p, int dh)
       for (int r = 0; r < 4; ++r) {
         const int kj = k0 + 16 * blk + 4 * kq + r;
         bool vis = kj < p.S;
-        if (causal) vis = vis && kj <= qi + p.start_pos;
+        if (causal) vis = vis && kj <= qi + start;
         if (haskp) vis = vis && kp[kj < p.S ? kj : 0] != 0;
         const float tv = vis ? sc[blk][r] : -INFINITY;
         sc[blk][r] = tv;
@@ -555,8 +598,8 @@ __global__ __launch_bounds__(256) void attn_fwd_gen_kernel(AttnParams p, int dh)
       vy_static_for<NDB>([&](auto n_c) {
         constexpr int n = decltype(n_c)::value;
         union { struct { s16x4 a, b; } h; bf16x8 v; } u;
-        u.h.a = vy_lds_tr16_off<n * 32>(vtr + (32 * tt) * PITCH);
-        u.h.b = vy_lds_tr16_off<n * 32>(vtr + (32 * tt + 16) * PITCH);
+        u.h.a = vy_lds_tr16_off<n * 32>(vtr + (32 * tt) * VPITCH);
+        u.h.b = vy_lds_tr16_off<n * 32>(vtr + (32 * tt + 16) * VPITCH);
         asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
         vy_tie(u.v);
         o[n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(u.v, pf, o[n], 0, 0, 0);
@@ -582,7 +625,7 @@ __global__ __launch_bounds__(256) void attn_fwd_gen_kernel(AttnParams p, int dh)
 #pragma unroll
       for (int n = 0; n < NDB; ++n) {
         const int d0 = 16 * n + 4 * kq;
-        if (d0 < dh) {
+        if (d0 < dv) {
           const bf16x4 v4 = *reinterpret_cast<const bf16x4*>(Vb + (int64_t)kj * p.v_sl + d0);
 #pragma unroll
           for (int r = 0; r < 4; ++r) o[n][r] += (float)v4[r];
@@ -594,14 +637,21 @@ __global__ __launch_bounds__(256) void attn_fwd_gen_kernel(AttnParams p, int dh)
   }
   const float inv = 1.0f / l_tot;
   if (qi < p.L) {
-    bf16* orow = (bf16*)p.out + (int64_t)b * p.o_sb + (int64_t)qi * p.o_sl + head * dh;
+    bf16* orow = (bf16*)p.out + (int64_t)b * p.o_sb + (int64_t)qi * p.o_sl + head * dv;
+    const bf16* grow = EXT && p.gate ? (const bf16*)p.gate + (int64_t)b * p.g_sb + (int64_t)qi * p.g_sl + head * dv : nullptr;
 #pragma unroll
     for (int n = 0; n < NDB; ++n) {
       const int d0 = 16 * n + 4 * kq;
-      if (d0 < dh) {
+      if (d0 < dv) {
         bf16x4 w;
+        float gt[4] = {1.f, 1.f, 1.f, 1.f};
+        if (grow) {
+          const bf16x4 g4 = *reinterpret_cast<const bf16x4*>(grow + d0);
 #pragma unroll
-        for (int r = 0; r < 4; ++r) w[r] = (bf16)(o[n][r] * inv);
+          for (int r = 0; r < 4; ++r) gt[r] = vy_sigmoid((float)g4[r]);
+        }
+#pragma unroll
+        for (int r = 0; r < 4; ++r) w[r] = (bf16)(o[n][r] * inv * gt[r]);
         *reinterpret_cast<bf16x4*>(orow + d0) = w;
       }
     }
@@ -634,7 +684,7 @@ template <> struct RowVec<float> {
 // NWV waves per workgroup: 4, or 16 for decode launches with few (batch x head) rows -- an MQA / small-batch
 // decode has only B*h workgroups, each walking its keys in dependent trips; four times the waves = a quarter
 // of the trips, combined through LDS as before (no workspace, no second launch)
-template <typename T, int CPR, int NWV = 4>  // CPR = dh / VEC lanes per key row, power of two <= 64
+template <typename T, int CPR, int NWV = 4, bool EXT = false>  // CPR = dh / VEC lanes per key row, power of two <= 64
 __global__ __launch_bounds__(64 * NWV) void attn_rowwise_kernel(AttnParams p, int dh) {
   constexpr int VEC = RowVec<T>::VEC;
   constexpr int KPP = 64 / CPR;  // keys per wave pass
@@ -651,6 +701,10 @@ __global__ __launch_bounds__(64 * NWV) void attn_rowwise_kernel(AttnParams p, in
   // next power of two lanes per key; the surplus lanes carry zeros and never store
   const bool ch_ok = ch * VEC < dh;
   const int chl = ch_ok ? ch : 0;  // a valid address for the idle lanes
+  const int dv = EXT ? p.dv : dh;          // EXT: value width, start position per sequence, output gate
+  const bool chv_ok = EXT ? ch * VEC < dv : ch_ok;
+  const int chv = EXT ? (chv_ok ? ch : 0) : chl;
+  const int start = EXT ? attn_start(p, b) : p.start_pos;
   float qv[VEC];
   RowVec<T>::load(Q + chl * VEC, qv);
   if (!ch_ok) {
@@ -665,7 +719,7 @@ __global__ __launch_bounds__(64 * NWV) void attn_rowwise_kernel(AttnParams p, in
   // pure causal: invisible keys contribute exactly 0 -> stop at the diagonal.  With key padding
   // every key is walked so a fully masked row reproduces the reference's uniform average.
   int S_eff = p.pos_dev ? *p.pos_dev + 1 : p.S;
-  if (causal && !haskp && !hasadd) S_eff = min(S_eff, qi + p.start_pos + 1);
+  if (causal && !haskp && !hasadd) S_eff = min(S_eff, qi + start + 1);
 
   float m = -FLT_MAX, l = 0.f, acc[VEC];
 #pragma unroll
@@ -693,7 +747,7 @@ __global__ __launch_bounds__(64 * NWV) void attn_rowwise_kernel(AttnParams p, in
     for (int u = 0; u < U; ++u) {
       bool ok;
       const int jc = key_of(j0, u, ok);
-      vr[u] = *reinterpret_cast<const raw16*>(Vb + (int64_t)jc * p.v_sl + chl * VEC);
+      vr[u] = *reinterpret_cast<const raw16*>(Vb + (int64_t)jc * p.v_sl + chv * VEC);
     }
   };
   auto widen = [&](const raw16& r, float (&o)[VEC]) {
@@ -729,7 +783,7 @@ __global__ __launch_bounds__(64 * NWV) void attn_rowwise_kernel(AttnParams p, in
       for (int o_ = CPR >> 1; o_ > 0; o_ >>= 1) d += __shfl_xor(d, o_, 64);
       float x = d * p.scale;
       if (hasadd) x = x + am[jc[u]];
-      if (causal && jc[u] > qi + p.start_pos) x = -FLT_MAX;
+      if (causal && jc[u] > qi + start) x = -FLT_MAX;
       if (haskp && !kp[jc[u]]) x = -FLT_MAX;
       x = fmaxf(x, -FLT_MAX);
       t[u] = x;
@@ -771,7 +825,7 @@ __global__ __launch_bounds__(64 * NWV) void attn_rowwise_kernel(AttnParams p, in
     for (int e = 0; e < VEC; ++e) red_o[(wave * 64 + ch) * VEC + e] = acc[e];
   }
   __syncthreads();
-  if (wave == 0 && grp == 0 && ch_ok) {
+  if (wave == 0 && grp == 0 && chv_ok) {
     float M_ = red_m[0];
     for (int w = 1; w < NWV; ++w) M_ = fmaxf(M_, red_m[w * KPP]);
     float Ls = 0.f, out[VEC];
@@ -783,31 +837,35 @@ __global__ __launch_bounds__(64 * NWV) void attn_rowwise_kernel(AttnParams p, in
 #pragma unroll
       for (int e = 0; e < VEC; ++e) out[e] += red_o[(w * 64 + ch) * VEC + e] * a;
     }
-    T* O = (T*)p.out + (int64_t)b * p.o_sb + (int64_t)qi * p.o_sl + head * dh + ch * VEC;
+    T* O = (T*)p.out + (int64_t)b * p.o_sb + (int64_t)qi * p.o_sl + head * dv + ch * VEC;
     const float inv = 1.0f / Ls;
 #pragma unroll
-    for (int e = 0; e < VEC; ++e) VyT<T>::st(O + e, out[e] * inv);
+    for (int e = 0; e < VEC; ++e) {
+      float x = out[e] * inv;
+      if (EXT && p.gate) x *= vy_sigmoid(VyT<T>::ld((const T*)p.gate + (int64_t)b * p.g_sb + (int64_t)qi * p.g_sl + head * dv + ch * VEC + e));
+      VyT<T>::st(O + e, x);
+    }
     if (p.lse && ch == 0) p.lse[((int64_t)b * p.h + head) * p.L + qi] = M_ + __logf(Ls);
   }
 }
 
-template <typename T>
+template <typename T, bool EXT = false>
 int launch_rowwise(const AttnParams& p, int dh, hipStream_t st, const char* who) {
   constexpr int VEC = RowVec<T>::VEC;
-  if (dh % VEC) VY_FAIL(VY_ERR_ARG, "%s: head_dim %d not a multiple of %d", who, dh, VEC);
+  if (dh % VEC || p.dv % VEC) VY_FAIL(VY_ERR_ARG, "%s: head_dim %d not a multiple of %d", who, p.dv % VEC ? p.dv : dh, VEC);
   int cpr = 1;
-  while (cpr * VEC < dh) cpr <<= 1;  // lanes per key row, rounded up to a power of two
+  while (cpr * VEC < (p.dv > dh ? p.dv : dh)) cpr <<= 1;  // lanes per key row, rounded up to a power of two
   const dim3 grid(p.L, p.h, p.B), block(256);
   static const int wide_wg = [] { const char* e = getenv("VY_DECODE_WIDE_WG"); return e ? atoi(e) : 1; }();
   static const int wide_rows = [] { const char* e = getenv("VY_DECODE_WIDE_ROWS"); return e ? atoi(e) : 128; }();
-  if (p.L == 1 && wide_wg && (int64_t)p.B * p.h <= wide_rows && p.S > 64 && std::is_same<T, bf16>::value && (cpr == 8 || cpr == 32)) {
+  if (!EXT && p.L == 1 && wide_wg && (int64_t)p.B * p.h <= wide_rows && p.S > 64 && std::is_same<T, bf16>::value && (cpr == 8 || cpr == 32)) {
     const dim3 block16(1024);
     if (cpr == 8) hipLaunchKernelGGL((attn_rowwise_kernel<T, 8, 16>), grid, block16, 0, st, p, dh);
     else hipLaunchKernelGGL((attn_rowwise_kernel<T, 32, 16>), grid, block16, 0, st, p, dh);
     VY_CHECK_LAUNCH(who);
     return VY_OK;
   }
-#define RW_GO(C) hipLaunchKernelGGL((attn_rowwise_kernel<T, C>), grid, block, 0, st, p, dh)
+#define RW_GO(C) hipLaunchKernelGGL((attn_rowwise_kernel<T, C, 4, EXT>), grid, block, 0, st, p, dh)
   switch (cpr) {
     case 1: RW_GO(1); break;
     case 2: RW_GO(2); break;
@@ -848,7 +906,7 @@ extern "C" int vy_attn_fwd(const void* q, int64_t q_sb, int64_t q_sh, int64_t q_
                            const float* addmask, int64_t am_sb, int64_t am_sl, int64_t B, int h, int hk,
                            int64_t L, int64_t S, int dh, float scale, int dtype, void* stream) {
   const char* who = "vy_attn_fwd";
-  AttnParams p;
+  AttnParams p{};
   p.q = q; p.q_sb = q_sb; p.q_sh = q_sh; p.q_sl = q_sl;
   p.k = k; p.k_sb = k_sb; p.k_sh = k_sh; p.k_sl = k_sl;
   p.v = v; p.v_sb = v_sb; p.v_sh = v_sh; p.v_sl = v_sl;
@@ -880,6 +938,54 @@ extern "C" int vy_attn_fwd(const void* q, int64_t q_sb, int64_t q_sh, int64_t q_
   }
   if (dtype == VY_BF16) return launch_rowwise<bf16>(p, dh, st, who);
   return launch_rowwise<float>(p, dh, st, who);
+}
+
+namespace {
+template <int DHP>
+void gen_go(const AttnParams& p, int dh, int dv, dim3 grid, hipStream_t st) {
+  const dim3 block(256);
+  if (dv <= 64) hipLaunchKernelGGL((attn_fwd_gen_kernel<DHP, 64, true>), grid, block, 0, st, p, dh);
+  else if (dv <= 96) hipLaunchKernelGGL((attn_fwd_gen_kernel<DHP, 96, true>), grid, block, 0, st, p, dh);
+  else if (dv <= 128) hipLaunchKernelGGL((attn_fwd_gen_kernel<DHP, 128, true>), grid, block, 0, st, p, dh);
+  else hipLaunchKernelGGL((attn_fwd_gen_kernel<DHP, 256, true>), grid, block, 0, st, p, dh);
+}
+}  // namespace
+
+extern "C" int vy_attn_fwd_ex(const void* q, int64_t q_sb, int64_t q_sh, int64_t q_sl, const void* k, int64_t k_sb,
+                              int64_t k_sh, int64_t k_sl, const void* v, int64_t v_sb, int64_t v_sh, int64_t v_sl,
+                              void* out, int64_t o_sb, int64_t o_sl, const void* gate, int64_t g_sb, int64_t g_sl,
+                              const int32_t* start, const int32_t* slots, int64_t B, int h, int hk, int64_t L, int64_t S,
+                              int dh, int dv, float scale, int dtype, void* stream) {
+  const char* who = "vy_attn_fwd_ex";
+  AttnParams p{};
+  p.q = q; p.q_sb = q_sb; p.q_sh = q_sh; p.q_sl = q_sl;
+  p.k = k; p.k_sb = k_sb; p.k_sh = k_sh; p.k_sl = k_sl;
+  p.v = v; p.v_sb = v_sb; p.v_sh = v_sh; p.v_sl = v_sl;
+  p.out = out; p.o_sb = o_sb; p.o_sl = o_sl;
+  p.gate = gate; p.g_sb = g_sb; p.g_sl = g_sl;
+  p.mask_kind = VY_MASK_CAUSAL; p.start_dev = start; p.slots = slots;
+  p.B = (int)B; p.h = h; p.hk = hk; p.L = (int)L; p.S = (int)S; p.scale = scale; p.dv = dv;
+  if (dtype != VY_BF16 && dtype != VY_F32) VY_FAIL(VY_ERR_ARG, "%s: bad dtype %d", who, dtype);
+  if (int rc = check_attn(who, p, dh, dtype)) return rc;
+  const int vec = dtype == VY_BF16 ? 8 : 4;
+  if (dv <= 0 || dh % vec || dv % vec) VY_FAIL(VY_ERR_ARG, "%s: head widths %d / %d must be multiples of %d", who, dh, dv, vec);
+  if (gate && (g_sb % vec || g_sl % vec || (uintptr_t)gate % 16)) VY_FAIL(VY_ERR_ARG, "%s: gate rows must be 16-byte aligned", who);
+  hipStream_t st = (hipStream_t)stream;
+  if (dtype == VY_BF16 && dh == dv && (dh == 64 || dh == 128)) {
+    const dim3 grid((unsigned)(h * B), (unsigned)((L + 127) / 128), 1), block(256);
+    if (dh == 64) hipLaunchKernelGGL((attn_fwd_mfma_kernel<64, true>), grid, block, 0, st, p);
+    else hipLaunchKernelGGL((attn_fwd_mfma_kernel<128, true>), grid, block, 0, st, p);
+  } else if (dtype == VY_BF16 && dh <= 256 && dv <= 256) {
+    const dim3 grid((unsigned)(h * B), (unsigned)((L + 63) / 64), 1);
+    if (dh <= 64) gen_go<64>(p, dh, dv, grid, st);
+    else if (dh <= 96) gen_go<96>(p, dh, dv, grid, st);
+    else if (dh <= 128) gen_go<128>(p, dh, dv, grid, st);
+    else gen_go<256>(p, dh, dv, grid, st);
+  } else {
+    return dtype == VY_BF16 ? launch_rowwise<bf16, true>(p, dh, st, who) : launch_rowwise<float, true>(p, dh, st, who);
+  }
+  VY_CHECK_LAUNCH(who);
+  return VY_OK;
 }
 
 int vy_attn_decode_ex(const void* q, int64_t q_sb, int64_t q_sh, const void* k, int64_t k_sb, int64_t k_sh,

@@ -152,10 +152,14 @@ __device__ __forceinline__ float vy_gelu_erf_grad_fast(float x) {
   return cdf + x * 0.39894228040143267794f * g;
 }
 
+__device__ __forceinline__ float vy_sigmoid(float x) { return 1.0f / (1.0f + __expf(-x)); }
+__device__ __forceinline__ float vy_silu(float x) { return x * vy_sigmoid(x); }
+
 template <int ACT>
 __device__ __forceinline__ float vy_act_fwd(float x) {
   if constexpr (ACT == VY_ACT_GELU_ERF) return vy_gelu_erf(x);
   else if constexpr (ACT == VY_ACT_GELU_TANH) return vy_gelu_tanh(x);
+  else if constexpr (ACT == VY_ACT_SILU) return vy_silu(x);
   else return x;
 }
 template <int ACT>
@@ -247,4 +251,42 @@ template <> struct VyT<float> {
 template <> struct VyT<bf16> {
   static __device__ __forceinline__ float ld(const bf16* p) { return (float)*p; }
   static __device__ __forceinline__ void st(bf16* p, float v) { *p = (bf16)v; }
+};
+
+template <typename T> struct VyChunk;  // one 16-byte chunk = VEC elements
+template <> struct VyChunk<bf16> {
+  static constexpr int VEC = 8;
+  typedef bf16x8 Raw;
+  static __device__ __forceinline__ void unpack(const Raw& t, float* v) {
+#pragma unroll
+    for (int e = 0; e < 8; ++e) v[e] = (float)t[e];
+  }
+  static __device__ __forceinline__ void load(const bf16* p, float* v) {
+    bf16x8 t = *reinterpret_cast<const bf16x8*>(p);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) v[e] = (float)t[e];
+  }
+  static __device__ __forceinline__ void store(bf16* p, const float* v) {
+    bf16x8 t;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) t[e] = (bf16)v[e];
+    *reinterpret_cast<bf16x8*>(p) = t;
+  }
+};
+template <> struct VyChunk<float> {
+  static constexpr int VEC = 4;
+  typedef f32x4 Raw;
+  static __device__ __forceinline__ void unpack(const Raw& t, float* v) {
+#pragma unroll
+    for (int e = 0; e < 4; ++e) v[e] = t[e];
+  }
+  static __device__ __forceinline__ void load(const float* p, float* v) {
+    f32x4 t = *reinterpret_cast<const f32x4*>(p);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) v[e] = t[e];
+  }
+  static __device__ __forceinline__ void store(float* p, const float* v) {
+    f32x4 t = {v[0], v[1], v[2], v[3]};
+    *reinterpret_cast<f32x4*>(p) = t;
+  }
 };

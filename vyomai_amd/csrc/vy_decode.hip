@@ -672,6 +672,7 @@ enum { GV_PLAIN = 0, GV_GATED = 1, GV_QKV = 2 };
 struct DecGemvArgs {
   const bf16* x; const bf16* w; const bf16* bias; const bf16* residual; bf16* y;
   int N, K, ldw;
+  int act;                                     // GV_GATED: VY_ACT_GELU_TANH or VY_ACT_SILU
   float eps;
   // GV_QKV
   bf16* q; bf16* k; bf16* v; long long c_sh;   // q [nq]; k / v: cache row of this position, head stride c_sh
@@ -742,7 +743,7 @@ __global__ __launch_bounds__(256) void dec_gemv1_kernel(const DecGemvArgs p) {
   } else if constexpr (EPI == GV_GATED) {
     if (lane == 0) {
       const float gte = vy_round_bf16(acc), up = vy_round_bf16(acc2);
-      p.y[n] = (bf16)(vy_gelu_tanh(gte) * up);
+      p.y[n] = (bf16)((p.act == VY_ACT_SILU ? vy_silu(gte) : vy_gelu_tanh(gte)) * up);
     }
   } else {
     float x = acc;
@@ -912,10 +913,11 @@ int vy_dec_gemv1(const void* x, const void* w, const void* bias, const void* res
   VY_CHECK_LAUNCH("vy_dec_gemv1");
   return VY_OK;
 }
-int vy_dec_gemv1_gated(const void* x, const void* wgu, void* y, int I, int K, int prescaled, float eps, hipStream_t st) {
+int vy_dec_gemv1_gated(const void* x, const void* wgu, void* y, int I, int K, int act, int prescaled, float eps, hipStream_t st) {
+  if (act != VY_ACT_GELU_TANH && act != VY_ACT_SILU) return VY_ERR_UNSUPPORTED;
   if (!gemv1_ok(x, wgu, I, K)) return VY_ERR_UNSUPPORTED;
   DecGemvArgs a{};
-  a.x = (const bf16*)x; a.w = (const bf16*)wgu; a.y = (bf16*)y; a.N = I; a.K = K; a.ldw = K; a.eps = eps;
+  a.x = (const bf16*)x; a.w = (const bf16*)wgu; a.y = (bf16*)y; a.N = I; a.K = K; a.ldw = K; a.act = act; a.eps = eps;
   if (prescaled ? dec_gemv1_go<GV_GATED, true>(a, st) : dec_gemv1_go<GV_GATED, false>(a, st)) return VY_ERR_UNSUPPORTED;
   VY_CHECK_LAUNCH("vy_dec_gemv1_gated");
   return VY_OK;

@@ -2434,23 +2434,29 @@ int vy_gemv_qkv_norm(const void* x, int64_t ldx, const void* w, int64_t ldw, con
   VY_CHECK_LAUNCH("vy_gemv_qkv_norm");
   return VY_OK;
 }
-int vy_gemv_gated(const void* x, int64_t ldx, const void* w, int64_t ldw, const void* norm_w, float eps, void* y, int64_t ldy,
-                  int64_t M, int64_t I, int64_t K, int act, void* stream) {
-  if (!gemv_ok(x, ldx, w, ldw, M, K)) VY_FAIL(VY_ERR_UNSUPPORTED, "vy_gemv_gated: needs M <= 4 and 16-byte aligned rows");
-  if (act != VY_ACT_GELU_TANH) VY_FAIL(VY_ERR_UNSUPPORTED, "vy_gemv_gated: gelu_tanh only");
+template <int ACT>
+static void gemv_gated_go(const void* x, int64_t ldx, const void* w, int64_t ldw, const void* norm_w, float eps, void* y, int64_t ldy,
+                          int64_t M, int64_t I, int64_t K, void* stream) {
   EpiPlain<bf16> ep{};
   ep.y = (bf16*)y; ep.ldy = ldy;
   EpiQkv<bf16> eq{};
   const dim3 grid((unsigned)vy_cdiv(I, 4)), block(256);
   if (norm_w == VY_NORM_PRESCALED)
-    hipLaunchKernelGGL((gemv_bf16_kernel<0, VY_ACT_GELU_TANH, 4, 2, true>), grid, block, 0, (hipStream_t)stream, (const bf16*)x, ldx,
+    hipLaunchKernelGGL((gemv_bf16_kernel<0, ACT, 4, 2, true>), grid, block, 0, (hipStream_t)stream, (const bf16*)x, ldx,
                        (const bf16*)w, ldw, (int)M, (int)I, (int)K, ep, eq, (const bf16*)nullptr, eps);
   else if (norm_w)
-    hipLaunchKernelGGL((gemv_bf16_kernel<0, VY_ACT_GELU_TANH, 4, 1, true>), grid, block, 0, (hipStream_t)stream, (const bf16*)x, ldx,
+    hipLaunchKernelGGL((gemv_bf16_kernel<0, ACT, 4, 1, true>), grid, block, 0, (hipStream_t)stream, (const bf16*)x, ldx,
                        (const bf16*)w, ldw, (int)M, (int)I, (int)K, ep, eq, (const bf16*)norm_w, eps);
   else
-    hipLaunchKernelGGL((gemv_bf16_kernel<0, VY_ACT_GELU_TANH, 4, 0, true>), grid, block, 0, (hipStream_t)stream, (const bf16*)x, ldx,
+    hipLaunchKernelGGL((gemv_bf16_kernel<0, ACT, 4, 0, true>), grid, block, 0, (hipStream_t)stream, (const bf16*)x, ldx,
                        (const bf16*)w, ldw, (int)M, (int)I, (int)K, ep, eq, (const bf16*)nullptr, 0.f);
+}
+int vy_gemv_gated(const void* x, int64_t ldx, const void* w, int64_t ldw, const void* norm_w, float eps, void* y, int64_t ldy,
+                  int64_t M, int64_t I, int64_t K, int act, void* stream) {
+  if (!gemv_ok(x, ldx, w, ldw, M, K)) VY_FAIL(VY_ERR_UNSUPPORTED, "vy_gemv_gated: needs M <= 4 and 16-byte aligned rows");
+  if (act == VY_ACT_GELU_TANH) gemv_gated_go<VY_ACT_GELU_TANH>(x, ldx, w, ldw, norm_w, eps, y, ldy, M, I, K, stream);
+  else if (act == VY_ACT_SILU) gemv_gated_go<VY_ACT_SILU>(x, ldx, w, ldw, norm_w, eps, y, ldy, M, I, K, stream);
+  else VY_FAIL(VY_ERR_UNSUPPORTED, "vy_gemv_gated: gelu_tanh and silu only");
   VY_CHECK_LAUNCH("vy_gemv_gated");
   return VY_OK;
 }

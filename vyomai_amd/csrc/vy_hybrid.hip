@@ -1,0 +1,134 @@
+// Native decode driver (host code) of decoders that mix layer kinds: one call runs a whole single-token step of a batch of
+// sequences of different lengths -- embedding, every layer (latent attention over its latent cache, or decayed linear
+// attention over its fp32 state), gated MLPs, final norm and vocabulary product.  See include/vyom_hip.h
+// (vy_hybrid_decoder_step).
+#include "vy_common.h"
+
+int vy_residual_norm_ex(float* x, int64_t ldx, const void* y, int64_t ldy, const void* table, int64_t ldt, const int64_t* ids,
+                        int64_t V, int32_t* err, const float* w_post, float eps_post, const float* w_pre, float eps_pre, void* h,
+                        int64_t ldh, int64_t M, int64_t N, int64_t NP, int rms, int* advance, const int* slots, int n_adv,
+                        int dtype, void* stream);
+int vy_dec_gemv1(const void* x, const void* w, const void* bias, const void* residual, void* y, int N, int K, int prescaled,
+                 float eps, hipStream_t st);
+int vy_dec_gemv1_gated(const void* x, const void* wgu, void* y, int I, int K, int act, int prescaled, float eps, hipStream_t st);
+int vy_gemv_gated(const void* x, int64_t ldx, const void* w, int64_t ldw, const void* norm_w, float eps, void* y, int64_t ldy,
+                  int64_t M, int64_t I, int64_t K, int act, void* stream);
+
+namespace {
+
+int64_t up(int64_t x) { return (x + 255) / 256 * 256; }
+
+struct Sizes { int64_t in, q, cq, ao, o, gu, ff, latent_ws; };   // widest of each over the layers
+
+Sizes sizes_of(const vy_hybrid_plan* p) {
+  Sizes s{};
+  auto mx = [](int64_t& a, int64_t b) { if (b > a) a = b; };
+  for (int l = 0; l < p->num_layers; ++l) {
+    const vy_hybrid_layer& L = p->layers[l];
+    mx(s.in, L.n_in);
+    mx(s.ao, (int64_t)L.heads * L.vdim);
+    if (L.mixer == VY_MIX_LATENT) {
+      mx(s.q, (int64_t)L.heads * L.dim);
+      mx(s.cq, L.q_rank_p);
+      mx(s.latent_ws, vy_latent_decode_ws_bytes(p->B, L.heads, L.kv_rank_p));
+    } else {
+      mx(s.o, (int64_t)L.heads * L.vdim);
+    }
+    mx(s.gu, 2 * (int64_t)L.ff);
+    mx(s.ff, L.ff);
+  }
+  return s;
+}
+
+// y[B, N] = x[B, K] W^T
+int product(const vy_hybrid_plan* p, const void* x, const void* w, void* y, int64_t ldy, int64_t N, int64_t K, void* stream) {
+  if (p->dtype == VY_BF16 && p->B == 1 && N <= INT32_MAX) {
+    const int rc = vy_dec_gemv1(x, w, nullptr, nullptr, y, (int)N, (int)K, 0, 0.f, (hipStream_t)stream);
+    if (rc != VY_ERR_UNSUPPORTED) return rc;
+  }
+  return vy_linear_fwd(x, K, w, K, nullptr, nullptr, 0, y, ldy, nullptr, p->B, N, K, VY_ACT_NONE, p->dtype, stream);
+}
+
+int gated(const vy_hybrid_plan* p, const vy_hybrid_layer& L, const void* x, void* gu, void* act, void* stream) {
+  if (p->dtype == VY_BF16 && p->B == 1) {
+    const int rc = vy_dec_gemv1_gated(x, L.w_gu, act, L.ff, p->dp, p->act, 0, 0.f, (hipStream_t)stream);
+    if (rc != VY_ERR_UNSUPPORTED) return rc;
+  }
+  if (p->dtype == VY_BF16 && p->B <= 4)
+    return vy_gemv_gated(x, p->dp, L.w_gu, p->dp, nullptr, 0.f, act, L.ff, p->B, L.ff, p->dp, p->act, stream);
+  const int rc = vy_linear_fwd(x, p->dp, L.w_gu, p->dp, nullptr, nullptr, 0, gu, 2 * (int64_t)L.ff, nullptr, p->B,
+                               2 * (int64_t)L.ff, p->dp, VY_ACT_NONE, p->dtype, stream);
+  return rc ? rc : vy_gated_act_fwd(gu, 2 * (int64_t)L.ff, act, L.ff, p->B, L.ff, p->act, p->dtype, stream);
+}
+
+}  // namespace
+
+extern "C" int64_t vy_hybrid_ws_bytes(const vy_hybrid_plan* p) {
+  if (!p || !p->layers) return -1;
+  const Sizes s = sizes_of(p);
+  const int64_t e = p->dtype == VY_BF16 ? 2 : 4, B = p->B;
+  return up(B * p->dp * 4) + 2 * up(B * p->dp * e) + up(B * s.in * e) + up(B * s.q * e) + up(B * s.cq * e) +
+         up(B * s.ao * e) + up(B * s.o * e) + up(B * s.gu * e) + up(B * s.ff * e) + up(s.latent_ws);
+}
+
+extern "C" int vy_hybrid_decoder_step(const vy_hybrid_plan* p, const int64_t* ids, const int32_t* slots, int32_t* lengths,
+                                      int64_t max_keys, void* logits, int64_t ldv, void* stream) {
+  const char* who = "vy_hybrid_decoder_step";
+  if (!p || !p->layers || !p->ws || !ids || !lengths || !logits) VY_FAIL(VY_ERR_ARG, "%s: null plan/input/workspace/output", who);
+  if (p->ws_bytes < vy_hybrid_ws_bytes(p)) VY_FAIL(VY_ERR_ARG, "%s: workspace too small", who);
+  if (max_keys < 1) VY_FAIL(VY_ERR_ARG, "%s: max_keys %ld", who, (long)max_keys);
+  const Sizes s = sizes_of(p);
+  const int64_t e = p->dtype == VY_BF16 ? 2 : 4, B = p->B, dp = p->dp;
+  char* w = (char*)p->ws;
+  auto take = [&](int64_t bytes) { char* r = w; w += up(bytes); return r; };
+  float* x = (float*)take(B * dp * 4);
+  void* h = take(B * dp * e);
+  void* y = take(B * dp * e);
+  void* in = take(B * s.in * e);
+  void* q = take(B * s.q * e);
+  void* cq = take(B * s.cq * e);
+  void* ao = take(B * s.ao * e);
+  void* o = take(B * s.o * e);
+  void* gu = take(B * s.gu * e);
+  void* act = take(B * s.ff * e);
+  void* lws = take(s.latent_ws);
+  int rc;
+  auto norm = [&](const void* yy, const float* post, const float* pre, bool last) {
+    return vy_residual_norm_ex(x, dp, yy, dp, p->embed, dp, yy ? nullptr : ids, p->vocab, p->err, post, p->eps, pre, p->eps, h,
+                               dp, B, p->d, dp, p->rms, last ? lengths : nullptr, slots, last ? (int)B : 0, p->dtype, stream);
+  };
+  if ((rc = norm(nullptr, nullptr, p->layers[0].norm1, false))) return rc;
+  for (int l = 0; l < p->num_layers; ++l) {
+    const vy_hybrid_layer& L = p->layers[l];
+    const bool last = l + 1 == p->num_layers;
+    const float* next = last ? p->final_norm : p->layers[l + 1].norm1;
+    const int64_t nv = (int64_t)L.heads * L.vdim, nk = (int64_t)L.heads * L.dim;
+    if ((rc = product(p, h, L.w_in, in, L.n_in, L.n_in, dp, stream))) return rc;
+    if (L.mixer == VY_MIX_LATENT) {
+      if (max_keys > L.cap) VY_FAIL(VY_ERR_ARG, "%s: %ld keys exceed the cache capacity %d", who, (long)max_keys, L.cap);
+      if ((rc = vy_latent_norm(in, L.n_in, L.q_norm, cq, L.q_rank_p, L.q_rank, L.q_rank_p, L.c_norm, nullptr, 0, L.kv_rank,
+                               L.kv_rank_p, L.cache, L.c_ss, L.c_st, L.cap, slots, lengths, nullptr, B, 1, p->eps, p->dtype,
+                               stream))) return rc;
+      if ((rc = product(p, cq, L.w_uq, q, nk, nk, L.q_rank_p, stream))) return rc;
+      const char* gate = (const char*)in + ((int64_t)L.q_rank_p + L.kv_rank_p) * e;
+      if ((rc = vy_latent_decode(q, nk, L.w_ukt, L.w_uv, L.cache, L.c_ss, L.c_st, slots, lengths, max_keys, ao, nv, gate, L.n_in,
+                                 (int)B, L.heads, L.dim, L.vdim, L.kv_rank_p, L.scale, lws, s.latent_ws, p->dtype, stream)))
+        return rc;
+    } else {
+      if ((rc = vy_decay_attn(in, L.n_in, 0, nk, 2 * nk, L.state, L.decay_pow, slots, lengths, nullptr, o, nv, B, 1, L.heads, L.dim,
+                              L.vdim, 1, nullptr, 0, p->dtype, stream))) return rc;
+      const char* gate = (const char*)in + (2 * nk + nv) * e;
+      if ((rc = vy_rmsnorm_gate(o, nv, L.mix_norm, gate, L.n_in, ao, nv, B, L.mix_n, nv, p->eps, p->dtype, stream))) return rc;
+    }
+    if ((rc = product(p, ao, L.w_o, y, dp, dp, nv, stream))) return rc;
+    if (L.ff) {
+      if ((rc = norm(y, L.norm1b, L.norm2, false))) return rc;
+      if ((rc = gated(p, L, h, gu, act, stream))) return rc;
+      if ((rc = product(p, act, L.w_down, y, dp, dp, L.ff, stream))) return rc;
+      if ((rc = norm(y, L.norm2b, next, last))) return rc;
+    } else if ((rc = norm(y, L.norm1b, next, last))) {
+      return rc;
+    }
+  }
+  return product(p, h, p->head, logits, ldv, p->vocab, dp, stream);
+}

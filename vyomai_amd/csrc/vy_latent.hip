@@ -1,0 +1,495 @@
+// Decode attention over a latent cache: one row c_j of R values per token serves every head as key AND value.
+//
+//   keys are W_uk,h c_j and values W_uv,h c_j, so the score of head h is q_h . (W_uk,h c_j) = (W_uk,h^T q_h) . c_j and the
+//   output W_uv,h (sum_j p_j c_j): the query is taken into the latent space once, the cache is streamed once for all heads
+//   (a multi-query problem whose keys and values are the same bytes), and the mean latent is expanded at the end.
+//
+// Three launches: latent_query_kernel (per-head W_uk^T q), latent_scan_kernel (flash attention over a slice of the keys,
+// fp32 partial sums), latent_value_kernel (adds the slices, expands with W_uv, applies the sigmoid output gate).
+// Precision: scores take the latent query as TWO bf16 numbers (hi + lo, ~16 bits of mantissa), so taking the query through
+// W_uk costs no accuracy against expanding the keys; likewise the mean latent in front of W_uv.
+//
+// f32 (and bf16 latents wider than 512): the same three steps with plain fp32 FMAs.
+#include "vy_common.h"
+#include <float.h>
+
+namespace {
+
+constexpr float LOG2E = 1.4426950408889634f;
+constexpr int MAX_SPLIT = 64;      // slices of the key range
+constexpr int KEYS_PER_TILE = 32;  // keys a wave takes at a time
+
+struct LatentArgs {
+  const void* q; int64_t ldq;
+  const void* wukt; const void* wuv;
+  const void* cache; int64_t c_ss, c_st;
+  const int* slots; const int* start;
+  void* out; int64_t ldo;
+  const void* gate; int64_t ldg;
+  int B, h, dh, dv, R, nsplit;
+  float c;                         // scale * log2(e)
+  // workspace
+  float* qf;                       // generic: latent queries [B][h][R]
+  bf16* qhi; bf16* qlo;            // MFMA: the same as two bf16 halves
+  float* part_o; float* part_ml;   // [B][h][nsplit][R], [B][h][nsplit][2]
+};
+
+__device__ __forceinline__ int row_keys(const LatentArgs& p, int b, int& slot) {
+  slot = p.slots ? p.slots[b] : b;
+  return p.start[slot] + 1;
+}
+// combine over the four lane groups (lane >> 4) of a 16 x 16 MFMA layout
+__device__ __forceinline__ float quad_max(float v) {
+  v = fmaxf(v, __shfl_xor(v, 16, 64));
+  return fmaxf(v, __shfl_xor(v, 32, 64));
+}
+__device__ __forceinline__ float quad_sum(float v) {
+  v += __shfl_xor(v, 16, 64);
+  return v + __shfl_xor(v, 32, 64);
+}
+__device__ __forceinline__ void split_bf16(float x, bf16& hi, bf16& lo) {
+  const float h = vy_round_bf16(x);
+  hi = (bf16)h;
+  lo = (bf16)(x - h);
+}
+
+// ---- MFMA path ------------------------------------------------------------------------------
+// q~[b][h][r] = sum_d W_uk^T[h][r][d] q[b][h][d]: workgroup = 64 latent columns of one head x 16 sequences
+__global__ __launch_bounds__(256) void latent_query_kernel(LatentArgs p) {
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const int r16 = lane & 15, kq = lane >> 4;
+  const int head = blockIdx.y, b = (int)blockIdx.z * 16 + r16;
+  const int r0 = (int)blockIdx.x * 64 + wave * 16;
+  const bf16x8 zero8 = {};
+  const bool wok = r0 + r16 < p.R, xok = b < p.B;
+  const bf16* w = (const bf16*)p.wukt + ((int64_t)head * p.R + (wok ? r0 + r16 : 0)) * p.dh;
+  const bf16* x = (const bf16*)p.q + (int64_t)(xok ? b : 0) * p.ldq + head * p.dh;
+  f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+  for (int k0 = 0; k0 < p.dh; k0 += 128) {
+    bf16x8 wf[4], xf[4];
+#pragma unroll
+    for (int u = 0; u < 4; ++u) {
+      const int k = k0 + 32 * u + 8 * kq;
+      const bool ok = k < p.dh;
+      wf[u] = ok && wok ? *reinterpret_cast<const bf16x8*>(w + k) : zero8;
+      xf[u] = ok && xok ? *reinterpret_cast<const bf16x8*>(x + k) : zero8;
+    }
+#pragma unroll
+    for (int u = 0; u < 4; ++u) acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[u], xf[u], acc, 0, 0, 0);
+  }
+  const int r = r0 + 4 * kq;   // R is a multiple of 8: the quad is inside or outside as a whole
+  if (xok && r < p.R) {
+    bf16x4 hi, lo;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) { bf16 a, c; split_bf16(acc[e], a, c); hi[e] = a; lo[e] = c; }
+    const int64_t o = ((int64_t)b * p.h + head) * p.R + r;
+    *reinterpret_cast<bf16x4*>(p.qhi + o) = hi;
+    *reinterpret_cast<bf16x4*>(p.qlo + o) = lo;
+  }
+}
+
+// grid (slices, head groups of 16, B); 4 waves, each walking its own 32-key tiles of the slice through a private LDS tile.
+// Swapped products as in attn_fwd_gen_kernel: S^T = c q~^T puts ONE head per lane column and four consecutive keys per
+// lane group, P^T is the B operand of U^T = c^T P^T as it sits, and the same LDS tile serves both products (row reads
+// for the scores, transposing reads for the mean).
+template <int RP>
+__global__ __launch_bounds__(256, 1) void latent_scan_kernel(LatentArgs p) {
+  constexpr int KT = KEYS_PER_TILE;
+  constexpr int PITCH = (RP + 8) * 2;
+  constexpr int TILE = KT * PITCH;
+  constexpr int KS = RP / 32, ND = RP / 16;
+  constexpr int CPR = RP / 8;                 // 16-byte chunks per row
+  constexpr int NCH = KT * CPR / 64;          // chunks per lane
+  // at the full width the low halves of the queries sit in LDS (one copy for the four waves) instead of 64 registers
+  constexpr bool QLDS = RP >= 512;
+  __shared__ __attribute__((aligned(16))) char smem[4 * TILE + 4 * 16 * 8 + (QLDS ? 16 * PITCH : 0)];
+  const int lane = threadIdx.x & 63;
+  const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const int r16 = lane & 15, kq = lane >> 4;
+  const int b = blockIdx.z, split = blockIdx.x;
+  const int head = (int)blockIdx.y * 16 + r16;
+  int slot;
+  const int n = row_keys(p, b, slot);
+  const int tiles = (n + KT - 1) / KT;
+  const int tps = (tiles + p.nsplit - 1) / p.nsplit;
+  const int t0 = split * tps, t1 = min(tiles, t0 + tps);
+  const bf16* C = (const bf16*)p.cache + (int64_t)slot * p.c_ss;
+  const bf16x8 zero8 = {};
+  char* tile = smem + wave * TILE;
+  float* red = reinterpret_cast<float*>(smem + 4 * TILE);   // [wave][16 heads][m, l]
+
+  char* qlt = smem + 4 * TILE + 4 * 16 * 8;
+  bf16x8 qh[KS], ql[QLDS ? 1 : KS];
+  const int64_t qo = ((int64_t)b * p.h + (head < p.h ? head : 0)) * p.R;
+#pragma unroll
+  for (int ks = 0; ks < KS; ++ks) {
+    const int k = 32 * ks + 8 * kq;
+    const bool ok = k < p.R && head < p.h;
+    qh[ks] = ok ? *reinterpret_cast<const bf16x8*>(p.qhi + qo + k) : zero8;
+    const bf16x8 low = ok ? *reinterpret_cast<const bf16x8*>(p.qlo + qo + k) : zero8;
+    if constexpr (!QLDS) ql[ks] = low;
+    else if (wave == (ks & 3)) *reinterpret_cast<bf16x8*>(qlt + r16 * PITCH + k * 2) = low;
+  }
+  if constexpr (QLDS) __syncthreads();
+  f32x4 o[ND];
+#pragma unroll
+  for (int i = 0; i < ND; ++i) o[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+  float m_run = -FLT_MAX, l_run = 0.f;
+
+  bf16x8 reg[NCH];
+  auto fetch = [&](int t) {
+#pragma unroll
+    for (int i = 0; i < NCH; ++i) {
+      const int cidx = lane + 64 * i;
+      const int row = cidx / CPR, ch = cidx % CPR;
+      const int kj = min(t * KT + row, n - 1);
+      reg[i] = ch * 8 < p.R ? __builtin_nontemporal_load(reinterpret_cast<const bf16x8*>(C + (int64_t)kj * p.c_st + ch * 8)) : zero8;
+    }
+  };
+  const unsigned vtr = vy_lds_addr(tile) + (4 * kq + (r16 >> 2)) * PITCH + (4 * (r16 & 3)) * 2;
+  int t = t0 + wave;
+  if (t < t1) fetch(t);
+  for (; t < t1; t += 4) {
+#pragma unroll
+    for (int i = 0; i < NCH; ++i) {
+      const int cidx = lane + 64 * i;
+      *reinterpret_cast<bf16x8*>(tile + (cidx / CPR) * PITCH + (cidx % CPR) * 16) = reg[i];
+    }
+    if (t + 4 < t1) fetch(t + 4);
+    f32x4 sc[2];
+#pragma unroll
+    for (int blk = 0; blk < 2; ++blk) {
+      sc[blk] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int ks = 0; ks < KS; ++ks) {
+        const bf16x8 kf = *reinterpret_cast<const bf16x8*>(tile + (16 * blk + r16) * PITCH + (32 * ks + 8 * kq) * 2);
+        bf16x8 low;
+        if constexpr (QLDS) low = *reinterpret_cast<const bf16x8*>(qlt + r16 * PITCH + (32 * ks + 8 * kq) * 2);
+        else low = ql[ks];
+        sc[blk] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, low, sc[blk], 0, 0, 0);
+        sc[blk] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qh[ks], sc[blk], 0, 0, 0);
+      }
+    }
+    float tmax = -INFINITY;
+#pragma unroll
+    for (int blk = 0; blk < 2; ++blk)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const bool vis = t * KT + 16 * blk + 4 * kq + r < n;
+        sc[blk][r] = vis ? sc[blk][r] * p.c : -INFINITY;
+        tmax = fmaxf(tmax, sc[blk][r]);
+      }
+    const float m_new = fmaxf(m_run, quad_max(tmax));
+    if (__any(m_new > m_run)) {
+      const float alpha = __builtin_amdgcn_exp2f(m_run - m_new);
+      m_run = m_new;
+      l_run *= alpha;
+#pragma unroll
+      for (int i = 0; i < ND; ++i)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) o[i][r] *= alpha;
+    }
+    bf16x8 pf;
+#pragma unroll
+    for (int blk = 0; blk < 2; ++blk)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const float e = __builtin_amdgcn_exp2f(sc[blk][r] - m_run);
+        l_run += e;
+        pf[4 * blk + r] = (bf16)e;
+      }
+    vy_static_for<ND / 4>([&](auto g_c) {
+      constexpr int g = decltype(g_c)::value;
+      union { struct { s16x4 a, b; } s; bf16x8 v; } u[4];
+      vy_static_for<4>([&](auto i_c) {
+        constexpr int i = decltype(i_c)::value;
+        u[i].s.a = vy_lds_tr16_off<(4 * g + i) * 32>(vtr);
+        u[i].s.b = vy_lds_tr16_off<(4 * g + i) * 32>(vtr + 16 * PITCH);
+      });
+      asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        vy_tie(u[i].v);
+        o[4 * g + i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(u[i].v, pf, o[4 * g + i], 0, 0, 0);
+      }
+    });
+  }
+  // the four waves' partial sums: each leaves [16 heads][RP] fp32 in its own tile
+  const float l_tot = quad_sum(l_run);
+  if (kq == 0) { red[(wave * 16 + r16) * 2] = m_run; red[(wave * 16 + r16) * 2 + 1] = l_tot; }
+  float* mine = reinterpret_cast<float*>(tile);
+#pragma unroll
+  for (int i = 0; i < ND; ++i) *reinterpret_cast<f32x4*>(mine + r16 * RP + 16 * i + 4 * kq) = o[i];
+  __syncthreads();
+  for (int idx = threadIdx.x; idx < 16 * (RP / 4); idx += 256) {
+    const int hr = idx / (RP / 4), col = (idx % (RP / 4)) * 4;
+    const int hd = (int)blockIdx.y * 16 + hr;
+    if (hd >= p.h || col >= p.R) continue;
+    float M = -FLT_MAX;
+#pragma unroll
+    for (int w = 0; w < 4; ++w) M = fmaxf(M, red[(w * 16 + hr) * 2]);
+    f32x4 s = {0.f, 0.f, 0.f, 0.f};
+    float l = 0.f;
+#pragma unroll
+    for (int w = 0; w < 4; ++w) {
+      const float a = __builtin_amdgcn_exp2f(red[(w * 16 + hr) * 2] - M);
+      l += a * red[(w * 16 + hr) * 2 + 1];
+      s += a * *reinterpret_cast<const f32x4*>(reinterpret_cast<const float*>(smem + w * TILE) + hr * RP + col);
+    }
+    const int64_t o_ = ((int64_t)b * p.h + hd) * p.nsplit + split;
+    *reinterpret_cast<f32x4*>(p.part_o + o_ * p.R + col) = s;
+    if (col == 0) { p.part_ml[o_ * 2] = M; p.part_ml[o_ * 2 + 1] = l; }
+  }
+}
+
+// weights of the slices of one (b, head): exp2(m_s - M) / L, 0 for an empty slice
+__device__ __forceinline__ void slice_weights(const LatentArgs& p, int b, int head, float* w, int lane) {
+  const float* ml = p.part_ml + ((int64_t)b * p.h + head) * p.nsplit * 2;
+  const float m = lane < p.nsplit ? ml[2 * lane] : -FLT_MAX;
+  const float l = lane < p.nsplit ? ml[2 * lane + 1] : 0.f;
+  const float M = vy_wave_max(l > 0.f ? m : -FLT_MAX);
+  const float e = l > 0.f ? __builtin_amdgcn_exp2f(m - M) : 0.f;
+  const float L = vy_wave_sum(e * l);
+  if (lane < p.nsplit) w[lane] = e / L;
+}
+
+// out[b][h][n] = (W_uv,h u_bh)_n * sigmoid(gate): workgroup = 64 value columns of one head x 16 sequences; the mean latents
+// are added up from the slices into LDS first
+__global__ __launch_bounds__(256) void latent_value_kernel(LatentArgs p) {
+  extern __shared__ __attribute__((aligned(16))) char dyn[];
+  const int RP = (p.R + 31) / 32 * 32, PITCH = (RP + 8) * 2;
+  float* sw = reinterpret_cast<float*>(dyn);                       // [16][MAX_SPLIT]
+  char* xh = dyn + 16 * MAX_SPLIT * 4;
+  char* xl = xh + 16 * PITCH;
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const int r16 = lane & 15, kq = lane >> 4;
+  const int head = blockIdx.y, b0 = (int)blockIdx.z * 16;
+  const int nb = min(16, p.B - b0);
+  const bf16x8 zero8 = {};
+  for (int i = wave; i < nb; i += 4) slice_weights(p, b0 + i, head, sw + i * MAX_SPLIT, lane);
+  __syncthreads();
+  const int q4 = RP / 4;
+  for (int idx = threadIdx.x; idx < nb * q4; idx += 256) {
+    const int i = idx / q4, col = (idx - i * q4) * 4;
+    f32x4 s = {0.f, 0.f, 0.f, 0.f};
+    if (col < p.R) {
+      const float* po = p.part_o + ((int64_t)(b0 + i) * p.h + head) * p.nsplit * p.R + col;
+#pragma unroll 4
+      for (int k = 0; k < p.nsplit; ++k) s += sw[i * MAX_SPLIT + k] * *reinterpret_cast<const f32x4*>(po + (int64_t)k * p.R);
+    }
+    bf16x4 hi, lo;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) { bf16 a, c; split_bf16(s[e], a, c); hi[e] = a; lo[e] = c; }
+    *reinterpret_cast<bf16x4*>(xh + i * PITCH + col * 2) = hi;
+    *reinterpret_cast<bf16x4*>(xl + i * PITCH + col * 2) = lo;
+  }
+  __syncthreads();
+  const int n0 = (int)blockIdx.x * 64 + wave * 16;
+  if (n0 >= p.dv) return;
+  const bool wok = n0 + r16 < p.dv;
+  const bf16* w = (const bf16*)p.wuv + ((int64_t)head * p.dv + (wok ? n0 + r16 : 0)) * p.R;
+  f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+  for (int k0 = 0; k0 < p.R; k0 += 128) {
+    bf16x8 wf[4];
+#pragma unroll
+    for (int u = 0; u < 4; ++u) {
+      const int k = k0 + 32 * u + 8 * kq;
+      wf[u] = wok && k < p.R ? *reinterpret_cast<const bf16x8*>(w + k) : zero8;
+    }
+#pragma unroll
+    for (int u = 0; u < 4; ++u) {
+      const int k = k0 + 32 * u + 8 * kq;
+      const bool ok = r16 < nb && k < RP;
+      const bf16x8 a = ok ? *reinterpret_cast<const bf16x8*>(xl + r16 * PITCH + k * 2) : zero8;
+      const bf16x8 c = ok ? *reinterpret_cast<const bf16x8*>(xh + r16 * PITCH + k * 2) : zero8;
+      acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[u], a, acc, 0, 0, 0);
+      acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[u], c, acc, 0, 0, 0);
+    }
+  }
+  const int nn = n0 + 4 * kq;
+  if (r16 < nb && nn < p.dv) {
+    const int64_t b = b0 + r16;
+    bf16x4 r;
+    float g[4] = {1.f, 1.f, 1.f, 1.f};
+    if (p.gate) {
+      const bf16x4 g4 = *reinterpret_cast<const bf16x4*>((const bf16*)p.gate + b * p.ldg + head * p.dv + nn);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) g[e] = vy_sigmoid((float)g4[e]);
+    }
+#pragma unroll
+    for (int e = 0; e < 4; ++e) r[e] = (bf16)(acc[e] * g[e]);
+    *reinterpret_cast<bf16x4*>((bf16*)p.out + b * p.ldo + head * p.dv + nn) = r;
+  }
+}
+
+// ---- generic path (fp32, or bf16 latents wider than 512): one wave per scalar product ------------
+template <typename T>
+__global__ __launch_bounds__(256) void latent_query_gen_kernel(LatentArgs p) {
+  const int lane = threadIdx.x & 63;
+  const int r = (int)blockIdx.x * 4 + (threadIdx.x >> 6), head = blockIdx.y, b = blockIdx.z;
+  if (r >= p.R) return;
+  const T* w = (const T*)p.wukt + ((int64_t)head * p.R + r) * p.dh;
+  const T* x = (const T*)p.q + (int64_t)b * p.ldq + head * p.dh;
+  float s = 0.f;
+  for (int k = lane; k < p.dh; k += 64) s = fmaf(VyT<T>::ld(w + k), VyT<T>::ld(x + k), s);
+  s = vy_wave_sum(s);
+  if (lane == 0) p.qf[((int64_t)b * p.h + head) * p.R + r] = s;
+}
+
+template <typename T, int NR>
+__global__ __launch_bounds__(256) void latent_scan_gen_kernel(LatentArgs p) {
+  __shared__ float so[4][NR * 64];
+  __shared__ float sm[4], sl[4];
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const int split = blockIdx.x, head = blockIdx.y, b = blockIdx.z;
+  int slot;
+  const int n = row_keys(p, b, slot);
+  const int kps = (n + p.nsplit - 1) / p.nsplit;
+  const int j1 = min(n, (split + 1) * kps);
+  const T* C = (const T*)p.cache + (int64_t)slot * p.c_ss;
+  const int64_t o_ = ((int64_t)b * p.h + head) * p.nsplit + split;
+  float q[NR], acc[NR];
+#pragma unroll
+  for (int i = 0; i < NR; ++i) {
+    const int col = lane + 64 * i;
+    q[i] = col < p.R ? p.qf[((int64_t)b * p.h + head) * p.R + col] : 0.f;
+    acc[i] = 0.f;
+  }
+  float m = -FLT_MAX, l = 0.f;
+  for (int j = split * kps + wave; j < j1; j += 4) {
+    float c[NR], d = 0.f;
+#pragma unroll
+    for (int i = 0; i < NR; ++i) {
+      const int col = lane + 64 * i;
+      c[i] = col < p.R ? VyT<T>::ld(C + (int64_t)j * p.c_st + col) : 0.f;
+      d = fmaf(q[i], c[i], d);
+    }
+    const float s = vy_wave_sum(d) * p.c;
+    const float mn = fmaxf(m, s);
+    const float a = exp2f(m - mn), e = exp2f(s - mn);
+    m = mn;
+    l = l * a + e;
+#pragma unroll
+    for (int i = 0; i < NR; ++i) acc[i] = acc[i] * a + e * c[i];
+  }
+#pragma unroll
+  for (int i = 0; i < NR; ++i) so[wave][lane + 64 * i] = acc[i];
+  if (lane == 0) { sm[wave] = m; sl[wave] = l; }
+  __syncthreads();
+  const float M = fmaxf(fmaxf(sm[0], sm[1]), fmaxf(sm[2], sm[3]));
+  float w[4], L = 0.f;
+#pragma unroll
+  for (int i = 0; i < 4; ++i) { w[i] = exp2f(sm[i] - M); L += w[i] * sl[i]; }
+  for (int col = threadIdx.x; col < p.R; col += 256)
+    p.part_o[o_ * p.R + col] = w[0] * so[0][col] + w[1] * so[1][col] + w[2] * so[2][col] + w[3] * so[3][col];
+  if (threadIdx.x == 0) { p.part_ml[o_ * 2] = M; p.part_ml[o_ * 2 + 1] = L; }
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void latent_value_gen_kernel(LatentArgs p) {
+  __shared__ float u[1024];
+  __shared__ float sw[MAX_SPLIT];
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const int head = blockIdx.y, b = blockIdx.z;
+  if (wave == 0) slice_weights(p, b, head, sw, lane);
+  __syncthreads();
+  const float* po = p.part_o + ((int64_t)b * p.h + head) * p.nsplit * p.R;
+  for (int col = threadIdx.x; col < p.R; col += 256) {
+    float s = 0.f;
+    for (int k = 0; k < p.nsplit; ++k) s = fmaf(sw[k], po[(int64_t)k * p.R + col], s);
+    u[col] = s;
+  }
+  __syncthreads();
+  const int n1 = min(p.dv, ((int)blockIdx.x + 1) * 64);
+  for (int n = (int)blockIdx.x * 64 + wave; n < n1; n += 4) {
+    const T* w = (const T*)p.wuv + ((int64_t)head * p.dv + n) * p.R;
+    float s = 0.f;
+    for (int k = lane; k < p.R; k += 64) s = fmaf(VyT<T>::ld(w + k), u[k], s);
+    s = vy_wave_sum(s);
+    if (lane == 0) {
+      if (p.gate) s *= vy_sigmoid(VyT<T>::ld((const T*)p.gate + (int64_t)b * p.ldg + head * p.dv + n));
+      VyT<T>::st((T*)p.out + (int64_t)b * p.ldo + head * p.dv + n, s);
+    }
+  }
+}
+
+int64_t up256(int64_t x) { return (x + 255) / 256 * 256; }
+int64_t query_bytes(int B, int h, int R) { return up256((int64_t)B * h * R * 4); }
+
+// slices of the key range: about two workgroups per CU in all (one where the LDS tile fills a CU), at least one tile per wave
+int pick_split(int B, int groups, int64_t max_keys, int R) {
+  const int64_t tiles = (max_keys + KEYS_PER_TILE - 1) / KEYS_PER_TILE;
+  const int64_t want = vy_cdiv(R > 256 ? 256 : 512, (int64_t)B * groups);
+  int64_t s = vy_cdiv(tiles, 4);
+  if (s > want) s = want;
+  if (s > MAX_SPLIT) s = MAX_SPLIT;
+  return (int)(s < 1 ? 1 : s);
+}
+
+template <typename T>
+int generic_go(LatentArgs& p, int64_t max_keys, hipStream_t st) {
+  int64_t s = vy_cdiv(512, (int64_t)p.B * p.h);
+  if (s > vy_cdiv(max_keys, 64)) s = vy_cdiv(max_keys, 64);
+  p.nsplit = (int)(s > MAX_SPLIT ? MAX_SPLIT : s < 1 ? 1 : s);
+  const dim3 block(256);
+  hipLaunchKernelGGL(latent_query_gen_kernel<T>, dim3((unsigned)vy_cdiv(p.R, 4), p.h, p.B), block, 0, st, p);
+  const dim3 grid(p.nsplit, p.h, p.B);
+  if (p.R <= 128) hipLaunchKernelGGL((latent_scan_gen_kernel<T, 2>), grid, block, 0, st, p);
+  else if (p.R <= 256) hipLaunchKernelGGL((latent_scan_gen_kernel<T, 4>), grid, block, 0, st, p);
+  else if (p.R <= 512) hipLaunchKernelGGL((latent_scan_gen_kernel<T, 8>), grid, block, 0, st, p);
+  else hipLaunchKernelGGL((latent_scan_gen_kernel<T, 16>), grid, block, 0, st, p);
+  hipLaunchKernelGGL(latent_value_gen_kernel<T>, dim3((unsigned)vy_cdiv(p.dv, 64), p.h, p.B), block, 0, st, p);
+  return 0;
+}
+
+}  // namespace
+
+// latent queries and the partial sums of at most max(512 / (B groups), 1) <= MAX_SPLIT slices
+extern "C" int64_t vy_latent_decode_ws_bytes(int32_t B, int32_t h, int32_t R) {
+  int64_t s = vy_cdiv(512, (int64_t)B * ((h + 15) / 16));
+  if (s > MAX_SPLIT) s = MAX_SPLIT;
+  return query_bytes(B, h, R) + up256((int64_t)B * h * s * R * 4) + up256((int64_t)B * h * s * 8);
+}
+
+extern "C" int vy_latent_decode(const void* q, int64_t ldq, const void* wukt, const void* wuv, const void* cache, int64_t c_ss,
+                                int64_t c_st, const int32_t* slots, const int32_t* start, int64_t max_keys, void* out,
+                                int64_t ldo, const void* gate, int64_t ldg, int32_t B, int32_t h, int32_t dh, int32_t dv,
+                                int32_t R, float scale, void* ws, int64_t ws_bytes, int dtype, void* stream) {
+  const char* who = "vy_latent_decode";
+  if (!q || !wukt || !wuv || !cache || !start || !out || !ws) VY_FAIL(VY_ERR_ARG, "%s: null pointer", who);
+  if (B <= 0 || h <= 0 || dh <= 0 || dv <= 0 || R <= 0 || max_keys <= 0) VY_FAIL(VY_ERR_ARG, "%s: empty problem", who);
+  if (dh % 8 || dv % 8 || R % 8 || ldq % 8 || ldo % 8 || ldg % 8 || c_ss % 8 || c_st % 8)
+    VY_FAIL(VY_ERR_ARG, "%s: widths and strides must be multiples of 8", who);
+  if (R > 1024) VY_FAIL(VY_ERR_UNSUPPORTED, "%s: latent width %d > 1024", who, R);
+  if (ws_bytes < vy_latent_decode_ws_bytes(B, h, R)) VY_FAIL(VY_ERR_ARG, "%s: workspace too small", who);
+  hipStream_t st = (hipStream_t)stream;
+  LatentArgs p{};
+  p.q = q; p.ldq = ldq; p.wukt = wukt; p.wuv = wuv; p.cache = cache; p.c_ss = c_ss; p.c_st = c_st;
+  p.slots = slots; p.start = start; p.out = out; p.ldo = ldo; p.gate = gate; p.ldg = ldg;
+  p.B = B; p.h = h; p.dh = dh; p.dv = dv; p.R = R; p.c = scale * LOG2E;
+  char* w = (char*)ws;
+  p.qf = (float*)w; p.qhi = (bf16*)w; p.qlo = p.qhi + (int64_t)B * h * R;
+  int64_t s = vy_cdiv(512, (int64_t)B * ((h + 15) / 16));
+  if (s > MAX_SPLIT) s = MAX_SPLIT;
+  p.part_o = (float*)(w + query_bytes(B, h, R));
+  p.part_ml = (float*)(w + query_bytes(B, h, R) + up256((int64_t)B * h * s * R * 4));
+  if (dtype == VY_F32) generic_go<float>(p, max_keys, st);
+  else if (dtype != VY_BF16) VY_FAIL(VY_ERR_ARG, "%s: bad dtype %d", who, dtype);
+  else if (R > 512) generic_go<bf16>(p, max_keys, st);
+  else {
+    const int groups = (h + 15) / 16, bt = (B + 15) / 16;
+    p.nsplit = pick_split(B, groups, max_keys, R);
+    const dim3 block(256);
+    hipLaunchKernelGGL(latent_query_kernel, dim3((unsigned)vy_cdiv(R, 64), h, bt), block, 0, st, p);
+    const dim3 grid(p.nsplit, groups, B);
+    if (R <= 64) hipLaunchKernelGGL(latent_scan_kernel<64>, grid, block, 0, st, p);
+    else if (R <= 128) hipLaunchKernelGGL(latent_scan_kernel<128>, grid, block, 0, st, p);
+    else if (R <= 256) hipLaunchKernelGGL(latent_scan_kernel<256>, grid, block, 0, st, p);
+    else hipLaunchKernelGGL(latent_scan_kernel<512>, grid, block, 0, st, p);
+    const int RP = (R + 31) / 32 * 32;
+    hipLaunchKernelGGL(latent_value_kernel, dim3((unsigned)vy_cdiv(dv, 64), h, bt), block,
+                       16 * MAX_SPLIT * 4 + 2 * 16 * (RP + 8) * 2, st, p);
+  }
+  VY_CHECK_LAUNCH(who);
+  return VY_OK;
+}

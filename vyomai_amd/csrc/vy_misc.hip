@@ -17,44 +17,6 @@ extern "C" int vy_abi_version(void) { return 5; }
 
 namespace {
 
-template <typename T> struct Chunk;  // one 16-byte chunk = VEC elements
-template <> struct Chunk<bf16> {
-  static constexpr int VEC = 8;
-  typedef bf16x8 Raw;
-  static __device__ __forceinline__ void unpack(const Raw& t, float* v) {
-#pragma unroll
-    for (int e = 0; e < 8; ++e) v[e] = (float)t[e];
-  }
-  static __device__ __forceinline__ void load(const bf16* p, float* v) {
-    bf16x8 t = *reinterpret_cast<const bf16x8*>(p);
-#pragma unroll
-    for (int e = 0; e < 8; ++e) v[e] = (float)t[e];
-  }
-  static __device__ __forceinline__ void store(bf16* p, const float* v) {
-    bf16x8 t;
-#pragma unroll
-    for (int e = 0; e < 8; ++e) t[e] = (bf16)v[e];
-    *reinterpret_cast<bf16x8*>(p) = t;
-  }
-};
-template <> struct Chunk<float> {
-  static constexpr int VEC = 4;
-  typedef f32x4 Raw;
-  static __device__ __forceinline__ void unpack(const Raw& t, float* v) {
-#pragma unroll
-    for (int e = 0; e < 4; ++e) v[e] = t[e];
-  }
-  static __device__ __forceinline__ void load(const float* p, float* v) {
-    f32x4 t = *reinterpret_cast<const f32x4*>(p);
-#pragma unroll
-    for (int e = 0; e < 4; ++e) v[e] = t[e];
-  }
-  static __device__ __forceinline__ void store(float* p, const float* v) {
-    f32x4 t = {v[0], v[1], v[2], v[3]};
-    *reinterpret_cast<f32x4*>(p) = t;
-  }
-};
-
 // ---- LayerNorm forward: one wave per row, CH chunks per lane -------------------------------
 // mean, then variance about the mean (two reductions on registers): the same two-pass
 // formulation as aten's CPU LayerNorm closely enough for 1e-6 agreement.
@@ -65,7 +27,7 @@ __global__ __launch_bounds__(256) void layernorm_fwd_kernel(const T* __restrict_
                                                             int64_t ldy, float* __restrict__ mean_out,
                                                             float* __restrict__ rstd_out, int64_t M, int N,
                                                             float eps) {
-  constexpr int VEC = Chunk<T>::VEC;
+  constexpr int VEC = VyChunk<T>::VEC;
   const int lane = threadIdx.x & 63;
   const int64_t row = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
   if (row >= M) return;
@@ -76,7 +38,7 @@ __global__ __launch_bounds__(256) void layernorm_fwd_kernel(const T* __restrict_
   for (int c = 0; c < CH; ++c) {
     const int ch = lane + 64 * c;
     if (ch < nch) {
-      Chunk<T>::load(x + row * ldx + (int64_t)ch * VEC, v[c]);
+      VyChunk<T>::load(x + row * ldx + (int64_t)ch * VEC, v[c]);
 #pragma unroll
       for (int e = 0; e < VEC; ++e) s += v[c][e];
     } else {
@@ -103,11 +65,11 @@ __global__ __launch_bounds__(256) void layernorm_fwd_kernel(const T* __restrict_
     const int ch = lane + 64 * c;
     if (ch < nch) {
       float g[VEC], b[VEC], o[VEC];
-      Chunk<T>::load(gamma + (int64_t)ch * VEC, g);
-      Chunk<T>::load(beta + (int64_t)ch * VEC, b);
+      VyChunk<T>::load(gamma + (int64_t)ch * VEC, g);
+      VyChunk<T>::load(beta + (int64_t)ch * VEC, b);
 #pragma unroll
       for (int e = 0; e < VEC; ++e) o[e] = (v[c][e] - mean) * rstd_r * g[e] + b[e];
-      Chunk<T>::store(y + row * ldy + (int64_t)ch * VEC, o);
+      VyChunk<T>::store(y + row * ldy + (int64_t)ch * VEC, o);
     }
   }
   if (lane == 0) {
@@ -122,7 +84,7 @@ template <typename T, int CH>
 __global__ __launch_bounds__(256) void rmsnorm_fwd_kernel(const T* __restrict__ x, int64_t ldx,
                                                           const T* __restrict__ w, T* __restrict__ y, int64_t ldy,
                                                           int64_t M, int N, float eps, float w_offset) {
-  constexpr int VEC = Chunk<T>::VEC;
+  constexpr int VEC = VyChunk<T>::VEC;
   const int lane = threadIdx.x & 63;
   const int64_t row = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
   if (row >= M) return;
@@ -133,7 +95,7 @@ __global__ __launch_bounds__(256) void rmsnorm_fwd_kernel(const T* __restrict__ 
   for (int c = 0; c < CH; ++c) {
     const int ch = lane + 64 * c;
     if (ch < nch) {
-      Chunk<T>::load(x + row * ldx + (int64_t)ch * VEC, v[c]);
+      VyChunk<T>::load(x + row * ldx + (int64_t)ch * VEC, v[c]);
 #pragma unroll
       for (int e = 0; e < VEC; ++e) q += v[c][e] * v[c][e];
     }
@@ -146,10 +108,10 @@ __global__ __launch_bounds__(256) void rmsnorm_fwd_kernel(const T* __restrict__ 
     const int ch = lane + 64 * c;
     if (ch < nch) {
       float g[VEC], o[VEC];
-      Chunk<T>::load(w + (int64_t)ch * VEC, g);
+      VyChunk<T>::load(w + (int64_t)ch * VEC, g);
 #pragma unroll
       for (int e = 0; e < VEC; ++e) o[e] = v[c][e] * r * (w_offset + g[e]);
-      Chunk<T>::store(y + row * ldy + (int64_t)ch * VEC, o);
+      VyChunk<T>::store(y + row * ldy + (int64_t)ch * VEC, o);
     }
   }
 }
@@ -158,18 +120,18 @@ __global__ __launch_bounds__(256) void rmsnorm_fwd_kernel(const T* __restrict__ 
 template <typename T, int ACT>
 __global__ void gated_act_kernel(const T* __restrict__ gu, int64_t ldg, T* __restrict__ out, int64_t ldo,
                                  int64_t M, int I) {
-  constexpr int VEC = Chunk<T>::VEC;
+  constexpr int VEC = VyChunk<T>::VEC;
   const int nch = I / VEC;
   const int64_t total = M * nch;
   for (int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x; i < total; i += (int64_t)gridDim.x * blockDim.x) {
     const int64_t m = i / nch;
     const int c = (int)(i - m * nch) * VEC;
     float a[VEC], b[VEC], o[VEC];
-    Chunk<T>::load(gu + m * ldg + c, a);
-    Chunk<T>::load(gu + m * ldg + I + c, b);
+    VyChunk<T>::load(gu + m * ldg + c, a);
+    VyChunk<T>::load(gu + m * ldg + I + c, b);
 #pragma unroll
     for (int e = 0; e < VEC; ++e) o[e] = vy_act_fwd<ACT>(a[e]) * b[e];
-    Chunk<T>::store(out + m * ldo + c, o);
+    VyChunk<T>::store(out + m * ldo + c, o);
   }
 }
 
@@ -181,7 +143,7 @@ __global__ __launch_bounds__(256) void layernorm_bwd_kernel(
     const T* __restrict__ dy, int64_t lddy, const T* __restrict__ x, int64_t ldx,
     const T* __restrict__ gamma, const float* __restrict__ mean, const float* __restrict__ rstd,
     T* __restrict__ dx, int64_t lddx, float* __restrict__ ws, int64_t M, int N, int W) {
-  constexpr int VEC = Chunk<T>::VEC;
+  constexpr int VEC = VyChunk<T>::VEC;
   const int lane = threadIdx.x & 63;
   const int wid = blockIdx.x * 4 + (threadIdx.x >> 6);  // W = 4 * gridDim.x waves walk the rows
   const int nch = N / VEC;
@@ -191,12 +153,12 @@ __global__ __launch_bounds__(256) void layernorm_bwd_kernel(
     const int ch = lane + 64 * c;
 #pragma unroll
     for (int e = 0; e < VEC; ++e) { dg[c][e] = 0.f; db[c][e] = 0.f; g[c][e] = 0.f; }
-    if (ch < nch) Chunk<T>::load(gamma + (int64_t)ch * VEC, g[c]);
+    if (ch < nch) VyChunk<T>::load(gamma + (int64_t)ch * VEC, g[c]);
   }
   // software pipeline over the rows of this wave: the 16-byte loads (and the row statistics) of
   // the NEXT row are issued before the reductions of the current one, so the HBM latency of a row
   // hides behind the previous row's math instead of serialising with it
-  typedef typename Chunk<T>::Raw Raw;
+  typedef typename VyChunk<T>::Raw Raw;
   Raw xr[CH], dr[CH], xn[CH], dn[CH];
   float mu = 0.f, rs = 0.f, mu_n = 0.f, rs_n = 0.f;
   auto fetch = [&](int64_t row, Raw (&xa)[CH], Raw (&da)[CH], float& m_, float& r_) {
@@ -221,8 +183,8 @@ __global__ __launch_bounds__(256) void layernorm_bwd_kernel(
       const int ch = lane + 64 * c;
       if (ch < nch) {
         float xv[VEC], dv[VEC];
-        Chunk<T>::unpack(xr[c], xv);
-        Chunk<T>::unpack(dr[c], dv);
+        VyChunk<T>::unpack(xr[c], xv);
+        VyChunk<T>::unpack(dr[c], dv);
 #pragma unroll
         for (int e = 0; e < VEC; ++e) {
           xh[c][e] = (xv[e] - mu) * rs;
@@ -243,7 +205,7 @@ __global__ __launch_bounds__(256) void layernorm_bwd_kernel(
         float o[VEC];
 #pragma unroll
         for (int e = 0; e < VEC; ++e) o[e] = rs * (gy[c][e] - s1 - xh[c][e] * s2);
-        Chunk<T>::store(dx + row * lddx + (int64_t)ch * VEC, o);
+        VyChunk<T>::store(dx + row * lddx + (int64_t)ch * VEC, o);
       }
     }
     if (more) {
@@ -440,7 +402,7 @@ __global__ __launch_bounds__(256) void transpose_batched_kernel(const vy_transpo
     const int gr = r0 + r, gc = c0 + cc;
     if (gr >= d.R) continue;
     if (vec_in && gc + VEC <= d.C) {
-      typedef typename Chunk<T>::Raw Raw;
+      typedef typename VyChunk<T>::Raw Raw;
       const Raw raw = *reinterpret_cast<const Raw*>(in + (int64_t)gr * d.ldin + gc);
       const T* e = reinterpret_cast<const T*>(&raw);
 #pragma unroll
@@ -456,7 +418,7 @@ __global__ __launch_bounds__(256) void transpose_batched_kernel(const vy_transpo
     const int gc = c0 + oc, gr = r0 + rr;
     if (gc >= d.C) continue;
     if (vec_out && gr + VEC <= d.R) {
-      typedef typename Chunk<T>::Raw Raw;
+      typedef typename VyChunk<T>::Raw Raw;
       Raw raw;
       T* e = reinterpret_cast<T*>(&raw);
 #pragma unroll
@@ -522,15 +484,15 @@ __global__ void adamw_kernel(float* __restrict__ p, const float* __restrict__ g,
 template <typename T, int ACT>
 __global__ void act_bwd_kernel(const T* __restrict__ dy, int64_t lddy, const T* __restrict__ pre, int64_t ldpre,
                                T* __restrict__ dx, int64_t lddx, int64_t M, int N) {
-  constexpr int VEC = Chunk<T>::VEC;
+  constexpr int VEC = VyChunk<T>::VEC;
   const int nch = N / VEC;
   const int64_t total = M * nch;
   for (int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x; i < total; i += (int64_t)gridDim.x * blockDim.x) {
     const int64_t m = i / nch;
     const int c = (int)(i - m * nch) * VEC;
     float a[VEC], b[VEC], o[VEC];
-    Chunk<T>::load(dy + m * lddy + c, a);
-    Chunk<T>::load(pre + m * ldpre + c, b);
+    VyChunk<T>::load(dy + m * lddy + c, a);
+    VyChunk<T>::load(pre + m * ldpre + c, b);
 #pragma unroll
     for (int e = 0; e < VEC; ++e) {
       // bf16: the derivative the GEMM epilogues use (vy_act_grad_fast: its error is below bf16 rounding; libm's erff made
@@ -538,7 +500,7 @@ __global__ void act_bwd_kernel(const T* __restrict__ dy, int64_t lddy, const T* 
       if constexpr (sizeof(T) == 2) o[e] = a[e] * vy_act_grad_fast<ACT>(b[e]);
       else o[e] = a[e] * vy_act_grad<ACT>(b[e]);
     }
-    Chunk<T>::store(dx + m * lddx + c, o);
+    VyChunk<T>::store(dx + m * lddx + c, o);
   }
 }
 
@@ -559,7 +521,7 @@ __global__ __launch_bounds__(256) void xent_fwd_kernel(const T* __restrict__ log
                                                        const int64_t* __restrict__ labels, int64_t ignore,
                                                        float* __restrict__ lse, float* __restrict__ loss_sum,
                                                        float* __restrict__ count, int V, int* __restrict__ err) {
-  constexpr int VEC = Chunk<T>::VEC;
+  constexpr int VEC = VyChunk<T>::VEC;
   __shared__ float red[4];
   const int64_t m = blockIdx.x;
   const int64_t label = labels[m];
@@ -573,7 +535,7 @@ __global__ __launch_bounds__(256) void xent_fwd_kernel(const T* __restrict__ log
   float mx = -INFINITY, sm = 0.f;
   for (int c = threadIdx.x; c < nch; c += blockDim.x) {
     float v[VEC];
-    Chunk<T>::load(row + (int64_t)c * VEC, v);  // the padded tail of the row is readable
+    VyChunk<T>::load(row + (int64_t)c * VEC, v);  // the padded tail of the row is readable
     float cm = -INFINITY;
 #pragma unroll
     for (int e = 0; e < VEC; ++e) if (c * VEC + e < V) cm = fmaxf(cm, v[e]);
@@ -599,7 +561,7 @@ __global__ __launch_bounds__(256) void xent_bwd_kernel(T* __restrict__ logits, i
                                                        const int64_t* __restrict__ labels, int64_t ignore,
                                                        const float* __restrict__ lse, const float* __restrict__ gscale,
                                                        const float* __restrict__ count, int V) {
-  constexpr int VEC = Chunk<T>::VEC;
+  constexpr int VEC = VyChunk<T>::VEC;
   const int64_t m = blockIdx.x;
   const int64_t label = labels[m];
   T* row = logits + m * ld;
@@ -609,7 +571,7 @@ __global__ __launch_bounds__(256) void xent_bwd_kernel(T* __restrict__ logits, i
   const float l = lse[m];
   for (int c = threadIdx.x; c < nch; c += blockDim.x) {
     float v[VEC], o[VEC];
-    Chunk<T>::load(row + (int64_t)c * VEC, v);
+    VyChunk<T>::load(row + (int64_t)c * VEC, v);
 #pragma unroll
     for (int e = 0; e < VEC; ++e) {
       const int col = c * VEC + e;
@@ -617,7 +579,7 @@ __global__ __launch_bounds__(256) void xent_bwd_kernel(T* __restrict__ logits, i
       if (!dead && col < V) g = (__expf(v[e] - l) - (col == label ? 1.f : 0.f)) * sc;
       o[e] = g;  // pad columns stay zero
     }
-    Chunk<T>::store(row + (int64_t)c * VEC, o);
+    VyChunk<T>::store(row + (int64_t)c * VEC, o);
   }
 }
 
@@ -702,7 +664,7 @@ __global__ __launch_bounds__(1024) void xent_fused_kernel(bf16* __restrict__ log
 template <typename T>
 int ln_fwd_dispatch(const void* x, int64_t ldx, const void* gamma, const void* beta, void* y, int64_t ldy,
                     float* mean, float* rstd, int64_t M, int64_t N, float eps, hipStream_t st) {
-  constexpr int VEC = Chunk<T>::VEC;
+  constexpr int VEC = VyChunk<T>::VEC;
   if (N % VEC || ldx % VEC || ldy % VEC) VY_FAIL(VY_ERR_ARG, "vy_layernorm_fwd: N/ld must be multiples of %d", VEC);
   const int nch = (int)(N / VEC);
   const dim3 grid((unsigned)vy_cdiv(M, 4)), block(256);
@@ -724,7 +686,7 @@ template <typename T>
 int ln_bwd_dispatch(const void* dy, int64_t lddy, const void* x, int64_t ldx, const void* gamma,
                     const float* mean, const float* rstd, void* dx, int64_t lddx, float* dgamma,
                     float* dbeta, float beta, float* ws, int64_t M, int64_t N, hipStream_t st) {
-  constexpr int VEC = Chunk<T>::VEC;
+  constexpr int VEC = VyChunk<T>::VEC;
   if (N % VEC || ldx % VEC || lddy % VEC || lddx % VEC) VY_FAIL(VY_ERR_ARG, "vy_layernorm_bwd: N/ld must be multiples of %d", VEC);
   const int nch = (int)(N / VEC);
   const int WB = (int)vy_layernorm_bwd_ws_rows(M);  // blocks = slab rows
@@ -803,6 +765,8 @@ extern "C" int vy_gated_act_fwd(const void* gate_up, int64_t ldg, void* out, int
 #define GA_GO(T, A) hipLaunchKernelGGL((gated_act_kernel<T, A>), grid, block, 0, st, (const T*)gate_up, ldg, (T*)out, ldo, M, (int)I)
   if (dtype == VY_BF16 && act == VY_ACT_GELU_TANH) GA_GO(bf16, VY_ACT_GELU_TANH);
   else if (dtype == VY_BF16 && act == VY_ACT_GELU_ERF) GA_GO(bf16, VY_ACT_GELU_ERF);
+  else if (dtype == VY_BF16 && act == VY_ACT_SILU) GA_GO(bf16, VY_ACT_SILU);
+  else if (dtype == VY_F32 && act == VY_ACT_SILU) GA_GO(float, VY_ACT_SILU);
   else if (dtype == VY_F32 && act == VY_ACT_GELU_TANH) GA_GO(float, VY_ACT_GELU_TANH);
   else if (dtype == VY_F32 && act == VY_ACT_GELU_ERF) GA_GO(float, VY_ACT_GELU_ERF);
   else VY_FAIL(VY_ERR_ARG, "vy_gated_act_fwd: unsupported act %d / dtype %d", act, dtype);
@@ -946,7 +910,7 @@ template <typename T>
 __global__ __launch_bounds__(256) void embedding_fwd_kernel(const T* __restrict__ table, int64_t ldt,
                                                             const int64_t* __restrict__ ids, T* __restrict__ out,
                                                             int64_t ldo, int64_t M, int d, int64_t V, int* err) {
-  constexpr int VEC = Chunk<T>::VEC;
+  constexpr int VEC = VyChunk<T>::VEC;
   const int lane = threadIdx.x & 63;
   const int64_t m = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
   if (m >= M) return;
@@ -959,9 +923,9 @@ __global__ __launch_bounds__(256) void embedding_fwd_kernel(const T* __restrict_
 #pragma unroll
       for (int e = 0; e < VEC; ++e) v[e] = 0.f;
     } else {
-      Chunk<T>::load(table + id * ldt + (int64_t)c * VEC, v);
+      VyChunk<T>::load(table + id * ldt + (int64_t)c * VEC, v);
     }
-    Chunk<T>::store(out + m * ldo + (int64_t)c * VEC, v);
+    VyChunk<T>::store(out + m * ldo + (int64_t)c * VEC, v);
   }
 }
 

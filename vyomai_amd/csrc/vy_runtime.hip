@@ -51,7 +51,7 @@ extern "C" int vy_debug_set_decode_lean(int v) { g_decode_lean = v; return 0; }
 
 int vy_dec_gemv1(const void* x, const void* w, const void* bias, const void* residual, void* y, int N, int K, int prescaled,
                  float eps, hipStream_t st);
-int vy_dec_gemv1_gated(const void* x, const void* wgu, void* y, int I, int K, int prescaled, float eps, hipStream_t st);
+int vy_dec_gemv1_gated(const void* x, const void* wgu, void* y, int I, int K, int act, int prescaled, float eps, hipStream_t st);
 int vy_dec_gemv1_qkv(const void* x, const void* w, const void* bias, void* q, void* k, void* v, int64_t c_sh, int h, int hk,
                      int dh, const float* cos_tab, const float* sin_tab, int64_t pos, int K, int prescaled, float eps,
                      hipStream_t st);
@@ -269,7 +269,7 @@ extern "C" int vy_gemma_decoder_step(const vy_gemma_plan* p, const void* x, int6
           if ((rc = vy_rmsnorm_fwd(x1, d, L.ln_post, n, d, B, d, p->eps, 1.0f, p->dtype, stream))) return rc;
           gin = n;
         }
-        if ((rc = vy_dec_gemv1_gated(gin, L.wgu, act, ffn, d, prescaled, p->eps, hs))) {
+        if ((rc = vy_dec_gemv1_gated(gin, L.wgu, act, ffn, d, VY_ACT_GELU_TANH, prescaled, p->eps, hs))) {
           if (rc != VY_ERR_UNSUPPORTED) return rc;
           if ((rc = vy_gemv_gated(gin, d, L.wgu, d, prescaled ? VY_NORM_PRESCALED : nullptr, p->eps, act, ffn, B, ffn, d,
                                   VY_ACT_GELU_TANH, stream))) return rc;

@@ -251,3 +251,91 @@ class GemmaDecodePlan:
         _lib.call("vy_gemma_decoder_step", C.byref(self.plan), x.data_ptr(), int(pos), logits.data_ptr(), self.ldv,
                   torch.cuda.current_stream().cuda_stream)
         return logits[:, : self.vocab]
+
+
+# ---- decoders that mix layer kinds (models/hybrid.py) --------------------------------------------------
+
+class VyHybridLayer(C.Structure):
+    _fields_ = [(n, C.c_int32) for n in ("mixer", "heads", "dim", "vdim", "n_in", "ff", "q_rank", "q_rank_p", "kv_rank",
+                                         "kv_rank_p", "cap", "mix_n")] + [("scale", C.c_float)] + \
+               [(n, C.c_void_p) for n in ("norm1", "norm1b", "norm2", "norm2b", "w_in", "w_o", "w_gu", "w_down", "q_norm",
+                                          "c_norm", "w_uq", "w_ukt", "w_uv", "cache")] + \
+               [("c_ss", C.c_int64), ("c_st", C.c_int64)] + \
+               [(n, C.c_void_p) for n in ("state", "decay_pow", "mix_norm")]
+
+
+class VyHybridPlan(C.Structure):
+    _fields_ = [(n, C.c_int32) for n in ("num_layers", "B", "d", "dp", "vocab", "dtype", "rms", "act")] + \
+               [("eps", C.c_float), ("layers", C.POINTER(VyHybridLayer))] + \
+               [(n, C.c_void_p) for n in ("embed", "head", "final_norm", "err", "ws")] + [("ws_bytes", C.c_int64)]
+
+
+MIX_LATENT, MIX_DECAY = 0, 1
+
+
+class HybridDecodePlan:
+    """vy_hybrid_plan of a models.hybrid.HybridDecoderModel over a SlotCache, for batches of `batch` sequences."""
+
+    def __init__(self, model, cache, batch: int):
+        lib = _lib.load()
+        self.keep: list = []
+        arr = (VyHybridLayer * len(model.layers))()
+        acts = set()
+        for i, layer in enumerate(model.layers):
+            m, L = layer.mixer, arr[i]
+            n, p = layer.packed(), m.packed()
+            self.keep += [n, p]
+            L.heads, L.dim, L.vdim = m.heads, (m.dim + 7) // 8 * 8, (m.vdim + 7) // 8 * 8
+            L.w_in, L.n_in, L.w_o = _ptr(p.w_in), p.w_in.shape[0], _ptr(p.w_o)
+            L.norm1, L.norm1b = _ptr(n.norm1), _ptr(n.norm1b)
+            buf = cache.buffers[i]
+            if m.kind == "latent":
+                L.mixer, L.scale = MIX_LATENT, m.scale
+                L.q_rank, L.q_rank_p, L.kv_rank, L.kv_rank_p = m.q_rank, p.q_norm.numel(), m.kv_rank, p.c_norm.numel()
+                L.q_norm, L.c_norm = _ptr(p.q_norm), _ptr(p.c_norm)
+                L.w_uq, L.w_ukt, L.w_uv = _ptr(p.w_uq), _ptr(p.w_ukt), _ptr(p.w_uv)
+                L.cache, L.c_ss, L.c_st, L.cap = buf.data_ptr(), buf.stride(0), buf.stride(1), buf.shape[1]
+            else:
+                L.mixer, L.state, L.decay_pow = MIX_DECAY, buf.data_ptr(), _ptr(p.decay_pow)
+                L.mix_norm, L.mix_n = _ptr(p.norm), m.heads * m.vdim
+            if layer.mlp is not None:
+                f = layer.mlp.packed()
+                self.keep.append(f)
+                L.norm2, L.norm2b, L.w_gu, L.w_down, L.ff = _ptr(n.norm2), _ptr(n.norm2b), _ptr(f.w_gu), _ptr(f.w_down), f.w_down.shape[1]
+                acts.add(layer.mlp.act)
+        if len(acts) > 1:
+            raise ValueError("the decode step takes one MLP activation")
+        t = model.packed()
+        self.keep.append(t)
+        self.layers = arr
+        p = VyHybridPlan()
+        p.num_layers, p.B, p.d, p.dp, p.vocab = len(model.layers), batch, model.width, t.embed.shape[1], model.vocab
+        p.dtype, p.rms, p.act, p.eps = _lib.dtype_code(model.dtype), int(model.rms), acts.pop() if acts else _lib.ACT_NONE, model.eps
+        p.layers = C.cast(arr, C.POINTER(VyHybridLayer))
+        p.embed, p.head, p.final_norm = _ptr(t.embed), _ptr(t.head), _ptr(t.final_norm)
+        nbytes = lib.vy_hybrid_ws_bytes(C.byref(p))
+        self.ws = torch.empty(nbytes, dtype=torch.uint8, device=model.device)
+        p.ws, p.ws_bytes = self.ws.data_ptr(), nbytes
+        self.plan, self.batch, self.cache, self.generation = p, batch, cache, cache.generation
+        self.vocab, self.ldv, self.dtype, self.device = model.vocab, (model.vocab + 7) // 8 * 8, model.dtype, model.device
+        self.weights = self._weights(model)
+
+    @staticmethod
+    def _weights(model):
+        return tuple((q.data_ptr(), q._version) for q in model.parameters())
+
+    def valid(self, model, cache) -> bool:
+        return self.cache is cache and self.generation == cache.generation and self.weights == self._weights(model)
+
+    def step(self, ids: torch.Tensor, batch) -> torch.Tensor:
+        """ids (B,) int64; batch: the cache's SlotBatch for one more token each -> logits (B, vocab) view."""
+        assert ids.shape == (self.batch,) and ids.dtype == torch.long and ids.is_contiguous() and ids.device == self.device
+        if batch.max_keys > self.cache.capacity:   # the kernels write the new row there
+            raise ValueError(f"{batch.max_keys} tokens exceed the cache capacity {self.cache.capacity}")
+        from .ops import _mid_ws
+        _mid_ws(self.batch)
+        logits = torch.empty((self.batch, self.ldv), dtype=self.dtype, device=self.device)
+        _lib.call("vy_hybrid_decoder_step", C.byref(self.plan), ids.data_ptr(), batch.slots.data_ptr(),
+                  self.cache.lengths.data_ptr(), int(batch.max_keys), logits.data_ptr(), self.ldv,
+                  torch.cuda.current_stream().cuda_stream)
+        return logits[:, : self.vocab]

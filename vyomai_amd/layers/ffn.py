@@ -11,7 +11,10 @@ from typing import Union
 import torch
 import torch.nn as nn
 
-from .._lib import ACT_GELU_ERF, ACT_GELU_TANH
+from .. import ops
+from .._lib import ACT_GELU_ERF, ACT_GELU_TANH, ACT_SILU
+from ..ops import up8
+from .packing import Packed, pad2
 
 # activations with a fused HIP epilogue; the reference's table (:7-15) also lists leaky_relu,
 # relu6, sigmoid, silu/swish, tanh, which no shipped model or test selects.
@@ -40,3 +43,28 @@ class FeedForward(nn.Module):
         return ffn_block(hidden_state, input_tensor, self.intermediate.weight, self.intermediate.bias,
                          self.out.weight, self.out.bias, self.layernorm.weight, self.layernorm.bias,
                          self.layernorm.eps, self.act, self.dropout.p, self.training)
+
+
+_GATED_ACT = {"silu": ACT_SILU, "gelu_tanh": ACT_GELU_TANH, "gelu": ACT_GELU_ERF}
+
+
+class GatedFeedForward(nn.Module):
+    """down(act(gate(x)) * up(x)), no biases: one packed [gate; up] product, the gated activation, one product."""
+
+    def __init__(self, width: int, inner: int, act: str = "silu") -> None:
+        super().__init__()
+        self.width, self.inner, self.act = width, inner, _GATED_ACT[act]
+        self.gate = nn.Linear(width, inner, bias=False)
+        self.up = nn.Linear(width, inner, bias=False)
+        self.down = nn.Linear(inner, width, bias=False)
+
+    def packed(self) -> Packed:
+        def build(p: Packed) -> None:
+            dp, ip = up8(self.width), up8(self.inner)
+            p.w_gu = torch.cat([pad2(self.gate.weight, ip, dp), pad2(self.up.weight, ip, dp)]).contiguous()
+            p.w_down = pad2(self.down.weight, dp, ip).contiguous()
+        return Packed.of(self, list(self.parameters()), build)
+
+    def forward(self, h: torch.Tensor) -> torch.Tensor:
+        p = self.packed()
+        return ops.linear(ops.gated_act(ops.linear(h, p.w_gu), self.act), p.w_down)

@@ -272,3 +272,115 @@ class StaticCacheOne:
 
     def get_max_length(self) -> Optional[int]:
         return None
+
+
+class SlotCache:
+    """Whole-model memory of sequences of DIFFERENT lengths, for decoders that mix layer kinds.
+
+    A sequence owns a slot while it lives (``allocate`` / ``free``); per layer a slot holds either cached rows
+    ("latent", width): a (slots, capacity, width) buffer, or a recurrent state ("state", shape): a (slots, *shape) fp32
+    buffer.  ``lengths`` (int32 on the device, one per slot) says how many tokens a slot holds: kernels place new rows
+    behind them, attend no further, and take the state of an empty slot as zero -- so nothing is cleared when a slot is
+    handed on.  The host keeps a mirror (``length``).  Slots and capacity grow by doubling.
+    """
+
+    def __init__(self, specs, dtype: torch.dtype, device, slots: int = 1, capacity: int = 64) -> None:
+        self.specs, self.dtype, self.device = list(specs), dtype, torch.device(device)
+        self.slots, self.capacity = max(1, slots), max(1, capacity)
+        self.buffers = [self._make(s, self.slots, self.capacity) for s in self.specs]
+        self.lengths = torch.zeros(self.slots, dtype=torch.int32, device=self.device)
+        self.length = [0] * self.slots
+        self._free = list(range(self.slots - 1, -1, -1))
+        self._tables = {}
+        self.generation = 0          # counts reallocations: whoever holds buffer addresses compares it
+
+    def _make(self, spec, slots: int, capacity: int) -> torch.Tensor:
+        kind, shape = spec
+        if kind == "latent":
+            return torch.zeros(slots, capacity, shape, dtype=self.dtype, device=self.device)
+        if kind == "state":
+            return torch.zeros(slots, *shape, dtype=torch.float32, device=self.device)
+        raise ValueError(f"cache kind {kind!r}")
+
+    def _regrow(self, slots: int, capacity: int) -> None:
+        for i, spec in enumerate(self.specs):
+            if spec[0] == "state" and slots == self.slots:
+                continue
+            old, new = self.buffers[i], self._make(spec, slots, capacity)
+            if spec[0] == "latent":
+                new[: old.shape[0], : old.shape[1]] = old
+            else:
+                new[: old.shape[0]] = old
+            self.buffers[i] = new
+        if slots != self.slots:
+            lengths = torch.zeros(slots, dtype=torch.int32, device=self.device)
+            lengths[: self.slots] = self.lengths
+            self.lengths = lengths
+            self.length += [0] * (slots - self.slots)
+            self._free = list(range(slots - 1, self.slots - 1, -1)) + self._free
+        self.slots, self.capacity = slots, capacity
+        self.generation += 1
+
+    # ---- slots -----------------------------------------------------------------------------
+    def allocate(self, n: int = 1) -> List[int]:
+        if n > len(self._free):
+            self._regrow(max(2 * self.slots, self.slots + n - len(self._free)), self.capacity)
+        got = [self._free.pop() for _ in range(n)]
+        if n:
+            self.lengths[self.table(got).long()] = 0
+        for s in got:
+            self.length[s] = 0
+        return got
+
+    def free(self, slots) -> None:
+        for s in slots:
+            if s in self._free or not 0 <= s < self.slots:
+                raise ValueError(f"slot {s} is not in use")
+            self._free.append(s)
+
+    @property
+    def free_slots(self) -> int:
+        return len(self._free)
+
+    def table(self, slots) -> torch.Tensor:
+        """Device int32 tensor of a slot list (kept: a batch decodes with the same list step after step)."""
+        key = tuple(slots)
+        if key not in self._tables:
+            if len(self._tables) > 64:
+                self._tables.clear()
+            self._tables[key] = torch.tensor(key, dtype=torch.int32, device=self.device)
+        return self._tables[key]
+
+    # ---- steps -----------------------------------------------------------------------------
+    def reserve(self, slots, counts) -> "SlotBatch":
+        """Room for counts[b] more tokens in slots[b] -> what a forward pass over them needs."""
+        if len(set(slots)) != len(slots):
+            raise ValueError("a sequence may appear once in a batch")
+        if min(counts) < 1:
+            raise ValueError("every sequence of a batch brings at least one token")
+        need = max(self.length[s] + c for s, c in zip(slots, counts))
+        if need > self.capacity:
+            self._regrow(self.slots, max(need, 2 * self.capacity))
+        return SlotBatch(self, slots, counts, need)
+
+    def advance(self, slots, counts, on_device: bool = True) -> None:
+        """The tokens of a step are in; on_device=False: the step's own kernels advanced ``lengths``."""
+        if on_device:
+            self.lengths[self.table(slots).long()] += torch.tensor(counts, dtype=torch.int32, device=self.device)
+        for s, c in zip(slots, counts):
+            self.length[s] += c
+
+
+class SlotBatch:
+    """One batch of a SlotCache during a forward pass over L tokens per sequence (shorter ones padded behind)."""
+
+    def __init__(self, cache: SlotCache, slots, counts, max_keys: int) -> None:
+        self.cache, self.max_keys = cache, max_keys
+        self.slots, self.start = cache.table(slots), cache.lengths
+        self.fresh = all(cache.length[s] == 0 for s in slots)
+        self.count = None if len(set(counts)) == 1 else torch.tensor(counts, dtype=torch.int32, device=cache.device)
+
+    def latents(self, layer: int) -> torch.Tensor:
+        return self.cache.buffers[layer]
+
+    states = latents

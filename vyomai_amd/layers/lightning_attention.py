@@ -1,0 +1,59 @@
+"""Lightning attention: linear attention with a constant decay per head,
+
+    S_t = decay S_(t-1) + k_t v_t^T ,   o_t = S_t^T q_t ,   q, k, v = silu of the projections,
+
+the concatenated heads RMS-normed together, multiplied by a sigmoid gate and projected.  The only memory of the past is
+the fp32 state S (one dk x dv matrix per head and sequence)."""
+from __future__ import annotations
+
+from typing import Sequence
+
+import torch
+import torch.nn as nn
+
+from .. import ops
+from .._lib import DECAY_CHUNK
+from ..ops import up8
+from .norms import WeightNorm
+from .packing import Packed, head_cols, head_rows, head_vec
+
+
+class LightningAttention(nn.Module):
+    kind = "decay"
+
+    def __init__(self, width: int, heads: int, dim: int, vdim: int, decay: Sequence[float], eps: float) -> None:
+        super().__init__()
+        if len(decay) != heads:
+            raise ValueError(f"{len(decay)} decays for {heads} heads")
+        self.width, self.heads, self.dim, self.vdim, self.eps = width, heads, dim, vdim, float(eps)
+        self.decay = tuple(float(d) for d in decay)
+        self.query = nn.Linear(width, heads * dim, bias=False)
+        self.key = nn.Linear(width, heads * dim, bias=False)
+        self.value = nn.Linear(width, heads * vdim, bias=False)
+        self.gate = nn.Linear(width, heads * vdim, bias=False)
+        self.norm = WeightNorm(heads * vdim, eps, "rms")
+        self.out = nn.Linear(heads * vdim, width, bias=False)
+
+    def cache_spec(self):
+        return ("state", (self.heads, up8(self.dim), up8(self.vdim)))
+
+    def packed(self) -> Packed:
+        def build(p: Packed) -> None:
+            H, dp = self.heads, up8(self.width)
+            p.w_in = torch.cat([head_rows(m.weight, H, dp)
+                                for m in (self.query, self.key, self.value, self.gate)]).contiguous()
+            p.norm = head_vec(self.norm.weight, H)
+            p.w_o = head_cols(self.out.weight, H, dp)
+            # powers of the decays in double precision, rounded once
+            t = torch.tensor([[d ** i for i in range(DECAY_CHUNK + 1)] for d in self.decay], dtype=torch.float64)
+            p.decay_pow = t.float().to(p.w_in.device)
+        return Packed.of(self, list(self.parameters()), build)
+
+    def forward(self, h: torch.Tensor, B: int, L: int, batch, layer: int) -> torch.Tensor:
+        p = self.packed()
+        H, dim, vdim = self.heads, up8(self.dim), up8(self.vdim)
+        rows = ops.linear(h, p.w_in)
+        o = ops.decay_attention(rows, H, dim, vdim, batch.states(layer), p.decay_pow, B, L, start=batch.start,
+                                slots=batch.slots, count=batch.count)
+        o = ops.rmsnorm_gate(o, p.norm, H * self.vdim, rows[:, H * (2 * dim + vdim):], self.eps)
+        return ops.linear(o, p.w_o)

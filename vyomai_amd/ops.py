@@ -630,3 +630,135 @@ def gated_act(gate_up: Tensor, act: int) -> Tensor:
     call("vy_gated_act_fwd", g2.data_ptr(), g2.stride(0), out.data_ptr(), out.stride(0), M, I, act,
          dtype_code(gate_up.dtype), _stream())
     return out.view(*gate_up.shape[:-1], I)
+
+
+# ------------------------------------------------------------------------------------------
+# decoders with an fp32 residual stream: norms, latent attention, decayed linear attention
+# ------------------------------------------------------------------------------------------
+
+
+def up8(n: int) -> int:
+    """Padded width of a row: the next multiple of 8 elements."""
+    return (n + 7) // 8 * 8
+
+
+def residual_norm(x: Tensor, width: int, *, y: Optional[Tensor] = None, post: Optional[Tensor] = None,
+                  pre: Optional[Tensor] = None, eps: float = 1e-5, rms: bool = False, table: Optional[Tensor] = None,
+                  ids: Optional[Tensor] = None, dtype: Optional[torch.dtype] = None,
+                  err_flag: Optional[Tensor] = None) -> Optional[Tensor]:
+    """x (M, padded width) fp32, in place: x += norm(y) * post (post None: x += y), or x = table[ids]; returns
+    norm(x) * pre in `dtype` (None without pre).  (vy_residual_norm)"""
+    _need_gpu(x, y, post, pre, table, ids)
+    assert x.dtype == torch.float32 and x.dim() == 2 and x.stride(1) == 1
+    for w in (post, pre):
+        assert w is None or (w.dtype == torch.float32 and w.numel() == x.shape[1] and w.is_contiguous())
+    M, NP = x.shape
+    src = y if y is not None else table
+    dt = dtype or src.dtype
+    assert src is None or (src.dtype == dt and src.shape[-1] == NP and src.stride(-1) == 1)
+    if y is not None:
+        y = _rows(y)
+        assert y.shape[0] == M
+    if ids is not None:
+        assert ids.dtype == torch.long and ids.is_contiguous() and ids.numel() == M and table is not None
+    h = torch.empty((M, NP), dtype=dt, device=x.device) if pre is not None else None
+    call("vy_residual_norm", x.data_ptr(), x.stride(0), _ptr(y), y.stride(0) if y is not None else 0, _ptr(table),
+         table.stride(0) if table is not None else 0, _ptr(ids), table.shape[0] if table is not None else 0, _ptr(err_flag),
+         _ptr(post), float(eps), _ptr(pre), float(eps), _ptr(h), NP, M, int(width), NP, int(rms), dtype_code(dt), _stream())
+    return h
+
+
+def _slot_args(slots: Optional[Tensor], start: Optional[Tensor], count: Optional[Tensor], B: int) -> None:
+    for t in (slots, start, count):
+        assert t is None or (t.dtype == torch.int32 and t.is_contiguous())
+    assert slots is None or slots.numel() == B
+    assert count is None or count.numel() == B
+
+
+def latent_norm(p: Tensor, w_q: Tensor, n_q: int, w_c: Tensor, n_c: int, B: int, L: int, eps: float, *,
+                cache: Optional[Tensor] = None, slots: Optional[Tensor] = None, start: Optional[Tensor] = None,
+                count: Optional[Tensor] = None, want_c: bool = True) -> Tuple[Tensor, Optional[Tensor]]:
+    """RMS norms of the two latents at the front of the packed rows p (B*L, .); the second one also goes to
+    cache[slot, start + l].  (vy_latent_norm)"""
+    _need_gpu(p, w_q, w_c, cache, slots, start, count)
+    _slot_args(slots, start, count, B)
+    npq, npc = w_q.numel(), w_c.numel()
+    assert p.shape[0] == B * L and p.stride(1) == 1 and p.shape[1] >= npq + npc
+    q = torch.empty((B * L, npq), dtype=p.dtype, device=p.device)
+    c = torch.empty((B * L, npc), dtype=p.dtype, device=p.device) if want_c else None
+    if cache is not None:
+        assert cache.dtype == p.dtype and cache.shape[2] == npc and cache.stride(2) == 1 and start is not None
+    call("vy_latent_norm", p.data_ptr(), p.stride(0), w_q.data_ptr(), q.data_ptr(), npq, int(n_q), npq, w_c.data_ptr(), _ptr(c),
+         npc, int(n_c), npc, _ptr(cache), cache.stride(0) if cache is not None else 0,
+         cache.stride(1) if cache is not None else 0, cache.shape[1] if cache is not None else 0, _ptr(slots), _ptr(start),
+         _ptr(count), B, L, float(eps), dtype_code(p.dtype), _stream())
+    return q, c
+
+
+def rmsnorm_gate(x: Tensor, w: Tensor, width: int, gate: Tensor, eps: float) -> Tensor:
+    """RMSNorm(x) * w * sigmoid(gate) over `width` of the padded columns.  (vy_rmsnorm_gate)"""
+    _need_gpu(x, w, gate)
+    M, NP = x.shape
+    assert gate.shape == x.shape and x.stride(1) == 1 and gate.stride(1) == 1 and w.numel() == NP and w.dtype == torch.float32
+    y = torch.empty((M, NP), dtype=x.dtype, device=x.device)
+    call("vy_rmsnorm_gate", x.data_ptr(), x.stride(0), w.data_ptr(), gate.data_ptr(), gate.stride(0), y.data_ptr(), NP, M,
+         int(width), NP, float(eps), dtype_code(x.dtype), _stream())
+    return y
+
+
+def attention_ex(q: Tensor, k: Tensor, v: Tensor, scale: float, *, gate: Optional[Tensor] = None,
+                 start: Optional[Tensor] = None, slots: Optional[Tensor] = None) -> Tensor:
+    """Causal attention with a value width of its own: q (B,h,L,dh), k (B,hk,S,dh), v (B,hk,S,dv) -> (B, L, h*dv); `start`
+    (int32, per slot) keys precede the queries; gate (B, L, h*dv): out *= sigmoid(gate).  (vy_attn_fwd_ex)"""
+    _need_gpu(q, k, v, gate, start, slots)
+    B, h, L, dh = q.shape
+    hk, S, dv = k.shape[1], k.shape[2], v.shape[3]
+    _slot_args(slots, start, None, B)
+    assert q.stride(3) == 1 and k.stride(3) == 1 and v.stride(3) == 1 and k.shape[3] == dh and v.shape[:3] == k.shape[:3]
+    out = torch.empty((B, L, h * dv), dtype=q.dtype, device=q.device)
+    assert gate is None or (gate.shape == out.shape and gate.stride(2) == 1)
+    call("vy_attn_fwd_ex", q.data_ptr(), q.stride(0), q.stride(1), q.stride(2), k.data_ptr(), k.stride(0), k.stride(1),
+         k.stride(2), v.data_ptr(), v.stride(0), v.stride(1), v.stride(2), out.data_ptr(), out.stride(0), out.stride(1),
+         _ptr(gate), gate.stride(0) if gate is not None else 0, gate.stride(1) if gate is not None else 0, _ptr(start),
+         _ptr(slots), B, h, hk, L, S, dh, dv, float(scale), dtype_code(q.dtype), _stream())
+    return out
+
+
+def latent_decode(q: Tensor, wukt: Tensor, wuv: Tensor, cache: Tensor, start: Tensor, max_keys: int, scale: float, *,
+                  slots: Optional[Tensor] = None, gate: Optional[Tensor] = None) -> Tensor:
+    """One query token per sequence against a latent cache (slots, cap, R); q (B, h*dh), wukt (h, R, dh), wuv (h, dv, R);
+    keys 0 .. start[slot] are attended (the newest row is in the cache already).  (vy_latent_decode)"""
+    _need_gpu(q, wukt, wuv, cache, start, slots, gate)
+    B = q.shape[0]
+    h, R, dh = wukt.shape
+    dv = wuv.shape[1]
+    _slot_args(slots, start, None, B)
+    assert q.shape == (B, h * dh) and q.stride(1) == 1 and wuv.shape == (h, dv, R) and cache.shape[2] == R
+    assert wukt.is_contiguous() and wuv.is_contiguous() and cache.stride(2) == 1 and 0 < max_keys <= cache.shape[1]
+    out = torch.empty((B, h * dv), dtype=q.dtype, device=q.device)
+    nws = _lib.load().vy_latent_decode_ws_bytes(B, h, R)
+    ws = torch.empty(nws, dtype=torch.uint8, device=q.device)
+    call("vy_latent_decode", q.data_ptr(), q.stride(0), wukt.data_ptr(), wuv.data_ptr(), cache.data_ptr(), cache.stride(0),
+         cache.stride(1), _ptr(slots), start.data_ptr(), int(max_keys), out.data_ptr(), out.stride(0), _ptr(gate),
+         gate.stride(0) if gate is not None else 0, B, h, dh, dv, R, float(scale), ws.data_ptr(), nws, dtype_code(q.dtype),
+         _stream())
+    return out
+
+
+def decay_attention(p: Tensor, heads: int, dk: int, dv: int, state: Tensor, decay_pow: Tensor, B: int, L: int, *,
+                    start: Tensor, slots: Optional[Tensor] = None, count: Optional[Tensor] = None,
+                    silu: bool = True) -> Tensor:
+    """Decayed linear attention over packed rows p = [q (heads*dk) | k (heads*dk) | v (heads*dv) | ...] of B sequences of L
+    tokens; state (slots, heads, dk, dv) fp32 is read (zero where start[slot] == 0) and updated.  (vy_decay_attn)"""
+    _need_gpu(p, state, decay_pow, start, slots, count)
+    _slot_args(slots, start, count, B)
+    assert p.shape[0] == B * L and p.stride(1) == 1 and p.shape[1] >= heads * (2 * dk + dv)
+    assert state.dtype == torch.float32 and state.is_contiguous() and state.shape[1:] == (heads, dk, dv)
+    assert decay_pow.dtype == torch.float32 and decay_pow.shape == (heads, _lib.DECAY_CHUNK + 1) and decay_pow.is_contiguous()
+    out = torch.empty((B * L, heads * dv), dtype=p.dtype, device=p.device)
+    nws = _lib.load().vy_decay_attn_ws_bytes(B, L, heads, dk, dv, dtype_code(p.dtype))
+    ws = torch.empty(nws, dtype=torch.uint8, device=p.device) if nws else None
+    call("vy_decay_attn", p.data_ptr(), p.stride(0), 0, heads * dk, 2 * heads * dk, state.data_ptr(), decay_pow.data_ptr(),
+         _ptr(slots), start.data_ptr(), _ptr(count), out.data_ptr(), out.stride(0), B, L, heads, dk, dv, int(silu), _ptr(ws),
+         nws, dtype_code(p.dtype), _stream())
+    return out
