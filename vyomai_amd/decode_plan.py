@@ -318,14 +318,15 @@ class HybridDecodePlan:
         p.ws, p.ws_bytes = self.ws.data_ptr(), nbytes
         self.plan, self.batch, self.cache, self.generation = p, batch, cache, cache.generation
         self.vocab, self.ldv, self.dtype, self.device = model.vocab, (model.vocab + 7) // 8 * 8, model.dtype, model.device
-        self.weights = self._weights(model)
+        self.params = list(model.parameters())
+        self.versions = self._versions()
 
-    @staticmethod
-    def _weights(model):
-        return tuple((q.data_ptr(), q._version) for q in model.parameters())
+    def _versions(self):
+        return sum(p._version for p in self.params)
 
-    def valid(self, model, cache) -> bool:
-        return self.cache is cache and self.generation == cache.generation and self.weights == self._weights(model)
+    def valid(self, cache) -> bool:
+        """Same buffers, and no weight written since (weights REPLACED are noticed by the next prefill, which drops plans)."""
+        return self.cache is cache and self.generation == cache.generation and self.versions == self._versions()
 
     def step(self, ids: torch.Tensor, batch) -> torch.Tensor:
         """ids (B,) int64; batch: the cache's SlotBatch for one more token each -> logits (B, vocab) view."""
