@@ -17,7 +17,6 @@ namespace {
 
 constexpr float LOG2E = 1.4426950408889634f;
 constexpr int MAX_SPLIT = 64;      // slices of the key range
-constexpr int KEYS_PER_TILE = 32;  // keys a wave takes at a time
 
 struct LatentArgs {
   const void* q; int64_t ldq;
@@ -26,7 +25,7 @@ struct LatentArgs {
   const int* slots; const int* start;
   void* out; int64_t ldo;
   const void* gate; int64_t ldg;
-  int B, h, dh, dv, R, nsplit;
+  int B, h, dh, dv, R, nsplit, seqs;
   float c;                         // scale * log2(e)
   // workspace
   float* qf;                       // generic: latent queries [B][h][R]
@@ -88,21 +87,34 @@ __global__ __launch_bounds__(256) void latent_query_kernel(LatentArgs p) {
   }
 }
 
-// grid (slices, head groups of 16, B); 4 waves, each walking its own 32-key tiles of the slice through a private LDS tile.
-// Swapped products as in attn_fwd_gen_kernel: S^T = c q~^T puts ONE head per lane column and four consecutive keys per
-// lane group, P^T is the B operand of U^T = c^T P^T as it sits, and the same LDS tile serves both products (row reads
-// for the scores, transposing reads for the mean).
+// asm forms of the score exchange: while LDS-DMA is in flight hipcc drains it (vmcnt(0)) in front of every LDS access it can
+// see; these are retired by counted / explicit waits instead (vy_common.h)
+__device__ __forceinline__ void lds_write4(unsigned addr, f32x4 v) {
+  asm volatile("ds_write_b128 %0, %1" ::"v"(addr), "v"(v) : "memory");
+}
+__device__ __forceinline__ bf16x8 lds_read16(unsigned addr) { return vy_lds_read128_off<0>(addr); }
+
+// grid (slices, head groups of 16, B); 4 waves share tiles of KT keys that LDS-DMA brings through a ring of NS buffers.
+//   scores  S^T = c q~^T, swapped as in attn_fwd_gen_kernel: one head per lane column, four consecutive keys per lane
+//           group.  A wave takes one block of 16 keys (KT = 64) or half of the contraction of one block (KT = 32); the
+//           scores are exchanged through LDS, and every wave then holds the same running maximum and sum;
+//   mean    U^T += c^T P^T: a wave owns RP / 4 of the latent columns, so nothing is combined across waves at the end.  The
+//           same LDS tile serves both products: row reads for the scores, transposing reads for the mean.
+// Rows are XOR-swizzled in 16-byte chunks with the low bits of the key index (applied to the DMA's source address).
 template <int RP>
-__global__ __launch_bounds__(256, 1) void latent_scan_kernel(LatentArgs p) {
-  constexpr int KT = KEYS_PER_TILE;
-  constexpr int PITCH = (RP + 8) * 2;
-  constexpr int TILE = KT * PITCH;
-  constexpr int KS = RP / 32, ND = RP / 16;
+__global__ __launch_bounds__(256) void latent_scan_kernel(LatentArgs p) {
+  constexpr int KT = RP >= 512 ? 32 : 64;     // keys per tile
+  constexpr int NS = RP >= 512 ? 4 : RP >= 256 ? 2 : 3;
+  constexpr int RB = RP * 2;                  // bytes per row
+  constexpr int TILE = KT * RB;
+  constexpr int NP = TILE / 1024 / 4;         // 1-KiB pieces per wave and tile
   constexpr int CPR = RP / 8;                 // 16-byte chunks per row
-  constexpr int NCH = KT * CPR / 64;          // chunks per lane
-  // at the full width the low halves of the queries sit in LDS (one copy for the four waves) instead of 64 registers
-  constexpr bool QLDS = RP >= 512;
-  __shared__ __attribute__((aligned(16))) char smem[4 * TILE + 4 * 16 * 8 + (QLDS ? 16 * PITCH : 0)];
+  constexpr int SWZ = CPR < 16 ? CPR - 1 : 15;
+  constexpr int KH = KT == 32 ? 2 : 1;        // waves per key block
+  constexpr int KS = RP / 32 / KH;            // k-steps of a wave
+  constexpr int ND = RP / 64;                 // 16-wide latent blocks of a wave
+  constexpr int SP = (KT + 4) * 4;            // bytes per score row (head)
+  __shared__ __attribute__((aligned(16))) char smem[NS * TILE + KH * 16 * SP];
   const int lane = threadIdx.x & 63;
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int r16 = lane & 15, kq = lane >> 4;
@@ -112,73 +124,122 @@ __global__ __launch_bounds__(256, 1) void latent_scan_kernel(LatentArgs p) {
   const int n = row_keys(p, b, slot);
   const int tiles = (n + KT - 1) / KT;
   const int tps = (tiles + p.nsplit - 1) / p.nsplit;
-  const int t0 = split * tps, t1 = min(tiles, t0 + tps);
-  const bf16* C = (const bf16*)p.cache + (int64_t)slot * p.c_ss;
-  const bf16x8 zero8 = {};
-  char* tile = smem + wave * TILE;
-  float* red = reinterpret_cast<float*>(smem + 4 * TILE);   // [wave][16 heads][m, l]
+  const int t0 = split * tps, nt = max(0, min(tiles, t0 + tps) - t0);
+  const bf16* Cs = (const bf16*)p.cache + (int64_t)slot * p.c_ss;
 
-  char* qlt = smem + 4 * TILE + 4 * 16 * 8;
-  bf16x8 qh[KS], ql[QLDS ? 1 : KS];
+  int ld_row[NP], ld_col[NP];                 // row and source column (< 0: padding) of this lane's 16 bytes of a piece
+#pragma unroll
+  for (int i = 0; i < NP; ++i) {
+    const int P = (wave * NP + i) * 1024 + lane * 16;
+    ld_row[i] = P / RB;
+    const int ch = ((P % RB) >> 4) ^ (ld_row[i] & SWZ);
+    ld_col[i] = ch * 8 < p.R ? ch * 8 : -1;
+  }
+  auto stage = [&](int t) {
+    const int k0 = (t0 + t) * KT;
+#pragma unroll
+    for (int i = 0; i < NP; ++i) {
+      const int kj = min(k0 + ld_row[i], n - 1);
+      const void* src = ld_col[i] < 0 ? (const void*)vy_zero16 : (const void*)(Cs + (int64_t)kj * p.c_st + ld_col[i]);
+      __builtin_amdgcn_global_load_lds((const VY_GLOBAL void*)src,
+                                       (VY_LDS void*)(smem + (t % NS) * TILE + (wave * NP + i) * 1024), 16, 0, 0);
+    }
+  };
+#pragma unroll
+  for (int t = 0; t < NS - 1; ++t)
+    if (t < nt) stage(t);
+
+  const int kblk = KH == 2 ? wave & 1 : wave, khalf = KH == 2 ? wave >> 1 : 0;
+  bf16x8 qh[KS], ql[KS];
   const int64_t qo = ((int64_t)b * p.h + (head < p.h ? head : 0)) * p.R;
+  const bf16x8 zero8 = {};
 #pragma unroll
   for (int ks = 0; ks < KS; ++ks) {
-    const int k = 32 * ks + 8 * kq;
+    const int k = 32 * (khalf * KS + ks) + 8 * kq;
     const bool ok = k < p.R && head < p.h;
     qh[ks] = ok ? *reinterpret_cast<const bf16x8*>(p.qhi + qo + k) : zero8;
-    const bf16x8 low = ok ? *reinterpret_cast<const bf16x8*>(p.qlo + qo + k) : zero8;
-    if constexpr (!QLDS) ql[ks] = low;
-    else if (wave == (ks & 3)) *reinterpret_cast<bf16x8*>(qlt + r16 * PITCH + k * 2) = low;
+    ql[ks] = ok ? *reinterpret_cast<const bf16x8*>(p.qlo + qo + k) : zero8;
   }
-  if constexpr (QLDS) __syncthreads();
+  // (retire the ordinary loads before the loop: a wait for them inside it would drain the ring)
+#pragma unroll
+  for (int ks = 0; ks < KS; ++ks) { asm volatile("" ::"v"(qh[ks])); asm volatile("" ::"v"(ql[ks])); }
+
+  const unsigned base = vy_lds_addr(smem), sbase = base + NS * TILE;
+  const int krow = 16 * kblk + r16;
+  unsigned ka[KS];                            // score fragments: key row krow, chunk 4 ks + kq
+#pragma unroll
+  for (int ks = 0; ks < KS; ++ks) ka[ks] = base + krow * RB + (((4 * (khalf * KS + ks) + kq) ^ (krow & SWZ)) << 4);
+  const int vrow = 4 * kq + (r16 >> 2);       // mean fragments: rows vrow and vrow + 16 (same swizzle), 8 bytes per lane
+  unsigned va[ND];
+#pragma unroll
+  for (int i = 0; i < ND; ++i) {
+    const int ch = 2 * (wave * ND + i) + ((r16 & 3) >> 1);
+    va[i] = base + vrow * RB + ((ch ^ (vrow & SWZ)) << 4) + (r16 & 1) * 8;
+  }
+  const unsigned sw_addr = sbase + khalf * 16 * SP + r16 * SP + (16 * kblk + 4 * kq) * 4;
+  const unsigned sr_addr = sbase + r16 * SP + 4 * kq * 4;
+
   f32x4 o[ND];
 #pragma unroll
   for (int i = 0; i < ND; ++i) o[i] = f32x4{0.f, 0.f, 0.f, 0.f};
   float m_run = -FLT_MAX, l_run = 0.f;
 
-  bf16x8 reg[NCH];
-  auto fetch = [&](int t) {
+  for (int t = 0; t < nt; ++t) {
+    const int younger = min(NS - 2, nt - 1 - t);      // tiles that may stay in flight
+    if (NS >= 4 && younger >= 2) asm volatile("s_waitcnt vmcnt(%0)" ::"n"(2 * NP) : "memory");
+    else if (NS >= 3 && younger >= 1) asm volatile("s_waitcnt vmcnt(%0)" ::"n"(NP) : "memory");
+    else asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+    __builtin_amdgcn_s_barrier();
+    asm volatile("" ::: "memory");
+    if (t + NS - 1 < nt) stage(t + NS - 1);           // into the buffer tile t - 1 was read from
+    const unsigned buf = (t % NS) * TILE;
+    f32x4 sh = {0.f, 0.f, 0.f, 0.f}, sl = {0.f, 0.f, 0.f, 0.f};
+    bf16x8 kf[KS];
 #pragma unroll
-    for (int i = 0; i < NCH; ++i) {
-      const int cidx = lane + 64 * i;
-      const int row = cidx / CPR, ch = cidx % CPR;
-      const int kj = min(t * KT + row, n - 1);
-      reg[i] = ch * 8 < p.R ? __builtin_nontemporal_load(reinterpret_cast<const bf16x8*>(C + (int64_t)kj * p.c_st + ch * 8)) : zero8;
-    }
-  };
-  const unsigned vtr = vy_lds_addr(tile) + (4 * kq + (r16 >> 2)) * PITCH + (4 * (r16 & 3)) * 2;
-  int t = t0 + wave;
-  if (t < t1) fetch(t);
-  for (; t < t1; t += 4) {
+    for (int ks = 0; ks < KS; ++ks) kf[ks] = lds_read16(ka[ks] + buf);
+    vy_static_for<KS>([&](auto i_c) {
+      constexpr int i = decltype(i_c)::value;
+      constexpr int left = KS - 1 - i;
+      if constexpr (left <= 15) asm volatile("s_waitcnt lgkmcnt(%0)" ::"n"(left) : "memory");
+      vy_tie(kf[i]);
+      sh = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[i], qh[i], sh, 0, 0, 0);
+      sl = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[i], ql[i], sl, 0, 0, 0);
+    });
+    lds_write4(sw_addr, sh + sl);
+    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+    __builtin_amdgcn_s_barrier();
+    asm volatile("" ::: "memory");
+    // scores of every key of the tile for this lane's head, in the key order of the transposed fragments
+    bf16x8 raw[KT / 16][KH];
 #pragma unroll
-    for (int i = 0; i < NCH; ++i) {
-      const int cidx = lane + 64 * i;
-      *reinterpret_cast<bf16x8*>(tile + (cidx / CPR) * PITCH + (cidx % CPR) * 16) = reg[i];
-    }
-    if (t + 4 < t1) fetch(t + 4);
-    f32x4 sc[2];
+    for (int g = 0; g < KT / 16; ++g)
 #pragma unroll
-    for (int blk = 0; blk < 2; ++blk) {
-      sc[blk] = f32x4{0.f, 0.f, 0.f, 0.f};
+      for (int hf = 0; hf < KH; ++hf) raw[g][hf] = lds_read16(sr_addr + hf * 16 * SP + g * 64);
+    bf16x8 vf[KT / 32][ND];
+    vy_static_for<KT / 32>([&](auto t_c) {
+      constexpr int tt = decltype(t_c)::value;
 #pragma unroll
-      for (int ks = 0; ks < KS; ++ks) {
-        const bf16x8 kf = *reinterpret_cast<const bf16x8*>(tile + (16 * blk + r16) * PITCH + (32 * ks + 8 * kq) * 2);
-        bf16x8 low;
-        if constexpr (QLDS) low = *reinterpret_cast<const bf16x8*>(qlt + r16 * PITCH + (32 * ks + 8 * kq) * 2);
-        else low = ql[ks];
-        sc[blk] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, low, sc[blk], 0, 0, 0);
-        sc[blk] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qh[ks], sc[blk], 0, 0, 0);
-      }
-    }
+      for (int i = 0; i < ND; ++i) vf[tt][i] = vy_lds_tr16_pair_off<32 * tt * RB, (32 * tt + 16) * RB>(va[i] + buf);
+    });
+    // (lgkmcnt has 4 bits: the scores are the oldest reads, the transposed fragments behind them may stay in flight)
+    constexpr int behind = 2 * ND * (KT / 32);
+    if constexpr (behind <= 15) asm volatile("s_waitcnt lgkmcnt(%0)" ::"n"(behind) : "memory");
+    else asm volatile("s_waitcnt lgkmcnt(15)" ::: "memory");
+    float sc[KT / 16][4];
     float tmax = -INFINITY;
+    const int kbase = (t0 + t) * KT + 4 * kq;
 #pragma unroll
-    for (int blk = 0; blk < 2; ++blk)
+    for (int g = 0; g < KT / 16; ++g) {
+#pragma unroll
+      for (int hf = 0; hf < KH; ++hf) vy_tie(raw[g][hf]);
+      f32x4 v = __builtin_bit_cast(f32x4, raw[g][0]);
+      if constexpr (KH == 2) v += __builtin_bit_cast(f32x4, raw[g][KH - 1]);
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
-        const bool vis = t * KT + 16 * blk + 4 * kq + r < n;
-        sc[blk][r] = vis ? sc[blk][r] * p.c : -INFINITY;
-        tmax = fmaxf(tmax, sc[blk][r]);
+        sc[g][r] = kbase + 16 * g + r < n ? v[r] * p.c : -INFINITY;
+        tmax = fmaxf(tmax, sc[g][r]);
       }
+    }
     const float m_new = fmaxf(m_run, quad_max(tmax));
     if (__any(m_new > m_run)) {
       const float alpha = __builtin_amdgcn_exp2f(m_run - m_new);
@@ -189,56 +250,33 @@ __global__ __launch_bounds__(256, 1) void latent_scan_kernel(LatentArgs p) {
 #pragma unroll
         for (int r = 0; r < 4; ++r) o[i][r] *= alpha;
     }
-    bf16x8 pf;
+    bf16x8 pf[KT / 32];
 #pragma unroll
-    for (int blk = 0; blk < 2; ++blk)
+    for (int g = 0; g < KT / 16; ++g)
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
-        const float e = __builtin_amdgcn_exp2f(sc[blk][r] - m_run);
+        const float e = __builtin_amdgcn_exp2f(sc[g][r] - m_run);
         l_run += e;
-        pf[4 * blk + r] = (bf16)e;
+        pf[g >> 1][4 * (g & 1) + r] = (bf16)e;
       }
-    vy_static_for<ND / 4>([&](auto g_c) {
-      constexpr int g = decltype(g_c)::value;
-      union { struct { s16x4 a, b; } s; bf16x8 v; } u[4];
-      vy_static_for<4>([&](auto i_c) {
-        constexpr int i = decltype(i_c)::value;
-        u[i].s.a = vy_lds_tr16_off<(4 * g + i) * 32>(vtr);
-        u[i].s.b = vy_lds_tr16_off<(4 * g + i) * 32>(vtr + 16 * PITCH);
-      });
-      asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
 #pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        vy_tie(u[i].v);
-        o[4 * g + i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(u[i].v, pf, o[4 * g + i], 0, 0, 0);
+    for (int tt = 0; tt < KT / 32; ++tt)
+#pragma unroll
+      for (int i = 0; i < ND; ++i) {
+        vy_tie(vf[tt][i]);
+        o[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[tt][i], pf[tt], o[i], 0, 0, 0);
       }
-    });
   }
-  // the four waves' partial sums: each leaves [16 heads][RP] fp32 in its own tile
-  const float l_tot = quad_sum(l_run);
-  if (kq == 0) { red[(wave * 16 + r16) * 2] = m_run; red[(wave * 16 + r16) * 2 + 1] = l_tot; }
-  float* mine = reinterpret_cast<float*>(tile);
+  if (head < p.h) {
+    const int64_t o_ = ((int64_t)b * p.h + head) * p.nsplit + split;
+    const float l = quad_sum(l_run);
+    if (wave == 0 && kq == 0) { p.part_ml[o_ * 2] = m_run; p.part_ml[o_ * 2 + 1] = l; }
 #pragma unroll
-  for (int i = 0; i < ND; ++i) *reinterpret_cast<f32x4*>(mine + r16 * RP + 16 * i + 4 * kq) = o[i];
-  __syncthreads();
-  for (int idx = threadIdx.x; idx < 16 * (RP / 4); idx += 256) {
-    const int hr = idx / (RP / 4), col = (idx % (RP / 4)) * 4;
-    const int hd = (int)blockIdx.y * 16 + hr;
-    if (hd >= p.h || col >= p.R) continue;
-    float M = -FLT_MAX;
-#pragma unroll
-    for (int w = 0; w < 4; ++w) M = fmaxf(M, red[(w * 16 + hr) * 2]);
-    f32x4 s = {0.f, 0.f, 0.f, 0.f};
-    float l = 0.f;
-#pragma unroll
-    for (int w = 0; w < 4; ++w) {
-      const float a = __builtin_amdgcn_exp2f(red[(w * 16 + hr) * 2] - M);
-      l += a * red[(w * 16 + hr) * 2 + 1];
-      s += a * *reinterpret_cast<const f32x4*>(reinterpret_cast<const float*>(smem + w * TILE) + hr * RP + col);
+    for (int i = 0; i < ND; ++i) {
+      const int col = 16 * (wave * ND + i) + 4 * kq;
+      if (col < p.R) *reinterpret_cast<f32x4*>(p.part_o + o_ * p.R + col) = o[i];
     }
-    const int64_t o_ = ((int64_t)b * p.h + hd) * p.nsplit + split;
-    *reinterpret_cast<f32x4*>(p.part_o + o_ * p.R + col) = s;
-    if (col == 0) { p.part_ml[o_ * 2] = M; p.part_ml[o_ * 2 + 1] = l; }
   }
 }
 
@@ -253,35 +291,48 @@ __device__ __forceinline__ void slice_weights(const LatentArgs& p, int b, int he
   if (lane < p.nsplit) w[lane] = e / L;
 }
 
-// out[b][h][n] = (W_uv,h u_bh)_n * sigmoid(gate): workgroup = 64 value columns of one head x 16 sequences; the mean latents
-// are added up from the slices into LDS first
+// out[b][h][n] = (W_uv,h u_bh)_n * sigmoid(gate): workgroup = 64 value columns of one head x p.seqs (<= 16) sequences; the
+// mean latents are added up from the slices into LDS first (few sequences: the slices are shared out over the threads)
 __global__ __launch_bounds__(256) void latent_value_kernel(LatentArgs p) {
   extern __shared__ __attribute__((aligned(16))) char dyn[];
   const int RP = (p.R + 31) / 32 * 32, PITCH = (RP + 8) * 2;
-  float* sw = reinterpret_cast<float*>(dyn);                       // [16][MAX_SPLIT]
-  char* xh = dyn + 16 * MAX_SPLIT * 4;
-  char* xl = xh + 16 * PITCH;
+  float* sw = reinterpret_cast<float*>(dyn);                       // [seqs][MAX_SPLIT]
+  f32x4* acc4 = reinterpret_cast<f32x4*>(dyn + p.seqs * MAX_SPLIT * 4);   // [256]
+  char* xh = dyn + p.seqs * MAX_SPLIT * 4 + 4096;
+  char* xl = xh + p.seqs * PITCH;
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int r16 = lane & 15, kq = lane >> 4;
-  const int head = blockIdx.y, b0 = (int)blockIdx.z * 16;
-  const int nb = min(16, p.B - b0);
+  const int head = blockIdx.y, b0 = (int)blockIdx.z * p.seqs;
+  const int nb = min(p.seqs, p.B - b0);
   const bf16x8 zero8 = {};
   for (int i = wave; i < nb; i += 4) slice_weights(p, b0 + i, head, sw + i * MAX_SPLIT, lane);
   __syncthreads();
-  const int q4 = RP / 4;
-  for (int idx = threadIdx.x; idx < nb * q4; idx += 256) {
-    const int i = idx / q4, col = (idx - i * q4) * 4;
+  const int q4 = RP / 4, items = nb * q4;
+  const int G = items >= 256 ? 1 : 256 / items;                    // groups of slices
+  for (int base = 0; base < items; base += 256) {
+    const int g = G > 1 ? (int)threadIdx.x / items : 0;
+    const int idx = base + (int)threadIdx.x - g * items;
+    const bool live = idx < items && g < G;
+    const int i = live ? idx / q4 : 0, col = (idx - i * q4) * 4;
     f32x4 s = {0.f, 0.f, 0.f, 0.f};
-    if (col < p.R) {
+    if (live && col < p.R) {
       const float* po = p.part_o + ((int64_t)(b0 + i) * p.h + head) * p.nsplit * p.R + col;
-#pragma unroll 4
-      for (int k = 0; k < p.nsplit; ++k) s += sw[i * MAX_SPLIT + k] * *reinterpret_cast<const f32x4*>(po + (int64_t)k * p.R);
+#pragma unroll 8
+      for (int k = g; k < p.nsplit; k += G) s += sw[i * MAX_SPLIT + k] * *reinterpret_cast<const f32x4*>(po + (int64_t)k * p.R);
     }
-    bf16x4 hi, lo;
+    if (G > 1) {   // (workgroup-uniform; then one pass covers every item)
+      acc4[threadIdx.x] = s;
+      __syncthreads();
+      if (live && g == 0)
+        for (int k = 1; k < G; ++k) s += acc4[k * items + idx];
+    }
+    if (live && g == 0) {
+      bf16x4 hi, lo;
 #pragma unroll
-    for (int e = 0; e < 4; ++e) { bf16 a, c; split_bf16(s[e], a, c); hi[e] = a; lo[e] = c; }
-    *reinterpret_cast<bf16x4*>(xh + i * PITCH + col * 2) = hi;
-    *reinterpret_cast<bf16x4*>(xl + i * PITCH + col * 2) = lo;
+      for (int e = 0; e < 4; ++e) { bf16 a, c; split_bf16(s[e], a, c); hi[e] = a; lo[e] = c; }
+      *reinterpret_cast<bf16x4*>(xh + i * PITCH + col * 2) = hi;
+      *reinterpret_cast<bf16x4*>(xl + i * PITCH + col * 2) = lo;
+    }
   }
   __syncthreads();
   const int n0 = (int)blockIdx.x * 64 + wave * 16;
@@ -416,11 +467,12 @@ __global__ __launch_bounds__(256) void latent_value_gen_kernel(LatentArgs p) {
 int64_t up256(int64_t x) { return (x + 255) / 256 * 256; }
 int64_t query_bytes(int B, int h, int R) { return up256((int64_t)B * h * R * 4); }
 
-// slices of the key range: about two workgroups per CU in all (one where the LDS tile fills a CU), at least one tile per wave
+int scan_tile(int R) { return R > 256 ? 32 : 64; }
+// slices of the key range: enough workgroups for the CUs' occupancy of the scan kernel, at least two tiles each
 int pick_split(int B, int groups, int64_t max_keys, int R) {
-  const int64_t tiles = (max_keys + KEYS_PER_TILE - 1) / KEYS_PER_TILE;
+  const int64_t tiles = vy_cdiv(max_keys, scan_tile(R));
   const int64_t want = vy_cdiv(R > 256 ? 256 : 512, (int64_t)B * groups);
-  int64_t s = vy_cdiv(tiles, 4);
+  int64_t s = vy_cdiv(tiles, 2);
   if (s > want) s = want;
   if (s > MAX_SPLIT) s = MAX_SPLIT;
   return (int)(s < 1 ? 1 : s);
@@ -486,9 +538,11 @@ extern "C" int vy_latent_decode(const void* q, int64_t ldq, const void* wukt, co
     else if (R <= 128) hipLaunchKernelGGL(latent_scan_kernel<128>, grid, block, 0, st, p);
     else if (R <= 256) hipLaunchKernelGGL(latent_scan_kernel<256>, grid, block, 0, st, p);
     else hipLaunchKernelGGL(latent_scan_kernel<512>, grid, block, 0, st, p);
-    const int RP = (R + 31) / 32 * 32;
-    hipLaunchKernelGGL(latent_value_kernel, dim3((unsigned)vy_cdiv(dv, 64), h, bt), block,
-                       16 * MAX_SPLIT * 4 + 2 * 16 * (RP + 8) * 2, st, p);
+    const int RP = (R + 31) / 32 * 32, nv = (int)vy_cdiv(dv, 64);
+    const int64_t per = vy_cdiv((int64_t)B * h * nv, 256);         // sequences per workgroup: fill the CUs first
+    p.seqs = (int)(per > 16 ? 16 : per);
+    hipLaunchKernelGGL(latent_value_kernel, dim3(nv, h, (unsigned)vy_cdiv(B, p.seqs)), block,
+                       p.seqs * MAX_SPLIT * 4 + 4096 + 2 * p.seqs * (RP + 8) * 2, st, p);
   }
   VY_CHECK_LAUNCH(who);
   return VY_OK;

@@ -35,16 +35,17 @@ __device__ __forceinline__ void split_bf16(float x, bf16& hi, bf16& lo) {
 }
 
 // ---- recurrence ------------------------------------------------------------------------------
-// workgroup = 16 value columns of one (b, head); thread (rg, col) keeps rows rg, rg + 16, ... of the state column.
-// TT tokens are staged at a time; the 16 partial dot products of an output are added after each stage.
-template <typename T, int RPT, int TT>
+// workgroup = COLS value columns of one (b, head); thread (rg, col) keeps rows rg, rg + RG, ... of the state column.
+// TT tokens are staged at a time; the RG partial dot products of an output are added after each stage.
+template <typename T, int COLS, int RPT, int TT>
 __global__ __launch_bounds__(256) void decay_recurrent_kernel(DecayArgs a) {
-  __shared__ float qs[TT][RPT * 16], ks[TT][RPT * 16];
-  __shared__ float vs[TT][16];
-  __shared__ float red[TT][16][17];
-  const int col = threadIdx.x & 15, rg = threadIdx.x >> 4;
+  constexpr int RG = 256 / COLS, DK = RG * RPT;
+  __shared__ float qs[TT][DK], ks[TT][DK];
+  __shared__ float vs[TT][COLS];
+  __shared__ float red[TT][RG][COLS + 1];
+  const int col = threadIdx.x % COLS, rg = threadIdx.x / COLS;
   const int head = blockIdx.y, b = blockIdx.z;
-  const int c0 = (int)blockIdx.x * 16, vc = c0 + col;
+  const int c0 = (int)blockIdx.x * COLS, vc = c0 + col;
   const int slot = a.slots ? a.slots[b] : b;
   const int n = a.count ? min(a.count[b], a.L) : a.L;
   const float decay = a.pow[(int64_t)head * (C + 1) + 1];
@@ -53,23 +54,23 @@ __global__ __launch_bounds__(256) void decay_recurrent_kernel(DecayArgs a) {
   const bool fresh = a.start[slot] == 0;
 #pragma unroll
   for (int i = 0; i < RPT; ++i) {
-    const int r = rg + 16 * i;
-    s[i] = !fresh && r < a.dk && vc < a.dv ? S[(int64_t)r * a.dv + vc] : 0.f;
+    const int r = rg + RG * i;
+    s[i] = r < a.dk && vc < a.dv ? S[(int64_t)r * a.dv + vc] : 0.f;
   }
   const T* P = (const T*)a.p + (int64_t)b * a.L * a.ldp;
   T* O = (T*)a.out + (int64_t)b * a.L * a.ldo + head * a.dv;
   for (int t0 = 0; t0 < n; t0 += TT) {
     const int m = min(TT, n - t0);
-    for (int i = threadIdx.x; i < m * RPT * 16; i += 256) {
-      const int t = i / (RPT * 16), d = i % (RPT * 16);
+    for (int i = threadIdx.x; i < m * DK; i += 256) {
+      const int t = i / DK, d = i % DK;
       const T* row = P + (int64_t)(t0 + t) * a.ldp + head * a.dk + d;
       const bool ok = d < a.dk;
       qs[t][d] = ok ? activate(VyT<T>::ld(row + a.oq), a.silu) : 0.f;
       ks[t][d] = ok ? activate(VyT<T>::ld(row + a.ok), a.silu) : 0.f;
     }
-    for (int i = threadIdx.x; i < m * 16; i += 256) {
-      const int t = i >> 4, d = c0 + (i & 15);
-      vs[t][i & 15] = d < a.dv ? activate(VyT<T>::ld(P + (int64_t)(t0 + t) * a.ldp + a.ov + head * a.dv + d), a.silu) : 0.f;
+    for (int i = threadIdx.x; i < m * COLS; i += 256) {
+      const int t = i / COLS, d = c0 + i % COLS;
+      vs[t][i % COLS] = d < a.dv ? activate(VyT<T>::ld(P + (int64_t)(t0 + t) * a.ldp + a.ov + head * a.dv + d), a.silu) : 0.f;
     }
     __syncthreads();
     for (int t = 0; t < m; ++t) {
@@ -77,26 +78,27 @@ __global__ __launch_bounds__(256) void decay_recurrent_kernel(DecayArgs a) {
       float o = 0.f;
 #pragma unroll
       for (int i = 0; i < RPT; ++i) {
-        s[i] = fmaf(decay, s[i], ks[t][rg + 16 * i] * v);
-        o = fmaf(s[i], qs[t][rg + 16 * i], o);
+        const float before = fresh && t0 + t == 0 ? 0.f : s[i];   // an empty slot's state is zero, whatever lies there
+        s[i] = fmaf(decay, before, ks[t][rg + RG * i] * v);
+        o = fmaf(s[i], qs[t][rg + RG * i], o);
       }
       red[t][rg][col] = o;
     }
     __syncthreads();
-    for (int i = threadIdx.x; i < m * 16; i += 256) {
-      const int t = i >> 4, cc = i & 15;
+    for (int i = threadIdx.x; i < m * COLS; i += 256) {
+      const int t = i / COLS, cc = i % COLS;
       float o = 0.f;
 #pragma unroll
-      for (int r = 0; r < 16; ++r) o += red[t][r][cc];
+      for (int r = 0; r < RG; ++r) o += red[t][r][cc];
       if (c0 + cc < a.dv) VyT<T>::st(O + (int64_t)(t0 + t) * a.ldo + c0 + cc, o);
     }
   }
   // the padding behind a short sequence: finite values for whatever reads whole batches
-  for (int64_t t = n + rg; t < a.L; t += 16)
+  for (int64_t t = n + rg; t < a.L; t += RG)
     if (vc < a.dv) VyT<T>::st(O + t * a.ldo + vc, 0.f);
 #pragma unroll
   for (int i = 0; i < RPT; ++i) {
-    const int r = rg + 16 * i;
+    const int r = rg + RG * i;
     if (r < a.dk && vc < a.dv) S[(int64_t)r * a.dv + vc] = s[i];
   }
 }
@@ -207,7 +209,7 @@ __global__ __launch_bounds__(256) void chunk_scan_kernel(DecayArgs a) {
   f32x4 s = {0.f, 0.f, 0.f, 0.f};
   if (a.start[slot] != 0) s = *reinterpret_cast<const f32x4*>(S);
   const float full = pw[C];
-  constexpr int UN = 4;
+  constexpr int UN = 8;
   for (int c0 = 0; c0 < a.nc; c0 += UN) {
     f32x4 u[UN];
 #pragma unroll
@@ -377,17 +379,22 @@ template <typename T>
 int recurrent_go(const DecayArgs& a, hipStream_t st) {
   const dim3 grid((unsigned)vy_cdiv(a.dv, 16), a.h, a.B), block(256);
   if (a.L == 1) {
-    if (a.dk <= 64) hipLaunchKernelGGL((decay_recurrent_kernel<T, 4, 1>), grid, block, 0, st, a);
-    else if (a.dk <= 128) hipLaunchKernelGGL((decay_recurrent_kernel<T, 8, 1>), grid, block, 0, st, a);
-    else if (a.dk <= 256) hipLaunchKernelGGL((decay_recurrent_kernel<T, 16, 1>), grid, block, 0, st, a);
-    else if (a.dk <= 512) hipLaunchKernelGGL((decay_recurrent_kernel<T, 32, 1>), grid, block, 0, st, a);
+    // a decode step streams the state: whole 256-byte row pieces where enough workgroups remain, else narrow columns
+    const int64_t wide = vy_cdiv(a.dv, 64) * a.h * a.B;
+    const dim3 wgrid((unsigned)vy_cdiv(a.dv, 64), a.h, a.B);
+    if (wide >= 512 && a.dk <= 64) hipLaunchKernelGGL((decay_recurrent_kernel<T, 64, 16, 1>), wgrid, block, 0, st, a);
+    else if (wide >= 512 && a.dk <= 128) hipLaunchKernelGGL((decay_recurrent_kernel<T, 64, 32, 1>), wgrid, block, 0, st, a);
+    else if (a.dk <= 64) hipLaunchKernelGGL((decay_recurrent_kernel<T, 16, 4, 1>), grid, block, 0, st, a);
+    else if (a.dk <= 128) hipLaunchKernelGGL((decay_recurrent_kernel<T, 16, 8, 1>), grid, block, 0, st, a);
+    else if (a.dk <= 256) hipLaunchKernelGGL((decay_recurrent_kernel<T, 16, 16, 1>), grid, block, 0, st, a);
+    else if (a.dk <= 512) hipLaunchKernelGGL((decay_recurrent_kernel<T, 16, 32, 1>), grid, block, 0, st, a);
     else return 1;
     return 0;
   }
-  if (a.dk <= 64) hipLaunchKernelGGL((decay_recurrent_kernel<T, 4, 16>), grid, block, 0, st, a);
-  else if (a.dk <= 128) hipLaunchKernelGGL((decay_recurrent_kernel<T, 8, 16>), grid, block, 0, st, a);
-  else if (a.dk <= 256) hipLaunchKernelGGL((decay_recurrent_kernel<T, 16, 8>), grid, block, 0, st, a);
-  else if (a.dk <= 512) hipLaunchKernelGGL((decay_recurrent_kernel<T, 32, 8>), grid, block, 0, st, a);
+  if (a.dk <= 64) hipLaunchKernelGGL((decay_recurrent_kernel<T, 16, 4, 16>), grid, block, 0, st, a);
+  else if (a.dk <= 128) hipLaunchKernelGGL((decay_recurrent_kernel<T, 16, 8, 16>), grid, block, 0, st, a);
+  else if (a.dk <= 256) hipLaunchKernelGGL((decay_recurrent_kernel<T, 16, 16, 8>), grid, block, 0, st, a);
+  else if (a.dk <= 512) hipLaunchKernelGGL((decay_recurrent_kernel<T, 16, 32, 8>), grid, block, 0, st, a);
   else return 1;
   return 0;
 }
