@@ -182,7 +182,7 @@ def latent_want(q, uk, uv, c, n, scale, gate):
 
 
 @pytest.mark.parametrize("dt", DT)
-@pytest.mark.parametrize("h,dh,dv,R", [(1, 16, 8, 8), (5, 24, 40, 72), (16, 64, 80, 96), (17, 8, 72, 200), (3, 136, 128, 512),
+@pytest.mark.parametrize("h,dh,dv,R", [(1, 16, 8, 8), (5, 24, 40, 72), (16, 64, 88, 104), (17, 8, 72, 200), (3, 136, 128, 512),
                                        (2, 16, 24, 640), (40, 16, 16, 264)])
 def test_latent_decode(dt, h, dh, dv, R):
     from vyomai_amd import ops
@@ -216,7 +216,7 @@ def test_latent_decode(dt, h, dh, dv, R):
 @pytest.mark.parametrize("dt", DT)
 def test_latent_decode_finds_one_key_among_many(dt):
     from vyomai_amd import ops
-    n, R, dh, dv = 777, 96, 96, 32
+    n, R, dh, dv = 777, 104, 104, 32
     uk = torch.eye(R, dtype=torch.float64)[None]         # the latent is the key
     uv = rnd(1, dv, R, seed=1, scale=R ** -0.5)
     q = rnd(1, dh, seed=2)

@@ -145,10 +145,6 @@ __global__ __launch_bounds__(256) void latent_scan_kernel(LatentArgs p) {
                                        (VY_LDS void*)(smem + (t % NS) * TILE + (wave * NP + i) * 1024), 16, 0, 0);
     }
   };
-#pragma unroll
-  for (int t = 0; t < NS - 1; ++t)
-    if (t < nt) stage(t);
-
   const int kblk = KH == 2 ? wave & 1 : wave, khalf = KH == 2 ? wave >> 1 : 0;
   bf16x8 qh[KS], ql[KS];
   const int64_t qo = ((int64_t)b * p.h + (head < p.h ? head : 0)) * p.R;
@@ -160,7 +156,10 @@ __global__ __launch_bounds__(256) void latent_scan_kernel(LatentArgs p) {
     qh[ks] = ok ? *reinterpret_cast<const bf16x8*>(p.qhi + qo + k) : zero8;
     ql[ks] = ok ? *reinterpret_cast<const bf16x8*>(p.qlo + qo + k) : zero8;
   }
-  // (retire the ordinary loads before the loop: a wait for them inside it would drain the ring)
+  // The ring is filled behind the query loads (without conditions, so that their wait can be counted: rows past the end are
+  // clamped), and the queries are retired before the loop: a wait for them inside it would drain the ring.
+#pragma unroll
+  for (int t = 0; t < NS - 1; ++t) stage(t);
 #pragma unroll
   for (int ks = 0; ks < KS; ++ks) { asm volatile("" ::"v"(qh[ks])); asm volatile("" ::"v"(ql[ks])); }
 
@@ -268,6 +267,7 @@ __global__ __launch_bounds__(256) void latent_scan_kernel(LatentArgs p) {
         o[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[tt][i], pf[tt], o[i], 0, 0, 0);
       }
   }
+  asm volatile("s_waitcnt vmcnt(0)" ::: "memory");   // tiles requested past the slice's end
   if (head < p.h) {
     const int64_t o_ = ((int64_t)b * p.h + head) * p.nsplit + split;
     const float l = quad_sum(l_run);
@@ -293,9 +293,12 @@ __device__ __forceinline__ void slice_weights(const LatentArgs& p, int b, int he
 
 // out[b][h][n] = (W_uv,h u_bh)_n * sigmoid(gate): workgroup = 64 value columns of one head x p.seqs (<= 16) sequences; the
 // mean latents are added up from the slices into LDS first (few sequences: the slices are shared out over the threads)
+// (RP: padded latent width.  The weights of the product are requested before anything else: one memory latency beside the
+// slices', not one after another behind them.)
+template <int RP>
 __global__ __launch_bounds__(256) void latent_value_kernel(LatentArgs p) {
   extern __shared__ __attribute__((aligned(16))) char dyn[];
-  const int RP = (p.R + 31) / 32 * 32, PITCH = (RP + 8) * 2;
+  constexpr int PITCH = (RP + 8) * 2, KS = RP / 32;
   float* sw = reinterpret_cast<float*>(dyn);                       // [seqs][MAX_SPLIT]
   f32x4* acc4 = reinterpret_cast<f32x4*>(dyn + p.seqs * MAX_SPLIT * 4);   // [256]
   char* xh = dyn + p.seqs * MAX_SPLIT * 4 + 4096;
@@ -305,9 +308,21 @@ __global__ __launch_bounds__(256) void latent_value_kernel(LatentArgs p) {
   const int head = blockIdx.y, b0 = (int)blockIdx.z * p.seqs;
   const int nb = min(p.seqs, p.B - b0);
   const bf16x8 zero8 = {};
+  const int n0 = (int)blockIdx.x * 64 + wave * 16;
+  const bool wok = n0 + r16 < p.dv;
+  bf16x8 wf[KS];
+  {
+    const bf16* w = (const bf16*)p.wuv + ((int64_t)head * p.dv + (wok ? n0 + r16 : 0)) * p.R;
+#pragma unroll
+    for (int ks = 0; ks < KS; ++ks) {
+      const int k = 32 * ks + 8 * kq;
+      wf[ks] = wok && k < p.R ? *reinterpret_cast<const bf16x8*>(w + k) : zero8;
+    }
+  }
   for (int i = wave; i < nb; i += 4) slice_weights(p, b0 + i, head, sw + i * MAX_SPLIT, lane);
   __syncthreads();
-  const int q4 = RP / 4, items = nb * q4;
+  constexpr int q4 = RP / 4;
+  const int items = nb * q4;
   const int G = items >= 256 ? 1 : 256 / items;                    // groups of slices
   for (int base = 0; base < items; base += 256) {
     const int g = G > 1 ? (int)threadIdx.x / items : 0;
@@ -316,9 +331,21 @@ __global__ __launch_bounds__(256) void latent_value_kernel(LatentArgs p) {
     const int i = live ? idx / q4 : 0, col = (idx - i * q4) * 4;
     f32x4 s = {0.f, 0.f, 0.f, 0.f};
     if (live && col < p.R) {
+      // batches of UB loads, all requested before the first is used (slices past the end: the last one, weight 0)
       const float* po = p.part_o + ((int64_t)(b0 + i) * p.h + head) * p.nsplit * p.R + col;
-#pragma unroll 8
-      for (int k = g; k < p.nsplit; k += G) s += sw[i * MAX_SPLIT + k] * *reinterpret_cast<const f32x4*>(po + (int64_t)k * p.R);
+      constexpr int UB = 8;
+      for (int k0 = g; k0 < p.nsplit; k0 += UB * G) {
+        f32x4 v[UB];
+        float wk[UB];
+#pragma unroll
+        for (int u = 0; u < UB; ++u) {
+          const int k = k0 + u * G, kc = min(k, p.nsplit - 1);
+          v[u] = *reinterpret_cast<const f32x4*>(po + (int64_t)kc * p.R);
+          wk[u] = k < p.nsplit ? sw[i * MAX_SPLIT + kc] : 0.f;
+        }
+#pragma unroll
+        for (int u = 0; u < UB; ++u) s += wk[u] * v[u];
+      }
     }
     if (G > 1) {   // (workgroup-uniform; then one pass covers every item)
       acc4[threadIdx.x] = s;
@@ -335,28 +362,18 @@ __global__ __launch_bounds__(256) void latent_value_kernel(LatentArgs p) {
     }
   }
   __syncthreads();
-  const int n0 = (int)blockIdx.x * 64 + wave * 16;
   if (n0 >= p.dv) return;
-  const bool wok = n0 + r16 < p.dv;
-  const bf16* w = (const bf16*)p.wuv + ((int64_t)head * p.dv + (wok ? n0 + r16 : 0)) * p.R;
-  f32x4 acc = {0.f, 0.f, 0.f, 0.f};
-  for (int k0 = 0; k0 < p.R; k0 += 128) {
-    bf16x8 wf[4];
+  f32x4 acc = {0.f, 0.f, 0.f, 0.f}, acl = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-    for (int u = 0; u < 4; ++u) {
-      const int k = k0 + 32 * u + 8 * kq;
-      wf[u] = wok && k < p.R ? *reinterpret_cast<const bf16x8*>(w + k) : zero8;
-    }
-#pragma unroll
-    for (int u = 0; u < 4; ++u) {
-      const int k = k0 + 32 * u + 8 * kq;
-      const bool ok = r16 < nb && k < RP;
-      const bf16x8 a = ok ? *reinterpret_cast<const bf16x8*>(xl + r16 * PITCH + k * 2) : zero8;
-      const bf16x8 c = ok ? *reinterpret_cast<const bf16x8*>(xh + r16 * PITCH + k * 2) : zero8;
-      acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[u], a, acc, 0, 0, 0);
-      acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[u], c, acc, 0, 0, 0);
-    }
+  for (int ks = 0; ks < KS; ++ks) {
+    const int k = 32 * ks + 8 * kq;
+    const bool ok = r16 < nb;
+    const bf16x8 a = ok ? *reinterpret_cast<const bf16x8*>(xl + r16 * PITCH + k * 2) : zero8;
+    const bf16x8 c = ok ? *reinterpret_cast<const bf16x8*>(xh + r16 * PITCH + k * 2) : zero8;
+    acl = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[ks], a, acl, 0, 0, 0);
+    acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[ks], c, acc, 0, 0, 0);
   }
+  acc += acl;
   const int nn = n0 + 4 * kq;
   if (r16 < nb && nn < p.dv) {
     const int64_t b = b0 + r16;
@@ -538,11 +555,15 @@ extern "C" int vy_latent_decode(const void* q, int64_t ldq, const void* wukt, co
     else if (R <= 128) hipLaunchKernelGGL(latent_scan_kernel<128>, grid, block, 0, st, p);
     else if (R <= 256) hipLaunchKernelGGL(latent_scan_kernel<256>, grid, block, 0, st, p);
     else hipLaunchKernelGGL(latent_scan_kernel<512>, grid, block, 0, st, p);
-    const int RP = (R + 31) / 32 * 32, nv = (int)vy_cdiv(dv, 64);
+    const int nv = (int)vy_cdiv(dv, 64);
     const int64_t per = vy_cdiv((int64_t)B * h * nv, 256);         // sequences per workgroup: fill the CUs first
     p.seqs = (int)(per > 16 ? 16 : per);
-    hipLaunchKernelGGL(latent_value_kernel, dim3(nv, h, (unsigned)vy_cdiv(B, p.seqs)), block,
-                       p.seqs * MAX_SPLIT * 4 + 4096 + 2 * p.seqs * (RP + 8) * 2, st, p);
+    const dim3 vgrid(nv, h, (unsigned)vy_cdiv(B, p.seqs));
+    auto lds = [&](int RP) { return p.seqs * MAX_SPLIT * 4 + 4096 + 2 * p.seqs * (RP + 8) * 2; };
+    if (R <= 64) hipLaunchKernelGGL(latent_value_kernel<64>, vgrid, block, lds(64), st, p);
+    else if (R <= 128) hipLaunchKernelGGL(latent_value_kernel<128>, vgrid, block, lds(128), st, p);
+    else if (R <= 256) hipLaunchKernelGGL(latent_value_kernel<256>, vgrid, block, lds(256), st, p);
+    else hipLaunchKernelGGL(latent_value_kernel<512>, vgrid, block, lds(512), st, p);
   }
   VY_CHECK_LAUNCH(who);
   return VY_OK;

@@ -209,12 +209,15 @@ __global__ __launch_bounds__(256) void chunk_scan_kernel(DecayArgs a) {
   f32x4 s = {0.f, 0.f, 0.f, 0.f};
   if (a.start[slot] != 0) s = *reinterpret_cast<const f32x4*>(S);
   const float full = pw[C];
-  constexpr int UN = 8;
-  for (int c0 = 0; c0 < a.nc; c0 += UN) {
-    f32x4 u[UN];
+  constexpr int UN = 4;                       // chunks per batch of loads; the next batch is requested before this one is used
+  f32x4 u[UN], nx[UN];
+  auto fetch = [&](int c0, f32x4 (&r)[UN]) {
 #pragma unroll
-    for (int i = 0; i < UN; ++i)
-      if (c0 + i < a.nc) u[i] = *reinterpret_cast<const f32x4*>(U + (c0 + i) * elems);
+    for (int i = 0; i < UN; ++i) r[i] = *reinterpret_cast<const f32x4*>(U + min(c0 + i, a.nc - 1) * elems);
+  };
+  fetch(0, u);
+  for (int c0 = 0; c0 < a.nc; c0 += UN) {
+    if (c0 + UN < a.nc) fetch(c0 + UN, nx);
 #pragma unroll
     for (int i = 0; i < UN; ++i) {
       if (c0 + i >= a.nc) break;
@@ -227,6 +230,8 @@ __global__ __launch_bounds__(256) void chunk_scan_kernel(DecayArgs a) {
 #pragma unroll
       for (int e = 0; e < 4; ++e) s[e] = fmaf(d, s[e], u[i][e]);
     }
+#pragma unroll
+    for (int i = 0; i < UN; ++i) u[i] = nx[i];
   }
   *reinterpret_cast<f32x4*>(S) = s;
 }
