@@ -289,6 +289,7 @@ class HybridDecodePlan:
             L.w_in, L.n_in, L.w_o = _ptr(p.w_in), p.w_in.shape[0], _ptr(p.w_o)
             L.norm1, L.norm1b = _ptr(n.norm1), _ptr(n.norm1b)
             buf = cache.buffers[i]
+            self.keep.append(buf)
             if m.kind == "latent":
                 L.mixer, L.scale = MIX_LATENT, m.scale
                 L.q_rank, L.q_rank_p, L.kv_rank, L.kv_rank_p = m.q_rank, p.q_norm.numel(), m.kv_rank, p.c_norm.numel()
@@ -316,7 +317,7 @@ class HybridDecodePlan:
         nbytes = lib.vy_hybrid_ws_bytes(C.byref(p))
         self.ws = torch.empty(nbytes, dtype=torch.uint8, device=model.device)
         p.ws, p.ws_bytes = self.ws.data_ptr(), nbytes
-        self.plan, self.batch, self.cache, self.generation = p, batch, cache, cache.generation
+        self.plan, self.batch, self.generation = p, batch, cache.generation
         self.vocab, self.ldv, self.dtype, self.device = model.vocab, (model.vocab + 7) // 8 * 8, model.dtype, model.device
         self.params = list(model.parameters())
         self.versions = self._versions()
@@ -325,18 +326,18 @@ class HybridDecodePlan:
         return sum(p._version for p in self.params)
 
     def valid(self, cache) -> bool:
-        """Same buffers, and no weight written since (weights REPLACED are noticed by the next prefill, which drops plans)."""
-        return self.cache is cache and self.generation == cache.generation and self.versions == self._versions()
+        """The cache's buffers have not moved and no weight was written since."""
+        return self.generation == cache.generation and self.versions == self._versions()
 
     def step(self, ids: torch.Tensor, batch) -> torch.Tensor:
         """ids (B,) int64; batch: the cache's SlotBatch for one more token each -> logits (B, vocab) view."""
         assert ids.shape == (self.batch,) and ids.dtype == torch.long and ids.is_contiguous() and ids.device == self.device
-        if batch.max_keys > self.cache.capacity:   # the kernels write the new row there
-            raise ValueError(f"{batch.max_keys} tokens exceed the cache capacity {self.cache.capacity}")
+        if batch.max_keys > batch.cache.capacity:   # the kernels write the new row there
+            raise ValueError(f"{batch.max_keys} tokens exceed the cache capacity {batch.cache.capacity}")
         from .ops import _mid_ws
         _mid_ws(self.batch)
         logits = torch.empty((self.batch, self.ldv), dtype=self.dtype, device=self.device)
         _lib.call("vy_hybrid_decoder_step", C.byref(self.plan), ids.data_ptr(), batch.slots.data_ptr(),
-                  self.cache.lengths.data_ptr(), int(batch.max_keys), logits.data_ptr(), self.ldv,
+                  batch.start.data_ptr(), int(batch.max_keys), logits.data_ptr(), self.ldv,
                   torch.cuda.current_stream().cuda_stream)
         return logits[:, : self.vocab]

@@ -293,6 +293,7 @@ class SlotCache:
         self._free = list(range(self.slots - 1, -1, -1))
         self._tables = {}
         self.generation = 0          # counts reallocations: whoever holds buffer addresses compares it
+        self.plans = {}              # native decode plans over these buffers (models/hybrid.py)
 
     def _make(self, spec, slots: int, capacity: int) -> torch.Tensor:
         kind, shape = spec

@@ -53,7 +53,6 @@ class HybridDecoderModel(nn.Module):
         self.layers = nn.ModuleList(layers)
         self.final_norm = WeightNorm(width, eps, norm)
         self.head = nn.Linear(width, vocab, bias=False)
-        self._plans, self._stamp = {}, None
         self._own_cache: Optional[SlotCache] = None
         self.requires_grad_(False)
 
@@ -89,9 +88,6 @@ class HybridDecoderModel(nn.Module):
                                "model and its inputs to 'cuda')")
         B, L = tokens.shape
         batch = cache.reserve(list(slots), list(counts))
-        stamp = tuple(q.data_ptr() for q in self.parameters())
-        if stamp != self._stamp:
-            self._plans, self._stamp = {}, stamp
         p = self.packed()
         dp = up8(self.width)
         x = torch.empty((B * L, dp), dtype=torch.float32, device=tokens.device)
@@ -124,12 +120,13 @@ class HybridDecoderModel(nn.Module):
         from ..decode_plan import HybridDecodePlan
         slots = list(slots)
         batch = cache.reserve(slots, [1] * len(slots))
-        key = id(cache), len(slots)
-        plan = self._plans.get(key)
+        # plans live with the cache whose buffers they point at; a model that was given other weights is another owner
+        key = id(self), self.word_embeddings.weight.data_ptr(), self.head.weight.data_ptr(), len(slots)
+        plan = cache.plans.get(key)
         if plan is None or not plan.valid(cache):
-            if len(self._plans) > 8:
-                self._plans.clear()
-            plan = self._plans[key] = HybridDecodePlan(self, cache, len(slots))
+            if len(cache.plans) > 8:
+                cache.plans.clear()
+            plan = cache.plans[key] = HybridDecodePlan(self, cache, len(slots))
         out = plan.step(ids, batch)
         cache.advance(slots, [1] * len(slots), on_device=False)
         return out
