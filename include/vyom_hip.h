@@ -153,6 +153,11 @@ int vy_rmsnorm_fwd(const void* x, int64_t ldx, const void* w, void* y, int64_t l
 int vy_gated_act_fwd(const void* gate_up, int64_t ldg, void* out, int64_t ldo, int64_t M, int64_t I,
                      int act, int dtype, void* stream);
 
+/* vy_clamped_act_fwd: with g = min(gate_up[m, i], limit), u = clamp(gate_up[m, I + i], -limit, limit):
+ * out[m, i] = g * sigmoid(alpha * g) * (u + 1). */
+int vy_clamped_act_fwd(const void* gate_up, int64_t ldg, void* out, int64_t ldo, int64_t M, int64_t I, float limit, float alpha,
+                       int dtype, void* stream);
+
 /* ------------------------------------------------------------------------------------------
  * Decoders with an fp32 residual stream (norm before and after every sublayer), latent attention and decayed linear
  * attention.  Conventions shared by this group:
@@ -164,6 +169,9 @@ int vy_gated_act_fwd(const void* gate_up, int64_t ldg, void* out, int64_t ldo, i
  * vy_residual_norm: x (fp32) += norm(y) * w_post ; h = norm(x) * w_pre.  ids given: x = table[ids] instead (an id outside
  *   [0, V) gives zeros and sets *err_flag); w_post NULL: plain add; y and ids NULL: x is only read; h NULL: no second norm.
  *   rms = 0: (v - mean) / sqrt(var + eps), rms = 1: v / sqrt(mean(v^2) + eps).
+ * vy_residual_norm_routed: the same with y += sum_k weight[row][k] * rows[pos[row][k]] ahead of the post norm (routed
+ *   nullable; weight fp32 and pos int32 are [M][top], pos NULL: row * top + k, pos < 0: left out; y NULL: the sum alone) and
+ *   x = table_scale * table[ids].
  * vy_latent_norm: p = packed rows [query latent (npq) | key/value latent (npc) | ...]: q_out = RMSNorm(latent) * w_q,
  *   c_out (nullable) = RMSNorm(latent) * w_c, also written to cache[slot][start + l] (strides c_ss / c_st, cap rows per slot).
  * vy_rmsnorm_gate: y = RMSNorm(x) * w * sigmoid(gate).
@@ -171,6 +179,14 @@ int vy_gated_act_fwd(const void* gate_up, int64_t ldg, void* out, int64_t ldo, i
 int vy_residual_norm(float* x, int64_t ldx, const void* y, int64_t ldy, const void* table, int64_t ldt, const int64_t* ids,
                      int64_t V, int32_t* err_flag, const float* w_post, float eps_post, const float* w_pre, float eps_pre,
                      void* h, int64_t ldh, int64_t M, int64_t N, int64_t NP, int rms, int dtype, void* stream);
+typedef struct vy_routed_rows {
+  const void* rows; int64_t ld;
+  const int32_t* pos; const float* weight; int32_t top;
+} vy_routed_rows;
+int vy_residual_norm_routed(float* x, int64_t ldx, const void* y, int64_t ldy, const void* table, int64_t ldt,
+                            const int64_t* ids, int64_t V, int32_t* err_flag, float table_scale, const vy_routed_rows* routed,
+                            const float* w_post, float eps_post, const float* w_pre, float eps_pre, void* h, int64_t ldh,
+                            int64_t M, int64_t N, int64_t NP, int rms, int dtype, void* stream);
 int vy_latent_norm(const void* p, int64_t ldp, const float* w_q, void* q_out, int64_t ldq, int32_t nq, int32_t npq,
                    const float* w_c, void* c_out, int64_t ldc, int32_t nc, int32_t npc, void* cache, int64_t c_ss,
                    int64_t c_st, int32_t cap, const int32_t* slots, const int32_t* start, const int32_t* count, int64_t B,
@@ -180,11 +196,63 @@ int vy_rmsnorm_gate(const void* x, int64_t ldx, const float* w, const void* gate
 
 /* vy_attn_fwd_ex: causal attention whose values may have a width of their own (dv), with a start position per sequence
  * (key j is visible to query i of sequence b iff j <= start[slot] + i; start NULL: 0) and an optional output gate:
- * out *= sigmoid(gate), gate laid out as out (strides g_sb, g_sl). */
+ * out *= sigmoid(gate), gate laid out as out (strides g_sb, g_sl).
+ * win (nullable) adds, with s_b = min(start[slot], start_cap) in the place of start[slot]:
+ *   window     query i sees only the keys j > s_b + i - window (0: every earlier key);
+ *   sink       one more term exp(0) in every softmax denominator, without a value;
+ *   rope       rotary positions of the queries: (cos, sin) pairs [rope_len][rope_dims / 2], fp32; columns 2c and 2c + 1 of the
+ *              first rope_dims turn by the angle of position start[slot] + i (the keys are rotated already);
+ *   kv_by_slot k and v are indexed by slots[b] instead of b (row-wise kernel). */
+typedef struct vy_attn_window {
+  int32_t window, sink, kv_by_slot, start_cap;
+  const float* rope; int32_t rope_dims, rope_len;
+} vy_attn_window;
 int vy_attn_fwd_ex(const void* q, int64_t q_sb, int64_t q_sh, int64_t q_sl, const void* k, int64_t k_sb, int64_t k_sh,
                    int64_t k_sl, const void* v, int64_t v_sb, int64_t v_sh, int64_t v_sl, void* out, int64_t o_sb,
                    int64_t o_sl, const void* gate, int64_t g_sb, int64_t g_sl, const int32_t* start, const int32_t* slots,
-                   int64_t B, int h, int hk, int64_t L, int64_t S, int dh, int dv, float scale, int dtype, void* stream);
+                   int64_t B, int h, int hk, int64_t L, int64_t S, int dh, int dv, float scale, const vy_attn_window* win,
+                   int dtype, void* stream);
+
+/* vy_moe_fwd: mixture of experts on rows h [M][width].  z = w_router h (fp32), scores softmax(z); experts form `groups` equal
+ * groups of neighbours, and only those of the `keep` groups with the best largest score can be chosen; the `top` best of them
+ * are, with weight = scale * score / (sum of the chosen scores + 1e-20).  Expert e: vy_clamped_act_fwd's activation between
+ * w_gu[e] (rows interleaved: 2j gate j, 2j + 1 up j) and w_down[e].  Nothing is added up here:
+ *   rows   the experts' outputs, row stride ldr, M * top of them in an order of its own,
+ *   pos    [M][top] a choice's row, weight [M][top] its weight (vy_residual_norm_routed takes the three), ids [M][top] its expert
+ *          (-1, 0 and -1 for padding tokens: those with l >= count[b], m = b L + l; count nullable).
+ * width and ff are padded to multiples of 8.  experts <= 1024, top <= 64. */
+typedef struct vy_moe {
+  int32_t experts, top, groups, keep, width, ff;
+  float scale, limit, alpha;
+  const void *w_router, *w_gu, *w_down;   /* [experts][width], [experts][2 ff][width], [experts][width][ff] */
+} vy_moe;
+int64_t vy_moe_ws_bytes(const vy_moe* d, int64_t M, int dtype);
+int vy_moe_fwd(const vy_moe* d, const void* h, int64_t ldh, int64_t M, const int32_t* count, int64_t L, void* rows, int64_t ldr,
+               int32_t* ids, int32_t* pos, float* weight, void* ws, int64_t ws_bytes, int dtype, void* stream);
+
+/* Sliding-window attention over a ring of keys and values.  Per slot and key/value head the ring holds R rows [key (dim) |
+ * value (vdim)] (strides r_ss per slot, r_sh per head), position p in row p % R; R is the window, or less while no sequence is
+ * longer than R.  Packed projection rows p (stride ldp): queries at column oq ([h][dim]), keys ok ([hk][dim]), values ov
+ * ([hk][vdim]), output gate og ([h][vdim], og < 0: none).  rope / rope_dims / rope_len as in vy_attn_window.
+ *
+ * vy_window_rows: rotate != 0: rotary positions on the new keys, in place; store != 0: the last R of the count[b] new rows of
+ *   every sequence to the ring.
+ * vy_window_context: ctx [B][hk][S][dim + vdim] = the last min(start, past) rows of the ring in order of position, then the L
+ *   new rows (rotated already), then zeros: what vy_attn_fwd_ex takes with start_cap = past.
+ * vy_window_decode: one new token per sequence (L = 1): its key and value to the ring, then attention of its queries over the
+ *   ring with sink and gate; max_keys >= every start + 1; ws: vy_window_decode_ws_bytes(...).  scale > 0. */
+int vy_window_rows(void* p, int64_t ldp, int64_t ok, int64_t ov, void* ring, int64_t r_ss, int64_t r_sh, int32_t R,
+                   const float* rope, int32_t rope_dims, int32_t rope_len, int rotate, int store, const int32_t* slots,
+                   const int32_t* start, const int32_t* count, int64_t B, int64_t L, int32_t hk, int32_t dim, int32_t vdim,
+                   int dtype, void* stream);
+int vy_window_context(const void* p, int64_t ldp, int64_t ok, int64_t ov, const void* ring, int64_t r_ss, int64_t r_sh,
+                      int32_t R, void* ctx, int32_t S, int32_t past, const int32_t* slots, const int32_t* start, int64_t B,
+                      int64_t L, int32_t hk, int32_t dim, int32_t vdim, int dtype, void* stream);
+int64_t vy_window_decode_ws_bytes(int32_t B, int32_t h, int32_t hk, int32_t vdim, int32_t R);
+int vy_window_decode(void* p, int64_t ldp, int64_t oq, int64_t ok, int64_t ov, int64_t og, void* ring, int64_t r_ss, int64_t r_sh,
+                     int32_t R, const float* rope, int32_t rope_dims, int32_t rope_len, const int32_t* slots,
+                     const int32_t* start, int64_t max_keys, void* out, int64_t ldo, int64_t B, int32_t h, int32_t hk,
+                     int32_t dim, int32_t vdim, float scale, int32_t sink, void* ws, int64_t ws_bytes, int dtype, void* stream);
 
 /* vy_latent_decode: one query token per sequence against a cache of latents c (one row of R per token, shared by all
  * heads).  Keys and values are never expanded:  q~_h = Wuk_h^T q_h,  s_j = scale * q~_h . c_j over j <= start[slot],
@@ -491,30 +559,42 @@ int vy_gemma_decoder_step(const vy_gemma_plan* plan, const void* x, int64_t pos,
 
 /* ------------------------------------------------------------------------------------------
  * vy_hybrid_decoder_step: one new token for each of B sequences of a decoder that mixes layer kinds over an fp32 residual
- * stream.  Per layer: h = norm(x) * norm1; mixer; x += norm(y) * norm1b; h = norm(x) * norm2; gated MLP; x += norm(y) * norm2b
- * (ff = 0: no MLP).  Mixers, all from ONE packed input projection w_in of h:
+ * stream.  Forms of a layer:
+ *   VY_FORM_SANDWICH  h = norm(x) * norm1; y = w_o mixer(h); x += norm(y) * norm1b;
+ *                     h = norm(x) * norm2; x += norm(ff(h)) * norm2b                       (ff = 0 and no moe: no second half)
+ *   VY_FORM_PARALLEL  h = norm(x) * norm1; x += w_o [mixer(h) | act(h)] + routed(h): one packed product w_in of h also gives the
+ *                     [gate; up] rows of a dense feed-forward of width ff (its last 2 ff rows), one product w_o takes both back
+ * norm1b / norm2b NULL: no norm on a sublayer's output.  moe (nullable): routed experts, added to the feed-forward's output.
+ * clamped: the feed-forward's activation is vy_clamped_act_fwd's (limit, alpha), else the plan's act.
+ * Mixers, all from ONE packed input projection w_in of h:
  *   VY_MIX_LATENT  rows [query latent | key/value latent | output gate]: vy_latent_norm, q = w_uq latent, vy_latent_decode
  *   VY_MIX_DECAY   rows [q | k | v | output gate]: vy_decay_attn, vy_rmsnorm_gate
- * then y = w_o (.).  Sequence b (ids[b]) lives in slot slots[b] (NULL: b) and holds lengths[slot] tokens, which the step
- * advances by one on the device; max_keys >= every lengths[slot] + 1.  Widths with _p, dim, vdim, ff and dp are padded to
- * multiples of 8; d, q_rank, kv_rank and mix_n are the true counts the norms divide by.  logits: (B, ldv).
+ *   VY_MIX_WINDOW  rows [q | k | v | output gate]: vy_window_decode on the ring `cache` (strides c_ss per slot, c_sh per head)
+ * Sequence b (ids[b]) lives in slot slots[b] (NULL: b) and holds lengths[slot] tokens, which the step advances by one on the
+ * device; max_keys >= every lengths[slot] + 1.  Widths with _p, dim, vdim, ff and dp are padded to multiples of 8; d, q_rank,
+ * kv_rank and mix_n are the true counts the norms divide by.  logits: (B, ldv).
  * -------------------------------------------------------------------------------------------- */
-enum { VY_MIX_LATENT = 0, VY_MIX_DECAY = 1 };
+enum { VY_MIX_LATENT = 0, VY_MIX_DECAY = 1, VY_MIX_WINDOW = 2 };
+enum { VY_FORM_SANDWICH = 0, VY_FORM_PARALLEL = 1 };
 typedef struct vy_hybrid_layer {
   int32_t mixer, heads, dim, vdim, n_in, ff;
   int32_t q_rank, q_rank_p, kv_rank, kv_rank_p;   /* VY_MIX_LATENT */
   int32_t cap, mix_n;                             /* cache rows per slot; VY_MIX_DECAY: width of mix_norm */
-  float scale;
+  int32_t form, clamped;
+  int32_t kv_heads, rope_dims, rope_len, sink;    /* VY_MIX_WINDOW */
+  float scale, limit, alpha;
   const float *norm1, *norm1b, *norm2, *norm2b;
-  const void *w_in, *w_o, *w_gu, *w_down;         /* w_gu: packed [gate; up] */
+  const void *w_in, *w_o, *w_gu, *w_down;         /* w_gu: packed [gate; up] (VY_FORM_SANDWICH) */
   const float *q_norm, *c_norm;
   const void *w_uq, *w_ukt, *w_uv;
-  void* cache; int64_t c_ss, c_st;
+  void* cache; int64_t c_ss, c_sh, c_st;
   float* state; const float *decay_pow, *mix_norm;
+  const float* rope;
+  const vy_moe* moe;
 } vy_hybrid_layer;
 typedef struct vy_hybrid_plan {
   int32_t num_layers, B, d, dp, vocab, dtype, rms, act;
-  float eps;
+  float eps, embed_scale;
   const vy_hybrid_layer* layers;                  /* host array [num_layers] */
   const void *embed, *head; const float* final_norm;
   int32_t* err;                                   /* nullable: set when an id is outside the vocabulary */

@@ -61,14 +61,22 @@ PROTOTYPES = {
     "vy_decoder_step": [_p, _p, _i64, _p, _p, _p, _i64, _p],
     "vy_gemma_decoder_step": [_p, _p, _i64, _p, _i64, _p],
     "vy_residual_norm": [_p, _i64, _p, _i64, _p, _i64, _p, _i64, _p, _p, _f, _p, _f, _p, _i64, _i64, _i64, _i64, _i, _i, _p],
+    "vy_residual_norm_routed": [_p, _i64, _p, _i64, _p, _i64, _p, _i64, _p, _f, _p, _p, _f, _p, _f, _p, _i64, _i64, _i64, _i64, _i,
+                                _i, _p],
     "vy_latent_norm": [_p, _i64, _p, _p, _i64, _i, _i, _p, _p, _i64, _i, _i, _p, _i64, _i64, _i, _p, _p, _p, _i64, _i64, _f,
                        _i, _p],
     "vy_rmsnorm_gate": [_p, _i64, _p, _p, _i64, _p, _i64, _i64, _i64, _i64, _f, _i, _p],
     "vy_attn_fwd_ex": [_p, _i64, _i64, _i64, _p, _i64, _i64, _i64, _p, _i64, _i64, _i64, _p, _i64, _i64, _p, _i64, _i64,
-                       _p, _p, _i64, _i, _i, _i64, _i64, _i, _i, _f, _i, _p],
+                       _p, _p, _i64, _i, _i, _i64, _i64, _i, _i, _f, _p, _i, _p],
     "vy_latent_decode": [_p, _i64, _p, _p, _p, _i64, _i64, _p, _p, _i64, _p, _i64, _p, _i64, _i, _i, _i, _i, _i, _f, _p, _i64,
                          _i, _p],
     "vy_decay_attn": [_p, _i64, _i64, _i64, _i64, _p, _p, _p, _p, _p, _p, _i64, _i64, _i64, _i, _i, _i, _i, _p, _i64, _i, _p],
+    "vy_window_rows": [_p, _i64, _i64, _i64, _p, _i64, _i64, _i, _p, _i, _i, _i, _i, _p, _p, _p, _i64, _i64, _i, _i, _i, _i, _p],
+    "vy_window_context": [_p, _i64, _i64, _i64, _p, _i64, _i64, _i, _p, _i, _i, _p, _p, _i64, _i64, _i, _i, _i, _i, _p],
+    "vy_window_decode": [_p, _i64, _i64, _i64, _i64, _i64, _p, _i64, _i64, _i, _p, _i, _i, _p, _p, _i64, _p, _i64, _i64, _i, _i, _i,
+                         _i, _f, _i, _p, _i64, _i, _p],
+    "vy_moe_fwd": [_p, _p, _i64, _i64, _p, _i64, _p, _i64, _p, _p, _p, _p, _i64, _i, _p],
+    "vy_clamped_act_fwd": [_p, _i64, _p, _i64, _i64, _i64, _f, _f, _i, _p],
     "vy_hybrid_decoder_step": [_p, _p, _p, _p, _i64, _p, _i64, _p],
     "vy_cast": [_p, _p, _i64, _i, _i, _p],
     "vy_ddp_unique_id": [_p],
@@ -80,7 +88,7 @@ PROTOTYPES = {
 }
 OTHER_SYMBOLS = ["vy_last_error", "vy_abi_version", "vy_layernorm_bwd_ws_rows", "vy_decode_ws_bytes",
                  "vy_gemma_ws_bytes", "vy_ddp_world", "vy_ddp_rank", "vy_latent_decode_ws_bytes", "vy_decay_attn_ws_bytes",
-                 "vy_hybrid_ws_bytes"]
+                 "vy_hybrid_ws_bytes", "vy_window_decode_ws_bytes", "vy_moe_ws_bytes"]
 DECAY_CHUNK = 64   # VY_DECAY_CHUNK
 ALL_SYMBOLS = list(PROTOTYPES) + OTHER_SYMBOLS
 
@@ -89,6 +97,23 @@ class VyWgradDesc(C.Structure):
     """vy_wgrad_desc of include/vyom_hip.h."""
     _fields_ = [("dy", _p), ("lddy", _i64), ("x", _p), ("ldx", _i64), ("dw", _p), ("lddw", _i64), ("db", _p),
                 ("M", _i64), ("N", _i64), ("K", _i64)]
+
+
+class VyAttnWindow(C.Structure):
+    """vy_attn_window of include/vyom_hip.h."""
+    _fields_ = [(n, C.c_int32) for n in ("window", "sink", "kv_by_slot", "start_cap")] + \
+               [("rope", _p), ("rope_dims", C.c_int32), ("rope_len", C.c_int32)]
+
+
+class VyRoutedRows(C.Structure):
+    """vy_routed_rows of include/vyom_hip.h."""
+    _fields_ = [("rows", _p), ("ld", _i64), ("pos", _p), ("weight", _p), ("top", C.c_int32)]
+
+
+class VyMoe(C.Structure):
+    """vy_moe of include/vyom_hip.h."""
+    _fields_ = [(n, C.c_int32) for n in ("experts", "top", "groups", "keep", "width", "ff")] + \
+               [(n, C.c_float) for n in ("scale", "limit", "alpha")] + [(n, _p) for n in ("w_router", "w_gu", "w_down")]
 
 
 class VyomHipError(RuntimeError):
@@ -121,7 +146,8 @@ def load() -> C.CDLL:
     lib.vy_decode_ws_bytes.restype = C.c_int64
     lib.vy_decode_ws_bytes.argtypes = [C.c_int32] * 7
     for name, argtypes in (("vy_latent_decode_ws_bytes", [_i, _i, _i]),
-                           ("vy_decay_attn_ws_bytes", [_i64, _i64, _i, _i, _i, _i]), ("vy_hybrid_ws_bytes", [_p])):
+                           ("vy_decay_attn_ws_bytes", [_i64, _i64, _i, _i, _i, _i]), ("vy_hybrid_ws_bytes", [_p]),
+                           ("vy_window_decode_ws_bytes", [_i, _i, _i, _i, _i]), ("vy_moe_ws_bytes", [_p, _i64, _i])):
         getattr(lib, name).restype = C.c_int64
         getattr(lib, name).argtypes = argtypes
     _lib = lib

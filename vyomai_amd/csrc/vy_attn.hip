@@ -45,17 +45,53 @@ struct AttnParams {
   const int* start_dev; const int* slots;
   int dv;              // value width (0 = as wide as the keys)
   const void* gate; int64_t g_sb, g_sl;   // output gate (nullable): out *= sigmoid(gate), laid out as out
+  // EXT = 2 only: sliding window (0 = none), a sink of score 0 without a value, keys / values indexed by slot instead of by
+  // sequence, an upper bound of the start position (older keys are not in the operands), and rotary positions of the queries
+  int window, sink, kv_by_slot, start_cap;
+  const float2* rope; int rope_half, rope_len;   // (cos, sin) [position][pair], pairs of neighbouring columns
   int diag;            // timing experiments only (VY_ATTN_DIAG): 1 = no output store, 2 = no tile loop
 };
 
 __device__ __forceinline__ int attn_start(const AttnParams& p, int b) {
   return p.start_dev ? p.start_dev[p.slots ? p.slots[b] : b] : p.start_pos;
 }
+template <int EXT> __device__ __forceinline__ int attn_first(const AttnParams& p, int b) {
+  if constexpr (EXT == 0) return p.start_pos;
+  else if constexpr (EXT == 1) return attn_start(p, b);
+  else return min(attn_start(p, b), p.start_cap);
+}
+// rotary positions on N consecutive columns d0 .. of a query row (d0, N even)
+template <int N>
+__device__ __forceinline__ void attn_rotate(const AttnParams& p, int b, int qi, int d0, float (&v)[N]) {
+  if (!p.rope) return;
+  int pos = attn_start(p, b) + qi;
+  pos = pos < p.rope_len ? pos : p.rope_len - 1;   // (padding rows only)
+  const float2* t = p.rope + (int64_t)pos * p.rope_half;
+#pragma unroll
+  for (int e = 0; e < N; e += 2) {
+    const int i = (d0 + e) >> 1;
+    if (i < p.rope_half) {
+      const float2 cs = t[i];
+      const float u = v[e], w = v[e + 1];
+      v[e] = u * cs.x - w * cs.y;
+      v[e + 1] = w * cs.x + u * cs.y;
+    }
+  }
+}
+__device__ __forceinline__ void attn_rotate8(const AttnParams& p, int b, int qi, int d0, bf16x8& q) {
+  float v[8];
+#pragma unroll
+  for (int e = 0; e < 8; ++e) v[e] = (float)q[e];
+  attn_rotate<8>(p, b, qi, d0, v);
+#pragma unroll
+  for (int e = 0; e < 8; ++e) q[e] = (bf16)v[e];
+}
 
 // ------------------------------------------------------------------------------------------
-// MFMA flash forward (bf16).  EXT: per-sequence start positions and the sigmoid output gate.
+// MFMA flash forward (bf16).  EXT = 1: per-sequence start positions and the sigmoid output gate; 2: also the sliding window,
+// the sink and the queries' rotary positions.
 // ------------------------------------------------------------------------------------------
-template <int DH, bool EXT = false>
+template <int DH, int EXT = 0>
 __global__ __launch_bounds__(256, DH == 64 ? 3 : 1) void attn_fwd_mfma_kernel(AttnParams p) {
   constexpr int RB = DH * 2;            // bytes per K/V row
   constexpr int TILE = 64 * RB;         // bytes per 64-key tile
@@ -84,7 +120,7 @@ __global__ __launch_bounds__(256, DH == 64 ? 3 : 1) void attn_fwd_mfma_kernel(At
   const int qrow = qi < p.L ? qi : p.L - 1;
 
   const bf16* Q = (const bf16*)p.q + (int64_t)b * p.q_sb + (int64_t)head * p.q_sh + (int64_t)qrow * p.q_sl;
-  const int start = EXT ? attn_start(p, b) : p.start_pos;
+  const int start = attn_first<EXT>(p, b);
   const bf16* Kb = (const bf16*)p.k + (int64_t)b * p.k_sb + (int64_t)kvh * p.k_sh;
   const bf16* Vb = (const bf16*)p.v + (int64_t)b * p.v_sb + (int64_t)kvh * p.v_sh;
 
@@ -165,6 +201,8 @@ __global__ __launch_bounds__(256, DH == 64 ? 3 : 1) void attn_fwd_mfma_kernel(At
   // rows with NO visible key are recognised by l == 0 after the loop and get the reference's
   // uniform average over all keys from the column-sum pass below.
   float m_run = -FLT_MAX, l_run = 0.f;
+  if constexpr (EXT == 2)
+    if (p.sink) { m_run = 0.f; l_run = fh == 0 ? 1.f : 0.f; }   // exp(0), counted by one of the row's two halves
   const float c = p.scale * LOG2E;
 
   // pure causal: keys beyond the diagonal of the block's last row are never visible -> skipped
@@ -176,6 +214,10 @@ __global__ __launch_bounds__(256, DH == 64 ? 3 : 1) void attn_fwd_mfma_kernel(At
     if (nt < 1) nt = 1;
   }
   const int wave_first = q0 + wave * 32, wave_last = wave_first + 31;
+  // sliding window: tiles wholly before the block's first row's window are never loaded
+  const int window = EXT == 2 ? p.window : 0;
+  int t0 = 0;
+  if (EXT == 2 && window) t0 = max(0, start + q0 - window + 1) >> 6;
 
   // key-padding mask -> one 64-bit visibility word per key tile, built once (an ordinary load inside
   // the tile loop would make the compiler drain the LDS-DMA ring with vmcnt(0) every tile)
@@ -194,6 +236,7 @@ __global__ __launch_bounds__(256, DH == 64 ? 3 : 1) void attn_fwd_mfma_kernel(At
     const int k0 = tile * 64;
     // wave-uniform skip of tiles wholly above this wave's diagonal
     if (causal && k0 > start + wave_last) return;
+    if (EXT == 2 && window && k0 + 63 < start + wave_first - window + 1) return;
     const char* kb_ = smem + buf * TILE;
     const char* vb_ = smem + (NS + buf) * TILE;
     f32x16 st[2];
@@ -237,7 +280,8 @@ __global__ __launch_bounds__(256, DH == 64 ? 3 : 1) void attn_fwd_mfma_kernel(At
     });
     unsigned long long vis = ~0ull;
     if (haskp) vis = kpbits[tile];
-    const bool need_mask = hasadd || (k0 + 64 > p.S) || (causal && k0 + 63 > start + wave_first) || vis != ~0ull;
+    const bool need_mask = hasadd || (k0 + 64 > p.S) || (causal && k0 + 63 > start + wave_first) || vis != ~0ull ||
+                           (EXT == 2 && window && k0 < start + wave_last - window + 1);
     // softmax runs on the RAW scores: max first, then p = exp2(fma(s, c, -m)) -- one FMA and one
     // v_exp_f32 per element (the VALU, not the MFMA pipe, bounds dh=64)
     float tmax = -INFINITY;
@@ -249,6 +293,10 @@ __global__ __launch_bounds__(256, DH == 64 ? 3 : 1) void attn_fwd_mfma_kernel(At
       if (causal) klim = min(klim, qi + start - k0 - 4 * fh);
       unsigned long long lm = klim >= 63 ? ~0ull : (klim < 0 ? 0ull : ((2ull << klim) - 1ull));
       lm &= vis >> (4 * fh);
+      if (EXT == 2 && window) {
+        const int klow = qi + start - window + 1 - k0 - 4 * fh;
+        if (klow > 0) lm &= klow > 63 ? 0ull : ~0ull << klow;
+      }
       const unsigned lmw[2] = {(unsigned)lm, (unsigned)(lm >> 32)};
 #pragma unroll
       for (int kb = 0; kb < 2; ++kb)
@@ -328,18 +376,24 @@ __global__ __launch_bounds__(256, DH == 64 ? 3 : 1) void attn_fwd_mfma_kernel(At
   // MFMA inside the loop as vmcnt(0) and drains the ring every tile.
 #pragma unroll
   for (int s_ = 0; s_ < NS - 1; ++s_)
-    if (s_ < nt) stage(s_, s_);
+    if (t0 + s_ < nt) stage(t0 + s_, s_);
   // Q after the first K/V tiles are requested: one memory latency for both, not two in a row
 #pragma unroll
   for (int ks = 0; ks < KS; ++ks) qf[ks] = *reinterpret_cast<const bf16x8*>(Q + ks * 16 + fh * 8);
 #pragma unroll
   for (int ks = 0; ks < KS; ++ks) asm volatile("" ::"v"(qf[ks]));
-  for (int t = 0; t < (p.diag == 2 ? 0 : nt); ++t) {
+  if constexpr (EXT == 2) {
+#pragma unroll
+    for (int ks = 0; ks < KS; ++ks) attn_rotate8(p, b, qi, ks * 16 + fh * 8, qf[ks]);
+#pragma unroll
+    for (int ks = 0; ks < KS; ++ks) asm volatile("" ::"v"(qf[ks]));
+  }
+  for (int t = t0; t < (p.diag == 2 ? 0 : nt); ++t) {
     wait_tile(min(NS - 2, nt - 1 - t));
     __builtin_amdgcn_s_barrier();
     asm volatile("" ::: "memory");
-    if (t + NS - 1 < nt) stage(t + NS - 1, (t + NS - 1) % NS);  // the buffer tile t-1 was read from
-    compute(t, t % NS);
+    if (t + NS - 1 < nt) stage(t + NS - 1, (t - t0 + NS - 1) % NS);  // the buffer tile t-1 was read from
+    compute(t, (t - t0) % NS);
   }
 
   float l_tot = l_run + __shfl_xor(l_run, 32, 64);
@@ -442,7 +496,7 @@ __global__ __launch_bounds__(256, DH == 64 ? 3 : 1) void attn_fwd_mfma_kernel(At
 // reference's uniform average; a dense additive mask goes to the row-wise kernel.
 // ------------------------------------------------------------------------------------------
 // DHP / DVP: padded widths of the keys and of the values (attention whose values have a width of their own).
-template <int DHP, int DVP = DHP, bool EXT = false>
+template <int DHP, int DVP = DHP, int EXT = 0>
 __global__ __launch_bounds__(256) void attn_fwd_gen_kernel(AttnParams p, int dh) {
   constexpr int KPITCH = (DHP + 8) * 2;      // bytes per LDS row (16 B of padding: conflict-free fragment reads)
   constexpr int VPITCH = (DVP + 8) * 2;
@@ -467,7 +521,7 @@ __global__ __launch_bounds__(256) void attn_fwd_gen_kernel(AttnParams p, int dh)
   const bf16* Q = (const bf16*)p.q + (int64_t)b * p.q_sb + (int64_t)head * p.q_sh + (int64_t)qrow * p.q_sl;
   const bf16* Kb = (const bf16*)p.k + (int64_t)b * p.k_sb + (int64_t)kvh * p.k_sh;
   const bf16* Vb = (const bf16*)p.v + (int64_t)b * p.v_sb + (int64_t)kvh * p.v_sh;
-  const int start = EXT ? attn_start(p, b) : p.start_pos;
+  const int start = attn_first<EXT>(p, b);
   const bool causal = p.mask_kind & VY_MASK_CAUSAL;
   const bool haskp = p.mask_kind & VY_MASK_KEYPAD;
   const uint8_t* kp = haskp ? p.keypad + (int64_t)b * p.kp_sb : nullptr;
@@ -478,12 +532,18 @@ __global__ __launch_bounds__(256) void attn_fwd_gen_kernel(AttnParams p, int dh)
   for (int ks = 0; ks < KS; ++ks) {
     const int d0 = 32 * ks + 8 * kq;
     qf[ks] = d0 < dh ? *reinterpret_cast<const bf16x8*>(Q + d0) : zero8;
+    if constexpr (EXT == 2) attn_rotate8(p, b, qi, d0, qf[ks]);
   }
   f32x4 o[NDB];
 #pragma unroll
   for (int n = 0; n < NDB; ++n) o[n] = f32x4{0.f, 0.f, 0.f, 0.f};
   float m_run = -FLT_MAX, l_run = 0.f;
+  if constexpr (EXT == 2)
+    if (p.sink) { m_run = 0.f; l_run = kq == 0 ? 1.f : 0.f; }   // exp(0), counted by one of the row's four lane groups
   const float c = p.scale * LOG2E;
+  const int window = EXT == 2 ? p.window : 0;
+  int t0 = 0;
+  if (EXT == 2 && window) t0 = max(0, start + q0 - window + 1) >> 6;
   int nt = (p.S + 63) / 64;
   if (causal) {
     const int kv_end = min(p.S, start + q0 + 64);
@@ -492,7 +552,7 @@ __global__ __launch_bounds__(256) void attn_fwd_gen_kernel(AttnParams p, int dh)
   // transposing-read addresses of the V tile: lane j of a 16-lane group supplies row (j >> 2), columns 4 (j & 3) ..
   const unsigned vtr = vy_lds_addr(vt) + (4 * kq + (r16 >> 2)) * VPITCH + (4 * (r16 & 3)) * 2;
 
-  for (int t = 0; t < nt; ++t) {
+  for (int t = t0; t < nt; ++t) {
     const int k0 = t * 64;
     // stage the tile: 16-byte chunks, zero beyond the head width and beyond the last key
     bf16x8 kreg[KCPT], vreg[VCPT];
@@ -557,6 +617,7 @@ __global__ __launch_bounds__(256) void attn_fwd_gen_kernel(AttnParams p, int dh)
         const int kj = k0 + 16 * blk + 4 * kq + r;
         bool vis = kj < p.S;
         if (causal) vis = vis && kj <= qi + start;
+        if (EXT == 2 && window) vis = vis && kj > qi + start - window;
         if (haskp) vis = vis && kp[kj < p.S ? kj : 0] != 0;
         const float tv = vis ? sc[blk][r] : -INFINITY;
         sc[blk][r] = tv;
@@ -684,7 +745,7 @@ template <> struct RowVec<float> {
 // NWV waves per workgroup: 4, or 16 for decode launches with few (batch x head) rows -- an MQA / small-batch
 // decode has only B*h workgroups, each walking its keys in dependent trips; four times the waves = a quarter
 // of the trips, combined through LDS as before (no workspace, no second launch)
-template <typename T, int CPR, int NWV = 4, bool EXT = false>  // CPR = dh / VEC lanes per key row, power of two <= 64
+template <typename T, int CPR, int NWV = 4, int EXT = 0>  // CPR = dh / VEC lanes per key row, power of two <= 64
 __global__ __launch_bounds__(64 * NWV) void attn_rowwise_kernel(AttnParams p, int dh) {
   constexpr int VEC = RowVec<T>::VEC;
   constexpr int KPP = 64 / CPR;  // keys per wave pass
@@ -695,8 +756,9 @@ __global__ __launch_bounds__(64 * NWV) void attn_rowwise_kernel(AttnParams p, in
   const int kvh = head / (p.h / p.hk);
   const int grp = lane / CPR, ch = lane % CPR;
   const T* Q = (const T*)p.q + (int64_t)b * p.q_sb + (int64_t)head * p.q_sh + (int64_t)qi * p.q_sl;
-  const T* Kb = (const T*)p.k + (int64_t)b * p.k_sb + (int64_t)kvh * p.k_sh;
-  const T* Vb = (const T*)p.v + (int64_t)b * p.v_sb + (int64_t)kvh * p.v_sh;
+  const int bk = EXT == 2 && p.kv_by_slot && p.slots ? p.slots[b] : b;
+  const T* Kb = (const T*)p.k + (int64_t)bk * p.k_sb + (int64_t)kvh * p.k_sh;
+  const T* Vb = (const T*)p.v + (int64_t)bk * p.v_sb + (int64_t)kvh * p.v_sh;
   // head dims whose chunk count is not a power of two (SigLIP: 72 = 9 chunks of 8) run with the
   // next power of two lanes per key; the surplus lanes carry zeros and never store
   const bool ch_ok = ch * VEC < dh;
@@ -704,9 +766,16 @@ __global__ __launch_bounds__(64 * NWV) void attn_rowwise_kernel(AttnParams p, in
   const int dv = EXT ? p.dv : dh;          // EXT: value width, start position per sequence, output gate
   const bool chv_ok = EXT ? ch * VEC < dv : ch_ok;
   const int chv = EXT ? (chv_ok ? ch : 0) : chl;
-  const int start = EXT ? attn_start(p, b) : p.start_pos;
+  const int start = attn_first<EXT>(p, b);
   float qv[VEC];
   RowVec<T>::load(Q + chl * VEC, qv);
+  if constexpr (EXT == 2) {
+    attn_rotate<VEC>(p, b, qi, chl * VEC, qv);
+    if constexpr (VEC == 8) {   // rounded as the MFMA kernels' operand
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) qv[e] = vy_round_bf16(qv[e]);
+    }
+  }
   if (!ch_ok) {
 #pragma unroll
     for (int e = 0; e < VEC; ++e) qv[e] = 0.f;
@@ -720,8 +789,11 @@ __global__ __launch_bounds__(64 * NWV) void attn_rowwise_kernel(AttnParams p, in
   // every key is walked so a fully masked row reproduces the reference's uniform average.
   int S_eff = p.pos_dev ? *p.pos_dev + 1 : p.S;
   if (causal && !haskp && !hasadd) S_eff = min(S_eff, qi + start + 1);
+  const int S_lo = EXT == 2 && p.window ? max(0, qi + start - p.window + 1) : 0;
 
   float m = -FLT_MAX, l = 0.f, acc[VEC];
+  if constexpr (EXT == 2)
+    if (p.sink && wave == 0 && grp == 0) { m = 0.f; l = 1.f; }   // exp(0), counted by one key group
 #pragma unroll
   for (int e = 0; e < VEC; ++e) acc[e] = 0.f;
   // U key groups per trip: their K and V chunks are all requested before the first dot product, AND the
@@ -761,7 +833,7 @@ __global__ __launch_bounds__(64 * NWV) void attn_rowwise_kernel(AttnParams p, in
     }
   };
   raw16 kcur[U], vcur[U];
-  int j0 = wave * KPP;
+  int j0 = S_lo + wave * KPP;
   if (j0 < S_eff) request(j0, kcur, vcur);
   for (; j0 < S_eff; j0 += STRIDE) {
     raw16 knext[U], vnext[U];
@@ -849,7 +921,7 @@ __global__ __launch_bounds__(64 * NWV) void attn_rowwise_kernel(AttnParams p, in
   }
 }
 
-template <typename T, bool EXT = false>
+template <typename T, int EXT = 0>
 int launch_rowwise(const AttnParams& p, int dh, hipStream_t st, const char* who) {
   constexpr int VEC = RowVec<T>::VEC;
   if (dh % VEC || p.dv % VEC) VY_FAIL(VY_ERR_ARG, "%s: head_dim %d not a multiple of %d", who, p.dv % VEC ? p.dv : dh, VEC);
@@ -941,13 +1013,33 @@ extern "C" int vy_attn_fwd(const void* q, int64_t q_sb, int64_t q_sh, int64_t q_
 }
 
 namespace {
-template <int DHP>
+template <int DHP, int EXT>
 void gen_go(const AttnParams& p, int dh, int dv, dim3 grid, hipStream_t st) {
   const dim3 block(256);
-  if (dv <= 64) hipLaunchKernelGGL((attn_fwd_gen_kernel<DHP, 64, true>), grid, block, 0, st, p, dh);
-  else if (dv <= 96) hipLaunchKernelGGL((attn_fwd_gen_kernel<DHP, 96, true>), grid, block, 0, st, p, dh);
-  else if (dv <= 128) hipLaunchKernelGGL((attn_fwd_gen_kernel<DHP, 128, true>), grid, block, 0, st, p, dh);
-  else hipLaunchKernelGGL((attn_fwd_gen_kernel<DHP, 256, true>), grid, block, 0, st, p, dh);
+  if (dv <= 64) hipLaunchKernelGGL((attn_fwd_gen_kernel<DHP, 64, EXT>), grid, block, 0, st, p, dh);
+  else if (dv <= 96) hipLaunchKernelGGL((attn_fwd_gen_kernel<DHP, 96, EXT>), grid, block, 0, st, p, dh);
+  else if (dv <= 128) hipLaunchKernelGGL((attn_fwd_gen_kernel<DHP, 128, EXT>), grid, block, 0, st, p, dh);
+  else hipLaunchKernelGGL((attn_fwd_gen_kernel<DHP, 256, EXT>), grid, block, 0, st, p, dh);
+}
+
+template <int EXT>
+int launch_ex(const AttnParams& p, int dh, int dtype, hipStream_t st, const char* who) {
+  const int dv = p.dv;
+  if (dtype == VY_BF16 && !p.kv_by_slot && dh == dv && (dh == 64 || dh == 128)) {
+    const dim3 grid((unsigned)(p.h * p.B), (unsigned)((p.L + 127) / 128), 1), block(256);
+    if (dh == 64) hipLaunchKernelGGL((attn_fwd_mfma_kernel<64, EXT>), grid, block, 0, st, p);
+    else hipLaunchKernelGGL((attn_fwd_mfma_kernel<128, EXT>), grid, block, 0, st, p);
+  } else if (dtype == VY_BF16 && !p.kv_by_slot && dh <= 256 && dv <= 256) {
+    const dim3 grid((unsigned)(p.h * p.B), (unsigned)((p.L + 63) / 64), 1);
+    if (dh <= 64) gen_go<64, EXT>(p, dh, dv, grid, st);
+    else if (dh <= 96) gen_go<96, EXT>(p, dh, dv, grid, st);
+    else if (dh <= 128) gen_go<128, EXT>(p, dh, dv, grid, st);
+    else gen_go<256, EXT>(p, dh, dv, grid, st);
+  } else {
+    return dtype == VY_BF16 ? launch_rowwise<bf16, EXT>(p, dh, st, who) : launch_rowwise<float, EXT>(p, dh, st, who);
+  }
+  VY_CHECK_LAUNCH(who);
+  return VY_OK;
 }
 }  // namespace
 
@@ -955,7 +1047,7 @@ extern "C" int vy_attn_fwd_ex(const void* q, int64_t q_sb, int64_t q_sh, int64_t
                               int64_t k_sh, int64_t k_sl, const void* v, int64_t v_sb, int64_t v_sh, int64_t v_sl,
                               void* out, int64_t o_sb, int64_t o_sl, const void* gate, int64_t g_sb, int64_t g_sl,
                               const int32_t* start, const int32_t* slots, int64_t B, int h, int hk, int64_t L, int64_t S,
-                              int dh, int dv, float scale, int dtype, void* stream) {
+                              int dh, int dv, float scale, const vy_attn_window* win, int dtype, void* stream) {
   const char* who = "vy_attn_fwd_ex";
   AttnParams p{};
   p.q = q; p.q_sb = q_sb; p.q_sh = q_sh; p.q_sl = q_sl;
@@ -970,22 +1062,15 @@ extern "C" int vy_attn_fwd_ex(const void* q, int64_t q_sb, int64_t q_sh, int64_t
   const int vec = dtype == VY_BF16 ? 8 : 4;
   if (dv <= 0 || dh % vec || dv % vec) VY_FAIL(VY_ERR_ARG, "%s: head widths %d / %d must be multiples of %d", who, dh, dv, vec);
   if (gate && (g_sb % vec || g_sl % vec || (uintptr_t)gate % 16)) VY_FAIL(VY_ERR_ARG, "%s: gate rows must be 16-byte aligned", who);
-  hipStream_t st = (hipStream_t)stream;
-  if (dtype == VY_BF16 && dh == dv && (dh == 64 || dh == 128)) {
-    const dim3 grid((unsigned)(h * B), (unsigned)((L + 127) / 128), 1), block(256);
-    if (dh == 64) hipLaunchKernelGGL((attn_fwd_mfma_kernel<64, true>), grid, block, 0, st, p);
-    else hipLaunchKernelGGL((attn_fwd_mfma_kernel<128, true>), grid, block, 0, st, p);
-  } else if (dtype == VY_BF16 && dh <= 256 && dv <= 256) {
-    const dim3 grid((unsigned)(h * B), (unsigned)((L + 63) / 64), 1);
-    if (dh <= 64) gen_go<64>(p, dh, dv, grid, st);
-    else if (dh <= 96) gen_go<96>(p, dh, dv, grid, st);
-    else if (dh <= 128) gen_go<128>(p, dh, dv, grid, st);
-    else gen_go<256>(p, dh, dv, grid, st);
-  } else {
-    return dtype == VY_BF16 ? launch_rowwise<bf16, true>(p, dh, st, who) : launch_rowwise<float, true>(p, dh, st, who);
-  }
-  VY_CHECK_LAUNCH(who);
-  return VY_OK;
+  if (!win) return launch_ex<1>(p, dh, dtype, (hipStream_t)stream, who);
+  if (win->window < 0 || win->start_cap < 0) VY_FAIL(VY_ERR_ARG, "%s: window %d, start_cap %d", who, win->window, win->start_cap);
+  if (!(scale > 0.f)) VY_FAIL(VY_ERR_ARG, "%s: scale %g", who, (double)scale);
+  if (win->rope && (win->rope_dims < 0 || win->rope_dims % 2 || win->rope_dims > dh || win->rope_len < 1))
+    VY_FAIL(VY_ERR_ARG, "%s: rotary table of %d columns, %d positions for heads of %d", who, win->rope_dims, win->rope_len, dh);
+  p.window = win->window; p.sink = win->sink; p.kv_by_slot = win->kv_by_slot; p.start_cap = win->start_cap;
+  p.rope = (const float2*)win->rope; p.rope_half = win->rope_dims / 2; p.rope_len = win->rope_len;
+  if (p.rope_half == 0) p.rope = nullptr;
+  return launch_ex<2>(p, dh, dtype, (hipStream_t)stream, who);
 }
 
 int vy_attn_decode_ex(const void* q, int64_t q_sb, int64_t q_sh, const void* k, int64_t k_sb, int64_t k_sh,

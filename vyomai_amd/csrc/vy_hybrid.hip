@@ -1,13 +1,13 @@
 // Native decode driver (host code) of decoders that mix layer kinds: one call runs a whole single-token step of a batch of
-// sequences of different lengths -- embedding, every layer (latent attention over its latent cache, or decayed linear
-// attention over its fp32 state), gated MLPs, final norm and vocabulary product.  See include/vyom_hip.h
-// (vy_hybrid_decoder_step).
+// sequences of different lengths -- embedding, every layer (latent attention over its latent cache, decayed linear attention
+// over its fp32 state, or windowed attention over its ring), dense or routed feed-forward behind or beside the mixer, final
+// norm and vocabulary product.  See include/vyom_hip.h (vy_hybrid_decoder_step).
 #include "vy_common.h"
 
 int vy_residual_norm_ex(float* x, int64_t ldx, const void* y, int64_t ldy, const void* table, int64_t ldt, const int64_t* ids,
-                        int64_t V, int32_t* err, const float* w_post, float eps_post, const float* w_pre, float eps_pre, void* h,
-                        int64_t ldh, int64_t M, int64_t N, int64_t NP, int rms, int* advance, const int* slots, int n_adv,
-                        int dtype, void* stream);
+                        int64_t V, int32_t* err, float table_scale, const vy_routed_rows* routed, const float* w_post,
+                        float eps_post, const float* w_pre, float eps_pre, void* h, int64_t ldh, int64_t M, int64_t N, int64_t NP,
+                        int rms, int* advance, const int* slots, int n_adv, int dtype, void* stream);
 int vy_dec_gemv1(const void* x, const void* w, const void* bias, const void* residual, void* y, int N, int K, int prescaled,
                  float eps, hipStream_t st);
 int vy_dec_gemv1_gated(const void* x, const void* wgu, void* y, int I, int K, int act, int prescaled, float eps, hipStream_t st);
@@ -18,7 +18,7 @@ namespace {
 
 int64_t up(int64_t x) { return (x + 255) / 256 * 256; }
 
-struct Sizes { int64_t in, q, cq, ao, o, gu, ff, latent_ws; };   // widest of each over the layers
+struct Sizes { int64_t in, q, cq, ao, o, gu, ff, mix_ws, top, moe_ws; };   // widest of each over the layers
 
 Sizes sizes_of(const vy_hybrid_plan* p) {
   Sizes s{};
@@ -26,16 +26,25 @@ Sizes sizes_of(const vy_hybrid_plan* p) {
   for (int l = 0; l < p->num_layers; ++l) {
     const vy_hybrid_layer& L = p->layers[l];
     mx(s.in, L.n_in);
-    mx(s.ao, (int64_t)L.heads * L.vdim);
+    const bool parallel = L.form == VY_FORM_PARALLEL;
+    mx(s.ao, (int64_t)L.heads * L.vdim + (parallel ? L.ff : 0));
     if (L.mixer == VY_MIX_LATENT) {
       mx(s.q, (int64_t)L.heads * L.dim);
       mx(s.cq, L.q_rank_p);
-      mx(s.latent_ws, vy_latent_decode_ws_bytes(p->B, L.heads, L.kv_rank_p));
+      mx(s.mix_ws, vy_latent_decode_ws_bytes(p->B, L.heads, L.kv_rank_p));
+    } else if (L.mixer == VY_MIX_WINDOW) {
+      mx(s.mix_ws, vy_window_decode_ws_bytes(p->B, L.heads, L.kv_heads, L.vdim, L.cap));
     } else {
       mx(s.o, (int64_t)L.heads * L.vdim);
     }
-    mx(s.gu, 2 * (int64_t)L.ff);
-    mx(s.ff, L.ff);
+    if (!parallel) {
+      mx(s.gu, 2 * (int64_t)L.ff);
+      mx(s.ff, L.ff);
+    }
+    if (L.moe) {
+      mx(s.top, L.moe->top);
+      mx(s.moe_ws, vy_moe_ws_bytes(L.moe, p->B, p->dtype));
+    }
   }
   return s;
 }
@@ -49,16 +58,22 @@ int product(const vy_hybrid_plan* p, const void* x, const void* w, void* y, int6
   return vy_linear_fwd(x, K, w, K, nullptr, nullptr, 0, y, ldy, nullptr, p->B, N, K, VY_ACT_NONE, p->dtype, stream);
 }
 
+// packed [gate | up] rows -> activation rows
+int activation(const vy_hybrid_plan* p, const vy_hybrid_layer& L, const void* gu, int64_t ldg, void* act, int64_t lda, void* stream) {
+  if (L.clamped) return vy_clamped_act_fwd(gu, ldg, act, lda, p->B, L.ff, L.limit, L.alpha, p->dtype, stream);
+  return vy_gated_act_fwd(gu, ldg, act, lda, p->B, L.ff, p->act, p->dtype, stream);
+}
+
 int gated(const vy_hybrid_plan* p, const vy_hybrid_layer& L, const void* x, void* gu, void* act, void* stream) {
-  if (p->dtype == VY_BF16 && p->B == 1) {
+  if (!L.clamped && p->dtype == VY_BF16 && p->B == 1) {
     const int rc = vy_dec_gemv1_gated(x, L.w_gu, act, L.ff, p->dp, p->act, 0, 0.f, (hipStream_t)stream);
     if (rc != VY_ERR_UNSUPPORTED) return rc;
   }
-  if (p->dtype == VY_BF16 && p->B <= 4)
+  if (!L.clamped && p->dtype == VY_BF16 && p->B <= 4)
     return vy_gemv_gated(x, p->dp, L.w_gu, p->dp, nullptr, 0.f, act, L.ff, p->B, L.ff, p->dp, p->act, stream);
   const int rc = vy_linear_fwd(x, p->dp, L.w_gu, p->dp, nullptr, nullptr, 0, gu, 2 * (int64_t)L.ff, nullptr, p->B,
                                2 * (int64_t)L.ff, p->dp, VY_ACT_NONE, p->dtype, stream);
-  return rc ? rc : vy_gated_act_fwd(gu, 2 * (int64_t)L.ff, act, L.ff, p->B, L.ff, p->act, p->dtype, stream);
+  return rc ? rc : activation(p, L, gu, 2 * (int64_t)L.ff, act, L.ff, stream);
 }
 
 }  // namespace
@@ -68,7 +83,8 @@ extern "C" int64_t vy_hybrid_ws_bytes(const vy_hybrid_plan* p) {
   const Sizes s = sizes_of(p);
   const int64_t e = p->dtype == VY_BF16 ? 2 : 4, B = p->B;
   return up(B * p->dp * 4) + 2 * up(B * p->dp * e) + up(B * s.in * e) + up(B * s.q * e) + up(B * s.cq * e) +
-         up(B * s.ao * e) + up(B * s.o * e) + up(B * s.gu * e) + up(B * s.ff * e) + up(s.latent_ws);
+         up(B * s.ao * e) + up(B * s.o * e) + up(B * s.gu * e) + up(B * s.ff * e) + up(s.mix_ws) + up(B * s.top * p->dp * e) +
+         3 * up(B * s.top * 4) + up(s.moe_ws);
 }
 
 extern "C" int vy_hybrid_decoder_step(const vy_hybrid_plan* p, const int64_t* ids, const int32_t* slots, int32_t* lengths,
@@ -91,18 +107,24 @@ extern "C" int vy_hybrid_decoder_step(const vy_hybrid_plan* p, const int64_t* id
   void* o = take(B * s.o * e);
   void* gu = take(B * s.gu * e);
   void* act = take(B * s.ff * e);
-  void* lws = take(s.latent_ws);
+  void* mws = take(s.mix_ws);
+  void* erows = take(B * s.top * dp * e);
+  int32_t* eids = (int32_t*)take(B * s.top * 4);
+  int32_t* epos = (int32_t*)take(B * s.top * 4);
+  float* ew = (float*)take(B * s.top * 4);
+  void* ews = take(s.moe_ws);
   int rc;
-  auto norm = [&](const void* yy, const float* post, const float* pre, bool last) {
-    return vy_residual_norm_ex(x, dp, yy, dp, p->embed, dp, yy ? nullptr : ids, p->vocab, p->err, post, p->eps, pre, p->eps, h,
-                               dp, B, p->d, dp, p->rms, last ? lengths : nullptr, slots, last ? (int)B : 0, p->dtype, stream);
+  auto norm = [&](const void* yy, const vy_routed_rows* routed, const float* post, const float* pre, bool last) {
+    return vy_residual_norm_ex(x, dp, yy, dp, p->embed, dp, yy || routed ? nullptr : ids, p->vocab, p->err, p->embed_scale, routed,
+                               post, p->eps, pre, p->eps, h, dp, B, p->d, dp, p->rms, last ? lengths : nullptr, slots,
+                               last ? (int)B : 0, p->dtype, stream);
   };
-  if ((rc = norm(nullptr, nullptr, p->layers[0].norm1, false))) return rc;
+  if ((rc = norm(nullptr, nullptr, nullptr, p->layers[0].norm1, false))) return rc;
   for (int l = 0; l < p->num_layers; ++l) {
     const vy_hybrid_layer& L = p->layers[l];
-    const bool last = l + 1 == p->num_layers;
+    const bool last = l + 1 == p->num_layers, parallel = L.form == VY_FORM_PARALLEL;
     const float* next = last ? p->final_norm : p->layers[l + 1].norm1;
-    const int64_t nv = (int64_t)L.heads * L.vdim, nk = (int64_t)L.heads * L.dim;
+    const int64_t nv = (int64_t)L.heads * L.vdim, nk = (int64_t)L.heads * L.dim, na = nv + (parallel ? L.ff : 0);
     if ((rc = product(p, h, L.w_in, in, L.n_in, L.n_in, dp, stream))) return rc;
     if (L.mixer == VY_MIX_LATENT) {
       if (max_keys > L.cap) VY_FAIL(VY_ERR_ARG, "%s: %ld keys exceed the cache capacity %d", who, (long)max_keys, L.cap);
@@ -111,24 +133,45 @@ extern "C" int vy_hybrid_decoder_step(const vy_hybrid_plan* p, const int64_t* id
                                stream))) return rc;
       if ((rc = product(p, cq, L.w_uq, q, nk, nk, L.q_rank_p, stream))) return rc;
       const char* gate = (const char*)in + ((int64_t)L.q_rank_p + L.kv_rank_p) * e;
-      if ((rc = vy_latent_decode(q, nk, L.w_ukt, L.w_uv, L.cache, L.c_ss, L.c_st, slots, lengths, max_keys, ao, nv, gate, L.n_in,
-                                 (int)B, L.heads, L.dim, L.vdim, L.kv_rank_p, L.scale, lws, s.latent_ws, p->dtype, stream)))
+      if ((rc = vy_latent_decode(q, nk, L.w_ukt, L.w_uv, L.cache, L.c_ss, L.c_st, slots, lengths, max_keys, ao, na, gate, L.n_in,
+                                 (int)B, L.heads, L.dim, L.vdim, L.kv_rank_p, L.scale, mws, s.mix_ws, p->dtype, stream)))
         return rc;
+    } else if (L.mixer == VY_MIX_WINDOW) {
+      const int64_t gk = (int64_t)L.kv_heads * L.dim, gv = (int64_t)L.kv_heads * L.vdim;
+      if ((rc = vy_window_decode(in, L.n_in, 0, nk, nk + gk, nk + gk + gv, L.cache, L.c_ss, L.c_sh, L.cap, L.rope, L.rope_dims,
+                                 L.rope_len, slots, lengths, max_keys, ao, na, B, L.heads, L.kv_heads, L.dim, L.vdim, L.scale,
+                                 L.sink, mws, s.mix_ws, p->dtype, stream))) return rc;
     } else {
       if ((rc = vy_decay_attn(in, L.n_in, 0, nk, 2 * nk, L.state, L.decay_pow, slots, lengths, nullptr, o, nv, B, 1, L.heads, L.dim,
                               L.vdim, 1, nullptr, 0, p->dtype, stream))) return rc;
       const char* gate = (const char*)in + (2 * nk + nv) * e;
-      if ((rc = vy_rmsnorm_gate(o, nv, L.mix_norm, gate, L.n_in, ao, nv, B, L.mix_n, nv, p->eps, p->dtype, stream))) return rc;
+      if ((rc = vy_rmsnorm_gate(o, nv, L.mix_norm, gate, L.n_in, ao, na, B, L.mix_n, nv, p->eps, p->dtype, stream))) return rc;
+    }
+    const vy_routed_rows rows{erows, dp, epos, ew, L.moe ? L.moe->top : 0};
+    const vy_routed_rows* routed = L.moe ? &rows : nullptr;
+    auto experts = [&]() {
+      return L.moe ? vy_moe_fwd(L.moe, h, dp, B, nullptr, 1, erows, dp, eids, epos, ew, ews, s.moe_ws, p->dtype, stream) : VY_OK;
+    };
+    if (parallel) {
+      if (L.ff && (rc = activation(p, L, (const char*)in + (L.n_in - 2 * (int64_t)L.ff) * e, L.n_in, (char*)ao + nv * e, na, stream)))
+        return rc;
+      if ((rc = experts())) return rc;
+      if ((rc = product(p, ao, L.w_o, y, dp, dp, na, stream))) return rc;
+      if ((rc = norm(y, routed, L.norm1b, next, last))) return rc;
+      continue;
     }
     if ((rc = product(p, ao, L.w_o, y, dp, dp, nv, stream))) return rc;
+    if (!L.ff && !L.moe) {
+      if ((rc = norm(y, nullptr, L.norm1b, next, last))) return rc;
+      continue;
+    }
+    if ((rc = norm(y, nullptr, L.norm1b, L.norm2, false))) return rc;
     if (L.ff) {
-      if ((rc = norm(y, L.norm1b, L.norm2, false))) return rc;
       if ((rc = gated(p, L, h, gu, act, stream))) return rc;
       if ((rc = product(p, act, L.w_down, y, dp, dp, L.ff, stream))) return rc;
-      if ((rc = norm(y, L.norm2b, next, last))) return rc;
-    } else if ((rc = norm(y, L.norm1b, next, last))) {
-      return rc;
     }
+    if ((rc = experts())) return rc;
+    if ((rc = norm(L.ff ? y : nullptr, routed, L.norm2b, next, last))) return rc;
   }
   return product(p, h, p->head, logits, ldv, p->vocab, dp, stream);
 }

@@ -3,7 +3,8 @@
 // every operand and kept zero in every result), so widths that are not a multiple of 8 run on the same kernels.
 //
 //   vy_residual_norm   x += norm(y) * w_post  (or x = table[ids], or x += y) and h = norm(x) * w_pre, one pass: the
-//                      end of one sublayer and the beginning of the next
+//                      end of one sublayer and the beginning of the next.  vy_residual_norm_routed: y also collects the
+//                      weighted rows of a token's experts
 //   vy_latent_norm     the two RMS norms behind a packed [query latent | key/value latent | ...] projection; the
 //                      key/value latent also goes to its cache rows
 //   vy_rmsnorm_gate    RMSNorm(x) * w * sigmoid(gate)
@@ -58,6 +59,8 @@ struct ResNormArgs {
   void* h; int64_t ldh;
   int64_t M; int N, NP; float eps_post, eps_pre;
   int* advance; const int* slots; int n_adv;   // decode: advance[slots[i]] += 1 once per step (workgroup 0)
+  float table_scale;                           // x = table_scale * table[ids]
+  const void* er; int64_t lder; const int* epos; const float* ew; int top;   // routed rows: y += sum_k ew[row][k] er[epos[row][k]]
 };
 
 // statistics of v (CH quads per thread) over the row's first N columns, then v <- (v - mean) * rstd (RMS: mean = 0)
@@ -85,7 +88,7 @@ __device__ __forceinline__ void row_stats(const float (&v)[CH][4], int t, int N,
   rstd = rsqrt_refined(row_sum<TPR>(q, red, slot + 1) / (float)N + eps);
 }
 
-template <typename T, int TPR, int CH, bool RMS>
+template <typename T, int TPR, int CH, bool RMS, bool ROUTED>
 __global__ __launch_bounds__(256) void residual_norm_kernel(ResNormArgs p) {
   __shared__ float red[16];
   const int t = TPR == 64 ? threadIdx.x & 63 : threadIdx.x;
@@ -113,7 +116,31 @@ __global__ __launch_bounds__(256) void residual_norm_kernel(ResNormArgs p) {
       if (!p.ids) load4<float>(xr + col, x[c]);
     }
   }
-  if (p.ids || p.y) {
+  if (p.ids) {
+#pragma unroll
+    for (int c = 0; c < CH; ++c)
+#pragma unroll
+      for (int e = 0; e < 4; ++e) y[c][e] *= p.table_scale;
+  }
+  if constexpr (ROUTED) {
+#pragma unroll 4
+    for (int k = 0; k < p.top; ++k) {
+      const int er = p.epos ? p.epos[row * p.top + k] : (int)(row * p.top + k);
+      const float w = er >= 0 ? p.ew[row * p.top + k] : 0.f;
+      const T* src_e = (const T*)p.er + (int64_t)(er >= 0 ? er : 0) * p.lder;
+#pragma unroll
+      for (int c = 0; c < CH; ++c) {
+        const int col = (t + TPR * c) * 4;
+        if (col < p.NP && er >= 0) {
+          float v[4];
+          load4<T>(src_e + col, v);
+#pragma unroll
+          for (int e = 0; e < 4; ++e) y[c][e] = fmaf(w, v[e], y[c][e]);
+        }
+      }
+    }
+  }
+  if (ROUTED || p.ids || p.y) {
     float mean = 0.f, rstd = 1.f;
     const bool post = !p.ids && p.w_post;
     if (post) row_stats<TPR, CH, RMS>(y, t, p.N, p.NP, p.eps_post, red, 0, mean, rstd);
@@ -152,25 +179,33 @@ __global__ __launch_bounds__(256) void residual_norm_kernel(ResNormArgs p) {
   }
 }
 
-template <typename T, bool RMS>
+template <typename T, bool RMS, bool ROUTED>
 int residual_norm_go(const ResNormArgs& a, hipStream_t st) {
   const dim3 block(256);
+#define RN_GO(TPR, CH) hipLaunchKernelGGL((residual_norm_kernel<T, TPR, CH, RMS, ROUTED>), grid, block, 0, st, a)
   // wide enough batches keep every CU busy with a wave per row; a decode step gives each row a workgroup
   if (a.M >= 1024 && a.NP <= 2048) {
     const dim3 grid((unsigned)vy_cdiv(a.M, 4));
-    if (a.NP <= 512) hipLaunchKernelGGL((residual_norm_kernel<T, 64, 2, RMS>), grid, block, 0, st, a);
-    else if (a.NP <= 1024) hipLaunchKernelGGL((residual_norm_kernel<T, 64, 4, RMS>), grid, block, 0, st, a);
-    else hipLaunchKernelGGL((residual_norm_kernel<T, 64, 8, RMS>), grid, block, 0, st, a);
+    if (a.NP <= 512) RN_GO(64, 2);
+    else if (a.NP <= 1024) RN_GO(64, 4);
+    else RN_GO(64, 8);
     return 0;
   }
   const dim3 grid((unsigned)a.M);
-  if (a.NP <= 1024) hipLaunchKernelGGL((residual_norm_kernel<T, 256, 1, RMS>), grid, block, 0, st, a);
-  else if (a.NP <= 2048) hipLaunchKernelGGL((residual_norm_kernel<T, 256, 2, RMS>), grid, block, 0, st, a);
-  else if (a.NP <= 4096) hipLaunchKernelGGL((residual_norm_kernel<T, 256, 4, RMS>), grid, block, 0, st, a);
-  else if (a.NP <= 8192) hipLaunchKernelGGL((residual_norm_kernel<T, 256, 8, RMS>), grid, block, 0, st, a);
-  else if (a.NP <= 16384) hipLaunchKernelGGL((residual_norm_kernel<T, 256, 16, RMS>), grid, block, 0, st, a);
+  if (a.NP <= 1024) RN_GO(256, 1);
+  else if (a.NP <= 2048) RN_GO(256, 2);
+  else if (a.NP <= 4096) RN_GO(256, 4);
+  else if (a.NP <= 8192) RN_GO(256, 8);
+  else if (a.NP <= 16384) RN_GO(256, 16);
   else return 1;
+#undef RN_GO
   return 0;
+}
+
+template <typename T>
+int residual_norm_any(const ResNormArgs& a, int rms, hipStream_t st) {
+  if (a.er) return rms ? residual_norm_go<T, true, true>(a, st) : residual_norm_go<T, false, true>(a, st);
+  return rms ? residual_norm_go<T, true, false>(a, st) : residual_norm_go<T, false, false>(a, st);
 }
 
 struct LatentNormArgs {
@@ -275,11 +310,11 @@ __global__ __launch_bounds__(256) void rmsnorm_gate_kernel(const T* __restrict__
 
 }  // namespace
 
-// internal: the step driver also advances the sequence lengths in this launch
+// internal: the step driver also advances the sequence lengths in this launch (advance[slots[i]] += 1 for i < n_adv)
 int vy_residual_norm_ex(float* x, int64_t ldx, const void* y, int64_t ldy, const void* table, int64_t ldt, const int64_t* ids,
-                        int64_t V, int32_t* err, const float* w_post, float eps_post, const float* w_pre, float eps_pre, void* h,
-                        int64_t ldh, int64_t M, int64_t N, int64_t NP, int rms, int* advance, const int* slots, int n_adv,
-                        int dtype, void* stream) {
+                        int64_t V, int32_t* err, float table_scale, const vy_routed_rows* routed, const float* w_post,
+                        float eps_post, const float* w_pre, float eps_pre, void* h, int64_t ldh, int64_t M, int64_t N, int64_t NP,
+                        int rms, int* advance, const int* slots, int n_adv, int dtype, void* stream) {
   const char* who = "vy_residual_norm";
   if (!x || M <= 0 || N <= 0 || NP < N) VY_FAIL(VY_ERR_ARG, "%s: bad arguments", who);
   if (NP % 4 || ldx % 4 || ldy % 4 || ldt % 4 || ldh % 4 || ldx < NP) VY_FAIL(VY_ERR_ARG, "%s: padded widths and row strides must be multiples of 4", who);
@@ -289,10 +324,16 @@ int vy_residual_norm_ex(float* x, int64_t ldx, const void* y, int64_t ldy, const
   a.x = x; a.ldx = ldx; a.y = y; a.ldy = ldy; a.table = table; a.ldt = ldt; a.ids = ids; a.V = V; a.err = err;
   a.w_post = w_post; a.w_pre = w_pre; a.h = h; a.ldh = ldh; a.M = M; a.N = (int)N; a.NP = (int)NP;
   a.eps_post = eps_post; a.eps_pre = eps_pre; a.advance = advance; a.slots = slots; a.n_adv = n_adv;
+  a.table_scale = table_scale;
+  if (routed) {
+    if (ids || !routed->rows || !routed->weight || routed->top <= 0 || routed->ld % 4 || routed->ld < NP)
+      VY_FAIL(VY_ERR_ARG, "%s: bad routed rows", who);
+    a.er = routed->rows; a.lder = routed->ld; a.epos = routed->pos; a.ew = routed->weight; a.top = routed->top;
+  }
   hipStream_t st = (hipStream_t)stream;
   int rc;
-  if (dtype == VY_BF16) rc = rms ? residual_norm_go<bf16, true>(a, st) : residual_norm_go<bf16, false>(a, st);
-  else if (dtype == VY_F32) rc = rms ? residual_norm_go<float, true>(a, st) : residual_norm_go<float, false>(a, st);
+  if (dtype == VY_BF16) rc = residual_norm_any<bf16>(a, rms, st);
+  else if (dtype == VY_F32) rc = residual_norm_any<float>(a, rms, st);
   else VY_FAIL(VY_ERR_ARG, "%s: bad dtype %d", who, dtype);
   if (rc) VY_FAIL(VY_ERR_UNSUPPORTED, "%s: width %ld", who, (long)NP);
   VY_CHECK_LAUNCH(who);
@@ -303,8 +344,17 @@ extern "C" int vy_residual_norm(float* x, int64_t ldx, const void* y, int64_t ld
                                 const int64_t* ids, int64_t V, int32_t* err_flag, const float* w_post, float eps_post,
                                 const float* w_pre, float eps_pre, void* h, int64_t ldh, int64_t M, int64_t N, int64_t NP,
                                 int rms, int dtype, void* stream) {
-  return vy_residual_norm_ex(x, ldx, y, ldy, table, ldt, ids, V, err_flag, w_post, eps_post, w_pre, eps_pre, h, ldh, M, N, NP,
-                             rms, nullptr, nullptr, 0, dtype, stream);
+  return vy_residual_norm_ex(x, ldx, y, ldy, table, ldt, ids, V, err_flag, 1.f, nullptr, w_post, eps_post, w_pre, eps_pre, h,
+                             ldh, M, N, NP, rms, nullptr, nullptr, 0, dtype, stream);
+}
+
+extern "C" int vy_residual_norm_routed(float* x, int64_t ldx, const void* y, int64_t ldy, const void* table, int64_t ldt,
+                                       const int64_t* ids, int64_t V, int32_t* err_flag, float table_scale,
+                                       const vy_routed_rows* routed, const float* w_post, float eps_post, const float* w_pre,
+                                       float eps_pre, void* h, int64_t ldh, int64_t M, int64_t N, int64_t NP, int rms, int dtype,
+                                       void* stream) {
+  return vy_residual_norm_ex(x, ldx, y, ldy, table, ldt, ids, V, err_flag, table_scale, routed, w_post, eps_post, w_pre, eps_pre,
+                             h, ldh, M, N, NP, rms, nullptr, nullptr, 0, dtype, stream);
 }
 
 extern "C" int vy_latent_norm(const void* p, int64_t ldp, const float* w_q, void* q_out, int64_t ldq, int32_t nq, int32_t npq,

@@ -11,6 +11,7 @@ import torch
 
 from . import _lib
 from .layers.attention import _shadow
+from .ops import up8
 
 
 class VyDecodeLayer(C.Structure):
@@ -257,20 +258,22 @@ class GemmaDecodePlan:
 
 class VyHybridLayer(C.Structure):
     _fields_ = [(n, C.c_int32) for n in ("mixer", "heads", "dim", "vdim", "n_in", "ff", "q_rank", "q_rank_p", "kv_rank",
-                                         "kv_rank_p", "cap", "mix_n")] + [("scale", C.c_float)] + \
+                                         "kv_rank_p", "cap", "mix_n", "form", "clamped", "kv_heads", "rope_dims", "rope_len", "sink")] + \
+               [(n, C.c_float) for n in ("scale", "limit", "alpha")] + \
                [(n, C.c_void_p) for n in ("norm1", "norm1b", "norm2", "norm2b", "w_in", "w_o", "w_gu", "w_down", "q_norm",
                                           "c_norm", "w_uq", "w_ukt", "w_uv", "cache")] + \
-               [("c_ss", C.c_int64), ("c_st", C.c_int64)] + \
-               [(n, C.c_void_p) for n in ("state", "decay_pow", "mix_norm")]
+               [(n, C.c_int64) for n in ("c_ss", "c_sh", "c_st")] + \
+               [(n, C.c_void_p) for n in ("state", "decay_pow", "mix_norm", "rope")] + [("moe", C.POINTER(_lib.VyMoe))]
 
 
 class VyHybridPlan(C.Structure):
     _fields_ = [(n, C.c_int32) for n in ("num_layers", "B", "d", "dp", "vocab", "dtype", "rms", "act")] + \
-               [("eps", C.c_float), ("layers", C.POINTER(VyHybridLayer))] + \
+               [("eps", C.c_float), ("embed_scale", C.c_float), ("layers", C.POINTER(VyHybridLayer))] + \
                [(n, C.c_void_p) for n in ("embed", "head", "final_norm", "err", "ws")] + [("ws_bytes", C.c_int64)]
 
 
-MIX_LATENT, MIX_DECAY = 0, 1
+MIX_LATENT, MIX_DECAY, MIX_WINDOW = 0, 1, 2
+FORMS = {"sandwich": 0, "parallel": 1}
 
 
 class HybridDecodePlan:
@@ -283,11 +286,16 @@ class HybridDecodePlan:
         acts = set()
         for i, layer in enumerate(model.layers):
             m, L = layer.mixer, arr[i]
-            n, p = layer.packed(), m.packed()
+            n = layer.packed()
+            parallel = layer.form == "parallel"
+            L.form = FORMS[layer.form]
+            # (a parallel layer holds the stacked products of mixer and dense feed-forward itself)
+            p = n if parallel and m.kind == "window" else m.packed()
             self.keep += [n, p]
-            L.heads, L.dim, L.vdim = m.heads, (m.dim + 7) // 8 * 8, (m.vdim + 7) // 8 * 8
-            L.w_in, L.n_in, L.w_o = _ptr(p.w_in), p.w_in.shape[0], _ptr(p.w_o)
-            L.norm1, L.norm1b = _ptr(n.norm1), _ptr(n.norm1b)
+            L.heads, L.dim, L.vdim = m.heads, up8(m.dim), up8(m.vdim)
+            w = n if parallel else p
+            L.w_in, L.n_in, L.w_o = _ptr(w.w_in), w.w_in.shape[0], _ptr(w.w_o)
+            L.norm1, L.norm1b = _ptr(n.norm1), None if parallel else _ptr(n.norm1b)
             buf = cache.buffers[i]
             self.keep.append(buf)
             if m.kind == "latent":
@@ -296,14 +304,31 @@ class HybridDecodePlan:
                 L.q_norm, L.c_norm = _ptr(p.q_norm), _ptr(p.c_norm)
                 L.w_uq, L.w_ukt, L.w_uv = _ptr(p.w_uq), _ptr(p.w_ukt), _ptr(p.w_uv)
                 L.cache, L.c_ss, L.c_st, L.cap = buf.data_ptr(), buf.stride(0), buf.stride(1), buf.shape[1]
+            elif m.kind == "window":
+                L.mixer, L.scale, L.kv_heads, L.sink = MIX_WINDOW, m.scale, m.kv_heads, int(m.sink)
+                L.cache, L.c_ss, L.c_sh, L.cap = buf.data_ptr(), buf.stride(0), buf.stride(1), buf.shape[2]
+                table = m.rotary.table(cache.capacity, model.device)
+                self.keep.append(table)
+                L.rope, L.rope_dims, L.rope_len = _ptr(table), m.rotary.dims, table.shape[0] if table is not None else 0
             else:
                 L.mixer, L.state, L.decay_pow = MIX_DECAY, buf.data_ptr(), _ptr(p.decay_pow)
                 L.mix_norm, L.mix_n = _ptr(p.norm), m.heads * m.vdim
             if layer.mlp is not None:
-                f = layer.mlp.packed()
-                self.keep.append(f)
-                L.norm2, L.norm2b, L.w_gu, L.w_down, L.ff = _ptr(n.norm2), _ptr(n.norm2b), _ptr(f.w_gu), _ptr(f.w_down), f.w_down.shape[1]
-                acts.add(layer.mlp.act)
+                dense = layer.mlp.dense
+                if not parallel:
+                    L.norm2, L.norm2b = _ptr(n.norm2), _ptr(n.norm2b)
+                if dense is not None:
+                    L.ff, L.clamped, L.limit, L.alpha = up8(dense.inner), int(dense.clamped), dense.limit, dense.alpha
+                    if not parallel:
+                        f = dense.packed()
+                        self.keep.append(f)
+                        L.w_gu, L.w_down = _ptr(f.w_gu), _ptr(f.w_down)
+                    if not dense.clamped:
+                        acts.add(dense.act)
+                if layer.mlp is not dense:
+                    f = layer.mlp.packed()
+                    self.keep.append(f)
+                    L.moe = C.pointer(f.desc)
         if len(acts) > 1:
             raise ValueError("the decode step takes one MLP activation")
         t = model.packed()
@@ -312,6 +337,7 @@ class HybridDecodePlan:
         p = VyHybridPlan()
         p.num_layers, p.B, p.d, p.dp, p.vocab = len(model.layers), batch, model.width, t.embed.shape[1], model.vocab
         p.dtype, p.rms, p.act, p.eps = _lib.dtype_code(model.dtype), int(model.rms), acts.pop() if acts else _lib.ACT_NONE, model.eps
+        p.embed_scale = model.embed_scale
         p.layers = C.cast(arr, C.POINTER(VyHybridLayer))
         p.embed, p.head, p.final_norm = _ptr(t.embed), _ptr(t.head), _ptr(t.final_norm)
         nbytes = lib.vy_hybrid_ws_bytes(C.byref(p))

@@ -6,13 +6,13 @@ MI355X: two MFMA GEMM launches -- bias+GELU in the first epilogue, bias+dropout+
 second -- and one LayerNorm launch."""
 from __future__ import annotations
 
-from typing import Union
+from typing import Optional, Union
 
 import torch
 import torch.nn as nn
 
 from .. import ops
-from .._lib import ACT_GELU_ERF, ACT_GELU_TANH, ACT_SILU
+from .._lib import ACT_GELU_ERF, ACT_GELU_TANH, ACT_SILU, VyMoe
 from ..ops import up8
 from .packing import Packed, pad2
 
@@ -49,22 +49,85 @@ _GATED_ACT = {"silu": ACT_SILU, "gelu_tanh": ACT_GELU_TANH, "gelu": ACT_GELU_ERF
 
 
 class GatedFeedForward(nn.Module):
-    """down(act(gate(x)) * up(x)), no biases: one packed [gate; up] product, the gated activation, one product."""
+    """down(act(gate(x)) * up(x)), no biases: one packed [gate; up] product, the gated activation, one product.
+    act "clamped": with g = min(gate, limit), u = clamp(up, -limit, limit): down(g sigmoid(alpha g) (u + 1))."""
 
-    def __init__(self, width: int, inner: int, act: str = "silu") -> None:
+    def __init__(self, width: int, inner: int, act: str = "silu", limit: float = 0.0, alpha: float = 1.702) -> None:
         super().__init__()
-        self.width, self.inner, self.act = width, inner, _GATED_ACT[act]
+        self.width, self.inner, self.limit, self.alpha = width, inner, float(limit), float(alpha)
+        self.clamped = act == "clamped"
+        self.act = None if self.clamped else _GATED_ACT[act]
         self.gate = nn.Linear(width, inner, bias=False)
         self.up = nn.Linear(width, inner, bias=False)
         self.down = nn.Linear(inner, width, bias=False)
 
+    def matrices(self):
+        """Padded [gate; up] and down matrices."""
+        dp, ip = up8(self.width), up8(self.inner)
+        return torch.cat([pad2(self.gate.weight, ip, dp), pad2(self.up.weight, ip, dp)]), pad2(self.down.weight, dp, ip)
+
     def packed(self) -> Packed:
         def build(p: Packed) -> None:
-            dp, ip = up8(self.width), up8(self.inner)
-            p.w_gu = torch.cat([pad2(self.gate.weight, ip, dp), pad2(self.up.weight, ip, dp)]).contiguous()
-            p.w_down = pad2(self.down.weight, dp, ip).contiguous()
+            p.w_gu, p.w_down = (w.contiguous() for w in self.matrices())
         return Packed.of(self, list(self.parameters()), build)
+
+    def activation(self, gate_up: torch.Tensor, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+        if self.clamped:
+            return ops.clamped_act(gate_up, self.limit, self.alpha, out)
+        return ops.gated_act(gate_up, self.act, out)
 
     def forward(self, h: torch.Tensor) -> torch.Tensor:
         p = self.packed()
-        return ops.linear(ops.gated_act(ops.linear(h, p.w_gu), self.act), p.w_down)
+        return ops.linear(self.activation(ops.linear(h, p.w_gu)), p.w_down)
+
+    # what a layer asks of its feed-forward: the part that runs on every token, and the routed rows beside it
+    @property
+    def dense(self) -> Optional["GatedFeedForward"]:
+        return self
+
+    def routed(self, h: torch.Tensor, L: int = 1, count: Optional[torch.Tensor] = None) -> Optional["ops.Routed"]:
+        return None
+
+
+class MixtureFeedForward(nn.Module):
+    """`top` of `experts` clamped gated feed-forwards per token and (shared may be None) one dense one for every token.
+
+    Router scores are softmax(router(x)) in fp32; experts form `groups` equal groups of neighbours and only those of the `keep`
+    groups with the best largest score can be chosen; the chosen scores are normalised to sum 1 and multiplied by `scale`.
+    The experts' weights are one tensor each (experts first); once packed, they are views of the packed storage, so there is one
+    copy of them in memory."""
+
+    def __init__(self, width: int, experts: int, top: int, inner: int, limit: float, groups: int = 1, keep: int = 1,
+                 scale: float = 1.0, alpha: float = 1.702, shared: Optional[GatedFeedForward] = None) -> None:
+        super().__init__()
+        if experts < 1 or groups < 1 or experts % groups or not 1 <= keep <= groups or not 1 <= top <= keep * (experts // groups):
+            raise ValueError(f"{top} of {experts} experts, {keep} of {groups} groups")
+        self.width, self.experts, self.top, self.inner, self.limit, self.alpha = width, experts, top, inner, float(limit), float(alpha)
+        self.groups, self.keep, self.scale = groups, keep, float(scale)
+        self.router = nn.Linear(width, experts, bias=False)
+        self.gate = nn.Parameter(torch.empty(experts, inner, width))
+        self.up = nn.Parameter(torch.empty(experts, inner, width))
+        self.down = nn.Parameter(torch.empty(experts, width, inner))
+        self.shared = shared
+
+    def packed(self) -> Packed:
+        def build(p: Packed) -> None:
+            dp, ip, n, w = up8(self.width), up8(self.inner), self.inner, self.width
+            dt, dev = self.gate.dtype, self.gate.device
+            p.w_router = pad2(self.router.weight, self.experts, dp).contiguous()
+            p.w_gu = torch.zeros(self.experts, 2 * ip, dp, dtype=dt, device=dev)      # rows interleaved: gate 0, up 0, gate 1, ...
+            p.w_down = torch.zeros(self.experts, dp, ip, dtype=dt, device=dev)
+            for param, place in ((self.gate, p.w_gu[:, 0:2 * n:2, :w]), (self.up, p.w_gu[:, 1:2 * n:2, :w]),
+                                 (self.down, p.w_down[:, :w, :n])):
+                place.copy_(param)
+                param.data = place
+            p.desc = VyMoe(self.experts, self.top, self.groups, self.keep, dp, ip, self.scale, self.limit, self.alpha,
+                           p.w_router.data_ptr(), p.w_gu.data_ptr(), p.w_down.data_ptr())
+        return Packed.of(self, [self.router.weight, self.gate, self.up, self.down], build)
+
+    @property
+    def dense(self) -> Optional[GatedFeedForward]:
+        return self.shared
+
+    def routed(self, h: torch.Tensor, L: int = 1, count: Optional[torch.Tensor] = None) -> "ops.Routed":
+        return ops.moe(h, self.packed().desc, L, count)

@@ -278,8 +278,9 @@ class SlotCache:
     """Whole-model memory of sequences of DIFFERENT lengths, for decoders that mix layer kinds.
 
     A sequence owns a slot while it lives (``allocate`` / ``free``); per layer a slot holds either cached rows
-    ("latent", width): a (slots, capacity, width) buffer, or a recurrent state ("state", shape): a (slots, *shape) fp32
-    buffer.  ``lengths`` (int32 on the device, one per slot) says how many tokens a slot holds: kernels place new rows
+    ("latent", width): a (slots, capacity, width) buffer, or a ring of the last tokens' keys and values ("window", (heads,
+    width, window)): a (slots, heads, rows, width) buffer of min(window, capacity) rows, position p in row p % rows, or a
+    recurrent state ("state", shape): a (slots, *shape) fp32 buffer.  ``lengths`` (int32 on the device, one per slot) says how many tokens a slot holds: kernels place new rows
     behind them, attend no further, and take the state of an empty slot as zero -- so nothing is cleared when a slot is
     handed on.  The host keeps a mirror (``length``).  Slots and capacity grow by doubling.
     """
@@ -299,6 +300,9 @@ class SlotCache:
         kind, shape = spec
         if kind == "latent":
             return torch.zeros(slots, capacity, shape, dtype=self.dtype, device=self.device)
+        if kind == "window":
+            heads, width, window = shape
+            return torch.zeros(slots, heads, min(window, capacity), width, dtype=self.dtype, device=self.device)
         if kind == "state":
             return torch.zeros(slots, *shape, dtype=torch.float32, device=self.device)
         raise ValueError(f"cache kind {kind!r}")
@@ -307,9 +311,13 @@ class SlotCache:
         for i, spec in enumerate(self.specs):
             if spec[0] == "state" and slots == self.slots:
                 continue
+            if spec[0] == "window" and slots == self.slots and self.buffers[i].shape[2] == spec[1][2]:
+                continue
             old, new = self.buffers[i], self._make(spec, slots, capacity)
             if spec[0] == "latent":
                 new[: old.shape[0], : old.shape[1]] = old
+            elif spec[0] == "window":   # (a ring that still grows has not wrapped: rows are positions)
+                new[: old.shape[0], :, : old.shape[2]] = old
             else:
                 new[: old.shape[0]] = old
             self.buffers[i] = new
@@ -378,10 +386,11 @@ class SlotBatch:
     def __init__(self, cache: SlotCache, slots, counts, max_keys: int) -> None:
         self.cache, self.max_keys = cache, max_keys
         self.slots, self.start = cache.table(slots), cache.lengths
-        self.fresh = all(cache.length[s] == 0 for s in slots)
+        self.past = max(cache.length[s] for s in slots)   # tokens before these, at most
+        self.fresh = self.past == 0
         self.count = None if len(set(counts)) == 1 else torch.tensor(counts, dtype=torch.int32, device=cache.device)
 
     def latents(self, layer: int) -> torch.Tensor:
         return self.cache.buffers[layer]
 
-    states = latents
+    states = ring = latents

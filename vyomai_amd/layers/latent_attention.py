@@ -52,12 +52,17 @@ class LatentAttention(nn.Module):
             p.w_o = head_cols(self.out.weight, H, dp)
         return Packed.of(self, list(self.parameters()), build)
 
-    def forward(self, h: torch.Tensor, B: int, L: int, batch, layer: int) -> torch.Tensor:
-        """h (B*L, padded width) of the new tokens -> mixer output (B*L, padded width).  The latents go to the cache."""
+    def matrices(self):
+        """Padded input (see packed) and output matrices."""
+        p = self.packed()
+        return p.w_in, p.w_o
+
+    def mix(self, rows: torch.Tensor, B: int, L: int, batch, layer: int, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+        """Packed projections (B*L, [q latent | kv latent | gate]) -> gated heads (B*L, heads * padded vdim).  The latents of
+        the new tokens go to the cache."""
         p = self.packed()
         H, dim, vdim = self.heads, up8(self.dim), up8(self.vdim)
         cache = batch.latents(layer)
-        rows = ops.linear(h, p.w_in)
         cq, c = ops.latent_norm(rows, p.q_norm, self.q_rank, p.c_norm, self.kv_rank, B, L, self.eps, cache=cache,
                                 slots=batch.slots, start=batch.start, count=batch.count, want_c=batch.fresh)
         q = ops.linear(cq, p.w_uq).view(B, L, H, dim).transpose(1, 2)
@@ -67,7 +72,13 @@ class LatentAttention(nn.Module):
         kv = ops.linear(c, p.w_ukv).view(B, S, -1)
         k = kv[..., : H * dim].unflatten(-1, (H, dim)).transpose(1, 2)
         v = kv[..., H * dim:].unflatten(-1, (H, vdim)).transpose(1, 2)
-        gate = rows[:, cq.shape[1] + p.c_norm.numel():].unflatten(0, (B, L))
+        g0 = cq.shape[1] + p.c_norm.numel()
+        gate = rows[:, g0: g0 + H * vdim].unflatten(0, (B, L))
         o = ops.attention_ex(q, k, v, self.scale, gate=gate, start=None if batch.fresh else batch.start,
-                             slots=None if batch.fresh else batch.slots)
-        return ops.linear(o.view(B * L, -1), p.w_o)
+                             slots=None if batch.fresh else batch.slots, out=None if out is None else out.unflatten(0, (B, L)))
+        return o.view(B * L, -1) if out is None else out
+
+    def forward(self, h: torch.Tensor, B: int, L: int, batch, layer: int) -> torch.Tensor:
+        """h (B*L, padded width) of the new tokens -> mixer output (B*L, padded width)."""
+        p = self.packed()
+        return ops.linear(self.mix(ops.linear(h, p.w_in), B, L, batch, layer), p.w_o)

@@ -6,7 +6,7 @@ the concatenated heads RMS-normed together, multiplied by a sigmoid gate and pro
 the fp32 state S (one dk x dv matrix per head and sequence)."""
 from __future__ import annotations
 
-from typing import Sequence
+from typing import Optional, Sequence
 
 import torch
 import torch.nn as nn
@@ -49,11 +49,20 @@ class LightningAttention(nn.Module):
             p.decay_pow = t.float().to(p.w_in.device)
         return Packed.of(self, list(self.parameters()), build)
 
-    def forward(self, h: torch.Tensor, B: int, L: int, batch, layer: int) -> torch.Tensor:
+    def matrices(self):
+        """Padded input (see packed) and output matrices."""
+        p = self.packed()
+        return p.w_in, p.w_o
+
+    def mix(self, rows: torch.Tensor, B: int, L: int, batch, layer: int, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+        """Packed projections (B*L, [q | k | v | gate]) -> gated heads (B*L, heads * padded vdim); the state advances."""
         p = self.packed()
         H, dim, vdim = self.heads, up8(self.dim), up8(self.vdim)
-        rows = ops.linear(h, p.w_in)
         o = ops.decay_attention(rows, H, dim, vdim, batch.states(layer), p.decay_pow, B, L, start=batch.start,
                                 slots=batch.slots, count=batch.count)
-        o = ops.rmsnorm_gate(o, p.norm, H * self.vdim, rows[:, H * (2 * dim + vdim):], self.eps)
-        return ops.linear(o, p.w_o)
+        g0 = H * (2 * dim + vdim)
+        return ops.rmsnorm_gate(o, p.norm, H * self.vdim, rows[:, g0: g0 + H * vdim], self.eps, out)
+
+    def forward(self, h: torch.Tensor, B: int, L: int, batch, layer: int) -> torch.Tensor:
+        p = self.packed()
+        return ops.linear(self.mix(ops.linear(h, p.w_in), B, L, batch, layer), p.w_o)

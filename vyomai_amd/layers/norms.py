@@ -7,11 +7,12 @@ import torch.nn as nn
 
 
 class WeightNorm(nn.Module):
-    """kind 'layer': (x - mean) / sqrt(var + eps) * w; kind 'rms': x / sqrt(mean(x^2) + eps) * w."""
+    """kind 'layer': (x - mean) / sqrt(var + eps) * w; kind 'rms': x / sqrt(mean(x^2) + eps) * w.  offset: the factor is
+    offset + w (1 for weights that are stored around zero)."""
 
-    def __init__(self, width: int, eps: float, kind: str = "layer") -> None:
+    def __init__(self, width: int, eps: float, kind: str = "layer", offset: float = 0.0) -> None:
         super().__init__()
         if kind not in ("layer", "rms"):
             raise ValueError(f"norm kind {kind!r}")
-        self.weight = nn.Parameter(torch.ones(width))
-        self.eps, self.kind = float(eps), kind
+        self.weight = nn.Parameter(torch.full((width,), 1.0 - offset))
+        self.eps, self.kind, self.offset = float(eps), kind, float(offset)

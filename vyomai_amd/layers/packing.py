@@ -26,6 +26,11 @@ def pad_vec(w: torch.Tensor, n: int) -> torch.Tensor:
     return out
 
 
+def norm_vec(norm, n: int) -> torch.Tensor:
+    """fp32 factors of a WeightNorm, zero-padded to n."""
+    return pad_vec(norm.weight.float() + norm.offset, n)
+
+
 def head_rows(w: torch.Tensor, heads: int, cols: int) -> torch.Tensor:
     """(heads * dim, k) -> (heads * up8(dim), cols): every head's rows padded by themselves."""
     dim = w.shape[0] // heads
@@ -51,16 +56,19 @@ def head_vec(w: torch.Tensor, heads: int) -> torch.Tensor:
 
 
 class Packed:
-    """Attribute bag of a module's kernel-side tensors, rebuilt when one of its parameters changed."""
+    """Attribute bag of a module's kernel-side tensors, rebuilt when one of its parameters changed.  (A build may turn a
+    parameter into a view of its packed copy: the parameters' state is noted after it.)"""
 
     @staticmethod
     def of(owner: nn.Module, params: Sequence[torch.Tensor], build: Callable[["Packed"], None]) -> "Packed":
-        key = tuple((p.data_ptr(), p._version, p.dtype) for p in params)
+        def state():
+            return tuple((p.data_ptr(), p._version, p.dtype) for p in params)
+        key = state()
         hit = owner.__dict__.get("_packed_cache")
         if hit is None or hit.key != key:
             hit = Packed()
-            hit.key = key
             with torch.no_grad():
                 build(hit)
+            hit.key = state()
             owner.__dict__["_packed_cache"] = hit
         return hit

@@ -100,6 +100,34 @@ def resolve_freqs(freqs, device):
     return a.cos().contiguous().to(device), a.sin().contiguous().to(device), 0
 
 
+class PairRotary:
+    """Rotary positions on neighbouring columns (2i, 2i + 1) of the first `dims` columns of a head, pair i turning by
+    position * base^(-2i / dims).  table(n): at least n positions of (cos, sin), fp32 (evaluated in double precision), shaped
+    (positions, dims / 2, 2); None without rotated columns.  Layers with equal constants share their tables."""
+
+    _tables: Dict[tuple, torch.Tensor] = {}
+
+    def __init__(self, base: float, dims: int) -> None:
+        if dims < 0 or dims % 2:
+            raise ValueError(f"{dims} rotated columns (an even number)")
+        self.base, self.dims = float(base), int(dims)
+
+    def table(self, positions: int, device) -> Optional[torch.Tensor]:
+        if self.dims == 0:
+            return None
+        key = self.base, self.dims, torch.device(device)
+        t = self._tables.get(key)
+        if t is None or t.shape[0] < positions:
+            n = 256
+            while n < positions:
+                n *= 2
+            f = torch.pow(torch.tensor(self.base, dtype=torch.float64, device=device),
+                          -torch.arange(0, self.dims, 2, dtype=torch.float64, device=device) / self.dims)
+            a = torch.arange(n, dtype=torch.float64, device=device)[:, None] * f[None, :]
+            t = self._tables[key] = torch.stack((a.cos(), a.sin()), -1).float().contiguous()
+        return t
+
+
 def apply_rotary_pos_emb(q, k, freqs, unsqueeze_dim=1) -> Tuple[torch.Tensor, torch.Tensor]:
     """q, k: (B, heads, L, dh); freqs: raw angles (1, L, dh/2).  Returns rotated copies
     (reference :155-182), computed by the vy_rope_fwd HIP kernel."""

@@ -1,13 +1,15 @@
-"""Decoder that mixes layer kinds over an fp32 residual stream: every layer is one mixer (latent attention, lightning
-attention, ...) and an optional gated MLP, each between a norm before and a norm after,
+"""Decoders that mix layer kinds over an fp32 residual stream: every layer is one mixer (latent attention, lightning attention,
+windowed attention, ...) and an optional feed-forward (gated, or a mixture of experts), in one of two forms:
 
-    x <- x + norm1b(mixer(norm1(x))) ;  x <- x + norm2b(mlp(norm2(x))) .
+    HybridLayer    x <- x + norm1b(mixer(norm1(x))) ;  x <- x + norm2b(ff(norm2(x)))
+    ParallelLayer  x <- x + (mixer(h) + ff(h)),  h = norm1(x)
 
-A design built from this file supplies its layers and its parameter names (models/gisitar.py); embedding, residual stream,
-slot cache, prefill, the native single-token step and generation are here.  Inference only.
+A design built from this file supplies its layers and its parameter names (models/gisitar.py, models/rivudra.py); embedding,
+residual stream, slot cache, prefill, the native single-token step and generation are here.  Inference only.
 """
 from __future__ import annotations
 
+import functools
 from typing import List, Optional, Sequence
 
 import torch
@@ -15,23 +17,23 @@ import torch.nn as nn
 
 from .. import ops
 from .._lib import VyomHipError
-from ..layers.ffn import GatedFeedForward
 from ..layers.kv_cache import SlotCache
 from ..layers.norms import WeightNorm
-from ..layers.packing import Packed, pad2, pad_vec
+from ..layers.packing import Packed, norm_vec, pad2
 from ..ops import up8
 from .decoder import CLMOutput
 
 
 class HybridLayer(nn.Module):
-    """One mixer and (mlp may be None) one gated MLP with their four norms."""
+    """One mixer and (mlp may be None) one feed-forward behind it, with their four norms."""
+    form = "sandwich"
 
-    def __init__(self, width: int, mixer: nn.Module, mlp: Optional[GatedFeedForward], eps: float, norm: str = "layer") -> None:
+    def __init__(self, width: int, mixer: nn.Module, mlp: Optional[nn.Module], eps: float, norm: str = "layer",
+                 offset: float = 0.0) -> None:
         super().__init__()
         self.mixer, self.mlp, self.width = mixer, mlp, width
-        self.norm1, self.norm1b = WeightNorm(width, eps, norm), WeightNorm(width, eps, norm)
-        if mlp is not None:
-            self.norm2, self.norm2b = WeightNorm(width, eps, norm), WeightNorm(width, eps, norm)
+        for n in self._norms():
+            setattr(self, n, WeightNorm(width, eps, norm, offset))
 
     def _norms(self) -> List[str]:
         return ["norm1", "norm1b"] + (["norm2", "norm2b"] if self.mlp is not None else [])
@@ -39,19 +41,71 @@ class HybridLayer(nn.Module):
     def packed(self) -> Packed:
         def build(p: Packed) -> None:
             for n in self._norms():
-                setattr(p, n, pad_vec(getattr(self, n).weight, up8(self.width)))
+                setattr(p, n, norm_vec(getattr(self, n), up8(self.width)))
         return Packed.of(self, [getattr(self, n).weight for n in self._norms()], build)
+
+    def run(self, norm, h: torch.Tensor, B: int, L: int, batch, layer: int, nxt: Optional[torch.Tensor]) -> Optional[torch.Tensor]:
+        """h = norm1(x) of the new tokens; norm(y=, post=, pre=, routed=) advances the residual stream x by a sublayer and
+        returns its next norm.  nxt: the norm of what follows this layer."""
+        p = self.packed()
+        y = self.mixer(h, B, L, batch, layer)
+        if self.mlp is None:
+            return norm(y=y, post=p.norm1b, pre=nxt)
+        h = norm(y=y, post=p.norm1b, pre=p.norm2)
+        routed = self.mlp.routed(h, L, batch.count)
+        return norm(y=self.mlp.dense(h) if self.mlp.dense is not None else None, routed=routed, post=p.norm2b, pre=nxt)
+
+
+class ParallelLayer(nn.Module):
+    """One norm whose output both the mixer and (mlp may be None) the feed-forward read.  The projections of the mixer and of
+    the feed-forward's dense part are ONE product of h, and their output products are one as well."""
+    form = "parallel"
+
+    def __init__(self, width: int, mixer: nn.Module, mlp: Optional[nn.Module], eps: float, norm: str = "rms",
+                 offset: float = 0.0) -> None:
+        super().__init__()
+        self.mixer, self.mlp, self.width = mixer, mlp, width
+        self.norm1 = WeightNorm(width, eps, norm, offset)
+
+    @property
+    def dense(self):
+        return self.mlp.dense if self.mlp is not None else None
+
+    def packed(self) -> Packed:
+        params = [self.norm1.weight, *self.mixer.parameters(), *(self.dense.parameters() if self.dense is not None else [])]
+
+        def build(p: Packed) -> None:
+            p.norm1 = norm_vec(self.norm1, up8(self.width))
+            p.w_in, p.w_o = self.mixer.matrices()
+            p.n_mix, p.n_heads = p.w_in.shape[0], p.w_o.shape[1]
+            if self.dense is not None:
+                gate_up, down = self.dense.matrices()
+                p.w_in, p.w_o = torch.cat([p.w_in, gate_up]), torch.cat([p.w_o, down], 1)
+            p.w_in, p.w_o = p.w_in.contiguous(), p.w_o.contiguous()
+        return Packed.of(self, params, build)
+
+    def run(self, norm, h: torch.Tensor, B: int, L: int, batch, layer: int, nxt: Optional[torch.Tensor]) -> Optional[torch.Tensor]:
+        p = self.packed()
+        rows = ops.linear(h, p.w_in)
+        both = torch.empty((B * L, p.w_o.shape[1]), dtype=h.dtype, device=h.device)
+        self.mixer.mix(rows[:, : p.n_mix], B, L, batch, layer, out=both[:, : p.n_heads])
+        if self.dense is not None:
+            self.dense.activation(rows[:, p.n_mix:], out=both[:, p.n_heads:])
+        routed = self.mlp.routed(h, L, batch.count) if self.mlp is not None else None
+        return norm(y=ops.linear(both, p.w_o), routed=routed, pre=nxt)
 
 
 class HybridDecoderModel(nn.Module):
-    """`layers` of HybridLayer between an embedding and a norm + vocabulary projection."""
+    """`layers` of HybridLayer / ParallelLayer between a (scaled) embedding and a norm + vocabulary projection."""
 
-    def __init__(self, config, width: int, vocab: int, layers: Sequence[HybridLayer], eps: float, norm: str = "layer") -> None:
+    def __init__(self, config, width: int, vocab: int, layers: Sequence[nn.Module], eps: float, norm: str = "layer",
+                 offset: float = 0.0, embed_scale: float = 1.0) -> None:
         super().__init__()
         self.config, self.width, self.vocab, self.eps, self.rms = config, width, vocab, float(eps), norm == "rms"
+        self.embed_scale = float(embed_scale)
         self.word_embeddings = nn.Embedding(vocab, width)
         self.layers = nn.ModuleList(layers)
-        self.final_norm = WeightNorm(width, eps, norm)
+        self.final_norm = WeightNorm(width, eps, norm, offset)
         self.head = nn.Linear(width, vocab, bias=False)
         self._own_cache: Optional[SlotCache] = None
         self.requires_grad_(False)
@@ -70,7 +124,7 @@ class HybridDecoderModel(nn.Module):
             dp = up8(self.width)
             p.embed = pad2(self.word_embeddings.weight, self.vocab, dp).contiguous()
             p.head = pad2(self.head.weight, self.vocab, dp).contiguous()
-            p.final_norm = pad_vec(self.final_norm.weight, dp)
+            p.final_norm = norm_vec(self.final_norm, dp)
         return Packed.of(self, [self.word_embeddings.weight, self.head.weight, self.final_norm.weight], build)
 
     # ---- cache ------------------------------------------------------------------------------
@@ -92,17 +146,11 @@ class HybridDecoderModel(nn.Module):
         dp = up8(self.width)
         x = torch.empty((B * L, dp), dtype=torch.float32, device=tokens.device)
         norms = [l.packed() for l in self.layers]
-        h = ops.residual_norm(x, self.width, table=p.embed, ids=tokens.reshape(-1).contiguous(), pre=norms[0].norm1,
-                              eps=self.eps, rms=self.rms)
+        norm = functools.partial(ops.residual_norm, x, self.width, eps=self.eps, rms=self.rms)
+        h = norm(table=p.embed, ids=tokens.reshape(-1).contiguous(), table_scale=self.embed_scale, pre=norms[0].norm1)
         for i, layer in enumerate(self.layers):
-            y = layer.mixer(h, B, L, batch, i)
             # (the last layer's stream is normed row by row in logits(): only the rows asked for)
-            nxt = norms[i + 1].norm1 if i + 1 < len(self.layers) else None
-            if layer.mlp is not None:
-                h = ops.residual_norm(x, self.width, y=y, post=norms[i].norm1b, pre=norms[i].norm2, eps=self.eps, rms=self.rms)
-                h = ops.residual_norm(x, self.width, y=layer.mlp(h), post=norms[i].norm2b, pre=nxt, eps=self.eps, rms=self.rms)
-            else:
-                h = ops.residual_norm(x, self.width, y=y, post=norms[i].norm1b, pre=nxt, eps=self.eps, rms=self.rms)
+            h = layer.run(norm, h, B, L, batch, i, norms[i + 1].norm1 if i + 1 < len(self.layers) else None)
             if layers_out is not None:
                 layers_out.append(x.view(B, L, dp)[..., : self.width].clone())
         cache.advance(list(slots), list(counts))

@@ -1,7 +1,7 @@
 """Model registry and checkpoint loading: a folder with config.json (its "architecture" chooses the class) and *.safetensors.
 
 A registered class has ``config_class`` (with ``from_dict``), takes the config, and may map its parameter names to the
-checkpoint's with ``checkpoint_name``.
+checkpoint's with ``checkpoint_name``: a name, or a list of names whose tensors are stacked (a mixture's experts).
 """
 from __future__ import annotations
 
@@ -29,7 +29,7 @@ def register_model(name: str) -> Callable[[type], type]:
 
 
 def model_class(architecture: str) -> type:
-    from . import gisitar  # noqa: F401  (registers itself)
+    from . import gisitar, rivudra  # noqa: F401  (they register themselves)
     if architecture not in MODELS:
         raise ValueError(f"architecture {architecture!r} is not registered (known: {sorted(MODELS)})")
     return MODELS[architecture]
@@ -68,15 +68,25 @@ def load_checkpoint(model: nn.Module, tensors: Dict[str, torch.Tensor], dtype: t
     rename = getattr(model, "checkpoint_name", lambda n: n)
     left = set(tensors)
     for name, p in list(model.named_parameters()):
-        key = rename(name)
-        if key not in tensors:
-            raise KeyError(f"the checkpoint lacks {key!r}")
-        t = tensors[key]
-        if tuple(t.shape) != tuple(p.shape):
-            raise ValueError(f"{key}: shape {tuple(t.shape)} in the checkpoint, {tuple(p.shape)} in the model")
-        left.discard(key)
+        keys = rename(name)
+        stacked = isinstance(keys, list)
+        parts = []
+        for key in keys if stacked else [keys]:
+            if key not in tensors:
+                raise KeyError(f"the checkpoint lacks {key!r}")
+            t, want = tensors[key], tuple(p.shape[1:] if stacked else p.shape)
+            if tuple(t.shape) != want:
+                raise ValueError(f"{key}: shape {tuple(t.shape)} in the checkpoint, {want} in the model")
+            left.discard(key)
+            parts.append(t)
+        if stacked:
+            full = torch.empty(p.shape, dtype=dtype, device=device)
+            for i, t in enumerate(parts):
+                full[i].copy_(t)
+        else:
+            full = parts[0].to(device=device, dtype=dtype)
         owner, _, leaf = name.rpartition(".")
-        setattr(model.get_submodule(owner), leaf, nn.Parameter(t.to(device=device, dtype=dtype), requires_grad=p.requires_grad))
+        setattr(model.get_submodule(owner), leaf, nn.Parameter(full, requires_grad=p.requires_grad))
     if left:
         raise KeyError(f"the model has no place for {sorted(left)[:4]}{' ...' if len(left) > 4 else ''}")
 

@@ -6,8 +6,9 @@ is no CPU or eager fallback.
 """
 from __future__ import annotations
 
+import ctypes as C
 import math
-from typing import Optional, Tuple
+from typing import NamedTuple, Optional, Tuple
 
 import torch
 
@@ -620,16 +621,34 @@ def rmsnorm(x: Tensor, w: Tensor, eps: float, w_offset: float = 1.0) -> Tensor:
     return y.view(x.shape)
 
 
-def gated_act(gate_up: Tensor, act: int) -> Tensor:
+def gated_act(gate_up: Tensor, act: int, out: Optional[Tensor] = None) -> Tensor:
     """act(gate_up[..., :I]) * gate_up[..., I:]  (vy_gated_act_fwd)."""
     _need_gpu(gate_up)
     g2 = _rows(gate_up)
     M, two_i = g2.shape
     I = two_i // 2
+    if out is not None:
+        assert out.shape == (M, I) and out.stride(1) == 1 and out.dtype == gate_up.dtype
+        call("vy_gated_act_fwd", g2.data_ptr(), g2.stride(0), out.data_ptr(), out.stride(0), M, I, act,
+             dtype_code(gate_up.dtype), _stream())
+        return out
     out = torch.empty((M, I), dtype=gate_up.dtype, device=gate_up.device)
     call("vy_gated_act_fwd", g2.data_ptr(), g2.stride(0), out.data_ptr(), out.stride(0), M, I, act,
          dtype_code(gate_up.dtype), _stream())
     return out.view(*gate_up.shape[:-1], I)
+
+
+def clamped_act(gate_up: Tensor, limit: float, alpha: float, out: Optional[Tensor] = None) -> Tensor:
+    """g * sigmoid(alpha g) * (u + 1) with g = min(gate, limit), u = clamp(up, -limit, limit)  (vy_clamped_act_fwd)."""
+    _need_gpu(gate_up, out)
+    g2 = _rows(gate_up)
+    M, two_i = g2.shape
+    if out is None:
+        out = torch.empty((M, two_i // 2), dtype=gate_up.dtype, device=gate_up.device)
+    assert out.shape == (M, two_i // 2) and out.stride(1) == 1 and out.dtype == gate_up.dtype
+    call("vy_clamped_act_fwd", g2.data_ptr(), g2.stride(0), out.data_ptr(), out.stride(0), M, two_i // 2, float(limit),
+         float(alpha), dtype_code(gate_up.dtype), _stream())
+    return out
 
 
 # ------------------------------------------------------------------------------------------
@@ -645,15 +664,17 @@ def up8(n: int) -> int:
 def residual_norm(x: Tensor, width: int, *, y: Optional[Tensor] = None, post: Optional[Tensor] = None,
                   pre: Optional[Tensor] = None, eps: float = 1e-5, rms: bool = False, table: Optional[Tensor] = None,
                   ids: Optional[Tensor] = None, dtype: Optional[torch.dtype] = None,
-                  err_flag: Optional[Tensor] = None) -> Optional[Tensor]:
-    """x (M, padded width) fp32, in place: x += norm(y) * post (post None: x += y), or x = table[ids]; returns
-    norm(x) * pre in `dtype` (None without pre).  (vy_residual_norm)"""
+                  err_flag: Optional[Tensor] = None, table_scale: float = 1.0,
+                  routed: Optional["Routed"] = None) -> Optional[Tensor]:
+    """x (M, padded width) fp32, in place: x += norm(y) * post (post None: x += y), or x = table_scale * table[ids]; routed:
+    y also gets the weighted rows of every token's experts (y None: they are all of it); returns norm(x) * pre in `dtype`
+    (None without pre).  (vy_residual_norm_routed)"""
     _need_gpu(x, y, post, pre, table, ids)
     assert x.dtype == torch.float32 and x.dim() == 2 and x.stride(1) == 1
     for w in (post, pre):
         assert w is None or (w.dtype == torch.float32 and w.numel() == x.shape[1] and w.is_contiguous())
     M, NP = x.shape
-    src = y if y is not None else table
+    src = y if y is not None else routed.rows if routed is not None else table
     dt = dtype or src.dtype
     assert src is None or (src.dtype == dt and src.shape[-1] == NP and src.stride(-1) == 1)
     if y is not None:
@@ -662,9 +683,15 @@ def residual_norm(x: Tensor, width: int, *, y: Optional[Tensor] = None, post: Op
     if ids is not None:
         assert ids.dtype == torch.long and ids.is_contiguous() and ids.numel() == M and table is not None
     h = torch.empty((M, NP), dtype=dt, device=x.device) if pre is not None else None
-    call("vy_residual_norm", x.data_ptr(), x.stride(0), _ptr(y), y.stride(0) if y is not None else 0, _ptr(table),
+    extra = None
+    if routed is not None:
+        r, top = routed.rows, routed.weight.shape[1]
+        assert ids is None and r.dtype == dt and r.shape[1] == NP and r.stride(1) == 1 and routed.weight.shape == (M, top)
+        assert routed.weight.dtype == torch.float32 and routed.pos.dtype == torch.int32 and routed.pos.shape == (M, top)
+        extra = _lib.VyRoutedRows(r.data_ptr(), r.stride(0), routed.pos.data_ptr(), routed.weight.data_ptr(), top)
+    call("vy_residual_norm_routed", x.data_ptr(), x.stride(0), _ptr(y), y.stride(0) if y is not None else 0, _ptr(table),
          table.stride(0) if table is not None else 0, _ptr(ids), table.shape[0] if table is not None else 0, _ptr(err_flag),
-         _ptr(post), float(eps), _ptr(pre), float(eps), _ptr(h), NP, M, int(width), NP, int(rms), dtype_code(dt), _stream())
+         float(table_scale), C.byref(extra) if extra is not None else None, _ptr(post), float(eps), _ptr(pre), float(eps), _ptr(h), NP, M, int(width), NP, int(rms), dtype_code(dt), _stream())
     return h
 
 
@@ -695,33 +722,131 @@ def latent_norm(p: Tensor, w_q: Tensor, n_q: int, w_c: Tensor, n_c: int, B: int,
     return q, c
 
 
-def rmsnorm_gate(x: Tensor, w: Tensor, width: int, gate: Tensor, eps: float) -> Tensor:
+def rmsnorm_gate(x: Tensor, w: Tensor, width: int, gate: Tensor, eps: float, out: Optional[Tensor] = None) -> Tensor:
     """RMSNorm(x) * w * sigmoid(gate) over `width` of the padded columns.  (vy_rmsnorm_gate)"""
     _need_gpu(x, w, gate)
     M, NP = x.shape
     assert gate.shape == x.shape and x.stride(1) == 1 and gate.stride(1) == 1 and w.numel() == NP and w.dtype == torch.float32
-    y = torch.empty((M, NP), dtype=x.dtype, device=x.device)
-    call("vy_rmsnorm_gate", x.data_ptr(), x.stride(0), w.data_ptr(), gate.data_ptr(), gate.stride(0), y.data_ptr(), NP, M,
+    y = torch.empty((M, NP), dtype=x.dtype, device=x.device) if out is None else out
+    assert y.shape == x.shape and y.stride(1) == 1 and y.dtype == x.dtype
+    call("vy_rmsnorm_gate", x.data_ptr(), x.stride(0), w.data_ptr(), gate.data_ptr(), gate.stride(0), y.data_ptr(), y.stride(0), M,
          int(width), NP, float(eps), dtype_code(x.dtype), _stream())
     return y
 
 
 def attention_ex(q: Tensor, k: Tensor, v: Tensor, scale: float, *, gate: Optional[Tensor] = None,
-                 start: Optional[Tensor] = None, slots: Optional[Tensor] = None) -> Tensor:
+                 start: Optional[Tensor] = None, slots: Optional[Tensor] = None, window: int = 0, sink: bool = False,
+                 rotary: Optional[Tensor] = None, start_cap: Optional[int] = None, out: Optional[Tensor] = None) -> Tensor:
     """Causal attention with a value width of its own: q (B,h,L,dh), k (B,hk,S,dh), v (B,hk,S,dv) -> (B, L, h*dv); `start`
-    (int32, per slot) keys precede the queries; gate (B, L, h*dv): out *= sigmoid(gate).  (vy_attn_fwd_ex)"""
+    (int32, per slot) keys precede the queries; gate (B, L, h*dv): out *= sigmoid(gate).  window: only the last `window` keys up
+    to a query's own are seen (0: all); sink: one more exp(0) in the denominators; rotary (positions, pairs, 2): the queries are
+    rotated by position start + i; start_cap: at most so many keys precede the queries.  (vy_attn_fwd_ex)"""
     _need_gpu(q, k, v, gate, start, slots)
     B, h, L, dh = q.shape
     hk, S, dv = k.shape[1], k.shape[2], v.shape[3]
     _slot_args(slots, start, None, B)
     assert q.stride(3) == 1 and k.stride(3) == 1 and v.stride(3) == 1 and k.shape[3] == dh and v.shape[:3] == k.shape[:3]
-    out = torch.empty((B, L, h * dv), dtype=q.dtype, device=q.device)
+    if out is None:
+        out = torch.empty((B, L, h * dv), dtype=q.dtype, device=q.device)
+    assert out.shape == (B, L, h * dv) and out.stride(2) == 1 and out.dtype == q.dtype
     assert gate is None or (gate.shape == out.shape and gate.stride(2) == 1)
+    win = None
+    if window or sink or rotary is not None or start_cap is not None:
+        _need_gpu(rotary)
+        win = _lib.VyAttnWindow(int(window), int(sink), 0, 2 ** 31 - 1 if start_cap is None else int(start_cap),
+                                *_rotary_args(rotary))
     call("vy_attn_fwd_ex", q.data_ptr(), q.stride(0), q.stride(1), q.stride(2), k.data_ptr(), k.stride(0), k.stride(1),
          k.stride(2), v.data_ptr(), v.stride(0), v.stride(1), v.stride(2), out.data_ptr(), out.stride(0), out.stride(1),
          _ptr(gate), gate.stride(0) if gate is not None else 0, gate.stride(1) if gate is not None else 0, _ptr(start),
-         _ptr(slots), B, h, hk, L, S, dh, dv, float(scale), dtype_code(q.dtype), _stream())
+         _ptr(slots), B, h, hk, L, S, dh, dv, float(scale), C.byref(win) if win is not None else None, dtype_code(q.dtype),
+         _stream())
     return out
+
+
+def _rotary_args(rotary: Optional[Tensor]):
+    """(pointer, rotated columns, positions) of a (positions, pairs, 2) fp32 table of cosines and sines."""
+    if rotary is None:
+        return None, 0, 0
+    assert rotary.dtype == torch.float32 and rotary.dim() == 3 and rotary.shape[2] == 2 and rotary.is_contiguous()
+    return rotary.data_ptr(), 2 * rotary.shape[1], rotary.shape[0]
+
+
+def _ring_args(ring: Optional[Tensor], hk: int, dim: int, vdim: int):
+    """(pointer, slot stride, head stride, rows) of a (slots, hk, rows, dim + vdim) ring."""
+    if ring is None:
+        return None, 0, 0, 0
+    assert ring.dim() == 4 and ring.shape[1] == hk and ring.shape[3] == dim + vdim and ring.is_contiguous()
+    return ring.data_ptr(), ring.stride(0), ring.stride(1), ring.shape[2]
+
+
+def window_rows(p: Tensor, B: int, L: int, hk: int, dim: int, vdim: int, ok: int, ov: int, *, rotary: Optional[Tensor] = None,
+                ring: Optional[Tensor] = None, slots: Optional[Tensor] = None, start: Optional[Tensor] = None,
+                count: Optional[Tensor] = None) -> None:
+    """Packed rows p (B*L, .) with keys at column ok and values at ov: rotary given: the keys are rotated in place; ring given:
+    the last rows of every sequence go to it.  (vy_window_rows)"""
+    _need_gpu(p, rotary, ring, slots, start, count)
+    _slot_args(slots, start, count, B)
+    assert p.shape[0] == B * L and p.stride(1) == 1 and (ring is None or ring.dtype == p.dtype)
+    call("vy_window_rows", p.data_ptr(), p.stride(0), ok, ov, *_ring_args(ring, hk, dim, vdim), *_rotary_args(rotary),
+         int(rotary is not None), int(ring is not None), _ptr(slots), _ptr(start), _ptr(count), B, L, hk, dim, vdim,
+         dtype_code(p.dtype), _stream())
+
+
+def window_context(p: Tensor, B: int, L: int, hk: int, dim: int, vdim: int, ok: int, ov: int, ring: Tensor, past: int,
+                   start: Tensor, slots: Optional[Tensor] = None) -> Tensor:
+    """(B, hk, past + L, dim + vdim): the last min(start, past) rows of every ring in order, then the new ones.
+    (vy_window_context)"""
+    _need_gpu(p, ring, slots, start)
+    _slot_args(slots, start, None, B)
+    assert p.shape[0] == B * L and p.stride(1) == 1 and ring.dtype == p.dtype
+    ctx = torch.empty((B, hk, past + L, dim + vdim), dtype=p.dtype, device=p.device)
+    call("vy_window_context", p.data_ptr(), p.stride(0), ok, ov, *_ring_args(ring, hk, dim, vdim), ctx.data_ptr(), past + L, past,
+         _ptr(slots), start.data_ptr(), B, L, hk, dim, vdim, dtype_code(p.dtype), _stream())
+    return ctx
+
+
+def window_decode(p: Tensor, h: int, hk: int, dim: int, vdim: int, ring: Tensor, scale: float, start: Tensor, max_keys: int, *,
+                  rotary: Optional[Tensor] = None, sink: bool = False, gate: bool = False,
+                  slots: Optional[Tensor] = None) -> Tensor:
+    """One token per sequence, packed rows p (B, [q | k | v | gate]): its key and value go to the ring, its queries attend
+    over it -> (B, h*vdim).  (vy_window_decode)"""
+    _need_gpu(p, ring, slots, start, rotary)
+    B = p.shape[0]
+    _slot_args(slots, start, None, B)
+    assert p.stride(1) == 1 and ring.dtype == p.dtype
+    nk, gk, gv = h * dim, hk * dim, hk * vdim
+    assert p.shape[1] >= nk + gk + gv + (h * vdim if gate else 0)
+    out = torch.empty((B, h * vdim), dtype=p.dtype, device=p.device)
+    nws = _lib.load().vy_window_decode_ws_bytes(B, h, hk, vdim, ring.shape[2])
+    ws = torch.empty(max(nws, 1), dtype=torch.uint8, device=p.device)
+    call("vy_window_decode", p.data_ptr(), p.stride(0), 0, nk, nk + gk, nk + gk + gv if gate else -1,
+         *_ring_args(ring, hk, dim, vdim), *_rotary_args(rotary), _ptr(slots), start.data_ptr(), int(max_keys), out.data_ptr(),
+         out.stride(0), B, h, hk, dim, vdim, float(scale), int(sink), ws.data_ptr(), nws, dtype_code(p.dtype), _stream())
+    return out
+
+
+class Routed(NamedTuple):
+    """Outputs of the experts of M tokens, not yet added up: sum_k weight[m, k] * rows[pos[m, k]] (pos < 0: nothing)."""
+    rows: Tensor
+    pos: Tensor
+    weight: Tensor
+    ids: Tensor
+
+
+def moe(h: Tensor, desc: "_lib.VyMoe", L: int = 1, count: Optional[Tensor] = None) -> Routed:
+    """Router and experts of `desc` on rows h (M, padded width); tokens l >= count[b] of a sequence are padding.
+    (vy_moe_fwd)"""
+    _need_gpu(h, count)
+    M, top = h.shape[0], desc.top
+    assert h.stride(1) == 1 and h.shape[1] == desc.width and (count is None or count.dtype == torch.int32)
+    rows = torch.empty((M * top, desc.width), dtype=h.dtype, device=h.device)
+    pos, ids = (torch.empty((M, top), dtype=torch.int32, device=h.device) for _ in range(2))
+    weight = torch.empty((M, top), dtype=torch.float32, device=h.device)
+    nws = _lib.load().vy_moe_ws_bytes(C.byref(desc), M, dtype_code(h.dtype))
+    ws = torch.empty(nws, dtype=torch.uint8, device=h.device)
+    call("vy_moe_fwd", C.byref(desc), h.data_ptr(), h.stride(0), M, _ptr(count), L, rows.data_ptr(), rows.stride(0),
+         ids.data_ptr(), pos.data_ptr(), weight.data_ptr(), ws.data_ptr(), nws, dtype_code(h.dtype), _stream())
+    return Routed(rows, pos, weight, ids)
 
 
 def latent_decode(q: Tensor, wukt: Tensor, wuv: Tensor, cache: Tensor, start: Tensor, max_keys: int, scale: float, *,
