@@ -30,13 +30,13 @@ def rotate(x: Tensor, base: float, dims: int, first: int = 0) -> Tensor:
     """Rotary positions on (T, dim) rows of one head at positions first, first + 1, ...: neighbours (2i, 2i + 1) among the
     first `dims` columns turn by position * base^(-2i / dims)."""
     y = x.clone()
-    for t in range(x.shape[0]):
-        for i in range(dims // 2):
-            angle = torch.tensor((first + t) * float(base) ** (-2.0 * i / dims), dtype=torch.float64)
-            c, s = torch.cos(angle).to(x.dtype), torch.sin(angle).to(x.dtype)
-            u, v = x[t, 2 * i], x[t, 2 * i + 1]
-            y[t, 2 * i] = u * c - v * s
-            y[t, 2 * i + 1] = v * c + u * s
+    position = torch.arange(first, first + x.shape[0], dtype=torch.float64)
+    for i in range(dims // 2):
+        angle = position * float(base) ** (-2.0 * i / dims)
+        c, s = torch.cos(angle).to(x.dtype), torch.sin(angle).to(x.dtype)
+        u, v = x[:, 2 * i], x[:, 2 * i + 1]
+        y[:, 2 * i] = u * c - v * s
+        y[:, 2 * i + 1] = v * c + u * s
     return y
 
 
