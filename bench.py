@@ -51,8 +51,8 @@ def parse():
     ap.add_argument("--no-cpu-baseline", action="store_true")
     ap.add_argument("--no-decode", action="store_true")
     ap.add_argument("--no-other-configs", action="store_true", help="skip the configs[3] / configs[4] side measurements")
-    ap.add_argument("--model", default="decoder", choices=["decoder", "gisitar"],
-                    help="gisitar: prefill / decode throughput of that design beside the Gemma-style stack at equal size (one "
+    ap.add_argument("--model", default="decoder", choices=["decoder", "gisitar", "rivudra"],
+                    help="gisitar / rivudra: prefill / decode throughput of that design beside the Gemma-style stack at equal size (one "
                          "GPU, serving only) instead of the headline workload")
     ap.add_argument("--backend", default="nccl", help="torch.distributed backend (nccl = RCCL; gloo for rehearsals)")
     ap.add_argument("--rehearse-launch", action="store_true",
@@ -394,20 +394,21 @@ def rehearse_launch(a) -> None:
         dist.destroy_process_group()
 
 
-def bench_gisitar(a) -> None:
-    """--model gisitar: one JSON line with the throughputs of tools/bench_gisitar.py."""
+def bench_serving(a) -> None:
+    """--model gisitar / rivudra: one JSON line with the throughputs of tools/bench_gisitar.py / bench_rivudra.py."""
     if a.gpus != 1:
-        raise SystemExit("bench.py --model gisitar measures one GPU")
+        raise SystemExit(f"bench.py --model {a.model} measures one GPU")
     json_fd = os.dup(1)
     os.dup2(2, 1)
-    from tools import bench_gisitar as G
+    import importlib
+    G = importlib.import_module(f"tools.bench_{a.model}")
     r = G.run()
     big = max(G.SIZES)
-    d = r[f"width {big}"]["gisitar"]["decode32"]
-    line = {"metric": f"decode tokens/sec (Gisitar, {G.LAYERS} layers, width {big}, batch {d['batch']}, context {d['context']})",
+    d = r[f"width {big}"][a.model]["decode32"]
+    line = {"metric": f"decode tokens/sec ({a.model.capitalize()}, {G.LAYERS} layers, width {big}, batch {d['batch']}, context {d['context']})",
             "value": d["tokens_per_sec"], "unit": "tokens/s", "n_gpus": 1, "ms_per_step": d["ms_per_step"],
             "higher_is_better": True, "vs_baseline": None, "dtype": "bf16", "data": "synthetic",
-            "config": {"model": "gisitar", "layers": G.LAYERS, "vocab": G.VOCAB, "sizes": {str(w): s for w, s in G.SIZES.items()}},
+            "config": {"model": a.model, "layers": G.LAYERS, "vocab": G.VOCAB, "sizes": {str(w): s for w, s in G.SIZES.items()}},
             "results": r}
     os.write(json_fd, (json.dumps(line) + "\n").encode())
     os.close(json_fd)
@@ -415,8 +416,8 @@ def bench_gisitar(a) -> None:
 
 def main():
     a = parse()
-    if a.model == "gisitar":
-        return bench_gisitar(a)
+    if a.model != "decoder":
+        return bench_serving(a)
     env_world = os.environ.get("WORLD_SIZE")
     if env_world is None and a.gpus > 1:
         raise SystemExit(spawn_ranks(a))

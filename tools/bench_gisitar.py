@@ -43,13 +43,12 @@ class GemmaStack(nn.Module):
     """The language model of models/paligemma.py without its vision tower."""
     ROPE_OFFSET = 0
 
-    def __init__(self, width, max_pos):
+    def __init__(self, width, max_pos, heads, kv_heads, ff):
         super().__init__()
         from vyomai_amd.layers.positional_embeddings import RopeTable
         from vyomai_amd.models import paligemma as P
-        H, _, _, ff = SIZES[width]
-        t = types.SimpleNamespace(hidden_size=width, intermediate_size=ff, num_hidden_layers=LAYERS, num_attention_heads=H,
-                                  num_key_value_heads=H, head_dim=DIM, vocab_size=VOCAB, rms_norm_eps=1e-6,
+        t = types.SimpleNamespace(hidden_size=width, intermediate_size=ff, num_hidden_layers=LAYERS, num_attention_heads=heads,
+                                  num_key_value_heads=kv_heads, head_dim=DIM, vocab_size=VOCAB, rms_norm_eps=1e-6,
                                   attention_bias=False, max_position_embeddings=max_pos, rope_theta=10000.0)
         self.shape = types.SimpleNamespace(text=t)
         self.embed_tokens = nn.Embedding(VOCAB, width)
@@ -118,11 +117,14 @@ def measure_gisitar(width, cases):
 
 
 @torch.no_grad()
-def measure_gemma(width, cases):
+def measure_gemma(width, cases, heads=None, kv_heads=None, ff=None):
     from vyomai_amd.decode_plan import GemmaDecodePlan
+    if heads is None:
+        heads, _, _, ff = SIZES[width]
+        kv_heads = heads
     torch.manual_seed(0)
     with torch.device("cuda"):
-        m = GemmaStack(width, 8192 + 64)
+        m = GemmaStack(width, 8192 + 64, heads, kv_heads, ff)
     m = m.to(torch.bfloat16).eval()
     out = {"parameters": sum(p.numel() for p in m.parameters())}
     for c in cases:
@@ -137,7 +139,7 @@ def measure_gemma(width, cases):
             plan = GemmaDecodePlan(m, m.caches(B, ctx + 8), B)
             x = torch.randn(B, width, device="cuda", dtype=torch.bfloat16)
             ms = timed(lambda: plan.step(x, ctx - 1), 35)
-            nbytes = sum(p.numel() for p in m.parameters()) * 2 + B * LAYERS * ctx * 2 * SIZES[width][0] * DIM * 2
+            nbytes = sum(p.numel() for p in m.parameters()) * 2 + B * LAYERS * ctx * 2 * kv_heads * DIM * 2
             out[c] = {"batch": B, "context": ctx, "ms_per_step": round(ms, 4), "tokens_per_sec": round(B / ms * 1e3, 1),
                       "bytes_per_step": int(nbytes), "achieved_GBps": round(nbytes / ms * 1e-6, 1)}
             del plan
