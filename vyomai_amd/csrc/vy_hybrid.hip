@@ -8,6 +8,9 @@ int vy_residual_norm_ex(float* x, int64_t ldx, const void* y, int64_t ldy, const
                         int64_t V, int32_t* err, float table_scale, const vy_routed_rows* routed, const float* w_post,
                         float eps_post, const float* w_pre, float eps_pre, void* h, int64_t ldh, int64_t M, int64_t N, int64_t NP,
                         int rms, int* advance, const int* slots, int n_adv, int dtype, void* stream);
+int vy_parallel_decode(const vy_hybrid_plan* p, const vy_hybrid_layer* L, const void* h, void* in, void* ao, void* y, void* erows,
+                       int32_t* eids, float* ew, void* moe_ws, int64_t moe_ws_bytes, const int32_t* slots, const int32_t* lengths,
+                       int64_t max_keys, void* mix_ws, int64_t mix_ws_bytes, void* stream);
 int vy_dec_gemv1(const void* x, const void* w, const void* bias, const void* residual, void* y, int N, int K, int prescaled,
                  float eps, hipStream_t st);
 int vy_dec_gemv1_gated(const void* x, const void* wgu, void* y, int I, int K, int act, int prescaled, float eps, hipStream_t st);
@@ -125,6 +128,15 @@ extern "C" int vy_hybrid_decoder_step(const vy_hybrid_plan* p, const int64_t* id
     const bool last = l + 1 == p->num_layers, parallel = L.form == VY_FORM_PARALLEL;
     const float* next = last ? p->final_norm : p->layers[l + 1].norm1;
     const int64_t nv = (int64_t)L.heads * L.vdim, nk = (int64_t)L.heads * L.dim, na = nv + (parallel ? L.ff : 0);
+    if (parallel) {   // windowed attention beside clamped feed-forwards: the pieces of the layer share launches
+      rc = vy_parallel_decode(p, &L, h, in, ao, y, erows, eids, ew, ews, s.moe_ws, slots, lengths, max_keys, mws, s.mix_ws, stream);
+      if (rc == VY_OK) {
+        const vy_routed_rows rows{erows, dp, nullptr, ew, L.moe ? L.moe->top : 0};
+        if ((rc = norm(y, L.moe ? &rows : nullptr, L.norm1b, next, last))) return rc;
+        continue;
+      }
+      if (rc != VY_ERR_UNSUPPORTED) return rc;
+    }
     if ((rc = product(p, h, L.w_in, in, L.n_in, L.n_in, dp, stream))) return rc;
     if (L.mixer == VY_MIX_LATENT) {
       if (max_keys > L.cap) VY_FAIL(VY_ERR_ARG, "%s: %ld keys exceed the cache capacity %d", who, (long)max_keys, L.cap);

@@ -8,17 +8,16 @@
 // with their rows interleaved (row 2j: gate j, row 2j + 1: up j): in the accumulators' layout (a lane owns 4 consecutive
 // output columns of one token) both halves of a pair sit in one lane and the activation is the product's epilogue.
 //
-// Few tokens (decode): expert_rows_kernel streams the weights of the experts in use straight into MFMA operands, one
+// Few tokens (decode): expert_rows_kernel streams the weights of the experts in use straight into MFMA operands (vy_rows.h), one
 // workgroup per 16 or 32 weight rows of an expert; which experts and tokens, every workgroup reads from the choice itself.
 // Many tokens (prefill): tokens are sorted by expert (ranks from the choice kernel, offsets in the scatter kernel) and
 // grouped_gemm_kernel runs 128 x 128 tiles over the experts' row ranges, gathering its rows of h on the way into LDS.
 // fp32 takes the same way with a plain tile kernel.  A row's result does not depend on its place or on other rows.
-#include "vy_common.h"
-#include <float.h>
+#include "vy_moe.h"
 
 namespace {
 
-constexpr int MAX_E = 1024, MAX_ENTRIES = 1024;
+using namespace vy_moe_dev;
 
 // ---- router -----------------------------------------------------------------------------------
 // logits[m][e] = sum_k h[m][k] w[e][k], fp32 accumulation and result.  One workgroup: 16 ET experts x 16 MT tokens; the four
@@ -42,7 +41,7 @@ __global__ __launch_bounds__(256) void router_logits_kernel(const bf16* __restri
 #pragma unroll
     for (int j = 0; j < MT; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
   const bf16x8 zero8 = {(bf16)0.f, (bf16)0.f, (bf16)0.f, (bf16)0.f, (bf16)0.f, (bf16)0.f, (bf16)0.f, (bf16)0.f};
-#pragma unroll 4
+#pragma unroll 8
   for (int k = 32 * wave; k < K; k += 128) {
     const bool in = k + 8 * kq < K;
     bf16x8 a[ET], b[MT];
@@ -98,102 +97,11 @@ __global__ __launch_bounds__(256) void router_logits_f32_kernel(const float* __r
 }
 
 // ---- choice of experts ------------------------------------------------------------------------
-struct ChooseArgs {
-  const float* logits; int64_t M;
-  int E, top, groups, keep;
-  float scale;
-  const int* count; int L;            // tokens l >= count[b] of a sequence are padding: no expert
-  int* ids; float* weight;            // [M][top]; id -1: none
-  int* pos;                           // nullable: choice -> its row where rows lie in the order of the choices
-  int* counts; int* rank;             // nullable: tokens per expert (zeroed by the caller), a choice's rank among its expert's
-};
-
-__device__ __forceinline__ unsigned ordered(float z) {
-  const unsigned u = __builtin_bit_cast(unsigned, z);
-  return u & 0x80000000u ? ~u : u | 0x80000000u;
-}
-
-// one wave per token; lane holds experts lane + 64 i.  Softmax is monotone: the choice is made on the logits.
-template <int EPL>
-__device__ __forceinline__ void choose_one(const ChooseArgs& a, int64_t m, int lane, float* gmax, int (&my_id), float (&my_w)) {
-  my_id = -1;
-  my_w = 0.f;
-  const int b = a.count ? (int)(m / a.L) : 0;
-  if (a.count && (int)(m - (int64_t)b * a.L) >= a.count[b]) return;
-  float z[EPL], zmax = -INFINITY;
-#pragma unroll
-  for (int i = 0; i < EPL; ++i) {
-    const int e = lane + 64 * i;
-    z[i] = e < a.E ? a.logits[m * a.E + e] : -INFINITY;
-    zmax = fmaxf(zmax, z[i]);
-  }
-  zmax = vy_wave_max(zmax);
-  float sum = 0.f;
-#pragma unroll
-  for (int i = 0; i < EPL; ++i) sum += expf(z[i] - zmax);   // (exp(-inf) = 0 behind the last expert)
-  sum = vy_wave_sum(sum);
-  unsigned key[EPL];
-#pragma unroll
-  for (int i = 0; i < EPL; ++i) key[i] = lane + 64 * i < a.E ? ordered(z[i]) : 0u;
-  if (a.keep < a.groups) {
-    // a group's score is its best expert's; a group stays if fewer than `keep` others are better (ties: the earlier one)
-    const int size = a.E / a.groups;
-    float* zs = gmax + MAX_E;
-#pragma unroll
-    for (int i = 0; i < EPL; ++i)
-      if (lane + 64 * i < a.E) zs[lane + 64 * i] = z[i];
-    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
-    for (int g = lane; g < a.groups; g += 64) {
-      float best = -INFINITY;
-      for (int j = 0; j < size; ++j) best = fmaxf(best, zs[g * size + j]);
-      gmax[g] = best;
-    }
-    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
-#pragma unroll
-    for (int i = 0; i < EPL; ++i) {
-      const int e = lane + 64 * i;
-      if (e < a.E) {
-        const int g = e / size;
-        const float mine = gmax[g];
-        int better = 0;
-        for (int j = 0; j < a.groups; ++j) better += gmax[j] > mine || (gmax[j] == mine && j < g);
-        if (better >= a.keep) key[i] = 0u;
-      }
-    }
-    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
-  }
-  float total = 0.f;
-  for (int k = 0; k < a.top; ++k) {
-    // best remaining key, the lower expert of equal ones
-    unsigned bk = 0u;
-    int be = MAX_E;
-#pragma unroll
-    for (int i = 0; i < EPL; ++i)
-      if (key[i] > bk) { bk = key[i]; be = lane + 64 * i; }
-#pragma unroll
-    for (int o = 32; o > 0; o >>= 1) {
-      const unsigned ok = (unsigned)__shfl_xor((int)bk, o, 64);
-      const int oe = __shfl_xor(be, o, 64);
-      if (ok > bk || (ok == bk && oe < be)) { bk = ok; be = oe; }
-    }
-    if (bk == 0u) break;
-    float ze = 0.f;
-#pragma unroll
-    for (int i = 0; i < EPL; ++i)
-      if (lane + 64 * i == be) { ze = z[i]; key[i] = 0u; }
-    ze = __shfl(ze, be & 63, 64);
-    const float s = expf(ze - zmax) / sum;
-    total += s;
-    if (lane == k) { my_id = be; my_w = s; }
-  }
-  my_w = my_w / (total + 1e-20f) * a.scale;
-}
-
 // TPW tokens per wave; ranks: the workgroup's choices are counted in LDS, one global add per expert and workgroup
 template <int EPL>
 __global__ __launch_bounds__(256) void choose_kernel(ChooseArgs a, int tpw) {
-  __shared__ float groups[4][2 * MAX_E];
-  __shared__ int hist[MAX_E], base[MAX_E];
+  __shared__ float groups[4][2 * 64 * EPL];
+  __shared__ int hist[64 * EPL], base[64 * EPL];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int64_t m0 = ((int64_t)blockIdx.x * 4 + wave) * tpw;
   if (a.counts) {
@@ -285,12 +193,6 @@ __global__ __launch_bounds__(256) void sort_kernel(SortArgs a) {
 }
 
 // ---- the experts, many tokens -----------------------------------------------------------------
-__device__ __forceinline__ float clamped_act(float g, float u, float limit, float alpha) {
-  g = fminf(g, limit);
-  u = fminf(fmaxf(u, -limit), limit);
-  return g * vy_sigmoid(alpha * g) * (u + 1.f);
-}
-
 __device__ __forceinline__ int xcd_remap(int bid, int nwg) {
   const int xcd = bid & 7, q = nwg >> 3, r = nwg & 7;
   return (xcd < r ? xcd * (q + 1) : r * (q + 1) + (xcd - r) * q) + (bid >> 3);
@@ -501,105 +403,10 @@ __global__ __launch_bounds__(256) void grouped_gemm_f32_kernel(GroupedArgs a) {
 }
 
 // ---- the experts, few tokens ------------------------------------------------------------------
-struct RowsArgs {
-  const bf16* x; int64_t ldx;          // GU: rows of h by token; else activation rows by choice
-  const int* ids; int n, top, E;       // n = tokens * top choices
-  const bf16* w; int N, K;             // [E][N][K]
-  bf16* y; int64_t ldy;                // rows by choice
-  float limit, alpha;
-};
-
-// The blockIdx.y-th expert in use (in order of its number) x 16 NT weight rows; the four waves split K.
 template <bool GU, int NT>
-__global__ __launch_bounds__(256) void expert_rows_kernel(RowsArgs a) {
-  __shared__ unsigned used[MAX_E / 32];
-  __shared__ int who, found, list[MAX_ENTRIES];
-  __shared__ f32x4 red[3][NT][64];
-  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, r16 = lane & 15, kq = lane >> 4;
-  if (tid < MAX_E / 32) used[tid] = 0u;
-  if (tid == 0) { who = -1; found = 0; }
-  __syncthreads();
-  for (int i = tid; i < a.n; i += 256) {
-    const int id = a.ids[i];
-    if (id >= 0) atomicOr(&used[id >> 5], 1u << (id & 31));
-  }
-  __syncthreads();
-  if (tid < 32) {
-    const unsigned bits = used[tid];
-    int before = __popc(bits);
-#pragma unroll
-    for (int o = 1; o < 32; o <<= 1) {
-      const int v = __shfl_up(before, o, 32);
-      if (lane >= o) before += v;
-    }
-    before -= __popc(bits);
-    int want = (int)blockIdx.y - before;
-    if (want >= 0 && want < __popc(bits)) {
-      unsigned rest = bits;
-      while (want--) rest &= rest - 1;
-      who = tid * 32 + __ffs((int)rest) - 1;
-    }
-  }
-  __syncthreads();
-  const int e = who;
-  if (e < 0) return;
-  for (int i = tid; i < a.n; i += 256)
-    if (a.ids[i] == e) list[atomicAdd(&found, 1)] = i;   // (any order: rows do not touch each other)
-  __syncthreads();
-  const int cnt = found, n0 = blockIdx.x * 16 * NT;
-  const bf16* ws[NT];
-#pragma unroll
-  for (int t = 0; t < NT; ++t) ws[t] = a.w + ((int64_t)e * a.N + min(n0 + 16 * t + r16, a.N - 1)) * a.K + 8 * kq;
-  const bf16x8 zero8 = {(bf16)0.f, (bf16)0.f, (bf16)0.f, (bf16)0.f, (bf16)0.f, (bf16)0.f, (bf16)0.f, (bf16)0.f};
-  for (int m0 = 0; m0 < cnt; m0 += 16) {
-    const int mine = list[m0 + r16 < cnt ? m0 + r16 : cnt - 1];
-    const bf16* xs = a.x + (int64_t)(GU ? mine / a.top : mine) * a.ldx + 8 * kq;
-    f32x4 acc[NT];
-#pragma unroll
-    for (int t = 0; t < NT; ++t) acc[t] = f32x4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll 8
-    for (int k = 32 * wave; k < a.K; k += 128) {
-      const bool in = k + 8 * kq < a.K;
-      const bf16x8 b = in ? *reinterpret_cast<const bf16x8*>(xs + k) : zero8;
-#pragma unroll
-      for (int t = 0; t < NT; ++t) {
-        const bf16x8 w8 = in ? *reinterpret_cast<const bf16x8*>(ws[t] + k) : zero8;
-        acc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(w8, b, acc[t], 0, 0, 0);
-      }
-    }
-    __syncthreads();
-    if (wave)
-#pragma unroll
-      for (int t = 0; t < NT; ++t) red[wave - 1][t][lane] = acc[t];
-    __syncthreads();
-    if (wave == 0 && m0 + r16 < cnt) {
-#pragma unroll
-      for (int t = 0; t < NT; ++t) {
-        f32x4 v = acc[t];
-#pragma unroll
-        for (int s = 0; s < 3; ++s) {
-          const f32x4 x = red[s][t][lane];
-#pragma unroll
-          for (int r = 0; r < 4; ++r) v[r] += x[r];
-        }
-        const int n = n0 + 16 * t + 4 * kq;
-        if (n < a.N) {
-          bf16* y = a.y + (int64_t)mine * a.ldy;
-          if constexpr (GU) {
-            bf16x2 w2;
-            w2[0] = (bf16)clamped_act(v[0], v[1], a.limit, a.alpha);
-            w2[1] = (bf16)clamped_act(v[2], v[3], a.limit, a.alpha);
-            *reinterpret_cast<bf16x2*>(y + n / 2) = w2;
-          } else {
-            bf16x4 w4;
-#pragma unroll
-            for (int r = 0; r < 4; ++r) w4[r] = (bf16)v[r];
-            *reinterpret_cast<bf16x4*>(y + n) = w4;
-          }
-        }
-      }
-    }
-  }
+__global__ __launch_bounds__(256) void expert_rows_kernel(ExpertRows a) {
+  __shared__ ExpertLds<NT> lds;
+  expert_rows<GU, NT>(a, lds, blockIdx.x, blockIdx.y);
 }
 
 // ---- activation of packed [gate | up] rows ----------------------------------------------------
@@ -696,11 +503,11 @@ extern "C" int vy_moe_fwd(const vy_moe* d, const void* h, int64_t ldh, int64_t M
     hipLaunchKernelGGL((router_logits_kernel<1, 1>), dim3((unsigned)vy_cdiv(E, 16), (unsigned)vy_cdiv(M, 16)), dim3(256), 0, st,
                        (const bf16*)h, ldh, (const bf16*)d->w_router, p.logits, M, K, E);
   } else {
-    hipLaunchKernelGGL((router_logits_kernel<4, 2>), dim3((unsigned)vy_cdiv(E, 64), (unsigned)vy_cdiv(M, 32)), dim3(256), 0, st,
+    hipLaunchKernelGGL((router_logits_kernel<4, 1>), dim3((unsigned)vy_cdiv(E, 64), (unsigned)vy_cdiv(M, 16)), dim3(256), 0, st,
                        (const bf16*)h, ldh, (const bf16*)d->w_router, p.logits, M, K, E);
   }
   ChooseArgs c{p.logits, M, E, d->top, d->groups, d->keep, d->scale, count, (int)L, ids, weight, small ? pos : nullptr, small ? nullptr : p.counts, p.rank};
-  const int tpw = small ? 1 : 8;
+  const int tpw = small ? 1 : 2;
   const dim3 cgrid((unsigned)vy_cdiv(M, 4 * tpw)), block(256);
   if (E <= 64) hipLaunchKernelGGL(choose_kernel<1>, cgrid, block, 0, st, c, tpw);
   else if (E <= 128) hipLaunchKernelGGL(choose_kernel<2>, cgrid, block, 0, st, c, tpw);
@@ -708,9 +515,9 @@ extern "C" int vy_moe_fwd(const vy_moe* d, const void* h, int64_t ldh, int64_t M
   else hipLaunchKernelGGL(choose_kernel<16>, cgrid, block, 0, st, c, tpw);
   if (small) {
     const unsigned active = (unsigned)(n < E ? n : E);
-    RowsArgs g{(const bf16*)h, ldh, ids, (int)n, d->top, E, (const bf16*)d->w_gu, 2 * d->ff, K, (bf16*)p.act, d->ff, d->limit, d->alpha};
-    RowsArgs o{(const bf16*)p.act, d->ff, ids, (int)n, d->top, E, (const bf16*)d->w_down, K, d->ff, (bf16*)rows, ldr, 0.f, 0.f};
-    auto go = [&](auto gu, RowsArgs& a) {
+    ExpertRows g{(const bf16*)h, ldh, ids, (int)n, d->top, (const bf16*)d->w_gu, 2 * d->ff, K, (bf16*)p.act, d->ff, d->limit, d->alpha};
+    ExpertRows o{(const bf16*)p.act, d->ff, ids, (int)n, d->top, (const bf16*)d->w_down, K, d->ff, (bf16*)rows, ldr, 0.f, 0.f};
+    auto go = [&](auto gu, ExpertRows& a) {
       constexpr bool GU = decltype(gu)::value;
       if (vy_cdiv(a.N, 16) * active > 1536) hipLaunchKernelGGL((expert_rows_kernel<GU, 2>), dim3((unsigned)vy_cdiv(a.N, 32), active), block, 0, st, a);
       else hipLaunchKernelGGL((expert_rows_kernel<GU, 1>), dim3((unsigned)vy_cdiv(a.N, 16), active), block, 0, st, a);

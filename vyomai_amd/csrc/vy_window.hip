@@ -9,19 +9,11 @@
 //   vy_window_decode   one query token per sequence: rotation of query and key, the new row to the ring, attention over the
 //                      ring, sink, output gate.  Every row of the ring that holds a token is inside the window, so decode
 //                      needs no mask but the row count -- and no order: softmax does not care where a row lies.
-//
-// window_decode_kernel (bf16): a workgroup takes one key/value head of one sequence with ALL its query heads (up to 16 per
-// pass: the ring is streamed once, not once per query head) and a slice of the ring; its four waves walk units of 32 rows on
-// their own.  Swapped products as in attn_fwd_gen_kernel: S^T = K Q^T straight from global memory into MFMA operands (a key
-// row is read once, nobody else needs it: no LDS), P stays in registers as the B operand of O^T = V^T P^T, V passes through a
-// wave-private LDS tile for the transposing reads.  Rows of the next unit are requested before the arithmetic of this one.
-// The token's own key and value never make the trip to memory and back: they replace row p % R in registers / LDS.
-#include "vy_common.h"
-#include <float.h>
+#include "vy_window.h"
 
 namespace {
 
-constexpr float LOG2E = 1.4426950408889634f;
+using namespace vy_window;
 
 struct RowsArgs {
   const void* p; int64_t ldp, ok, ov;       // packed rows; key / value columns
@@ -104,309 +96,15 @@ __global__ __launch_bounds__(256) void window_context_kernel(ContextArgs a) {
 }
 
 // ---- decode ---------------------------------------------------------------------------------
-struct DecodeArgs {
-  const bf16* p; int64_t ldp, oq, ok, ov, og;
-  bf16* ring; int64_t r_ss, r_sh; int R;
-  const float2* rope; int half, rope_len;
-  const int* slots; const int* start;
-  bf16* out; int64_t ldo;
-  int h, hk, dim, vdim, ns, passes, sink;   // ns slices of the ring, passes of 16 query heads per key/value head
-  float scale;
-  float* part_o; float* part_ml;            // ns > 1: [b][head][slice][vdim] and [b][head][slice][2]
-};
-
-__device__ __forceinline__ float group_max(float v) {   // over the four lane groups (lane >> 4)
-  const unsigned u = __builtin_bit_cast(unsigned, v);
-  auto s = __builtin_amdgcn_permlane16_swap(u, u, false, false);
-  v = fmaxf(__builtin_bit_cast(float, (unsigned)s[0]), __builtin_bit_cast(float, (unsigned)s[1]));
-  const unsigned w = __builtin_bit_cast(unsigned, v);
-  auto t = __builtin_amdgcn_permlane32_swap(w, w, false, false);
-  return fmaxf(__builtin_bit_cast(float, (unsigned)t[0]), __builtin_bit_cast(float, (unsigned)t[1]));
-}
-__device__ __forceinline__ float group_sum(float v) {
-  const unsigned u = __builtin_bit_cast(unsigned, v);
-  auto s = __builtin_amdgcn_permlane16_swap(u, u, false, false);
-  v = __builtin_bit_cast(float, (unsigned)s[0]) + __builtin_bit_cast(float, (unsigned)s[1]);
-  const unsigned w = __builtin_bit_cast(unsigned, v);
-  auto t = __builtin_amdgcn_permlane32_swap(w, w, false, false);
-  return __builtin_bit_cast(float, (unsigned)t[0]) + __builtin_bit_cast(float, (unsigned)t[1]);
-}
-
-__device__ __forceinline__ bf16x8 rotate8(const DecodeArgs& a, const float2* t, int d0, bf16x8 x) {
-  if (d0 >= 2 * a.half) return x;
-  bf16x8 y = x;
-#pragma unroll
-  for (int e = 0; e < 8; e += 2) {
-    const int i = (d0 + e) >> 1;
-    if (i < a.half) {
-      const float2 cs = t[i];
-      const float u = (float)x[e], w = (float)x[e + 1];
-      y[e] = (bf16)(u * cs.x - w * cs.y);
-      y[e + 1] = (bf16)(w * cs.x + u * cs.y);
-    }
-  }
-  return y;
-}
-
 template <int DHP, int DVP>
 __global__ __launch_bounds__(256) void window_decode_kernel(DecodeArgs a) {
-  constexpr int KS = DHP / 32, NDB = DVP / 16;
-  constexpr int VPITCH = (DVP + 8) * 2;              // bytes per row of a wave's value tile
-  constexpr int VROWS = 32 * VPITCH, VC = DVP / 8;   // 16-byte chunks per value row
-  constexpr int VPL = 32 * VC / 64;                  // value chunks per lane and unit
-  constexpr int QP = DHP + 8;                        // query pitch (elements)
-  // [value tiles, later the waves' results | queries | new key | new value | m, l of the waves]
-  constexpr int O_Q = 4 * VROWS, O_K = O_Q + 16 * QP * 2, O_V = O_K + DHP * 2, O_ML = O_V + DVP * 2;
-  static_assert(4 * 16 * DVP * 4 <= 4 * VROWS, "the waves' results fit over the value tiles");
-  __shared__ __attribute__((aligned(16))) char smem[O_ML + 2 * 64 * 4];
-  const int tid = threadIdx.x, lane = tid & 63;
-  const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
-  const int r16 = lane & 15, kq = lane >> 4;
-  const int slice = blockIdx.x, b = blockIdx.z;
-  const int g = (int)blockIdx.y / a.passes, pass = (int)blockIdx.y - g * a.passes;
-  const int rep = a.h / a.hk, h0 = g * rep + pass * 16, nh = min(16, rep - pass * 16);
-  const int slot = a.slots ? a.slots[b] : b;
-  const int pos = a.start[slot];
-  const int n = min(pos + 1, a.R), fresh = pos % a.R;
-  const int W = a.dim + a.vdim;
-  const bf16* row = a.p + (int64_t)b * a.ldp;
-  bf16* ring = a.ring + (int64_t)slot * a.r_ss + (int64_t)g * a.r_sh;
-  const float2* trig = a.rope + (int64_t)min(pos, a.rope_len - 1) * a.half;
-  const bf16x8 zero8 = {(bf16)0.f, (bf16)0.f, (bf16)0.f, (bf16)0.f, (bf16)0.f, (bf16)0.f, (bf16)0.f, (bf16)0.f};
-  const int units = (n + 31) / 32, step = a.ns * 4;
-  int u = slice * 4 + wave;
-
-  // keys and values of a unit in registers: key rows as MFMA operands, values chunk by chunk (whole rows per instruction)
-  bf16x8 kf[2][KS], vr[VPL];
-  auto request = [&](int unit, bf16x8 (&kd)[2][KS], bf16x8 (&vd)[VPL]) {
-#pragma unroll
-    for (int blk = 0; blk < 2; ++blk) {
-      const int j = min(unit * 32 + 16 * blk + r16, n - 1);
-#pragma unroll
-      for (int ks = 0; ks < KS; ++ks) {
-        const int d0 = 32 * ks + 8 * kq;
-        kd[blk][ks] = d0 < a.dim ? *reinterpret_cast<const bf16x8*>(ring + (int64_t)j * W + d0) : zero8;
-      }
-    }
-#pragma unroll
-    for (int i = 0; i < VPL; ++i) {
-      const int c = lane + 64 * i, j = min(unit * 32 + c / VC, n - 1), d0 = (c % VC) * 8;
-      vd[i] = d0 < a.vdim ? *reinterpret_cast<const bf16x8*>(ring + (int64_t)j * W + a.dim + d0) : zero8;
-    }
-  };
-  if (u < units) request(u, kf, vr);
-
-  // rotated queries, new key, new value
-  bf16* lq = reinterpret_cast<bf16*>(smem + O_Q);
-  bf16* lk = reinterpret_cast<bf16*>(smem + O_K);
-  bf16* lv = reinterpret_cast<bf16*>(smem + O_V);
-  for (int i = tid; i < 16 * (DHP / 8); i += 256) {
-    const int hh = i / (DHP / 8), d0 = (i % (DHP / 8)) * 8;
-    const bool ok = hh < nh && d0 < a.dim;
-    bf16x8 q = zero8;
-    if (ok) q = rotate8(a, trig, d0, *reinterpret_cast<const bf16x8*>(row + a.oq + (int64_t)(h0 + hh) * a.dim + d0));
-    *reinterpret_cast<bf16x8*>(lq + hh * QP + d0) = q;
-  }
-  const bool owner = pass == 0 && (fresh / 32) % step / 4 == slice;   // the workgroup whose units hold the new row
-  if (tid >= 192 && tid - 192 < DHP / 8) {
-    const int d0 = (tid - 192) * 8;
-    bf16x8 k8 = zero8;
-    if (d0 < a.dim) {
-      k8 = rotate8(a, trig, d0, *reinterpret_cast<const bf16x8*>(row + a.ok + (int64_t)g * a.dim + d0));
-      if (owner) *reinterpret_cast<bf16x8*>(ring + (int64_t)fresh * W + d0) = k8;
-    }
-    *reinterpret_cast<bf16x8*>(lk + d0) = k8;
-  } else if (tid >= 128 && tid < 192 && tid - 128 < VC) {
-    const int d0 = (tid - 128) * 8;
-    bf16x8 v8 = zero8;
-    if (d0 < a.vdim) {
-      v8 = *reinterpret_cast<const bf16x8*>(row + a.ov + (int64_t)g * a.vdim + d0);
-      if (owner) *reinterpret_cast<bf16x8*>(ring + (int64_t)fresh * W + a.dim + d0) = v8;
-    }
-    *reinterpret_cast<bf16x8*>(lv + d0) = v8;
-  }
-  __syncthreads();
-  bf16x8 qf[KS];
-#pragma unroll
-  for (int ks = 0; ks < KS; ++ks) qf[ks] = *reinterpret_cast<const bf16x8*>(lq + r16 * QP + 32 * ks + 8 * kq);
-
-  f32x4 o[NDB];
-#pragma unroll
-  for (int d = 0; d < NDB; ++d) o[d] = f32x4{0.f, 0.f, 0.f, 0.f};
-  float m_run = -FLT_MAX, l_run = 0.f;
-  const float c = a.scale * LOG2E;
-  char* vt = smem + wave * VROWS;
-  const unsigned vtr = vy_lds_addr(vt) + (4 * kq + (r16 >> 2)) * VPITCH + (4 * (r16 & 3)) * 2;
-  for (; u < units; u += step) {
-    const int j0 = u * 32;
-    if (fresh >= j0 && fresh < j0 + 32) {   // wave-uniform
-      if (r16 == (fresh & 15)) {
-#pragma unroll
-        for (int blk = 0; blk < 2; ++blk)
-          if (blk == ((fresh >> 4) & 1))
-#pragma unroll
-            for (int ks = 0; ks < KS; ++ks) kf[blk][ks] = *reinterpret_cast<const bf16x8*>(lk + 32 * ks + 8 * kq);
-      }
-#pragma unroll
-      for (int i = 0; i < VPL; ++i) {
-        const int cc = lane + 64 * i;
-        if (cc / VC == (fresh & 31)) vr[i] = *reinterpret_cast<const bf16x8*>(lv + (cc % VC) * 8);
-      }
-    }
-    if (j0 + 32 > n) {   // rows behind the last one weigh 0, whatever an earlier owner of the slot left there
-#pragma unroll
-      for (int i = 0; i < VPL; ++i)
-        if (j0 + (lane + 64 * i) / VC >= n) vr[i] = zero8;
-    }
-#pragma unroll
-    for (int i = 0; i < VPL; ++i) {
-      const int cc = lane + 64 * i;
-      *reinterpret_cast<bf16x8*>(vt + (cc / VC) * VPITCH + (cc % VC) * 16) = vr[i];
-    }
-    f32x4 sc[2];
-#pragma unroll
-    for (int blk = 0; blk < 2; ++blk) {
-      sc[blk] = f32x4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-      for (int ks = 0; ks < KS; ++ks) sc[blk] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[blk][ks], qf[ks], sc[blk], 0, 0, 0);
-    }
-    if (u + step < units) request(u + step, kf, vr);   // lands under this unit's softmax and value product
-    float tmax = -INFINITY;
-#pragma unroll
-    for (int blk = 0; blk < 2; ++blk)
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        if (j0 + 16 * blk + 4 * kq + r >= n) sc[blk][r] = -INFINITY;
-        tmax = fmaxf(tmax, sc[blk][r]);
-      }
-    const float m_new = fmaxf(m_run, group_max(tmax) * c);
-    const float alpha = __builtin_amdgcn_exp2f(m_run - m_new);
-    m_run = m_new;
-    l_run *= alpha;
-#pragma unroll
-    for (int d = 0; d < NDB; ++d)
-#pragma unroll
-      for (int r = 0; r < 4; ++r) o[d][r] *= alpha;
-    bf16x8 pf;
-#pragma unroll
-    for (int blk = 0; blk < 2; ++blk)
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const float e = __builtin_amdgcn_exp2f(fmaf(sc[blk][r], c, -m_run));
-        l_run += e;
-        pf[4 * blk + r] = (bf16)e;
-      }
-    vy_static_for<NDB>([&](auto d_c) {
-      constexpr int d = decltype(d_c)::value;
-      union { struct { s16x4 a, b; } hh; bf16x8 v; } uu;
-      uu.hh.a = vy_lds_tr16_off<d * 32>(vtr);
-      uu.hh.b = vy_lds_tr16_off<d * 32 + 16 * VPITCH>(vtr);
-      asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
-      vy_tie(uu.v);
-      o[d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(uu.v, pf, o[d], 0, 0, 0);
-    });
-  }
-  l_run = group_sum(l_run);
-
-  // the four waves' results through LDS
-  __syncthreads();
-  float* lo = reinterpret_cast<float*>(smem);                    // [wave][head][DVP]
-  float* lml = reinterpret_cast<float*>(smem + O_ML);            // m [wave][16], l [wave][16]
-#pragma unroll
-  for (int d = 0; d < NDB; ++d) *reinterpret_cast<f32x4*>(lo + (wave * 16 + r16) * DVP + 16 * d + 4 * kq) = o[d];
-  if (kq == 0) {
-    lml[wave * 16 + r16] = m_run;
-    lml[64 + wave * 16 + r16] = l_run;
-  }
-  __syncthreads();
-  for (int i = tid; i < nh * (a.vdim / 8); i += 256) {
-    const int hh = i / (a.vdim / 8), d0 = (i % (a.vdim / 8)) * 8, head = h0 + hh;
-    float m = fmaxf(fmaxf(lml[hh], lml[16 + hh]), fmaxf(lml[32 + hh], lml[48 + hh]));
-    if (a.ns == 1 && a.sink) m = fmaxf(m, 0.f);
-    float l = a.ns == 1 && a.sink ? __builtin_amdgcn_exp2f(-m) : 0.f, v[8];
-#pragma unroll
-    for (int e = 0; e < 8; ++e) v[e] = 0.f;
-#pragma unroll
-    for (int w = 0; w < 4; ++w) {
-      const float s = __builtin_amdgcn_exp2f(lml[w * 16 + hh] - m);
-      l += s * lml[64 + w * 16 + hh];
-#pragma unroll
-      for (int e = 0; e < 8; ++e) v[e] = fmaf(s, lo[(w * 16 + hh) * DVP + d0 + e], v[e]);
-    }
-    if (a.ns == 1) {
-      const float inv = 1.f / l;
-      bf16x8 w8;
-#pragma unroll
-      for (int e = 0; e < 8; ++e) v[e] *= inv;
-      if (a.og >= 0) {
-        const bf16x8 g8 = *reinterpret_cast<const bf16x8*>(row + a.og + (int64_t)head * a.vdim + d0);
-#pragma unroll
-        for (int e = 0; e < 8; ++e) v[e] *= vy_sigmoid((float)g8[e]);
-      }
-#pragma unroll
-      for (int e = 0; e < 8; ++e) w8[e] = (bf16)v[e];
-      *reinterpret_cast<bf16x8*>(a.out + (int64_t)b * a.ldo + (int64_t)head * a.vdim + d0) = w8;
-    } else {
-      const int64_t at = ((int64_t)b * a.h + head) * a.ns + slice;
-      VyChunk<float>::store(a.part_o + at * a.vdim + d0, v);
-      VyChunk<float>::store(a.part_o + at * a.vdim + d0 + 4, v + 4);
-      if (d0 == 0) { a.part_ml[2 * at] = m; a.part_ml[2 * at + 1] = l; }
-    }
-  }
+  __shared__ __attribute__((aligned(16))) char smem[WindowDecode<DHP, DVP>::LDS];
+  WindowDecode<DHP, DVP>::run(a, smem, blockIdx.x, blockIdx.y, blockIdx.z);
 }
 
-// one workgroup per (sequence, head): sink, slices, gate
 __global__ __launch_bounds__(256) void window_finish_kernel(DecodeArgs a) {
-  __shared__ float red[256 * 4];
-  const int head = blockIdx.x, b = blockIdx.y, tid = threadIdx.x;
-  const float* ml = a.part_ml + ((int64_t)b * a.h + head) * a.ns * 2;
-  const float* po = a.part_o + ((int64_t)b * a.h + head) * a.ns * a.vdim;
-  const int nc = a.vdim / 4, lanes = nc <= 64 ? 64 : nc <= 128 ? 128 : 256, groups = 256 / lanes;
-  const int ch = tid % lanes, grp = tid / lanes;
-  float m = a.sink ? 0.f : -FLT_MAX;
-  for (int s = 0; s < a.ns; ++s) m = fmaxf(m, ml[2 * s]);
-  float l = a.sink ? __builtin_amdgcn_exp2f(-m) : 0.f;
-  f32x4 v = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll 4
-  for (int s = 0; s < a.ns; ++s) l += ml[2 * s + 1] * __builtin_amdgcn_exp2f(ml[2 * s] - m);
-  if (ch < nc) {
-#pragma unroll 4
-    for (int s = grp; s < a.ns; s += groups) {
-      const float f = __builtin_amdgcn_exp2f(ml[2 * s] - m);
-      const f32x4 x = *reinterpret_cast<const f32x4*>(po + (int64_t)s * a.vdim + ch * 4);
-#pragma unroll
-      for (int e = 0; e < 4; ++e) v[e] = fmaf(f, x[e], v[e]);
-    }
-  }
-  *reinterpret_cast<f32x4*>(red + tid * 4) = v;
-  __syncthreads();
-  if (grp == 0 && ch < nc) {
-    for (int s = 1; s < groups; ++s) {
-      const f32x4 x = *reinterpret_cast<const f32x4*>(red + (s * lanes + ch) * 4);
-#pragma unroll
-      for (int e = 0; e < 4; ++e) v[e] += x[e];
-    }
-    const float inv = 1.f / l;
-#pragma unroll
-    for (int e = 0; e < 4; ++e) v[e] *= inv;
-    if (a.og >= 0) {
-      const bf16x4 g4 = *reinterpret_cast<const bf16x4*>(a.p + (int64_t)b * a.ldp + a.og + (int64_t)head * a.vdim + ch * 4);
-#pragma unroll
-      for (int e = 0; e < 4; ++e) v[e] *= vy_sigmoid((float)g4[e]);
-    }
-    bf16x4 w;
-#pragma unroll
-    for (int e = 0; e < 4; ++e) w[e] = (bf16)v[e];
-    *reinterpret_cast<bf16x4*>(a.out + (int64_t)b * a.ldo + (int64_t)head * a.vdim + ch * 4) = w;
-  }
-}
-
-// slices of the ring: about 512 workgroups in all, at least 128 rows (one unit per wave) each
-int slices_of(int64_t workgroups, int64_t rows) {
-  int64_t ns = (512 + workgroups - 1) / workgroups;
-  const int64_t most = (rows + 127) / 128;
-  if (ns > most) ns = most;
-  return (int)(ns < 1 ? 1 : ns > 64 ? 64 : ns);
+  __shared__ __attribute__((aligned(16))) float red[FINISH_LDS / 4];
+  window_finish(a, red, blockIdx.x, blockIdx.y);
 }
 
 template <int DHP>
