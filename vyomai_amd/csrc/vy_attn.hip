@@ -67,6 +67,18 @@ __device__ __forceinline__ void attn_rotate(const AttnParams& p, int b, int qi, 
   int pos = attn_start(p, b) + qi;
   pos = pos < p.rope_len ? pos : p.rope_len - 1;   // (padding rows only)
   const float2* t = p.rope + (int64_t)pos * p.rope_half;
+  if (d0 + N <= 2 * p.rope_half && (p.rope_half & 1) == 0 && N % 4 == 0) {   // whole 16-byte pieces of the table's row
+#pragma unroll
+    for (int e = 0; e < N; e += 4) {
+      const f32x4 cs = *reinterpret_cast<const f32x4*>(t + ((d0 + e) >> 1));
+      const float u = v[e], w = v[e + 1], x = v[e + 2], y = v[e + 3];
+      v[e] = u * cs[0] - w * cs[1];
+      v[e + 1] = w * cs[0] + u * cs[1];
+      v[e + 2] = x * cs[2] - y * cs[3];
+      v[e + 3] = y * cs[2] + x * cs[3];
+    }
+    return;
+  }
 #pragma unroll
   for (int e = 0; e < N; e += 2) {
     const int i = (d0 + e) >> 1;
@@ -441,6 +453,18 @@ __global__ __launch_bounds__(256, DH == 64 ? 3 : 1) void attn_fwd_mfma_kernel(At
     }
   }
   const float inv = 1.0f / l_tot;
+  constexpr int LPR = RB / 16;                         // lanes per output row
+  // gate chunks are requested together here: behind the first store each load would wait for its own round trip
+  bf16x8 g8[EXT ? 32 * LPR / 64 : 1];
+  if constexpr (EXT != 0) {
+    if (p.gate) {
+#pragma unroll
+      for (int it = 0; it < 32 * LPR / 64; ++it) {
+        const int r = q0 + wave * 32 + (it * 64 + lane) / LPR, ch = (it * 64 + lane) % LPR;
+        g8[it] = *reinterpret_cast<const bf16x8*>((const bf16*)p.gate + (int64_t)b * p.g_sb + (int64_t)min(r, p.L - 1) * p.g_sl + head * DH + ch * 8);
+      }
+    }
+  }
   // The wave's 32 x DH output tile goes through LDS so that HBM sees whole 16-byte-per-lane row
   // segments (8 or 16 lanes = one row's DH*2 bytes) instead of 8-byte pieces of 32 different rows per
   // store instruction.  Every wave has left the tile loop once the barrier below is passed; each wave
@@ -459,17 +483,15 @@ __global__ __launch_bounds__(256, DH == 64 ? 3 : 1) void attn_fwd_mfma_kernel(At
       *reinterpret_cast<bf16x4*>(ot + fr * OROW + (32 * n + 8 * rg + 4 * fh) * 2) = w;
     }
   asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");   // wave-private tile: no barrier needed
-  constexpr int LPR = RB / 16;                         // lanes per output row
 #pragma unroll
   for (int it = 0; it < 32 * LPR / 64; ++it) {
     const int r = (it * 64 + lane) / LPR, ch = (it * 64 + lane) % LPR;
     const int qrow_ = q0 + wave * 32 + r;
     bf16x8 vv = *reinterpret_cast<const bf16x8*>(ot + r * OROW + ch * 16);
     if constexpr (EXT) {
-      if (p.gate && qrow_ < p.L) {
-        const bf16x8 g8 = *reinterpret_cast<const bf16x8*>((const bf16*)p.gate + (int64_t)b * p.g_sb + (int64_t)qrow_ * p.g_sl + head * DH + ch * 8);
+      if (p.gate) {
 #pragma unroll
-        for (int e = 0; e < 8; ++e) vv[e] = (bf16)((float)vv[e] * vy_sigmoid((float)g8[e]));
+        for (int e = 0; e < 8; ++e) vv[e] = (bf16)((float)vv[e] * vy_sigmoid((float)g8[it][e]));
       }
     }
     if (qrow_ < p.L)
@@ -700,16 +722,20 @@ __global__ __launch_bounds__(256) void attn_fwd_gen_kernel(AttnParams p, int dh)
   if (qi < p.L) {
     bf16* orow = (bf16*)p.out + (int64_t)b * p.o_sb + (int64_t)qi * p.o_sl + head * dv;
     const bf16* grow = EXT && p.gate ? (const bf16*)p.gate + (int64_t)b * p.g_sb + (int64_t)qi * p.g_sl + head * dv : nullptr;
+    bf16x4 g4[EXT ? NDB : 1];   // requested together: behind the first store each load would wait for its own round trip
+    if (EXT && grow) {
+#pragma unroll
+      for (int n = 0; n < NDB; ++n) g4[n] = *reinterpret_cast<const bf16x4*>(grow + (16 * n + 4 * kq < dv ? 16 * n + 4 * kq : 0));
+    }
 #pragma unroll
     for (int n = 0; n < NDB; ++n) {
       const int d0 = 16 * n + 4 * kq;
       if (d0 < dv) {
         bf16x4 w;
         float gt[4] = {1.f, 1.f, 1.f, 1.f};
-        if (grow) {
-          const bf16x4 g4 = *reinterpret_cast<const bf16x4*>(grow + d0);
+        if (EXT && grow) {
 #pragma unroll
-          for (int r = 0; r < 4; ++r) gt[r] = vy_sigmoid((float)g4[r]);
+          for (int r = 0; r < 4; ++r) gt[r] = vy_sigmoid((float)g4[n][r]);
         }
 #pragma unroll
         for (int r = 0; r < 4; ++r) w[r] = (bf16)(o[n][r] * inv * gt[r]);

@@ -20,13 +20,12 @@ namespace {
 using namespace vy_moe_dev;
 
 // ---- router -----------------------------------------------------------------------------------
-// logits[m][e] = sum_k h[m][k] w[e][k], fp32 accumulation and result.  One workgroup: 16 ET experts x 16 MT tokens; the four
-// waves split K.
+// logits[m][e] = sum_k h[m][k] w[e][k], fp32 accumulation and result.  One workgroup: 16 ET experts x 16 MT tokens.
 template <int ET, int MT>
 __global__ __launch_bounds__(256) void router_logits_kernel(const bf16* __restrict__ h, int64_t ldh, const bf16* __restrict__ w,
                                                             float* __restrict__ logits, int64_t M, int K, int E) {
-  __shared__ f32x4 red[3][ET * MT][64];
-  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, r16 = lane & 15, kq = lane >> 4;
+  __shared__ f32x4 red[vy_rows::RED<ET, MT>];
+  const int lane = threadIdx.x & 63, r16 = lane & 15, kq = lane >> 4;
   const int e0 = blockIdx.x * 16 * ET;
   const int64_t m0 = (int64_t)blockIdx.y * 16 * MT;
   const bf16* ws[ET];
@@ -36,48 +35,18 @@ __global__ __launch_bounds__(256) void router_logits_kernel(const bf16* __restri
 #pragma unroll
   for (int j = 0; j < MT; ++j) hs[j] = h + (m0 + 16 * j + r16 < M ? m0 + 16 * j + r16 : M - 1) * ldh + 8 * kq;
   f32x4 acc[ET][MT];
-#pragma unroll
-  for (int i = 0; i < ET; ++i)
-#pragma unroll
-    for (int j = 0; j < MT; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
-  const bf16x8 zero8 = {(bf16)0.f, (bf16)0.f, (bf16)0.f, (bf16)0.f, (bf16)0.f, (bf16)0.f, (bf16)0.f, (bf16)0.f};
-#pragma unroll 8
-  for (int k = 32 * wave; k < K; k += 128) {
-    const bool in = k + 8 * kq < K;
-    bf16x8 a[ET], b[MT];
-#pragma unroll
-    for (int i = 0; i < ET; ++i) a[i] = in ? *reinterpret_cast<const bf16x8*>(ws[i] + k) : zero8;
-#pragma unroll
-    for (int j = 0; j < MT; ++j) b[j] = in ? *reinterpret_cast<const bf16x8*>(hs[j] + k) : zero8;
-#pragma unroll
-    for (int i = 0; i < ET; ++i)
-#pragma unroll
-      for (int j = 0; j < MT; ++j) acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a[i], b[j], acc[i][j], 0, 0, 0);
-  }
-  if (wave)
-#pragma unroll
-    for (int i = 0; i < ET; ++i)
-#pragma unroll
-      for (int j = 0; j < MT; ++j) red[wave - 1][i * MT + j][lane] = acc[i][j];
-  __syncthreads();
-  if (wave) return;
+  vy_rows::stream<ET, MT, false>(ws, hs, K, acc, red);
+  if (threadIdx.x >= 64) return;
 #pragma unroll
   for (int i = 0; i < ET; ++i)
 #pragma unroll
     for (int j = 0; j < MT; ++j) {
-      f32x4 v = acc[i][j];
-#pragma unroll
-      for (int s = 0; s < 3; ++s) {
-        const f32x4 x = red[s][i * MT + j][lane];
-#pragma unroll
-        for (int r = 0; r < 4; ++r) v[r] += x[r];
-      }
       const int64_t m = m0 + 16 * j + r16;
       const int e = e0 + 16 * i + 4 * kq;   // a lane: token r16, experts 4 kq .. + 3
       if (m < M)
 #pragma unroll
         for (int r = 0; r < 4; ++r)
-          if (e + r < E) logits[m * E + e + r] = v[r];
+          if (e + r < E) logits[m * E + e + r] = acc[i][j][r];
     }
 }
 
@@ -98,14 +67,14 @@ __global__ __launch_bounds__(256) void router_logits_f32_kernel(const float* __r
 
 // ---- choice of experts ------------------------------------------------------------------------
 // TPW tokens per wave; ranks: the workgroup's choices are counted in LDS, one global add per expert and workgroup
-template <int EPL>
-__global__ __launch_bounds__(256) void choose_kernel(ChooseArgs a, int tpw) {
-  __shared__ float groups[4][2 * 64 * EPL];
+template <int EPL, int NW>
+__global__ __launch_bounds__(64 * NW) void choose_kernel(ChooseArgs a, int tpw) {
+  __shared__ float groups[NW][2 * 64 * EPL];
   __shared__ int hist[64 * EPL], base[64 * EPL];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-  const int64_t m0 = ((int64_t)blockIdx.x * 4 + wave) * tpw;
+  const int64_t m0 = ((int64_t)blockIdx.x * NW + wave) * tpw;
   if (a.counts) {
-    for (int e = threadIdx.x; e < a.E; e += 256) hist[e] = 0;
+    for (int e = threadIdx.x; e < a.E; e += 64 * NW) hist[e] = 0;
     __syncthreads();
   }
   for (int t = 0; t < tpw; ++t) {
@@ -123,7 +92,7 @@ __global__ __launch_bounds__(256) void choose_kernel(ChooseArgs a, int tpw) {
   }
   if (!a.counts) return;
   __syncthreads();
-  for (int e = threadIdx.x; e < a.E; e += 256) base[e] = hist[e] ? atomicAdd(&a.counts[e], hist[e]) : 0;
+  for (int e = threadIdx.x; e < a.E; e += 64 * NW) base[e] = hist[e] ? atomicAdd(&a.counts[e], hist[e]) : 0;
   __syncthreads();
   for (int t = 0; t < tpw; ++t) {
     const int64_t m = m0 + t;
@@ -503,16 +472,22 @@ extern "C" int vy_moe_fwd(const vy_moe* d, const void* h, int64_t ldh, int64_t M
     hipLaunchKernelGGL((router_logits_kernel<1, 1>), dim3((unsigned)vy_cdiv(E, 16), (unsigned)vy_cdiv(M, 16)), dim3(256), 0, st,
                        (const bf16*)h, ldh, (const bf16*)d->w_router, p.logits, M, K, E);
   } else {
-    hipLaunchKernelGGL((router_logits_kernel<4, 1>), dim3((unsigned)vy_cdiv(E, 64), (unsigned)vy_cdiv(M, 16)), dim3(256), 0, st,
+    hipLaunchKernelGGL((router_logits_kernel<4, 2>), dim3((unsigned)vy_cdiv(E, 64), (unsigned)vy_cdiv(M, 32)), dim3(256), 0, st,
                        (const bf16*)h, ldh, (const bf16*)d->w_router, p.logits, M, K, E);
   }
   ChooseArgs c{p.logits, M, E, d->top, d->groups, d->keep, d->scale, count, (int)L, ids, weight, small ? pos : nullptr, small ? nullptr : p.counts, p.rank};
-  const int tpw = small ? 1 : 2;
-  const dim3 cgrid((unsigned)vy_cdiv(M, 4 * tpw)), block(256);
-  if (E <= 64) hipLaunchKernelGGL(choose_kernel<1>, cgrid, block, 0, st, c, tpw);
-  else if (E <= 128) hipLaunchKernelGGL(choose_kernel<2>, cgrid, block, 0, st, c, tpw);
-  else if (E <= 256) hipLaunchKernelGGL(choose_kernel<4>, cgrid, block, 0, st, c, tpw);
-  else hipLaunchKernelGGL(choose_kernel<16>, cgrid, block, 0, st, c, tpw);
+  // few tokens: a wave each, spread over the CUs; many: 32 per workgroup, so that few global adds count them
+  const dim3 block(256);
+#define CHOOSE(EPL, NW, TPW) hipLaunchKernelGGL((choose_kernel<EPL, NW>), dim3((unsigned)vy_cdiv(M, NW * TPW)), dim3(64 * NW), 0, st, c, TPW)
+  if (small || E > 256) {
+    if (E <= 64) CHOOSE(1, 4, 1);
+    else if (E <= 128) CHOOSE(2, 4, 1);
+    else if (E <= 256) CHOOSE(4, 4, 1);
+    else CHOOSE(16, 4, 2);
+  } else if (E <= 64) CHOOSE(1, 16, 2);
+  else if (E <= 128) CHOOSE(2, 16, 2);
+  else CHOOSE(4, 16, 2);
+#undef CHOOSE
   if (small) {
     const unsigned active = (unsigned)(n < E ? n : E);
     ExpertRows g{(const bf16*)h, ldh, ids, (int)n, d->top, (const bf16*)d->w_gu, 2 * d->ff, K, (bf16*)p.act, d->ff, d->limit, d->alpha};

@@ -1,7 +1,8 @@
 // Weight-streaming products of few rows (decode): a workgroup of four waves takes 16 NT rows of W [N][K] against 16 MB rows of X
 // on mfma_f32_16x16x32_bf16 (A = weight rows, B = rows of X), both straight from memory into operand registers: a weight is used
-// once, and X is small enough for L2.  The waves split K; every wave requests its loads of up to STEPS k-steps before the first
-// product, so a pass over K = 128 STEPS costs one memory latency.  W is streamed past the caches (non-temporal).
+// once, and X is small enough for L2.  The waves split K by whole 128-byte lines (two k-steps of 32); every wave requests its
+// loads of up to STEPS k-steps before the first product, so a pass over K = 128 STEPS costs one memory latency.  W is streamed
+// past the caches (non-temporal) unless other workgroups read it too.
 #pragma once
 #include "vy_common.h"
 
@@ -12,7 +13,7 @@ template <int NT, int MB> constexpr int STEPS = NT * MB == 1 ? 16 : NT + MB <= 3
 
 // acc[t][j] (in wave 0 only) = 16 rows ws[t] x 16 rows xs[j]; a lane's pointers are its row (lane & 15) + 8 (lane >> 4).
 // D: a lane owns row lane & 15 of X and rows 4 (lane >> 4) .. + 3 of W.
-template <int NT, int MB>
+template <int NT, int MB, bool ONCE = true>
 __device__ __forceinline__ void stream(const bf16* const (&ws)[NT], const bf16* const (&xs)[MB], int K, f32x4 (&acc)[NT][MB],
                                        f32x4* red) {
   constexpr int U = STEPS<NT, MB>;
@@ -23,14 +24,18 @@ __device__ __forceinline__ void stream(const bf16* const (&ws)[NT], const bf16* 
   for (int t = 0; t < NT; ++t)
 #pragma unroll
     for (int j = 0; j < MB; ++j) acc[t][j] = f32x4{0.f, 0.f, 0.f, 0.f};
-  for (int k0 = 32 * wave; k0 < K; k0 += 128 * U) {
+  for (int k0 = 64 * wave; k0 < K; k0 += 128 * U) {
     bf16x8 w[U][NT], x[U][MB];
 #pragma unroll
     for (int u = 0; u < U; ++u) {
-      const int k = k0 + 128 * u;
+      const int k = k0 + 256 * (u >> 1) + 32 * (u & 1);
       const bool in = k + 8 * kq < K;
 #pragma unroll
-      for (int t = 0; t < NT; ++t) w[u][t] = in ? __builtin_nontemporal_load(reinterpret_cast<const bf16x8*>(ws[t] + k)) : zero8;
+      for (int t = 0; t < NT; ++t) {
+        const bf16x8* at = reinterpret_cast<const bf16x8*>(ws[t] + k);
+        if constexpr (ONCE) w[u][t] = in ? __builtin_nontemporal_load(at) : zero8;
+        else w[u][t] = in ? *at : zero8;
+      }
 #pragma unroll
       for (int j = 0; j < MB; ++j) x[u][j] = in ? *reinterpret_cast<const bf16x8*>(xs[j] + k) : zero8;
     }
