@@ -196,4 +196,22 @@ __device__ __forceinline__ void expert_rows(const ExpertRows& a, ExpertLds<NT>& 
   }
 }
 
+// a single token: its y-th choice x 8 weight rows (GU: 4 pairs)
+template <bool GU>
+__device__ __forceinline__ void expert_rows1(const ExpertRows& a, int x, int y) {
+  const int e = a.ids[y], n = 8 * x + 2 * (threadIdx.x >> 6);
+  if (e < 0 || n >= a.N) return;   // (N is a multiple of 8)
+  const bf16* w = a.w + ((int64_t)e * a.N + n) * a.K;
+  float s0, s1;
+  vy_rows::gemv2(w, w + a.K, a.x + (GU ? 0 : (int64_t)y * a.ldx), a.K, s0, s1);
+  if (threadIdx.x & 63) return;
+  bf16* yr = a.y + (int64_t)y * a.ldy;
+  if constexpr (GU) {
+    yr[n / 2] = (bf16)clamped_act(s0, s1, a.limit, a.alpha);
+  } else {
+    yr[n] = (bf16)s0;
+    yr[n + 1] = (bf16)s1;
+  }
+}
+
 }  // namespace vy_moe_dev

@@ -19,12 +19,14 @@ namespace {
 
 using namespace vy_moe_dev;
 
+constexpr int COUNT_STRIDE = 32;   // the experts' counters, one per 128-byte line: adds to one line queue up
+
 // ---- router -----------------------------------------------------------------------------------
 // logits[m][e] = sum_k h[m][k] w[e][k], fp32 accumulation and result.  One workgroup: 16 ET experts x 16 MT tokens.
-template <int ET, int MT>
-__global__ __launch_bounds__(256) void router_logits_kernel(const bf16* __restrict__ h, int64_t ldh, const bf16* __restrict__ w,
+template <int ET, int MT, int NW>
+__global__ __launch_bounds__(64 * NW) void router_logits_kernel(const bf16* __restrict__ h, int64_t ldh, const bf16* __restrict__ w,
                                                             float* __restrict__ logits, int64_t M, int K, int E) {
-  __shared__ f32x4 red[vy_rows::RED<ET, MT>];
+  __shared__ f32x4 red[vy_rows::RED<ET, MT, NW>];
   const int lane = threadIdx.x & 63, r16 = lane & 15, kq = lane >> 4;
   const int e0 = blockIdx.x * 16 * ET;
   const int64_t m0 = (int64_t)blockIdx.y * 16 * MT;
@@ -35,7 +37,7 @@ __global__ __launch_bounds__(256) void router_logits_kernel(const bf16* __restri
 #pragma unroll
   for (int j = 0; j < MT; ++j) hs[j] = h + (m0 + 16 * j + r16 < M ? m0 + 16 * j + r16 : M - 1) * ldh + 8 * kq;
   f32x4 acc[ET][MT];
-  vy_rows::stream<ET, MT, false>(ws, hs, K, acc, red);
+  vy_rows::stream<ET, MT, false, NW>(ws, hs, K, acc, red);
   if (threadIdx.x >= 64) return;
 #pragma unroll
   for (int i = 0; i < ET; ++i)
@@ -92,7 +94,7 @@ __global__ __launch_bounds__(64 * NW) void choose_kernel(ChooseArgs a, int tpw) 
   }
   if (!a.counts) return;
   __syncthreads();
-  for (int e = threadIdx.x; e < a.E; e += 64 * NW) base[e] = hist[e] ? atomicAdd(&a.counts[e], hist[e]) : 0;
+  for (int e = threadIdx.x; e < a.E; e += 64 * NW) base[e] = hist[e] ? atomicAdd(&a.counts[e * COUNT_STRIDE], hist[e]) : 0;
   __syncthreads();
   for (int t = 0; t < tpw; ++t) {
     const int64_t m = m0 + t;
@@ -107,10 +109,10 @@ __global__ __launch_bounds__(64 * NW) void choose_kernel(ChooseArgs a, int tpw) 
 // ---- sorting by expert ------------------------------------------------------------------------
 struct Tile { int expert, first, tiles, pad; };   // the expert of a tile, the expert's first tile and tile count
 struct SortArgs {
-  const int* ids; const int* rank; const int* counts;
+  const int* ids; const int* rank; const int* counts;   // counts COUNT_STRIDE apart
   int64_t n; int top, E, bm;
   int* pos; int* token;                // choice -> sorted row, sorted row -> token
-  int* offset;                         // [E] first sorted row of an expert
+  int* offset; int* rows;              // [E] first sorted row and row count of an expert
   Tile* tiles; int* ntiles;
 };
 
@@ -123,7 +125,7 @@ __global__ __launch_bounds__(256) void sort_kernel(SortArgs a) {
 #pragma unroll
   for (int i = 0; i < 4; ++i) {
     const int e = tid * 4 + i;
-    c[i] = e < a.E ? a.counts[e] : 0;
+    c[i] = e < a.E ? a.counts[e * COUNT_STRIDE] : 0;
     rows += c[i];
     tiles += (c[i] + a.bm - 1) / a.bm;
   }
@@ -144,6 +146,7 @@ __global__ __launch_bounds__(256) void sort_kernel(SortArgs a) {
       off[e] = r0;
       if (blockIdx.x == 0) {
         a.offset[e] = r0;
+        a.rows[e] = c[i];
         for (int t = 0; t < nt; ++t) a.tiles[t0 + t] = Tile{e, t0, nt, 0};
       }
     }
@@ -169,7 +172,7 @@ __device__ __forceinline__ int xcd_remap(int bid, int nwg) {
 
 struct GroupedArgs {
   const void* x; int64_t ldx;          // rows of h (gathered by `token`) or sorted activation rows (token NULL)
-  const int* token; const int* offset; const int* counts;
+  const int* token; const int* offset; const int* count;
   const Tile* tiles; const int* ntiles;
   const void* w; int N, K;             // [E][N][K]
   void* y; int64_t ldy;                // sorted rows
@@ -201,7 +204,7 @@ __global__ __launch_bounds__(256) void grouped_gemm_kernel(GroupedArgs a) {
   __shared__ __attribute__((aligned(16))) char smem[2 * STAGE];
   int e, mt, nt;
   if (!grouped_tile(a, (a.N + BN - 1) / BN, e, mt, nt)) return;
-  const int rows = a.counts[e] - mt * BM, row0 = a.offset[e] + mt * BM, n0 = nt * BN;
+  const int rows = a.count[e] - mt * BM, row0 = a.offset[e] + mt * BM, n0 = nt * BN;
   const int N = a.N, K = a.K;
   const bf16* W = (const bf16*)a.w + (int64_t)e * N * K;
   const int tid = threadIdx.x, lane = tid & 63;
@@ -333,7 +336,7 @@ __global__ __launch_bounds__(256) void grouped_gemm_f32_kernel(GroupedArgs a) {
   __shared__ float xs[KB][T + 4], ws[KB][T + 4];
   int e, mt, nt;
   if (!grouped_tile(a, (a.N + T - 1) / T, e, mt, nt)) return;
-  const int rows = a.counts[e] - mt * T, row0 = a.offset[e] + mt * T, n0 = nt * T;
+  const int rows = a.count[e] - mt * T, row0 = a.offset[e] + mt * T, n0 = nt * T;
   const float* W = (const float*)a.w + (int64_t)e * a.N * a.K;
   const int tid = threadIdx.x, lr = tid >> 2, lk = (tid & 3) * 4, ty = tid >> 4, tx = tid & 15;
   const int r = row0 + (lr < rows ? lr : rows - 1);
@@ -410,7 +413,7 @@ int64_t max_tiles(const vy_moe* d, int64_t M, int dtype) {   // every expert in 
   return n / tile_rows(dtype) + e;
 }
 
-struct Parts { float* logits; char* act; int* counts; int* rank; int* token; int* offset; int* ntiles; Tile* tiles; };
+struct Parts { float* logits; char* act; int* counts; int* rank; int* token; int* offset; int* rows; int* ntiles; Tile* tiles; };
 
 int64_t lay_out(const vy_moe* d, int64_t M, int dtype, char* ws, Parts& p) {
   const int64_t n = M * d->top, e = dtype == VY_BF16 ? 2 : 4;
@@ -418,10 +421,11 @@ int64_t lay_out(const vy_moe* d, int64_t M, int dtype, char* ws, Parts& p) {
   auto take = [&](int64_t bytes) { char* r = at; at += up(bytes); return r; };
   p.logits = (float*)take(M * d->experts * 4);
   p.act = take(n * d->ff * e);
-  p.counts = (int*)take(d->experts * 4);
+  p.counts = (int*)take((int64_t)d->experts * COUNT_STRIDE * 4);
   p.rank = (int*)take(n * 4);
   p.token = (int*)take(n * 4);
   p.offset = (int*)take(d->experts * 4);
+  p.rows = (int*)take(d->experts * 4);
   p.ntiles = (int*)take(4);
   p.tiles = (Tile*)take(max_tiles(d, M, dtype) * (int64_t)sizeof(Tile));
   return at - ws;
@@ -464,19 +468,19 @@ extern "C" int vy_moe_fwd(const vy_moe* d, const void* h, int64_t ldh, int64_t M
   const int E = d->experts, K = d->width;
   const int64_t n = M * d->top;
   const bool small = few(d, M, dtype);
-  if (!small) hipLaunchKernelGGL(zero_kernel, dim3((unsigned)vy_cdiv(E, 256)), dim3(256), 0, st, p.counts, E);
+  if (!small) hipLaunchKernelGGL(zero_kernel, dim3((unsigned)vy_cdiv((int64_t)E * COUNT_STRIDE, 256)), dim3(256), 0, st, p.counts, E * COUNT_STRIDE);
   if (dtype == VY_F32) {
     hipLaunchKernelGGL(router_logits_f32_kernel, dim3((unsigned)M, (unsigned)vy_cdiv(E, 4)), dim3(256), 0, st, (const float*)h, ldh,
                        (const float*)d->w_router, p.logits, K, E);
   } else if (M <= 256) {
-    hipLaunchKernelGGL((router_logits_kernel<1, 1>), dim3((unsigned)vy_cdiv(E, 16), (unsigned)vy_cdiv(M, 16)), dim3(256), 0, st,
+    hipLaunchKernelGGL((router_logits_kernel<1, 1, 4>), dim3((unsigned)vy_cdiv(E, 16), (unsigned)vy_cdiv(M, 16)), dim3(256), 0, st,
                        (const bf16*)h, ldh, (const bf16*)d->w_router, p.logits, M, K, E);
   } else {
-    hipLaunchKernelGGL((router_logits_kernel<4, 2>), dim3((unsigned)vy_cdiv(E, 64), (unsigned)vy_cdiv(M, 32)), dim3(256), 0, st,
+    hipLaunchKernelGGL((router_logits_kernel<4, 2, 8>), dim3((unsigned)vy_cdiv(E, 64), (unsigned)vy_cdiv(M, 32)), dim3(512), 0, st,
                        (const bf16*)h, ldh, (const bf16*)d->w_router, p.logits, M, K, E);
   }
   ChooseArgs c{p.logits, M, E, d->top, d->groups, d->keep, d->scale, count, (int)L, ids, weight, small ? pos : nullptr, small ? nullptr : p.counts, p.rank};
-  // few tokens: a wave each, spread over the CUs; many: 32 per workgroup, so that few global adds count them
+  // few tokens: a wave each, spread over the CUs; many: several per workgroup, so that few global adds count them
   const dim3 block(256);
 #define CHOOSE(EPL, NW, TPW) hipLaunchKernelGGL((choose_kernel<EPL, NW>), dim3((unsigned)vy_cdiv(M, NW * TPW)), dim3(64 * NW), 0, st, c, TPW)
   if (small || E > 256) {
@@ -503,10 +507,10 @@ extern "C" int vy_moe_fwd(const vy_moe* d, const void* h, int64_t ldh, int64_t M
     return VY_OK;
   }
   const int bm = tile_rows(dtype);
-  SortArgs s{ids, p.rank, p.counts, n, d->top, E, bm, pos, p.token, p.offset, p.tiles, p.ntiles};
+  SortArgs s{ids, p.rank, p.counts, n, d->top, E, bm, pos, p.token, p.offset, p.rows, p.tiles, p.ntiles};
   hipLaunchKernelGGL(sort_kernel, dim3((unsigned)vy_cdiv(n, 256)), block, 0, st, s);
-  GroupedArgs g{h, ldh, p.token, p.offset, p.counts, p.tiles, p.ntiles, d->w_gu, 2 * d->ff, K, p.act, d->ff, d->limit, d->alpha};
-  GroupedArgs o{p.act, d->ff, nullptr, p.offset, p.counts, p.tiles, p.ntiles, d->w_down, K, d->ff, rows, ldr, 0.f, 0.f};
+  GroupedArgs g{h, ldh, p.token, p.offset, p.rows, p.tiles, p.ntiles, d->w_gu, 2 * d->ff, K, p.act, d->ff, d->limit, d->alpha};
+  GroupedArgs o{p.act, d->ff, nullptr, p.offset, p.rows, p.tiles, p.ntiles, d->w_down, K, d->ff, rows, ldr, 0.f, 0.f};
   const int64_t tiles = max_tiles(d, M, dtype);
   const dim3 ggrid((unsigned)(tiles * vy_cdiv(g.N, bm))), ogrid((unsigned)(tiles * vy_cdiv(o.N, bm)));
   if (dtype == VY_BF16) {

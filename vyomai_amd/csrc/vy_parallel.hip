@@ -17,11 +17,17 @@ using namespace vy_moe_dev;
 using namespace vy_window;
 using vy_rows::Dense;
 
+// MB: blocks of 16 sequences; 0: one sequence (8 weight rows per workgroup instead of 16)
 template <int MB>
 __global__ __launch_bounds__(256) void parallel_in_kernel(Dense in, Dense router, int n_in) {
-  __shared__ f32x4 red[vy_rows::RED<1, MB>];
   const bool first = (int)blockIdx.x < n_in;
-  vy_rows::dense<MB>(first ? in : router, red, first ? blockIdx.x : blockIdx.x - n_in);
+  const int tile = first ? blockIdx.x : blockIdx.x - n_in;
+  if constexpr (MB == 0) {
+    vy_rows::dense1(first ? in : router, tile);
+  } else {
+    __shared__ f32x4 red[vy_rows::RED<1, MB>];
+    vy_rows::dense<MB>(first ? in : router, red, tile);
+  }
 }
 
 struct MixArgs {
@@ -72,18 +78,29 @@ __global__ __launch_bounds__(256) void parallel_mix_kernel(MixArgs a) {
 
 template <int NT>
 __global__ __launch_bounds__(256) void parallel_experts_kernel(DecodeArgs win, int n_finish, ExpertRows ex, int tiles) {
-  __shared__ union { ExpertLds<NT> ex; float red[FINISH_LDS / 4]; } lds;
   const int id = blockIdx.x;
-  if (id < n_finish) window_finish(win, lds.red, id % win.h, id / win.h);
-  else expert_rows<true, NT>(ex, lds.ex, (id - n_finish) % tiles, (id - n_finish) / tiles);
+  if constexpr (NT == 0) {   // one sequence
+    __shared__ __attribute__((aligned(16))) float red[FINISH_LDS / 4];
+    if (id < n_finish) window_finish(win, red, id % win.h, id / win.h);
+    else expert_rows1<true>(ex, (id - n_finish) % tiles, (id - n_finish) / tiles);
+  } else {
+    __shared__ union { ExpertLds<NT> ex; float red[FINISH_LDS / 4]; } lds;
+    if (id < n_finish) window_finish(win, lds.red, id % win.h, id / win.h);
+    else expert_rows<true, NT>(ex, lds.ex, (id - n_finish) % tiles, (id - n_finish) / tiles);
+  }
 }
 
 template <int MB, int NT>
 __global__ __launch_bounds__(256) void parallel_out_kernel(Dense out, int n_out, ExpertRows ex, int tiles) {
-  __shared__ union { ExpertLds<NT> ex; f32x4 red[vy_rows::RED<1, MB>]; } lds;
   const int id = blockIdx.x;
-  if (id < n_out) vy_rows::dense<MB>(out, lds.red, id);
-  else expert_rows<false, NT>(ex, lds.ex, (id - n_out) % tiles, (id - n_out) / tiles);
+  if constexpr (MB == 0) {   // one sequence
+    if (id < n_out) vy_rows::dense1(out, id);
+    else expert_rows1<false>(ex, (id - n_out) % tiles, (id - n_out) / tiles);
+  } else {
+    __shared__ union { ExpertLds<NT> ex; f32x4 red[vy_rows::RED<1, MB>]; } lds;
+    if (id < n_out) vy_rows::dense<MB>(out, lds.red, id);
+    else expert_rows<false, NT>(ex, lds.ex, (id - n_out) % tiles, (id - n_out) / tiles);
+  }
 }
 
 template <int DHP>
@@ -130,7 +147,7 @@ int vy_parallel_decode(const vy_hybrid_plan* p, const vy_hybrid_layer* L, const 
     VY_FAIL(VY_ERR_ARG, "%s: bad mixture", who);
   hipStream_t st = (hipStream_t)stream;
   const dim3 block(256);
-  auto tiles16 = [](int64_t rows) { return (int)((rows + 15) / 16); };
+  auto tiles_of = [&](int64_t rows) { return (int)(B == 1 ? (rows + 7) / 8 : (rows + 15) / 16); };
 
   // input products and router logits
   float* logits = (float*)moe_ws;
@@ -138,10 +155,12 @@ int vy_parallel_decode(const vy_hybrid_plan* p, const vy_hybrid_layer* L, const 
   const Dense din{(const bf16*)h, p->dp, B, (const bf16*)L->w_in, (int)n_in, p->dp, in, n_in, 0};
   const Dense drouter{(const bf16*)h, p->dp, B, d ? (const bf16*)d->w_router : nullptr, d ? d->experts : 0, p->dp, logits,
                       d ? d->experts : 0, 1};
-  const dim3 g_in((unsigned)(tiles16(n_in) + (d ? tiles16(d->experts) : 0)));
-  if (B <= 16) hipLaunchKernelGGL(parallel_in_kernel<1>, g_in, block, 0, st, din, drouter, tiles16(n_in));
-  else if (B <= 32) hipLaunchKernelGGL(parallel_in_kernel<2>, g_in, block, 0, st, din, drouter, tiles16(n_in));
-  else hipLaunchKernelGGL(parallel_in_kernel<4>, g_in, block, 0, st, din, drouter, tiles16(n_in));
+  const int t_in = tiles_of(n_in);
+  const dim3 g_in((unsigned)(t_in + (d ? tiles_of(d->experts) : 0)));
+  if (B == 1) hipLaunchKernelGGL(parallel_in_kernel<0>, g_in, block, 0, st, din, drouter, t_in);
+  else if (B <= 16) hipLaunchKernelGGL(parallel_in_kernel<1>, g_in, block, 0, st, din, drouter, t_in);
+  else if (B <= 32) hipLaunchKernelGGL(parallel_in_kernel<2>, g_in, block, 0, st, din, drouter, t_in);
+  else hipLaunchKernelGGL(parallel_in_kernel<4>, g_in, block, 0, st, din, drouter, t_in);
 
   // attention, choice, shared activation
   MixArgs m{};
@@ -177,18 +196,22 @@ int vy_parallel_decode(const vy_hybrid_plan* p, const vy_hybrid_layer* L, const 
     up = ExpertRows{(const bf16*)h, p->dp, eids, (int)n, d->top, (const bf16*)d->w_gu, 2 * d->ff, p->dp, act, d->ff, d->limit, d->alpha};
     down = ExpertRows{act, d->ff, eids, (int)n, d->top, (const bf16*)d->w_down, p->dp, d->ff, (bf16*)erows, p->dp, 0.f, 0.f};
   }
-  // 16 weight rows per workgroup, 32 where there are plenty
-  auto wide = [&](const ExpertRows& e) { return (int64_t)tiles16(e.N) * active > 1536; };
+  // 16 weight rows per workgroup, 32 where there are plenty (one sequence: 8)
+  auto wide = [&](const ExpertRows& e) { return B > 1 && (int64_t)tiles_of(e.N) * active > 1536; };
+  auto ex_tiles = [&](const ExpertRows& e) { return wide(e) ? (e.N + 31) / 32 : tiles_of(e.N); };
   if (n_finish + active) {
-    if (wide(up)) hipLaunchKernelGGL(parallel_experts_kernel<2>, dim3((unsigned)(n_finish + (up.N + 31) / 32 * active)), block, 0, st, w, n_finish, up, (up.N + 31) / 32);
-    else hipLaunchKernelGGL(parallel_experts_kernel<1>, dim3((unsigned)(n_finish + tiles16(up.N) * active)), block, 0, st, w, n_finish, up, tiles16(up.N));
+    const dim3 grid((unsigned)(n_finish + ex_tiles(up) * active));
+    if (B == 1) hipLaunchKernelGGL(parallel_experts_kernel<0>, grid, block, 0, st, w, n_finish, up, ex_tiles(up));
+    else if (wide(up)) hipLaunchKernelGGL(parallel_experts_kernel<2>, grid, block, 0, st, w, n_finish, up, ex_tiles(up));
+    else hipLaunchKernelGGL(parallel_experts_kernel<1>, grid, block, 0, st, w, n_finish, up, ex_tiles(up));
   }
 
   // output products
   const Dense dout{(const bf16*)ao, na, B, (const bf16*)L->w_o, p->dp, (int)na, y, p->dp, 0};
-  const int n_out = tiles16(p->dp);
-  if (wide(down)) out_go<2>(B, dout, n_out, down, (down.N + 31) / 32, n_out + (down.N + 31) / 32 * active, st);
-  else out_go<1>(B, dout, n_out, down, active ? tiles16(down.N) : 1, n_out + tiles16(down.N) * active, st);
+  const int n_out = tiles_of(p->dp), t_down = ex_tiles(down), blocks_out = n_out + t_down * active;
+  if (B == 1) hipLaunchKernelGGL((parallel_out_kernel<0, 0>), dim3((unsigned)blocks_out), block, 0, st, dout, n_out, down, t_down);
+  else if (wide(down)) out_go<2>(B, dout, n_out, down, t_down, blocks_out, st);
+  else out_go<1>(B, dout, n_out, down, t_down, blocks_out, st);
   VY_CHECK_LAUNCH(who);
   return VY_OK;
 }
