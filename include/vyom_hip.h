@@ -167,7 +167,8 @@ int vy_clamped_act_fwd(const void* gate_up, int64_t ldg, void* out, int64_t ldo,
  *     already holds start[slot] tokens; count[b] <= L of its tokens are real (NULL: all L), the rest is padding behind them.
  *
  * vy_residual_norm: x (fp32) += norm(y) * w_post ; h = norm(x) * w_pre.  ids given: x = table[ids] instead (an id outside
- *   [0, V) gives zeros and sets *err_flag); w_post NULL: plain add; y and ids NULL: x is only read; h NULL: no second norm.
+ *   [0, V) gives zeros and sets *err_flag); w_post NULL: plain add; y and ids NULL: x is only read; h NULL: no second norm;
+ *   h without w_pre: h = x, rounded to h's type.
  *   rms = 0: (v - mean) / sqrt(var + eps), rms = 1: v / sqrt(mean(v^2) + eps).
  * vy_residual_norm_routed: the same with y += sum_k weight[row][k] * rows[pos[row][k]] ahead of the post norm (routed
  *   nullable; weight fp32 and pos int32 are [M][top], pos NULL: row * top + k, pos < 0: left out; y NULL: the sum alone) and
@@ -193,12 +194,16 @@ int vy_latent_norm(const void* p, int64_t ldp, const float* w_q, void* q_out, in
                    int64_t L, float eps, int dtype, void* stream);
 int vy_rmsnorm_gate(const void* x, int64_t ldx, const float* w, const void* gate, int64_t ldg, void* y, int64_t ldy, int64_t M,
                     int64_t N, int64_t NP, float eps, int dtype, void* stream);
+/* vy_head_norm_gate: every head of a row by itself, without a weight: y = x / rms(x) * silu(gate); heads of NP columns, N used. */
+int vy_head_norm_gate(const void* x, int64_t ldx, const void* gate, int64_t ldg, void* y, int64_t ldy, int64_t M, int32_t heads,
+                      int64_t N, int64_t NP, float eps, int dtype, void* stream);
 
 /* vy_attn_fwd_ex: causal attention whose values may have a width of their own (dv), with a start position per sequence
  * (key j is visible to query i of sequence b iff j <= start[slot] + i; start NULL: 0) and an optional output gate:
  * out *= sigmoid(gate), gate laid out as out (strides g_sb, g_sl).
  * win (nullable) adds, with s_b = min(start[slot], start_cap) in the place of start[slot]:
- *   window     query i sees only the keys j > s_b + i - window (0: every earlier key);
+ *   window     query i sees only the keys j > s_b + i - window (0: every earlier key) ...
+ *   keep       ... and, whatever the window, the keys j < keep up to its own;
  *   sink       one more term exp(0) in every softmax denominator, without a value;
  *   rope       rotary positions of the queries: (cos, sin) pairs [rope_len][rope_dims / 2], fp32; columns 2c and 2c + 1 of the
  *              first rope_dims turn by the angle of position start[slot] + i (the keys are rotated already);
@@ -206,6 +211,7 @@ int vy_rmsnorm_gate(const void* x, int64_t ldx, const float* w, const void* gate
 typedef struct vy_attn_window {
   int32_t window, sink, kv_by_slot, start_cap;
   const float* rope; int32_t rope_dims, rope_len;
+  int32_t keep;
 } vy_attn_window;
 int vy_attn_fwd_ex(const void* q, int64_t q_sb, int64_t q_sh, int64_t q_sl, const void* k, int64_t k_sb, int64_t k_sh,
                    int64_t k_sl, const void* v, int64_t v_sb, int64_t v_sh, int64_t v_sl, void* out, int64_t o_sb,
@@ -213,45 +219,65 @@ int vy_attn_fwd_ex(const void* q, int64_t q_sb, int64_t q_sh, int64_t q_sl, cons
                    int64_t B, int h, int hk, int64_t L, int64_t S, int dh, int dv, float scale, const vy_attn_window* win,
                    int dtype, void* stream);
 
-/* vy_moe_fwd: mixture of experts on rows h [M][width].  z = w_router h (fp32), scores softmax(z); experts form `groups` equal
- * groups of neighbours, and only those of the `keep` groups with the best largest score can be chosen; the `top` best of them
- * are, with weight = scale * score / (sum of the chosen scores + 1e-20).  Expert e: vy_clamped_act_fwd's activation between
- * w_gu[e] (rows interleaved: 2j gate j, 2j + 1 up j) and w_down[e].  Nothing is added up here:
+/* vy_moe_fwd: mixture of experts on rows h [M][width].  z = w_router h (fp32), scores softmax(z) or sigmoid(z); experts form
+ * `groups` equal groups of neighbours, and only those of the `keep` best groups can be chosen (a group's score: the sum of its
+ * group_best largest scores, 1 or 2); the `top` best of them are, with weight = scale * score, divided by (sum of the chosen
+ * scores + 1e-20) if normalize.  Expert e, by `act`: VY_MOE_CLAMPED vy_clamped_act_fwd's activation between w_gu[e] (rows
+ * interleaved: 2j gate j, 2j + 1 up j) and w_down[e]; VY_MOE_GELU the exact GELU between w_gu[e] (the up rows alone) and
+ * w_down[e].  Nothing is added up here:
  *   rows   the experts' outputs, row stride ldr, M * top of them in an order of its own,
  *   pos    [M][top] a choice's row, weight [M][top] its weight (vy_residual_norm_routed takes the three), ids [M][top] its expert
  *          (-1, 0 and -1 for padding tokens: those with l >= count[b], m = b L + l; count nullable).
  * width and ff are padded to multiples of 8.  experts <= 1024, top <= 64. */
+enum { VY_MOE_CLAMPED = 0, VY_MOE_GELU = 1 };
+enum { VY_SCORE_SOFTMAX = 0, VY_SCORE_SIGMOID = 1 };
 typedef struct vy_moe {
   int32_t experts, top, groups, keep, width, ff;
+  int32_t act, score, group_best, normalize;
   float scale, limit, alpha;
-  const void *w_router, *w_gu, *w_down;   /* [experts][width], [experts][2 ff][width], [experts][width][ff] */
+  const void *w_router, *w_gu, *w_down;   /* [experts][width], [experts][2 ff or ff][width], [experts][width][ff] */
 } vy_moe;
 int64_t vy_moe_ws_bytes(const vy_moe* d, int64_t M, int dtype);
 int vy_moe_fwd(const vy_moe* d, const void* h, int64_t ldh, int64_t M, const int32_t* count, int64_t L, void* rows, int64_t ldr,
                int32_t* ids, int32_t* pos, float* weight, void* ws, int64_t ws_bytes, int dtype, void* stream);
 
 /* Sliding-window attention over a ring of keys and values.  Per slot and key/value head the ring holds R rows [key (dim) |
- * value (vdim)] (strides r_ss per slot, r_sh per head), position p in row p % R; R is the window, or less while no sequence is
- * longer than R.  Packed projection rows p (stride ldp): queries at column oq ([h][dim]), keys ok ([hk][dim]), values ov
+ * value (vdim)] (strides r_ss per slot, r_sh per head).  The first `keep` tokens of a sequence stay visible for good: position p
+ * lives in row p while p < R, later ones in row keep + (p - keep) % (R - keep); R is keep + the window, or less while no sequence
+ * is longer than R.  Packed projection rows p (stride ldp): queries at column oq ([h][dim]), keys ok ([hk][dim]), values ov
  * ([hk][vdim]), output gate og ([h][vdim], og < 0: none).  rope / rope_dims / rope_len as in vy_attn_window.
  *
- * vy_window_rows: rotate != 0: rotary positions on the new keys, in place; store != 0: the last R of the count[b] new rows of
- *   every sequence to the ring.
- * vy_window_context: ctx [B][hk][S][dim + vdim] = the last min(start, past) rows of the ring in order of position, then the L
- *   new rows (rotated already), then zeros: what vy_attn_fwd_ex takes with start_cap = past.
+ * vy_window_rows: rotate != 0: rotary positions on the new keys, in place; store != 0: those of the count[b] new rows of every
+ *   sequence that its ring still holds behind them, to the ring.
+ * vy_window_context: ctx [B][hk][S][dim + vdim] = min(start, past) rows of the ring in order of position (the kept ones, then the
+ *   last of the others), then the L new rows (rotated already), then zeros: what vy_attn_fwd_ex takes with start_cap = past.
+ * vy_qkv_rows: what a vy_qkv_prep asks for, in place on the packed rows: RMS norms of the whole query and of the whole key
+ *   projection, rotary positions on both, values mixed; store != 0: as vy_window_rows.
  * vy_window_decode: one new token per sequence (L = 1): its key and value to the ring, then attention of its queries over the
- *   ring with sink and gate; max_keys >= every start + 1; ws: vy_window_decode_ws_bytes(...).  scale > 0. */
-int vy_window_rows(void* p, int64_t ldp, int64_t ok, int64_t ov, void* ring, int64_t r_ss, int64_t r_sh, int32_t R,
+ *   ring with sink and gate, prep (nullable) as in vy_qkv_rows; max_keys >= every start + 1; ws: vy_window_decode_ws_bytes(...).
+ *   scale > 0. */
+typedef struct vy_qkv_prep {
+  const float *q_norm, *k_norm;     /* [h][dim], [hk][dim] factors (NULL: no norms), zero in padded columns */
+  int32_t n_q, n_k;                 /* columns the norms divide by */
+  float eps, lambda;
+  const void* v_mix; int64_t ldm;   /* nullable: v <- (1 - lambda) v + lambda v_mix, rows of [hk][vdim] */
+  void* v_out; int64_t ldo;         /* nullable: receives the values as they were before mixing */
+} vy_qkv_prep;
+int vy_qkv_rows(void* p, int64_t ldp, int64_t oq, int64_t ok, int64_t ov, const vy_qkv_prep* prep, void* ring, int64_t r_ss,
+                int64_t r_sh, int32_t R, int32_t keep, const float* rope, int32_t rope_dims, int32_t rope_len, int store,
+                const int32_t* slots, const int32_t* start, const int32_t* count, int64_t B, int64_t L, int32_t h, int32_t hk,
+                int32_t dim, int32_t vdim, int dtype, void* stream);
+int vy_window_rows(void* p, int64_t ldp, int64_t ok, int64_t ov, void* ring, int64_t r_ss, int64_t r_sh, int32_t R, int32_t keep,
                    const float* rope, int32_t rope_dims, int32_t rope_len, int rotate, int store, const int32_t* slots,
                    const int32_t* start, const int32_t* count, int64_t B, int64_t L, int32_t hk, int32_t dim, int32_t vdim,
                    int dtype, void* stream);
 int vy_window_context(const void* p, int64_t ldp, int64_t ok, int64_t ov, const void* ring, int64_t r_ss, int64_t r_sh,
-                      int32_t R, void* ctx, int32_t S, int32_t past, const int32_t* slots, const int32_t* start, int64_t B,
+                      int32_t R, int32_t keep, void* ctx, int32_t S, int32_t past, const int32_t* slots, const int32_t* start, int64_t B,
                       int64_t L, int32_t hk, int32_t dim, int32_t vdim, int dtype, void* stream);
 int64_t vy_window_decode_ws_bytes(int32_t B, int32_t h, int32_t hk, int32_t vdim, int32_t R);
 int vy_window_decode(void* p, int64_t ldp, int64_t oq, int64_t ok, int64_t ov, int64_t og, void* ring, int64_t r_ss, int64_t r_sh,
-                     int32_t R, const float* rope, int32_t rope_dims, int32_t rope_len, const int32_t* slots,
-                     const int32_t* start, int64_t max_keys, void* out, int64_t ldo, int64_t B, int32_t h, int32_t hk,
+                     int32_t R, int32_t keep, const float* rope, int32_t rope_dims, int32_t rope_len, const vy_qkv_prep* prep,
+                     const int32_t* slots, const int32_t* start, int64_t max_keys, void* out, int64_t ldo, int64_t B, int32_t h, int32_t hk,
                      int32_t dim, int32_t vdim, float scale, int32_t sink, void* ws, int64_t ws_bytes, int dtype, void* stream);
 
 /* vy_latent_decode: one query token per sequence against a cache of latents c (one row of R per token, shared by all
@@ -268,7 +294,8 @@ int vy_latent_decode(const void* q, int64_t ldq, const void* wukt, const void* w
 
 /* vy_decay_attn: linear attention with a per-head decay on packed rows p (row stride ldp; q / k / v of head a at columns
  * oq + a*dk, ok + a*dk, ov + a*dv):  S_t = decay_a S_(t-1) + k_t v_t^T,  o_t = S_t^T q_t  with q, k, v = silu of the
- * projections (silu = 0: taken as they are).  state: fp32 [slot][h][dk][dv], taken as zero where start[slot] == 0 and left as
+ * projections (silu = 0: taken as they are).  rope (nullable; as in vy_attn_window): rotary positions on q and k, in fp32 and
+ * not rounded before the recurrence; k is multiplied by k_scale behind it.  state: fp32 [slot][h][dk][dv], taken as zero where start[slot] == 0 and left as
  * S after the sequence's last real token.  decay_pow: fp32 [h][VY_DECAY_CHUNK + 1], decay_a^0 .. decay_a^CHUNK.
  * out rows [h*dv].  ws: vy_decay_attn_ws_bytes(...) of scratch (chunked prefill: bf16, L > 1, dk <= 128; otherwise the
  * token-by-token recurrence runs and ws may be NULL).  dk, dv multiples of 8, dk <= 512. */
@@ -276,8 +303,8 @@ int vy_latent_decode(const void* q, int64_t ldq, const void* wukt, const void* w
 int64_t vy_decay_attn_ws_bytes(int64_t B, int64_t L, int32_t h, int32_t dk, int32_t dv, int dtype);
 int vy_decay_attn(const void* p, int64_t ldp, int64_t oq, int64_t ok, int64_t ov, float* state, const float* decay_pow,
                   const int32_t* slots, const int32_t* start, const int32_t* count, void* out, int64_t ldo, int64_t B,
-                  int64_t L, int32_t h, int32_t dk, int32_t dv, int silu, void* ws, int64_t ws_bytes, int dtype,
-                  void* stream);
+                  int64_t L, int32_t h, int32_t dk, int32_t dv, int silu, const float* rope, int32_t rope_dims, int32_t rope_len,
+                  float k_scale, void* ws, int64_t ws_bytes, int dtype, void* stream);
 
 /* vy_rope_fwd: in-place rotary embedding on a (B,heads,L,dh) tensor (strides as above);
  * used when the fused epilogue does not apply.  `inverse` != 0 applies the transpose rotation
@@ -562,27 +589,33 @@ int vy_gemma_decoder_step(const vy_gemma_plan* plan, const void* x, int64_t pos,
  * stream.  Forms of a layer:
  *   VY_FORM_SANDWICH  h = norm(x) * norm1; y = w_o mixer(h); x += norm(y) * norm1b;
  *                     h = norm(x) * norm2; x += norm(ff(h)) * norm2b                       (ff = 0 and no moe: no second half)
+ *                     norm1 / norm2 NULL: the sublayers read x itself
  *   VY_FORM_PARALLEL  h = norm(x) * norm1; x += w_o [mixer(h) | act(h)] + routed(h): one packed product w_in of h also gives the
  *                     [gate; up] rows of a dense feed-forward of width ff (its last 2 ff rows), one product w_o takes both back
  * norm1b / norm2b NULL: no norm on a sublayer's output.  moe (nullable): routed experts, added to the feed-forward's output.
  * clamped: the feed-forward's activation is vy_clamped_act_fwd's (limit, alpha), else the plan's act.
  * Mixers, all from ONE packed input projection w_in of h:
  *   VY_MIX_LATENT  rows [query latent | key/value latent | output gate]: vy_latent_norm, q = w_uq latent, vy_latent_decode
- *   VY_MIX_DECAY   rows [q | k | v | output gate]: vy_decay_attn, vy_rmsnorm_gate
- *   VY_MIX_WINDOW  rows [q | k | v | output gate]: vy_window_decode on the ring `cache` (strides c_ss per slot, c_sh per head)
+ *   VY_MIX_DECAY   rows [q | k | v | output gate]: vy_decay_attn (silu, rope, k_scale), then vy_rmsnorm_gate, or without
+ *                  mix_norm vy_head_norm_gate (mix_n: columns of a head)
+ *   VY_MIX_WINDOW  rows [q | k | v | output gate if gate]: vy_window_decode on the ring `cache` (strides c_ss per slot, c_sh per
+ *                  head); prep (nullable): its norms, and lambda; values: VY_VALUES_FIRST keeps this layer's values,
+ *                  VY_VALUES_MIX mixes them in (the step's own buffer is prep's v_out / v_mix)
  * Sequence b (ids[b]) lives in slot slots[b] (NULL: b) and holds lengths[slot] tokens, which the step advances by one on the
  * device; max_keys >= every lengths[slot] + 1.  Widths with _p, dim, vdim, ff and dp are padded to multiples of 8; d, q_rank,
  * kv_rank and mix_n are the true counts the norms divide by.  logits: (B, ldv).
  * -------------------------------------------------------------------------------------------- */
 enum { VY_MIX_LATENT = 0, VY_MIX_DECAY = 1, VY_MIX_WINDOW = 2 };
 enum { VY_FORM_SANDWICH = 0, VY_FORM_PARALLEL = 1 };
+enum { VY_VALUES_OWN = 0, VY_VALUES_FIRST = 1, VY_VALUES_MIX = 2 };
 typedef struct vy_hybrid_layer {
   int32_t mixer, heads, dim, vdim, n_in, ff;
   int32_t q_rank, q_rank_p, kv_rank, kv_rank_p;   /* VY_MIX_LATENT */
   int32_t cap, mix_n;                             /* cache rows per slot; VY_MIX_DECAY: width of mix_norm */
   int32_t form, clamped;
-  int32_t kv_heads, rope_dims, rope_len, sink;    /* VY_MIX_WINDOW */
-  float scale, limit, alpha;
+  int32_t kv_heads, rope_dims, rope_len, sink;    /* VY_MIX_WINDOW (rope_*: VY_MIX_DECAY too) */
+  int32_t keep, gate, values, silu;               /* VY_MIX_WINDOW, the last one VY_MIX_DECAY */
+  float scale, limit, alpha, k_scale;
   const float *norm1, *norm1b, *norm2, *norm2b;
   const void *w_in, *w_o, *w_gu, *w_down;         /* w_gu: packed [gate; up] (VY_FORM_SANDWICH) */
   const float *q_norm, *c_norm;
@@ -590,6 +623,7 @@ typedef struct vy_hybrid_layer {
   void* cache; int64_t c_ss, c_sh, c_st;
   float* state; const float *decay_pow, *mix_norm;
   const float* rope;
+  const vy_qkv_prep* prep;
   const vy_moe* moe;
 } vy_hybrid_layer;
 typedef struct vy_hybrid_plan {

@@ -194,7 +194,7 @@ def test_argument_errors_without_a_gpu():
     with pytest.raises(_lib.VyomHipError, match="workspace"):
         _lib.call("vy_latent_decode", p, 8, p, p, p, 8, 8, None, p, 1, p, 8, None, 0, 1, 1, 8, 8, 8, 1.0, p, 16, 1, None)
     with pytest.raises(_lib.VyomHipError, match="multiples of 8"):
-        _lib.call("vy_decay_attn", p, 24, 0, 8, 20, p, p, None, p, None, p, 8, 1, 1, 1, 8, 8, 1, None, 0, 1, None)
+        _lib.call("vy_decay_attn", p, 24, 0, 8, 20, p, p, None, p, None, p, 8, 1, 1, 1, 8, 8, 1, None, 0, 0, 1.0, None, 0, 1, None)
     with pytest.raises(_lib.VyomHipError, match="null"):
         _lib.call("vy_hybrid_decoder_step", None, p, None, p, 1, p, 8, None)
 

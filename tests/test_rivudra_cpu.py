@@ -196,7 +196,7 @@ def test_argument_errors_without_a_gpu():
     from vyomai_amd import _lib
     buf = (ctypes.c_char * 4096)()
     p = (ctypes.addressof(buf) + 63) // 64 * 64
-    win = [p, 64, 0, 8, 16, 24, p, 64, 64, 4, None, 0, 0, None, p, 1, p, 8, 1, 1, 1, 8, 8]
+    win = [p, 64, 0, 8, 16, 24, p, 64, 64, 4, 0, None, 0, 0, None, None, p, 1, p, 8, 1, 1, 1, 8, 8]
 
     def decode(**kw):
         a = list(win)
@@ -206,14 +206,16 @@ def test_argument_errors_without_a_gpu():
     with pytest.raises(_lib.VyomHipError, match="ring strides"):
         _lib.call("vy_window_decode", *decode(_8=56, _7=56), 1.0, 1, None, 0, 1, None)
     with pytest.raises(_lib.VyomHipError, match="rotary table"):
-        _lib.call("vy_window_decode", *decode(_10=p, _11=10, _12=5), 1.0, 1, None, 0, 1, None)
+        _lib.call("vy_window_decode", *decode(_11=p, _12=10, _13=5), 1.0, 1, None, 0, 1, None)
     with pytest.raises(_lib.VyomHipError, match="5 positions, rotary table of 4"):
-        _lib.call("vy_window_decode", *decode(_10=p, _11=8, _12=4, _15=5), 1.0, 1, None, 0, 1, None)
+        _lib.call("vy_window_decode", *decode(_11=p, _12=8, _13=4, _17=5), 1.0, 1, None, 0, 1, None)
     with pytest.raises(_lib.VyomHipError, match="bad arguments"):
         _lib.call("vy_window_decode", *win, 0.0, 1, None, 0, 1, None)
+    with pytest.raises(_lib.VyomHipError, match="4 kept of 4 rows"):
+        _lib.call("vy_window_decode", *decode(_10=4), 1.0, 1, None, 0, 1, None)
     with pytest.raises(_lib.VyomHipError, match="multiples of 8"):
         _lib.call("vy_window_decode", *decode(_2=4), 1.0, 1, None, 0, 1, None)
-    moe = _lib.VyMoe(4, 3, 2, 1, 8, 8, 1.0, 1.0, 1.0, p, p, p)
+    moe = _lib.VyMoe(4, 3, 2, 1, 8, 8, 0, 0, 1, 1, 1.0, 1.0, 1.0, p, p, p)
     with pytest.raises(_lib.VyomHipError, match="3 of 4 experts, 1 of 2 groups"):
         _lib.call("vy_moe_fwd", ctypes.byref(moe), p, 8, 1, None, 1, p, 8, p, p, p, p, 4096, 1, None)
     moe.top = 2
@@ -233,10 +235,11 @@ def test_layout_of_the_plan_structures():
     from vyomai_amd import _lib, decode_plan as D
     root = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
     names = {"vy_hybrid_layer": D.VyHybridLayer, "vy_hybrid_plan": D.VyHybridPlan, "vy_moe": _lib.VyMoe,
-             "vy_attn_window": _lib.VyAttnWindow, "vy_routed_rows": _lib.VyRoutedRows}
+             "vy_attn_window": _lib.VyAttnWindow, "vy_qkv_prep": _lib.VyQkvPrep, "vy_routed_rows": _lib.VyRoutedRows}
     src = "#include <stdio.h>\n#include <stddef.h>\n#include \"vyom_hip.h\"\nint main(){\n"
     for n, cls in names.items():
-        src += f'printf("%zu", sizeof({n}));\n' + "".join(f'printf(" %zu", offsetof({n}, {f[0]}));\n' for f in cls._fields_)
+        fields = [f[0].rstrip("_") for f in cls._fields_]    # (lambda_: a keyword in Python)
+        src += f'printf("%zu", sizeof({n}));\n' + "".join(f'printf(" %zu", offsetof({n}, {f}));\n' for f in fields)
         src += 'printf("\\n");\n'
     with tempfile.TemporaryDirectory() as d:
         with open(os.path.join(d, "t.c"), "w") as f:

@@ -11,6 +11,7 @@ from .models.vision_encoder import Vit  # noqa: F401
 from .models.multimodel import VisionLanguageModel  # noqa: F401
 from .models.encoder_decoder import EncoderDecoderModel  # noqa: F401
 from .models.gisitar import GisitarConfig, GisitarModel  # noqa: F401
+from .models.padulorn import PadulornConfig, PadulornModel  # noqa: F401
 from .models.rivudra import RivudraConfig, RivudraModel  # noqa: F401
 from .models.registry import load_pretrained, register_model  # noqa: F401
 from .generation_utils import generate, generate_multimodel, generate_seq2seq  # noqa: F401

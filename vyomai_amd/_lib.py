@@ -16,6 +16,8 @@ LIB_PATH = os.environ.get("VY_LIB_PATH") or os.path.join(_HERE, "lib", "libvyom_
 VY_F32, VY_BF16 = 0, 1
 ACT_NONE, ACT_GELU_ERF, ACT_GELU_TANH, ACT_SILU = 0, 1, 2, 3
 ACT_SAVE_DERIV = 0x100   # saved tensor = act'(pre) instead of pre (include/vyom_hip.h)
+MOE_CLAMPED, MOE_GELU = 0, 1
+SCORE_SOFTMAX, SCORE_SIGMOID = 0, 1
 MASK_NONE, MASK_CAUSAL, MASK_KEYPAD, MASK_ADDITIVE = 0, 1, 2, 4
 
 _p, _i64, _i, _f, _u64 = C.c_void_p, C.c_int64, C.c_int, C.c_float, C.c_uint64
@@ -66,15 +68,19 @@ PROTOTYPES = {
     "vy_latent_norm": [_p, _i64, _p, _p, _i64, _i, _i, _p, _p, _i64, _i, _i, _p, _i64, _i64, _i, _p, _p, _p, _i64, _i64, _f,
                        _i, _p],
     "vy_rmsnorm_gate": [_p, _i64, _p, _p, _i64, _p, _i64, _i64, _i64, _i64, _f, _i, _p],
+    "vy_head_norm_gate": [_p, _i64, _p, _i64, _p, _i64, _i64, _i, _i64, _i64, _f, _i, _p],
     "vy_attn_fwd_ex": [_p, _i64, _i64, _i64, _p, _i64, _i64, _i64, _p, _i64, _i64, _i64, _p, _i64, _i64, _p, _i64, _i64,
                        _p, _p, _i64, _i, _i, _i64, _i64, _i, _i, _f, _p, _i, _p],
     "vy_latent_decode": [_p, _i64, _p, _p, _p, _i64, _i64, _p, _p, _i64, _p, _i64, _p, _i64, _i, _i, _i, _i, _i, _f, _p, _i64,
                          _i, _p],
-    "vy_decay_attn": [_p, _i64, _i64, _i64, _i64, _p, _p, _p, _p, _p, _p, _i64, _i64, _i64, _i, _i, _i, _i, _p, _i64, _i, _p],
-    "vy_window_rows": [_p, _i64, _i64, _i64, _p, _i64, _i64, _i, _p, _i, _i, _i, _i, _p, _p, _p, _i64, _i64, _i, _i, _i, _i, _p],
-    "vy_window_context": [_p, _i64, _i64, _i64, _p, _i64, _i64, _i, _p, _i, _i, _p, _p, _i64, _i64, _i, _i, _i, _i, _p],
-    "vy_window_decode": [_p, _i64, _i64, _i64, _i64, _i64, _p, _i64, _i64, _i, _p, _i, _i, _p, _p, _i64, _p, _i64, _i64, _i, _i, _i,
-                         _i, _f, _i, _p, _i64, _i, _p],
+    "vy_decay_attn": [_p, _i64, _i64, _i64, _i64, _p, _p, _p, _p, _p, _p, _i64, _i64, _i64, _i, _i, _i, _i, _p, _i, _i, _f, _p, _i64,
+                      _i, _p],
+    "vy_window_rows": [_p, _i64, _i64, _i64, _p, _i64, _i64, _i, _i, _p, _i, _i, _i, _i, _p, _p, _p, _i64, _i64, _i, _i, _i, _i, _p],
+    "vy_qkv_rows": [_p, _i64, _i64, _i64, _i64, _p, _p, _i64, _i64, _i, _i, _p, _i, _i, _i, _p, _p, _p, _i64, _i64, _i, _i, _i, _i, _i,
+                    _p],
+    "vy_window_context": [_p, _i64, _i64, _i64, _p, _i64, _i64, _i, _i, _p, _i, _i, _p, _p, _i64, _i64, _i, _i, _i, _i, _p],
+    "vy_window_decode": [_p, _i64, _i64, _i64, _i64, _i64, _p, _i64, _i64, _i, _i, _p, _i, _i, _p, _p, _p, _i64, _p, _i64, _i64, _i, _i,
+                         _i, _i, _f, _i, _p, _i64, _i, _p],
     "vy_moe_fwd": [_p, _p, _i64, _i64, _p, _i64, _p, _i64, _p, _p, _p, _p, _i64, _i, _p],
     "vy_clamped_act_fwd": [_p, _i64, _p, _i64, _i64, _i64, _f, _f, _i, _p],
     "vy_hybrid_decoder_step": [_p, _p, _p, _p, _i64, _p, _i64, _p],
@@ -102,7 +108,13 @@ class VyWgradDesc(C.Structure):
 class VyAttnWindow(C.Structure):
     """vy_attn_window of include/vyom_hip.h."""
     _fields_ = [(n, C.c_int32) for n in ("window", "sink", "kv_by_slot", "start_cap")] + \
-               [("rope", _p), ("rope_dims", C.c_int32), ("rope_len", C.c_int32)]
+               [("rope", _p), ("rope_dims", C.c_int32), ("rope_len", C.c_int32), ("keep", C.c_int32)]
+
+
+class VyQkvPrep(C.Structure):
+    """vy_qkv_prep of include/vyom_hip.h."""
+    _fields_ = [("q_norm", _p), ("k_norm", _p), ("n_q", C.c_int32), ("n_k", C.c_int32), ("eps", C.c_float), ("lambda_", C.c_float),
+                ("v_mix", _p), ("ldm", _i64), ("v_out", _p), ("ldo", _i64)]
 
 
 class VyRoutedRows(C.Structure):
@@ -112,7 +124,8 @@ class VyRoutedRows(C.Structure):
 
 class VyMoe(C.Structure):
     """vy_moe of include/vyom_hip.h."""
-    _fields_ = [(n, C.c_int32) for n in ("experts", "top", "groups", "keep", "width", "ff")] + \
+    _fields_ = [(n, C.c_int32) for n in ("experts", "top", "groups", "keep", "width", "ff", "act", "score", "group_best",
+                                         "normalize")] + \
                [(n, C.c_float) for n in ("scale", "limit", "alpha")] + [(n, _p) for n in ("w_router", "w_gu", "w_down")]
 
 

@@ -48,6 +48,7 @@ struct AttnParams {
   // EXT = 2 only: sliding window (0 = none), a sink of score 0 without a value, keys / values indexed by slot instead of by
   // sequence, an upper bound of the start position (older keys are not in the operands), and rotary positions of the queries
   int window, sink, kv_by_slot, start_cap;
+  int keep;            // keys j < keep are seen whatever the window
   const float2* rope; int rope_half, rope_len;   // (cos, sin) [position][pair], pairs of neighbouring columns
   int diag;            // timing experiments only (VY_ATTN_DIAG): 1 = no output store, 2 = no tile loop
 };
@@ -230,6 +231,10 @@ __global__ __launch_bounds__(256, DH == 64 ? 3 : 1) void attn_fwd_mfma_kernel(At
   const int window = EXT == 2 ? p.window : 0;
   int t0 = 0;
   if (EXT == 2 && window) t0 = max(0, start + q0 - window + 1) >> 6;
+  // tiles of kept keys ahead of them: step u of the walk takes tile tile_at(u), steps u0 .. nt - 1
+  const int keep = EXT == 2 && window ? p.keep : 0;
+  const int kept = EXT == 2 ? min((keep + 63) >> 6, t0) : 0, u0 = t0 - kept;
+  auto tile_at = [&](int u) { return EXT == 2 && u < t0 ? u - u0 : u; };
 
   // key-padding mask -> one 64-bit visibility word per key tile, built once (an ordinary load inside
   // the tile loop would make the compiler drain the LDS-DMA ring with vmcnt(0) every tile)
@@ -248,7 +253,7 @@ __global__ __launch_bounds__(256, DH == 64 ? 3 : 1) void attn_fwd_mfma_kernel(At
     const int k0 = tile * 64;
     // wave-uniform skip of tiles wholly above this wave's diagonal
     if (causal && k0 > start + wave_last) return;
-    if (EXT == 2 && window && k0 + 63 < start + wave_first - window + 1) return;
+    if (EXT == 2 && window && k0 + 63 < start + wave_first - window + 1 && k0 >= keep) return;
     const char* kb_ = smem + buf * TILE;
     const char* vb_ = smem + (NS + buf) * TILE;
     f32x16 st[2];
@@ -307,7 +312,10 @@ __global__ __launch_bounds__(256, DH == 64 ? 3 : 1) void attn_fwd_mfma_kernel(At
       lm &= vis >> (4 * fh);
       if (EXT == 2 && window) {
         const int klow = qi + start - window + 1 - k0 - 4 * fh;
-        if (klow > 0) lm &= klow > 63 ? 0ull : ~0ull << klow;
+        unsigned long long in = klow > 63 ? 0ull : klow > 0 ? ~0ull << klow : ~0ull;
+        const int kk = keep - k0 - 4 * fh;
+        in |= kk > 63 ? ~0ull : kk > 0 ? (1ull << kk) - 1ull : 0ull;
+        lm &= in;
       }
       const unsigned lmw[2] = {(unsigned)lm, (unsigned)(lm >> 32)};
 #pragma unroll
@@ -388,7 +396,7 @@ __global__ __launch_bounds__(256, DH == 64 ? 3 : 1) void attn_fwd_mfma_kernel(At
   // MFMA inside the loop as vmcnt(0) and drains the ring every tile.
 #pragma unroll
   for (int s_ = 0; s_ < NS - 1; ++s_)
-    if (t0 + s_ < nt) stage(t0 + s_, s_);
+    if (u0 + s_ < nt) stage(tile_at(u0 + s_), s_);
   // Q after the first K/V tiles are requested: one memory latency for both, not two in a row
 #pragma unroll
   for (int ks = 0; ks < KS; ++ks) qf[ks] = *reinterpret_cast<const bf16x8*>(Q + ks * 16 + fh * 8);
@@ -400,12 +408,12 @@ __global__ __launch_bounds__(256, DH == 64 ? 3 : 1) void attn_fwd_mfma_kernel(At
 #pragma unroll
     for (int ks = 0; ks < KS; ++ks) asm volatile("" ::"v"(qf[ks]));
   }
-  for (int t = t0; t < (p.diag == 2 ? 0 : nt); ++t) {
+  for (int t = u0; t < (p.diag == 2 ? 0 : nt); ++t) {
     wait_tile(min(NS - 2, nt - 1 - t));
     __builtin_amdgcn_s_barrier();
     asm volatile("" ::: "memory");
-    if (t + NS - 1 < nt) stage(t + NS - 1, (t - t0 + NS - 1) % NS);  // the buffer tile t-1 was read from
-    compute(t, (t - t0) % NS);
+    if (t + NS - 1 < nt) stage(tile_at(t + NS - 1), (t - u0 + NS - 1) % NS);  // the buffer tile t-1 was read from
+    compute(tile_at(t), (t - u0) % NS);
   }
 
   float l_tot = l_run + __shfl_xor(l_run, 32, 64);
@@ -566,6 +574,8 @@ __global__ __launch_bounds__(256) void attn_fwd_gen_kernel(AttnParams p, int dh)
   const int window = EXT == 2 ? p.window : 0;
   int t0 = 0;
   if (EXT == 2 && window) t0 = max(0, start + q0 - window + 1) >> 6;
+  const int keep = EXT == 2 && window ? p.keep : 0;
+  const int u0 = EXT == 2 ? t0 - min((keep + 63) >> 6, t0) : t0;   // tiles of kept keys ahead of the window's
   int nt = (p.S + 63) / 64;
   if (causal) {
     const int kv_end = min(p.S, start + q0 + 64);
@@ -574,8 +584,8 @@ __global__ __launch_bounds__(256) void attn_fwd_gen_kernel(AttnParams p, int dh)
   // transposing-read addresses of the V tile: lane j of a 16-lane group supplies row (j >> 2), columns 4 (j & 3) ..
   const unsigned vtr = vy_lds_addr(vt) + (4 * kq + (r16 >> 2)) * VPITCH + (4 * (r16 & 3)) * 2;
 
-  for (int t = t0; t < nt; ++t) {
-    const int k0 = t * 64;
+  for (int t = u0; t < nt; ++t) {
+    const int k0 = (EXT == 2 && t < t0 ? t - u0 : t) * 64;
     // stage the tile: 16-byte chunks, zero beyond the head width and beyond the last key
     bf16x8 kreg[KCPT], vreg[VCPT];
     if constexpr (!EXT && DHP == DVP) {
@@ -639,7 +649,7 @@ __global__ __launch_bounds__(256) void attn_fwd_gen_kernel(AttnParams p, int dh)
         const int kj = k0 + 16 * blk + 4 * kq + r;
         bool vis = kj < p.S;
         if (causal) vis = vis && kj <= qi + start;
-        if (EXT == 2 && window) vis = vis && kj > qi + start - window;
+        if (EXT == 2 && window) vis = vis && (kj > qi + start - window || kj < keep);
         if (haskp) vis = vis && kp[kj < p.S ? kj : 0] != 0;
         const float tv = vis ? sc[blk][r] : -INFINITY;
         sc[blk][r] = tv;
@@ -815,7 +825,9 @@ __global__ __launch_bounds__(64 * NWV) void attn_rowwise_kernel(AttnParams p, in
   // every key is walked so a fully masked row reproduces the reference's uniform average.
   int S_eff = p.pos_dev ? *p.pos_dev + 1 : p.S;
   if (causal && !haskp && !hasadd) S_eff = min(S_eff, qi + start + 1);
+  // (window: key index u of the walk is key u - gap below S_lo, the kept keys, and key u from there on)
   const int S_lo = EXT == 2 && p.window ? max(0, qi + start - p.window + 1) : 0;
+  const int gap = EXT == 2 && p.window ? S_lo - min(p.keep, S_lo) : 0;
 
   float m = -FLT_MAX, l = 0.f, acc[VEC];
   if constexpr (EXT == 2)
@@ -832,6 +844,7 @@ __global__ __launch_bounds__(64 * NWV) void attn_rowwise_kernel(AttnParams p, in
   auto key_of = [&](int j0, int u, bool& valid) {
     const int j = j0 + u * NWV * KPP + grp;
     valid = j < S_eff;
+    if (EXT == 2 && j < S_lo) return j - gap;
     return valid ? j : S_eff - 1;
   };
   auto request = [&](int j0, raw16 (&kr)[U], raw16 (&vr)[U]) {
@@ -859,7 +872,7 @@ __global__ __launch_bounds__(64 * NWV) void attn_rowwise_kernel(AttnParams p, in
     }
   };
   raw16 kcur[U], vcur[U];
-  int j0 = S_lo + wave * KPP;
+  int j0 = gap + wave * KPP;
   if (j0 < S_eff) request(j0, kcur, vcur);
   for (; j0 < S_eff; j0 += STRIDE) {
     raw16 knext[U], vnext[U];
@@ -1089,11 +1102,12 @@ extern "C" int vy_attn_fwd_ex(const void* q, int64_t q_sb, int64_t q_sh, int64_t
   if (dv <= 0 || dh % vec || dv % vec) VY_FAIL(VY_ERR_ARG, "%s: head widths %d / %d must be multiples of %d", who, dh, dv, vec);
   if (gate && (g_sb % vec || g_sl % vec || (uintptr_t)gate % 16)) VY_FAIL(VY_ERR_ARG, "%s: gate rows must be 16-byte aligned", who);
   if (!win) return launch_ex<1>(p, dh, dtype, (hipStream_t)stream, who);
+  if (win->keep < 0) VY_FAIL(VY_ERR_ARG, "%s: %d kept keys", who, win->keep);
   if (win->window < 0 || win->start_cap < 0) VY_FAIL(VY_ERR_ARG, "%s: window %d, start_cap %d", who, win->window, win->start_cap);
   if (!(scale > 0.f)) VY_FAIL(VY_ERR_ARG, "%s: scale %g", who, (double)scale);
   if (win->rope && (win->rope_dims < 0 || win->rope_dims % 2 || win->rope_dims > dh || win->rope_len < 1))
     VY_FAIL(VY_ERR_ARG, "%s: rotary table of %d columns, %d positions for heads of %d", who, win->rope_dims, win->rope_len, dh);
-  p.window = win->window; p.sink = win->sink; p.kv_by_slot = win->kv_by_slot; p.start_cap = win->start_cap;
+  p.window = win->window; p.sink = win->sink; p.kv_by_slot = win->kv_by_slot; p.start_cap = win->start_cap; p.keep = win->keep;
   p.rope = (const float2*)win->rope; p.rope_half = win->rope_dims / 2; p.rope_len = win->rope_len;
   if (p.rope_half == 0) p.rope = nullptr;
   return launch_ex<2>(p, dh, dtype, (hipStream_t)stream, who);

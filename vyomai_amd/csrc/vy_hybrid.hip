@@ -21,7 +21,7 @@ namespace {
 
 int64_t up(int64_t x) { return (x + 255) / 256 * 256; }
 
-struct Sizes { int64_t in, q, cq, ao, o, gu, ff, mix_ws, top, moe_ws; };   // widest of each over the layers
+struct Sizes { int64_t in, q, cq, ao, o, gu, ff, mix_ws, top, moe_ws, values; };   // widest of each over the layers
 
 Sizes sizes_of(const vy_hybrid_plan* p) {
   Sizes s{};
@@ -37,6 +37,7 @@ Sizes sizes_of(const vy_hybrid_plan* p) {
       mx(s.mix_ws, vy_latent_decode_ws_bytes(p->B, L.heads, L.kv_rank_p));
     } else if (L.mixer == VY_MIX_WINDOW) {
       mx(s.mix_ws, vy_window_decode_ws_bytes(p->B, L.heads, L.kv_heads, L.vdim, L.cap));
+      if (L.values != VY_VALUES_OWN) mx(s.values, (int64_t)L.kv_heads * L.vdim);
     } else {
       mx(s.o, (int64_t)L.heads * L.vdim);
     }
@@ -87,7 +88,7 @@ extern "C" int64_t vy_hybrid_ws_bytes(const vy_hybrid_plan* p) {
   const int64_t e = p->dtype == VY_BF16 ? 2 : 4, B = p->B;
   return up(B * p->dp * 4) + 2 * up(B * p->dp * e) + up(B * s.in * e) + up(B * s.q * e) + up(B * s.cq * e) +
          up(B * s.ao * e) + up(B * s.o * e) + up(B * s.gu * e) + up(B * s.ff * e) + up(s.mix_ws) + up(B * s.top * p->dp * e) +
-         3 * up(B * s.top * 4) + up(s.moe_ws);
+         3 * up(B * s.top * 4) + up(s.moe_ws) + up(B * s.values * e);
 }
 
 extern "C" int vy_hybrid_decoder_step(const vy_hybrid_plan* p, const int64_t* ids, const int32_t* slots, int32_t* lengths,
@@ -116,6 +117,8 @@ extern "C" int vy_hybrid_decoder_step(const vy_hybrid_plan* p, const int64_t* id
   int32_t* epos = (int32_t*)take(B * s.top * 4);
   float* ew = (float*)take(B * s.top * 4);
   void* ews = take(s.moe_ws);
+  void* values = take(B * s.values * e);
+  int64_t values_ld = 0;   // set by the layer that fills them
   int rc;
   auto norm = [&](const void* yy, const vy_routed_rows* routed, const float* post, const float* pre, bool last) {
     return vy_residual_norm_ex(x, dp, yy, dp, p->embed, dp, yy || routed ? nullptr : ids, p->vocab, p->err, p->embed_scale, routed,
@@ -150,14 +153,26 @@ extern "C" int vy_hybrid_decoder_step(const vy_hybrid_plan* p, const int64_t* id
         return rc;
     } else if (L.mixer == VY_MIX_WINDOW) {
       const int64_t gk = (int64_t)L.kv_heads * L.dim, gv = (int64_t)L.kv_heads * L.vdim;
-      if ((rc = vy_window_decode(in, L.n_in, 0, nk, nk + gk, nk + gk + gv, L.cache, L.c_ss, L.c_sh, L.cap, L.rope, L.rope_dims,
-                                 L.rope_len, slots, lengths, max_keys, ao, na, B, L.heads, L.kv_heads, L.dim, L.vdim, L.scale,
+      vy_qkv_prep prep{};
+      if (L.prep) prep = *L.prep;
+      if (L.values == VY_VALUES_FIRST) {
+        prep.v_out = values;
+        prep.ldo = values_ld = gv;
+      } else if (L.values == VY_VALUES_MIX) {
+        if (values_ld != gv) VY_FAIL(VY_ERR_ARG, "%s: layer %d mixes values of %ld columns with %ld", who, l, (long)gv, (long)values_ld);
+        prep.v_mix = values;
+        prep.ldm = gv;
+      }
+      if ((rc = vy_window_decode(in, L.n_in, 0, nk, nk + gk, L.gate ? nk + gk + gv : -1, L.cache, L.c_ss, L.c_sh, L.cap, L.keep, L.rope,
+                                 L.rope_dims, L.rope_len, L.prep || L.values != VY_VALUES_OWN ? &prep : nullptr, slots, lengths, max_keys, ao, na, B, L.heads, L.kv_heads, L.dim, L.vdim, L.scale,
                                  L.sink, mws, s.mix_ws, p->dtype, stream))) return rc;
     } else {
       if ((rc = vy_decay_attn(in, L.n_in, 0, nk, 2 * nk, L.state, L.decay_pow, slots, lengths, nullptr, o, nv, B, 1, L.heads, L.dim,
-                              L.vdim, 1, nullptr, 0, p->dtype, stream))) return rc;
+                              L.vdim, L.silu, L.rope, L.rope_dims, L.rope_len, L.k_scale, nullptr, 0, p->dtype, stream))) return rc;
       const char* gate = (const char*)in + (2 * nk + nv) * e;
-      if ((rc = vy_rmsnorm_gate(o, nv, L.mix_norm, gate, L.n_in, ao, na, B, L.mix_n, nv, p->eps, p->dtype, stream))) return rc;
+      if (!L.mix_norm) {
+        if ((rc = vy_head_norm_gate(o, nv, gate, L.n_in, ao, na, B, L.heads, L.mix_n, L.vdim, p->eps, p->dtype, stream))) return rc;
+      } else if ((rc = vy_rmsnorm_gate(o, nv, L.mix_norm, gate, L.n_in, ao, na, B, L.mix_n, nv, p->eps, p->dtype, stream))) return rc;
     }
     const vy_routed_rows rows{erows, dp, epos, ew, L.moe ? L.moe->top : 0};
     const vy_routed_rows* routed = L.moe ? &rows : nullptr;

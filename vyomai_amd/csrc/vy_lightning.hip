@@ -1,5 +1,6 @@
-// Linear attention with a per-head decay (lightning attention):
-//   S_t = decay S_(t-1) + k_t v_t^T ,  o_t = S_t^T q_t ,  q, k, v = silu of the projections.
+// Linear attention with a per-head decay:
+//   S_t = decay S_(t-1) + k_t v_t^T ,  o_t = S_t^T q_t
+// with q, k, v = silu of the projections (lightning attention), or q and k rotated by their position and k scaled (retention).
 //
 // Two forms of the same sums:
 //   * decay_recurrent_kernel: token by token, the state in registers (fp32).  Decode steps, fp32 models, and head widths
@@ -11,7 +12,8 @@
 //
 // 32-bit throughout where it enters the recurrence: decays are fp32 tables made in double precision on the host, the state
 // is fp32, and every MFMA operand that carries a decay or a state (decayed keys, decayed scores, S_c) is fed as TWO bf16
-// numbers hi + lo (~16 bits of mantissa); only q, k, v themselves -- projections -- are plain bf16.
+// numbers hi + lo (~16 bits of mantissa); only q, k, v themselves -- projections -- are plain bf16.  Rotated q and k (ROT) are no
+// projections any more: they are made in fp32 on the way in and go on as hi + lo as well.
 #include "vy_common.h"
 
 namespace {
@@ -25,7 +27,40 @@ struct DecayArgs {
   void* out; int64_t ldo;
   int B, L, h, dk, dv, silu, nc;
   float* U;                                // [B * h][nc][dk][dv]
+  const float2* rope; int half, rope_len;  // half = 0: no rotation; pairs of neighbouring columns
+  float k_scale;
 };
+
+// (cos, sin) of the first pair of a token's row of the table (clamped: padding rows only)
+__device__ __forceinline__ const float2* trig_row(const DecayArgs& a, int pos) {
+  return a.rope + (int64_t)(pos < a.rope_len ? pos : a.rope_len - 1) * a.half;
+}
+// N consecutive columns d0 .. (both even) of a row
+template <int N>
+__device__ __forceinline__ void rotate(const float2* trig, int half, int d0, float (&v)[N]) {
+  if (d0 + N <= 2 * half && (half & 1) == 0 && N % 4 == 0) {   // whole 16-byte pieces of the table's row
+#pragma unroll
+    for (int e = 0; e < N; e += 4) {
+      const f32x4 cs = *reinterpret_cast<const f32x4*>(trig + ((d0 + e) >> 1));
+      const float u = v[e], w = v[e + 1], x = v[e + 2], y = v[e + 3];
+      v[e] = u * cs[0] - w * cs[1];
+      v[e + 1] = w * cs[0] + u * cs[1];
+      v[e + 2] = x * cs[2] - y * cs[3];
+      v[e + 3] = y * cs[2] + x * cs[3];
+    }
+    return;
+  }
+#pragma unroll
+  for (int e = 0; e < N; e += 2) {
+    const int i = (d0 + e) >> 1;
+    if (i < half) {
+      const float2 cs = trig[i];
+      const float u = v[e], w = v[e + 1];
+      v[e] = u * cs.x - w * cs.y;
+      v[e + 1] = w * cs.x + u * cs.y;
+    }
+  }
+}
 
 __device__ __forceinline__ float activate(float x, int silu) { return silu ? vy_silu(x) : x; }
 __device__ __forceinline__ void split_bf16(float x, bf16& hi, bf16& lo) {
@@ -51,7 +86,8 @@ __global__ __launch_bounds__(256) void decay_recurrent_kernel(DecayArgs a) {
   const float decay = a.pow[(int64_t)head * (C + 1) + 1];
   float* S = a.state + ((int64_t)slot * a.h + head) * a.dk * a.dv;
   float s[RPT];
-  const bool fresh = a.start[slot] == 0;
+  const int first = a.start[slot];
+  const bool fresh = first == 0;
 #pragma unroll
   for (int i = 0; i < RPT; ++i) {
     const int r = rg + RG * i;
@@ -65,8 +101,17 @@ __global__ __launch_bounds__(256) void decay_recurrent_kernel(DecayArgs a) {
       const int t = i / DK, d = i % DK;
       const T* row = P + (int64_t)(t0 + t) * a.ldp + head * a.dk + d;
       const bool ok = d < a.dk;
-      qs[t][d] = ok ? activate(VyT<T>::ld(row + a.oq), a.silu) : 0.f;
-      ks[t][d] = ok ? activate(VyT<T>::ld(row + a.ok), a.silu) : 0.f;
+      float q = ok ? activate(VyT<T>::ld(row + a.oq), a.silu) : 0.f;
+      float k = ok ? activate(VyT<T>::ld(row + a.ok), a.silu) : 0.f;
+      if (d < 2 * a.half) {
+        const int to = d & 1 ? -1 : 1;   // the other column of the pair
+        const float2 cs = trig_row(a, first + t0 + t)[d >> 1];
+        const float s = d & 1 ? cs.y : -cs.y;
+        q = q * cs.x + activate(VyT<T>::ld(row + a.oq + to), a.silu) * s;
+        k = k * cs.x + activate(VyT<T>::ld(row + a.ok + to), a.silu) * s;
+      }
+      qs[t][d] = q;
+      ks[t][d] = k * a.k_scale;
     }
     for (int i = threadIdx.x; i < m * COLS; i += 256) {
       const int t = i / COLS, d = c0 + i % COLS;
@@ -125,8 +170,21 @@ __device__ __forceinline__ bf16x8 tr_frag(unsigned lane_addr, int pitch) {
   return u.v;
 }
 
+// eight key columns d .. of a chunk's token t: rotated and scaled (ROT), else as loaded
+template <bool ROT>
+__device__ __forceinline__ void key8(const DecayArgs& a, const bf16* p, bool ok, int pos, int d, float (&v)[8]) {
+  const bf16x8 k8 = load8(p, ok, a.silu);
+#pragma unroll
+  for (int e = 0; e < 8; ++e) v[e] = (float)k8[e];
+  if constexpr (ROT) {
+    if (a.half) rotate(trig_row(a, pos), a.half, d, v);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) v[e] *= a.k_scale;
+  }
+}
+
 // grid (chunks, value blocks of 64, B * h)
-template <int DKP>
+template <int DKP, bool ROT>
 __global__ __launch_bounds__(256) void chunk_kv_kernel(DecayArgs a) {
   constexpr int KP = (DKP + 8) * 2, VP = (64 + 8) * 2;
   __shared__ __attribute__((aligned(16))) char smem[C * (2 * KP + VP)];
@@ -140,16 +198,18 @@ __global__ __launch_bounds__(256) void chunk_kv_kernel(DecayArgs a) {
   const int v0 = (int)blockIdx.y * 64;
   const int n = a.count ? min(a.count[b], a.L) : a.L;
   const int m = max(0, min(C, n - ch * C));            // tokens of this chunk
+  const int first = ROT ? a.start[a.slots ? a.slots[b] : b] + ch * C : 0;
   const float* pw = a.pow + (int64_t)head * (C + 1);
   const bf16* P = (const bf16*)a.p + ((int64_t)b * a.L + ch * C) * a.ldp;
   for (int i = threadIdx.x; i < C * (DKP / 8); i += 256) {
     const int t = i / (DKP / 8), d = (i % (DKP / 8)) * 8;
     const bool ok = t < m && d < a.dk;
-    const bf16x8 k8 = load8(P + (int64_t)t * a.ldp + a.ok + head * a.dk + d, ok, a.silu);
+    float k8[8];
+    key8<ROT>(a, P + (int64_t)t * a.ldp + a.ok + head * a.dk + d, ok, first + t, d, k8);
     const float w = t < m ? pw[m - 1 - t] : 0.f;
     bf16x8 hi, lo;
 #pragma unroll
-    for (int e = 0; e < 8; ++e) { bf16 x, y; split_bf16((float)k8[e] * w, x, y); hi[e] = x; lo[e] = y; }
+    for (int e = 0; e < 8; ++e) { bf16 x, y; split_bf16(k8[e] * w, x, y); hi[e] = x; lo[e] = y; }
     *reinterpret_cast<bf16x8*>(kh + t * KP + d * 2) = hi;
     *reinterpret_cast<bf16x8*>(kl + t * KP + d * 2) = lo;
   }
@@ -237,14 +297,14 @@ __global__ __launch_bounds__(256) void chunk_scan_kernel(DecayArgs a) {
 }
 
 // grid (chunks, value blocks of 64, B * h): wave w computes rows 16 w .. + 15 of the chunk (C = 64)
-template <int DKP>
+template <int DKP, bool ROT>
 __global__ __launch_bounds__(256) void chunk_out_kernel(DecayArgs a) {
   static_assert(C == 64, "one 16-row block per wave");
   constexpr int KP = (DKP + 8) * 2, VP = (64 + 8) * 2;
-  constexpr int KS = DKP / 32;
-  __shared__ __attribute__((aligned(16))) char smem[C * (KP + VP) + 2 * DKP * VP + (C + 1) * 4];
+  constexpr int KS = DKP / 32, KB = ROT ? 2 : 1;        // key images: hi, lo
+  __shared__ __attribute__((aligned(16))) char smem[C * (KB * KP + VP) + 2 * DKP * VP + (C + 1) * 4];
   char* kt = smem;
-  char* vt = smem + C * KP;
+  char* vt = smem + KB * C * KP;
   char* sh = vt + C * VP;
   char* sl = sh + DKP * VP;
   float* pw = reinterpret_cast<float*>(sl + DKP * VP);
@@ -256,10 +316,22 @@ __global__ __launch_bounds__(256) void chunk_out_kernel(DecayArgs a) {
   const int rows = min(C, a.L - ch * C);
   const bf16* P = (const bf16*)a.p + ((int64_t)b * a.L + ch * C) * a.ldp;
   const float* Sg = a.U + ((int64_t)bh * a.nc + ch) * a.dk * a.dv;
+  const int first = ROT ? a.start[a.slots ? a.slots[b] : b] + ch * C : 0;
   for (int i = threadIdx.x; i < C * (DKP / 8); i += 256) {
     const int t = i / (DKP / 8), d = (i % (DKP / 8)) * 8;
-    *reinterpret_cast<bf16x8*>(kt + t * KP + d * 2) =
-        load8(P + (int64_t)t * a.ldp + a.ok + head * a.dk + d, t < rows && d < a.dk, a.silu);
+    const bf16* src = P + (int64_t)t * a.ldp + a.ok + head * a.dk + d;
+    const bool ok = t < rows && d < a.dk;
+    if constexpr (ROT) {
+      float k8[8];
+      key8<true>(a, src, ok, first + t, d, k8);
+      bf16x8 hi, lo;
+#pragma unroll
+      for (int e = 0; e < 8; ++e) { bf16 x, y; split_bf16(k8[e], x, y); hi[e] = x; lo[e] = y; }
+      *reinterpret_cast<bf16x8*>(kt + t * KP + d * 2) = hi;
+      *reinterpret_cast<bf16x8*>(kt + C * KP + t * KP + d * 2) = lo;
+    } else {
+      *reinterpret_cast<bf16x8*>(kt + t * KP + d * 2) = load8(src, ok, a.silu);
+    }
   }
   for (int i = threadIdx.x; i < C * 8; i += 256) {
     const int t = i >> 3, d = (i & 7) * 8;
@@ -277,7 +349,7 @@ __global__ __launch_bounds__(256) void chunk_out_kernel(DecayArgs a) {
   for (int i = threadIdx.x; i <= C; i += 256) pw[i] = a.pow[(int64_t)head * (C + 1) + i];
   // the wave's query rows, in the k order of the transposed state fragments (4 kq .. and 16 + 4 kq ..)
   const int qi = 16 * wave + r16;
-  bf16x8 qf[KS];
+  bf16x8 qf[KS], ql[ROT ? KS : 1];
   {
     const bf16* Q = P + (int64_t)min(qi, rows - 1) * a.ldp + a.oq + head * a.dk;
 #pragma unroll
@@ -287,8 +359,17 @@ __global__ __launch_bounds__(256) void chunk_out_kernel(DecayArgs a) {
         const int d = 32 * ks + 16 * hf + 4 * kq;
         bf16x4 q4 = {};
         if (d < a.dk) q4 = *reinterpret_cast<const bf16x4*>(Q + d);
+        if constexpr (ROT) {
+          float v[4];
 #pragma unroll
-        for (int e = 0; e < 4; ++e) qf[ks][4 * hf + e] = (bf16)activate((float)q4[e], a.silu);
+          for (int e = 0; e < 4; ++e) v[e] = activate((float)q4[e], a.silu);
+          if (a.half) rotate(trig_row(a, first + qi), a.half, d, v);
+#pragma unroll
+          for (int e = 0; e < 4; ++e) { bf16 x, y; split_bf16(v[e], x, y); qf[ks][4 * hf + e] = x; ql[ks][4 * hf + e] = y; }
+        } else {
+#pragma unroll
+          for (int e = 0; e < 4; ++e) qf[ks][4 * hf + e] = (bf16)activate((float)q4[e], a.silu);
+        }
       }
     }
   }
@@ -313,6 +394,7 @@ __global__ __launch_bounds__(256) void chunk_out_kernel(DecayArgs a) {
       vy_tie(fh[i]);
       vy_tie(fl[i]);
       o[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(fl[i], qf[ks], o[i], 0, 0, 0);
+      if constexpr (ROT) o[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(fh[i], ql[ks], o[i], 0, 0, 0);
       o[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(fh[i], qf[ks], o[i], 0, 0, 0);
     }
   }
@@ -335,6 +417,13 @@ __global__ __launch_bounds__(256) void chunk_out_kernel(DecayArgs a) {
         const char* kr = kt + (32 * tt + 16 * blk + r16) * KP + (32 * ks + 4 * kq) * 2;
         kf.h.a = *reinterpret_cast<const bf16x4*>(kr);
         kf.h.b = *reinterpret_cast<const bf16x4*>(kr + 32);
+        if constexpr (ROT) {
+          union { struct { bf16x4 a, b; } h; bf16x8 v; } kl;
+          kl.h.a = *reinterpret_cast<const bf16x4*>(kr + C * KP);
+          kl.h.b = *reinterpret_cast<const bf16x4*>(kr + C * KP + 32);
+          sc[blk] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kl.v, qf[ks], sc[blk], 0, 0, 0);
+          sc[blk] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf.v, ql[ks], sc[blk], 0, 0, 0);
+        }
         sc[blk] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf.v, qf[ks], sc[blk], 0, 0, 0);
       }
     }
@@ -413,29 +502,33 @@ extern "C" int64_t vy_decay_attn_ws_bytes(int64_t B, int64_t L, int32_t h, int32
 extern "C" int vy_decay_attn(const void* p, int64_t ldp, int64_t oq, int64_t ok, int64_t ov, float* state,
                              const float* decay_pow, const int32_t* slots, const int32_t* start, const int32_t* count,
                              void* out, int64_t ldo, int64_t B, int64_t L, int32_t h, int32_t dk, int32_t dv, int silu,
-                             void* ws, int64_t ws_bytes, int dtype, void* stream) {
+                             const float* rope, int32_t rope_dims, int32_t rope_len, float k_scale, void* ws, int64_t ws_bytes,
+                             int dtype, void* stream) {
   const char* who = "vy_decay_attn";
   if (!p || !state || !decay_pow || !start || !out) VY_FAIL(VY_ERR_ARG, "%s: null pointer", who);
   if (B <= 0 || L <= 0 || h <= 0 || dk <= 0 || dv <= 0 || L > INT32_MAX) VY_FAIL(VY_ERR_ARG, "%s: empty problem", who);
   if (dk % 8 || dv % 8 || ldp % 8 || ldo % 8 || oq % 8 || ok % 8 || ov % 8) VY_FAIL(VY_ERR_ARG, "%s: widths, strides and offsets must be multiples of 8", who);
   if (dtype != VY_BF16 && dtype != VY_F32) VY_FAIL(VY_ERR_ARG, "%s: bad dtype %d", who, dtype);
   if (B * h > 65535) VY_FAIL(VY_ERR_UNSUPPORTED, "%s: %ld (sequence, head) pairs", who, (long)(B * h));
+  if (rope_dims < 0 || rope_dims % 2 || rope_dims > dk || (rope_dims && (!rope || rope_len < 1)))
+    VY_FAIL(VY_ERR_ARG, "%s: rotary table of %d columns, %d positions for heads of %d", who, rope_dims, rope_len, dk);
   hipStream_t st = (hipStream_t)stream;
   DecayArgs a{p, ldp, oq, ok, ov, state, decay_pow, slots, start, count, out, ldo, (int)B, (int)L, h, dk, dv, silu,
-              (int)vy_cdiv(L, C), (float*)ws};
+              (int)vy_cdiv(L, C), (float*)ws, (const float2*)rope, rope_dims / 2, rope_len > 0 ? rope_len : 1, k_scale};
   if (chunked(L, dk, dtype)) {
     if (!ws || ws_bytes < vy_decay_attn_ws_bytes(B, L, h, dk, dv, dtype)) VY_FAIL(VY_ERR_ARG, "%s: workspace too small", who);
     const dim3 grid(a.nc, (unsigned)vy_cdiv(dv, 64), (unsigned)(B * h)), block(256);
     const dim3 sgrid((unsigned)vy_cdiv((int64_t)dk * dv, 1024), (unsigned)(B * h));
-#define CH_GO(D)                                                                \
+#define CH_GO(D, ROT)                                                           \
   do {                                                                          \
-    hipLaunchKernelGGL(chunk_kv_kernel<D>, grid, block, 0, st, a);              \
+    hipLaunchKernelGGL((chunk_kv_kernel<D, ROT>), grid, block, 0, st, a);       \
     hipLaunchKernelGGL(chunk_scan_kernel, sgrid, block, 0, st, a);              \
-    hipLaunchKernelGGL(chunk_out_kernel<D>, grid, block, 0, st, a);             \
+    hipLaunchKernelGGL((chunk_out_kernel<D, ROT>), grid, block, 0, st, a);      \
   } while (0)
-    if (dk <= 32) CH_GO(32);
-    else if (dk <= 64) CH_GO(64);
-    else CH_GO(128);
+    const bool rot = a.half || k_scale != 1.f;
+    if (dk <= 32) { if (rot) CH_GO(32, true); else CH_GO(32, false); }
+    else if (dk <= 64) { if (rot) CH_GO(64, true); else CH_GO(64, false); }
+    else { if (rot) CH_GO(128, true); else CH_GO(128, false); }
 #undef CH_GO
   } else if (dtype == VY_BF16 ? recurrent_go<bf16>(a, st) : recurrent_go<float>(a, st)) {
     VY_FAIL(VY_ERR_UNSUPPORTED, "%s: key width %d > 512", who, dk);

@@ -11,6 +11,7 @@ constexpr int MAX_E = 1024, MAX_ENTRIES = 1024;
 struct ChooseArgs {
   const float* logits; int64_t M;
   int E, top, groups, keep;
+  int sigmoid, best, normalize;       // scores sigmoid or softmax; largest scores summed for a group's (1 or 2)
   float scale;
   const int* count; int L;            // tokens l >= count[b] of a sequence are padding: no expert
   int* ids; float* weight;            // [M][top]; id -1: none
@@ -23,8 +24,8 @@ __device__ __forceinline__ unsigned ordered(float z) {
   return u & 0x80000000u ? ~u : u | 0x80000000u;
 }
 
-// one wave per token; lane holds experts lane + 64 i.  Softmax is monotone: the choice is made on the logits.  gmax: 2 * 64 EPL
-// floats of LDS of the wave's own
+// one wave per token; lane holds experts lane + 64 i.  Both scores are monotone: the choice is made on the logits (of groups only
+// if a group's score is its best expert's).  gmax: 2 * 64 EPL floats of LDS of the wave's own
 template <int EPL>
 __device__ __forceinline__ void choose_one(const ChooseArgs& a, int64_t m, int lane, float* gmax, int (&my_id), float (&my_w)) {
   my_id = -1;
@@ -38,26 +39,34 @@ __device__ __forceinline__ void choose_one(const ChooseArgs& a, int64_t m, int l
     z[i] = e < a.E ? a.logits[m * a.E + e] : -INFINITY;
     zmax = fmaxf(zmax, z[i]);
   }
-  zmax = vy_wave_max(zmax);
-  float sum = 0.f;
+  float sum = 1.f;
+  if (!a.sigmoid) {
+    zmax = vy_wave_max(zmax);
+    sum = 0.f;
 #pragma unroll
-  for (int i = 0; i < EPL; ++i) sum += expf(z[i] - zmax);   // (exp(-inf) = 0 behind the last expert)
-  sum = vy_wave_sum(sum);
+    for (int i = 0; i < EPL; ++i) sum += expf(z[i] - zmax);   // (exp(-inf) = 0 behind the last expert)
+    sum = vy_wave_sum(sum);
+  }
+  auto score = [&](float x) { return a.sigmoid ? 1.f / (1.f + expf(-x)) : expf(x - zmax) / sum; };
   unsigned key[EPL];
 #pragma unroll
   for (int i = 0; i < EPL; ++i) key[i] = lane + 64 * i < a.E ? ordered(z[i]) : 0u;
   if (a.keep < a.groups) {
-    // a group's score is its best expert's; a group stays if fewer than `keep` others are better (ties: the earlier one)
+    // a group stays if fewer than `keep` others are better (ties: the earlier one)
     const int size = a.E / a.groups;
     float* zs = gmax + 64 * EPL;
 #pragma unroll
     for (int i = 0; i < EPL; ++i)
-      if (lane + 64 * i < a.E) zs[lane + 64 * i] = z[i];
+      if (lane + 64 * i < a.E) zs[lane + 64 * i] = a.best == 1 ? z[i] : score(z[i]);
     __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
     for (int g = lane; g < a.groups; g += 64) {
-      float best = -INFINITY;
-      for (int j = 0; j < size; ++j) best = fmaxf(best, zs[g * size + j]);
-      gmax[g] = best;
+      float best = -INFINITY, second = -INFINITY;
+      for (int j = 0; j < size; ++j) {
+        const float s = zs[g * size + j];
+        second = fmaxf(second, fminf(best, s));
+        best = fmaxf(best, s);
+      }
+      gmax[g] = a.best == 1 || size == 1 ? best : best + second;
     }
     __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
 #pragma unroll
@@ -93,12 +102,17 @@ __device__ __forceinline__ void choose_one(const ChooseArgs& a, int64_t m, int l
     for (int i = 0; i < EPL; ++i)
       if (lane + 64 * i == be) { ze = z[i]; key[i] = 0u; }
     ze = __shfl(ze, be & 63, 64);
-    const float s = expf(ze - zmax) / sum;
+    const float s = score(ze);
     total += s;
     if (lane == k) { my_id = be; my_w = s; }
   }
-  my_w = my_w / (total + 1e-20f) * a.scale;
+  my_w = (a.normalize ? my_w / (total + 1e-20f) : my_w) * a.scale;
 }
+
+// what an expert product does with its rows
+constexpr int DOWN = 0;      // rows by choice in and out
+constexpr int GATE_UP = 1;   // rows by token in, pairs of neighbouring results -> clamped gated activation
+constexpr int UP = 2;        // rows by token in, exact GELU
 
 __device__ __forceinline__ float clamped_act(float g, float u, float limit, float alpha) {
   g = fminf(g, limit);
@@ -108,7 +122,7 @@ __device__ __forceinline__ float clamped_act(float g, float u, float limit, floa
 
 // ---- the experts, few tokens ------------------------------------------------------------------
 struct ExpertRows {
-  const bf16* x; int64_t ldx;          // GU: rows of h by token; else activation rows by choice
+  const bf16* x; int64_t ldx;          // DOWN: activation rows by choice; else rows of h by token
   const int* ids; int n, top;          // n = tokens * top choices
   const bf16* w; int N, K;             // [E][N][K]
   bf16* y; int64_t ldy;                // rows by choice
@@ -122,7 +136,7 @@ template <int NT> struct ExpertLds {
 };
 
 // The y-th expert in use (in order of its number; of a single token: its y-th choice) x 16 NT weight rows.
-template <bool GU, int NT>
+template <int KIND, int NT>
 __device__ __forceinline__ void expert_rows(const ExpertRows& a, ExpertLds<NT>& lds, int x, int y) {
   const int tid = threadIdx.x, lane = tid & 63, r16 = lane & 15, kq = lane >> 4;
   int e, cnt;
@@ -169,7 +183,7 @@ __device__ __forceinline__ void expert_rows(const ExpertRows& a, ExpertLds<NT>& 
   for (int t = 0; t < NT; ++t) ws[t] = a.w + ((int64_t)e * a.N + min(n0 + 16 * t + r16, a.N - 1)) * a.K + 8 * kq;
   for (int m0 = 0; m0 < cnt; m0 += 16) {
     const int mine = a.n == a.top ? y : lds.list[m0 + r16 < cnt ? m0 + r16 : cnt - 1];
-    const bf16* xs[1] = {a.x + (int64_t)(GU ? mine / a.top : mine) * a.ldx + 8 * kq};
+    const bf16* xs[1] = {a.x + (int64_t)(KIND != DOWN ? mine / a.top : mine) * a.ldx + 8 * kq};
     f32x4 acc[NT][1];
     vy_rows::stream<NT, 1>(ws, xs, a.K, acc, lds.red);
     if (tid < 64 && m0 + r16 < cnt) {
@@ -179,7 +193,7 @@ __device__ __forceinline__ void expert_rows(const ExpertRows& a, ExpertLds<NT>& 
         const int n = n0 + 16 * t + 4 * kq;
         if (n < a.N) {
           bf16* yr = a.y + (int64_t)mine * a.ldy;
-          if constexpr (GU) {
+          if constexpr (KIND == GATE_UP) {
             bf16x2 w2;
             w2[0] = (bf16)clamped_act(v[0], v[1], a.limit, a.alpha);
             w2[1] = (bf16)clamped_act(v[2], v[3], a.limit, a.alpha);
@@ -187,7 +201,7 @@ __device__ __forceinline__ void expert_rows(const ExpertRows& a, ExpertLds<NT>& 
           } else {
             bf16x4 w4;
 #pragma unroll
-            for (int r = 0; r < 4; ++r) w4[r] = (bf16)v[r];
+            for (int r = 0; r < 4; ++r) w4[r] = (bf16)(KIND == UP ? vy_gelu_erf_fast(v[r]) : v[r]);
             *reinterpret_cast<bf16x4*>(yr + n) = w4;
           }
         }
@@ -196,18 +210,21 @@ __device__ __forceinline__ void expert_rows(const ExpertRows& a, ExpertLds<NT>& 
   }
 }
 
-// a single token: its y-th choice x 8 weight rows (GU: 4 pairs)
-template <bool GU>
+// a single token: its y-th choice x 8 weight rows (GATE_UP: 4 pairs)
+template <int KIND>
 __device__ __forceinline__ void expert_rows1(const ExpertRows& a, int x, int y) {
   const int e = a.ids[y], n = 8 * x + 2 * (threadIdx.x >> 6);
   if (e < 0 || n >= a.N) return;   // (N is a multiple of 8)
   const bf16* w = a.w + ((int64_t)e * a.N + n) * a.K;
   float s0, s1;
-  vy_rows::gemv2(w, w + a.K, a.x + (GU ? 0 : (int64_t)y * a.ldx), a.K, s0, s1);
+  vy_rows::gemv2(w, w + a.K, a.x + (KIND != DOWN ? 0 : (int64_t)y * a.ldx), a.K, s0, s1);
   if (threadIdx.x & 63) return;
   bf16* yr = a.y + (int64_t)y * a.ldy;
-  if constexpr (GU) {
+  if constexpr (KIND == GATE_UP) {
     yr[n / 2] = (bf16)clamped_act(s0, s1, a.limit, a.alpha);
+  } else if constexpr (KIND == UP) {
+    yr[n] = (bf16)vy_gelu_erf_fast(s0);
+    yr[n + 1] = (bf16)vy_gelu_erf_fast(s1);
   } else {
     yr[n] = (bf16)s0;
     yr[n + 1] = (bf16)s1;

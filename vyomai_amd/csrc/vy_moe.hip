@@ -1,11 +1,11 @@
-// Mixture of experts: every token goes through `top` of E small gated feed-forward layers.
+// Mixture of experts: every token goes through `top` of E small feed-forward layers.
 //
 //   vy_moe_fwd   router logits (fp32), choice of experts, the experts, their outputs left as rows for
 //                vy_residual_norm_routed (which adds them up, weighted, in fp32)
 //   vy_clamped_act_fwd   the experts' activation on packed [gate | up] rows (a shared expert's)
 //
-// Expert e: g = min(Wg h, limit), u = clamp(Wu h, -limit, limit), y = Wd (g sigmoid(alpha g) (u + 1)).  Wg and Wu are packed
-// with their rows interleaved (row 2j: gate j, row 2j + 1: up j): in the accumulators' layout (a lane owns 4 consecutive
+// Expert e, gated and clamped: g = min(Wg h, limit), u = clamp(Wu h, -limit, limit), y = Wd (g sigmoid(alpha g) (u + 1)); or
+// plain: y = Wd gelu(Wu h).  Wg and Wu are packed with their rows interleaved (row 2j: gate j, row 2j + 1: up j): in the accumulators' layout (a lane owns 4 consecutive
 // output columns of one token) both halves of a pair sit in one lane and the activation is the product's epilogue.
 //
 // Few tokens (decode): expert_rows_kernel streams the weights of the experts in use straight into MFMA operands (vy_rows.h), one
@@ -196,10 +196,10 @@ constexpr int BK = 64, ROWB = BK * 2;
 
 // 128 x 128 x 64 tiles, two LDS stages, four waves of 64 x 64 on mfma_f32_16x16x32_bf16 (the structure of
 // gemm_nt_bf16_m16_kernel).  GU: rows gathered, activation in the epilogue, half as many output columns.
-template <bool GU>
+template <int KIND>
 __global__ __launch_bounds__(256) void grouped_gemm_kernel(GroupedArgs a) {
   constexpr int BM = 128, BN = 128, NW = 4, TM = 4, TN = 4, GX = BM / 8 / NW, GW = BN / 8 / NW;
-  constexpr int STAGE = (BM + BN) * ROWB, ON = GU ? BN / 2 : BN, OROW = ON * 2 + 16;
+  constexpr int STAGE = (BM + BN) * ROWB, ON = KIND == GATE_UP ? BN / 2 : BN, OROW = ON * 2 + 16;
   static_assert(BM * OROW <= 2 * STAGE, "the output tile fits");
   __shared__ __attribute__((aligned(16))) char smem[2 * STAGE];
   int e, mt, nt;
@@ -216,7 +216,7 @@ __global__ __launch_bounds__(256) void grouped_gemm_kernel(GroupedArgs a) {
   for (int t = 0; t < GX; ++t) {
     const int R = (wave + NW * t) * 8 + lrow, g = slot ^ ((R >> 1) & 7);
     const int r = row0 + (R < rows ? R : rows - 1);
-    xsrc[t] = (const bf16*)a.x + (int64_t)(GU ? a.token[r] : r) * a.ldx + g * 8;
+    xsrc[t] = (const bf16*)a.x + (int64_t)(KIND != DOWN ? a.token[r] : r) * a.ldx + g * 8;
     xk[t] = g * 8;
   }
 #pragma unroll
@@ -307,7 +307,7 @@ __global__ __launch_bounds__(256) void grouped_gemm_kernel(GroupedArgs a) {
       char* at = smem + (wm * 16 * TM + 16 * j + r16) * OROW;
       const int n = wn * 16 * TN + 16 * i + 4 * kq;
       const f32x4 v = acc[i][j];
-      if constexpr (GU) {
+      if constexpr (KIND == GATE_UP) {
         bf16x2 w2;
         w2[0] = (bf16)clamped_act(v[0], v[1], a.limit, a.alpha);
         w2[1] = (bf16)clamped_act(v[2], v[3], a.limit, a.alpha);
@@ -315,13 +315,13 @@ __global__ __launch_bounds__(256) void grouped_gemm_kernel(GroupedArgs a) {
       } else {
         bf16x4 w4;
 #pragma unroll
-        for (int r = 0; r < 4; ++r) w4[r] = (bf16)v[r];
+        for (int r = 0; r < 4; ++r) w4[r] = (bf16)(KIND == UP ? vy_gelu_erf_fast(v[r]) : v[r]);
         *reinterpret_cast<bf16x4*>(at + 2 * n) = w4;
       }
     }
   __syncthreads();
   constexpr int CPR = ON / 8;
-  const int NO = GU ? N / 2 : N, c0 = GU ? n0 / 2 : n0;
+  const int NO = KIND == GATE_UP ? N / 2 : N, c0 = KIND == GATE_UP ? n0 / 2 : n0;
   for (int i = tid; i < BM * CPR; i += 256) {
     const int r = i / CPR, ch = (i % CPR) * 8;
     if (r < rows && c0 + ch < NO)
@@ -330,7 +330,7 @@ __global__ __launch_bounds__(256) void grouped_gemm_kernel(GroupedArgs a) {
 }
 
 // fp32: 64 x 64 x 16 tiles, 4 x 4 outputs per thread, fused multiply-adds in order of k
-template <bool GU>
+template <int KIND>
 __global__ __launch_bounds__(256) void grouped_gemm_f32_kernel(GroupedArgs a) {
   constexpr int T = 64, KB = 16;
   __shared__ float xs[KB][T + 4], ws[KB][T + 4];
@@ -340,7 +340,7 @@ __global__ __launch_bounds__(256) void grouped_gemm_f32_kernel(GroupedArgs a) {
   const float* W = (const float*)a.w + (int64_t)e * a.N * a.K;
   const int tid = threadIdx.x, lr = tid >> 2, lk = (tid & 3) * 4, ty = tid >> 4, tx = tid & 15;
   const int r = row0 + (lr < rows ? lr : rows - 1);
-  const float* xr = (const float*)a.x + (int64_t)(GU ? a.token[r] : r) * a.ldx;
+  const float* xr = (const float*)a.x + (int64_t)(KIND != DOWN ? a.token[r] : r) * a.ldx;
   const float* wr = W + (int64_t)min(n0 + lr, a.N - 1) * a.K;
   float acc[4][4] = {};
   for (int k0 = 0; k0 < a.K; k0 += KB) {
@@ -364,21 +364,24 @@ __global__ __launch_bounds__(256) void grouped_gemm_f32_kernel(GroupedArgs a) {
   for (int i = 0; i < 4; ++i) {
     const int m = ty * 4 + i, n = n0 + tx * 4;
     if (m >= rows || n >= a.N) continue;
-    if constexpr (GU) {
+    if constexpr (KIND == GATE_UP) {
       float* y = (float*)a.y + (int64_t)(row0 + m) * a.ldy + n / 2;
       y[0] = clamped_act(acc[i][0], acc[i][1], a.limit, a.alpha);
       y[1] = clamped_act(acc[i][2], acc[i][3], a.limit, a.alpha);
     } else {
-      *reinterpret_cast<f32x4*>((float*)a.y + (int64_t)(row0 + m) * a.ldy + n) = f32x4{acc[i][0], acc[i][1], acc[i][2], acc[i][3]};
+      f32x4 v;
+#pragma unroll
+      for (int j = 0; j < 4; ++j) v[j] = KIND == UP ? vy_gelu_erf(acc[i][j]) : acc[i][j];
+      *reinterpret_cast<f32x4*>((float*)a.y + (int64_t)(row0 + m) * a.ldy + n) = v;
     }
   }
 }
 
 // ---- the experts, few tokens ------------------------------------------------------------------
-template <bool GU, int NT>
+template <int KIND, int NT>
 __global__ __launch_bounds__(256) void expert_rows_kernel(ExpertRows a) {
   __shared__ ExpertLds<NT> lds;
-  expert_rows<GU, NT>(a, lds, blockIdx.x, blockIdx.y);
+  expert_rows<KIND, NT>(a, lds, blockIdx.x, blockIdx.y);
 }
 
 // ---- activation of packed [gate | up] rows ----------------------------------------------------
@@ -437,6 +440,9 @@ int check_moe(const char* who, const vy_moe* d, int dtype) {
   if (d->experts < 1 || d->experts > MAX_E || d->top < 1 || d->top > 64 || d->groups < 1 || d->experts % d->groups ||
       d->keep < 1 || d->keep > d->groups || d->top > d->keep * (d->experts / d->groups))
     VY_FAIL(VY_ERR_UNSUPPORTED, "%s: %d of %d experts, %d of %d groups", who, d->top, d->experts, d->keep, d->groups);
+  if ((d->act != VY_MOE_CLAMPED && d->act != VY_MOE_GELU) || (d->score != VY_SCORE_SOFTMAX && d->score != VY_SCORE_SIGMOID) ||
+      d->group_best < 1 || d->group_best > 2)
+    VY_FAIL(VY_ERR_ARG, "%s: activation %d, score %d, groups by %d scores", who, d->act, d->score, d->group_best);
   if (d->width < 8 || d->ff < 8 || d->width % 8 || d->ff % 8) VY_FAIL(VY_ERR_ARG, "%s: widths %d / %d must be multiples of 8", who, d->width, d->ff);
   return VY_OK;
 }
@@ -467,7 +473,8 @@ extern "C" int vy_moe_fwd(const vy_moe* d, const void* h, int64_t ldh, int64_t M
   hipStream_t st = (hipStream_t)stream;
   const int E = d->experts, K = d->width;
   const int64_t n = M * d->top;
-  const bool small = few(d, M, dtype);
+  const bool small = few(d, M, dtype), gated = d->act == VY_MOE_CLAMPED;
+  const int up_rows = gated ? 2 * d->ff : d->ff;
   if (!small) hipLaunchKernelGGL(zero_kernel, dim3((unsigned)vy_cdiv((int64_t)E * COUNT_STRIDE, 256)), dim3(256), 0, st, p.counts, E * COUNT_STRIDE);
   if (dtype == VY_F32) {
     hipLaunchKernelGGL(router_logits_f32_kernel, dim3((unsigned)M, (unsigned)vy_cdiv(E, 4)), dim3(256), 0, st, (const float*)h, ldh,
@@ -479,7 +486,7 @@ extern "C" int vy_moe_fwd(const vy_moe* d, const void* h, int64_t ldh, int64_t M
     hipLaunchKernelGGL((router_logits_kernel<4, 2, 8>), dim3((unsigned)vy_cdiv(E, 64), (unsigned)vy_cdiv(M, 32)), dim3(512), 0, st,
                        (const bf16*)h, ldh, (const bf16*)d->w_router, p.logits, M, K, E);
   }
-  ChooseArgs c{p.logits, M, E, d->top, d->groups, d->keep, d->scale, count, (int)L, ids, weight, small ? pos : nullptr, small ? nullptr : p.counts, p.rank};
+  ChooseArgs c{p.logits, M, E, d->top, d->groups, d->keep, d->score == VY_SCORE_SIGMOID, d->group_best, d->normalize, d->scale, count, (int)L, ids, weight, small ? pos : nullptr, small ? nullptr : p.counts, p.rank};
   // few tokens: a wave each, spread over the CUs; many: several per workgroup, so that few global adds count them
   const dim3 block(256);
 #define CHOOSE(EPL, NW, TPW) hipLaunchKernelGGL((choose_kernel<EPL, NW>), dim3((unsigned)vy_cdiv(M, NW * TPW)), dim3(64 * NW), 0, st, c, TPW)
@@ -494,31 +501,34 @@ extern "C" int vy_moe_fwd(const vy_moe* d, const void* h, int64_t ldh, int64_t M
 #undef CHOOSE
   if (small) {
     const unsigned active = (unsigned)(n < E ? n : E);
-    ExpertRows g{(const bf16*)h, ldh, ids, (int)n, d->top, (const bf16*)d->w_gu, 2 * d->ff, K, (bf16*)p.act, d->ff, d->limit, d->alpha};
+    ExpertRows g{(const bf16*)h, ldh, ids, (int)n, d->top, (const bf16*)d->w_gu, up_rows, K, (bf16*)p.act, d->ff, d->limit, d->alpha};
     ExpertRows o{(const bf16*)p.act, d->ff, ids, (int)n, d->top, (const bf16*)d->w_down, K, d->ff, (bf16*)rows, ldr, 0.f, 0.f};
-    auto go = [&](auto gu, ExpertRows& a) {
-      constexpr bool GU = decltype(gu)::value;
-      if (vy_cdiv(a.N, 16) * active > 1536) hipLaunchKernelGGL((expert_rows_kernel<GU, 2>), dim3((unsigned)vy_cdiv(a.N, 32), active), block, 0, st, a);
-      else hipLaunchKernelGGL((expert_rows_kernel<GU, 1>), dim3((unsigned)vy_cdiv(a.N, 16), active), block, 0, st, a);
+    auto go = [&](auto kind, ExpertRows& a) {
+      constexpr int KIND = decltype(kind)::value;
+      if (vy_cdiv(a.N, 16) * active > 1536) hipLaunchKernelGGL((expert_rows_kernel<KIND, 2>), dim3((unsigned)vy_cdiv(a.N, 32), active), block, 0, st, a);
+      else hipLaunchKernelGGL((expert_rows_kernel<KIND, 1>), dim3((unsigned)vy_cdiv(a.N, 16), active), block, 0, st, a);
     };
-    go(std::true_type{}, g);
-    go(std::false_type{}, o);
+    if (gated) go(std::integral_constant<int, GATE_UP>{}, g);
+    else go(std::integral_constant<int, UP>{}, g);
+    go(std::integral_constant<int, DOWN>{}, o);
     VY_CHECK_LAUNCH(who);
     return VY_OK;
   }
   const int bm = tile_rows(dtype);
   SortArgs s{ids, p.rank, p.counts, n, d->top, E, bm, pos, p.token, p.offset, p.rows, p.tiles, p.ntiles};
   hipLaunchKernelGGL(sort_kernel, dim3((unsigned)vy_cdiv(n, 256)), block, 0, st, s);
-  GroupedArgs g{h, ldh, p.token, p.offset, p.rows, p.tiles, p.ntiles, d->w_gu, 2 * d->ff, K, p.act, d->ff, d->limit, d->alpha};
+  GroupedArgs g{h, ldh, p.token, p.offset, p.rows, p.tiles, p.ntiles, d->w_gu, up_rows, K, p.act, d->ff, d->limit, d->alpha};
   GroupedArgs o{p.act, d->ff, nullptr, p.offset, p.rows, p.tiles, p.ntiles, d->w_down, K, d->ff, rows, ldr, 0.f, 0.f};
   const int64_t tiles = max_tiles(d, M, dtype);
   const dim3 ggrid((unsigned)(tiles * vy_cdiv(g.N, bm))), ogrid((unsigned)(tiles * vy_cdiv(o.N, bm)));
   if (dtype == VY_BF16) {
-    hipLaunchKernelGGL((grouped_gemm_kernel<true>), ggrid, block, 0, st, g);
-    hipLaunchKernelGGL((grouped_gemm_kernel<false>), ogrid, block, 0, st, o);
+    if (gated) hipLaunchKernelGGL((grouped_gemm_kernel<GATE_UP>), ggrid, block, 0, st, g);
+    else hipLaunchKernelGGL((grouped_gemm_kernel<UP>), ggrid, block, 0, st, g);
+    hipLaunchKernelGGL((grouped_gemm_kernel<DOWN>), ogrid, block, 0, st, o);
   } else {
-    hipLaunchKernelGGL((grouped_gemm_f32_kernel<true>), ggrid, block, 0, st, g);
-    hipLaunchKernelGGL((grouped_gemm_f32_kernel<false>), ogrid, block, 0, st, o);
+    if (gated) hipLaunchKernelGGL((grouped_gemm_f32_kernel<GATE_UP>), ggrid, block, 0, st, g);
+    else hipLaunchKernelGGL((grouped_gemm_f32_kernel<UP>), ggrid, block, 0, st, g);
+    hipLaunchKernelGGL((grouped_gemm_f32_kernel<DOWN>), ogrid, block, 0, st, o);
   }
   VY_CHECK_LAUNCH(who);
   return VY_OK;

@@ -8,6 +8,7 @@
 //   vy_latent_norm     the two RMS norms behind a packed [query latent | key/value latent | ...] projection; the
 //                      key/value latent also goes to its cache rows
 //   vy_rmsnorm_gate    RMSNorm(x) * w * sigmoid(gate)
+//   vy_head_norm_gate  x / rms(x) * silu(gate), every head by itself
 #include "vy_common.h"
 
 namespace {
@@ -161,7 +162,14 @@ __global__ __launch_bounds__(256) void residual_norm_kernel(ResNormArgs p) {
       }
     }
   }
-  if (p.h) {
+  if (p.h && !p.w_pre) {   // no norm: the stream itself
+    T* hr = (T*)p.h + row * p.ldh;
+#pragma unroll
+    for (int c = 0; c < CH; ++c) {
+      const int col = (t + TPR * c) * 4;
+      if (col < p.NP) store4<T>(hr + col, x[c]);
+    }
+  } else if (p.h) {
     float mean, rstd;
     row_stats<TPR, CH, RMS>(x, t, p.N, p.NP, p.eps_pre, red, 2, mean, rstd);
     T* hr = (T*)p.h + row * p.ldh;
@@ -308,6 +316,55 @@ __global__ __launch_bounds__(256) void rmsnorm_gate_kernel(const T* __restrict__
   }
 }
 
+// LPH lanes per head (a power of two up to a wave), one 16-byte chunk per lane and pass
+template <typename T, int LPH>
+__global__ __launch_bounds__(256) void head_norm_gate_kernel(const T* __restrict__ x, int64_t ldx, const T* __restrict__ gate,
+                                                             int64_t ldg, T* __restrict__ y, int64_t ldy, int64_t units, int heads,
+                                                             int N, int NP, float eps) {
+  constexpr int VEC = VyChunk<T>::VEC;
+  const int sub = threadIdx.x % LPH;
+  const int64_t u = (int64_t)blockIdx.x * (256 / LPH) + threadIdx.x / LPH;
+  const int64_t uc = u < units ? u : units - 1, row = uc / heads;
+  const int head = (int)(uc - row * heads);
+  const T* xr = x + row * ldx + (int64_t)head * NP;
+  const T* gr = gate + row * ldg + (int64_t)head * NP;
+  float v[VEC], g[VEC], q = 0.f;
+  for (int c = sub * VEC; c < NP; c += LPH * VEC) {
+    VyChunk<T>::load(xr + c, v);
+    VyChunk<T>::load(gr + c, g);
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) q += v[e] * v[e];   // (the padding columns are zero)
+  }
+#pragma unroll
+  for (int o = LPH / 2; o > 0; o >>= 1) q += __shfl_xor(q, o, 64);
+  const float rstd = rsqrt_refined(q / (float)N + eps);
+  if (u >= units) return;
+  for (int c = sub * VEC; c < NP; c += LPH * VEC) {
+    if (LPH * VEC < NP) {   // several passes: read again (from cache)
+      VyChunk<T>::load(xr + c, v);
+      VyChunk<T>::load(gr + c, g);
+    }
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) v[e] = v[e] * rstd * vy_silu(g[e]);
+    VyChunk<T>::store(y + row * ldy + (int64_t)head * NP + c, v);
+  }
+}
+
+template <typename T>
+void head_norm_gate_go(const void* x, int64_t ldx, const void* gate, int64_t ldg, void* y, int64_t ldy, int64_t M, int heads, int N,
+                       int NP, float eps, hipStream_t st) {
+  const int nch = NP / VyChunk<T>::VEC;
+  const int64_t units = M * heads;
+#define HN_GO(L) hipLaunchKernelGGL((head_norm_gate_kernel<T, L>), dim3((unsigned)vy_cdiv(units, 256 / L)), dim3(256), 0, st, (const T*)x, ldx, (const T*)gate, ldg, (T*)y, ldy, units, heads, N, NP, eps)
+  if (nch <= 1) HN_GO(1);
+  else if (nch <= 4) HN_GO(4);
+  else if (nch <= 8) HN_GO(8);
+  else if (nch <= 16) HN_GO(16);
+  else if (nch <= 32) HN_GO(32);
+  else HN_GO(64);
+#undef HN_GO
+}
+
 }  // namespace
 
 // internal: the step driver also advances the sequence lengths in this launch (advance[slots[i]] += 1 for i < n_adv)
@@ -319,7 +376,6 @@ int vy_residual_norm_ex(float* x, int64_t ldx, const void* y, int64_t ldy, const
   if (!x || M <= 0 || N <= 0 || NP < N) VY_FAIL(VY_ERR_ARG, "%s: bad arguments", who);
   if (NP % 4 || ldx % 4 || ldy % 4 || ldt % 4 || ldh % 4 || ldx < NP) VY_FAIL(VY_ERR_ARG, "%s: padded widths and row strides must be multiples of 4", who);
   if (ids && !table) VY_FAIL(VY_ERR_ARG, "%s: token ids without a table", who);
-  if (h && !w_pre) VY_FAIL(VY_ERR_ARG, "%s: h without w_pre", who);
   ResNormArgs a{};
   a.x = x; a.ldx = ldx; a.y = y; a.ldy = ldy; a.table = table; a.ldt = ldt; a.ids = ids; a.V = V; a.err = err;
   a.w_post = w_post; a.w_pre = w_pre; a.h = h; a.ldh = ldh; a.M = M; a.N = (int)N; a.NP = (int)NP;
@@ -374,6 +430,20 @@ extern "C" int vy_latent_norm(const void* p, int64_t ldp, const float* w_q, void
   else if (dtype == VY_F32) rc = latent_norm_go<float>(a, (hipStream_t)stream);
   else VY_FAIL(VY_ERR_ARG, "%s: bad dtype %d", who, dtype);
   if (rc) VY_FAIL(VY_ERR_UNSUPPORTED, "%s: latent width %d / %d", who, npq, npc);
+  VY_CHECK_LAUNCH(who);
+  return VY_OK;
+}
+
+extern "C" int vy_head_norm_gate(const void* x, int64_t ldx, const void* gate, int64_t ldg, void* y, int64_t ldy, int64_t M,
+                                 int32_t heads, int64_t N, int64_t NP, float eps, int dtype, void* stream) {
+  const char* who = "vy_head_norm_gate";
+  if (dtype != VY_BF16 && dtype != VY_F32) VY_FAIL(VY_ERR_ARG, "%s: bad dtype %d", who, dtype);
+  const int vec = dtype == VY_BF16 ? 8 : 4;
+  if (!x || !gate || !y || M <= 0 || heads <= 0 || N <= 0 || NP < N || NP > 1 << 20 || M * heads > INT32_MAX)
+    VY_FAIL(VY_ERR_ARG, "%s: bad arguments", who);
+  if (NP % vec || ldx % vec || ldg % vec || ldy % vec) VY_FAIL(VY_ERR_ARG, "%s: widths and strides must be multiples of %d", who, vec);
+  if (dtype == VY_BF16) head_norm_gate_go<bf16>(x, ldx, gate, ldg, y, ldy, M, heads, (int)N, (int)NP, eps, (hipStream_t)stream);
+  else head_norm_gate_go<float>(x, ldx, gate, ldg, y, ldy, M, heads, (int)N, (int)NP, eps, (hipStream_t)stream);
   VY_CHECK_LAUNCH(who);
   return VY_OK;
 }

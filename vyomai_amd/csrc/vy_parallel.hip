@@ -82,11 +82,11 @@ __global__ __launch_bounds__(256) void parallel_experts_kernel(DecodeArgs win, i
   if constexpr (NT == 0) {   // one sequence
     __shared__ __attribute__((aligned(16))) float red[FINISH_LDS / 4];
     if (id < n_finish) window_finish(win, red, id % win.h, id / win.h);
-    else expert_rows1<true>(ex, (id - n_finish) % tiles, (id - n_finish) / tiles);
+    else expert_rows1<GATE_UP>(ex, (id - n_finish) % tiles, (id - n_finish) / tiles);
   } else {
     __shared__ union { ExpertLds<NT> ex; float red[FINISH_LDS / 4]; } lds;
     if (id < n_finish) window_finish(win, lds.red, id % win.h, id / win.h);
-    else expert_rows<true, NT>(ex, lds.ex, (id - n_finish) % tiles, (id - n_finish) / tiles);
+    else expert_rows<GATE_UP, NT>(ex, lds.ex, (id - n_finish) % tiles, (id - n_finish) / tiles);
   }
 }
 
@@ -95,11 +95,11 @@ __global__ __launch_bounds__(256) void parallel_out_kernel(Dense out, int n_out,
   const int id = blockIdx.x;
   if constexpr (MB == 0) {   // one sequence
     if (id < n_out) vy_rows::dense1(out, id);
-    else expert_rows1<false>(ex, (id - n_out) % tiles, (id - n_out) / tiles);
+    else expert_rows1<DOWN>(ex, (id - n_out) % tiles, (id - n_out) / tiles);
   } else {
     __shared__ union { ExpertLds<NT> ex; f32x4 red[vy_rows::RED<1, MB>]; } lds;
     if (id < n_out) vy_rows::dense<MB>(out, lds.red, id);
-    else expert_rows<false, NT>(ex, lds.ex, (id - n_out) % tiles, (id - n_out) / tiles);
+    else expert_rows<DOWN, NT>(ex, lds.ex, (id - n_out) % tiles, (id - n_out) / tiles);
   }
 }
 
@@ -131,7 +131,7 @@ int vy_parallel_decode(const vy_hybrid_plan* p, const vy_hybrid_layer* L, const 
   const int B = p->B;
   const int64_t n = d ? (int64_t)B * d->top : 0;
   if (p->dtype != VY_BF16 || L->form != VY_FORM_PARALLEL || L->mixer != VY_MIX_WINDOW || B > 64 || L->dim > 256 || L->vdim > 256 ||
-      (L->ff && !L->clamped) || n > MAX_ENTRIES || (d && d->experts > 256))
+      (L->ff && !L->clamped) || n > MAX_ENTRIES || (d && (d->experts > 256 || d->act != VY_MOE_CLAMPED)) || !L->gate || L->prep)
     return VY_ERR_UNSUPPORTED;
   const int64_t nk = (int64_t)L->heads * L->dim, gk = (int64_t)L->kv_heads * L->dim, gv = (int64_t)L->kv_heads * L->vdim,
                 nv = (int64_t)L->heads * L->vdim, na = nv + L->ff, n_in = nk + gk + gv + nv + 2 * (int64_t)L->ff;
@@ -143,7 +143,7 @@ int vy_parallel_decode(const vy_hybrid_plan* p, const vy_hybrid_layer* L, const 
     VY_FAIL(VY_ERR_ARG, "%s: %ld positions, rotary table of %d", who, (long)max_keys, L->rope_len);
   if (d && (!d->w_router || !d->w_gu || !d->w_down || d->experts < 1 || d->top < 1 || d->top > 64 || d->groups < 1 || d->keep < 1 ||
             d->experts % d->groups || d->keep > d->groups || d->top > d->keep * (d->experts / d->groups) || d->width != p->dp ||
-            d->ff < 8 || d->ff % 8 || moe_ws_bytes < vy_moe_ws_bytes(d, B, p->dtype)))
+            d->group_best < 1 || d->group_best > 2 || d->ff < 8 || d->ff % 8 || moe_ws_bytes < vy_moe_ws_bytes(d, B, p->dtype)))
     VY_FAIL(VY_ERR_ARG, "%s: bad mixture", who);
   hipStream_t st = (hipStream_t)stream;
   const dim3 block(256);
@@ -166,7 +166,7 @@ int vy_parallel_decode(const vy_hybrid_plan* p, const vy_hybrid_layer* L, const 
   MixArgs m{};
   DecodeArgs& w = m.win;
   w.p = (const bf16*)in; w.ldp = n_in; w.oq = 0; w.ok = nk; w.ov = nk + gk; w.og = nk + gk + gv;
-  w.ring = (bf16*)L->cache; w.r_ss = L->c_ss; w.r_sh = L->c_sh; w.R = L->cap;
+  w.ring = (bf16*)L->cache; w.r_ss = L->c_ss; w.r_sh = L->c_sh; w.R = L->cap; w.keep = L->keep;
   w.rope = (const float2*)L->rope; w.half = L->rope_dims / 2; w.rope_len = L->rope_len > 0 ? L->rope_len : 1;
   w.slots = slots; w.start = lengths; w.out = (bf16*)ao; w.ldo = na;
   w.h = L->heads; w.hk = L->kv_heads; w.dim = L->dim; w.vdim = L->vdim; w.scale = L->scale; w.sink = L->sink;
@@ -179,7 +179,7 @@ int vy_parallel_decode(const vy_hybrid_plan* p, const vy_hybrid_layer* L, const 
   }
   m.n_win = w.ns * w.hk * w.passes * B;
   if (d) {
-    m.choose = ChooseArgs{logits, B, d->experts, d->top, d->groups, d->keep, d->scale, nullptr, 1, eids, ew, nullptr, nullptr, nullptr};
+    m.choose = ChooseArgs{logits, B, d->experts, d->top, d->groups, d->keep, d->score == VY_SCORE_SIGMOID, d->group_best, d->normalize, d->scale, nullptr, 1, eids, ew, nullptr, nullptr, nullptr};
     m.n_choose = (B + 3) / 4;
   }
   m.gu = (const bf16*)in + (n_in - 2 * (int64_t)L->ff); m.ldg = n_in; m.act = (bf16*)ao + nv; m.lda = na; m.B = B; m.ff = L->ff;

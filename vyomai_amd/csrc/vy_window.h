@@ -6,7 +6,10 @@
 // Swapped products as in attn_fwd_gen_kernel: S^T = K Q^T straight from global memory into MFMA operands (a key row is read
 // once, nobody else needs it: no LDS), P stays in registers as the B operand of O^T = V^T P^T, V passes through a wave-private
 // LDS tile for the transposing reads.  Rows of the next unit are requested before the arithmetic of this one.  The token's own
-// key and value never make the trip to memory and back: they replace row p % R in registers / LDS.
+// key and value never make the trip to memory and back: they replace its row of the ring in registers / LDS.
+//
+// The norms over the whole query and key projection (DecodeArgs::q_norm) are part of it: every workgroup adds up the squares of
+// the sequence's projection rows itself (a few KB from L2), in fp32, and the rotated operand is rounded once.
 #pragma once
 #include "vy_common.h"
 #include <float.h>
@@ -17,8 +20,11 @@ constexpr float LOG2E = 1.4426950408889634f;
 
 struct DecodeArgs {
   const bf16* p; int64_t ldp, oq, ok, ov, og;
-  bf16* ring; int64_t r_ss, r_sh; int R;
+  bf16* ring; int64_t r_ss, r_sh; int R, keep;
   const float2* rope; int half, rope_len;
+  const float* q_norm; const float* k_norm; int n_q, n_k; float eps;   // nullable: norms over the whole projections
+  const bf16* vm; int64_t ldm; float lambda;                           // nullable: values mixed in
+  bf16* vo; int64_t ldvo;                                              // nullable: receives the token's own values
   const int* slots; const int* start;
   bf16* out; int64_t ldo;
   int h, hk, dim, vdim, ns, passes, sink;   // ns slices of the ring, passes of 16 query heads per key/value head
@@ -43,20 +49,40 @@ __device__ __forceinline__ float group_sum(float v) {
   return __builtin_bit_cast(float, (unsigned)t[0]) + __builtin_bit_cast(float, (unsigned)t[1]);
 }
 
-__device__ __forceinline__ bf16x8 rotate8(const DecodeArgs& a, const float2* t, int d0, bf16x8 x) {
-  if (d0 >= 2 * a.half) return x;
-  bf16x8 y = x;
+// row of position p in a ring of R rows whose first `keep` stay
+__device__ __forceinline__ int ring_row(int p, int R, int keep) { return p < R ? p : keep + (p - keep) % (R - keep); }
+
+// 8 columns d0 .. of a head times r w (w nullable: as they are), rotated, rounded once
+__device__ __forceinline__ bf16x8 rotate8(const DecodeArgs& a, const float2* t, int d0, bf16x8 x, const float* w, float r) {
+  if (!w && d0 >= 2 * a.half) return x;
+  float v[8];
+#pragma unroll
+  for (int e = 0; e < 8; ++e) v[e] = (float)x[e];
+  if (w) {
+    float f[8];
+    VyChunk<float>::load(w, f);
+    VyChunk<float>::load(w + 4, f + 4);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) v[e] *= r * f[e];
+  }
 #pragma unroll
   for (int e = 0; e < 8; e += 2) {
     const int i = (d0 + e) >> 1;
     if (i < a.half) {
       const float2 cs = t[i];
-      const float u = (float)x[e], w = (float)x[e + 1];
-      y[e] = (bf16)(u * cs.x - w * cs.y);
-      y[e + 1] = (bf16)(w * cs.x + u * cs.y);
+      const float u = v[e], y = v[e + 1];
+      v[e] = u * cs.x - y * cs.y;
+      v[e + 1] = y * cs.x + u * cs.y;
     }
   }
+  bf16x8 y;
+#pragma unroll
+  for (int e = 0; e < 8; ++e) y[e] = (bf16)v[e];
   return y;
+}
+__device__ __forceinline__ float rms_factor(float sum, int n, float eps) {
+  const float ms = sum / (float)n + eps, r = rsqrtf(ms);
+  return r * (1.5f - 0.5f * ms * r * r);
 }
 
 template <int DHP, int DVP>
@@ -69,6 +95,7 @@ struct WindowDecode {
   // [value tiles, later the waves' results | queries | new key | new value | m, l of the waves]
   static constexpr int O_Q = 4 * VROWS, O_K = O_Q + 16 * QP * 2, O_V = O_K + DHP * 2, O_ML = O_V + DVP * 2;
   static_assert(4 * 16 * DVP * 4 <= 4 * VROWS, "the waves' results fit over the value tiles");
+  static_assert(2 * 64 * 4 >= 8 * 4, "the norms' partial sums fit over m, l");
   static constexpr int LDS = O_ML + 2 * 64 * 4;
 
   // slice of the ring, y = key/value head * passes + pass, b = sequence
@@ -80,7 +107,7 @@ struct WindowDecode {
   const int rep = a.h / a.hk, h0 = g * rep + pass * 16, nh = min(16, rep - pass * 16);
   const int slot = a.slots ? a.slots[b] : b;
   const int pos = a.start[slot];
-  const int n = min(pos + 1, a.R), fresh = pos % a.R;
+  const int n = min(pos + 1, a.R), fresh = ring_row(pos, a.R, a.keep);
   const int W = a.dim + a.vdim;
   const bf16* row = a.p + (int64_t)b * a.ldp;
   bf16* ring = a.ring + (int64_t)slot * a.r_ss + (int64_t)g * a.r_sh;
@@ -109,6 +136,28 @@ struct WindowDecode {
   };
   if (u < units) request(u, kf, vr);
 
+  // sums of squares of the sequence's whole query and key projections
+  float rq = 1.f, rk = 1.f;
+  if (a.q_norm) {
+    float* red = reinterpret_cast<float*>(smem + O_ML);
+    float sq = 0.f, sk = 0.f;
+    auto squares = [&](const bf16* p, int cols, float& s) {
+      for (int i = tid * 8; i < cols; i += 2048) {
+        const bf16x8 x = *reinterpret_cast<const bf16x8*>(p + i);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) s = fmaf((float)x[e], (float)x[e], s);
+      }
+    };
+    squares(row + a.oq, a.h * a.dim, sq);
+    squares(row + a.ok, a.hk * a.dim, sk);
+    sq = vy_wave_sum(sq);
+    sk = vy_wave_sum(sk);
+    if (lane == 0) { red[wave] = sq; red[4 + wave] = sk; }
+    __syncthreads();
+    rq = rms_factor(red[0] + red[1] + red[2] + red[3], a.n_q, a.eps);
+    rk = rms_factor(red[4] + red[5] + red[6] + red[7], a.n_k, a.eps);
+  }
+
   // rotated queries, new key, new value
   bf16* lq = reinterpret_cast<bf16*>(smem + O_Q);
   bf16* lk = reinterpret_cast<bf16*>(smem + O_K);
@@ -117,7 +166,8 @@ struct WindowDecode {
     const int hh = i / (DHP / 8), d0 = (i % (DHP / 8)) * 8;
     const bool ok = hh < nh && d0 < a.dim;
     bf16x8 q = zero8;
-    if (ok) q = rotate8(a, trig, d0, *reinterpret_cast<const bf16x8*>(row + a.oq + (int64_t)(h0 + hh) * a.dim + d0));
+    const int at = (h0 + hh) * a.dim + d0;
+    if (ok) q = rotate8(a, trig, d0, *reinterpret_cast<const bf16x8*>(row + a.oq + at), a.q_norm ? a.q_norm + at : nullptr, rq);
     *reinterpret_cast<bf16x8*>(lq + hh * QP + d0) = q;
   }
   const bool owner = pass == 0 && (fresh / 32) % step / 4 == slice;   // the workgroup whose units hold the new row
@@ -125,7 +175,8 @@ struct WindowDecode {
     const int d0 = (tid - 192) * 8;
     bf16x8 k8 = zero8;
     if (d0 < a.dim) {
-      k8 = rotate8(a, trig, d0, *reinterpret_cast<const bf16x8*>(row + a.ok + (int64_t)g * a.dim + d0));
+      const int at = g * a.dim + d0;
+      k8 = rotate8(a, trig, d0, *reinterpret_cast<const bf16x8*>(row + a.ok + at), a.k_norm ? a.k_norm + at : nullptr, rk);
       if (owner) *reinterpret_cast<bf16x8*>(ring + (int64_t)fresh * W + d0) = k8;
     }
     *reinterpret_cast<bf16x8*>(lk + d0) = k8;
@@ -134,6 +185,12 @@ struct WindowDecode {
     bf16x8 v8 = zero8;
     if (d0 < a.vdim) {
       v8 = *reinterpret_cast<const bf16x8*>(row + a.ov + (int64_t)g * a.vdim + d0);
+      if (owner && a.vo) *reinterpret_cast<bf16x8*>(a.vo + (int64_t)b * a.ldvo + (int64_t)g * a.vdim + d0) = v8;
+      if (a.vm) {
+        const bf16x8 m8 = *reinterpret_cast<const bf16x8*>(a.vm + (int64_t)b * a.ldm + (int64_t)g * a.vdim + d0);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) v8[e] = (bf16)((1.f - a.lambda) * (float)v8[e] + a.lambda * (float)m8[e]);
+      }
       if (owner) *reinterpret_cast<bf16x8*>(ring + (int64_t)fresh * W + a.dim + d0) = v8;
     }
     *reinterpret_cast<bf16x8*>(lv + d0) = v8;

@@ -1,10 +1,13 @@
 // Sliding-window attention over a ring of keys and values, for decoders whose queries see only the last `window` tokens.
 //
-// Memory: per sequence (slot) and key/value head a ring of R rows [key (dim) | value (vdim)], R = the window (or less while
-// sequences are shorter): position p lives in row p % R, so a sequence never holds more than its window.
+// Memory: per sequence (slot) and key/value head a ring of R rows [key (dim) | value (vdim)], R = keep + the window (or less while
+// sequences are shorter): the first `keep` positions stay in their rows, later ones go round the others, so a sequence never
+// holds more than its window and its kept tokens.
 //
-//   vy_window_rows     prefill: rotary positions on the new keys (in place in the packed projection rows) and the last R new
+//   vy_window_rows     prefill: rotary positions on the new keys (in place in the packed projection rows) and the last new
 //                      rows to the ring
+//   vy_qkv_rows        the same for designs that norm their queries and keys (over the whole projection) and mix their values:
+//                      queries, keys and values in place
 //   vy_window_context  prefill behind a past: the ring's rows and the new ones as one contiguous context for vy_attn_fwd_ex
 //   vy_window_decode   one query token per sequence: rotation of query and key, the new row to the ring, attention over the
 //                      ring, sink, output gate.  Every row of the ring that holds a token is inside the window, so decode
@@ -17,11 +20,16 @@ using namespace vy_window;
 
 struct RowsArgs {
   const void* p; int64_t ldp, ok, ov;       // packed rows; key / value columns
-  void* ring; int64_t r_ss, r_sh; int R;    // ring rows of dim + vdim elements
+  void* ring; int64_t r_ss, r_sh; int R, keep;   // ring rows of dim + vdim elements
   const float2* rope; int half, rope_len;
   const int* slots; const int* start; const int* count;
   int64_t M; int L, hk, dim, vdim, rotate, store;
 };
+
+// whether the ring still holds a token once its sequence's n new tokens are in (position first + l)
+__device__ __forceinline__ bool stays(int first, int l, int n, int R, int keep) {
+  return l < n && (first + l < keep || l + (R - keep) >= n);
+}
 
 // one 16-byte chunk of a token's keys or values per thread
 template <typename T>
@@ -36,7 +44,7 @@ __global__ __launch_bounds__(256) void window_rows_kernel(RowsArgs a) {
     const int slot = a.slots ? a.slots[b] : b;
     const int first = a.start ? a.start[slot] : 0, n = a.count ? a.count[b] : a.L;
     const int pos = first + l;
-    const bool keep = a.store && l < n && l + a.R >= n;
+    const bool keep = a.store && stays(first, l, n, a.R, a.keep);
     const bool key = c < kc;
     if (!keep && !(key && a.rotate)) continue;
     T* src = (T*)a.p + row * a.ldp + (key ? a.ok + (int64_t)g * a.dim + c * VEC : a.ov + (int64_t)g * a.vdim + (c - kc) * VEC);
@@ -56,19 +64,134 @@ __global__ __launch_bounds__(256) void window_rows_kernel(RowsArgs a) {
       }
       VyChunk<T>::store(src, v);
     }
-    if (keep) VyChunk<T>::store((T*)a.ring + (int64_t)slot * a.r_ss + (int64_t)g * a.r_sh + (int64_t)(pos % a.R) * (a.dim + a.vdim) + c * VEC, v);
+    if (keep) VyChunk<T>::store((T*)a.ring + (int64_t)slot * a.r_ss + (int64_t)g * a.r_sh + (int64_t)ring_row(pos, a.R, a.keep) * (a.dim + a.vdim) + c * VEC, v);
+  }
+}
+
+struct QkvArgs {
+  RowsArgs r;
+  int64_t oq; int h;
+  const float* q_norm; const float* k_norm; int n_q, n_k; float eps, lambda;
+  const void* vm; int64_t ldm;
+  void* vo; int64_t ldvo;
+};
+
+// WPR waves per token: sums of squares of its query and key projections, then every chunk once more (from cache) to be scaled,
+// rotated, rounded once and written back.  CH chunks per lane are held between the two (more are read again).
+template <typename T, int WPR, int CH>
+__global__ __launch_bounds__(256) void qkv_rows_kernel(QkvArgs a) {
+  constexpr int VEC = VyChunk<T>::VEC, LPR = 64 * WPR;
+  __shared__ float red[8];
+  const RowsArgs& r = a.r;
+  const int t = threadIdx.x % LPR;
+  const int64_t m0 = (int64_t)blockIdx.x * (4 / WPR) + threadIdx.x / LPR, row = m0 < r.M ? m0 : r.M - 1;
+  T* p = (T*)r.p + row * r.ldp;
+  const int b = (int)(row / r.L), l = (int)(row - (int64_t)b * r.L);
+  const int slot = r.slots ? r.slots[b] : b;
+  const int first = r.start ? r.start[slot] : 0, n = r.count ? r.count[b] : r.L, pos = first + l;
+  const int nq = a.h * r.dim / VEC, nk = r.hk * r.dim / VEC, nv = r.hk * r.vdim / VEC;
+  float held[CH][VEC];
+  float sq = 0.f, sk = 0.f;
+#pragma unroll
+  for (int c = 0; c < CH; ++c) {
+    const int i = t + LPR * c;
+    if (i < nq + nk) {
+      VyChunk<T>::load(i < nq ? p + a.oq + i * VEC : p + r.ok + (i - nq) * VEC, held[c]);
+      float s = 0.f;
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) s = fmaf(held[c][e], held[c][e], s);
+      if (i < nq) sq += s;
+      else sk += s;
+    }
+  }
+  for (int i = t + LPR * CH; i < nq + nk; i += LPR) {
+    float v[VEC], s = 0.f;
+    VyChunk<T>::load(i < nq ? p + a.oq + i * VEC : p + r.ok + (i - nq) * VEC, v);
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) s = fmaf(v[e], v[e], s);
+    if (i < nq) sq += s;
+    else sk += s;
+  }
+  sq = vy_wave_sum(sq);
+  sk = vy_wave_sum(sk);
+  if constexpr (WPR == 4) {
+    const int wave = threadIdx.x >> 6;
+    if ((threadIdx.x & 63) == 0) { red[wave] = sq; red[4 + wave] = sk; }
+    __syncthreads();
+    sq = red[0] + red[1] + red[2] + red[3];
+    sk = red[4] + red[5] + red[6] + red[7];
+  }
+  if (m0 >= r.M) return;
+  const float rq = a.q_norm ? rms_factor(sq, a.n_q, a.eps) : 1.f, rk = a.k_norm ? rms_factor(sk, a.n_k, a.eps) : 1.f;
+  const float2* trig = r.rope + (int64_t)(pos < r.rope_len ? pos : r.rope_len - 1) * r.half;   // (clamped: padding rows only)
+  const bool keep = r.store && stays(first, l, n, r.R, r.keep);
+  T* ring = keep ? (T*)r.ring + (int64_t)slot * r.r_ss + (int64_t)ring_row(pos, r.R, r.keep) * (r.dim + r.vdim) : nullptr;
+  auto finish = [&](int i, float (&v)[VEC]) {   // chunk i of [queries | keys]
+    const bool key = i >= nq;
+    const int col = (key ? i - nq : i) * VEC, g = col / r.dim, d = col - g * r.dim;
+    const float* w = key ? a.k_norm : a.q_norm;
+    if (w) {
+      const float f = key ? rk : rq;
+#pragma unroll
+      for (int e = 0; e < VEC; e += 4) {
+        float w4[4];
+        VyChunk<float>::load(w + col + e, w4);
+#pragma unroll
+        for (int c = 0; c < 4; ++c) v[e + c] *= f * w4[c];
+      }
+    }
+    if (d < 2 * r.half) {
+#pragma unroll
+      for (int e = 0; e < VEC; e += 2) {
+        const int j = (d + e) >> 1;
+        if (j < r.half) {
+          const float2 cs = trig[j];
+          const float x = v[e], y = v[e + 1];
+          v[e] = x * cs.x - y * cs.y;
+          v[e + 1] = y * cs.x + x * cs.y;
+        }
+      }
+    }
+    VyChunk<T>::store(p + (key ? r.ok : a.oq) + col, v);
+    if (key && keep) VyChunk<T>::store(ring + (int64_t)g * r.r_sh + d, v);
+  };
+#pragma unroll
+  for (int c = 0; c < CH; ++c) {
+    const int i = t + LPR * c;
+    if (i < nq + nk) finish(i, held[c]);
+  }
+  for (int i = t + LPR * CH; i < nq + nk; i += LPR) {
+    float v[VEC];
+    VyChunk<T>::load(i < nq ? p + a.oq + i * VEC : p + r.ok + (i - nq) * VEC, v);
+    finish(i, v);
+  }
+  if (!a.vm && !a.vo && !keep) return;
+  for (int i = t; i < nv; i += LPR) {
+    const int col = i * VEC, g = col / r.vdim, d = col - g * r.vdim;
+    float v[VEC];
+    VyChunk<T>::load(p + r.ov + col, v);
+    if (a.vo) VyChunk<T>::store((T*)a.vo + row * a.ldvo + col, v);
+    if (a.vm) {
+      float m[VEC];
+      VyChunk<T>::load((const T*)a.vm + row * a.ldm + col, m);
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) v[e] = (1.f - a.lambda) * v[e] + a.lambda * m[e];
+      VyChunk<T>::store(p + r.ov + col, v);
+    }
+    if (keep) VyChunk<T>::store(ring + (int64_t)g * r.r_sh + r.dim + d, v);
   }
 }
 
 struct ContextArgs {
   const void* p; int64_t ldp, ok, ov;
-  const void* ring; int64_t r_ss, r_sh; int R;
+  const void* ring; int64_t r_ss, r_sh; int R, keep;
   void* ctx; int S, past;                   // ctx [B][hk][S][dim + vdim]; past rows of the ring at most
   const int* slots; const int* start;
   int B, L, hk, dim, vdim;
 };
 
-// row s of sequence b: position (start - k) + s with k = min(start, past); the first k rows come from the ring
+// row s of sequence b, k = min(start, past): the first k rows come from the ring, positions 0 .. keep - 1, then the k - keep last;
+// the new tokens follow
 template <typename T>
 __global__ __launch_bounds__(256) void window_context_kernel(ContextArgs a) {
   constexpr int VEC = VyChunk<T>::VEC;
@@ -86,7 +209,7 @@ __global__ __launch_bounds__(256) void window_context_kernel(ContextArgs a) {
 #pragma unroll
     for (int e = 0; e < VEC; ++e) v[e] = 0.f;
     if (s < k) {
-      VyChunk<T>::load((const T*)a.ring + (int64_t)slot * a.r_ss + (int64_t)g * a.r_sh + (int64_t)((first - k + s) % a.R) * W + c, v);
+      VyChunk<T>::load((const T*)a.ring + (int64_t)slot * a.r_ss + (int64_t)g * a.r_sh + (int64_t)ring_row(s < a.keep ? s : first - k + s, a.R, a.keep) * W + c, v);
     } else if (s - k < a.L) {
       const T* row = (const T*)a.p + ((int64_t)b * a.L + s - k) * a.ldp;
       VyChunk<T>::load(c < a.dim ? row + a.ok + (int64_t)g * a.dim + c : row + a.ov + (int64_t)g * a.vdim + (c - a.dim), v);
@@ -115,11 +238,21 @@ void decode_go(const DecodeArgs& a, dim3 grid, hipStream_t st) {
   else hipLaunchKernelGGL((window_decode_kernel<DHP, 256>), grid, block, 0, st, a);
 }
 
-int check_ring(const char* who, const void* ring, int64_t r_ss, int64_t r_sh, int32_t R, int32_t hk, int32_t dim, int32_t vdim,
-               int vec) {
+int check_ring(const char* who, const void* ring, int64_t r_ss, int64_t r_sh, int32_t R, int32_t keep, int32_t hk, int32_t dim,
+               int32_t vdim, int vec) {
   if (!ring || R < 1 || hk < 1 || dim < 1 || vdim < 1) VY_FAIL(VY_ERR_ARG, "%s: bad ring", who);
+  if (keep < 0 || keep >= R) VY_FAIL(VY_ERR_ARG, "%s: %d kept of %d rows", who, keep, R);
   if (dim % vec || vdim % vec || r_ss % vec || r_sh % vec) VY_FAIL(VY_ERR_ARG, "%s: widths and strides must be multiples of %d", who, vec);
   if (r_sh < (int64_t)R * (dim + vdim) || r_ss < hk * r_sh) VY_FAIL(VY_ERR_ARG, "%s: ring strides do not hold %d rows", who, R);
+  return VY_OK;
+}
+
+int check_prep(const char* who, const vy_qkv_prep* q, int32_t h, int32_t hk, int32_t dim, int32_t vdim, int vec) {
+  if (!q) return VY_OK;
+  if (!q->q_norm != !q->k_norm || (q->q_norm && (q->n_q < 1 || q->n_k < 1 || q->n_q > h * dim || q->n_k > hk * dim)))
+    VY_FAIL(VY_ERR_ARG, "%s: bad query / key norms", who);
+  if ((q->v_mix && (q->ldm % vec || q->ldm < (int64_t)hk * vdim)) || (q->v_out && (q->ldo % vec || q->ldo < (int64_t)hk * vdim)))
+    VY_FAIL(VY_ERR_ARG, "%s: bad value rows", who);
   return VY_OK;
 }
 
@@ -132,7 +265,7 @@ int check_rope(const char* who, const float* rope, int32_t rope_dims, int32_t ro
 }  // namespace
 
 extern "C" int vy_window_rows(void* p, int64_t ldp, int64_t ok, int64_t ov, void* ring, int64_t r_ss, int64_t r_sh, int32_t R,
-                              const float* rope, int32_t rope_dims, int32_t rope_len, int rotate, int store,
+                              int32_t keep, const float* rope, int32_t rope_dims, int32_t rope_len, int rotate, int store,
                               const int32_t* slots, const int32_t* start, const int32_t* count, int64_t B, int64_t L, int32_t hk,
                               int32_t dim, int32_t vdim, int dtype, void* stream) {
   const char* who = "vy_window_rows";
@@ -142,12 +275,12 @@ extern "C" int vy_window_rows(void* p, int64_t ldp, int64_t ok, int64_t ov, void
     VY_FAIL(VY_ERR_ARG, "%s: bad arguments", who);
   if (store) {
     if (!start) VY_FAIL(VY_ERR_ARG, "%s: ring without start positions", who);
-    if (int rc = check_ring(who, ring, r_ss, r_sh, R, hk, dim, vdim, vec)) return rc;
+    if (int rc = check_ring(who, ring, r_ss, r_sh, R, keep, hk, dim, vdim, vec)) return rc;
   }
   if (rotate)
     if (int rc = check_rope(who, rope, rope_dims, rope_len, dim)) return rc;
   if (!rotate && !store) return VY_OK;
-  RowsArgs a{p, ldp, ok, ov, ring, r_ss, r_sh, store ? R : 1, (const float2*)rope, rope_dims / 2, rope_len, slots, start, count,
+  RowsArgs a{p, ldp, ok, ov, ring, r_ss, r_sh, store ? R : 1, store ? keep : 0, (const float2*)rope, rope_dims / 2, rope_len, slots, start, count,
              B * L, (int)L, hk, dim, vdim, rotate && rope_dims > 0, store};
   const int64_t want = vy_cdiv(a.M * hk * ((dim + vdim) / vec), 256);
   const dim3 grid((unsigned)(want < 16384 ? want : 16384)), block(256);
@@ -157,16 +290,55 @@ extern "C" int vy_window_rows(void* p, int64_t ldp, int64_t ok, int64_t ov, void
   return VY_OK;
 }
 
+extern "C" int vy_qkv_rows(void* p, int64_t ldp, int64_t oq, int64_t ok, int64_t ov, const vy_qkv_prep* prep, void* ring, int64_t r_ss,
+                           int64_t r_sh, int32_t R, int32_t keep, const float* rope, int32_t rope_dims, int32_t rope_len, int store,
+                           const int32_t* slots, const int32_t* start, const int32_t* count, int64_t B, int64_t L, int32_t h,
+                           int32_t hk, int32_t dim, int32_t vdim, int dtype, void* stream) {
+  const char* who = "vy_qkv_rows";
+  if (dtype != VY_BF16 && dtype != VY_F32) VY_FAIL(VY_ERR_ARG, "%s: bad dtype %d", who, dtype);
+  const int vec = dtype == VY_BF16 ? 8 : 4;
+  if (!p || !prep || B <= 0 || L <= 0 || h <= 0 || hk <= 0 || dim <= 0 || vdim <= 0 || dim % vec || vdim % vec || ldp % vec || oq % vec ||
+      ok % vec || ov % vec || L > INT32_MAX || (int64_t)(h + hk) * dim > 1 << 24)
+    VY_FAIL(VY_ERR_ARG, "%s: bad arguments", who);
+  if (int rc = check_prep(who, prep, h, hk, dim, vdim, vec)) return rc;
+  if (int rc = check_rope(who, rope, rope_dims, rope_len, dim)) return rc;
+  if (store) {
+    if (!start) VY_FAIL(VY_ERR_ARG, "%s: ring without start positions", who);
+    if (int rc = check_ring(who, ring, r_ss, r_sh, R, keep, hk, dim, vdim, vec)) return rc;
+  }
+  QkvArgs a{};
+  a.r = RowsArgs{p, ldp, ok, ov, ring, r_ss, r_sh, store ? R : 1, store ? keep : 0, (const float2*)rope, rope_dims / 2,
+                 rope_len > 0 ? rope_len : 1, slots, start, count, B * L, (int)L, hk, dim, vdim, rope_dims > 0, store};
+  a.oq = oq; a.h = h; a.q_norm = prep->q_norm; a.k_norm = prep->k_norm; a.n_q = prep->n_q; a.n_k = prep->n_k;
+  a.eps = prep->eps; a.lambda = prep->lambda; a.vm = prep->v_mix; a.ldm = prep->ldm; a.vo = prep->v_out; a.ldvo = prep->ldo;
+  hipStream_t st = (hipStream_t)stream;
+  const int chunks = (h + hk) * dim / vec;
+  // narrow rows: a wave each
+  const bool narrow = chunks <= 64 * 4 && B * L >= 1024;
+  const dim3 grid((unsigned)(narrow ? vy_cdiv(B * L, 4) : B * L)), block(256);
+#define QKV_GO(T)                                                                              \
+  do {                                                                                         \
+    if (narrow) hipLaunchKernelGGL((qkv_rows_kernel<T, 1, 4>), grid, block, 0, st, a);         \
+    else if (chunks <= 512) hipLaunchKernelGGL((qkv_rows_kernel<T, 4, 2>), grid, block, 0, st, a); \
+    else hipLaunchKernelGGL((qkv_rows_kernel<T, 4, 4>), grid, block, 0, st, a);                \
+  } while (0)
+  if (dtype == VY_BF16) QKV_GO(bf16);
+  else QKV_GO(float);
+#undef QKV_GO
+  VY_CHECK_LAUNCH(who);
+  return VY_OK;
+}
+
 extern "C" int vy_window_context(const void* p, int64_t ldp, int64_t ok, int64_t ov, const void* ring, int64_t r_ss, int64_t r_sh,
-                                 int32_t R, void* ctx, int32_t S, int32_t past, const int32_t* slots, const int32_t* start,
+                                 int32_t R, int32_t keep, void* ctx, int32_t S, int32_t past, const int32_t* slots, const int32_t* start,
                                  int64_t B, int64_t L, int32_t hk, int32_t dim, int32_t vdim, int dtype, void* stream) {
   const char* who = "vy_window_context";
   if (dtype != VY_BF16 && dtype != VY_F32) VY_FAIL(VY_ERR_ARG, "%s: bad dtype %d", who, dtype);
   const int vec = dtype == VY_BF16 ? 8 : 4;
   if (!p || !ctx || !start || B <= 0 || L <= 0 || S < L || past < 0 || past > R || ldp % vec || ok % vec || ov % vec)
     VY_FAIL(VY_ERR_ARG, "%s: bad arguments", who);
-  if (int rc = check_ring(who, ring, r_ss, r_sh, R, hk, dim, vdim, vec)) return rc;
-  ContextArgs a{p, ldp, ok, ov, ring, r_ss, r_sh, R, ctx, S, past, slots, start, (int)B, (int)L, hk, dim, vdim};
+  if (int rc = check_ring(who, ring, r_ss, r_sh, R, keep, hk, dim, vdim, vec)) return rc;
+  ContextArgs a{p, ldp, ok, ov, ring, r_ss, r_sh, R, keep, ctx, S, past, slots, start, (int)B, (int)L, hk, dim, vdim};
   const int64_t want = vy_cdiv(B * hk * S * ((dim + vdim) / vec), 256);
   const dim3 grid((unsigned)(want < 16384 ? want : 16384)), block(256);
   if (dtype == VY_BF16) hipLaunchKernelGGL((window_context_kernel<bf16>), grid, block, 0, (hipStream_t)stream, a);
@@ -182,8 +354,8 @@ extern "C" int64_t vy_window_decode_ws_bytes(int32_t B, int32_t h, int32_t hk, i
 }
 
 extern "C" int vy_window_decode(void* p, int64_t ldp, int64_t oq, int64_t ok, int64_t ov, int64_t og, void* ring, int64_t r_ss,
-                                int64_t r_sh, int32_t R, const float* rope, int32_t rope_dims, int32_t rope_len,
-                                const int32_t* slots, const int32_t* start, int64_t max_keys, void* out, int64_t ldo, int64_t B,
+                                int64_t r_sh, int32_t R, int32_t keep, const float* rope, int32_t rope_dims, int32_t rope_len,
+                                const vy_qkv_prep* prep, const int32_t* slots, const int32_t* start, int64_t max_keys, void* out, int64_t ldo, int64_t B,
                                 int32_t h, int32_t hk, int32_t dim, int32_t vdim, float scale, int32_t sink, void* ws,
                                 int64_t ws_bytes, int dtype, void* stream) {
   const char* who = "vy_window_decode";
@@ -193,16 +365,21 @@ extern "C" int vy_window_decode(void* p, int64_t ldp, int64_t oq, int64_t ok, in
     VY_FAIL(VY_ERR_ARG, "%s: bad arguments", who);
   if (ldp % vec || oq % vec || ok % vec || ov % vec || ldo % vec || (og >= 0 && og % vec))
     VY_FAIL(VY_ERR_ARG, "%s: columns and strides must be multiples of %d", who, vec);
-  if (int rc = check_ring(who, ring, r_ss, r_sh, R, hk, dim, vdim, vec)) return rc;
+  if (int rc = check_ring(who, ring, r_ss, r_sh, R, keep, hk, dim, vdim, vec)) return rc;
+  if (int rc = check_prep(who, prep, h, hk, dim, vdim, vec)) return rc;
   if (int rc = check_rope(who, rope, rope_dims, rope_len, dim)) return rc;
   if (rope_dims && max_keys > rope_len) VY_FAIL(VY_ERR_ARG, "%s: %ld positions, rotary table of %d", who, (long)max_keys, rope_len);
   hipStream_t st = (hipStream_t)stream;
   if (dtype == VY_F32 || dim > 256 || vdim > 256) {
     // row-wise kernel over the ring: the new row goes in first
-    if (int rc = vy_window_rows(p, ldp, ok, ov, ring, r_ss, r_sh, R, rope, rope_dims, rope_len, 1, 1, slots, start, nullptr, B, 1,
-                                hk, dim, vdim, dtype, stream)) return rc;
+    int rc;
+    if (prep) rc = vy_qkv_rows(p, ldp, oq, ok, ov, prep, ring, r_ss, r_sh, R, keep, rope, rope_dims, rope_len, 1, slots, start, nullptr, B, 1,
+                               h, hk, dim, vdim, dtype, stream);
+    else rc = vy_window_rows(p, ldp, ok, ov, ring, r_ss, r_sh, R, keep, rope, rope_dims, rope_len, 1, 1, slots, start, nullptr, B, 1,
+                             hk, dim, vdim, dtype, stream);
+    if (rc) return rc;
     const int64_t e = dtype == VY_BF16 ? 2 : 4;
-    const vy_attn_window win{0, sink, 1, INT32_MAX, rope, rope_dims, rope_len};
+    const vy_attn_window win{0, sink, 1, INT32_MAX, prep ? nullptr : rope, prep ? 0 : rope_dims, rope_len, 0};   // (prep: rotated already)
     const char* gate = og >= 0 ? (const char*)p + og * e : nullptr;
     return vy_attn_fwd_ex((const char*)p + oq * e, ldp, dim, ldp, ring, r_ss, r_sh, dim + vdim, (const char*)ring + (int64_t)dim * e,
                           r_ss, r_sh, dim + vdim, out, ldo, ldo, gate, ldp, ldp, start, slots, B, h, hk, 1, R, dim, vdim, scale,
@@ -210,7 +387,11 @@ extern "C" int vy_window_decode(void* p, int64_t ldp, int64_t oq, int64_t ok, in
   }
   DecodeArgs a{};
   a.p = (const bf16*)p; a.ldp = ldp; a.oq = oq; a.ok = ok; a.ov = ov; a.og = og;
-  a.ring = (bf16*)ring; a.r_ss = r_ss; a.r_sh = r_sh; a.R = R;
+  a.ring = (bf16*)ring; a.r_ss = r_ss; a.r_sh = r_sh; a.R = R; a.keep = keep;
+  if (prep) {
+    a.q_norm = prep->q_norm; a.k_norm = prep->k_norm; a.n_q = prep->n_q; a.n_k = prep->n_k; a.eps = prep->eps; a.lambda = prep->lambda;
+    a.vm = (const bf16*)prep->v_mix; a.ldm = prep->ldm; a.vo = (bf16*)prep->v_out; a.ldvo = prep->ldo;
+  }
   a.rope = (const float2*)rope; a.half = rope_dims / 2; a.rope_len = rope_len > 0 ? rope_len : 1;
   a.slots = slots; a.start = start; a.out = (bf16*)out; a.ldo = ldo;
   a.h = h; a.hk = hk; a.dim = dim; a.vdim = vdim; a.scale = scale; a.sink = sink;

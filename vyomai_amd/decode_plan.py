@@ -29,7 +29,7 @@ class VyDecodePlan(C.Structure):
 
 
 def _ptr(t):
-    return None if t is None else t.data_ptr()
+    return None if t is None or isinstance(t, str) else t.data_ptr()   # (ops.PLAIN: no norm)
 
 
 class DecodePlan:
@@ -258,12 +258,14 @@ class GemmaDecodePlan:
 
 class VyHybridLayer(C.Structure):
     _fields_ = [(n, C.c_int32) for n in ("mixer", "heads", "dim", "vdim", "n_in", "ff", "q_rank", "q_rank_p", "kv_rank",
-                                         "kv_rank_p", "cap", "mix_n", "form", "clamped", "kv_heads", "rope_dims", "rope_len", "sink")] + \
-               [(n, C.c_float) for n in ("scale", "limit", "alpha")] + \
+                                         "kv_rank_p", "cap", "mix_n", "form", "clamped", "kv_heads", "rope_dims", "rope_len", "sink", "keep",
+                                         "gate", "values", "silu")] + \
+               [(n, C.c_float) for n in ("scale", "limit", "alpha", "k_scale")] + \
                [(n, C.c_void_p) for n in ("norm1", "norm1b", "norm2", "norm2b", "w_in", "w_o", "w_gu", "w_down", "q_norm",
                                           "c_norm", "w_uq", "w_ukt", "w_uv", "cache")] + \
                [(n, C.c_int64) for n in ("c_ss", "c_sh", "c_st")] + \
-               [(n, C.c_void_p) for n in ("state", "decay_pow", "mix_norm", "rope")] + [("moe", C.POINTER(_lib.VyMoe))]
+               [(n, C.c_void_p) for n in ("state", "decay_pow", "mix_norm", "rope")] + \
+               [("prep", C.POINTER(_lib.VyQkvPrep)), ("moe", C.POINTER(_lib.VyMoe))]
 
 
 class VyHybridPlan(C.Structure):
@@ -306,13 +308,21 @@ class HybridDecodePlan:
                 L.cache, L.c_ss, L.c_st, L.cap = buf.data_ptr(), buf.stride(0), buf.stride(1), buf.shape[1]
             elif m.kind == "window":
                 L.mixer, L.scale, L.kv_heads, L.sink = MIX_WINDOW, m.scale, m.kv_heads, int(m.sink)
+                L.keep, L.gate, L.values = m.keep_first, int(m.gate is not None), m.values
+                c = m.constants()
+                self.keep.append(c)
+                if c.prep is not None:
+                    q = c.prep
+                    L.prep = C.pointer(_lib.VyQkvPrep(_ptr(q.q_norm), _ptr(q.k_norm), q.n_q, q.n_k, q.eps, q.mix))
                 L.cache, L.c_ss, L.c_sh, L.cap = buf.data_ptr(), buf.stride(0), buf.stride(1), buf.shape[2]
+            else:
+                L.mixer, L.state, L.decay_pow = MIX_DECAY, buf.data_ptr(), _ptr(p.decay_pow)
+                L.mix_norm, L.mix_n = _ptr(p.norm), m.heads * m.vdim if p.norm is not None else m.vdim
+                L.silu, L.k_scale = int(m.silu), m.k_scale
+            if getattr(m, "rotary", None) is not None:
                 table = m.rotary.table(cache.capacity, model.device)
                 self.keep.append(table)
                 L.rope, L.rope_dims, L.rope_len = _ptr(table), m.rotary.dims, table.shape[0] if table is not None else 0
-            else:
-                L.mixer, L.state, L.decay_pow = MIX_DECAY, buf.data_ptr(), _ptr(p.decay_pow)
-                L.mix_norm, L.mix_n = _ptr(p.norm), m.heads * m.vdim
             if layer.mlp is not None:
                 dense = layer.mlp.dense
                 if not parallel:

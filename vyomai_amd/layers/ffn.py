@@ -12,7 +12,7 @@ import torch
 import torch.nn as nn
 
 from .. import ops
-from .._lib import ACT_GELU_ERF, ACT_GELU_TANH, ACT_SILU, VyMoe
+from .._lib import (ACT_GELU_ERF, ACT_GELU_TANH, ACT_SILU, MOE_CLAMPED, MOE_GELU, SCORE_SIGMOID, SCORE_SOFTMAX, VyMoe)
 from ..ops import up8
 from .packing import Packed, pad2
 
@@ -89,23 +89,32 @@ class GatedFeedForward(nn.Module):
         return None
 
 
-class MixtureFeedForward(nn.Module):
-    """`top` of `experts` clamped gated feed-forwards per token and (shared may be None) one dense one for every token.
+_EXPERT_ACT = {"clamped": MOE_CLAMPED, "gelu": MOE_GELU}
+_SCORE = {"softmax": SCORE_SOFTMAX, "sigmoid": SCORE_SIGMOID}
 
-    Router scores are softmax(router(x)) in fp32; experts form `groups` equal groups of neighbours and only those of the `keep`
-    groups with the best largest score can be chosen; the chosen scores are normalised to sum 1 and multiplied by `scale`.
-    The experts' weights are one tensor each (experts first); once packed, they are views of the packed storage, so there is one
+
+class MixtureFeedForward(nn.Module):
+    """`top` of `experts` small feed-forwards per token and (shared may be None) one dense one for every token.  act "clamped":
+    the clamped gated one of GatedFeedForward; "gelu": down(gelu(up(x))), the exact GELU, no gate.
+
+    Router scores are softmax(router(x)) or sigmoid(router(x)) (`score`) in fp32; experts form `groups` equal groups of neighbours
+    and only those of the `keep` best groups can be chosen (a group's score: the sum of its `group_best` largest scores, 1 or 2);
+    the chosen scores are normalised to sum 1 (if `normalize`) and multiplied by `scale`.  The experts' weights are one tensor each (experts first); once packed, they are views of the packed storage, so there is one
     copy of them in memory."""
 
-    def __init__(self, width: int, experts: int, top: int, inner: int, limit: float, groups: int = 1, keep: int = 1,
-                 scale: float = 1.0, alpha: float = 1.702, shared: Optional[GatedFeedForward] = None) -> None:
+    def __init__(self, width: int, experts: int, top: int, inner: int, limit: float = 0.0, groups: int = 1, keep: int = 1,
+                 scale: float = 1.0, alpha: float = 1.702, shared: Optional[GatedFeedForward] = None, act: str = "clamped",
+                 score: str = "softmax", group_best: int = 1, normalize: bool = True) -> None:
         super().__init__()
         if experts < 1 or groups < 1 or experts % groups or not 1 <= keep <= groups or not 1 <= top <= keep * (experts // groups):
             raise ValueError(f"{top} of {experts} experts, {keep} of {groups} groups")
+        if act not in _EXPERT_ACT or score not in _SCORE or group_best not in (1, 2):
+            raise ValueError(f"experts' activation {act!r}, scores {score!r}, groups by {group_best} scores")
         self.width, self.experts, self.top, self.inner, self.limit, self.alpha = width, experts, top, inner, float(limit), float(alpha)
         self.groups, self.keep, self.scale = groups, keep, float(scale)
+        self.act, self.score, self.group_best, self.normalize = _EXPERT_ACT[act], _SCORE[score], int(group_best), bool(normalize)
         self.router = nn.Linear(width, experts, bias=False)
-        self.gate = nn.Parameter(torch.empty(experts, inner, width))
+        self.gate = nn.Parameter(torch.empty(experts, inner, width)) if self.act == MOE_CLAMPED else None
         self.up = nn.Parameter(torch.empty(experts, inner, width))
         self.down = nn.Parameter(torch.empty(experts, width, inner))
         self.shared = shared
@@ -113,17 +122,20 @@ class MixtureFeedForward(nn.Module):
     def packed(self) -> Packed:
         def build(p: Packed) -> None:
             dp, ip, n, w = up8(self.width), up8(self.inner), self.inner, self.width
-            dt, dev = self.gate.dtype, self.gate.device
+            dt, dev = self.up.dtype, self.up.device
             p.w_router = pad2(self.router.weight, self.experts, dp).contiguous()
-            p.w_gu = torch.zeros(self.experts, 2 * ip, dp, dtype=dt, device=dev)      # rows interleaved: gate 0, up 0, gate 1, ...
+            rows = 1 if self.gate is None else 2      # rows interleaved: gate 0, up 0, gate 1, ...
+            p.w_gu = torch.zeros(self.experts, rows * ip, dp, dtype=dt, device=dev)
             p.w_down = torch.zeros(self.experts, dp, ip, dtype=dt, device=dev)
-            for param, place in ((self.gate, p.w_gu[:, 0:2 * n:2, :w]), (self.up, p.w_gu[:, 1:2 * n:2, :w]),
+            for param, place in ((self.gate, p.w_gu[:, 0:2 * n:2, :w]), (self.up, p.w_gu[:, rows - 1:rows * n:rows, :w]),
                                  (self.down, p.w_down[:, :w, :n])):
-                place.copy_(param)
-                param.data = place
-            p.desc = VyMoe(self.experts, self.top, self.groups, self.keep, dp, ip, self.scale, self.limit, self.alpha,
-                           p.w_router.data_ptr(), p.w_gu.data_ptr(), p.w_down.data_ptr())
-        return Packed.of(self, [self.router.weight, self.gate, self.up, self.down], build)
+                if param is not None:
+                    place.copy_(param)
+                    param.data = place
+            p.desc = VyMoe(self.experts, self.top, self.groups, self.keep, dp, ip, self.act, self.score, self.group_best,
+                           int(self.normalize), self.scale, self.limit, self.alpha, p.w_router.data_ptr(), p.w_gu.data_ptr(),
+                           p.w_down.data_ptr())
+        return Packed.of(self, [p for p in (self.router.weight, self.gate, self.up, self.down) if p is not None], build)
 
     @property
     def dense(self) -> Optional[GatedFeedForward]:

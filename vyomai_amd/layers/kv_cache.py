@@ -279,8 +279,9 @@ class SlotCache:
 
     A sequence owns a slot while it lives (``allocate`` / ``free``); per layer a slot holds either cached rows
     ("latent", width): a (slots, capacity, width) buffer, or a ring of the last tokens' keys and values ("window", (heads,
-    width, window)): a (slots, heads, rows, width) buffer of min(window, capacity) rows, position p in row p % rows, or a
-    recurrent state ("state", shape): a (slots, *shape) fp32 buffer.  ``lengths`` (int32 on the device, one per slot) says how many tokens a slot holds: kernels place new rows
+    width, rows[, keep])): a (slots, heads, rows, width) buffer (fewer rows while the capacity is less), position p in row p, and
+    from `rows` on round and round the rows behind the `keep` first, or a recurrent state ("state", shape): a (slots, *shape)
+    fp32 buffer.  ``lengths`` (int32 on the device, one per slot) says how many tokens a slot holds: kernels place new rows
     behind them, attend no further, and take the state of an empty slot as zero -- so nothing is cleared when a slot is
     handed on.  The host keeps a mirror (``length``).  Slots and capacity grow by doubling.
     """
@@ -301,8 +302,9 @@ class SlotCache:
         if kind == "latent":
             return torch.zeros(slots, capacity, shape, dtype=self.dtype, device=self.device)
         if kind == "window":
-            heads, width, window = shape
-            return torch.zeros(slots, heads, min(window, capacity), width, dtype=self.dtype, device=self.device)
+            heads, width, rows, *keep = shape
+            rows = min(rows, max(capacity, keep[0] + 1 if keep else 1))
+            return torch.zeros(slots, heads, rows, width, dtype=self.dtype, device=self.device)
         if kind == "state":
             return torch.zeros(slots, *shape, dtype=torch.float32, device=self.device)
         raise ValueError(f"cache kind {kind!r}")
@@ -388,6 +390,7 @@ class SlotBatch:
         self.slots, self.start = cache.table(slots), cache.lengths
         self.past = max(cache.length[s] for s in slots)   # tokens before these, at most
         self.fresh = self.past == 0
+        self.shared_values = None                         # what one layer of this pass leaves to later ones (window attention)
         self.count = None if len(set(counts)) == 1 else torch.tensor(counts, dtype=torch.int32, device=cache.device)
 
     def latents(self, layer: int) -> torch.Tensor:

@@ -18,8 +18,15 @@ from .norms import WeightNorm
 from .packing import Packed, head_cols, head_rows, head_vec
 
 
+def decay_powers(decay: Sequence[float], device) -> torch.Tensor:
+    """(heads, DECAY_CHUNK + 1) fp32: powers of the decays, made in double precision and rounded once."""
+    t = torch.tensor([[d ** i for i in range(DECAY_CHUNK + 1)] for d in decay], dtype=torch.float64)
+    return t.float().to(device)
+
+
 class LightningAttention(nn.Module):
     kind = "decay"
+    silu, rotary, k_scale = True, None, 1.0     # of q, k, v; rotary positions and factor on the keys: none
 
     def __init__(self, width: int, heads: int, dim: int, vdim: int, decay: Sequence[float], eps: float) -> None:
         super().__init__()
@@ -44,9 +51,7 @@ class LightningAttention(nn.Module):
                                 for m in (self.query, self.key, self.value, self.gate)]).contiguous()
             p.norm = head_vec(self.norm.weight, H)
             p.w_o = head_cols(self.out.weight, H, dp)
-            # powers of the decays in double precision, rounded once
-            t = torch.tensor([[d ** i for i in range(DECAY_CHUNK + 1)] for d in self.decay], dtype=torch.float64)
-            p.decay_pow = t.float().to(p.w_in.device)
+            p.decay_pow = decay_powers(self.decay, p.w_in.device)
         return Packed.of(self, list(self.parameters()), build)
 
     def matrices(self):

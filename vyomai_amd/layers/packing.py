@@ -26,9 +26,9 @@ def pad_vec(w: torch.Tensor, n: int) -> torch.Tensor:
     return out
 
 
-def norm_vec(norm, n: int) -> torch.Tensor:
-    """fp32 factors of a WeightNorm, zero-padded to n."""
-    return pad_vec(norm.weight.float() + norm.offset, n)
+def norm_vec(norm, n: int, mult: float = 1.0) -> torch.Tensor:
+    """fp32 factors of a WeightNorm (times mult), zero-padded to n."""
+    return pad_vec((norm.weight.float() + norm.offset) * mult, n)
 
 
 def head_rows(w: torch.Tensor, heads: int, cols: int) -> torch.Tensor:
@@ -47,6 +47,14 @@ def head_cols(w: torch.Tensor, heads: int, rows: int) -> torch.Tensor:
     return out.view(rows, heads * up8(dim))
 
 
+def halves_to_pairs(w: torch.Tensor, heads: int, dims: int) -> torch.Tensor:
+    """Rows of every head put in another order: row i and row i + dims / 2 of its first `dims` become neighbours (2i, 2i + 1).
+    Queries and keys whose rotary pairs are halves apart run on kernels that rotate neighbours: dot products do not see it."""
+    dim, half = w.shape[0] // heads, dims // 2
+    order = [c for i in range(half) for c in (i, i + half)] + list(range(dims, dim))
+    return w.view(heads, dim, *w.shape[1:])[:, order].reshape(w.shape)
+
+
 def head_vec(w: torch.Tensor, heads: int) -> torch.Tensor:
     """fp32 copy of a norm weight over concatenated heads, every head padded by itself."""
     dim = w.numel() // heads
@@ -60,15 +68,15 @@ class Packed:
     parameter into a view of its packed copy: the parameters' state is noted after it.)"""
 
     @staticmethod
-    def of(owner: nn.Module, params: Sequence[torch.Tensor], build: Callable[["Packed"], None]) -> "Packed":
+    def of(owner: nn.Module, params: Sequence[torch.Tensor], build: Callable[["Packed"], None], name: str = "_packed_cache") -> "Packed":
         def state():
             return tuple((p.data_ptr(), p._version, p.dtype) for p in params)
         key = state()
-        hit = owner.__dict__.get("_packed_cache")
+        hit = owner.__dict__.get(name)
         if hit is None or hit.key != key:
             hit = Packed()
             with torch.no_grad():
                 build(hit)
             hit.key = state()
-            owner.__dict__["_packed_cache"] = hit
+            owner.__dict__[name] = hit
         return hit

@@ -4,7 +4,8 @@ QKV projection epilogue on the model path, or by ``vy_rope_fwd`` through
 ``apply_rotary_pos_emb``; the additive encodings are table lookups kept in PyTorch."""
 from __future__ import annotations
 
-from typing import Dict, Optional, Tuple
+import math
+from typing import Dict, List, Optional, Tuple
 
 import torch
 import torch.nn as nn
@@ -103,28 +104,44 @@ def resolve_freqs(freqs, device):
 class PairRotary:
     """Rotary positions on neighbouring columns (2i, 2i + 1) of the first `dims` columns of a head, pair i turning by
     position * base^(-2i / dims).  table(n): at least n positions of (cos, sin), fp32 (evaluated in double precision), shaped
-    (positions, dims / 2, 2); None without rotated columns.  Layers with equal constants share their tables."""
+    (positions, dims / 2, 2); None without rotated columns.  Layers with equal constants share their tables.
+
+    scaling (factor, original, fast, slow): YaRN.  Pairs that turn more than `fast` times within `original` positions keep their
+    frequency, those that turn less than `slow` times have it divided by `factor`, a ramp over the pairs lies between; cosines
+    and sines carry the factor 0.1 ln(factor) + 1."""
 
     _tables: Dict[tuple, torch.Tensor] = {}
 
-    def __init__(self, base: float, dims: int) -> None:
+    def __init__(self, base: float, dims: int, scaling: Optional[Dict[str, float]] = None) -> None:
         if dims < 0 or dims % 2:
             raise ValueError(f"{dims} rotated columns (an even number)")
         self.base, self.dims = float(base), int(dims)
+        self.scaling = None if scaling is None else tuple(float(scaling[k]) for k in ("factor", "original", "fast", "slow"))
+
+    def frequencies(self) -> Tuple[List[float], float]:
+        """Angle per position of every pair, and the factor on cosines and sines."""
+        n = self.dims // 2
+        f = [self.base ** (-2.0 * i / self.dims) for i in range(n)]
+        if self.scaling is None:
+            return f, 1.0
+        factor, original, fast, slow = self.scaling
+        pair = [self.dims * math.log(original / (2.0 * math.pi * turns)) / (2.0 * math.log(self.base)) for turns in (fast, slow)]
+        lo, hi = max(math.floor(pair[0]), 0), min(math.ceil(pair[1]), self.dims - 1)
+        ramp = [min(max((i - lo) / max(hi - lo, 0.001), 0.0), 1.0) for i in range(n)]
+        return [a / factor * r + a * (1.0 - r) for a, r in zip(f, ramp)], 0.1 * math.log(factor) + 1.0
 
     def table(self, positions: int, device) -> Optional[torch.Tensor]:
         if self.dims == 0:
             return None
-        key = self.base, self.dims, torch.device(device)
+        key = self.base, self.dims, self.scaling, torch.device(device)
         t = self._tables.get(key)
         if t is None or t.shape[0] < positions:
             n = 256
             while n < positions:
                 n *= 2
-            f = torch.pow(torch.tensor(self.base, dtype=torch.float64, device=device),
-                          -torch.arange(0, self.dims, 2, dtype=torch.float64, device=device) / self.dims)
-            a = torch.arange(n, dtype=torch.float64, device=device)[:, None] * f[None, :]
-            t = self._tables[key] = torch.stack((a.cos(), a.sin()), -1).float().contiguous()
+            f, factor = self.frequencies()
+            a = torch.arange(n, dtype=torch.float64, device=device)[:, None] * torch.tensor(f, dtype=torch.float64, device=device)[None, :]
+            t = self._tables[key] = (torch.stack((a.cos(), a.sin()), -1) * factor).float().contiguous()
         return t
 
 

@@ -1,10 +1,10 @@
 """Decoders that mix layer kinds over an fp32 residual stream: every layer is one mixer (latent attention, lightning attention,
 windowed attention, ...) and an optional feed-forward (gated, or a mixture of experts), in one of two forms:
 
-    HybridLayer    x <- x + norm1b(mixer(norm1(x))) ;  x <- x + norm2b(ff(norm2(x)))
+    HybridLayer    x <- x + m norm1b(mixer(norm1(x))) ;  x <- x + m norm2b(ff(norm2(x)))    (without norm1 / norm2: of x itself)
     ParallelLayer  x <- x + (mixer(h) + ff(h)),  h = norm1(x)
 
-A design built from this file supplies its layers and its parameter names (models/gisitar.py, models/rivudra.py); embedding,
+A design built from this file supplies its layers and its parameter names (models/gisitar.py, rivudra.py, padulorn.py); embedding,
 residual stream, slot cache, prefill, the native single-token step and generation are here.  Inference only.
 """
 from __future__ import annotations
@@ -25,27 +25,30 @@ from .decoder import CLMOutput
 
 
 class HybridLayer(nn.Module):
-    """One mixer and (mlp may be None) one feed-forward behind it, with their four norms."""
+    """One mixer and (mlp may be None) one feed-forward behind it, with norms ahead of them (pre) and on their outputs, which
+    join the residual stream times `mult`."""
     form = "sandwich"
 
     def __init__(self, width: int, mixer: nn.Module, mlp: Optional[nn.Module], eps: float, norm: str = "layer",
-                 offset: float = 0.0) -> None:
+                 offset: float = 0.0, pre: bool = True, mult: float = 1.0) -> None:
         super().__init__()
-        self.mixer, self.mlp, self.width = mixer, mlp, width
+        self.mixer, self.mlp, self.width, self.pre, self.mult = mixer, mlp, width, pre, float(mult)
         for n in self._norms():
             setattr(self, n, WeightNorm(width, eps, norm, offset))
 
     def _norms(self) -> List[str]:
-        return ["norm1", "norm1b"] + (["norm2", "norm2b"] if self.mlp is not None else [])
+        names = ["norm1", "norm1b"] + (["norm2", "norm2b"] if self.mlp is not None else [])
+        return [n for n in names if self.pre or n.endswith("b")]
 
     def packed(self) -> Packed:
         def build(p: Packed) -> None:
+            p.norm1 = p.norm2 = ops.PLAIN
             for n in self._norms():
-                setattr(p, n, norm_vec(getattr(self, n), up8(self.width)))
+                setattr(p, n, norm_vec(getattr(self, n), up8(self.width), self.mult if n.endswith("b") else 1.0))
         return Packed.of(self, [getattr(self, n).weight for n in self._norms()], build)
 
     def run(self, norm, h: torch.Tensor, B: int, L: int, batch, layer: int, nxt: Optional[torch.Tensor]) -> Optional[torch.Tensor]:
-        """h = norm1(x) of the new tokens; norm(y=, post=, pre=, routed=) advances the residual stream x by a sublayer and
+        """h = norm1(x) (or x) of the new tokens; norm(y=, post=, pre=, routed=) advances the residual stream x by a sublayer and
         returns its next norm.  nxt: the norm of what follows this layer."""
         p = self.packed()
         y = self.mixer(h, B, L, batch, layer)
@@ -99,10 +102,10 @@ class HybridDecoderModel(nn.Module):
     """`layers` of HybridLayer / ParallelLayer between a (scaled) embedding and a norm + vocabulary projection."""
 
     def __init__(self, config, width: int, vocab: int, layers: Sequence[nn.Module], eps: float, norm: str = "layer",
-                 offset: float = 0.0, embed_scale: float = 1.0) -> None:
+                 offset: float = 0.0, embed_scale: float = 1.0, logit_scale: float = 1.0) -> None:
         super().__init__()
         self.config, self.width, self.vocab, self.eps, self.rms = config, width, vocab, float(eps), norm == "rms"
-        self.embed_scale = float(embed_scale)
+        self.embed_scale, self.logit_scale = float(embed_scale), float(logit_scale)
         self.word_embeddings = nn.Embedding(vocab, width)
         self.layers = nn.ModuleList(layers)
         self.final_norm = WeightNorm(width, eps, norm, offset)
@@ -124,7 +127,7 @@ class HybridDecoderModel(nn.Module):
             dp = up8(self.width)
             p.embed = pad2(self.word_embeddings.weight, self.vocab, dp).contiguous()
             p.head = pad2(self.head.weight, self.vocab, dp).contiguous()
-            p.final_norm = norm_vec(self.final_norm, dp)
+            p.final_norm = norm_vec(self.final_norm, dp, self.logit_scale)   # (the head is linear)
         return Packed.of(self, [self.word_embeddings.weight, self.head.weight, self.final_norm.weight], build)
 
     # ---- cache ------------------------------------------------------------------------------

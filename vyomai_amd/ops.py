@@ -8,7 +8,7 @@ from __future__ import annotations
 
 import ctypes as C
 import math
-from typing import NamedTuple, Optional, Tuple
+from typing import NamedTuple, Optional, Tuple, Union
 
 import torch
 
@@ -661,14 +661,20 @@ def up8(n: int) -> int:
     return (n + 7) // 8 * 8
 
 
+PLAIN = "plain"   # in the place of a norm's factors: no norm, the stream itself in the compute dtype
+
+
 def residual_norm(x: Tensor, width: int, *, y: Optional[Tensor] = None, post: Optional[Tensor] = None,
-                  pre: Optional[Tensor] = None, eps: float = 1e-5, rms: bool = False, table: Optional[Tensor] = None,
+                  pre: Union[Tensor, str, None] = None, eps: float = 1e-5, rms: bool = False, table: Optional[Tensor] = None,
                   ids: Optional[Tensor] = None, dtype: Optional[torch.dtype] = None,
                   err_flag: Optional[Tensor] = None, table_scale: float = 1.0,
                   routed: Optional["Routed"] = None) -> Optional[Tensor]:
     """x (M, padded width) fp32, in place: x += norm(y) * post (post None: x += y), or x = table_scale * table[ids]; routed:
     y also gets the weighted rows of every token's experts (y None: they are all of it); returns norm(x) * pre in `dtype`
-    (None without pre).  (vy_residual_norm_routed)"""
+    (pre PLAIN: x itself; None without pre).  (vy_residual_norm_routed)"""
+    want_h = pre is not None
+    if pre is PLAIN:
+        pre = None
     _need_gpu(x, y, post, pre, table, ids)
     assert x.dtype == torch.float32 and x.dim() == 2 and x.stride(1) == 1
     for w in (post, pre):
@@ -682,7 +688,7 @@ def residual_norm(x: Tensor, width: int, *, y: Optional[Tensor] = None, post: Op
         assert y.shape[0] == M
     if ids is not None:
         assert ids.dtype == torch.long and ids.is_contiguous() and ids.numel() == M and table is not None
-    h = torch.empty((M, NP), dtype=dt, device=x.device) if pre is not None else None
+    h = torch.empty((M, NP), dtype=dt, device=x.device) if want_h else None
     extra = None
     if routed is not None:
         r, top = routed.rows, routed.weight.shape[1]
@@ -734,12 +740,25 @@ def rmsnorm_gate(x: Tensor, w: Tensor, width: int, gate: Tensor, eps: float, out
     return y
 
 
+def head_norm_gate(x: Tensor, heads: int, width: int, gate: Tensor, eps: float, out: Optional[Tensor] = None) -> Tensor:
+    """x / rms(x) * silu(gate), every head (`width` of its padded columns) by itself.  (vy_head_norm_gate)"""
+    _need_gpu(x, gate, out)
+    M, NP = x.shape
+    assert NP % heads == 0 and gate.shape == x.shape and x.stride(1) == 1 and gate.stride(1) == 1
+    y = torch.empty((M, NP), dtype=x.dtype, device=x.device) if out is None else out
+    assert y.shape == x.shape and y.stride(1) == 1 and y.dtype == x.dtype
+    call("vy_head_norm_gate", x.data_ptr(), x.stride(0), gate.data_ptr(), gate.stride(0), y.data_ptr(), y.stride(0), M, heads,
+         int(width), NP // heads, float(eps), dtype_code(x.dtype), _stream())
+    return y
+
+
 def attention_ex(q: Tensor, k: Tensor, v: Tensor, scale: float, *, gate: Optional[Tensor] = None,
                  start: Optional[Tensor] = None, slots: Optional[Tensor] = None, window: int = 0, sink: bool = False,
-                 rotary: Optional[Tensor] = None, start_cap: Optional[int] = None, out: Optional[Tensor] = None) -> Tensor:
+                 rotary: Optional[Tensor] = None, start_cap: Optional[int] = None, keep: int = 0,
+                 out: Optional[Tensor] = None) -> Tensor:
     """Causal attention with a value width of its own: q (B,h,L,dh), k (B,hk,S,dh), v (B,hk,S,dv) -> (B, L, h*dv); `start`
     (int32, per slot) keys precede the queries; gate (B, L, h*dv): out *= sigmoid(gate).  window: only the last `window` keys up
-    to a query's own are seen (0: all); sink: one more exp(0) in the denominators; rotary (positions, pairs, 2): the queries are
+    to a query's own are seen (0: all), and the first `keep` of all; sink: one more exp(0) in the denominators; rotary (positions, pairs, 2): the queries are
     rotated by position start + i; start_cap: at most so many keys precede the queries.  (vy_attn_fwd_ex)"""
     _need_gpu(q, k, v, gate, start, slots)
     B, h, L, dh = q.shape
@@ -754,7 +773,7 @@ def attention_ex(q: Tensor, k: Tensor, v: Tensor, scale: float, *, gate: Optiona
     if window or sink or rotary is not None or start_cap is not None:
         _need_gpu(rotary)
         win = _lib.VyAttnWindow(int(window), int(sink), 0, 2 ** 31 - 1 if start_cap is None else int(start_cap),
-                                *_rotary_args(rotary))
+                                *_rotary_args(rotary), int(keep))
     call("vy_attn_fwd_ex", q.data_ptr(), q.stride(0), q.stride(1), q.stride(2), k.data_ptr(), k.stride(0), k.stride(1),
          k.stride(2), v.data_ptr(), v.stride(0), v.stride(1), v.stride(2), out.data_ptr(), out.stride(0), out.stride(1),
          _ptr(gate), gate.stride(0) if gate is not None else 0, gate.stride(1) if gate is not None else 0, _ptr(start),
@@ -780,36 +799,77 @@ def _ring_args(ring: Optional[Tensor], hk: int, dim: int, vdim: int):
 
 
 def window_rows(p: Tensor, B: int, L: int, hk: int, dim: int, vdim: int, ok: int, ov: int, *, rotary: Optional[Tensor] = None,
-                ring: Optional[Tensor] = None, slots: Optional[Tensor] = None, start: Optional[Tensor] = None,
+                ring: Optional[Tensor] = None, keep: int = 0, slots: Optional[Tensor] = None, start: Optional[Tensor] = None,
                 count: Optional[Tensor] = None) -> None:
     """Packed rows p (B*L, .) with keys at column ok and values at ov: rotary given: the keys are rotated in place; ring given:
-    the last rows of every sequence go to it.  (vy_window_rows)"""
+    the rows that it holds behind them (the first `keep` of a sequence and its last ones) go to it.  (vy_window_rows)"""
     _need_gpu(p, rotary, ring, slots, start, count)
     _slot_args(slots, start, count, B)
     assert p.shape[0] == B * L and p.stride(1) == 1 and (ring is None or ring.dtype == p.dtype)
-    call("vy_window_rows", p.data_ptr(), p.stride(0), ok, ov, *_ring_args(ring, hk, dim, vdim), *_rotary_args(rotary),
+    call("vy_window_rows", p.data_ptr(), p.stride(0), ok, ov, *_ring_args(ring, hk, dim, vdim), int(keep), *_rotary_args(rotary),
          int(rotary is not None), int(ring is not None), _ptr(slots), _ptr(start), _ptr(count), B, L, hk, dim, vdim,
          dtype_code(p.dtype), _stream())
 
 
+class QkvPrep(NamedTuple):
+    """What happens to packed queries, keys and values ahead of attention: RMS norms over the whole query and key projection
+    (fp32 factors over the padded heads, zero in the padding; n_q / n_k true columns), and a share `mix` of the values
+    `values` (rows of another layer's) in the values.  `keep_values`: receives the values before mixing."""
+    q_norm: Optional[Tensor] = None
+    k_norm: Optional[Tensor] = None
+    n_q: int = 0
+    n_k: int = 0
+    eps: float = 0.0
+    mix: float = 0.0
+    values: Optional[Tensor] = None
+    keep_values: Optional[Tensor] = None
+
+
+def _prep_args(prep: Optional[QkvPrep], M: int, h: int, hk: int, dim: int, vdim: int, dtype: torch.dtype):
+    if prep is None:
+        return None
+    _need_gpu(prep.q_norm, prep.k_norm, prep.values, prep.keep_values)
+    for w, n in ((prep.q_norm, h * dim), (prep.k_norm, hk * dim)):
+        assert w is None or (w.dtype == torch.float32 and w.numel() == n and w.is_contiguous())
+    for t in (prep.values, prep.keep_values):
+        assert t is None or (t.shape == (M, hk * vdim) and t.dtype == dtype and t.stride(1) == 1)
+    v, k = prep.values, prep.keep_values
+    return _lib.VyQkvPrep(_ptr(prep.q_norm), _ptr(prep.k_norm), int(prep.n_q), int(prep.n_k), float(prep.eps), float(prep.mix), _ptr(v),
+                          v.stride(0) if v is not None else 0, _ptr(k), k.stride(0) if k is not None else 0)
+
+
+def qkv_rows(p: Tensor, B: int, L: int, h: int, hk: int, dim: int, vdim: int, oq: int, ok: int, ov: int, prep: QkvPrep, *,
+             rotary: Optional[Tensor] = None, ring: Optional[Tensor] = None, keep: int = 0, slots: Optional[Tensor] = None,
+             start: Optional[Tensor] = None, count: Optional[Tensor] = None) -> None:
+    """Packed rows p (B*L, .) in place: queries and keys normed and rotated, values mixed, as `prep` and `rotary` say; ring
+    given: as window_rows.  (vy_qkv_rows)"""
+    _need_gpu(p, rotary, ring, slots, start, count)
+    _slot_args(slots, start, count, B)
+    assert p.shape[0] == B * L and p.stride(1) == 1 and (ring is None or ring.dtype == p.dtype)
+    call("vy_qkv_rows", p.data_ptr(), p.stride(0), oq, ok, ov, C.byref(_prep_args(prep, B * L, h, hk, dim, vdim, p.dtype)),
+         *_ring_args(ring, hk, dim, vdim), int(keep), *_rotary_args(rotary), int(ring is not None), _ptr(slots), _ptr(start),
+         _ptr(count), B, L, h, hk, dim, vdim, dtype_code(p.dtype), _stream())
+
+
 def window_context(p: Tensor, B: int, L: int, hk: int, dim: int, vdim: int, ok: int, ov: int, ring: Tensor, past: int,
-                   start: Tensor, slots: Optional[Tensor] = None) -> Tensor:
-    """(B, hk, past + L, dim + vdim): the last min(start, past) rows of every ring in order, then the new ones.
+                   start: Tensor, slots: Optional[Tensor] = None, keep: int = 0) -> Tensor:
+    """(B, hk, past + L, dim + vdim): min(start, past) rows of every ring in order of position (the `keep` first, then the last
+    of the others), then the new ones.
     (vy_window_context)"""
     _need_gpu(p, ring, slots, start)
     _slot_args(slots, start, None, B)
     assert p.shape[0] == B * L and p.stride(1) == 1 and ring.dtype == p.dtype
     ctx = torch.empty((B, hk, past + L, dim + vdim), dtype=p.dtype, device=p.device)
-    call("vy_window_context", p.data_ptr(), p.stride(0), ok, ov, *_ring_args(ring, hk, dim, vdim), ctx.data_ptr(), past + L, past,
+    call("vy_window_context", p.data_ptr(), p.stride(0), ok, ov, *_ring_args(ring, hk, dim, vdim), int(keep), ctx.data_ptr(), past + L, past,
          _ptr(slots), start.data_ptr(), B, L, hk, dim, vdim, dtype_code(p.dtype), _stream())
     return ctx
 
 
 def window_decode(p: Tensor, h: int, hk: int, dim: int, vdim: int, ring: Tensor, scale: float, start: Tensor, max_keys: int, *,
-                  rotary: Optional[Tensor] = None, sink: bool = False, gate: bool = False,
-                  slots: Optional[Tensor] = None) -> Tensor:
+                  rotary: Optional[Tensor] = None, sink: bool = False, gate: bool = False, keep: int = 0,
+                  prep: Optional[QkvPrep] = None, slots: Optional[Tensor] = None) -> Tensor:
     """One token per sequence, packed rows p (B, [q | k | v | gate]): its key and value go to the ring, its queries attend
-    over it -> (B, h*vdim).  (vy_window_decode)"""
+    over it -> (B, h*vdim); prep: see qkv_rows.  (vy_window_decode)"""
     _need_gpu(p, ring, slots, start, rotary)
     B = p.shape[0]
     _slot_args(slots, start, None, B)
@@ -820,8 +880,9 @@ def window_decode(p: Tensor, h: int, hk: int, dim: int, vdim: int, ring: Tensor,
     nws = _lib.load().vy_window_decode_ws_bytes(B, h, hk, vdim, ring.shape[2])
     ws = torch.empty(max(nws, 1), dtype=torch.uint8, device=p.device)
     call("vy_window_decode", p.data_ptr(), p.stride(0), 0, nk, nk + gk, nk + gk + gv if gate else -1,
-         *_ring_args(ring, hk, dim, vdim), *_rotary_args(rotary), _ptr(slots), start.data_ptr(), int(max_keys), out.data_ptr(),
-         out.stride(0), B, h, hk, dim, vdim, float(scale), int(sink), ws.data_ptr(), nws, dtype_code(p.dtype), _stream())
+         *_ring_args(ring, hk, dim, vdim), int(keep), *_rotary_args(rotary),
+         C.byref(_prep_args(prep, B, h, hk, dim, vdim, p.dtype)) if prep is not None else None, _ptr(slots), start.data_ptr(),
+         int(max_keys), out.data_ptr(), out.stride(0), B, h, hk, dim, vdim, float(scale), int(sink), ws.data_ptr(), nws, dtype_code(p.dtype), _stream())
     return out
 
 
@@ -871,10 +932,12 @@ def latent_decode(q: Tensor, wukt: Tensor, wuv: Tensor, cache: Tensor, start: Te
 
 
 def decay_attention(p: Tensor, heads: int, dk: int, dv: int, state: Tensor, decay_pow: Tensor, B: int, L: int, *,
-                    start: Tensor, slots: Optional[Tensor] = None, count: Optional[Tensor] = None,
-                    silu: bool = True) -> Tensor:
+                    start: Tensor, slots: Optional[Tensor] = None, count: Optional[Tensor] = None, silu: bool = True,
+                    rotary: Optional[Tensor] = None, k_scale: float = 1.0) -> Tensor:
     """Decayed linear attention over packed rows p = [q (heads*dk) | k (heads*dk) | v (heads*dv) | ...] of B sequences of L
-    tokens; state (slots, heads, dk, dv) fp32 is read (zero where start[slot] == 0) and updated.  (vy_decay_attn)"""
+    tokens; state (slots, heads, dk, dv) fp32 is read (zero where start[slot] == 0) and updated.  rotary: q and k are rotated by
+    their positions; k_scale: factor on k.  (vy_decay_attn)"""
+    _need_gpu(rotary)
     _need_gpu(p, state, decay_pow, start, slots, count)
     _slot_args(slots, start, count, B)
     assert p.shape[0] == B * L and p.stride(1) == 1 and p.shape[1] >= heads * (2 * dk + dv)
@@ -884,6 +947,6 @@ def decay_attention(p: Tensor, heads: int, dk: int, dv: int, state: Tensor, deca
     nws = _lib.load().vy_decay_attn_ws_bytes(B, L, heads, dk, dv, dtype_code(p.dtype))
     ws = torch.empty(nws, dtype=torch.uint8, device=p.device) if nws else None
     call("vy_decay_attn", p.data_ptr(), p.stride(0), 0, heads * dk, 2 * heads * dk, state.data_ptr(), decay_pow.data_ptr(),
-         _ptr(slots), start.data_ptr(), _ptr(count), out.data_ptr(), out.stride(0), B, L, heads, dk, dv, int(silu), _ptr(ws),
-         nws, dtype_code(p.dtype), _stream())
+         _ptr(slots), start.data_ptr(), _ptr(count), out.data_ptr(), out.stride(0), B, L, heads, dk, dv, int(silu),
+         *_rotary_args(rotary), float(k_scale), _ptr(ws), nws, dtype_code(p.dtype), _stream())
     return out
