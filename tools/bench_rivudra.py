@@ -17,13 +17,21 @@ from tools.bench_gisitar import DECODE, DIM, LAYERS, PREFILL, VOCAB, measure_gem
 SIZES = {1024: (8, 2, 1024, 32, 4, 4, 2, 512, 1024), 2048: (16, 4, 1024, 64, 4, 8, 4, 1024, 2048)}
 
 
-def rivudra(width):
+def init_experts(m):
+    with torch.no_grad():
+        for l in m.layers:
+            for p in (l.mlp.gate, l.mlp.up, l.mlp.down):
+                if p is not None:
+                    p.normal_(std=p.shape[-1] ** -0.5)
+
+
+def rivudra(width, size=None):
     from vyomai_amd import RivudraConfig, RivudraModel
-    H, G, window, E, top, groups, keep, ff, shared = SIZES[width]
+    H, G, window, E, top, groups, keep, ff, shared = size or SIZES[width]
     layer = {"type": "attention", "mixer": {"heads": H, "kv_heads": G, "dim": DIM, "vdim": DIM, "scale": DIM ** -0.5,
                                             "mask": {"size": window}, "rot": {"base": 10000.0, "dims": DIM}},
              "mlp": {"kind": "moe", "router": {"experts": E, "top": top, "scale": 1.0, "groups": {"count": groups, "keep": keep}},
-                     "expert": {"ff": ff, "limit": 7.0}, "shared": {"ff": shared, "limit": 7.0}}}
+                     "expert": {"ff": ff, "limit": 7.0}, "shared": {"ff": shared, "limit": 7.0} if shared else None}}
     torch.manual_seed(0)
     with torch.device("cuda"):
         torch.set_default_dtype(torch.bfloat16)
@@ -31,19 +39,23 @@ def rivudra(width):
             m = RivudraModel(RivudraConfig(vocab=VOCAB, width=width, layers=[layer] * LAYERS))
         finally:
             torch.set_default_dtype(torch.float32)
-    with torch.no_grad():
-        for l in m.layers:
-            for p in (l.mlp.gate, l.mlp.up, l.mlp.down):
-                p.normal_(std=p.shape[-1] ** -0.5)
+    init_experts(m)
     return m.eval()
 
 
+def measure_rivudra(width, cases, size=None):
+    H, G, window, E, top, _, _, ff, _ = size or SIZES[width]
+
+    def cached(B, ctx):
+        return LAYERS * B * min(ctx, window) * G * 2 * DIM * 2
+    return measure_routed(rivudra(width, size), width, cases, E, top, 3 * width * ff, cached)
+
+
 @torch.no_grad()
-def measure_rivudra(width, cases):
-    H, G, window, E, top, _, _, ff, _ = SIZES[width]
-    m = rivudra(width)
+def measure_routed(m, width, cases, E, top, expert, cached):
+    """Throughputs of a hybrid decoder whose layers all have a mixture: `expert` weights per expert, cached(B, context) bytes read
+    per decode step besides weights."""
     total = sum(p.numel() for p in m.parameters())
-    expert = 3 * width * ff
     out = {"parameters": total, "active_parameters": total - LAYERS * (E - top) * expert}
     for c in cases:
         if c in PREFILL:
@@ -69,8 +81,7 @@ def measure_rivudra(width, cases):
             h = torch.randn(B, width, device="cuda", dtype=torch.bfloat16)
             used = sum(int(l.mlp.routed(h).ids.unique().numel()) for l in m.layers)
             ms = timed(lambda: m.decode(ids, cache, slots), n - 5)
-            cached = LAYERS * B * min(ctx, window) * G * 2 * DIM * 2
-            nbytes = (total - VOCAB * width - LAYERS * E * expert + used * expert) * 2 + cached
+            nbytes = (total - VOCAB * width - LAYERS * E * expert + used * expert) * 2 + cached(B, ctx)
             out[c] = {"batch": B, "context": ctx, "ms_per_step": round(ms, 4), "tokens_per_sec": round(B / ms * 1e3, 1),
                       "experts_per_layer": round(used / LAYERS, 1), "bytes_per_step": int(nbytes),
                       "achieved_GBps": round(nbytes / ms * 1e-6, 1)}
