@@ -260,7 +260,8 @@ typedef struct vy_qkv_prep {
   const float *q_norm, *k_norm;     /* [h][dim], [hk][dim] factors (NULL: no norms), zero in padded columns */
   int32_t n_q, n_k;                 /* columns the norms divide by */
   float eps, lambda;
-  const void* v_mix; int64_t ldm;   /* nullable: v <- (1 - lambda) v + lambda v_mix, rows of [hk][vdim] */
+  const void* v_mix; int64_t ldm;   /* nullable: v <- (1 - lambda) v + lambda v_mix, both as flat rows of their used columns */
+  int32_t n_v, m_v, m_vp;           /* used columns of a value head; of v_mix's heads, and those with their padding (m_v 0: as v's) */
   void* v_out; int64_t ldo;         /* nullable: receives the values as they were before mixing */
 } vy_qkv_prep;
 int vy_qkv_rows(void* p, int64_t ldp, int64_t oq, int64_t ok, int64_t ov, const vy_qkv_prep* prep, void* ring, int64_t r_ss,

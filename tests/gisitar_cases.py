@@ -94,7 +94,7 @@ def write_folder(folder, cfg, w):
         json.dump(cfg, f)
     header, blob = {}, b""
     for n, t in w.items():
-        raw = t.to(torch.bfloat16).contiguous().view(torch.uint8).numpy().tobytes()
+        raw = t.to(torch.bfloat16).reshape(-1).view(torch.uint8).numpy().tobytes()
         header[n] = {"dtype": "BF16", "shape": list(t.shape), "data_offsets": [len(blob), len(blob) + len(raw)]}
         blob += raw
     head = json.dumps(header).encode()

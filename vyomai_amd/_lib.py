@@ -114,7 +114,7 @@ class VyAttnWindow(C.Structure):
 class VyQkvPrep(C.Structure):
     """vy_qkv_prep of include/vyom_hip.h."""
     _fields_ = [("q_norm", _p), ("k_norm", _p), ("n_q", C.c_int32), ("n_k", C.c_int32), ("eps", C.c_float), ("lambda_", C.c_float),
-                ("v_mix", _p), ("ldm", _i64), ("v_out", _p), ("ldo", _i64)]
+                ("v_mix", _p), ("ldm", _i64), ("n_v", C.c_int32), ("m_v", C.c_int32), ("m_vp", C.c_int32), ("v_out", _p), ("ldo", _i64)]
 
 
 class VyRoutedRows(C.Structure):

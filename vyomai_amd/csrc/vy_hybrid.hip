@@ -118,7 +118,7 @@ extern "C" int vy_hybrid_decoder_step(const vy_hybrid_plan* p, const int64_t* id
   float* ew = (float*)take(B * s.top * 4);
   void* ews = take(s.moe_ws);
   void* values = take(B * s.values * e);
-  int64_t values_ld = 0;   // set by the layer that fills them
+  const vy_hybrid_layer* values_of = nullptr;   // the layer that filled them
   int rc;
   auto norm = [&](const void* yy, const vy_routed_rows* routed, const float* post, const float* pre, bool last) {
     return vy_residual_norm_ex(x, dp, yy, dp, p->embed, dp, yy || routed ? nullptr : ids, p->vocab, p->err, p->embed_scale, routed,
@@ -157,11 +157,16 @@ extern "C" int vy_hybrid_decoder_step(const vy_hybrid_plan* p, const int64_t* id
       if (L.prep) prep = *L.prep;
       if (L.values == VY_VALUES_FIRST) {
         prep.v_out = values;
-        prep.ldo = values_ld = gv;
+        prep.ldo = gv;
+        values_of = &L;
       } else if (L.values == VY_VALUES_MIX) {
-        if (values_ld != gv) VY_FAIL(VY_ERR_ARG, "%s: layer %d mixes values of %ld columns with %ld", who, l, (long)gv, (long)values_ld);
+        const vy_hybrid_layer* F = values_of;
+        if (!F || !F->prep || F->kv_heads * F->prep->n_v != L.kv_heads * prep.n_v)
+          VY_FAIL(VY_ERR_ARG, "%s: layer %d has no values to mix in", who, l);
         prep.v_mix = values;
-        prep.ldm = gv;
+        prep.ldm = (int64_t)F->kv_heads * F->vdim;
+        prep.m_v = F->prep->n_v;
+        prep.m_vp = F->vdim;
       }
       if ((rc = vy_window_decode(in, L.n_in, 0, nk, nk + gk, L.gate ? nk + gk + gv : -1, L.cache, L.c_ss, L.c_sh, L.cap, L.keep, L.rope,
                                  L.rope_dims, L.rope_len, L.prep || L.values != VY_VALUES_OWN ? &prep : nullptr, slots, lengths, max_keys, ao, na, B, L.heads, L.kv_heads, L.dim, L.vdim, L.scale,

@@ -24,6 +24,7 @@ struct DecodeArgs {
   const float2* rope; int half, rope_len;
   const float* q_norm; const float* k_norm; int n_q, n_k; float eps;   // nullable: norms over the whole projections
   const bf16* vm; int64_t ldm; float lambda;                           // nullable: values mixed in
+  int n_v, m_v, m_vp;                                                  // used columns of v's heads and of vm's, and vm's padded ones
   bf16* vo; int64_t ldvo;                                              // nullable: receives the token's own values
   const int* slots; const int* start;
   bf16* out; int64_t ldo;
@@ -79,6 +80,23 @@ __device__ __forceinline__ bf16x8 rotate8(const DecodeArgs& a, const float2* t, 
 #pragma unroll
   for (int e = 0; e < 8; ++e) y[e] = (bf16)v[e];
   return y;
+}
+// v <- (1 - lambda) v + lambda m on VEC columns d .. of head g; the rows m have heads of their own width (m_v of m_vp columns used,
+// against n_v of vdim) and agree as flat rows of used columns
+template <typename T, int VEC>
+__device__ __forceinline__ void mix_values(float (&v)[VEC], const T* m, float lambda, int g, int d, int vdim, int n_v, int m_v, int m_vp) {
+  float x[VEC];
+  if (m_v == n_v) {
+    VyChunk<T>::load(m + g * vdim + d, x);
+  } else {
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) {
+      const int f = g * n_v + d + e;
+      x[e] = d + e < n_v ? VyT<T>::ld(m + (f / m_v) * m_vp + f % m_v) : 0.f;
+    }
+  }
+#pragma unroll
+  for (int e = 0; e < VEC; ++e) v[e] = (1.f - lambda) * v[e] + lambda * x[e];
 }
 __device__ __forceinline__ float rms_factor(float sum, int n, float eps) {
   const float ms = sum / (float)n + eps, r = rsqrtf(ms);
@@ -187,9 +205,11 @@ struct WindowDecode {
       v8 = *reinterpret_cast<const bf16x8*>(row + a.ov + (int64_t)g * a.vdim + d0);
       if (owner && a.vo) *reinterpret_cast<bf16x8*>(a.vo + (int64_t)b * a.ldvo + (int64_t)g * a.vdim + d0) = v8;
       if (a.vm) {
-        const bf16x8 m8 = *reinterpret_cast<const bf16x8*>(a.vm + (int64_t)b * a.ldm + (int64_t)g * a.vdim + d0);
+        float v[8];
+        VyChunk<bf16>::unpack(v8, v);
+        mix_values(v, a.vm + (int64_t)b * a.ldm, a.lambda, g, d0, a.vdim, a.n_v, a.m_v, a.m_vp);
 #pragma unroll
-        for (int e = 0; e < 8; ++e) v8[e] = (bf16)((1.f - a.lambda) * (float)v8[e] + a.lambda * (float)m8[e]);
+        for (int e = 0; e < 8; ++e) v8[e] = (bf16)v[e];
       }
       if (owner) *reinterpret_cast<bf16x8*>(ring + (int64_t)fresh * W + a.dim + d0) = v8;
     }

@@ -72,7 +72,7 @@ struct QkvArgs {
   RowsArgs r;
   int64_t oq; int h;
   const float* q_norm; const float* k_norm; int n_q, n_k; float eps, lambda;
-  const void* vm; int64_t ldm;
+  const void* vm; int64_t ldm; int n_v, m_v, m_vp;
   void* vo; int64_t ldvo;
 };
 
@@ -172,10 +172,7 @@ __global__ __launch_bounds__(256) void qkv_rows_kernel(QkvArgs a) {
     VyChunk<T>::load(p + r.ov + col, v);
     if (a.vo) VyChunk<T>::store((T*)a.vo + row * a.ldvo + col, v);
     if (a.vm) {
-      float m[VEC];
-      VyChunk<T>::load((const T*)a.vm + row * a.ldm + col, m);
-#pragma unroll
-      for (int e = 0; e < VEC; ++e) v[e] = (1.f - a.lambda) * v[e] + a.lambda * m[e];
+      mix_values(v, (const T*)a.vm + row * a.ldm, a.lambda, g, d, r.vdim, a.n_v, a.m_v, a.m_vp);
       VyChunk<T>::store(p + r.ov + col, v);
     }
     if (keep) VyChunk<T>::store(ring + (int64_t)g * r.r_sh + r.dim + d, v);
@@ -251,7 +248,11 @@ int check_prep(const char* who, const vy_qkv_prep* q, int32_t h, int32_t hk, int
   if (!q) return VY_OK;
   if (!q->q_norm != !q->k_norm || (q->q_norm && (q->n_q < 1 || q->n_k < 1 || q->n_q > h * dim || q->n_k > hk * dim)))
     VY_FAIL(VY_ERR_ARG, "%s: bad query / key norms", who);
-  if ((q->v_mix && (q->ldm % vec || q->ldm < (int64_t)hk * vdim)) || (q->v_out && (q->ldo % vec || q->ldo < (int64_t)hk * vdim)))
+  const int m_v = q->m_v ? q->m_v : q->n_v, m_vp = q->m_v ? q->m_vp : vdim;
+  if (q->v_mix && (q->n_v < 1 || q->n_v > vdim || m_v < 1 || m_v > m_vp || hk * q->n_v % m_v || (m_v == q->n_v && m_vp != vdim) ||
+                   q->ldm < (int64_t)(hk * q->n_v / m_v) * m_vp))
+    VY_FAIL(VY_ERR_ARG, "%s: bad value rows", who);
+  if ((q->v_mix && q->ldm % vec) || (q->v_out && (q->ldo % vec || q->ldo < (int64_t)hk * vdim)))
     VY_FAIL(VY_ERR_ARG, "%s: bad value rows", who);
   return VY_OK;
 }
@@ -310,7 +311,8 @@ extern "C" int vy_qkv_rows(void* p, int64_t ldp, int64_t oq, int64_t ok, int64_t
   a.r = RowsArgs{p, ldp, ok, ov, ring, r_ss, r_sh, store ? R : 1, store ? keep : 0, (const float2*)rope, rope_dims / 2,
                  rope_len > 0 ? rope_len : 1, slots, start, count, B * L, (int)L, hk, dim, vdim, rope_dims > 0, store};
   a.oq = oq; a.h = h; a.q_norm = prep->q_norm; a.k_norm = prep->k_norm; a.n_q = prep->n_q; a.n_k = prep->n_k;
-  a.eps = prep->eps; a.lambda = prep->lambda; a.vm = prep->v_mix; a.ldm = prep->ldm; a.vo = prep->v_out; a.ldvo = prep->ldo;
+  a.eps = prep->eps; a.lambda = prep->lambda; a.vm = prep->v_mix; a.ldm = prep->ldm;
+  a.n_v = prep->n_v; a.m_v = prep->m_v ? prep->m_v : prep->n_v; a.m_vp = prep->m_v ? prep->m_vp : vdim; a.vo = prep->v_out; a.ldvo = prep->ldo;
   hipStream_t st = (hipStream_t)stream;
   const int chunks = (h + hk) * dim / vec;
   // narrow rows: a wave each
@@ -390,7 +392,9 @@ extern "C" int vy_window_decode(void* p, int64_t ldp, int64_t oq, int64_t ok, in
   a.ring = (bf16*)ring; a.r_ss = r_ss; a.r_sh = r_sh; a.R = R; a.keep = keep;
   if (prep) {
     a.q_norm = prep->q_norm; a.k_norm = prep->k_norm; a.n_q = prep->n_q; a.n_k = prep->n_k; a.eps = prep->eps; a.lambda = prep->lambda;
-    a.vm = (const bf16*)prep->v_mix; a.ldm = prep->ldm; a.vo = (bf16*)prep->v_out; a.ldvo = prep->ldo;
+    a.vm = (const bf16*)prep->v_mix; a.ldm = prep->ldm;
+    a.n_v = prep->n_v; a.m_v = prep->m_v ? prep->m_v : prep->n_v; a.m_vp = prep->m_v ? prep->m_vp : vdim;
+    a.vo = (bf16*)prep->v_out; a.ldvo = prep->ldo;
   }
   a.rope = (const float2*)rope; a.half = rope_dims / 2; a.rope_len = rope_len > 0 ? rope_len : 1;
   a.slots = slots; a.start = start; a.out = (bf16*)out; a.ldo = ldo;

@@ -313,7 +313,7 @@ class HybridDecodePlan:
                 self.keep.append(c)
                 if c.prep is not None:
                     q = c.prep
-                    L.prep = C.pointer(_lib.VyQkvPrep(_ptr(q.q_norm), _ptr(q.k_norm), q.n_q, q.n_k, q.eps, q.mix))
+                    L.prep = C.pointer(_lib.VyQkvPrep(_ptr(q.q_norm), _ptr(q.k_norm), q.n_q, q.n_k, q.eps, q.mix, n_v=q.n_v))
                 L.cache, L.c_ss, L.c_sh, L.cap = buf.data_ptr(), buf.stride(0), buf.stride(1), buf.shape[2]
             else:
                 L.mixer, L.state, L.decay_pow = MIX_DECAY, buf.data_ptr(), _ptr(p.decay_pow)

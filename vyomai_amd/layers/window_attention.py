@@ -75,7 +75,7 @@ class WindowAttention(nn.Module):
                 p.prep = ops.QkvPrep(head_vec(self.q_norm.weight, self.heads) if n else None,
                                      head_vec(self.k_norm.weight, self.kv_heads) if n else None, self.heads * self.dim,
                                      self.kv_heads * self.dim, self.q_norm.eps if n else 0.0,
-                                     float(self.value_mix) if self.values == VALUES_MIX else 0.0)
+                                     float(self.value_mix) if self.values == VALUES_MIX else 0.0, self.vdim)
         return Packed.of(self, params, build, "_constants")
 
     def packed(self) -> Packed:
@@ -92,9 +92,9 @@ class WindowAttention(nn.Module):
         table = self.rotary.table(batch.max_keys, rows.device)
         prep = self.constants().prep
         if self.values == VALUES_FIRST:
-            batch.shared_values = rows[:, nk + gk: nk + gk + gv]
+            batch.shared_values = rows[:, nk + gk: nk + gk + gv], self.vdim
         elif self.values == VALUES_MIX:
-            prep = prep._replace(values=batch.shared_values)
+            prep = prep._replace(values=batch.shared_values[0], values_dim=batch.shared_values[1])
         q = rows[:, :nk].unflatten(0, (B, L)).unflatten(2, (H, dim)).transpose(1, 2)
         gate = rows[:, nk + gk + gv: nk + gk + gv + nv].unflatten(0, (B, L)) if self.gate is not None else None
         out = torch.empty((B * L, nv), dtype=rows.dtype, device=rows.device) if out is None else out

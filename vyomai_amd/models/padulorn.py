@@ -78,7 +78,7 @@ class PadulornModel(HybridDecoderModel):
     config_class = PadulornConfig
 
     def __init__(self, config: PadulornConfig) -> None:
-        layers, mixes = [], False      # mixes: a layer whose values later ones mix in has been there
+        layers, mixes = [], 0      # mixes: columns of the values that later layers mix in
         for i, spec in enumerate(config.layers):
             kind, mlp = spec["type"], spec.get("mlp")
             if kind not in MIXERS:
@@ -87,7 +87,10 @@ class PadulornModel(HybridDecoderModel):
                 raise ValueError(f"layer {i}: feed-forward {mlp['kind']!r} is not one of {sorted(FEED_FORWARDS)}")
             values = VALUES_OWN
             if spec["mixer"].get("v_mix"):
-                values, mixes = VALUES_MIX if mixes else VALUES_FIRST, True
+                values, columns = VALUES_MIX if mixes else VALUES_FIRST, spec["mixer"]["kv_heads"] * spec["mixer"]["vdim"]
+                if mixes not in (0, columns):
+                    raise ValueError(f"layer {i}: values of {columns} columns cannot be mixed with {mixes}")
+                mixes = columns
             layers.append(HybridLayer(config.width, MIXERS[kind](config, spec["mixer"], values),
                                       FEED_FORWARDS[mlp["kind"]](config, mlp) if mlp is not None else None, config.norm_eps, "rms",
                                       pre=False, mult=config.residual_mult))

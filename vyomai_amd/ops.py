@@ -814,14 +814,17 @@ def window_rows(p: Tensor, B: int, L: int, hk: int, dim: int, vdim: int, ok: int
 class QkvPrep(NamedTuple):
     """What happens to packed queries, keys and values ahead of attention: RMS norms over the whole query and key projection
     (fp32 factors over the padded heads, zero in the padding; n_q / n_k true columns), and a share `mix` of the values
-    `values` (rows of another layer's) in the values.  `keep_values`: receives the values before mixing."""
+    `values` (rows of another layer's, whose heads have `values_dim` true columns) in the values, whose heads have n_v.
+    `keep_values`: receives the values before mixing."""
     q_norm: Optional[Tensor] = None
     k_norm: Optional[Tensor] = None
     n_q: int = 0
     n_k: int = 0
     eps: float = 0.0
     mix: float = 0.0
+    n_v: int = 0
     values: Optional[Tensor] = None
+    values_dim: int = 0
     keep_values: Optional[Tensor] = None
 
 
@@ -831,11 +834,13 @@ def _prep_args(prep: Optional[QkvPrep], M: int, h: int, hk: int, dim: int, vdim:
     _need_gpu(prep.q_norm, prep.k_norm, prep.values, prep.keep_values)
     for w, n in ((prep.q_norm, h * dim), (prep.k_norm, hk * dim)):
         assert w is None or (w.dtype == torch.float32 and w.numel() == n and w.is_contiguous())
-    for t in (prep.values, prep.keep_values):
-        assert t is None or (t.shape == (M, hk * vdim) and t.dtype == dtype and t.stride(1) == 1)
     v, k = prep.values, prep.keep_values
+    for t in (v, k):
+        assert t is None or (t.shape[0] == M and t.dtype == dtype and t.stride(1) == 1)
+    assert k is None or k.shape[1] == hk * vdim
+    assert v is None or v.shape[1] * prep.values_dim == hk * prep.n_v * up8(prep.values_dim)
     return _lib.VyQkvPrep(_ptr(prep.q_norm), _ptr(prep.k_norm), int(prep.n_q), int(prep.n_k), float(prep.eps), float(prep.mix), _ptr(v),
-                          v.stride(0) if v is not None else 0, _ptr(k), k.stride(0) if k is not None else 0)
+                          v.stride(0) if v is not None else 0, int(prep.n_v), int(prep.values_dim), up8(prep.values_dim), _ptr(k), k.stride(0) if k is not None else 0)
 
 
 def qkv_rows(p: Tensor, B: int, L: int, h: int, hk: int, dim: int, vdim: int, oq: int, ok: int, ov: int, prep: QkvPrep, *,
