@@ -8,6 +8,11 @@ int vy_residual_norm_ex(float* x, int64_t ldx, const void* y, int64_t ldy, const
                         int64_t V, int32_t* err, float table_scale, const vy_routed_rows* routed, const float* w_post,
                         float eps_post, const float* w_pre, float eps_pre, void* h, int64_t ldh, int64_t M, int64_t N, int64_t NP,
                         int rms, int* advance, const int* slots, int n_adv, int dtype, void* stream);
+int vy_residual_route(float* x, int64_t ldx, const void* y, int64_t ldy, const float* w_post, const float* w_pre, float eps, void* h,
+                      int64_t ldh, int64_t M, int64_t N, int64_t NP, int rms, const vy_moe* d, int32_t* ids, float* weight, int dtype,
+                      void* stream);
+int vy_moe_few(const vy_moe* d, const void* h, int64_t ldh, int64_t M, const int32_t* ids, void* rows, int64_t ldr, void* ws,
+               int64_t ws_bytes, int dtype, void* stream);
 int vy_parallel_decode(const vy_hybrid_plan* p, const vy_hybrid_layer* L, const void* h, void* in, void* ao, void* y, void* erows,
                        int32_t* eids, float* ew, void* moe_ws, int64_t moe_ws_bytes, const int32_t* slots, const int32_t* lengths,
                        int64_t max_keys, void* mix_ws, int64_t mix_ws_bytes, void* stream);
@@ -179,7 +184,7 @@ extern "C" int vy_hybrid_decoder_step(const vy_hybrid_plan* p, const int64_t* id
         if ((rc = vy_head_norm_gate(o, nv, gate, L.n_in, ao, na, B, L.heads, L.mix_n, L.vdim, p->eps, p->dtype, stream))) return rc;
       } else if ((rc = vy_rmsnorm_gate(o, nv, L.mix_norm, gate, L.n_in, ao, na, B, L.mix_n, nv, p->eps, p->dtype, stream))) return rc;
     }
-    const vy_routed_rows rows{erows, dp, epos, ew, L.moe ? L.moe->top : 0};
+    vy_routed_rows rows{erows, dp, epos, ew, L.moe ? L.moe->top : 0};
     const vy_routed_rows* routed = L.moe ? &rows : nullptr;
     auto experts = [&]() {
       return L.moe ? vy_moe_fwd(L.moe, h, dp, B, nullptr, 1, erows, dp, eids, epos, ew, ews, s.moe_ws, p->dtype, stream) : VY_OK;
@@ -197,12 +202,27 @@ extern "C" int vy_hybrid_decoder_step(const vy_hybrid_plan* p, const int64_t* id
       if ((rc = norm(y, nullptr, L.norm1b, next, last))) return rc;
       continue;
     }
-    if ((rc = norm(y, nullptr, L.norm1b, L.norm2, false))) return rc;
+    // few tokens: the choice of experts comes with the residual sum
+    bool chosen = false;
+    if (L.moe) {
+      rc = vy_moe_few(L.moe, nullptr, 0, B, nullptr, nullptr, 0, nullptr, 0, p->dtype, stream);
+      if (rc == VY_OK)
+        rc = vy_residual_route(x, dp, y, dp, L.norm1b, L.norm2, p->eps, h, dp, B, p->d, dp, p->rms, L.moe, eids, ew, p->dtype, stream);
+      if (rc && rc != VY_ERR_UNSUPPORTED) return rc;
+      chosen = rc == VY_OK;
+    }
+    if (!chosen && (rc = norm(y, nullptr, L.norm1b, L.norm2, false))) return rc;
     if (L.ff) {
       if ((rc = gated(p, L, h, gu, act, stream))) return rc;
       if ((rc = product(p, act, L.w_down, y, dp, dp, L.ff, stream))) return rc;
     }
-    if ((rc = experts())) return rc;
+    if (chosen) {
+      rows.pos = nullptr;
+      rc = vy_moe_few(L.moe, h, dp, B, eids, erows, dp, ews, s.moe_ws, p->dtype, stream);
+    } else {
+      rc = experts();
+    }
+    if (rc) return rc;
     if ((rc = norm(L.ff ? y : nullptr, routed, L.norm2b, next, last))) return rc;
   }
   return product(p, h, p->head, logits, ldv, p->vocab, dp, stream);

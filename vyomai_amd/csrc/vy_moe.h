@@ -1,5 +1,5 @@
 // Mixture of experts, the device code of decode steps: the choice of a token's experts and the weight-streaming products of few
-// tokens.  Used by vy_moe.hip (launches of their own) and vy_parallel.hip (one launch with other work of the same step).
+// tokens.  Used by vy_moe.hip (launches of their own), vy_parallel.hip and vy_route.hip (one launch with other work of the same step).
 #pragma once
 #include "vy_rows.h"
 #include <float.h>
@@ -25,9 +25,11 @@ __device__ __forceinline__ unsigned ordered(float z) {
 }
 
 // one wave per token; lane holds experts lane + 64 i.  Both scores are monotone: the choice is made on the logits (of groups only
-// if a group's score is its best expert's).  gmax: 2 * 64 EPL floats of LDS of the wave's own
+// if a group's score is its best expert's).  logits: the token's, in global memory or
+// LDS; gmax: 2 * 64 EPL floats of LDS of the wave's own
 template <int EPL>
-__device__ __forceinline__ void choose_one(const ChooseArgs& a, int64_t m, int lane, float* gmax, int (&my_id), float (&my_w)) {
+__device__ __forceinline__ void choose_one(const ChooseArgs& a, int64_t m, const float* logits, int lane, float* gmax, int (&my_id),
+                                           float (&my_w)) {
   my_id = -1;
   my_w = 0.f;
   const int b = a.count ? (int)(m / a.L) : 0;
@@ -36,7 +38,7 @@ __device__ __forceinline__ void choose_one(const ChooseArgs& a, int64_t m, int l
 #pragma unroll
   for (int i = 0; i < EPL; ++i) {
     const int e = lane + 64 * i;
-    z[i] = e < a.E ? a.logits[m * a.E + e] : -INFINITY;
+    z[i] = e < a.E ? logits[e] : -INFINITY;
     zmax = fmaxf(zmax, z[i]);
   }
   float sum = 1.f;

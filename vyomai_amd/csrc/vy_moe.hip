@@ -84,7 +84,7 @@ __global__ __launch_bounds__(64 * NW) void choose_kernel(ChooseArgs a, int tpw) 
     if (m >= a.M) break;
     int id;
     float w;
-    choose_one<EPL>(a, m, lane, groups[wave], id, w);
+    choose_one<EPL>(a, m, a.logits + m * a.E, lane, groups[wave], id, w);
     if (lane < a.top) {
       a.ids[m * a.top + lane] = id;
       a.weight[m * a.top + lane] = w;
@@ -383,6 +383,10 @@ __global__ __launch_bounds__(256) void expert_rows_kernel(ExpertRows a) {
   __shared__ ExpertLds<NT> lds;
   expert_rows<KIND, NT>(a, lds, blockIdx.x, blockIdx.y);
 }
+template <int KIND>
+__global__ __launch_bounds__(256) void expert_rows1_kernel(ExpertRows a) {   // a single token
+  expert_rows1<KIND>(a, blockIdx.x, blockIdx.y);
+}
 
 // ---- activation of packed [gate | up] rows ----------------------------------------------------
 template <typename T>
@@ -447,6 +451,25 @@ int check_moe(const char* who, const vy_moe* d, int dtype) {
   return VY_OK;
 }
 
+// the experts of few tokens whose choice is made; rows by choice
+void few_experts(const vy_moe* d, const void* h, int64_t ldh, int64_t M, const int* ids, void* act, void* rows, int64_t ldr, hipStream_t st) {
+  const bool gated = d->act == VY_MOE_CLAMPED;
+  const int K = d->width, n = (int)(M * d->top);
+  const unsigned active = (unsigned)(n < d->experts ? n : d->experts);
+  ExpertRows g{(const bf16*)h, ldh, ids, n, d->top, (const bf16*)d->w_gu, gated ? 2 * d->ff : d->ff, K, (bf16*)act, d->ff, d->limit, d->alpha};
+  ExpertRows o{(const bf16*)act, d->ff, ids, n, d->top, (const bf16*)d->w_down, K, d->ff, (bf16*)rows, ldr, 0.f, 0.f};
+  auto go = [&](auto kind, ExpertRows& a) {
+    constexpr int KIND = decltype(kind)::value;
+    const dim3 block(256);
+    if (M == 1) hipLaunchKernelGGL((expert_rows1_kernel<KIND>), dim3((unsigned)vy_cdiv(a.N, 8), active), block, 0, st, a);
+    else if (vy_cdiv(a.N, 16) * active > 1536) hipLaunchKernelGGL((expert_rows_kernel<KIND, 2>), dim3((unsigned)vy_cdiv(a.N, 32), active), block, 0, st, a);
+    else hipLaunchKernelGGL((expert_rows_kernel<KIND, 1>), dim3((unsigned)vy_cdiv(a.N, 16), active), block, 0, st, a);
+  };
+  if (gated) go(std::integral_constant<int, GATE_UP>{}, g);
+  else go(std::integral_constant<int, UP>{}, g);
+  go(std::integral_constant<int, DOWN>{}, o);
+}
+
 __global__ void zero_kernel(int* p, int n) {
   const int i = blockIdx.x * 256 + threadIdx.x;
   if (i < n) p[i] = 0;
@@ -500,17 +523,7 @@ extern "C" int vy_moe_fwd(const vy_moe* d, const void* h, int64_t ldh, int64_t M
   else CHOOSE(4, 16, 2);
 #undef CHOOSE
   if (small) {
-    const unsigned active = (unsigned)(n < E ? n : E);
-    ExpertRows g{(const bf16*)h, ldh, ids, (int)n, d->top, (const bf16*)d->w_gu, up_rows, K, (bf16*)p.act, d->ff, d->limit, d->alpha};
-    ExpertRows o{(const bf16*)p.act, d->ff, ids, (int)n, d->top, (const bf16*)d->w_down, K, d->ff, (bf16*)rows, ldr, 0.f, 0.f};
-    auto go = [&](auto kind, ExpertRows& a) {
-      constexpr int KIND = decltype(kind)::value;
-      if (vy_cdiv(a.N, 16) * active > 1536) hipLaunchKernelGGL((expert_rows_kernel<KIND, 2>), dim3((unsigned)vy_cdiv(a.N, 32), active), block, 0, st, a);
-      else hipLaunchKernelGGL((expert_rows_kernel<KIND, 1>), dim3((unsigned)vy_cdiv(a.N, 16), active), block, 0, st, a);
-    };
-    if (gated) go(std::integral_constant<int, GATE_UP>{}, g);
-    else go(std::integral_constant<int, UP>{}, g);
-    go(std::integral_constant<int, DOWN>{}, o);
+    few_experts(d, h, ldh, M, ids, p.act, rows, ldr, st);
     VY_CHECK_LAUNCH(who);
     return VY_OK;
   }
@@ -530,6 +543,21 @@ extern "C" int vy_moe_fwd(const vy_moe* d, const void* h, int64_t ldh, int64_t M
     else hipLaunchKernelGGL((grouped_gemm_f32_kernel<UP>), ggrid, block, 0, st, g);
     hipLaunchKernelGGL((grouped_gemm_f32_kernel<DOWN>), ogrid, block, 0, st, o);
   }
+  VY_CHECK_LAUNCH(who);
+  return VY_OK;
+}
+
+// internal (vy_hybrid.hip): the experts alone, behind a choice made elsewhere (no padding tokens); rows by choice.
+// VY_ERR_UNSUPPORTED: too many tokens for that
+int vy_moe_few(const vy_moe* d, const void* h, int64_t ldh, int64_t M, const int32_t* ids, void* rows, int64_t ldr, void* ws,
+               int64_t ws_bytes, int dtype, void* stream) {
+  const char* who = "vy_moe_fwd";
+  if (int rc = check_moe(who, d, dtype)) return rc;
+  if (!few(d, M, dtype)) return VY_ERR_UNSUPPORTED;
+  if (!h) return VY_OK;   // (asked whether it would)
+  Parts p;
+  if (!ids || !rows || !ws || ws_bytes < lay_out(d, M, dtype, (char*)ws, p)) VY_FAIL(VY_ERR_ARG, "%s: workspace too small", who);
+  few_experts(d, h, ldh, M, ids, p.act, rows, ldr, (hipStream_t)stream);
   VY_CHECK_LAUNCH(who);
   return VY_OK;
 }

@@ -56,9 +56,10 @@ __global__ __launch_bounds__(256) void parallel_mix_kernel(MixArgs a) {
     int e;
     float w;
     float* lds = reinterpret_cast<float*>(smem) + wave * 512;
-    if (a.choose.E <= 64) choose_one<1>(a.choose, m, lane, lds, e, w);
-    else if (a.choose.E <= 128) choose_one<2>(a.choose, m, lane, lds, e, w);
-    else choose_one<4>(a.choose, m, lane, lds, e, w);
+    const float* z = a.choose.logits + m * a.choose.E;
+    if (a.choose.E <= 64) choose_one<1>(a.choose, m, z, lane, lds, e, w);
+    else if (a.choose.E <= 128) choose_one<2>(a.choose, m, z, lane, lds, e, w);
+    else choose_one<4>(a.choose, m, z, lane, lds, e, w);
     if (lane < a.choose.top) {
       a.choose.ids[m * a.choose.top + lane] = e;
       a.choose.weight[m * a.choose.top + lane] = w;
