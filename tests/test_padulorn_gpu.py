@@ -687,6 +687,99 @@ def test_decode_of_larger_batches(batch):
         compare(logits[some], torch.stack([reference("plain", seqs[b])[0][-1] for b in some]), dt)
 
 
+# ---- the parts in other arrangements --------------------------------------------------------------
+@pytest.mark.parametrize("dt", DT)
+def test_parts_fit_other_layers(dt):
+    """Retention and normed, mixed attention in parallel layers and between norms on both sides (layer norms too), with gate and
+    sink, plain and gated experts: against the oracle's pieces."""
+    from vyomai_amd.layers.ffn import GatedFeedForward, MixtureFeedForward
+    from vyomai_amd.layers.retention import Retention
+    from vyomai_amd.layers.window_attention import VALUES_FIRST, VALUES_MIX, WindowAttention
+    from vyomai_amd.models.hybrid import HybridDecoderModel, HybridLayer, ParallelLayer
+    from oracle import gisitar_oracle as GO
+    from oracle import rivudra_oracle as RO
+    width, vocab, eps = 40, 50, 1e-5
+    att = P.attention(4, 2, 16, 8, 11, 3, rot=8, scaling=P.yarn())["mixer"]
+    ret = P.retention(2, 24, 16, rot=10)["mixer"]
+    plain, gated = P.moe(6, 2, 16, 3, 2), {"router": {"experts": 8, "top": 3, "scale": 1.5, "groups": {"count": 4, "keep": 2}},
+                                           "expert": {"ff": 24, "limit": 0.8}}
+
+    def window(values, gate=False):
+        return WindowAttention(width, 4, 2, 16, 8, att["scale"], 11, att["rot"]["base"], 8, sink=False, gate=gate, keep_first=3,
+                               rot_scaling=att["rot"]["scaling"], qk_norm_eps=eps, values=values)
+
+    def retain():
+        return Retention(width, 2, 24, 16, ret["decay"], eps, ret["rot"]["base"], 10)
+
+    def experts(cfg, **kw):
+        r = cfg["router"]
+        return MixtureFeedForward(width, r["experts"], r["top"], cfg["expert"]["ff"], groups=r["groups"]["count"], keep=r["groups"]["keep"], **kw)
+
+    def plain_experts(shared=None):
+        return experts(plain, act="gelu", score="sigmoid", group_best=2, normalize=False, shared=shared)
+    layers = [ParallelLayer(width, window(VALUES_FIRST, gate=True), plain_experts(), eps),
+              HybridLayer(width, retain(), experts(gated, limit=0.8, scale=1.5), eps, "rms", mult=0.5),
+              ParallelLayer(width, retain(), GatedFeedForward(width, 32), eps),
+              HybridLayer(width, window(VALUES_MIX), plain_experts(GatedFeedForward(width, 24)), eps, "rms", pre=False),
+              HybridLayer(width, retain(), None, eps, "rms", pre=False, mult=2.0)]
+    m = HybridDecoderModel(None, width, vocab, layers, eps, "rms", embed_scale=2.0, logit_scale=0.7).to(dt).cuda().eval()
+    w = {}
+    with torch.no_grad():
+        for i, (n, p) in enumerate(m.named_parameters()):
+            if p.dim() > 1:
+                t = rnd(*p.shape, seed=i, scale=2.0 if "router" in n else 1.0) / p.shape[-1] ** 0.5
+            else:
+                t = 1 + 0.2 * rnd(*p.shape, seed=i) if p.dim() else torch.tensor(0.375)
+            t = t.to(torch.bfloat16).double()
+            p.copy_(t)
+            w[n[:-7] if n.endswith(".weight") else n] = t
+
+    def sub(prefix, names):
+        return {short: w[f"{prefix}.{long}"] for short, long in names.items() if f"{prefix}.{long}" in w}
+
+    first = []
+
+    def mixer(i, h):
+        p = sub(f"layers.{i}.mixer", {"q": "query", "k": "key", "v": "value", "g": "gate", "o": "out", "q.norm": "q_norm", "k.norm": "k_norm",
+                                      "vmix": "value_mix"})
+        if m.layers[i].mixer.kind == "decay":
+            return O.retention(h, p, ret, eps)
+        if not first:                     # (gated: the heads before the output product)
+            heads, own = O.attention(h, {**p, "o": torch.eye(32, dtype=torch.float64)}, att, eps)
+            first.append(own)
+            return (heads * O.sigmoid(h @ p["g"].T)) @ p["o"].T
+        return O.attention(h, p, att, eps, first[0])[0]
+
+    def feed_forward(i, h):
+        p, mlp = f"layers.{i}.mlp", m.layers[i].mlp
+        dense = {n: n for n in ("gate", "up", "down")}
+        if i == 2:
+            return GO.gated_mlp(h, sub(p, dense))
+        q = {"router": w[p + ".router"]}
+        for e in range(mlp.experts):
+            q.update({f"e{e}.{n}": w[f"{p}.{n}"][e] for n in dense if f"{p}.{n}" in w})
+        if i == 1:
+            return RO.mixture(h, q, gated)
+        y = O.mixture(h, q, plain)
+        return y + GO.gated_mlp(h, sub(p + ".shared", dense)) if mlp.shared is not None else y
+
+    ids = torch.randint(0, vocab, (70,), generator=torch.Generator().manual_seed(1)).tolist()
+    x = 2.0 * w["word_embeddings"][ids]
+    for i, l in enumerate(m.layers):
+        def norm(t, name):
+            return O.rms_norm(t, w[f"layers.{i}.{name}"], eps)
+        if l.form == "parallel":
+            h = norm(x, "norm1")
+            x = x + mixer(i, h) + feed_forward(i, h)
+        else:
+            x = x + l.mult * norm(mixer(i, norm(x, "norm1") if l.pre else x), "norm1b")
+            if l.mlp is not None:
+                x = x + l.mult * norm(feed_forward(i, norm(x, "norm2") if l.pre else x), "norm2b")
+    want = 0.7 * O.rms_norm(x, w["final_norm"], eps) @ w["head"].T
+    for cuts in ([70], [1] * 70, [2, 1, 30, 1, 36]):
+        compare(run(m, ids, cuts), want, dt)
+
+
 # ---- entry points ---------------------------------------------------------------------------------
 @pytest.mark.parametrize("name", list(P.CONFIGS))
 def test_greedy_generation(name):

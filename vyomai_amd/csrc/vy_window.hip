@@ -316,11 +316,12 @@ extern "C" int vy_qkv_rows(void* p, int64_t ldp, int64_t oq, int64_t ok, int64_t
   hipStream_t st = (hipStream_t)stream;
   const int chunks = (h + hk) * dim / vec;
   // narrow rows: a wave each
-  const bool narrow = chunks <= 64 * 4 && B * L >= 1024;
+  const bool narrow = chunks <= 64 * 8 && B * L >= 1024;
   const dim3 grid((unsigned)(narrow ? vy_cdiv(B * L, 4) : B * L)), block(256);
 #define QKV_GO(T)                                                                              \
   do {                                                                                         \
-    if (narrow) hipLaunchKernelGGL((qkv_rows_kernel<T, 1, 4>), grid, block, 0, st, a);         \
+    if (narrow && chunks <= 256) hipLaunchKernelGGL((qkv_rows_kernel<T, 1, 4>), grid, block, 0, st, a); \
+    else if (narrow) hipLaunchKernelGGL((qkv_rows_kernel<T, 1, 8>), grid, block, 0, st, a);    \
     else if (chunks <= 512) hipLaunchKernelGGL((qkv_rows_kernel<T, 4, 2>), grid, block, 0, st, a); \
     else hipLaunchKernelGGL((qkv_rows_kernel<T, 4, 4>), grid, block, 0, st, a);                \
   } while (0)
