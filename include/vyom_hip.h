@@ -34,7 +34,9 @@ typedef enum {
 } vy_status;
 
 typedef enum { VY_ACT_NONE = 0, VY_ACT_GELU_ERF = 1, VY_ACT_GELU_TANH = 2,
-               VY_ACT_SILU = 3 /* gated products only (vy_gated_act_fwd, the decode steps) */ } vy_act;
+               VY_ACT_SILU = 3, /* gated products only (vy_gated_act_fwd, the decode steps) */
+               VY_ACT_RELU2 = 4, /* max(x, 0)^2; products only */
+               VY_ACT_SOFTCAP = 5 /* vy_linear_softcap_fwd */ } vy_act;
 /* OR-ed into `act` of vy_linear_fwd / vy_linear_dgrad (training): the tensor saved for backward is act'(x W^T + b)
  * instead of the pre-activation -- the forward epilogue has Phi and the Gaussian of the erf GELU at hand anyway, and
  * the dgrad epilogue (dX = (dY W) * act') becomes one multiply per element instead of an erf + exp evaluation.
@@ -76,6 +78,9 @@ int vy_workspace_set(void* stream, void* ws, int64_t bytes);
 int vy_linear_fwd(const void* x, int64_t ldx, const void* w, int64_t ldw, const void* bias,
                   const void* residual, int64_t ldr, void* y, int64_t ldy, void* pre_out,
                   int64_t M, int64_t N, int64_t K, int act, int dtype, void* stream);
+/* vy_linear_softcap_fwd: Y = cap * tanh(X . W^T / cap), a vocabulary product whose logits stay within +-cap. */
+int vy_linear_softcap_fwd(const void* x, int64_t ldx, const void* w, int64_t ldw, void* y, int64_t ldy, int64_t M, int64_t N,
+                          int64_t K, float cap, int dtype, void* stream);
 
 /* ------------------------------------------------------------------------------------------
  * vy_qkv_rope_fwd: fused Q/K/V projection + bias + rotary embedding + head split.
@@ -175,6 +180,8 @@ int vy_clamped_act_fwd(const void* gate_up, int64_t ldg, void* out, int64_t ldo,
  *   x = table_scale * table[ids].
  * vy_latent_norm: p = packed rows [query latent (npq) | key/value latent (npc) | ...]: q_out = RMSNorm(latent) * w_q,
  *   c_out (nullable) = RMSNorm(latent) * w_c, also written to cache[slot][start + l] (strides c_ss / c_st, cap rows per slot).
+ *   w_q NULL: the first npq columns are no latent and left alone.  ring != 0: the cap rows are a ring, position p lives in row
+ *   p % cap, and only the last cap tokens are written.
  * vy_rmsnorm_gate: y = RMSNorm(x) * w * sigmoid(gate).
  * ------------------------------------------------------------------------------------------ */
 int vy_residual_norm(float* x, int64_t ldx, const void* y, int64_t ldy, const void* table, int64_t ldt, const int64_t* ids,
@@ -190,13 +197,14 @@ int vy_residual_norm_routed(float* x, int64_t ldx, const void* y, int64_t ldy, c
                             int64_t M, int64_t N, int64_t NP, int rms, int dtype, void* stream);
 int vy_latent_norm(const void* p, int64_t ldp, const float* w_q, void* q_out, int64_t ldq, int32_t nq, int32_t npq,
                    const float* w_c, void* c_out, int64_t ldc, int32_t nc, int32_t npc, void* cache, int64_t c_ss,
-                   int64_t c_st, int32_t cap, const int32_t* slots, const int32_t* start, const int32_t* count, int64_t B,
+                   int64_t c_st, int32_t cap, int ring, const int32_t* slots, const int32_t* start, const int32_t* count, int64_t B,
                    int64_t L, float eps, int dtype, void* stream);
 int vy_rmsnorm_gate(const void* x, int64_t ldx, const float* w, const void* gate, int64_t ldg, void* y, int64_t ldy, int64_t M,
                     int64_t N, int64_t NP, float eps, int dtype, void* stream);
-/* vy_head_norm_gate: every head of a row by itself, without a weight: y = x / rms(x) * silu(gate); heads of NP columns, N used. */
-int vy_head_norm_gate(const void* x, int64_t ldx, const void* gate, int64_t ldg, void* y, int64_t ldy, int64_t M, int32_t heads,
-                      int64_t N, int64_t NP, float eps, int dtype, void* stream);
+/* vy_head_norm_gate: every head of a row by itself: y = x / rms(x) * w * silu(gate); heads of NP columns, N used; w (nullable): NP
+ * factors shared by the heads, zero in the padding; gate nullable. */
+int vy_head_norm_gate(const void* x, int64_t ldx, const float* w, const void* gate, int64_t ldg, void* y, int64_t ldy, int64_t M,
+                      int32_t heads, int64_t N, int64_t NP, float eps, int dtype, void* stream);
 
 /* vy_attn_fwd_ex: causal attention whose values may have a width of their own (dv), with a start position per sequence
  * (key j is visible to query i of sequence b iff j <= start[slot] + i; start NULL: 0) and an optional output gate:
@@ -207,11 +215,12 @@ int vy_head_norm_gate(const void* x, int64_t ldx, const void* gate, int64_t ldg,
  *   sink       one more term exp(0) in every softmax denominator, without a value;
  *   rope       rotary positions of the queries: (cos, sin) pairs [rope_len][rope_dims / 2], fp32; columns 2c and 2c + 1 of the
  *              first rope_dims turn by the angle of position start[slot] + i (the keys are rotated already);
- *   kv_by_slot k and v are indexed by slots[b] instead of b (row-wise kernel). */
+ *   kv_by_slot k and v are indexed by slots[b] instead of b (row-wise kernel);
+ *   gate_heads the gate is one number per head, gate rows [h]. */
 typedef struct vy_attn_window {
   int32_t window, sink, kv_by_slot, start_cap;
   const float* rope; int32_t rope_dims, rope_len;
-  int32_t keep;
+  int32_t keep, gate_heads;
 } vy_attn_window;
 int vy_attn_fwd_ex(const void* q, int64_t q_sb, int64_t q_sh, int64_t q_sl, const void* k, int64_t k_sb, int64_t k_sh,
                    int64_t k_sl, const void* v, int64_t v_sb, int64_t v_sh, int64_t v_sl, void* out, int64_t o_sb,
@@ -247,15 +256,21 @@ int vy_moe_fwd(const vy_moe* d, const void* h, int64_t ldh, int64_t M, const int
  * is longer than R.  Packed projection rows p (stride ldp): queries at column oq ([h][dim]), keys ok ([hk][dim]), values ov
  * ([hk][vdim]), output gate og ([h][vdim], og < 0: none).  rope / rope_dims / rope_len as in vy_attn_window.
  *
+ * (vdim 0: rows of one part, the keys', for vy_window_rows and vy_window_context.)
+ *
  * vy_window_rows: rotate != 0: rotary positions on the new keys, in place; store != 0: those of the count[b] new rows of every
  *   sequence that its ring still holds behind them, to the ring.
  * vy_window_context: ctx [B][hk][S][dim + vdim] = min(start, past) rows of the ring in order of position (the kept ones, then the
  *   last of the others), then the L new rows (rotated already), then zeros: what vy_attn_fwd_ex takes with start_cap = past.
  * vy_qkv_rows: what a vy_qkv_prep asks for, in place on the packed rows: RMS norms of the whole query and of the whole key
- *   projection, rotary positions on both, values mixed; store != 0: as vy_window_rows.
+ *   projection or of groups of their columns, rotary positions on both, a temperature on the queries, values mixed; store != 0:
+ *   as vy_window_rows.
  * vy_window_decode: one new token per sequence (L = 1): its key and value to the ring, then attention of its queries over the
- *   ring with sink and gate, prep (nullable) as in vy_qkv_rows; max_keys >= every start + 1; ws: vy_window_decode_ws_bytes(...).
- *   scale > 0. */
+ *   ring with sink and gate, prep (nullable) as in vy_qkv_rows; diff (nullable): differential attention, without sink, gate and
+ *   rope; max_keys >= every start + 1; ws: vy_window_decode_ws_bytes(...).  scale > 0.
+ * vy_diff_attn_fwd: causal differential attention of packed queries (B sequences of L rows, row stride ldq, heads of dim columns)
+ *   over keys and values that lie in a ring which has not wrapped (row = position): the new tokens' rows are in it already.
+ *   out rows [h][vdim]; rows behind count[b] hold finite numbers. */
 typedef struct vy_qkv_prep {
   const float *q_norm, *k_norm;     /* [h][dim], [hk][dim] factors (NULL: no norms), zero in padded columns */
   int32_t n_q, n_k;                 /* columns the norms divide by */
@@ -263,7 +278,17 @@ typedef struct vy_qkv_prep {
   const void* v_mix; int64_t ldm;   /* nullable: v <- (1 - lambda) v + lambda v_mix, both as flat rows of their used columns */
   int32_t n_v, m_v, m_vp;           /* used columns of a value head; of v_mix's heads, and those with their padding (m_v 0: as v's) */
   void* v_out; int64_t ldo;         /* nullable: receives the values as they were before mixing */
+  int32_t group;                    /* 0: norms over whole projections; else over every `group` neighbouring columns by themselves
+                                       (n_q = n_k of them used; dim a multiple of group); no v_mix / v_out then */
+  int32_t temp_every; float temp_coef;  /* temp_every > 0 (with group): the query of position p times
+                                       1 + temp_coef * ln(floor((p + 1) / temp_every) + 1) */
 } vy_qkv_prep;
+/* Differential attention: a head's dim columns of queries and keys are [map 1 | map 2], two attentions over the same values.  With
+ * their outputs a1, a2: o = a1 - lambda a2, out = o / rms(o) * out_scale over a head's n_v used value columns. */
+typedef struct vy_diff {
+  float lambda, out_scale, eps;
+  int32_t n_v;
+} vy_diff;
 int vy_qkv_rows(void* p, int64_t ldp, int64_t oq, int64_t ok, int64_t ov, const vy_qkv_prep* prep, void* ring, int64_t r_ss,
                 int64_t r_sh, int32_t R, int32_t keep, const float* rope, int32_t rope_dims, int32_t rope_len, int store,
                 const int32_t* slots, const int32_t* start, const int32_t* count, int64_t B, int64_t L, int32_t h, int32_t hk,
@@ -275,23 +300,28 @@ int vy_window_rows(void* p, int64_t ldp, int64_t ok, int64_t ov, void* ring, int
 int vy_window_context(const void* p, int64_t ldp, int64_t ok, int64_t ov, const void* ring, int64_t r_ss, int64_t r_sh,
                       int32_t R, int32_t keep, void* ctx, int32_t S, int32_t past, const int32_t* slots, const int32_t* start, int64_t B,
                       int64_t L, int32_t hk, int32_t dim, int32_t vdim, int dtype, void* stream);
-int64_t vy_window_decode_ws_bytes(int32_t B, int32_t h, int32_t hk, int32_t vdim, int32_t R);
+int64_t vy_window_decode_ws_bytes(int32_t B, int32_t h, int32_t hk, int32_t vdim, int32_t R, int diff);
 int vy_window_decode(void* p, int64_t ldp, int64_t oq, int64_t ok, int64_t ov, int64_t og, void* ring, int64_t r_ss, int64_t r_sh,
                      int32_t R, int32_t keep, const float* rope, int32_t rope_dims, int32_t rope_len, const vy_qkv_prep* prep,
-                     const int32_t* slots, const int32_t* start, int64_t max_keys, void* out, int64_t ldo, int64_t B, int32_t h, int32_t hk,
+                     const vy_diff* diff, const int32_t* slots, const int32_t* start, int64_t max_keys, void* out, int64_t ldo, int64_t B, int32_t h, int32_t hk,
                      int32_t dim, int32_t vdim, float scale, int32_t sink, void* ws, int64_t ws_bytes, int dtype, void* stream);
+
+int vy_diff_attn_fwd(const void* q, int64_t ldq, const void* ring, int64_t r_ss, int64_t r_sh, int32_t R, const vy_diff* diff,
+                     const int32_t* slots, const int32_t* start, const int32_t* count, void* out, int64_t ldo, int64_t B, int64_t L,
+                     int32_t h, int32_t hk, int32_t dim, int32_t vdim, float scale, int dtype, void* stream);
 
 /* vy_latent_decode: one query token per sequence against a cache of latents c (one row of R per token, shared by all
  * heads).  Keys and values are never expanded:  q~_h = Wuk_h^T q_h,  s_j = scale * q~_h . c_j over j <= start[slot],
  * u_h = sum_j softmax(s)_j c_j,  out_h = (Wuv_h u_h) * sigmoid(gate_h)  (gate nullable).
  *   q [B][h*dh] (row stride ldq), wukt [h][R][dh] (= Wuk_h transposed), wuv [h][dv][R], out / gate rows [h*dv];
  *   cache rows cache[slot][j] with strides c_ss / c_st; max_keys >= every start + 1 (sizes the grid, cap rows per slot);
- *   ws: vy_latent_decode_ws_bytes(...) of scratch.  dh, dv, R multiples of 8, R <= 1024. */
+ *   ring > 0: a slot's rows are a ring of that many (vy_latent_norm), all of whose tokens are seen; gate_heads != 0: gate rows [h],
+ *   one number per head.  ws: vy_latent_decode_ws_bytes(...) of scratch.  dh, dv, R multiples of 8, R <= 1024. */
 int64_t vy_latent_decode_ws_bytes(int32_t B, int32_t h, int32_t R);
 int vy_latent_decode(const void* q, int64_t ldq, const void* wukt, const void* wuv, const void* cache, int64_t c_ss,
                      int64_t c_st, const int32_t* slots, const int32_t* start, int64_t max_keys, void* out, int64_t ldo,
-                     const void* gate, int64_t ldg, int32_t B, int32_t h, int32_t dh, int32_t dv, int32_t R, float scale,
-                     void* ws, int64_t ws_bytes, int dtype, void* stream);
+                     const void* gate, int64_t ldg, int gate_heads, int32_t ring, int32_t B, int32_t h, int32_t dh, int32_t dv,
+                     int32_t R, float scale, void* ws, int64_t ws_bytes, int dtype, void* stream);
 
 /* vy_decay_attn: linear attention with a per-head decay on packed rows p (row stride ldp; q / k / v of head a at columns
  * oq + a*dk, ok + a*dk, ov + a*dv):  S_t = decay_a S_(t-1) + k_t v_t^T,  o_t = S_t^T q_t  with q, k, v = silu of the
@@ -306,6 +336,17 @@ int vy_decay_attn(const void* p, int64_t ldp, int64_t oq, int64_t ok, int64_t ov
                   const int32_t* slots, const int32_t* start, const int32_t* count, void* out, int64_t ldo, int64_t B,
                   int64_t L, int32_t h, int32_t dk, int32_t dv, int silu, const float* rope, int32_t rope_dims, int32_t rope_len,
                   float k_scale, void* ws, int64_t ws_bytes, int dtype, void* stream);
+
+/* vy_gated_attn: linear attention with a forget gate per key channel that also decides what is written, on packed rows p (q, gate
+ * logits z and v of head a at columns oq + a*dk, of + a*dk, ov + a*dv):
+ *   f = lower + (1 - lower) * sigmoid(z + bias),   S_t = diag(f_t) S_(t-1) + (1 - f_t) v_t^T,   o_t = S_t^T q_t
+ * with q = silu of its projection (silu = 0: taken as it is); bias (nullable) and lower fp32 [h][dk] (lower 1 in padded channels).
+ * Everything else as in vy_decay_attn; ws: vy_gated_attn_ws_bytes(...). */
+int64_t vy_gated_attn_ws_bytes(int64_t B, int64_t L, int32_t h, int32_t dk, int32_t dv, int dtype);
+int vy_gated_attn(const void* p, int64_t ldp, int64_t oq, int64_t of, int64_t ov, float* state, const float* bias,
+                  const float* lower, const int32_t* slots, const int32_t* start, const int32_t* count, void* out, int64_t ldo,
+                  int64_t B, int64_t L, int32_t h, int32_t dk, int32_t dv, int silu, void* ws, int64_t ws_bytes, int dtype,
+                  void* stream);
 
 /* vy_rope_fwd: in-place rotary embedding on a (B,heads,L,dh) tensor (strides as above);
  * used when the fused epilogue does not apply.  `inverse` != 0 applies the transpose rotation
@@ -593,20 +634,26 @@ int vy_gemma_decoder_step(const vy_gemma_plan* plan, const void* x, int64_t pos,
  *                     norm1 / norm2 NULL: the sublayers read x itself
  *   VY_FORM_PARALLEL  h = norm(x) * norm1; x += w_o [mixer(h) | act(h)] + routed(h): one packed product w_in of h also gives the
  *                     [gate; up] rows of a dense feed-forward of width ff (its last 2 ff rows), one product w_o takes both back
+ * w_up instead of w_gu: a feed-forward without a gate, w_down act(w_up h) with the plan's act (VY_FORM_SANDWICH).
  * norm1b / norm2b NULL: no norm on a sublayer's output.  moe (nullable): routed experts, added to the feed-forward's output.
  * clamped: the feed-forward's activation is vy_clamped_act_fwd's (limit, alpha), else the plan's act.
  * Mixers, all from ONE packed input projection w_in of h:
- *   VY_MIX_LATENT  rows [query latent | key/value latent | output gate]: vy_latent_norm, q = w_uq latent, vy_latent_decode
+ *   VY_MIX_LATENT  rows [query latent | key/value latent | output gate]: vy_latent_norm, q = w_uq latent, vy_latent_decode;
+ *                  w_uq NULL: rows [q | key/value latent | output gate]; ring: the cache is a ring of cap rows; gate 0: none;
+ *                  gate_heads: one gate per head
  *   VY_MIX_DECAY   rows [q | k | v | output gate]: vy_decay_attn (silu, rope, k_scale), then vy_rmsnorm_gate, or without
  *                  mix_norm vy_head_norm_gate (mix_n: columns of a head)
+ *   VY_MIX_GATED   rows [q | gate logits | v]: vy_gated_attn (f_bias, f_lower, silu), then vy_head_norm_gate with mix_norm
  *   VY_MIX_WINDOW  rows [q | k | v | output gate if gate]: vy_window_decode on the ring `cache` (strides c_ss per slot, c_sh per
  *                  head); prep (nullable): its norms, and lambda; values: VY_VALUES_FIRST keeps this layer's values,
- *                  VY_VALUES_MIX mixes them in (the step's own buffer is prep's v_out / v_mix)
+ *                  VY_VALUES_MIX mixes them in (the step's own buffer is prep's v_out / v_mix); diff (nullable): differential
+ *                  attention (dim: both maps' columns of a head)
+ * b_in (nullable): bias of w_in.  softcap > 0: logits <- softcap tanh(logits / softcap).
  * Sequence b (ids[b]) lives in slot slots[b] (NULL: b) and holds lengths[slot] tokens, which the step advances by one on the
  * device; max_keys >= every lengths[slot] + 1.  Widths with _p, dim, vdim, ff and dp are padded to multiples of 8; d, q_rank,
  * kv_rank and mix_n are the true counts the norms divide by.  logits: (B, ldv).
  * -------------------------------------------------------------------------------------------- */
-enum { VY_MIX_LATENT = 0, VY_MIX_DECAY = 1, VY_MIX_WINDOW = 2 };
+enum { VY_MIX_LATENT = 0, VY_MIX_DECAY = 1, VY_MIX_WINDOW = 2, VY_MIX_GATED = 3 };
 enum { VY_FORM_SANDWICH = 0, VY_FORM_PARALLEL = 1 };
 enum { VY_VALUES_OWN = 0, VY_VALUES_FIRST = 1, VY_VALUES_MIX = 2 };
 typedef struct vy_hybrid_layer {
@@ -615,21 +662,23 @@ typedef struct vy_hybrid_layer {
   int32_t cap, mix_n;                             /* cache rows per slot; VY_MIX_DECAY: width of mix_norm */
   int32_t form, clamped;
   int32_t kv_heads, rope_dims, rope_len, sink;    /* VY_MIX_WINDOW (rope_*: VY_MIX_DECAY too) */
-  int32_t keep, gate, values, silu;               /* VY_MIX_WINDOW, the last one VY_MIX_DECAY */
+  int32_t keep, gate, values, silu;               /* VY_MIX_WINDOW, the last one VY_MIX_DECAY and VY_MIX_GATED */
+  int32_t ring, gate_heads;                       /* VY_MIX_LATENT */
   float scale, limit, alpha, k_scale;
   const float *norm1, *norm1b, *norm2, *norm2b;
-  const void *w_in, *w_o, *w_gu, *w_down;         /* w_gu: packed [gate; up] (VY_FORM_SANDWICH) */
+  const void *w_in, *b_in, *w_o, *w_gu, *w_up, *w_down;   /* w_gu: packed [gate; up] (VY_FORM_SANDWICH) */
   const float *q_norm, *c_norm;
   const void *w_uq, *w_ukt, *w_uv;
   void* cache; int64_t c_ss, c_sh, c_st;
-  float* state; const float *decay_pow, *mix_norm;
+  float* state; const float *decay_pow, *mix_norm, *f_bias, *f_lower;
   const float* rope;
   const vy_qkv_prep* prep;
+  const vy_diff* diff;
   const vy_moe* moe;
 } vy_hybrid_layer;
 typedef struct vy_hybrid_plan {
   int32_t num_layers, B, d, dp, vocab, dtype, rms, act;
-  float eps, embed_scale;
+  float eps, embed_scale, softcap;
   const vy_hybrid_layer* layers;                  /* host array [num_layers] */
   const void *embed, *head; const float* final_norm;
   int32_t* err;                                   /* nullable: set when an id is outside the vocabulary */

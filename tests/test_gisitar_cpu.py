@@ -190,9 +190,9 @@ def test_argument_errors_without_a_gpu():
     with pytest.raises(_lib.VyomHipError, match="multiples of 4"):
         _lib.call("vy_residual_norm", p, 8, p, 8, None, 0, None, 0, None, None, 1e-5, p, 1e-5, p, 8, 1, 5, 6, 0, 1, None)
     with pytest.raises(_lib.VyomHipError, match="multiples of 8"):
-        _lib.call("vy_latent_decode", p, 8, p, p, p, 8, 8, None, p, 1, p, 8, None, 0, 1, 1, 8, 8, 12, 1.0, p, 4096, 1, None)
+        _lib.call("vy_latent_decode", p, 8, p, p, p, 8, 8, None, p, 1, p, 8, None, 0, 0, 0, 1, 1, 8, 8, 12, 1.0, p, 4096, 1, None)
     with pytest.raises(_lib.VyomHipError, match="workspace"):
-        _lib.call("vy_latent_decode", p, 8, p, p, p, 8, 8, None, p, 1, p, 8, None, 0, 1, 1, 8, 8, 8, 1.0, p, 16, 1, None)
+        _lib.call("vy_latent_decode", p, 8, p, p, p, 8, 8, None, p, 1, p, 8, None, 0, 0, 0, 1, 1, 8, 8, 8, 1.0, p, 16, 1, None)
     with pytest.raises(_lib.VyomHipError, match="multiples of 8"):
         _lib.call("vy_decay_attn", p, 24, 0, 8, 20, p, p, None, p, None, p, 8, 1, 1, 1, 8, 8, 1, None, 0, 0, 1.0, None, 0, 1, None)
     with pytest.raises(_lib.VyomHipError, match="null"):

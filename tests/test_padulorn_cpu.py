@@ -249,7 +249,7 @@ def test_argument_errors_without_a_gpu():
     with pytest.raises(_lib.VyomHipError, match="rotary table"):
         _lib.call("vy_decay_attn", p, 24, 0, 8, 16, p, p, None, p, None, p, 8, 1, 1, 1, 8, 8, 1, p, 10, 4, 1.0, None, 0, 1, None)
     with pytest.raises(_lib.VyomHipError, match="multiples of 8"):
-        _lib.call("vy_head_norm_gate", p, 8, p, 8, p, 8, 1, 1, 5, 6, 1e-5, 1, None)
+        _lib.call("vy_head_norm_gate", p, 8, None, p, 8, p, 8, 1, 1, 5, 6, 1e-5, 1, None)
     moe = _lib.VyMoe(4, 2, 2, 1, 8, 8, 2, 0, 1, 1, 1.0, 1.0, 1.0, p, p, p)
     for field, value in (("act", 2), ("score", 2), ("group_best", 3)):
         moe.act, moe.score, moe.group_best = 0, 0, 1

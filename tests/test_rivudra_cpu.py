@@ -196,7 +196,7 @@ def test_argument_errors_without_a_gpu():
     from vyomai_amd import _lib
     buf = (ctypes.c_char * 4096)()
     p = (ctypes.addressof(buf) + 63) // 64 * 64
-    win = [p, 64, 0, 8, 16, 24, p, 64, 64, 4, 0, None, 0, 0, None, None, p, 1, p, 8, 1, 1, 1, 8, 8]
+    win = [p, 64, 0, 8, 16, 24, p, 64, 64, 4, 0, None, 0, 0, None, None, None, p, 1, p, 8, 1, 1, 1, 8, 8]
 
     def decode(**kw):
         a = list(win)
@@ -208,7 +208,7 @@ def test_argument_errors_without_a_gpu():
     with pytest.raises(_lib.VyomHipError, match="rotary table"):
         _lib.call("vy_window_decode", *decode(_11=p, _12=10, _13=5), 1.0, 1, None, 0, 1, None)
     with pytest.raises(_lib.VyomHipError, match="5 positions, rotary table of 4"):
-        _lib.call("vy_window_decode", *decode(_11=p, _12=8, _13=4, _17=5), 1.0, 1, None, 0, 1, None)
+        _lib.call("vy_window_decode", *decode(_11=p, _12=8, _13=4, _18=5), 1.0, 1, None, 0, 1, None)
     with pytest.raises(_lib.VyomHipError, match="bad arguments"):
         _lib.call("vy_window_decode", *win, 0.0, 1, None, 0, 1, None)
     with pytest.raises(_lib.VyomHipError, match="4 kept of 4 rows"):

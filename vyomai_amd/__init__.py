@@ -10,6 +10,7 @@ from .models.decoder import DecoderModel  # noqa: F401
 from .models.vision_encoder import Vit  # noqa: F401
 from .models.multimodel import VisionLanguageModel  # noqa: F401
 from .models.encoder_decoder import EncoderDecoderModel  # noqa: F401
+from .models.biruvik import BiruvikConfig, BiruvikModel  # noqa: F401
 from .models.gisitar import GisitarConfig, GisitarModel  # noqa: F401
 from .models.padulorn import PadulornConfig, PadulornModel  # noqa: F401
 from .models.rivudra import RivudraConfig, RivudraModel  # noqa: F401

@@ -14,7 +14,7 @@ _HERE = os.path.dirname(os.path.abspath(__file__))
 LIB_PATH = os.environ.get("VY_LIB_PATH") or os.path.join(_HERE, "lib", "libvyom_hip.so")
 
 VY_F32, VY_BF16 = 0, 1
-ACT_NONE, ACT_GELU_ERF, ACT_GELU_TANH, ACT_SILU = 0, 1, 2, 3
+ACT_NONE, ACT_GELU_ERF, ACT_GELU_TANH, ACT_SILU, ACT_RELU2 = 0, 1, 2, 3, 4
 ACT_SAVE_DERIV = 0x100   # saved tensor = act'(pre) instead of pre (include/vyom_hip.h)
 MOE_CLAMPED, MOE_GELU = 0, 1
 SCORE_SOFTMAX, SCORE_SIGMOID = 0, 1
@@ -25,6 +25,7 @@ _p, _i64, _i, _f, _u64 = C.c_void_p, C.c_int64, C.c_int, C.c_float, C.c_uint64
 # name -> argtypes, exactly the prototypes of include/vyom_hip.h
 PROTOTYPES = {
     "vy_linear_fwd": [_p, _i64, _p, _i64, _p, _p, _i64, _p, _i64, _p, _i64, _i64, _i64, _i, _i, _p],
+    "vy_linear_softcap_fwd": [_p, _i64, _p, _i64, _p, _i64, _i64, _i64, _i64, _f, _i, _p],
     "vy_qkv_rope_fwd": [_p, _i64, _p, _i64, _p, _p, _p, _i64,
                         _p, _i64, _i64, _i64, _p, _i64, _i64, _i64, _p, _i64, _i64, _i64,
                         _i64, _i64, _i64, _i, _i, _i, _i, _p],
@@ -65,21 +66,23 @@ PROTOTYPES = {
     "vy_residual_norm": [_p, _i64, _p, _i64, _p, _i64, _p, _i64, _p, _p, _f, _p, _f, _p, _i64, _i64, _i64, _i64, _i, _i, _p],
     "vy_residual_norm_routed": [_p, _i64, _p, _i64, _p, _i64, _p, _i64, _p, _f, _p, _p, _f, _p, _f, _p, _i64, _i64, _i64, _i64, _i,
                                 _i, _p],
-    "vy_latent_norm": [_p, _i64, _p, _p, _i64, _i, _i, _p, _p, _i64, _i, _i, _p, _i64, _i64, _i, _p, _p, _p, _i64, _i64, _f,
+    "vy_latent_norm": [_p, _i64, _p, _p, _i64, _i, _i, _p, _p, _i64, _i, _i, _p, _i64, _i64, _i, _i, _p, _p, _p, _i64, _i64, _f,
                        _i, _p],
     "vy_rmsnorm_gate": [_p, _i64, _p, _p, _i64, _p, _i64, _i64, _i64, _i64, _f, _i, _p],
-    "vy_head_norm_gate": [_p, _i64, _p, _i64, _p, _i64, _i64, _i, _i64, _i64, _f, _i, _p],
+    "vy_head_norm_gate": [_p, _i64, _p, _p, _i64, _p, _i64, _i64, _i, _i64, _i64, _f, _i, _p],
     "vy_attn_fwd_ex": [_p, _i64, _i64, _i64, _p, _i64, _i64, _i64, _p, _i64, _i64, _i64, _p, _i64, _i64, _p, _i64, _i64,
                        _p, _p, _i64, _i, _i, _i64, _i64, _i, _i, _f, _p, _i, _p],
-    "vy_latent_decode": [_p, _i64, _p, _p, _p, _i64, _i64, _p, _p, _i64, _p, _i64, _p, _i64, _i, _i, _i, _i, _i, _f, _p, _i64,
+    "vy_latent_decode": [_p, _i64, _p, _p, _p, _i64, _i64, _p, _p, _i64, _p, _i64, _p, _i64, _i, _i, _i, _i, _i, _i, _i, _f, _p, _i64,
                          _i, _p],
+    "vy_gated_attn": [_p, _i64, _i64, _i64, _i64, _p, _p, _p, _p, _p, _p, _p, _i64, _i64, _i64, _i, _i, _i, _i, _p, _i64, _i, _p],
+    "vy_diff_attn_fwd": [_p, _i64, _p, _i64, _i64, _i, _p, _p, _p, _p, _p, _i64, _i64, _i64, _i, _i, _i, _i, _f, _i, _p],
     "vy_decay_attn": [_p, _i64, _i64, _i64, _i64, _p, _p, _p, _p, _p, _p, _i64, _i64, _i64, _i, _i, _i, _i, _p, _i, _i, _f, _p, _i64,
                       _i, _p],
     "vy_window_rows": [_p, _i64, _i64, _i64, _p, _i64, _i64, _i, _i, _p, _i, _i, _i, _i, _p, _p, _p, _i64, _i64, _i, _i, _i, _i, _p],
     "vy_qkv_rows": [_p, _i64, _i64, _i64, _i64, _p, _p, _i64, _i64, _i, _i, _p, _i, _i, _i, _p, _p, _p, _i64, _i64, _i, _i, _i, _i, _i,
                     _p],
     "vy_window_context": [_p, _i64, _i64, _i64, _p, _i64, _i64, _i, _i, _p, _i, _i, _p, _p, _i64, _i64, _i, _i, _i, _i, _p],
-    "vy_window_decode": [_p, _i64, _i64, _i64, _i64, _i64, _p, _i64, _i64, _i, _i, _p, _i, _i, _p, _p, _p, _i64, _p, _i64, _i64, _i, _i,
+    "vy_window_decode": [_p, _i64, _i64, _i64, _i64, _i64, _p, _i64, _i64, _i, _i, _p, _i, _i, _p, _p, _p, _p, _i64, _p, _i64, _i64, _i, _i,
                          _i, _i, _f, _i, _p, _i64, _i, _p],
     "vy_moe_fwd": [_p, _p, _i64, _i64, _p, _i64, _p, _i64, _p, _p, _p, _p, _i64, _i, _p],
     "vy_clamped_act_fwd": [_p, _i64, _p, _i64, _i64, _i64, _f, _f, _i, _p],
@@ -94,7 +97,7 @@ PROTOTYPES = {
 }
 OTHER_SYMBOLS = ["vy_last_error", "vy_abi_version", "vy_layernorm_bwd_ws_rows", "vy_decode_ws_bytes",
                  "vy_gemma_ws_bytes", "vy_ddp_world", "vy_ddp_rank", "vy_latent_decode_ws_bytes", "vy_decay_attn_ws_bytes",
-                 "vy_hybrid_ws_bytes", "vy_window_decode_ws_bytes", "vy_moe_ws_bytes"]
+                 "vy_hybrid_ws_bytes", "vy_window_decode_ws_bytes", "vy_moe_ws_bytes", "vy_gated_attn_ws_bytes"]
 DECAY_CHUNK = 64   # VY_DECAY_CHUNK
 ALL_SYMBOLS = list(PROTOTYPES) + OTHER_SYMBOLS
 
@@ -108,13 +111,19 @@ class VyWgradDesc(C.Structure):
 class VyAttnWindow(C.Structure):
     """vy_attn_window of include/vyom_hip.h."""
     _fields_ = [(n, C.c_int32) for n in ("window", "sink", "kv_by_slot", "start_cap")] + \
-               [("rope", _p), ("rope_dims", C.c_int32), ("rope_len", C.c_int32), ("keep", C.c_int32)]
+               [("rope", _p), ("rope_dims", C.c_int32), ("rope_len", C.c_int32), ("keep", C.c_int32), ("gate_heads", C.c_int32)]
 
 
 class VyQkvPrep(C.Structure):
     """vy_qkv_prep of include/vyom_hip.h."""
     _fields_ = [("q_norm", _p), ("k_norm", _p), ("n_q", C.c_int32), ("n_k", C.c_int32), ("eps", C.c_float), ("lambda_", C.c_float),
-                ("v_mix", _p), ("ldm", _i64), ("n_v", C.c_int32), ("m_v", C.c_int32), ("m_vp", C.c_int32), ("v_out", _p), ("ldo", _i64)]
+                ("v_mix", _p), ("ldm", _i64), ("n_v", C.c_int32), ("m_v", C.c_int32), ("m_vp", C.c_int32), ("v_out", _p), ("ldo", _i64),
+                ("group", C.c_int32), ("temp_every", C.c_int32), ("temp_coef", C.c_float)]
+
+
+class VyDiff(C.Structure):
+    """vy_diff of include/vyom_hip.h."""
+    _fields_ = [("lambda_", C.c_float), ("out_scale", C.c_float), ("eps", C.c_float), ("n_v", C.c_int32)]
 
 
 class VyRoutedRows(C.Structure):
@@ -160,7 +169,8 @@ def load() -> C.CDLL:
     lib.vy_decode_ws_bytes.argtypes = [C.c_int32] * 7
     for name, argtypes in (("vy_latent_decode_ws_bytes", [_i, _i, _i]),
                            ("vy_decay_attn_ws_bytes", [_i64, _i64, _i, _i, _i, _i]), ("vy_hybrid_ws_bytes", [_p]),
-                           ("vy_window_decode_ws_bytes", [_i, _i, _i, _i, _i]), ("vy_moe_ws_bytes", [_p, _i64, _i])):
+                           ("vy_window_decode_ws_bytes", [_i, _i, _i, _i, _i, _i]), ("vy_moe_ws_bytes", [_p, _i64, _i]),
+                           ("vy_gated_attn_ws_bytes", [_i64, _i64, _i, _i, _i, _i])):
         getattr(lib, name).restype = C.c_int64
         getattr(lib, name).argtypes = argtypes
     _lib = lib

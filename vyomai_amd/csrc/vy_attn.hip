@@ -49,6 +49,7 @@ struct AttnParams {
   // sequence, an upper bound of the start position (older keys are not in the operands), and rotary positions of the queries
   int window, sink, kv_by_slot, start_cap;
   int keep;            // keys j < keep are seen whatever the window
+  int gate_heads;      // the gate is one number per head: rows [h]
   const float2* rope; int rope_half, rope_len;   // (cos, sin) [position][pair], pairs of neighbouring columns
   int diag;            // timing experiments only (VY_ATTN_DIAG): 1 = no output store, 2 = no tile loop
 };
@@ -469,7 +470,9 @@ __global__ __launch_bounds__(256, DH == 64 ? 3 : 1) void attn_fwd_mfma_kernel(At
 #pragma unroll
       for (int it = 0; it < 32 * LPR / 64; ++it) {
         const int r = q0 + wave * 32 + (it * 64 + lane) / LPR, ch = (it * 64 + lane) % LPR;
-        g8[it] = *reinterpret_cast<const bf16x8*>((const bf16*)p.gate + (int64_t)b * p.g_sb + (int64_t)min(r, p.L - 1) * p.g_sl + head * DH + ch * 8);
+        const bf16* gr = (const bf16*)p.gate + (int64_t)b * p.g_sb + (int64_t)min(r, p.L - 1) * p.g_sl;
+        if (EXT == 2 && p.gate_heads) g8[it][0] = gr[head];
+        else g8[it] = *reinterpret_cast<const bf16x8*>(gr + head * DH + ch * 8);
       }
     }
   }
@@ -499,7 +502,7 @@ __global__ __launch_bounds__(256, DH == 64 ? 3 : 1) void attn_fwd_mfma_kernel(At
     if constexpr (EXT) {
       if (p.gate) {
 #pragma unroll
-        for (int e = 0; e < 8; ++e) vv[e] = (bf16)((float)vv[e] * vy_sigmoid((float)g8[it][e]));
+        for (int e = 0; e < 8; ++e) vv[e] = (bf16)((float)vv[e] * vy_sigmoid((float)g8[it][EXT == 2 && p.gate_heads ? 0 : e]));
       }
     }
     if (qrow_ < p.L)
@@ -731,7 +734,10 @@ __global__ __launch_bounds__(256) void attn_fwd_gen_kernel(AttnParams p, int dh)
   const float inv = 1.0f / l_tot;
   if (qi < p.L) {
     bf16* orow = (bf16*)p.out + (int64_t)b * p.o_sb + (int64_t)qi * p.o_sl + head * dv;
-    const bf16* grow = EXT && p.gate ? (const bf16*)p.gate + (int64_t)b * p.g_sb + (int64_t)qi * p.g_sl + head * dv : nullptr;
+    const bool one_gate = EXT == 2 && p.gate && p.gate_heads;
+    const bf16* grow = EXT && p.gate ? (const bf16*)p.gate + (int64_t)b * p.g_sb + (int64_t)qi * p.g_sl + (one_gate ? head : head * dv) : nullptr;
+    const float gh = one_gate ? vy_sigmoid((float)*grow) : 1.f;
+    if (one_gate) grow = nullptr;
     bf16x4 g4[EXT ? NDB : 1];   // requested together: behind the first store each load would wait for its own round trip
     if (EXT && grow) {
 #pragma unroll
@@ -742,7 +748,7 @@ __global__ __launch_bounds__(256) void attn_fwd_gen_kernel(AttnParams p, int dh)
       const int d0 = 16 * n + 4 * kq;
       if (d0 < dv) {
         bf16x4 w;
-        float gt[4] = {1.f, 1.f, 1.f, 1.f};
+        float gt[4] = {gh, gh, gh, gh};
         if (EXT && grow) {
 #pragma unroll
           for (int r = 0; r < 4; ++r) gt[r] = vy_sigmoid((float)g4[n][r]);
@@ -953,7 +959,7 @@ __global__ __launch_bounds__(64 * NWV) void attn_rowwise_kernel(AttnParams p, in
 #pragma unroll
     for (int e = 0; e < VEC; ++e) {
       float x = out[e] * inv;
-      if (EXT && p.gate) x *= vy_sigmoid(VyT<T>::ld((const T*)p.gate + (int64_t)b * p.g_sb + (int64_t)qi * p.g_sl + head * dv + ch * VEC + e));
+      if (EXT && p.gate) x *= vy_sigmoid(VyT<T>::ld((const T*)p.gate + (int64_t)b * p.g_sb + (int64_t)qi * p.g_sl + (EXT == 2 && p.gate_heads ? head : head * dv + ch * VEC + e)));
       VyT<T>::st(O + e, x);
     }
     if (p.lse && ch == 0) p.lse[((int64_t)b * p.h + head) * p.L + qi] = M_ + __logf(Ls);
@@ -1107,7 +1113,7 @@ extern "C" int vy_attn_fwd_ex(const void* q, int64_t q_sb, int64_t q_sh, int64_t
   if (!(scale > 0.f)) VY_FAIL(VY_ERR_ARG, "%s: scale %g", who, (double)scale);
   if (win->rope && (win->rope_dims < 0 || win->rope_dims % 2 || win->rope_dims > dh || win->rope_len < 1))
     VY_FAIL(VY_ERR_ARG, "%s: rotary table of %d columns, %d positions for heads of %d", who, win->rope_dims, win->rope_len, dh);
-  p.window = win->window; p.sink = win->sink; p.kv_by_slot = win->kv_by_slot; p.start_cap = win->start_cap; p.keep = win->keep;
+  p.window = win->window; p.sink = win->sink; p.kv_by_slot = win->kv_by_slot; p.start_cap = win->start_cap; p.keep = win->keep; p.gate_heads = win->gate_heads;
   p.rope = (const float2*)win->rope; p.rope_half = win->rope_dims / 2; p.rope_len = win->rope_len;
   if (p.rope_half == 0) p.rope = nullptr;
   return launch_ex<2>(p, dh, dtype, (hipStream_t)stream, who);

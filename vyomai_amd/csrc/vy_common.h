@@ -155,11 +155,14 @@ __device__ __forceinline__ float vy_gelu_erf_grad_fast(float x) {
 __device__ __forceinline__ float vy_sigmoid(float x) { return 1.0f / (1.0f + __expf(-x)); }
 __device__ __forceinline__ float vy_silu(float x) { return x * vy_sigmoid(x); }
 
+// arg: the cap of VY_ACT_SOFTCAP
 template <int ACT>
-__device__ __forceinline__ float vy_act_fwd(float x) {
+__device__ __forceinline__ float vy_act_fwd(float x, float arg = 0.f) {
   if constexpr (ACT == VY_ACT_GELU_ERF) return vy_gelu_erf(x);
   else if constexpr (ACT == VY_ACT_GELU_TANH) return vy_gelu_tanh(x);
   else if constexpr (ACT == VY_ACT_SILU) return vy_silu(x);
+  else if constexpr (ACT == VY_ACT_RELU2) { const float r = fmaxf(x, 0.f); return r * r; }
+  else if constexpr (ACT == VY_ACT_SOFTCAP) return arg * tanhf(x / arg);
   else return x;
 }
 template <int ACT>
@@ -182,9 +185,9 @@ __device__ __forceinline__ float vy_wave_max(float v) {
 
 // reduced-cost variants for bf16 storage (results are rounded to 8 bits of mantissa anyway)
 template <int ACT>
-__device__ __forceinline__ float vy_act_fwd_fast(float x) {
+__device__ __forceinline__ float vy_act_fwd_fast(float x, float arg = 0.f) {
   if constexpr (ACT == VY_ACT_GELU_ERF) return vy_gelu_erf_fast(x);
-  else return vy_act_fwd<ACT>(x);
+  else return vy_act_fwd<ACT>(x, arg);
 }
 template <int ACT>
 __device__ __forceinline__ float vy_act_grad_fast(float x) {

@@ -672,7 +672,8 @@ enum { GV_PLAIN = 0, GV_GATED = 1, GV_QKV = 2 };
 struct DecGemvArgs {
   const bf16* x; const bf16* w; const bf16* bias; const bf16* residual; bf16* y;
   int N, K, ldw;
-  int act;                                     // GV_GATED: VY_ACT_GELU_TANH or VY_ACT_SILU
+  int act;                                     // GV_GATED: VY_ACT_GELU_TANH or VY_ACT_SILU; GV_PLAIN: none, RELU2 or SOFTCAP
+  float act_arg;
   float eps;
   // GV_QKV
   bf16* q; bf16* k; bf16* v; long long c_sh;   // q [nq]; k / v: cache row of this position, head stride c_sh
@@ -737,6 +738,8 @@ __global__ __launch_bounds__(256) void dec_gemv1_kernel(const DecGemvArgs p) {
     if (lane == 0) {
       float x = acc;
       if (p.bias) x += (float)p.bias[n];
+      if (p.act == VY_ACT_RELU2) x = vy_act_fwd<VY_ACT_RELU2>(x);
+      else if (p.act == VY_ACT_SOFTCAP) x = vy_act_fwd<VY_ACT_SOFTCAP>(x, p.act_arg);
       if (p.residual) x += (float)p.residual[n];
       p.y[n] = (bf16)x;
     }
@@ -911,6 +914,16 @@ int vy_dec_gemv1(const void* x, const void* w, const void* bias, const void* res
   a.N = N; a.K = K; a.ldw = K; a.eps = eps;
   if (prescaled ? dec_gemv1_go<GV_PLAIN, true>(a, st) : dec_gemv1_go<GV_PLAIN, false>(a, st)) return VY_ERR_UNSUPPORTED;
   VY_CHECK_LAUNCH("vy_dec_gemv1");
+  return VY_OK;
+}
+// act(x W^T + bias), act none, VY_ACT_RELU2 or VY_ACT_SOFTCAP
+int vy_dec_gemv1_act(const void* x, const void* w, const void* bias, int act, float act_arg, void* y, int N, int K, hipStream_t st) {
+  if (!gemv1_ok(x, w, N, K) || (act != VY_ACT_NONE && act != VY_ACT_RELU2 && act != VY_ACT_SOFTCAP)) return VY_ERR_UNSUPPORTED;
+  DecGemvArgs a{};
+  a.x = (const bf16*)x; a.w = (const bf16*)w; a.bias = (const bf16*)bias; a.y = (bf16*)y;
+  a.N = N; a.K = K; a.ldw = K; a.act = act; a.act_arg = act_arg;
+  if (dec_gemv1_go<GV_PLAIN, false>(a, st)) return VY_ERR_UNSUPPORTED;
+  VY_CHECK_LAUNCH("vy_dec_gemv1_act");
   return VY_OK;
 }
 int vy_dec_gemv1_gated(const void* x, const void* wgu, void* y, int I, int K, int act, int prescaled, float eps, hipStream_t st) {

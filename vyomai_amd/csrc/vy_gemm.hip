@@ -82,6 +82,7 @@ struct EpiPlain {
   int vec_ok;  // all row strides % 4 == 0 and base pointers 4-element aligned
   VyDrop drop; // dropout on act(x W^T + b) before the residual add (thr == 0: none)
   int wt_store; // large outputs: write-through (sc1) stores from the staged epilogue
+  float act_arg; // VY_ACT_SOFTCAP: the cap
   int pre_deriv; // VY_ACT_SAVE_DERIV: `pre` receives act'(x W^T + b) / `gradpre` already holds act' (see include/vyom_hip.h)
 };
 
@@ -103,7 +104,7 @@ __device__ __forceinline__ void epi_plain_quad(const EpiPlain<T>& e, float (&v)[
     }
     if constexpr (!GRAD) {
 #pragma unroll
-      for (int i = 0; i < 4; ++i) v[i] = vy_act_fwd<ACT>(v[i]);
+      for (int i = 0; i < 4; ++i) v[i] = vy_act_fwd<ACT>(v[i], e.act_arg);
       if (e.drop.thr) {
         uint32_t lots[4];
         vy_drop_lots(e.drop, m, n >> 3, lots);
@@ -130,7 +131,7 @@ __device__ __forceinline__ void epi_plain_quad(const EpiPlain<T>& e, float (&v)[
       if (e.bias) x += VyT<T>::ld(e.bias + n + i);
       if (e.pre) VyT<T>::st(e.pre + m * e.ldy + n + i, e.pre_deriv ? vy_act_grad<ACT>(round_like<T>(x)) : x);
       if constexpr (!GRAD) {
-        x = vy_act_fwd<ACT>(x);
+        x = vy_act_fwd<ACT>(x, e.act_arg);
         if (e.drop.thr) {
           uint32_t lots[4];
           vy_drop_lots(e.drop, m, (n + i) >> 3, lots);
@@ -447,7 +448,7 @@ __device__ __forceinline__ void gemm_epilogue(typename AccTile<BM, BN, WGM, WGN,
                 v[e] = v[e] * cdf;
               } else {
                 d8[e] = (bf16)vy_act_grad_fast<ACT>(v[e]);
-                v[e] = vy_act_fwd_fast<ACT>(v[e]);
+                v[e] = vy_act_fwd_fast<ACT>(v[e], ep.act_arg);
               }
             }
             if (ep.vec_ok && n + 8 <= N) {
@@ -459,7 +460,7 @@ __device__ __forceinline__ void gemm_epilogue(typename AccTile<BM, BN, WGM, WGN,
             }
           } else {
 #pragma unroll
-            for (int e = 0; e < 8; ++e) v[e] = vy_act_fwd_fast<ACT>(v[e]);
+            for (int e = 0; e < 8; ++e) v[e] = vy_act_fwd_fast<ACT>(v[e], ep.act_arg);
           }
         }
         if constexpr (!GRAD) {
@@ -1766,7 +1767,7 @@ __global__ __launch_bounds__(256) void gemm_skinny16_bf16_kernel(
     if constexpr (EPI == 0) {
       if (fast && !ep.pre && !ep.residual2 && !ep.drop.thr) {   // epi_plain_quad on the prefetched operands
 #pragma unroll
-        for (int i = 0; i < 4; ++i) v[i] = vy_act_fwd<ACT>(v[i] + (float)bias4[i]);
+        for (int i = 0; i < 4; ++i) v[i] = vy_act_fwd<ACT>(v[i] + (float)bias4[i], ep.act_arg);
         if (ep.residual) {
 #pragma unroll
           for (int i = 0; i < 4; ++i) v[i] += (float)res4[blk][i];
@@ -2019,7 +2020,7 @@ __global__ __launch_bounds__(256) void gemv_bf16_kernel(const bf16* __restrict__
     } else if constexpr (EPI == 0) {
       if (ep.bias) x += (float)ep.bias[n];
       if (ep.pre) ep.pre[m * ep.ldy + n] = (bf16)(ep.pre_deriv ? vy_act_grad<ACT>(vy_round_bf16(x)) : x);
-      x = vy_act_fwd<ACT>(x);
+      x = vy_act_fwd<ACT>(x, ep.act_arg);
       if (ep.drop.thr) {
         uint32_t lots[4];
         vy_drop_lots(ep.drop, m, n >> 3, lots);
@@ -2142,11 +2143,12 @@ int linear_impl(const void* x, int64_t ldx, const void* w, int64_t ldw, const vo
                 const void* residual, int64_t ldr, const void* gradpre, int64_t ldg, void* y,
                 int64_t ldy, void* pre_out, int64_t M, int64_t N, int64_t K, int act, bool grad,
                 hipStream_t st, const char* who, const void* residual2 = nullptr, int64_t ldr2 = 0,
-                VyDrop drop = VyDrop{}) {
+                VyDrop drop = VyDrop{}, float act_arg = 0.f) {
   if (int rc = check_operands<T>(who, x, ldx, w, ldw, M, N, K)) return rc;
   if (!y) VY_FAIL(VY_ERR_ARG, "%s: null output", who);
   if (ldy < N) VY_FAIL(VY_ERR_ARG, "%s: ldy < N", who);
   EpiPlain<T> ep;
+  ep.act_arg = act_arg;
   ep.pre_deriv = (act & VY_ACT_SAVE_DERIV) ? 1 : 0;
   act &= ~VY_ACT_SAVE_DERIV;
   ep.bias = (const T*)bias; ep.residual = (const T*)residual; ep.ldr = ldr;
@@ -2176,6 +2178,8 @@ int linear_impl(const void* x, int64_t ldx, const void* w, int64_t ldw, const vo
     if (act == VY_ACT_NONE) VY_GO(VY_ACT_NONE, false);
     else if (act == VY_ACT_GELU_ERF) VY_GO(VY_ACT_GELU_ERF, false);
     else if (act == VY_ACT_GELU_TANH) VY_GO(VY_ACT_GELU_TANH, false);
+    else if (act == VY_ACT_RELU2 && !pre_out) VY_GO(VY_ACT_RELU2, false);
+    else if (act == VY_ACT_SOFTCAP && !pre_out && act_arg > 0.f) VY_GO(VY_ACT_SOFTCAP, false);
     else VY_FAIL(VY_ERR_ARG, "%s: unknown activation %d", who, act);
   } else {
     if (act == VY_ACT_NONE || !gradpre) VY_GO(VY_ACT_NONE, true);
@@ -2249,6 +2253,18 @@ extern "C" int vy_linear_fwd(const void* x, int64_t ldx, const void* w, int64_t 
   if (dtype == VY_F32)
     return linear_impl<float>(x, ldx, w, ldw, bias, residual, ldr, nullptr, 0, y, ldy, pre_out, M, N, K, act, false, st, "vy_linear_fwd");
   VY_FAIL(VY_ERR_ARG, "vy_linear_fwd: bad dtype %d", dtype);
+}
+
+extern "C" int vy_linear_softcap_fwd(const void* x, int64_t ldx, const void* w, int64_t ldw, void* y, int64_t ldy, int64_t M,
+                                     int64_t N, int64_t K, float cap, int dtype, void* stream) {
+  const char* who = "vy_linear_softcap_fwd";
+  hipStream_t st = (hipStream_t)stream;
+  if (!(cap > 0.f)) VY_FAIL(VY_ERR_ARG, "%s: cap %g", who, (double)cap);
+  if (dtype == VY_BF16)
+    return linear_impl<bf16>(x, ldx, w, ldw, nullptr, nullptr, 0, nullptr, 0, y, ldy, nullptr, M, N, K, VY_ACT_SOFTCAP, false, st, who, nullptr, 0, VyDrop{}, cap);
+  if (dtype == VY_F32)
+    return linear_impl<float>(x, ldx, w, ldw, nullptr, nullptr, 0, nullptr, 0, y, ldy, nullptr, M, N, K, VY_ACT_SOFTCAP, false, st, who, nullptr, 0, VyDrop{}, cap);
+  VY_FAIL(VY_ERR_ARG, "%s: bad dtype %d", who, dtype);
 }
 
 extern "C" int vy_linear_dropout_fwd(const void* x, int64_t ldx, const void* w, int64_t ldw, const void* bias,

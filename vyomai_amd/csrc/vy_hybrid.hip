@@ -1,7 +1,7 @@
 // Native decode driver (host code) of decoders that mix layer kinds: one call runs a whole single-token step of a batch of
-// sequences of different lengths -- embedding, every layer (latent attention over its latent cache, decayed linear attention
-// over its fp32 state, or windowed attention over its ring), dense or routed feed-forward behind or beside the mixer, final
-// norm and vocabulary product.  See include/vyom_hip.h (vy_hybrid_decoder_step).
+// sequences of different lengths -- embedding, every layer (latent attention over its latent cache or ring, decayed or gated
+// linear attention over its fp32 state, or windowed or differential attention over its ring), dense or routed feed-forward behind
+// or beside the mixer, final norm and vocabulary product.  See include/vyom_hip.h (vy_hybrid_decoder_step).
 #include "vy_common.h"
 
 int vy_residual_norm_ex(float* x, int64_t ldx, const void* y, int64_t ldy, const void* table, int64_t ldt, const int64_t* ids,
@@ -16,8 +16,7 @@ int vy_moe_few(const vy_moe* d, const void* h, int64_t ldh, int64_t M, const int
 int vy_parallel_decode(const vy_hybrid_plan* p, const vy_hybrid_layer* L, const void* h, void* in, void* ao, void* y, void* erows,
                        int32_t* eids, float* ew, void* moe_ws, int64_t moe_ws_bytes, const int32_t* slots, const int32_t* lengths,
                        int64_t max_keys, void* mix_ws, int64_t mix_ws_bytes, void* stream);
-int vy_dec_gemv1(const void* x, const void* w, const void* bias, const void* residual, void* y, int N, int K, int prescaled,
-                 float eps, hipStream_t st);
+int vy_dec_gemv1_act(const void* x, const void* w, const void* bias, int act, float act_arg, void* y, int N, int K, hipStream_t st);
 int vy_dec_gemv1_gated(const void* x, const void* wgu, void* y, int I, int K, int act, int prescaled, float eps, hipStream_t st);
 int vy_gemv_gated(const void* x, int64_t ldx, const void* w, int64_t ldw, const void* norm_w, float eps, void* y, int64_t ldy,
                   int64_t M, int64_t I, int64_t K, int act, void* stream);
@@ -37,11 +36,11 @@ Sizes sizes_of(const vy_hybrid_plan* p) {
     const bool parallel = L.form == VY_FORM_PARALLEL;
     mx(s.ao, (int64_t)L.heads * L.vdim + (parallel ? L.ff : 0));
     if (L.mixer == VY_MIX_LATENT) {
-      mx(s.q, (int64_t)L.heads * L.dim);
-      mx(s.cq, L.q_rank_p);
+      if (L.w_uq) mx(s.q, (int64_t)L.heads * L.dim);
+      if (L.w_uq) mx(s.cq, L.q_rank_p);
       mx(s.mix_ws, vy_latent_decode_ws_bytes(p->B, L.heads, L.kv_rank_p));
     } else if (L.mixer == VY_MIX_WINDOW) {
-      mx(s.mix_ws, vy_window_decode_ws_bytes(p->B, L.heads, L.kv_heads, L.vdim, L.cap));
+      mx(s.mix_ws, vy_window_decode_ws_bytes(p->B, L.heads, L.kv_heads, L.vdim, L.cap, L.diff != nullptr));
       if (L.values != VY_VALUES_OWN) mx(s.values, (int64_t)L.kv_heads * L.vdim);
     } else {
       mx(s.o, (int64_t)L.heads * L.vdim);
@@ -58,13 +57,15 @@ Sizes sizes_of(const vy_hybrid_plan* p) {
   return s;
 }
 
-// y[B, N] = x[B, K] W^T
-int product(const vy_hybrid_plan* p, const void* x, const void* w, void* y, int64_t ldy, int64_t N, int64_t K, void* stream) {
+// y[B, N] = act(x[B, K] W^T + bias); cap: of VY_ACT_SOFTCAP
+int product(const vy_hybrid_plan* p, const void* x, const void* w, void* y, int64_t ldy, int64_t N, int64_t K, void* stream,
+            const void* bias = nullptr, int act = VY_ACT_NONE, float cap = 0.f) {
   if (p->dtype == VY_BF16 && p->B == 1 && N <= INT32_MAX) {
-    const int rc = vy_dec_gemv1(x, w, nullptr, nullptr, y, (int)N, (int)K, 0, 0.f, (hipStream_t)stream);
+    const int rc = vy_dec_gemv1_act(x, w, bias, act, cap, y, (int)N, (int)K, (hipStream_t)stream);
     if (rc != VY_ERR_UNSUPPORTED) return rc;
   }
-  return vy_linear_fwd(x, K, w, K, nullptr, nullptr, 0, y, ldy, nullptr, p->B, N, K, VY_ACT_NONE, p->dtype, stream);
+  if (act == VY_ACT_SOFTCAP) return vy_linear_softcap_fwd(x, K, w, K, y, ldy, p->B, N, K, cap, p->dtype, stream);
+  return vy_linear_fwd(x, K, w, K, bias, nullptr, 0, y, ldy, nullptr, p->B, N, K, act, p->dtype, stream);
 }
 
 // packed [gate | up] rows -> activation rows
@@ -145,16 +146,18 @@ extern "C" int vy_hybrid_decoder_step(const vy_hybrid_plan* p, const int64_t* id
       }
       if (rc != VY_ERR_UNSUPPORTED) return rc;
     }
-    if ((rc = product(p, h, L.w_in, in, L.n_in, L.n_in, dp, stream))) return rc;
+    if ((rc = product(p, h, L.w_in, in, L.n_in, L.n_in, dp, stream, L.b_in))) return rc;
     if (L.mixer == VY_MIX_LATENT) {
-      if (max_keys > L.cap) VY_FAIL(VY_ERR_ARG, "%s: %ld keys exceed the cache capacity %d", who, (long)max_keys, L.cap);
-      if ((rc = vy_latent_norm(in, L.n_in, L.q_norm, cq, L.q_rank_p, L.q_rank, L.q_rank_p, L.c_norm, nullptr, 0, L.kv_rank,
-                               L.kv_rank_p, L.cache, L.c_ss, L.c_st, L.cap, slots, lengths, nullptr, B, 1, p->eps, p->dtype,
+      if (!L.ring && max_keys > L.cap) VY_FAIL(VY_ERR_ARG, "%s: %ld keys exceed the cache capacity %d", who, (long)max_keys, L.cap);
+      const int64_t nq = L.w_uq ? L.q_rank_p : nk;   // columns ahead of the key/value latent: the queries' latent, or the queries
+      if ((rc = vy_latent_norm(in, L.n_in, L.w_uq ? L.q_norm : nullptr, cq, L.q_rank_p, L.q_rank, (int)nq, L.c_norm, nullptr, 0, L.kv_rank,
+                               L.kv_rank_p, L.cache, L.c_ss, L.c_st, L.cap, L.ring, slots, lengths, nullptr, B, 1, p->eps, p->dtype,
                                stream))) return rc;
-      if ((rc = product(p, cq, L.w_uq, q, nk, nk, L.q_rank_p, stream))) return rc;
-      const char* gate = (const char*)in + ((int64_t)L.q_rank_p + L.kv_rank_p) * e;
-      if ((rc = vy_latent_decode(q, nk, L.w_ukt, L.w_uv, L.cache, L.c_ss, L.c_st, slots, lengths, max_keys, ao, na, gate, L.n_in,
-                                 (int)B, L.heads, L.dim, L.vdim, L.kv_rank_p, L.scale, mws, s.mix_ws, p->dtype, stream)))
+      if (L.w_uq && (rc = product(p, cq, L.w_uq, q, nk, nk, L.q_rank_p, stream))) return rc;
+      const char* gate = L.gate ? (const char*)in + (nq + L.kv_rank_p) * e : nullptr;
+      if ((rc = vy_latent_decode(L.w_uq ? q : in, L.w_uq ? nk : L.n_in, L.w_ukt, L.w_uv, L.cache, L.c_ss, L.c_st, slots, lengths, max_keys, ao,
+                                 na, gate, L.n_in, L.gate_heads, L.ring ? L.cap : 0, (int)B, L.heads, L.dim, L.vdim, L.kv_rank_p,
+                                 L.scale, mws, s.mix_ws, p->dtype, stream)))
         return rc;
     } else if (L.mixer == VY_MIX_WINDOW) {
       const int64_t gk = (int64_t)L.kv_heads * L.dim, gv = (int64_t)L.kv_heads * L.vdim;
@@ -174,14 +177,18 @@ extern "C" int vy_hybrid_decoder_step(const vy_hybrid_plan* p, const int64_t* id
         prep.m_vp = F->vdim;
       }
       if ((rc = vy_window_decode(in, L.n_in, 0, nk, nk + gk, L.gate ? nk + gk + gv : -1, L.cache, L.c_ss, L.c_sh, L.cap, L.keep, L.rope,
-                                 L.rope_dims, L.rope_len, L.prep || L.values != VY_VALUES_OWN ? &prep : nullptr, slots, lengths, max_keys, ao, na, B, L.heads, L.kv_heads, L.dim, L.vdim, L.scale,
+                                 L.rope_dims, L.rope_len, L.prep || L.values != VY_VALUES_OWN ? &prep : nullptr, L.diff, slots, lengths, max_keys, ao, na, B, L.heads, L.kv_heads, L.dim, L.vdim, L.scale,
                                  L.sink, mws, s.mix_ws, p->dtype, stream))) return rc;
+    } else if (L.mixer == VY_MIX_GATED) {
+      if ((rc = vy_gated_attn(in, L.n_in, 0, nk, 2 * nk, L.state, L.f_bias, L.f_lower, slots, lengths, nullptr, o, nv, B, 1, L.heads, L.dim,
+                              L.vdim, L.silu, nullptr, 0, p->dtype, stream))) return rc;
+      if ((rc = vy_head_norm_gate(o, nv, L.mix_norm, nullptr, 0, ao, na, B, L.heads, L.mix_n, L.vdim, p->eps, p->dtype, stream))) return rc;
     } else {
       if ((rc = vy_decay_attn(in, L.n_in, 0, nk, 2 * nk, L.state, L.decay_pow, slots, lengths, nullptr, o, nv, B, 1, L.heads, L.dim,
                               L.vdim, L.silu, L.rope, L.rope_dims, L.rope_len, L.k_scale, nullptr, 0, p->dtype, stream))) return rc;
       const char* gate = (const char*)in + (2 * nk + nv) * e;
       if (!L.mix_norm) {
-        if ((rc = vy_head_norm_gate(o, nv, gate, L.n_in, ao, na, B, L.heads, L.mix_n, L.vdim, p->eps, p->dtype, stream))) return rc;
+        if ((rc = vy_head_norm_gate(o, nv, nullptr, gate, L.n_in, ao, na, B, L.heads, L.mix_n, L.vdim, p->eps, p->dtype, stream))) return rc;
       } else if ((rc = vy_rmsnorm_gate(o, nv, L.mix_norm, gate, L.n_in, ao, na, B, L.mix_n, nv, p->eps, p->dtype, stream))) return rc;
     }
     vy_routed_rows rows{erows, dp, epos, ew, L.moe ? L.moe->top : 0};
@@ -213,7 +220,9 @@ extern "C" int vy_hybrid_decoder_step(const vy_hybrid_plan* p, const int64_t* id
     }
     if (!chosen && (rc = norm(y, nullptr, L.norm1b, L.norm2, false))) return rc;
     if (L.ff) {
-      if ((rc = gated(p, L, h, gu, act, stream))) return rc;
+      if (L.w_up) rc = product(p, h, L.w_up, act, L.ff, L.ff, dp, stream, nullptr, p->act);
+      else rc = gated(p, L, h, gu, act, stream);
+      if (rc) return rc;
       if ((rc = product(p, act, L.w_down, y, dp, dp, L.ff, stream))) return rc;
     }
     if (chosen) {
@@ -225,5 +234,5 @@ extern "C" int vy_hybrid_decoder_step(const vy_hybrid_plan* p, const int64_t* id
     if (rc) return rc;
     if ((rc = norm(L.ff ? y : nullptr, routed, L.norm2b, next, last))) return rc;
   }
-  return product(p, h, p->head, logits, ldv, p->vocab, dp, stream);
+  return product(p, h, p->head, logits, ldv, p->vocab, dp, stream, nullptr, p->softcap > 0.f ? VY_ACT_SOFTCAP : VY_ACT_NONE, p->softcap);
 }

@@ -26,6 +26,7 @@ struct LatentArgs {
   void* out; int64_t ldo;
   const void* gate; int64_t ldg;
   int B, h, dh, dv, R, nsplit, seqs;
+  int ring, gate_heads;            // rows of a slot's ring (0: rows are positions); one gate per head
   float c;                         // scale * log2(e)
   // workspace
   float* qf;                       // generic: latent queries [B][h][R]
@@ -35,7 +36,8 @@ struct LatentArgs {
 
 __device__ __forceinline__ int row_keys(const LatentArgs& p, int b, int& slot) {
   slot = p.slots ? p.slots[b] : b;
-  return p.start[slot] + 1;
+  const int n = p.start[slot] + 1;
+  return p.ring ? min(n, p.ring) : n;   // (every row of a ring is inside the window: order does not matter)
 }
 // combine over the four lane groups (lane >> 4) of a 16 x 16 MFMA layout
 __device__ __forceinline__ float quad_max(float v) {
@@ -379,7 +381,11 @@ __global__ __launch_bounds__(256) void latent_value_kernel(LatentArgs p) {
     const int64_t b = b0 + r16;
     bf16x4 r;
     float g[4] = {1.f, 1.f, 1.f, 1.f};
-    if (p.gate) {
+    if (p.gate && p.gate_heads) {
+      const float gh = vy_sigmoid((float)((const bf16*)p.gate)[b * p.ldg + head]);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) g[e] = gh;
+    } else if (p.gate) {
       const bf16x4 g4 = *reinterpret_cast<const bf16x4*>((const bf16*)p.gate + b * p.ldg + head * p.dv + nn);
 #pragma unroll
       for (int e = 0; e < 4; ++e) g[e] = vy_sigmoid((float)g4[e]);
@@ -475,7 +481,7 @@ __global__ __launch_bounds__(256) void latent_value_gen_kernel(LatentArgs p) {
     for (int k = lane; k < p.R; k += 64) s = fmaf(VyT<T>::ld(w + k), u[k], s);
     s = vy_wave_sum(s);
     if (lane == 0) {
-      if (p.gate) s *= vy_sigmoid(VyT<T>::ld((const T*)p.gate + (int64_t)b * p.ldg + head * p.dv + n));
+      if (p.gate) s *= vy_sigmoid(VyT<T>::ld((const T*)p.gate + (int64_t)b * p.ldg + (p.gate_heads ? head : head * p.dv + n)));
       VyT<T>::st((T*)p.out + (int64_t)b * p.ldo + head * p.dv + n, s);
     }
   }
@@ -522,11 +528,11 @@ extern "C" int64_t vy_latent_decode_ws_bytes(int32_t B, int32_t h, int32_t R) {
 
 extern "C" int vy_latent_decode(const void* q, int64_t ldq, const void* wukt, const void* wuv, const void* cache, int64_t c_ss,
                                 int64_t c_st, const int32_t* slots, const int32_t* start, int64_t max_keys, void* out,
-                                int64_t ldo, const void* gate, int64_t ldg, int32_t B, int32_t h, int32_t dh, int32_t dv,
+                                int64_t ldo, const void* gate, int64_t ldg, int gate_heads, int32_t ring, int32_t B, int32_t h, int32_t dh, int32_t dv,
                                 int32_t R, float scale, void* ws, int64_t ws_bytes, int dtype, void* stream) {
   const char* who = "vy_latent_decode";
   if (!q || !wukt || !wuv || !cache || !start || !out || !ws) VY_FAIL(VY_ERR_ARG, "%s: null pointer", who);
-  if (B <= 0 || h <= 0 || dh <= 0 || dv <= 0 || R <= 0 || max_keys <= 0) VY_FAIL(VY_ERR_ARG, "%s: empty problem", who);
+  if (B <= 0 || h <= 0 || dh <= 0 || dv <= 0 || R <= 0 || max_keys <= 0 || ring < 0) VY_FAIL(VY_ERR_ARG, "%s: empty problem", who);
   if (dh % 8 || dv % 8 || R % 8 || ldq % 8 || ldo % 8 || ldg % 8 || c_ss % 8 || c_st % 8)
     VY_FAIL(VY_ERR_ARG, "%s: widths and strides must be multiples of 8", who);
   if (R > 1024) VY_FAIL(VY_ERR_UNSUPPORTED, "%s: latent width %d > 1024", who, R);
@@ -535,7 +541,8 @@ extern "C" int vy_latent_decode(const void* q, int64_t ldq, const void* wukt, co
   LatentArgs p{};
   p.q = q; p.ldq = ldq; p.wukt = wukt; p.wuv = wuv; p.cache = cache; p.c_ss = c_ss; p.c_st = c_st;
   p.slots = slots; p.start = start; p.out = out; p.ldo = ldo; p.gate = gate; p.ldg = ldg;
-  p.B = B; p.h = h; p.dh = dh; p.dv = dv; p.R = R; p.c = scale * LOG2E;
+  p.B = B; p.h = h; p.dh = dh; p.dv = dv; p.R = R; p.c = scale * LOG2E; p.ring = ring; p.gate_heads = gate_heads;
+  if (ring && max_keys > ring) max_keys = ring;
   char* w = (char*)ws;
   p.qf = (float*)w; p.qhi = (bf16*)w; p.qlo = p.qhi + (int64_t)B * h * R;
   int64_t s = vy_cdiv(512, (int64_t)B * ((h + 15) / 16));

@@ -8,7 +8,7 @@
 //   vy_latent_norm     the two RMS norms behind a packed [query latent | key/value latent | ...] projection; the
 //                      key/value latent also goes to its cache rows
 //   vy_rmsnorm_gate    RMSNorm(x) * w * sigmoid(gate)
-//   vy_head_norm_gate  x / rms(x) * silu(gate), every head by itself
+//   vy_head_norm_gate  x / rms(x) * w * silu(gate), every head by itself
 #include "vy_common.h"
 
 namespace {
@@ -218,9 +218,9 @@ int residual_norm_any(const ResNormArgs& a, int rms, hipStream_t st) {
 
 struct LatentNormArgs {
   const void* p; int64_t ldp;
-  const float* w_q; void* q_out; int64_t ldq; int nq, npq;        // columns [0, npq), nq of them used
+  const float* w_q; void* q_out; int64_t ldq; int nq, npq;        // columns [0, npq), nq of them used (w_q NULL: no latent)
   const float* w_c; void* c_out; int64_t ldc; int nc, npc;        // columns [npq, npq + npc)
-  void* cache; int64_t c_ss, c_st; int cap;                       // cache rows: strides per slot and per token
+  void* cache; int64_t c_ss, c_st; int cap, ring;                 // cache rows: strides per slot and per token
   const int* slots; const int* start; const int* count;
   int64_t M; int L; float eps;
 };
@@ -231,9 +231,10 @@ __global__ __launch_bounds__(256) void latent_norm_kernel(LatentNormArgs a) {
   constexpr int VEC = VyChunk<T>::VEC;
   const int lane = threadIdx.x & 63;
   const int64_t u = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
-  if (u >= 2 * a.M) return;
-  const bool kv = u & 1;
-  const int64_t row = u >> 1;
+  const bool both = a.w_q != nullptr;
+  if (u >= (both ? 2 * a.M : a.M)) return;
+  const bool kv = !both || (u & 1);
+  const int64_t row = both ? u >> 1 : u;
   const int n = kv ? a.nc : a.nq, np = kv ? a.npc : a.npq;
   const T* src = (const T*)a.p + row * a.ldp + (kv ? a.npq : 0);
   const float* w = kv ? a.w_c : a.w_q;
@@ -254,8 +255,9 @@ __global__ __launch_bounds__(256) void latent_norm_kernel(LatentNormArgs a) {
   if (kv && a.cache) {
     const int b = (int)(row / a.L), l = (int)(row - (int64_t)b * a.L);
     const int slot = a.slots ? a.slots[b] : b;
-    const int pos = a.start[slot] + l;
-    if (l < (a.count ? a.count[b] : a.L) && pos < a.cap) cdst = (T*)a.cache + slot * a.c_ss + pos * a.c_st;
+    const int pos = a.start[slot] + l, n = a.count ? a.count[b] : a.L;
+    const bool held = a.ring ? l + a.cap >= n : pos < a.cap;      // (of a ring: not overwritten by a later one of these tokens)
+    if (l < n && held) cdst = (T*)a.cache + slot * a.c_ss + (a.ring ? pos % a.cap : pos) * a.c_st;
   }
 #pragma unroll
   for (int c = 0; c < CH; ++c) {
@@ -272,9 +274,9 @@ __global__ __launch_bounds__(256) void latent_norm_kernel(LatentNormArgs a) {
 
 template <typename T>
 int latent_norm_go(const LatentNormArgs& a, hipStream_t st) {
-  const int np = a.npq > a.npc ? a.npq : a.npc;
+  const int np = a.w_q && a.npq > a.npc ? a.npq : a.npc;
   const int nch = (np + VyChunk<T>::VEC - 1) / VyChunk<T>::VEC;
-  const dim3 grid((unsigned)vy_cdiv(2 * a.M, 4)), block(256);
+  const dim3 grid((unsigned)vy_cdiv(a.w_q ? 2 * a.M : a.M, 4)), block(256);
   if (nch <= 64) hipLaunchKernelGGL((latent_norm_kernel<T, 1>), grid, block, 0, st, a);
   else if (nch <= 128) hipLaunchKernelGGL((latent_norm_kernel<T, 2>), grid, block, 0, st, a);
   else if (nch <= 256) hipLaunchKernelGGL((latent_norm_kernel<T, 4>), grid, block, 0, st, a);
@@ -318,8 +320,8 @@ __global__ __launch_bounds__(256) void rmsnorm_gate_kernel(const T* __restrict__
 
 // LPH lanes per head (a power of two up to a wave), one 16-byte chunk per lane and pass
 template <typename T, int LPH>
-__global__ __launch_bounds__(256) void head_norm_gate_kernel(const T* __restrict__ x, int64_t ldx, const T* __restrict__ gate,
-                                                             int64_t ldg, T* __restrict__ y, int64_t ldy, int64_t units, int heads,
+__global__ __launch_bounds__(256) void head_norm_gate_kernel(const T* __restrict__ x, int64_t ldx, const float* __restrict__ w,
+                                                             const T* __restrict__ gate, int64_t ldg, T* __restrict__ y, int64_t ldy, int64_t units, int heads,
                                                              int N, int NP, float eps) {
   constexpr int VEC = VyChunk<T>::VEC;
   const int sub = threadIdx.x % LPH;
@@ -327,11 +329,11 @@ __global__ __launch_bounds__(256) void head_norm_gate_kernel(const T* __restrict
   const int64_t uc = u < units ? u : units - 1, row = uc / heads;
   const int head = (int)(uc - row * heads);
   const T* xr = x + row * ldx + (int64_t)head * NP;
-  const T* gr = gate + row * ldg + (int64_t)head * NP;
+  const T* gr = gate ? gate + row * ldg + (int64_t)head * NP : nullptr;
   float v[VEC], g[VEC], q = 0.f;
   for (int c = sub * VEC; c < NP; c += LPH * VEC) {
     VyChunk<T>::load(xr + c, v);
-    VyChunk<T>::load(gr + c, g);
+    if (gr) VyChunk<T>::load(gr + c, g);
 #pragma unroll
     for (int e = 0; e < VEC; ++e) q += v[e] * v[e];   // (the padding columns are zero)
   }
@@ -342,20 +344,33 @@ __global__ __launch_bounds__(256) void head_norm_gate_kernel(const T* __restrict
   for (int c = sub * VEC; c < NP; c += LPH * VEC) {
     if (LPH * VEC < NP) {   // several passes: read again (from cache)
       VyChunk<T>::load(xr + c, v);
-      VyChunk<T>::load(gr + c, g);
+      if (gr) VyChunk<T>::load(gr + c, g);
     }
 #pragma unroll
-    for (int e = 0; e < VEC; ++e) v[e] = v[e] * rstd * vy_silu(g[e]);
+    for (int e = 0; e < VEC; ++e) v[e] *= rstd;
+    if (w) {
+#pragma unroll
+      for (int e = 0; e < VEC; e += 4) {
+        float f[4];
+        load4<float>(w + c + e, f);
+#pragma unroll
+        for (int i = 0; i < 4; ++i) v[e + i] *= f[i];
+      }
+    }
+    if (gr) {
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) v[e] *= vy_silu(g[e]);
+    }
     VyChunk<T>::store(y + row * ldy + (int64_t)head * NP + c, v);
   }
 }
 
 template <typename T>
-void head_norm_gate_go(const void* x, int64_t ldx, const void* gate, int64_t ldg, void* y, int64_t ldy, int64_t M, int heads, int N,
+void head_norm_gate_go(const void* x, int64_t ldx, const float* w, const void* gate, int64_t ldg, void* y, int64_t ldy, int64_t M, int heads, int N,
                        int NP, float eps, hipStream_t st) {
   const int nch = NP / VyChunk<T>::VEC;
   const int64_t units = M * heads;
-#define HN_GO(L) hipLaunchKernelGGL((head_norm_gate_kernel<T, L>), dim3((unsigned)vy_cdiv(units, 256 / L)), dim3(256), 0, st, (const T*)x, ldx, (const T*)gate, ldg, (T*)y, ldy, units, heads, N, NP, eps)
+#define HN_GO(L) hipLaunchKernelGGL((head_norm_gate_kernel<T, L>), dim3((unsigned)vy_cdiv(units, 256 / L)), dim3(256), 0, st, (const T*)x, ldx, w, (const T*)gate, ldg, (T*)y, ldy, units, heads, N, NP, eps)
   if (nch <= 1) HN_GO(1);
   else if (nch <= 4) HN_GO(4);
   else if (nch <= 8) HN_GO(8);
@@ -415,15 +430,15 @@ extern "C" int vy_residual_norm_routed(float* x, int64_t ldx, const void* y, int
 
 extern "C" int vy_latent_norm(const void* p, int64_t ldp, const float* w_q, void* q_out, int64_t ldq, int32_t nq, int32_t npq,
                               const float* w_c, void* c_out, int64_t ldc, int32_t nc, int32_t npc, void* cache, int64_t c_ss,
-                              int64_t c_st, int32_t cap, const int32_t* slots, const int32_t* start, const int32_t* count,
-                              int64_t B, int64_t L, float eps, int dtype, void* stream) {
+                              int64_t c_st, int32_t cap, int ring, const int32_t* slots, const int32_t* start,
+                              const int32_t* count, int64_t B, int64_t L, float eps, int dtype, void* stream) {
   const char* who = "vy_latent_norm";
   const int vec = dtype == VY_BF16 ? 8 : 4;
-  if (!p || !w_q || !q_out || !w_c || B <= 0 || L <= 0 || nq <= 0 || nc <= 0 || npq < nq || npc < nc) VY_FAIL(VY_ERR_ARG, "%s: bad arguments", who);
+  if (!p || !w_c || B <= 0 || L <= 0 || nc <= 0 || npq < 0 || npc < nc || (w_q && (!q_out || nq <= 0 || npq < nq))) VY_FAIL(VY_ERR_ARG, "%s: bad arguments", who);
   if (npq % vec || npc % vec || ldp % vec || ldq % vec || ldc % vec || c_ss % vec || c_st % vec)
     VY_FAIL(VY_ERR_ARG, "%s: widths and strides must be multiples of %d", who, vec);
   if (cache && (!start || cap <= 0)) VY_FAIL(VY_ERR_ARG, "%s: cache without start positions / capacity", who);
-  LatentNormArgs a{p, ldp, w_q, q_out, ldq, nq, npq, w_c, c_out, ldc, nc, npc, cache, c_ss, c_st, cap, slots, start, count,
+  LatentNormArgs a{p, ldp, w_q, q_out, ldq, nq, npq, w_c, c_out, ldc, nc, npc, cache, c_ss, c_st, cap, ring, slots, start, count,
                    B * L, (int)L, eps};
   int rc;
   if (dtype == VY_BF16) rc = latent_norm_go<bf16>(a, (hipStream_t)stream);
@@ -434,16 +449,16 @@ extern "C" int vy_latent_norm(const void* p, int64_t ldp, const float* w_q, void
   return VY_OK;
 }
 
-extern "C" int vy_head_norm_gate(const void* x, int64_t ldx, const void* gate, int64_t ldg, void* y, int64_t ldy, int64_t M,
-                                 int32_t heads, int64_t N, int64_t NP, float eps, int dtype, void* stream) {
+extern "C" int vy_head_norm_gate(const void* x, int64_t ldx, const float* w, const void* gate, int64_t ldg, void* y, int64_t ldy,
+                                 int64_t M, int32_t heads, int64_t N, int64_t NP, float eps, int dtype, void* stream) {
   const char* who = "vy_head_norm_gate";
   if (dtype != VY_BF16 && dtype != VY_F32) VY_FAIL(VY_ERR_ARG, "%s: bad dtype %d", who, dtype);
   const int vec = dtype == VY_BF16 ? 8 : 4;
-  if (!x || !gate || !y || M <= 0 || heads <= 0 || N <= 0 || NP < N || NP > 1 << 20 || M * heads > INT32_MAX)
+  if (!x || !y || M <= 0 || heads <= 0 || N <= 0 || NP < N || NP > 1 << 20 || M * heads > INT32_MAX)
     VY_FAIL(VY_ERR_ARG, "%s: bad arguments", who);
   if (NP % vec || ldx % vec || ldg % vec || ldy % vec) VY_FAIL(VY_ERR_ARG, "%s: widths and strides must be multiples of %d", who, vec);
-  if (dtype == VY_BF16) head_norm_gate_go<bf16>(x, ldx, gate, ldg, y, ldy, M, heads, (int)N, (int)NP, eps, (hipStream_t)stream);
-  else head_norm_gate_go<float>(x, ldx, gate, ldg, y, ldy, M, heads, (int)N, (int)NP, eps, (hipStream_t)stream);
+  if (dtype == VY_BF16) head_norm_gate_go<bf16>(x, ldx, w, gate, ldg, y, ldy, M, heads, (int)N, (int)NP, eps, (hipStream_t)stream);
+  else head_norm_gate_go<float>(x, ldx, w, gate, ldg, y, ldy, M, heads, (int)N, (int)NP, eps, (hipStream_t)stream);
   VY_CHECK_LAUNCH(who);
   return VY_OK;
 }

@@ -132,7 +132,7 @@ int vy_parallel_decode(const vy_hybrid_plan* p, const vy_hybrid_layer* L, const 
   const int B = p->B;
   const int64_t n = d ? (int64_t)B * d->top : 0;
   if (p->dtype != VY_BF16 || L->form != VY_FORM_PARALLEL || L->mixer != VY_MIX_WINDOW || B > 64 || L->dim > 256 || L->vdim > 256 ||
-      (L->ff && !L->clamped) || n > MAX_ENTRIES || (d && (d->experts > 256 || d->act != VY_MOE_CLAMPED)) || !L->gate || L->prep)
+      (L->ff && !L->clamped) || n > MAX_ENTRIES || (d && (d->experts > 256 || d->act != VY_MOE_CLAMPED)) || !L->gate || L->prep || L->diff || L->b_in)
     return VY_ERR_UNSUPPORTED;
   const int64_t nk = (int64_t)L->heads * L->dim, gk = (int64_t)L->kv_heads * L->dim, gv = (int64_t)L->kv_heads * L->vdim,
                 nv = (int64_t)L->heads * L->vdim, na = nv + L->ff, n_in = nk + gk + gv + nv + 2 * (int64_t)L->ff;

@@ -9,7 +9,12 @@
 // key and value never make the trip to memory and back: they replace its row of the ring in registers / LDS.
 //
 // The norms over the whole query and key projection (DecodeArgs::q_norm) are part of it: every workgroup adds up the squares of
-// the sequence's projection rows itself (a few KB from L2), in fp32, and the rotated operand is rounded once.
+// the sequence's projection rows itself (a few KB from L2), in fp32, and the rotated operand is rounded once.  Norms over groups
+// of columns (DecodeArgs::group) need no more than the group's own lanes.
+//
+// MAPS = 2, differential attention: a head's queries and keys are two maps side by side (a row of the ring is [key 1 | key 2 |
+// value]), each with a softmax of its own over the same values: one stream of the ring, one value fragment for both.  The maps'
+// partial results always go through window_finish_diff.
 #pragma once
 #include "vy_common.h"
 #include <float.h>
@@ -22,7 +27,8 @@ struct DecodeArgs {
   const bf16* p; int64_t ldp, oq, ok, ov, og;
   bf16* ring; int64_t r_ss, r_sh; int R, keep;
   const float2* rope; int half, rope_len;
-  const float* q_norm; const float* k_norm; int n_q, n_k; float eps;   // nullable: norms over the whole projections
+  const float* q_norm; const float* k_norm; int n_q, n_k; float eps;   // nullable: norms over the whole projections ...
+  int group, temp_every; float temp_coef;                              // ... or (group > 0) over groups; temperature of the query
   const bf16* vm; int64_t ldm; float lambda;                           // nullable: values mixed in
   int n_v, m_v, m_vp;                                                  // used columns of v's heads and of vm's, and vm's padded ones
   bf16* vo; int64_t ldvo;                                              // nullable: receives the token's own values
@@ -30,7 +36,8 @@ struct DecodeArgs {
   bf16* out; int64_t ldo;
   int h, hk, dim, vdim, ns, passes, sink;   // ns slices of the ring, passes of 16 query heads per key/value head
   float scale;
-  float* part_o; float* part_ml;            // ns > 1: [b][head][slice][vdim] and [b][head][slice][2]
+  float* part_o; float* part_ml;            // ns > 1: [b][head][slice][vdim] and [b][head][slice][2] (head: head * MAPS + map)
+  float lambda2, out_scale, eps_out;        // MAPS = 2: the difference's weight, the outputs' factor and norm
 };
 
 __device__ __forceinline__ float group_max(float v) {   // over the four lane groups (lane >> 4)
@@ -52,6 +59,11 @@ __device__ __forceinline__ float group_sum(float v) {
 
 // row of position p in a ring of R rows whose first `keep` stay
 __device__ __forceinline__ int ring_row(int p, int R, int keep) { return p < R ? p : keep + (p - keep) % (R - keep); }
+
+// factor on the query of a position
+__device__ __forceinline__ float query_temperature(int pos, int every, float coef) {
+  return every > 0 ? 1.f + coef * logf((float)((pos + 1) / every + 1)) : 1.f;
+}
 
 // 8 columns d0 .. of a head times r w (w nullable: as they are), rotated, rounded once
 __device__ __forceinline__ bf16x8 rotate8(const DecodeArgs& a, const float2* t, int d0, bf16x8 x, const float* w, float r) {
@@ -103,7 +115,8 @@ __device__ __forceinline__ float rms_factor(float sum, int n, float eps) {
   return r * (1.5f - 0.5f * ms * r * r);
 }
 
-template <int DHP, int DVP>
+// DHP, DVP: padded widths of a map's keys and of the values (DecodeArgs::dim is a map's)
+template <int DHP, int DVP, int MAPS = 1>
 struct WindowDecode {
   static constexpr int KS = DHP / 32, NDB = DVP / 16;
   static constexpr int VPITCH = (DVP + 8) * 2;              // bytes per row of a wave's value tile
@@ -111,7 +124,7 @@ struct WindowDecode {
   static constexpr int VPL = 32 * VC / 64;                  // value chunks per lane and unit
   static constexpr int QP = DHP + 8;                        // query pitch (elements)
   // [value tiles, later the waves' results | queries | new key | new value | m, l of the waves]
-  static constexpr int O_Q = 4 * VROWS, O_K = O_Q + 16 * QP * 2, O_V = O_K + DHP * 2, O_ML = O_V + DVP * 2;
+  static constexpr int O_Q = 4 * VROWS, O_K = O_Q + MAPS * 16 * QP * 2, O_V = O_K + MAPS * DHP * 2, O_ML = O_V + DVP * 2;
   static_assert(4 * 16 * DVP * 4 <= 4 * VROWS, "the waves' results fit over the value tiles");
   static_assert(2 * 64 * 4 >= 8 * 4, "the norms' partial sums fit over m, l");
   static constexpr int LDS = O_ML + 2 * 64 * 4;
@@ -126,7 +139,7 @@ struct WindowDecode {
   const int slot = a.slots ? a.slots[b] : b;
   const int pos = a.start[slot];
   const int n = min(pos + 1, a.R), fresh = ring_row(pos, a.R, a.keep);
-  const int W = a.dim + a.vdim;
+  const int KW = MAPS * a.dim, W = KW + a.vdim;
   const bf16* row = a.p + (int64_t)b * a.ldp;
   bf16* ring = a.ring + (int64_t)slot * a.r_ss + (int64_t)g * a.r_sh;
   const float2* trig = a.rope + (int64_t)min(pos, a.rope_len - 1) * a.half;
@@ -135,28 +148,30 @@ struct WindowDecode {
   int u = slice * 4 + wave;
 
   // keys and values of a unit in registers: key rows as MFMA operands, values chunk by chunk (whole rows per instruction)
-  bf16x8 kf[2][KS], vr[VPL];
-  auto request = [&](int unit, bf16x8 (&kd)[2][KS], bf16x8 (&vd)[VPL]) {
+  bf16x8 kf[MAPS][2][KS], vr[VPL];
+  auto request = [&](int unit, bf16x8 (&kd)[MAPS][2][KS], bf16x8 (&vd)[VPL]) {
 #pragma unroll
     for (int blk = 0; blk < 2; ++blk) {
       const int j = min(unit * 32 + 16 * blk + r16, n - 1);
 #pragma unroll
-      for (int ks = 0; ks < KS; ++ks) {
-        const int d0 = 32 * ks + 8 * kq;
-        kd[blk][ks] = d0 < a.dim ? *reinterpret_cast<const bf16x8*>(ring + (int64_t)j * W + d0) : zero8;
-      }
+      for (int m = 0; m < MAPS; ++m)
+#pragma unroll
+        for (int ks = 0; ks < KS; ++ks) {
+          const int d0 = 32 * ks + 8 * kq;
+          kd[m][blk][ks] = d0 < a.dim ? *reinterpret_cast<const bf16x8*>(ring + (int64_t)j * W + m * a.dim + d0) : zero8;
+        }
     }
 #pragma unroll
     for (int i = 0; i < VPL; ++i) {
       const int c = lane + 64 * i, j = min(unit * 32 + c / VC, n - 1), d0 = (c % VC) * 8;
-      vd[i] = d0 < a.vdim ? *reinterpret_cast<const bf16x8*>(ring + (int64_t)j * W + a.dim + d0) : zero8;
+      vd[i] = d0 < a.vdim ? *reinterpret_cast<const bf16x8*>(ring + (int64_t)j * W + KW + d0) : zero8;
     }
   };
   if (u < units) request(u, kf, vr);
 
   // sums of squares of the sequence's whole query and key projections
   float rq = 1.f, rk = 1.f;
-  if (a.q_norm) {
+  if (a.q_norm && a.group == 0) {
     float* red = reinterpret_cast<float*>(smem + O_ML);
     float sq = 0.f, sk = 0.f;
     auto squares = [&](const bf16* p, int cols, float& s) {
@@ -180,24 +195,43 @@ struct WindowDecode {
   bf16* lq = reinterpret_cast<bf16*>(smem + O_Q);
   bf16* lk = reinterpret_cast<bf16*>(smem + O_K);
   bf16* lv = reinterpret_cast<bf16*>(smem + O_V);
-  for (int i = tid; i < 16 * (DHP / 8); i += 256) {
-    const int hh = i / (DHP / 8), d0 = (i % (DHP / 8)) * 8;
+  constexpr int CPG = DHP / 8;                 // lanes (chunks) of a head's map, neighbours
+  auto group_factor = [&](const bf16x8 x, int count) {   // every lane of the wave is here: rms of the map's columns
+    float s = 0.f;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) s = fmaf((float)x[e], (float)x[e], s);
+#pragma unroll
+    for (int o = CPG / 2; o > 0; o >>= 1) s += __shfl_xor(s, o, 64);
+    return rms_factor(s, count, a.eps);
+  };
+  const float temp = query_temperature(pos, a.temp_every, a.temp_coef);
+  static_assert(MAPS * 16 * CPG % 64 == 0, "whole waves");
+  for (int i = tid; i < MAPS * 16 * CPG; i += 256) {
+    const int hm = i / CPG, hh = hm / MAPS, mp = hm % MAPS, d0 = (i % CPG) * 8;
     const bool ok = hh < nh && d0 < a.dim;
     bf16x8 q = zero8;
-    const int at = (h0 + hh) * a.dim + d0;
-    if (ok) q = rotate8(a, trig, d0, *reinterpret_cast<const bf16x8*>(row + a.oq + at), a.q_norm ? a.q_norm + at : nullptr, rq);
-    *reinterpret_cast<bf16x8*>(lq + hh * QP + d0) = q;
+    const int at = (h0 + hh) * KW + mp * a.dim + d0;
+    if (ok) q = *reinterpret_cast<const bf16x8*>(row + a.oq + at);
+    float f = rq;
+    if (a.q_norm && a.group) f = group_factor(q, a.n_q) * temp;
+    if (ok) q = rotate8(a, trig, d0, q, a.q_norm ? a.q_norm + at : nullptr, f);
+    *reinterpret_cast<bf16x8*>(lq + (mp * 16 + hh) * QP + d0) = q;
   }
   const bool owner = pass == 0 && (fresh / 32) % step / 4 == slice;   // the workgroup whose units hold the new row
-  if (tid >= 192 && tid - 192 < DHP / 8) {
-    const int d0 = (tid - 192) * 8;
+  static_assert(MAPS * CPG <= 64, "a new key is one wave's");
+  if (tid >= 192) {
+    const int mp = (tid - 192) / CPG, d0 = (tid - 192) % CPG * 8;
+    const bool ok = mp < MAPS && d0 < a.dim;
     bf16x8 k8 = zero8;
-    if (d0 < a.dim) {
-      const int at = g * a.dim + d0;
-      k8 = rotate8(a, trig, d0, *reinterpret_cast<const bf16x8*>(row + a.ok + at), a.k_norm ? a.k_norm + at : nullptr, rk);
-      if (owner) *reinterpret_cast<bf16x8*>(ring + (int64_t)fresh * W + d0) = k8;
+    const int at = g * KW + mp * a.dim + d0;
+    if (ok) k8 = *reinterpret_cast<const bf16x8*>(row + a.ok + at);
+    float f = rk;
+    if (a.k_norm && a.group) f = group_factor(k8, a.n_k);
+    if (ok) {
+      k8 = rotate8(a, trig, d0, k8, a.k_norm ? a.k_norm + at : nullptr, f);
+      if (owner) *reinterpret_cast<bf16x8*>(ring + (int64_t)fresh * W + mp * a.dim + d0) = k8;
     }
-    *reinterpret_cast<bf16x8*>(lk + d0) = k8;
+    if (mp < MAPS) *reinterpret_cast<bf16x8*>(lk + mp * DHP + d0) = k8;
   } else if (tid >= 128 && tid < 192 && tid - 128 < VC) {
     const int d0 = (tid - 128) * 8;
     bf16x8 v8 = zero8;
@@ -211,19 +245,26 @@ struct WindowDecode {
 #pragma unroll
         for (int e = 0; e < 8; ++e) v8[e] = (bf16)v[e];
       }
-      if (owner) *reinterpret_cast<bf16x8*>(ring + (int64_t)fresh * W + a.dim + d0) = v8;
+      if (owner) *reinterpret_cast<bf16x8*>(ring + (int64_t)fresh * W + KW + d0) = v8;
     }
     *reinterpret_cast<bf16x8*>(lv + d0) = v8;
   }
   __syncthreads();
-  bf16x8 qf[KS];
+  bf16x8 qf[MAPS][KS];
 #pragma unroll
-  for (int ks = 0; ks < KS; ++ks) qf[ks] = *reinterpret_cast<const bf16x8*>(lq + r16 * QP + 32 * ks + 8 * kq);
+  for (int m = 0; m < MAPS; ++m)
+#pragma unroll
+    for (int ks = 0; ks < KS; ++ks) qf[m][ks] = *reinterpret_cast<const bf16x8*>(lq + (m * 16 + r16) * QP + 32 * ks + 8 * kq);
 
-  f32x4 o[NDB];
+  f32x4 o[MAPS][NDB];
+  float m_run[MAPS], l_run[MAPS];
 #pragma unroll
-  for (int d = 0; d < NDB; ++d) o[d] = f32x4{0.f, 0.f, 0.f, 0.f};
-  float m_run = -FLT_MAX, l_run = 0.f;
+  for (int m = 0; m < MAPS; ++m) {
+    m_run[m] = -FLT_MAX;
+    l_run[m] = 0.f;
+#pragma unroll
+    for (int d = 0; d < NDB; ++d) o[m][d] = f32x4{0.f, 0.f, 0.f, 0.f};
+  }
   const float c = a.scale * LOG2E;
   char* vt = smem + wave * VROWS;
   const unsigned vtr = vy_lds_addr(vt) + (4 * kq + (r16 >> 2)) * VPITCH + (4 * (r16 & 3)) * 2;
@@ -235,7 +276,9 @@ struct WindowDecode {
         for (int blk = 0; blk < 2; ++blk)
           if (blk == ((fresh >> 4) & 1))
 #pragma unroll
-            for (int ks = 0; ks < KS; ++ks) kf[blk][ks] = *reinterpret_cast<const bf16x8*>(lk + 32 * ks + 8 * kq);
+            for (int m = 0; m < MAPS; ++m)
+#pragma unroll
+              for (int ks = 0; ks < KS; ++ks) kf[m][blk][ks] = *reinterpret_cast<const bf16x8*>(lk + m * DHP + 32 * ks + 8 * kq);
       }
 #pragma unroll
       for (int i = 0; i < VPL; ++i) {
@@ -253,39 +296,44 @@ struct WindowDecode {
       const int cc = lane + 64 * i;
       *reinterpret_cast<bf16x8*>(vt + (cc / VC) * VPITCH + (cc % VC) * 16) = vr[i];
     }
-    f32x4 sc[2];
+    f32x4 sc[MAPS][2];
 #pragma unroll
-    for (int blk = 0; blk < 2; ++blk) {
-      sc[blk] = f32x4{0.f, 0.f, 0.f, 0.f};
+    for (int m = 0; m < MAPS; ++m)
 #pragma unroll
-      for (int ks = 0; ks < KS; ++ks) sc[blk] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[blk][ks], qf[ks], sc[blk], 0, 0, 0);
-    }
+      for (int blk = 0; blk < 2; ++blk) {
+        sc[m][blk] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int ks = 0; ks < KS; ++ks) sc[m][blk] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[m][blk][ks], qf[m][ks], sc[m][blk], 0, 0, 0);
+      }
     if (u + step < units) request(u + step, kf, vr);   // lands under this unit's softmax and value product
-    float tmax = -INFINITY;
+    bf16x8 pf[MAPS];
 #pragma unroll
-    for (int blk = 0; blk < 2; ++blk)
+    for (int m = 0; m < MAPS; ++m) {
+      float tmax = -INFINITY;
 #pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        if (j0 + 16 * blk + 4 * kq + r >= n) sc[blk][r] = -INFINITY;
-        tmax = fmaxf(tmax, sc[blk][r]);
-      }
-    const float m_new = fmaxf(m_run, group_max(tmax) * c);
-    const float alpha = __builtin_amdgcn_exp2f(m_run - m_new);
-    m_run = m_new;
-    l_run *= alpha;
+      for (int blk = 0; blk < 2; ++blk)
 #pragma unroll
-    for (int d = 0; d < NDB; ++d)
+        for (int r = 0; r < 4; ++r) {
+          if (j0 + 16 * blk + 4 * kq + r >= n) sc[m][blk][r] = -INFINITY;
+          tmax = fmaxf(tmax, sc[m][blk][r]);
+        }
+      const float m_new = fmaxf(m_run[m], group_max(tmax) * c);
+      const float alpha = __builtin_amdgcn_exp2f(m_run[m] - m_new);
+      m_run[m] = m_new;
+      l_run[m] *= alpha;
 #pragma unroll
-      for (int r = 0; r < 4; ++r) o[d][r] *= alpha;
-    bf16x8 pf;
+      for (int d = 0; d < NDB; ++d)
 #pragma unroll
-    for (int blk = 0; blk < 2; ++blk)
+        for (int r = 0; r < 4; ++r) o[m][d][r] *= alpha;
 #pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const float e = __builtin_amdgcn_exp2f(fmaf(sc[blk][r], c, -m_run));
-        l_run += e;
-        pf[4 * blk + r] = (bf16)e;
-      }
+      for (int blk = 0; blk < 2; ++blk)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const float e = __builtin_amdgcn_exp2f(fmaf(sc[m][blk][r], c, -m_run[m]));
+          l_run[m] += e;
+          pf[m][4 * blk + r] = (bf16)e;
+        }
+    }
     vy_static_for<NDB>([&](auto d_c) {
       constexpr int d = decltype(d_c)::value;
       union { struct { s16x4 a, b; } hh; bf16x8 v; } uu;
@@ -293,27 +341,30 @@ struct WindowDecode {
       uu.hh.b = vy_lds_tr16_off<d * 32 + 16 * VPITCH>(vtr);
       asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
       vy_tie(uu.v);
-      o[d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(uu.v, pf, o[d], 0, 0, 0);
+#pragma unroll
+      for (int m = 0; m < MAPS; ++m) o[m][d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(uu.v, pf[m], o[m][d], 0, 0, 0);
     });
   }
-  l_run = group_sum(l_run);
 
-  // the four waves' results through LDS
+  // the four waves' results through LDS, map by map
+#pragma unroll
+  for (int mp = 0; mp < MAPS; ++mp) {
+  l_run[mp] = group_sum(l_run[mp]);
   __syncthreads();
   float* lo = reinterpret_cast<float*>(smem);                    // [wave][head][DVP]
   float* lml = reinterpret_cast<float*>(smem + O_ML);            // m [wave][16], l [wave][16]
 #pragma unroll
-  for (int d = 0; d < NDB; ++d) *reinterpret_cast<f32x4*>(lo + (wave * 16 + r16) * DVP + 16 * d + 4 * kq) = o[d];
+  for (int d = 0; d < NDB; ++d) *reinterpret_cast<f32x4*>(lo + (wave * 16 + r16) * DVP + 16 * d + 4 * kq) = o[mp][d];
   if (kq == 0) {
-    lml[wave * 16 + r16] = m_run;
-    lml[64 + wave * 16 + r16] = l_run;
+    lml[wave * 16 + r16] = m_run[mp];
+    lml[64 + wave * 16 + r16] = l_run[mp];
   }
   __syncthreads();
   for (int i = tid; i < nh * (a.vdim / 8); i += 256) {
     const int hh = i / (a.vdim / 8), d0 = (i % (a.vdim / 8)) * 8, head = h0 + hh;
     float m = fmaxf(fmaxf(lml[hh], lml[16 + hh]), fmaxf(lml[32 + hh], lml[48 + hh]));
-    if (a.ns == 1 && a.sink) m = fmaxf(m, 0.f);
-    float l = a.ns == 1 && a.sink ? __builtin_amdgcn_exp2f(-m) : 0.f, v[8];
+    if (MAPS == 1 && a.ns == 1 && a.sink) m = fmaxf(m, 0.f);
+    float l = MAPS == 1 && a.ns == 1 && a.sink ? __builtin_amdgcn_exp2f(-m) : 0.f, v[8];
 #pragma unroll
     for (int e = 0; e < 8; ++e) v[e] = 0.f;
 #pragma unroll
@@ -323,7 +374,7 @@ struct WindowDecode {
 #pragma unroll
       for (int e = 0; e < 8; ++e) v[e] = fmaf(s, lo[(w * 16 + hh) * DVP + d0 + e], v[e]);
     }
-    if (a.ns == 1) {
+    if (MAPS == 1 && a.ns == 1) {
       const float inv = 1.f / l;
       bf16x8 w8;
 #pragma unroll
@@ -337,11 +388,12 @@ struct WindowDecode {
       for (int e = 0; e < 8; ++e) w8[e] = (bf16)v[e];
       *reinterpret_cast<bf16x8*>(a.out + (int64_t)b * a.ldo + (int64_t)head * a.vdim + d0) = w8;
     } else {
-      const int64_t at = ((int64_t)b * a.h + head) * a.ns + slice;
+      const int64_t at = (((int64_t)b * a.h + head) * MAPS + mp) * a.ns + slice;
       VyChunk<float>::store(a.part_o + at * a.vdim + d0, v);
       VyChunk<float>::store(a.part_o + at * a.vdim + d0 + 4, v + 4);
       if (d0 == 0) { a.part_ml[2 * at] = m; a.part_ml[2 * at + 1] = l; }
     }
+  }
   }
 }
 };
@@ -388,6 +440,56 @@ __device__ __forceinline__ void window_finish(const DecodeArgs& a, float* red, i
     bf16x4 w;
 #pragma unroll
     for (int e = 0; e < 4; ++e) w[e] = (bf16)v[e];
+    *reinterpret_cast<bf16x4*>(a.out + (int64_t)b * a.ldo + (int64_t)head * a.vdim + ch * 4) = w;
+  }
+}
+
+// one workgroup per (sequence, head): both maps' slices, their difference, the head's norm.  vdim <= 1024.
+constexpr int FINISH_DIFF_LDS = FINISH_LDS + 16;
+__device__ __forceinline__ void window_finish_diff(const DecodeArgs& a, float* red, int head, int b) {
+  const int tid = threadIdx.x;
+  const int nc = a.vdim / 4, lanes = nc <= 64 ? 64 : nc <= 128 ? 128 : 256, groups = 256 / lanes;
+  const int ch = tid % lanes, grp = tid / lanes;
+  f32x4 o = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+  for (int mp = 0; mp < 2; ++mp) {
+    const float* ml = a.part_ml + (((int64_t)b * a.h + head) * 2 + mp) * a.ns * 2;
+    const float* po = a.part_o + (((int64_t)b * a.h + head) * 2 + mp) * a.ns * a.vdim;
+    float m = -FLT_MAX, l = 0.f;
+    for (int s = 0; s < a.ns; ++s) m = fmaxf(m, ml[2 * s]);
+#pragma unroll 4
+    for (int s = 0; s < a.ns; ++s) l += ml[2 * s + 1] * __builtin_amdgcn_exp2f(ml[2 * s] - m);
+    const float w = (mp ? -a.lambda2 : 1.f) / l;
+    if (ch < nc) {
+#pragma unroll 4
+      for (int s = grp; s < a.ns; s += groups) {
+        const float f = __builtin_amdgcn_exp2f(ml[2 * s] - m) * w;
+        const f32x4 x = *reinterpret_cast<const f32x4*>(po + (int64_t)s * a.vdim + ch * 4);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) o[e] = fmaf(f, x[e], o[e]);
+      }
+    }
+  }
+  *reinterpret_cast<f32x4*>(red + tid * 4) = o;
+  __syncthreads();
+  float sq = 0.f;
+  if (grp == 0 && ch < nc) {
+    for (int s = 1; s < groups; ++s) {
+      const f32x4 x = *reinterpret_cast<const f32x4*>(red + (s * lanes + ch) * 4);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) o[e] += x[e];
+    }
+#pragma unroll
+    for (int e = 0; e < 4; ++e) sq = fmaf(o[e], o[e], sq);   // (padded columns are zero)
+  }
+  sq = vy_wave_sum(sq);
+  if ((tid & 63) == 0) red[1024 + (tid >> 6)] = sq;
+  __syncthreads();
+  if (grp == 0 && ch < nc) {
+    const float f = rms_factor(red[1024] + red[1025] + red[1026] + red[1027], a.n_v, a.eps_out) * a.out_scale;
+    bf16x4 w;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) w[e] = (bf16)(o[e] * f);
     *reinterpret_cast<bf16x4*>(a.out + (int64_t)b * a.ldo + (int64_t)head * a.vdim + ch * 4) = w;
   }
 }

@@ -6,12 +6,13 @@
 //
 //   vy_window_rows     prefill: rotary positions on the new keys (in place in the packed projection rows) and the last new
 //                      rows to the ring
-//   vy_qkv_rows        the same for designs that norm their queries and keys (over the whole projection) and mix their values:
-//                      queries, keys and values in place
+//   vy_qkv_rows        the same for designs that norm their queries and keys (over the whole projection, or over heads or other
+//                      groups of columns by themselves), scale their queries by position and mix their values: in place
 //   vy_window_context  prefill behind a past: the ring's rows and the new ones as one contiguous context for vy_attn_fwd_ex
 //   vy_window_decode   one query token per sequence: rotation of query and key, the new row to the ring, attention over the
 //                      ring, sink, output gate.  Every row of the ring that holds a token is inside the window, so decode
-//                      needs no mask but the row count -- and no order: softmax does not care where a row lies.
+//                      needs no mask but the row count -- and no order: softmax does not care where a row lies.  Also
+//                      differential attention (vy_diff.hip has its prompts).
 #include "vy_window.h"
 
 namespace {
@@ -179,6 +180,81 @@ __global__ __launch_bounds__(256) void qkv_rows_kernel(QkvArgs a) {
   }
 }
 
+// norms over groups of columns: LPG lanes per unit, a unit being a group of a token's queries or keys, or a head of its values
+// (which are only copied to the ring)
+template <typename T, int LPG>
+__global__ __launch_bounds__(256) void group_rows_kernel(QkvArgs a, int group, int temp_every, float temp_coef) {
+  constexpr int VEC = VyChunk<T>::VEC;
+  const RowsArgs& r = a.r;
+  const int sub = threadIdx.x % LPG;
+  const int gq = a.h * r.dim / group, gk = r.hk * r.dim / group, per_row = gq + gk + (r.store ? r.hk : 0);
+  const int64_t units = r.M * per_row, u0 = (int64_t)blockIdx.x * (256 / LPG) + threadIdx.x / LPG, u = u0 < units ? u0 : units - 1;
+  const int64_t row = u / per_row;
+  const int x = (int)(u - row * per_row);
+  const int b = (int)(row / r.L), l = (int)(row - (int64_t)b * r.L);
+  const int slot = r.slots ? r.slots[b] : b;
+  const int first = r.start ? r.start[slot] : 0, n = r.count ? r.count[b] : r.L, pos = first + l;
+  const bool keep = r.store && stays(first, l, n, r.R, r.keep);
+  T* p = (T*)r.p + row * r.ldp;
+  T* ring = keep ? (T*)r.ring + (int64_t)slot * r.r_ss + (int64_t)ring_row(pos, r.R, r.keep) * (r.dim + r.vdim) : nullptr;
+  const bool value = x >= gq + gk, key = !value && x >= gq;
+  const int col = key ? (x - gq) * group : x * group;              // of the group, in its projection
+  T* src = value ? p + r.ov + (int64_t)(x - gq - gk) * r.vdim : p + (key ? r.ok : a.oq) + col;
+  const int width = value ? r.vdim : group;
+  float v[VEC], s = 0.f;
+  for (int c = sub * VEC; c < width; c += LPG * VEC) {
+    VyChunk<T>::load(src + c, v);
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) s = fmaf(v[e], v[e], s);
+  }
+#pragma unroll
+  for (int o = LPG / 2; o > 0; o >>= 1) s += __shfl_xor(s, o, 64);
+  if (u0 >= units || (value && !keep)) return;
+  const float f = value ? 1.f : rms_factor(s, key ? a.n_k : a.n_q, a.eps) * (key ? 1.f : query_temperature(pos, temp_every, temp_coef));
+  const float* w = key ? a.k_norm : a.q_norm;
+  const float2* trig = r.rope + (int64_t)(pos < r.rope_len ? pos : r.rope_len - 1) * r.half;   // (clamped: padding rows only)
+  const int head = value ? x - gq - gk : col / r.dim, d0 = value ? r.dim : col - head * r.dim;
+  for (int c = sub * VEC; c < width; c += LPG * VEC) {
+    if (LPG * VEC < width) VyChunk<T>::load(src + c, v);           // (several passes: read again, from cache)
+    if (!value) {
+      if (w) {
+#pragma unroll
+        for (int e = 0; e < VEC; e += 4) {
+          float w4[4];
+          VyChunk<float>::load(w + col + c + e, w4);
+#pragma unroll
+          for (int i = 0; i < 4; ++i) v[e + i] *= f * w4[i];
+        }
+      }
+#pragma unroll
+      for (int e = 0; e < VEC; e += 2) {
+        const int j = (d0 + c + e) >> 1;
+        if (j < r.half) {
+          const float2 cs = trig[j];
+          const float y = v[e], z = v[e + 1];
+          v[e] = y * cs.x - z * cs.y;
+          v[e + 1] = z * cs.x + y * cs.y;
+        }
+      }
+      VyChunk<T>::store(src + c, v);
+    }
+    if (keep && (key || value)) VyChunk<T>::store(ring + (int64_t)head * r.r_sh + d0 + c, v);
+  }
+}
+
+template <typename T>
+void group_rows_go(const QkvArgs& a, int group, int temp_every, float temp_coef, hipStream_t st) {
+  const int widest = a.r.store && a.r.vdim > group ? a.r.vdim : group, nch = widest / VyChunk<T>::VEC;
+  const int64_t units = a.r.M * ((int64_t)(a.h + a.r.hk) * a.r.dim / group + (a.r.store ? a.r.hk : 0));
+#define GR_GO(LPG) hipLaunchKernelGGL((group_rows_kernel<T, LPG>), dim3((unsigned)vy_cdiv(units, 256 / LPG)), dim3(256), 0, st, a, group, temp_every, temp_coef)
+  if (nch <= 4) GR_GO(4);
+  else if (nch <= 8) GR_GO(8);
+  else if (nch <= 16) GR_GO(16);
+  else if (nch <= 32) GR_GO(32);
+  else GR_GO(64);
+#undef GR_GO
+}
+
 struct ContextArgs {
   const void* p; int64_t ldp, ok, ov;
   const void* ring; int64_t r_ss, r_sh; int R, keep;
@@ -216,10 +292,10 @@ __global__ __launch_bounds__(256) void window_context_kernel(ContextArgs a) {
 }
 
 // ---- decode ---------------------------------------------------------------------------------
-template <int DHP, int DVP>
+template <int DHP, int DVP, int MAPS>
 __global__ __launch_bounds__(256) void window_decode_kernel(DecodeArgs a) {
-  __shared__ __attribute__((aligned(16))) char smem[WindowDecode<DHP, DVP>::LDS];
-  WindowDecode<DHP, DVP>::run(a, smem, blockIdx.x, blockIdx.y, blockIdx.z);
+  __shared__ __attribute__((aligned(16))) char smem[WindowDecode<DHP, DVP, MAPS>::LDS];
+  WindowDecode<DHP, DVP, MAPS>::run(a, smem, blockIdx.x, blockIdx.y, blockIdx.z);
 }
 
 __global__ __launch_bounds__(256) void window_finish_kernel(DecodeArgs a) {
@@ -227,17 +303,22 @@ __global__ __launch_bounds__(256) void window_finish_kernel(DecodeArgs a) {
   window_finish(a, red, blockIdx.x, blockIdx.y);
 }
 
-template <int DHP>
+__global__ __launch_bounds__(256) void window_finish_diff_kernel(DecodeArgs a) {
+  __shared__ __attribute__((aligned(16))) float red[FINISH_DIFF_LDS / 4];
+  window_finish_diff(a, red, blockIdx.x, blockIdx.y);
+}
+
+template <int DHP, int MAPS = 1>
 void decode_go(const DecodeArgs& a, dim3 grid, hipStream_t st) {
   const dim3 block(256);
-  if (a.vdim <= 64) hipLaunchKernelGGL((window_decode_kernel<DHP, 64>), grid, block, 0, st, a);
-  else if (a.vdim <= 128) hipLaunchKernelGGL((window_decode_kernel<DHP, 128>), grid, block, 0, st, a);
-  else hipLaunchKernelGGL((window_decode_kernel<DHP, 256>), grid, block, 0, st, a);
+  if (a.vdim <= 64) hipLaunchKernelGGL((window_decode_kernel<DHP, 64, MAPS>), grid, block, 0, st, a);
+  else if (a.vdim <= 128) hipLaunchKernelGGL((window_decode_kernel<DHP, 128, MAPS>), grid, block, 0, st, a);
+  else hipLaunchKernelGGL((window_decode_kernel<DHP, 256, MAPS>), grid, block, 0, st, a);
 }
 
 int check_ring(const char* who, const void* ring, int64_t r_ss, int64_t r_sh, int32_t R, int32_t keep, int32_t hk, int32_t dim,
                int32_t vdim, int vec) {
-  if (!ring || R < 1 || hk < 1 || dim < 1 || vdim < 1) VY_FAIL(VY_ERR_ARG, "%s: bad ring", who);
+  if (!ring || R < 1 || hk < 1 || dim < 1 || vdim < 0) VY_FAIL(VY_ERR_ARG, "%s: bad ring", who);
   if (keep < 0 || keep >= R) VY_FAIL(VY_ERR_ARG, "%s: %d kept of %d rows", who, keep, R);
   if (dim % vec || vdim % vec || r_ss % vec || r_sh % vec) VY_FAIL(VY_ERR_ARG, "%s: widths and strides must be multiples of %d", who, vec);
   if (r_sh < (int64_t)R * (dim + vdim) || r_ss < hk * r_sh) VY_FAIL(VY_ERR_ARG, "%s: ring strides do not hold %d rows", who, R);
@@ -246,6 +327,13 @@ int check_ring(const char* who, const void* ring, int64_t r_ss, int64_t r_sh, in
 
 int check_prep(const char* who, const vy_qkv_prep* q, int32_t h, int32_t hk, int32_t dim, int32_t vdim, int vec) {
   if (!q) return VY_OK;
+  if (q->group) {
+    if (q->group < 1 || q->group % vec || dim % q->group || !q->q_norm || !q->k_norm || q->n_q < 1 || q->n_q > q->group || q->n_k != q->n_q ||
+        q->temp_every < 0 || q->v_mix || q->v_out)
+      VY_FAIL(VY_ERR_ARG, "%s: norms over %d of %d columns of heads of %d", who, q->n_q, q->group, dim);
+    return VY_OK;
+  }
+  if (q->temp_every) VY_FAIL(VY_ERR_ARG, "%s: a temperature without norms over groups", who);
   if (!q->q_norm != !q->k_norm || (q->q_norm && (q->n_q < 1 || q->n_k < 1 || q->n_q > h * dim || q->n_k > hk * dim)))
     VY_FAIL(VY_ERR_ARG, "%s: bad query / key norms", who);
   const int m_v = q->m_v ? q->m_v : q->n_v, m_vp = q->m_v ? q->m_vp : vdim;
@@ -272,7 +360,7 @@ extern "C" int vy_window_rows(void* p, int64_t ldp, int64_t ok, int64_t ov, void
   const char* who = "vy_window_rows";
   if (dtype != VY_BF16 && dtype != VY_F32) VY_FAIL(VY_ERR_ARG, "%s: bad dtype %d", who, dtype);
   const int vec = dtype == VY_BF16 ? 8 : 4;
-  if (!p || B <= 0 || L <= 0 || hk <= 0 || dim <= 0 || vdim <= 0 || dim % vec || vdim % vec || ldp % vec || ok % vec || ov % vec)
+  if (!p || B <= 0 || L <= 0 || hk <= 0 || dim <= 0 || vdim < 0 || dim % vec || vdim % vec || ldp % vec || ok % vec || ov % vec)
     VY_FAIL(VY_ERR_ARG, "%s: bad arguments", who);
   if (store) {
     if (!start) VY_FAIL(VY_ERR_ARG, "%s: ring without start positions", who);
@@ -315,6 +403,13 @@ extern "C" int vy_qkv_rows(void* p, int64_t ldp, int64_t oq, int64_t ok, int64_t
   a.n_v = prep->n_v; a.m_v = prep->m_v ? prep->m_v : prep->n_v; a.m_vp = prep->m_v ? prep->m_vp : vdim; a.vo = prep->v_out; a.ldvo = prep->ldo;
   hipStream_t st = (hipStream_t)stream;
   const int chunks = (h + hk) * dim / vec;
+  if (prep->group) {
+    if (a.r.M * ((int64_t)(h + hk) * dim / prep->group + hk) > INT32_MAX) VY_FAIL(VY_ERR_UNSUPPORTED, "%s: %ld rows", who, (long)a.r.M);
+    if (dtype == VY_BF16) group_rows_go<bf16>(a, prep->group, prep->temp_every, prep->temp_coef, st);
+    else group_rows_go<float>(a, prep->group, prep->temp_every, prep->temp_coef, st);
+    VY_CHECK_LAUNCH(who);
+    return VY_OK;
+  }
   // narrow rows: a wave each
   const bool narrow = chunks <= 64 * 8 && B * L >= 1024;
   const dim3 grid((unsigned)(narrow ? vy_cdiv(B * L, 4) : B * L)), block(256);
@@ -350,15 +445,16 @@ extern "C" int vy_window_context(const void* p, int64_t ldp, int64_t ok, int64_t
   return VY_OK;
 }
 
-extern "C" int64_t vy_window_decode_ws_bytes(int32_t B, int32_t h, int32_t hk, int32_t vdim, int32_t R) {
+extern "C" int64_t vy_window_decode_ws_bytes(int32_t B, int32_t h, int32_t hk, int32_t vdim, int32_t R, int diff) {
   if (B < 1 || h < 1 || hk < 1 || vdim < 1 || R < 1) return 0;
   const int ns = slices_of((int64_t)B * hk * ((h / hk + 15) / 16), R);
-  return ns == 1 ? 0 : (int64_t)B * h * ns * (vdim + 2) * 4 + 256;
+  return ns == 1 && !diff ? 0 : (int64_t)B * h * (diff ? 2 : 1) * ns * (vdim + 2) * 4 + 256;
 }
 
 extern "C" int vy_window_decode(void* p, int64_t ldp, int64_t oq, int64_t ok, int64_t ov, int64_t og, void* ring, int64_t r_ss,
                                 int64_t r_sh, int32_t R, int32_t keep, const float* rope, int32_t rope_dims, int32_t rope_len,
-                                const vy_qkv_prep* prep, const int32_t* slots, const int32_t* start, int64_t max_keys, void* out, int64_t ldo, int64_t B,
+                                const vy_qkv_prep* prep, const vy_diff* diff, const int32_t* slots, const int32_t* start, int64_t max_keys, void* out,
+                                int64_t ldo, int64_t B,
                                 int32_t h, int32_t hk, int32_t dim, int32_t vdim, float scale, int32_t sink, void* ws,
                                 int64_t ws_bytes, int dtype, void* stream) {
   const char* who = "vy_window_decode";
@@ -372,8 +468,18 @@ extern "C" int vy_window_decode(void* p, int64_t ldp, int64_t oq, int64_t ok, in
   if (int rc = check_prep(who, prep, h, hk, dim, vdim, vec)) return rc;
   if (int rc = check_rope(who, rope, rope_dims, rope_len, dim)) return rc;
   if (rope_dims && max_keys > rope_len) VY_FAIL(VY_ERR_ARG, "%s: %ld positions, rotary table of %d", who, (long)max_keys, rope_len);
+  if (diff && (dim % (2 * vec) || sink || og >= 0 || rope_dims || keep || max_keys > R || diff->n_v < 1 || diff->n_v > vdim || vdim < 1 ||
+               !prep || (prep->group && prep->group != dim / 2)))
+    VY_FAIL(VY_ERR_ARG, "%s: bad differential attention", who);
   hipStream_t st = (hipStream_t)stream;
-  if (dtype == VY_F32 || dim > 256 || vdim > 256) {
+  const int map_dim = diff ? dim / 2 : dim;
+  if (diff && (dtype == VY_F32 || map_dim > 256 || vdim > 256)) {
+    if (int rc = vy_qkv_rows(p, ldp, oq, ok, ov, prep, ring, r_ss, r_sh, R, keep, rope, rope_dims, rope_len, 1, slots, start, nullptr, B, 1, h,
+                             hk, dim, vdim, dtype, stream)) return rc;
+    return vy_diff_attn_fwd((const char*)p + oq * (dtype == VY_BF16 ? 2 : 4), ldp, ring, r_ss, r_sh, R, diff, slots, start, nullptr, out, ldo,
+                            B, 1, h, hk, dim, vdim, scale, dtype, stream);
+  }
+  if (dtype == VY_F32 || map_dim > 256 || vdim > 256) {
     // row-wise kernel over the ring: the new row goes in first
     int rc;
     if (prep) rc = vy_qkv_rows(p, ldp, oq, ok, ov, prep, ring, r_ss, r_sh, R, keep, rope, rope_dims, rope_len, 1, slots, start, nullptr, B, 1,
@@ -382,7 +488,7 @@ extern "C" int vy_window_decode(void* p, int64_t ldp, int64_t oq, int64_t ok, in
                              hk, dim, vdim, dtype, stream);
     if (rc) return rc;
     const int64_t e = dtype == VY_BF16 ? 2 : 4;
-    const vy_attn_window win{0, sink, 1, INT32_MAX, prep ? nullptr : rope, prep ? 0 : rope_dims, rope_len, 0};   // (prep: rotated already)
+    const vy_attn_window win{0, sink, 1, INT32_MAX, prep ? nullptr : rope, prep ? 0 : rope_dims, rope_len, 0, 0};   // (prep: rotated already)
     const char* gate = og >= 0 ? (const char*)p + og * e : nullptr;
     return vy_attn_fwd_ex((const char*)p + oq * e, ldp, dim, ldp, ring, r_ss, r_sh, dim + vdim, (const char*)ring + (int64_t)dim * e,
                           r_ss, r_sh, dim + vdim, out, ldo, ldo, gate, ldp, ldp, start, slots, B, h, hk, 1, R, dim, vdim, scale,
@@ -393,23 +499,33 @@ extern "C" int vy_window_decode(void* p, int64_t ldp, int64_t oq, int64_t ok, in
   a.ring = (bf16*)ring; a.r_ss = r_ss; a.r_sh = r_sh; a.R = R; a.keep = keep;
   if (prep) {
     a.q_norm = prep->q_norm; a.k_norm = prep->k_norm; a.n_q = prep->n_q; a.n_k = prep->n_k; a.eps = prep->eps; a.lambda = prep->lambda;
+    a.group = prep->group; a.temp_every = prep->temp_every; a.temp_coef = prep->temp_coef;
     a.vm = (const bf16*)prep->v_mix; a.ldm = prep->ldm;
     a.n_v = prep->n_v; a.m_v = prep->m_v ? prep->m_v : prep->n_v; a.m_vp = prep->m_v ? prep->m_vp : vdim;
     a.vo = (bf16*)prep->v_out; a.ldvo = prep->ldo;
   }
   a.rope = (const float2*)rope; a.half = rope_dims / 2; a.rope_len = rope_len > 0 ? rope_len : 1;
   a.slots = slots; a.start = start; a.out = (bf16*)out; a.ldo = ldo;
-  a.h = h; a.hk = hk; a.dim = dim; a.vdim = vdim; a.scale = scale; a.sink = sink;
+  a.h = h; a.hk = hk; a.dim = map_dim; a.vdim = vdim; a.scale = scale; a.sink = sink;
+  if (diff) { a.lambda2 = diff->lambda; a.out_scale = diff->out_scale; a.eps_out = diff->eps; a.n_v = diff->n_v; }
   a.passes = (h / hk + 15) / 16;
   const int64_t rows = max_keys < R ? max_keys : R;
   a.ns = slices_of(B * hk * a.passes, rows);
-  if (a.ns > 1) {
-    const int64_t need = B * h * a.ns * ((int64_t)vdim + 2) * 4;
+  if (a.ns > 1 || diff) {
+    const int64_t parts = B * h * (diff ? 2 : 1) * a.ns, need = parts * ((int64_t)vdim + 2) * 4;
     if (!ws || ws_bytes < need || (uintptr_t)ws % 16) VY_FAIL(VY_ERR_ARG, "%s: workspace too small or unaligned", who);
     a.part_o = (float*)ws;
-    a.part_ml = a.part_o + B * h * a.ns * (int64_t)vdim;
+    a.part_ml = a.part_o + parts * vdim;
   }
   const dim3 grid((unsigned)a.ns, (unsigned)(hk * a.passes), (unsigned)B);
+  if (diff) {
+    if (map_dim <= 64) decode_go<64, 2>(a, grid, st);
+    else if (map_dim <= 128) decode_go<128, 2>(a, grid, st);
+    else decode_go<256, 2>(a, grid, st);
+    hipLaunchKernelGGL(window_finish_diff_kernel, dim3((unsigned)h, (unsigned)B), dim3(256), 0, st, a);
+    VY_CHECK_LAUNCH(who);
+    return VY_OK;
+  }
   if (dim <= 64) decode_go<64>(a, grid, st);
   else if (dim <= 128) decode_go<128>(a, grid, st);
   else decode_go<256>(a, grid, st);

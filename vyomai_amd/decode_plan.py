@@ -9,7 +9,7 @@ from typing import List
 
 import torch
 
-from . import _lib
+from . import _lib, ops
 from .layers.attention import _shadow
 from .ops import up8
 
@@ -259,22 +259,22 @@ class GemmaDecodePlan:
 class VyHybridLayer(C.Structure):
     _fields_ = [(n, C.c_int32) for n in ("mixer", "heads", "dim", "vdim", "n_in", "ff", "q_rank", "q_rank_p", "kv_rank",
                                          "kv_rank_p", "cap", "mix_n", "form", "clamped", "kv_heads", "rope_dims", "rope_len", "sink", "keep",
-                                         "gate", "values", "silu")] + \
+                                         "gate", "values", "silu", "ring", "gate_heads")] + \
                [(n, C.c_float) for n in ("scale", "limit", "alpha", "k_scale")] + \
-               [(n, C.c_void_p) for n in ("norm1", "norm1b", "norm2", "norm2b", "w_in", "w_o", "w_gu", "w_down", "q_norm",
+               [(n, C.c_void_p) for n in ("norm1", "norm1b", "norm2", "norm2b", "w_in", "b_in", "w_o", "w_gu", "w_up", "w_down", "q_norm",
                                           "c_norm", "w_uq", "w_ukt", "w_uv", "cache")] + \
                [(n, C.c_int64) for n in ("c_ss", "c_sh", "c_st")] + \
-               [(n, C.c_void_p) for n in ("state", "decay_pow", "mix_norm", "rope")] + \
-               [("prep", C.POINTER(_lib.VyQkvPrep)), ("moe", C.POINTER(_lib.VyMoe))]
+               [(n, C.c_void_p) for n in ("state", "decay_pow", "mix_norm", "f_bias", "f_lower", "rope")] + \
+               [("prep", C.POINTER(_lib.VyQkvPrep)), ("diff", C.POINTER(_lib.VyDiff)), ("moe", C.POINTER(_lib.VyMoe))]
 
 
 class VyHybridPlan(C.Structure):
     _fields_ = [(n, C.c_int32) for n in ("num_layers", "B", "d", "dp", "vocab", "dtype", "rms", "act")] + \
-               [("eps", C.c_float), ("embed_scale", C.c_float), ("layers", C.POINTER(VyHybridLayer))] + \
+               [("eps", C.c_float), ("embed_scale", C.c_float), ("softcap", C.c_float), ("layers", C.POINTER(VyHybridLayer))] + \
                [(n, C.c_void_p) for n in ("embed", "head", "final_norm", "err", "ws")] + [("ws_bytes", C.c_int64)]
 
 
-MIX_LATENT, MIX_DECAY, MIX_WINDOW = 0, 1, 2
+MIX_LATENT, MIX_DECAY, MIX_WINDOW, MIX_GATED = 0, 1, 2, 3
 FORMS = {"sandwich": 0, "parallel": 1}
 
 
@@ -297,15 +297,18 @@ class HybridDecodePlan:
             L.heads, L.dim, L.vdim = m.heads, up8(m.dim), up8(m.vdim)
             w = n if parallel else p
             L.w_in, L.n_in, L.w_o = _ptr(w.w_in), w.w_in.shape[0], _ptr(w.w_o)
+            L.b_in = _ptr(getattr(w, "b_in", None))
             L.norm1, L.norm1b = _ptr(n.norm1), None if parallel else _ptr(n.norm1b)
             buf = cache.buffers[i]
             self.keep.append(buf)
             if m.kind == "latent":
                 L.mixer, L.scale = MIX_LATENT, m.scale
-                L.q_rank, L.q_rank_p, L.kv_rank, L.kv_rank_p = m.q_rank, p.q_norm.numel(), m.kv_rank, p.c_norm.numel()
-                L.q_norm, L.c_norm = _ptr(p.q_norm), _ptr(p.c_norm)
-                L.w_uq, L.w_ukt, L.w_uv = _ptr(p.w_uq), _ptr(p.w_ukt), _ptr(p.w_uv)
-                L.cache, L.c_ss, L.c_st, L.cap = buf.data_ptr(), buf.stride(0), buf.stride(1), buf.shape[1]
+                L.kv_rank, L.kv_rank_p, L.c_norm = m.kv_rank, p.c_norm.numel(), _ptr(p.c_norm)
+                if m.q_rank:
+                    L.q_rank, L.q_rank_p, L.q_norm, L.w_uq = m.q_rank, p.q_norm.numel(), _ptr(p.q_norm), _ptr(p.w_uq)
+                L.w_ukt, L.w_uv, L.gate, L.gate_heads, L.ring = _ptr(p.w_ukt), _ptr(p.w_uv), 1, int(m.head_gate), int(m.window is not None)
+                rows = buf.dim() - 2             # (slots, rows, width), or a ring (slots, 1, rows, width)
+                L.cache, L.c_ss, L.c_st, L.cap = buf.data_ptr(), buf.stride(0), buf.stride(rows), buf.shape[rows]
             elif m.kind == "window":
                 L.mixer, L.scale, L.kv_heads, L.sink = MIX_WINDOW, m.scale, m.kv_heads, int(m.sink)
                 L.keep, L.gate, L.values = m.keep_first, int(m.gate is not None), m.values
@@ -313,8 +316,17 @@ class HybridDecodePlan:
                 self.keep.append(c)
                 if c.prep is not None:
                     q = c.prep
-                    L.prep = C.pointer(_lib.VyQkvPrep(_ptr(q.q_norm), _ptr(q.k_norm), q.n_q, q.n_k, q.eps, q.mix, n_v=q.n_v))
+                    L.prep = C.pointer(ops.prep_struct(q))
                 L.cache, L.c_ss, L.c_sh, L.cap = buf.data_ptr(), buf.stride(0), buf.stride(1), buf.shape[2]
+            elif m.kind == "differential":
+                c = m.constants()
+                self.keep.append(c)
+                L.mixer, L.scale, L.kv_heads, L.dim = MIX_WINDOW, m.scale, m.kv_heads, 2 * up8(m.dim)
+                L.prep, L.diff = C.pointer(ops.prep_struct(c.prep)), C.pointer(c.diff)
+                L.cache, L.c_ss, L.c_sh, L.cap = buf.data_ptr(), buf.stride(0), buf.stride(1), buf.shape[2]
+            elif m.kind == "gated":
+                L.mixer, L.state, L.silu = MIX_GATED, buf.data_ptr(), int(m.silu)
+                L.f_bias, L.f_lower, L.mix_norm, L.mix_n = _ptr(p.f_bias), _ptr(p.f_lower), _ptr(p.norm), m.vdim
             else:
                 L.mixer, L.state, L.decay_pow = MIX_DECAY, buf.data_ptr(), _ptr(p.decay_pow)
                 L.mix_norm, L.mix_n = _ptr(p.norm), m.heads * m.vdim if p.norm is not None else m.vdim
@@ -332,7 +344,7 @@ class HybridDecodePlan:
                     if not parallel:
                         f = dense.packed()
                         self.keep.append(f)
-                        L.w_gu, L.w_down = _ptr(f.w_gu), _ptr(f.w_down)
+                        L.w_gu, L.w_up, L.w_down = _ptr(getattr(f, "w_gu", None)), _ptr(getattr(f, "w_up", None)), _ptr(f.w_down)
                     if not dense.clamped:
                         acts.add(dense.act)
                 if layer.mlp is not dense:
@@ -347,7 +359,7 @@ class HybridDecodePlan:
         p = VyHybridPlan()
         p.num_layers, p.B, p.d, p.dp, p.vocab = len(model.layers), batch, model.width, t.embed.shape[1], model.vocab
         p.dtype, p.rms, p.act, p.eps = _lib.dtype_code(model.dtype), int(model.rms), acts.pop() if acts else _lib.ACT_NONE, model.eps
-        p.embed_scale = model.embed_scale
+        p.embed_scale, p.softcap = model.embed_scale, model.softcap or 0.0
         p.layers = C.cast(arr, C.POINTER(VyHybridLayer))
         p.embed, p.head, p.final_norm = _ptr(t.embed), _ptr(t.head), _ptr(t.final_norm)
         nbytes = lib.vy_hybrid_ws_bytes(C.byref(p))

@@ -12,7 +12,7 @@ import torch
 import torch.nn as nn
 
 from .. import ops
-from .._lib import (ACT_GELU_ERF, ACT_GELU_TANH, ACT_SILU, MOE_CLAMPED, MOE_GELU, SCORE_SIGMOID, SCORE_SOFTMAX, VyMoe)
+from .._lib import (ACT_GELU_ERF, ACT_GELU_TANH, ACT_RELU2, ACT_SILU, MOE_CLAMPED, MOE_GELU, SCORE_SIGMOID, SCORE_SOFTMAX, VyMoe)
 from ..ops import up8
 from .packing import Packed, pad2
 
@@ -83,6 +83,40 @@ class GatedFeedForward(nn.Module):
     # what a layer asks of its feed-forward: the part that runs on every token, and the routed rows beside it
     @property
     def dense(self) -> Optional["GatedFeedForward"]:
+        return self
+
+    def routed(self, h: torch.Tensor, L: int = 1, count: Optional[torch.Tensor] = None) -> Optional["ops.Routed"]:
+        return None
+
+
+_PLAIN_ACT = {"relu2": ACT_RELU2, "gelu_tanh": ACT_GELU_TANH, "gelu": ACT_GELU_ERF}
+
+
+class PlainFeedForward(nn.Module):
+    """down(act(up(x))), no gate and no biases: the activation is the first product's epilogue.  act "relu2": max(z, 0)^2."""
+    clamped, limit, alpha = False, 0.0, 0.0
+
+    def __init__(self, width: int, inner: int, act: str = "relu2") -> None:
+        super().__init__()
+        self.width, self.inner, self.act = width, inner, _PLAIN_ACT[act]
+        self.up = nn.Linear(width, inner, bias=False)
+        self.down = nn.Linear(inner, width, bias=False)
+
+    def matrices(self):
+        raise ValueError("a feed-forward without a gate does not share its products with a mixer's (no parallel layers)")
+
+    def packed(self) -> Packed:
+        def build(p: Packed) -> None:
+            dp, ip = up8(self.width), up8(self.inner)
+            p.w_up, p.w_down = pad2(self.up.weight, ip, dp).contiguous(), pad2(self.down.weight, dp, ip).contiguous()
+        return Packed.of(self, list(self.parameters()), build)
+
+    def forward(self, h: torch.Tensor) -> torch.Tensor:
+        p = self.packed()
+        return ops.linear(ops.linear(h, p.w_up, act=self.act), p.w_down)
+
+    @property
+    def dense(self) -> Optional["PlainFeedForward"]:
         return self
 
     def routed(self, h: torch.Tensor, L: int = 1, count: Optional[torch.Tensor] = None) -> Optional["ops.Routed"]:

@@ -274,13 +274,17 @@ class StaticCacheOne:
         return None
 
 
+EVERY_TOKEN = 2 ** 31 - 1   # rows of a ring that never wraps: it grows with the capacity
+
+
 class SlotCache:
     """Whole-model memory of sequences of DIFFERENT lengths, for decoders that mix layer kinds.
 
     A sequence owns a slot while it lives (``allocate`` / ``free``); per layer a slot holds either cached rows
     ("latent", width): a (slots, capacity, width) buffer, or a ring of the last tokens' keys and values ("window", (heads,
     width, rows[, keep])): a (slots, heads, rows, width) buffer (fewer rows while the capacity is less), position p in row p, and
-    from `rows` on round and round the rows behind the `keep` first, or a recurrent state ("state", shape): a (slots, *shape)
+    from `rows` on round and round the rows behind the `keep` first (rows = EVERY_TOKEN: never; a windowed latent is a ring of one
+    head), or a recurrent state ("state", shape): a (slots, *shape)
     fp32 buffer.  ``lengths`` (int32 on the device, one per slot) says how many tokens a slot holds: kernels place new rows
     behind them, attend no further, and take the state of an empty slot as zero -- so nothing is cleared when a slot is
     handed on.  The host keeps a mirror (``length``).  Slots and capacity grow by doubling.

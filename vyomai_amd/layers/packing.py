@@ -28,11 +28,11 @@ def pad_vec(w: torch.Tensor, n: int) -> torch.Tensor:
 
 def norm_vec(norm, n: int, mult: float = 1.0) -> torch.Tensor:
     """fp32 factors of a WeightNorm (times mult), zero-padded to n."""
-    return pad_vec((norm.weight.float() + norm.offset) * mult, n)
+    return pad_vec(((norm.weight.float() + norm.offset) * mult).expand(norm.width), n)
 
 
 def head_rows(w: torch.Tensor, heads: int, cols: int) -> torch.Tensor:
-    """(heads * dim, k) -> (heads * up8(dim), cols): every head's rows padded by themselves."""
+    """(heads * dim, k <= cols) -> (heads * up8(dim), cols): every head's rows padded by themselves."""
     dim = w.shape[0] // heads
     out = torch.zeros(heads, up8(dim), cols, dtype=w.dtype, device=w.device)
     out[:, :dim, : w.shape[1]] = w.view(heads, dim, w.shape[1])
@@ -61,6 +61,11 @@ def head_vec(w: torch.Tensor, heads: int) -> torch.Tensor:
     out = torch.zeros(heads, up8(dim), dtype=torch.float32, device=w.device)
     out[:, :dim] = w.float().view(heads, dim)
     return out.view(-1)
+
+
+def head_bias(b: torch.Tensor, heads: int) -> torch.Tensor:
+    """A bias over concatenated heads in its own type, every head padded by itself (as head_rows pads the weights)."""
+    return head_rows(b[:, None], heads, 1)[:, 0]
 
 
 class Packed:

@@ -1,11 +1,11 @@
 """Decoders that mix layer kinds over an fp32 residual stream: every layer is one mixer (latent attention, lightning attention,
-windowed attention, ...) and an optional feed-forward (gated, or a mixture of experts), in one of two forms:
+windowed attention, ...) and an optional feed-forward (gated, plain, or a mixture of experts), in one of two forms:
 
     HybridLayer    x <- x + m norm1b(mixer(norm1(x))) ;  x <- x + m norm2b(ff(norm2(x)))    (without norm1 / norm2: of x itself)
     ParallelLayer  x <- x + (mixer(h) + ff(h)),  h = norm1(x)
 
-A design built from this file supplies its layers and its parameter names (models/gisitar.py, rivudra.py, padulorn.py); embedding,
-residual stream, slot cache, prefill, the native single-token step and generation are here.  Inference only.
+A design built from this file supplies its layers and its parameter names (models/gisitar.py, rivudra.py, padulorn.py,
+biruvik.py); embedding, residual stream, slot cache, prefill, the native single-token step and generation are here.  Inference only.
 """
 from __future__ import annotations
 
@@ -30,11 +30,12 @@ class HybridLayer(nn.Module):
     form = "sandwich"
 
     def __init__(self, width: int, mixer: nn.Module, mlp: Optional[nn.Module], eps: float, norm: str = "layer",
-                 offset: float = 0.0, pre: bool = True, mult: float = 1.0) -> None:
+                 offset: float = 0.0, pre: bool = True, mult: float = 1.0, scalar: bool = False) -> None:
+        """scalar: the norms' weights are one number each."""
         super().__init__()
         self.mixer, self.mlp, self.width, self.pre, self.mult = mixer, mlp, width, pre, float(mult)
         for n in self._norms():
-            setattr(self, n, WeightNorm(width, eps, norm, offset))
+            setattr(self, n, WeightNorm(width, eps, norm, offset, scalar))
 
     def _norms(self) -> List[str]:
         names = ["norm1", "norm1b"] + (["norm2", "norm2b"] if self.mlp is not None else [])
@@ -79,6 +80,8 @@ class ParallelLayer(nn.Module):
 
         def build(p: Packed) -> None:
             p.norm1 = norm_vec(self.norm1, up8(self.width))
+            if getattr(self.mixer, "query", None) is not None and self.mixer.query.bias is not None:
+                raise ValueError("a mixer with biases does not share its products (no parallel layers)")
             p.w_in, p.w_o = self.mixer.matrices()
             p.n_mix, p.n_heads = p.w_in.shape[0], p.w_o.shape[1]
             if self.dense is not None:
@@ -99,16 +102,21 @@ class ParallelLayer(nn.Module):
 
 
 class HybridDecoderModel(nn.Module):
-    """`layers` of HybridLayer / ParallelLayer between a (scaled) embedding and a norm + vocabulary projection."""
+    """`layers` of HybridLayer / ParallelLayer between a (scaled) embedding and a norm + vocabulary projection (softcap: logits
+    become softcap tanh(logits / softcap); scalar: the norm's weight is one number)."""
 
     def __init__(self, config, width: int, vocab: int, layers: Sequence[nn.Module], eps: float, norm: str = "layer",
-                 offset: float = 0.0, embed_scale: float = 1.0, logit_scale: float = 1.0) -> None:
+                 offset: float = 0.0, embed_scale: float = 1.0, logit_scale: float = 1.0, softcap: Optional[float] = None,
+                 scalar: bool = False) -> None:
         super().__init__()
         self.config, self.width, self.vocab, self.eps, self.rms = config, width, vocab, float(eps), norm == "rms"
         self.embed_scale, self.logit_scale = float(embed_scale), float(logit_scale)
+        self.softcap = float(softcap) if softcap is not None else None
+        if softcap is not None and not softcap > 0:
+            raise ValueError(f"logits capped at {softcap}")
         self.word_embeddings = nn.Embedding(vocab, width)
         self.layers = nn.ModuleList(layers)
-        self.final_norm = WeightNorm(width, eps, norm, offset)
+        self.final_norm = WeightNorm(width, eps, norm, offset, scalar)
         self.head = nn.Linear(width, vocab, bias=False)
         self._own_cache: Optional[SlotCache] = None
         self.requires_grad_(False)
@@ -164,7 +172,7 @@ class HybridDecoderModel(nn.Module):
         p = self.packed()
         rows = rows if rows.stride(1) == 1 else rows.contiguous()
         h = ops.residual_norm(rows, self.width, pre=p.final_norm, eps=self.eps, rms=self.rms, dtype=self.dtype)
-        return ops.linear(h, p.head)
+        return ops.linear(h, p.head) if self.softcap is None else ops.linear_softcap(h, p.head, self.softcap)
 
     def decode(self, ids: torch.Tensor, cache: SlotCache, slots: Sequence[int]) -> torch.Tensor:
         """One more token (ids (B,) int64 on the device) for each sequence: ONE native call -> logits (B, vocab)."""

@@ -29,7 +29,7 @@ def register_model(name: str) -> Callable[[type], type]:
 
 
 def model_class(architecture: str) -> type:
-    from . import gisitar, padulorn, rivudra  # noqa: F401  (they register themselves)
+    from . import biruvik, gisitar, padulorn, rivudra  # noqa: F401  (they register themselves)
     if architecture not in MODELS:
         raise ValueError(f"architecture {architecture!r} is not registered (known: {sorted(MODELS)})")
     return MODELS[architecture]

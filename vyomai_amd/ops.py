@@ -207,6 +207,18 @@ def linear(x: Tensor, w: Tensor, bias: Optional[Tensor] = None, act: int = _lib.
     return ret
 
 
+def linear_softcap(x: Tensor, w: Tensor, cap: float) -> Tensor:
+    """cap * tanh(x @ w.T / cap), x (M, K); rows of the result are padded to 8 elements.  (vy_linear_softcap_fwd)"""
+    _need_gpu(x, w)
+    (M, K), N = x.shape, w.shape[0]
+    assert w.shape[1] == K and w.stride(1) == 1 and x.stride(1) == 1
+    y = torch.empty((M, up8(N)), dtype=x.dtype, device=x.device)
+    _mid_ws(M)
+    call("vy_linear_softcap_fwd", x.data_ptr(), x.stride(0), w.data_ptr(), w.stride(0), y.data_ptr(), y.stride(0), M, N, K, float(cap),
+         dtype_code(x.dtype), _stream())
+    return y[:, :N]
+
+
 def qkv_rope(x: Tensor, w_packed: Tensor, b_packed: Optional[Tensor], h: int, hk: int, dh: int,
              cos: Optional[Tensor], sin: Optional[Tensor], pos0: int,
              q: Tensor, k: Tensor, v: Tensor) -> None:
@@ -708,23 +720,25 @@ def _slot_args(slots: Optional[Tensor], start: Optional[Tensor], count: Optional
     assert count is None or count.numel() == B
 
 
-def latent_norm(p: Tensor, w_q: Tensor, n_q: int, w_c: Tensor, n_c: int, B: int, L: int, eps: float, *,
+def latent_norm(p: Tensor, w_q: Optional[Tensor], n_q: int, w_c: Tensor, n_c: int, B: int, L: int, eps: float, *,
                 cache: Optional[Tensor] = None, slots: Optional[Tensor] = None, start: Optional[Tensor] = None,
-                count: Optional[Tensor] = None, want_c: bool = True) -> Tuple[Tensor, Optional[Tensor]]:
+                count: Optional[Tensor] = None, want_c: bool = True) -> Tuple[Optional[Tensor], Optional[Tensor]]:
     """RMS norms of the two latents at the front of the packed rows p (B*L, .); the second one also goes to
-    cache[slot, start + l].  (vy_latent_norm)"""
+    cache[slot, start + l], or to a ring: cache (slots, 1, rows, width), row (start + l) % rows.  w_q None: no first latent, n_q
+    columns ahead of the second one are left alone.  (vy_latent_norm)"""
     _need_gpu(p, w_q, w_c, cache, slots, start, count)
     _slot_args(slots, start, count, B)
-    npq, npc = w_q.numel(), w_c.numel()
+    npq, npc = w_q.numel() if w_q is not None else int(n_q), w_c.numel()
     assert p.shape[0] == B * L and p.stride(1) == 1 and p.shape[1] >= npq + npc
-    q = torch.empty((B * L, npq), dtype=p.dtype, device=p.device)
+    q = torch.empty((B * L, npq), dtype=p.dtype, device=p.device) if w_q is not None else None
     c = torch.empty((B * L, npc), dtype=p.dtype, device=p.device) if want_c else None
+    at = (None, 0, 0, 0, 0)
     if cache is not None:
-        assert cache.dtype == p.dtype and cache.shape[2] == npc and cache.stride(2) == 1 and start is not None
-    call("vy_latent_norm", p.data_ptr(), p.stride(0), w_q.data_ptr(), q.data_ptr(), npq, int(n_q), npq, w_c.data_ptr(), _ptr(c),
-         npc, int(n_c), npc, _ptr(cache), cache.stride(0) if cache is not None else 0,
-         cache.stride(1) if cache is not None else 0, cache.shape[1] if cache is not None else 0, _ptr(slots), _ptr(start),
-         _ptr(count), B, L, float(eps), dtype_code(p.dtype), _stream())
+        r = cache.dim() - 2
+        assert cache.dtype == p.dtype and cache.shape[r + 1] == npc and cache.stride(r + 1) == 1 and start is not None
+        at = cache.data_ptr(), cache.stride(0), cache.stride(r), cache.shape[r], int(r == 2)
+    call("vy_latent_norm", p.data_ptr(), p.stride(0), _ptr(w_q), _ptr(q), npq, int(n_q), npq, w_c.data_ptr(), _ptr(c),
+         npc, int(n_c), npc, *at, _ptr(slots), _ptr(start), _ptr(count), B, L, float(eps), dtype_code(p.dtype), _stream())
     return q, c
 
 
@@ -740,26 +754,31 @@ def rmsnorm_gate(x: Tensor, w: Tensor, width: int, gate: Tensor, eps: float, out
     return y
 
 
-def head_norm_gate(x: Tensor, heads: int, width: int, gate: Tensor, eps: float, out: Optional[Tensor] = None) -> Tensor:
-    """x / rms(x) * silu(gate), every head (`width` of its padded columns) by itself.  (vy_head_norm_gate)"""
-    _need_gpu(x, gate, out)
+def head_norm_gate(x: Tensor, heads: int, width: int, gate: Optional[Tensor], eps: float, out: Optional[Tensor] = None,
+                   w: Optional[Tensor] = None) -> Tensor:
+    """x / rms(x) * w * silu(gate), every head (`width` of its padded columns) by itself; w: fp32 factors of a head's padded
+    columns, shared by the heads; gate and w may be None.  (vy_head_norm_gate)"""
+    _need_gpu(x, gate, out, w)
     M, NP = x.shape
-    assert NP % heads == 0 and gate.shape == x.shape and x.stride(1) == 1 and gate.stride(1) == 1
+    assert NP % heads == 0 and x.stride(1) == 1 and (gate is None or (gate.shape == x.shape and gate.stride(1) == 1))
+    assert w is None or (w.dtype == torch.float32 and w.numel() == NP // heads and w.is_contiguous())
     y = torch.empty((M, NP), dtype=x.dtype, device=x.device) if out is None else out
     assert y.shape == x.shape and y.stride(1) == 1 and y.dtype == x.dtype
-    call("vy_head_norm_gate", x.data_ptr(), x.stride(0), gate.data_ptr(), gate.stride(0), y.data_ptr(), y.stride(0), M, heads,
+    call("vy_head_norm_gate", x.data_ptr(), x.stride(0), _ptr(w), _ptr(gate), gate.stride(0) if gate is not None else 0,
+         y.data_ptr(), y.stride(0), M, heads,
          int(width), NP // heads, float(eps), dtype_code(x.dtype), _stream())
     return y
 
 
 def attention_ex(q: Tensor, k: Tensor, v: Tensor, scale: float, *, gate: Optional[Tensor] = None,
                  start: Optional[Tensor] = None, slots: Optional[Tensor] = None, window: int = 0, sink: bool = False,
-                 rotary: Optional[Tensor] = None, start_cap: Optional[int] = None, keep: int = 0,
+                 rotary: Optional[Tensor] = None, start_cap: Optional[int] = None, keep: int = 0, gate_heads: bool = False,
                  out: Optional[Tensor] = None) -> Tensor:
     """Causal attention with a value width of its own: q (B,h,L,dh), k (B,hk,S,dh), v (B,hk,S,dv) -> (B, L, h*dv); `start`
     (int32, per slot) keys precede the queries; gate (B, L, h*dv): out *= sigmoid(gate).  window: only the last `window` keys up
     to a query's own are seen (0: all), and the first `keep` of all; sink: one more exp(0) in the denominators; rotary (positions, pairs, 2): the queries are
-    rotated by position start + i; start_cap: at most so many keys precede the queries.  (vy_attn_fwd_ex)"""
+    rotated by position start + i; start_cap: at most so many keys precede the queries; gate_heads: gate (B, L, >= h) holds one
+    number per head.  (vy_attn_fwd_ex)"""
     _need_gpu(q, k, v, gate, start, slots)
     B, h, L, dh = q.shape
     hk, S, dv = k.shape[1], k.shape[2], v.shape[3]
@@ -768,12 +787,12 @@ def attention_ex(q: Tensor, k: Tensor, v: Tensor, scale: float, *, gate: Optiona
     if out is None:
         out = torch.empty((B, L, h * dv), dtype=q.dtype, device=q.device)
     assert out.shape == (B, L, h * dv) and out.stride(2) == 1 and out.dtype == q.dtype
-    assert gate is None or (gate.shape == out.shape and gate.stride(2) == 1)
+    assert gate is None or (gate.stride(2) == 1 and (gate.shape[:2] == (B, L) and gate.shape[2] >= h if gate_heads else gate.shape == out.shape))
     win = None
-    if window or sink or rotary is not None or start_cap is not None:
+    if window or sink or gate_heads or rotary is not None or start_cap is not None:
         _need_gpu(rotary)
         win = _lib.VyAttnWindow(int(window), int(sink), 0, 2 ** 31 - 1 if start_cap is None else int(start_cap),
-                                *_rotary_args(rotary), int(keep))
+                                *_rotary_args(rotary), int(keep), int(gate_heads))
     call("vy_attn_fwd_ex", q.data_ptr(), q.stride(0), q.stride(1), q.stride(2), k.data_ptr(), k.stride(0), k.stride(1),
          k.stride(2), v.data_ptr(), v.stride(0), v.stride(1), v.stride(2), out.data_ptr(), out.stride(0), out.stride(1),
          _ptr(gate), gate.stride(0) if gate is not None else 0, gate.stride(1) if gate is not None else 0, _ptr(start),
@@ -815,7 +834,9 @@ class QkvPrep(NamedTuple):
     """What happens to packed queries, keys and values ahead of attention: RMS norms over the whole query and key projection
     (fp32 factors over the padded heads, zero in the padding; n_q / n_k true columns), and a share `mix` of the values
     `values` (rows of another layer's, whose heads have `values_dim` true columns) in the values, whose heads have n_v.
-    `keep_values`: receives the values before mixing."""
+    `keep_values`: receives the values before mixing.  group > 0: the norms go over every `group` padded columns by themselves
+    (n_q = n_k true ones), and the query of position p is multiplied by 1 + temp_coef ln(floor((p + 1) / temp_every) + 1)
+    (temp_every 0: no temperature); values stay as they are then."""
     q_norm: Optional[Tensor] = None
     k_norm: Optional[Tensor] = None
     n_q: int = 0
@@ -826,6 +847,17 @@ class QkvPrep(NamedTuple):
     values: Optional[Tensor] = None
     values_dim: int = 0
     keep_values: Optional[Tensor] = None
+    group: int = 0
+    temp_every: int = 0
+    temp_coef: float = 0.0
+
+
+def prep_struct(prep: QkvPrep) -> "_lib.VyQkvPrep":
+    """vy_qkv_prep of a QkvPrep; the rows of `values` and `keep_values` are filled in with their strides."""
+    v, k, d = prep.values, prep.keep_values, int(prep.values_dim)
+    return _lib.VyQkvPrep(_ptr(prep.q_norm), _ptr(prep.k_norm), int(prep.n_q), int(prep.n_k), float(prep.eps), float(prep.mix), _ptr(v),
+                          v.stride(0) if v is not None else 0, int(prep.n_v), d, up8(d), _ptr(k), k.stride(0) if k is not None else 0,
+                          int(prep.group), int(prep.temp_every), float(prep.temp_coef))
 
 
 def _prep_args(prep: Optional[QkvPrep], M: int, h: int, hk: int, dim: int, vdim: int, dtype: torch.dtype):
@@ -839,8 +871,7 @@ def _prep_args(prep: Optional[QkvPrep], M: int, h: int, hk: int, dim: int, vdim:
         assert t is None or (t.shape[0] == M and t.dtype == dtype and t.stride(1) == 1)
     assert k is None or k.shape[1] == hk * vdim
     assert v is None or v.shape[1] * prep.values_dim == hk * prep.n_v * up8(prep.values_dim)
-    return _lib.VyQkvPrep(_ptr(prep.q_norm), _ptr(prep.k_norm), int(prep.n_q), int(prep.n_k), float(prep.eps), float(prep.mix), _ptr(v),
-                          v.stride(0) if v is not None else 0, int(prep.n_v), int(prep.values_dim), up8(prep.values_dim), _ptr(k), k.stride(0) if k is not None else 0)
+    return prep_struct(prep)
 
 
 def qkv_rows(p: Tensor, B: int, L: int, h: int, hk: int, dim: int, vdim: int, oq: int, ok: int, ov: int, prep: QkvPrep, *,
@@ -872,9 +903,9 @@ def window_context(p: Tensor, B: int, L: int, hk: int, dim: int, vdim: int, ok: 
 
 def window_decode(p: Tensor, h: int, hk: int, dim: int, vdim: int, ring: Tensor, scale: float, start: Tensor, max_keys: int, *,
                   rotary: Optional[Tensor] = None, sink: bool = False, gate: bool = False, keep: int = 0,
-                  prep: Optional[QkvPrep] = None, slots: Optional[Tensor] = None) -> Tensor:
+                  prep: Optional[QkvPrep] = None, diff: Optional["_lib.VyDiff"] = None, slots: Optional[Tensor] = None) -> Tensor:
     """One token per sequence, packed rows p (B, [q | k | v | gate]): its key and value go to the ring, its queries attend
-    over it -> (B, h*vdim); prep: see qkv_rows.  (vy_window_decode)"""
+    over it -> (B, h*vdim); prep: see qkv_rows; diff: differential attention (dim: both maps' columns).  (vy_window_decode)"""
     _need_gpu(p, ring, slots, start, rotary)
     B = p.shape[0]
     _slot_args(slots, start, None, B)
@@ -882,12 +913,29 @@ def window_decode(p: Tensor, h: int, hk: int, dim: int, vdim: int, ring: Tensor,
     nk, gk, gv = h * dim, hk * dim, hk * vdim
     assert p.shape[1] >= nk + gk + gv + (h * vdim if gate else 0)
     out = torch.empty((B, h * vdim), dtype=p.dtype, device=p.device)
-    nws = _lib.load().vy_window_decode_ws_bytes(B, h, hk, vdim, ring.shape[2])
+    nws = _lib.load().vy_window_decode_ws_bytes(B, h, hk, vdim, ring.shape[2], int(diff is not None))
     ws = torch.empty(max(nws, 1), dtype=torch.uint8, device=p.device)
     call("vy_window_decode", p.data_ptr(), p.stride(0), 0, nk, nk + gk, nk + gk + gv if gate else -1,
          *_ring_args(ring, hk, dim, vdim), int(keep), *_rotary_args(rotary),
-         C.byref(_prep_args(prep, B, h, hk, dim, vdim, p.dtype)) if prep is not None else None, _ptr(slots), start.data_ptr(),
+         C.byref(_prep_args(prep, B, h, hk, dim, vdim, p.dtype)) if prep is not None else None,
+         C.byref(diff) if diff is not None else None, _ptr(slots), start.data_ptr(),
          int(max_keys), out.data_ptr(), out.stride(0), B, h, hk, dim, vdim, float(scale), int(sink), ws.data_ptr(), nws, dtype_code(p.dtype), _stream())
+    return out
+
+
+def diff_attention(q: Tensor, B: int, L: int, h: int, hk: int, dim: int, vdim: int, ring: Tensor, scale: float, diff: "_lib.VyDiff",
+                   start: Tensor, *, slots: Optional[Tensor] = None, count: Optional[Tensor] = None,
+                   out: Optional[Tensor] = None) -> Tensor:
+    """Causal differential attention of packed queries q (B*L, >= h*dim), heads [map 1 | map 2], over a ring (slots, hk, rows,
+    dim + vdim) that holds every token of the sequences, the new ones too, in order -> (B*L, h*vdim).  (vy_diff_attn_fwd)"""
+    _need_gpu(q, ring, start, slots, count)
+    _slot_args(slots, start, count, B)
+    assert q.shape[0] == B * L and q.shape[1] >= h * dim and q.stride(1) == 1 and ring.dtype == q.dtype
+    if out is None:
+        out = torch.empty((B * L, h * vdim), dtype=q.dtype, device=q.device)
+    assert out.shape == (B * L, h * vdim) and out.stride(1) == 1 and out.dtype == q.dtype
+    call("vy_diff_attn_fwd", q.data_ptr(), q.stride(0), *_ring_args(ring, hk, dim, vdim), C.byref(diff), _ptr(slots), start.data_ptr(),
+         _ptr(count), out.data_ptr(), out.stride(0), B, L, h, hk, dim, vdim, float(scale), dtype_code(q.dtype), _stream())
     return out
 
 
@@ -916,22 +964,24 @@ def moe(h: Tensor, desc: "_lib.VyMoe", L: int = 1, count: Optional[Tensor] = Non
 
 
 def latent_decode(q: Tensor, wukt: Tensor, wuv: Tensor, cache: Tensor, start: Tensor, max_keys: int, scale: float, *,
-                  slots: Optional[Tensor] = None, gate: Optional[Tensor] = None) -> Tensor:
+                  slots: Optional[Tensor] = None, gate: Optional[Tensor] = None, gate_heads: bool = False) -> Tensor:
     """One query token per sequence against a latent cache (slots, cap, R); q (B, h*dh), wukt (h, R, dh), wuv (h, dv, R);
-    keys 0 .. start[slot] are attended (the newest row is in the cache already).  (vy_latent_decode)"""
+    keys 0 .. start[slot] are attended (the newest row is in the cache already).  cache (slots, 1, rows, R): a ring, all of whose
+    tokens are seen.  gate_heads: gate (B, >= h) holds one number per head.  (vy_latent_decode)"""
     _need_gpu(q, wukt, wuv, cache, start, slots, gate)
     B = q.shape[0]
     h, R, dh = wukt.shape
     dv = wuv.shape[1]
     _slot_args(slots, start, None, B)
-    assert q.shape == (B, h * dh) and q.stride(1) == 1 and wuv.shape == (h, dv, R) and cache.shape[2] == R
-    assert wukt.is_contiguous() and wuv.is_contiguous() and cache.stride(2) == 1 and 0 < max_keys <= cache.shape[1]
+    assert q.shape == (B, h * dh) and q.stride(1) == 1 and wuv.shape == (h, dv, R) and cache.shape[-1] == R
+    r = cache.dim() - 2
+    assert wukt.is_contiguous() and wuv.is_contiguous() and cache.stride(-1) == 1 and 0 < max_keys and (r == 2 or max_keys <= cache.shape[1])
     out = torch.empty((B, h * dv), dtype=q.dtype, device=q.device)
     nws = _lib.load().vy_latent_decode_ws_bytes(B, h, R)
     ws = torch.empty(nws, dtype=torch.uint8, device=q.device)
     call("vy_latent_decode", q.data_ptr(), q.stride(0), wukt.data_ptr(), wuv.data_ptr(), cache.data_ptr(), cache.stride(0),
-         cache.stride(1), _ptr(slots), start.data_ptr(), int(max_keys), out.data_ptr(), out.stride(0), _ptr(gate),
-         gate.stride(0) if gate is not None else 0, B, h, dh, dv, R, float(scale), ws.data_ptr(), nws, dtype_code(q.dtype),
+         cache.stride(r), _ptr(slots), start.data_ptr(), int(max_keys), out.data_ptr(), out.stride(0), _ptr(gate),
+         gate.stride(0) if gate is not None else 0, int(gate_heads), cache.shape[2] if r == 2 else 0, B, h, dh, dv, R, float(scale), ws.data_ptr(), nws, dtype_code(q.dtype),
          _stream())
     return out
 
@@ -954,4 +1004,23 @@ def decay_attention(p: Tensor, heads: int, dk: int, dv: int, state: Tensor, deca
     call("vy_decay_attn", p.data_ptr(), p.stride(0), 0, heads * dk, 2 * heads * dk, state.data_ptr(), decay_pow.data_ptr(),
          _ptr(slots), start.data_ptr(), _ptr(count), out.data_ptr(), out.stride(0), B, L, heads, dk, dv, int(silu),
          *_rotary_args(rotary), float(k_scale), _ptr(ws), nws, dtype_code(p.dtype), _stream())
+    return out
+
+
+def gated_attention(p: Tensor, heads: int, dk: int, dv: int, state: Tensor, lower: Tensor, bias: Optional[Tensor], B: int, L: int, *,
+                    start: Tensor, slots: Optional[Tensor] = None, count: Optional[Tensor] = None, silu: bool = True) -> Tensor:
+    """Linear attention with a forget gate per key channel over packed rows p = [q (heads*dk) | gate logits (heads*dk) | v
+    (heads*dv) | ...] of B sequences of L tokens; lower and bias fp32 (heads*dk,); state as in decay_attention.  (vy_gated_attn)"""
+    _need_gpu(p, state, lower, bias, start, slots, count)
+    _slot_args(slots, start, count, B)
+    assert p.shape[0] == B * L and p.stride(1) == 1 and p.shape[1] >= heads * (2 * dk + dv)
+    assert state.dtype == torch.float32 and state.is_contiguous() and state.shape[1:] == (heads, dk, dv)
+    for t in (lower, bias):
+        assert t is None or (t.dtype == torch.float32 and t.numel() == heads * dk and t.is_contiguous())
+    out = torch.empty((B * L, heads * dv), dtype=p.dtype, device=p.device)
+    nws = _lib.load().vy_gated_attn_ws_bytes(B, L, heads, dk, dv, dtype_code(p.dtype))
+    ws = torch.empty(nws, dtype=torch.uint8, device=p.device) if nws else None
+    call("vy_gated_attn", p.data_ptr(), p.stride(0), 0, heads * dk, 2 * heads * dk, state.data_ptr(), _ptr(bias), lower.data_ptr(),
+         _ptr(slots), start.data_ptr(), _ptr(count), out.data_ptr(), out.stride(0), B, L, heads, dk, dv, int(silu), _ptr(ws), nws,
+         dtype_code(p.dtype), _stream())
     return out
