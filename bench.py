@@ -51,8 +51,8 @@ def parse():
     ap.add_argument("--no-cpu-baseline", action="store_true")
     ap.add_argument("--no-decode", action="store_true")
     ap.add_argument("--no-other-configs", action="store_true", help="skip the configs[3] / configs[4] side measurements")
-    ap.add_argument("--model", default="decoder", choices=["decoder", "gisitar", "rivudra", "padulorn"],
-                    help="gisitar / rivudra / padulorn: prefill / decode throughput of that design beside its closest other model at equal size (one "
+    ap.add_argument("--model", default="decoder", choices=["decoder", "gisitar", "rivudra", "padulorn", "biruvik"],
+                    help="gisitar / rivudra / padulorn / biruvik: prefill / decode throughput of that design beside its closest other model at equal size (one "
                          "GPU, serving only) instead of the headline workload")
     ap.add_argument("--backend", default="nccl", help="torch.distributed backend (nccl = RCCL; gloo for rehearsals)")
     ap.add_argument("--rehearse-launch", action="store_true",
@@ -395,7 +395,7 @@ def rehearse_launch(a) -> None:
 
 
 def bench_serving(a) -> None:
-    """--model gisitar / rivudra / padulorn: one JSON line with the throughputs of tools/bench_<model>.py."""
+    """--model gisitar / rivudra / padulorn / biruvik: one JSON line with the throughputs of tools/bench_<model>.py."""
     if a.gpus != 1:
         raise SystemExit(f"bench.py --model {a.model} measures one GPU")
     json_fd = os.dup(1)

@@ -82,9 +82,17 @@ def timed(fn, iters, warm=2):
     return s.elapsed_time(e) / iters
 
 
-@torch.no_grad()
 def measure_gisitar(width, cases):
+    H, _, kr, _ = SIZES[width]
     m = gisitar(width)
+    return measure_hybrid(m, width, cases, lambda B, ctx: B * sum(ctx * kr * 2 if l.mixer.kind == "latent" else 2 * H * DIM * DIM * 4
+                                                                  for l in m.layers))
+
+
+@torch.no_grad()
+def measure_hybrid(m, width, cases, cached):
+    """Throughputs of a hybrid decoder with dense feed-forwards; cached(B, context): bytes read and written per decode step besides
+    the weights."""
     out = {"parameters": sum(p.numel() for p in m.parameters())}
     for c in cases:
         if c in PREFILL:
@@ -107,9 +115,7 @@ def measure_gisitar(width, cases):
             cache.advance(slots, [ctx - n // 2] * B)          # a context of zeros: the kernels' work does not depend on it
             ids = torch.randint(0, VOCAB, (B,), device="cuda")
             ms = timed(lambda: m.decode(ids, cache, slots), n - 5)
-            H, _, kr, _ = SIZES[width]
-            cached = sum(ctx * kr * 2 if l.mixer.kind == "latent" else 2 * H * DIM * DIM * 4 for l in m.layers) * B
-            nbytes = sum(p.numel() for p in m.parameters()) * 2 - VOCAB * width * 2 + cached
+            nbytes = sum(p.numel() for p in m.parameters()) * 2 - VOCAB * width * 2 + cached(B, ctx)
             out[c] = {"batch": B, "context": ctx, "ms_per_step": round(ms, 4), "tokens_per_sec": round(B / ms * 1e3, 1),
                       "bytes_per_step": int(nbytes), "achieved_GBps": round(nbytes / ms * 1e-6, 1)}
         torch.cuda.empty_cache()
