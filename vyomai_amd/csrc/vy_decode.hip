@@ -780,7 +780,10 @@ template <int EPI, bool NORM>
 int dec_gemv1_go(const DecGemvArgs& a, hipStream_t st) {
   const dim3 grid((unsigned)(a.N / 4)), block(256);
   if (a.K == 2048) hipLaunchKernelGGL((dec_gemv1_kernel<EPI, 4, 1, NORM>), grid, block, 0, st, a);
+  else if (a.K == 1024) hipLaunchKernelGGL((dec_gemv1_kernel<EPI, 2, 1, NORM>), grid, block, 0, st, a);
   else if (a.K == 4096) hipLaunchKernelGGL((dec_gemv1_kernel<EPI, 8, 1, NORM>), grid, block, 0, st, a);
+  else if (a.K == 6144) hipLaunchKernelGGL((dec_gemv1_kernel<EPI, 4, 3, NORM>), grid, block, 0, st, a);
+  else if (a.K == 12288) hipLaunchKernelGGL((dec_gemv1_kernel<EPI, 8, 3, NORM>), grid, block, 0, st, a);
   else if (a.K == 8192) hipLaunchKernelGGL((dec_gemv1_kernel<EPI, 8, 2, NORM>), grid, block, 0, st, a);
   else if (a.K == 16384) hipLaunchKernelGGL((dec_gemv1_kernel<EPI, 8, 4, NORM>), grid, block, 0, st, a);
   else return 1;
@@ -904,7 +907,7 @@ extern "C" int vy_debug_set_decode_stamps(void* buf, int launches, int max_wg) {
 // ---- single-sequence (B = 1) products of the Gemma-style decode step; return VY_ERR_UNSUPPORTED (without an error
 // message being fatal: the driver falls back to the general kernels) for shapes the straight-line kernels do not cover
 static bool gemv1_ok(const void* x, const void* w, int N, int K) {
-  return N % 4 == 0 && (K == 2048 || K == 4096 || K == 8192 || K == 16384) && ((uintptr_t)x % 16 == 0) && ((uintptr_t)w % 16 == 0);
+  return N % 4 == 0 && (K == 1024 || K == 2048 || K == 4096 || K == 6144 || K == 8192 || K == 12288 || K == 16384) && ((uintptr_t)x % 16 == 0) && ((uintptr_t)w % 16 == 0);
 }
 int vy_dec_gemv1(const void* x, const void* w, const void* bias, const void* residual, void* y, int N, int K, int prescaled,
                  float eps, hipStream_t st) {

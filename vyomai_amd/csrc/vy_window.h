@@ -445,30 +445,41 @@ __device__ __forceinline__ void window_finish(const DecodeArgs& a, float* red, i
 }
 
 // one workgroup per (sequence, head): both maps' slices, their difference, the head's norm.  vdim <= 1024.
-constexpr int FINISH_DIFF_LDS = FINISH_LDS + 16;
+// A lane holds one slice's statistics (at most 64): one memory latency for all of them, and every partial row's factor is known
+// before the first is added.
+constexpr int FINISH_DIFF_LDS = FINISH_LDS + 16 + 2 * 64 * 4;
 __device__ __forceinline__ void window_finish_diff(const DecodeArgs& a, float* red, int head, int b) {
   const int tid = threadIdx.x;
   const int nc = a.vdim / 4, lanes = nc <= 64 ? 64 : nc <= 128 ? 128 : 256, groups = 256 / lanes;
   const int ch = tid % lanes, grp = tid / lanes;
+  float* sw = red + 1024 + 4;                // [map][slice]
+  const int64_t at = ((int64_t)b * a.h + head) * 2 * a.ns;
+  if (tid < 128) {
+    const int mp = tid >> 6, s = tid & 63;
+    const float2 ml = s < a.ns ? *reinterpret_cast<const float2*>(a.part_ml + (at + mp * a.ns + s) * 2) : make_float2(-FLT_MAX, 0.f);
+    const float e = __builtin_amdgcn_exp2f(ml.x - vy_wave_max(ml.x));
+    sw[mp * 64 + s] = e * (mp ? -a.lambda2 : 1.f) / vy_wave_sum(e * ml.y);
+  }
+  // the maps' slices as one list: 2 ns rows; the first batch is requested ahead of the factors
+  const float* po = a.part_o + at * a.vdim;
+  constexpr int UB = 8;
+  f32x4 x[UB];
+  auto fetch = [&](int k0) {
+#pragma unroll
+    for (int u = 0; u < UB; ++u) x[u] = *reinterpret_cast<const f32x4*>(po + (int64_t)min(k0 + u * groups, 2 * a.ns - 1) * a.vdim + (ch < nc ? ch : 0) * 4);
+  };
+  fetch(grp);
+  __syncthreads();
   f32x4 o = {0.f, 0.f, 0.f, 0.f};
+  for (int k0 = grp; k0 < 2 * a.ns; k0 += UB * groups) {
 #pragma unroll
-  for (int mp = 0; mp < 2; ++mp) {
-    const float* ml = a.part_ml + (((int64_t)b * a.h + head) * 2 + mp) * a.ns * 2;
-    const float* po = a.part_o + (((int64_t)b * a.h + head) * 2 + mp) * a.ns * a.vdim;
-    float m = -FLT_MAX, l = 0.f;
-    for (int s = 0; s < a.ns; ++s) m = fmaxf(m, ml[2 * s]);
-#pragma unroll 4
-    for (int s = 0; s < a.ns; ++s) l += ml[2 * s + 1] * __builtin_amdgcn_exp2f(ml[2 * s] - m);
-    const float w = (mp ? -a.lambda2 : 1.f) / l;
-    if (ch < nc) {
-#pragma unroll 4
-      for (int s = grp; s < a.ns; s += groups) {
-        const float f = __builtin_amdgcn_exp2f(ml[2 * s] - m) * w;
-        const f32x4 x = *reinterpret_cast<const f32x4*>(po + (int64_t)s * a.vdim + ch * 4);
+    for (int u = 0; u < UB; ++u) {
+      const int k = k0 + u * groups;
+      const float f = k < 2 * a.ns ? sw[k < a.ns ? k : 64 + k - a.ns] : 0.f;
 #pragma unroll
-        for (int e = 0; e < 4; ++e) o[e] = fmaf(f, x[e], o[e]);
-      }
+      for (int e = 0; e < 4; ++e) o[e] = fmaf(f, x[u][e], o[e]);
     }
+    if (k0 + UB * groups < 2 * a.ns) fetch(k0 + UB * groups);
   }
   *reinterpret_cast<f32x4*>(red + tid * 4) = o;
   __syncthreads();

@@ -244,7 +244,7 @@ __global__ __launch_bounds__(256) void group_rows_kernel(QkvArgs a, int group, i
 
 template <typename T>
 void group_rows_go(const QkvArgs& a, int group, int temp_every, float temp_coef, hipStream_t st) {
-  const int widest = a.r.store && a.r.vdim > group ? a.r.vdim : group, nch = widest / VyChunk<T>::VEC;
+  const int nch = group / VyChunk<T>::VEC;   // (wider values take more passes)
   const int64_t units = a.r.M * ((int64_t)(a.h + a.r.hk) * a.r.dim / group + (a.r.store ? a.r.hk : 0));
 #define GR_GO(LPG) hipLaunchKernelGGL((group_rows_kernel<T, LPG>), dim3((unsigned)vy_cdiv(units, 256 / LPG)), dim3(256), 0, st, a, group, temp_every, temp_coef)
   if (nch <= 4) GR_GO(4);
