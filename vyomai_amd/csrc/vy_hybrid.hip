@@ -17,6 +17,8 @@ int vy_parallel_decode(const vy_hybrid_plan* p, const vy_hybrid_layer* L, const 
                        int32_t* eids, float* ew, void* moe_ws, int64_t moe_ws_bytes, const int32_t* slots, const int32_t* lengths,
                        int64_t max_keys, void* mix_ws, int64_t mix_ws_bytes, void* stream);
 int vy_dec_gemv1_act(const void* x, const void* w, const void* bias, int act, float act_arg, void* y, int N, int K, hipStream_t st);
+int vy_rows_linear(const void* x, const void* w, const void* bias, int act, float act_arg, void* y, int64_t ldy, int64_t M, int64_t N,
+                   int64_t K, hipStream_t st);
 int vy_dec_gemv1_gated(const void* x, const void* wgu, void* y, int I, int K, int act, int prescaled, float eps, hipStream_t st);
 int vy_gemv_gated(const void* x, int64_t ldx, const void* w, int64_t ldw, const void* norm_w, float eps, void* y, int64_t ldy,
                   int64_t M, int64_t I, int64_t K, int act, void* stream);
@@ -64,6 +66,10 @@ int product(const vy_hybrid_plan* p, const void* x, const void* w, void* y, int6
     const int rc = vy_dec_gemv1_act(x, w, bias, act, cap, y, (int)N, (int)K, (hipStream_t)stream);
     if (rc != VY_ERR_UNSUPPORTED) return rc;
   }
+  if (p->dtype == VY_BF16) {
+    const int rc = vy_rows_linear(x, w, bias, act, cap, y, ldy, p->B, N, K, (hipStream_t)stream);
+    if (rc != VY_ERR_UNSUPPORTED) return rc;
+  }
   if (act == VY_ACT_SOFTCAP) return vy_linear_softcap_fwd(x, K, w, K, y, ldy, p->B, N, K, cap, p->dtype, stream);
   return vy_linear_fwd(x, K, w, K, bias, nullptr, 0, y, ldy, nullptr, p->B, N, K, act, p->dtype, stream);
 }
@@ -81,8 +87,7 @@ int gated(const vy_hybrid_plan* p, const vy_hybrid_layer& L, const void* x, void
   }
   if (!L.clamped && p->dtype == VY_BF16 && p->B <= 4)
     return vy_gemv_gated(x, p->dp, L.w_gu, p->dp, nullptr, 0.f, act, L.ff, p->B, L.ff, p->dp, p->act, stream);
-  const int rc = vy_linear_fwd(x, p->dp, L.w_gu, p->dp, nullptr, nullptr, 0, gu, 2 * (int64_t)L.ff, nullptr, p->B,
-                               2 * (int64_t)L.ff, p->dp, VY_ACT_NONE, p->dtype, stream);
+  const int rc = product(p, x, L.w_gu, gu, 2 * (int64_t)L.ff, 2 * (int64_t)L.ff, p->dp, stream);
   return rc ? rc : activation(p, L, gu, 2 * (int64_t)L.ff, act, L.ff, stream);
 }
 

@@ -70,25 +70,34 @@ struct Dense {
   const bf16* x; int64_t ldx; int M;   // M <= 16 MB
   const bf16* w; int N, K;             // [N][K]
   void* y; int64_t ldy; int f32;       // f32: fp32 results
+  const bf16* bias; int act; float act_arg;   // of bf16 results: act(x W^T + bias), act none, VY_ACT_RELU2 or VY_ACT_SOFTCAP
 };
 
-// rows 16 tile .. + 15 of W against all of X
-template <int MB>
+__device__ __forceinline__ float finish(const Dense& a, float v, int n) {
+  if (a.bias) v += (float)a.bias[n];
+  if (a.act == VY_ACT_RELU2) v = vy_act_fwd<VY_ACT_RELU2>(v);
+  else if (a.act == VY_ACT_SOFTCAP) v = vy_act_fwd<VY_ACT_SOFTCAP>(v, a.act_arg);
+  return v;
+}
+
+// rows 16 NT tile .. + 16 NT - 1 of W against all of X
+template <int MB, int NW = 4, int NT = 1>
 __device__ __forceinline__ void dense(const Dense& a, f32x4* red, int tile) {
   const int lane = threadIdx.x & 63, r16 = lane & 15, kq = lane >> 4;
-  const bf16* ws[1] = {a.w + (int64_t)min(16 * tile + r16, a.N - 1) * a.K + 8 * kq};
+  const bf16* ws[NT];
+#pragma unroll
+  for (int t = 0; t < NT; ++t) ws[t] = a.w + (int64_t)min(16 * (NT * tile + t) + r16, a.N - 1) * a.K + 8 * kq;
   const bf16* xs[MB];
 #pragma unroll
   for (int j = 0; j < MB; ++j) xs[j] = a.x + (int64_t)min(16 * j + r16, a.M - 1) * a.ldx + 8 * kq;
-  f32x4 acc[1][MB];
-  stream<1, MB>(ws, xs, a.K, acc, red);
+  f32x4 acc[NT][MB];
+  stream<NT, MB, true, NW>(ws, xs, a.K, acc, red);
   if (threadIdx.x >= 64) return;
-  const int n = 16 * tile + 4 * kq;
 #pragma unroll
-  for (int j = 0; j < MB; ++j) {
-    const int m = 16 * j + r16;
+  for (int i = 0; i < NT * MB; ++i) {
+    const int m = 16 * (i % MB) + r16, n = 16 * (NT * tile + i / MB) + 4 * kq;
     if (m >= a.M) continue;
-    const f32x4 v = acc[0][j];
+    const f32x4 v = acc[i / MB][i % MB];
     if (a.f32) {
 #pragma unroll
       for (int r = 0; r < 4; ++r)
@@ -96,12 +105,12 @@ __device__ __forceinline__ void dense(const Dense& a, f32x4* red, int tile) {
     } else if (n + 4 <= a.N) {
       bf16x4 w4;
 #pragma unroll
-      for (int r = 0; r < 4; ++r) w4[r] = (bf16)v[r];
+      for (int r = 0; r < 4; ++r) w4[r] = (bf16)finish(a, v[r], n + r);
       *reinterpret_cast<bf16x4*>((bf16*)a.y + (int64_t)m * a.ldy + n) = w4;
     } else {
 #pragma unroll
       for (int r = 0; r < 4; ++r)
-        if (n + r < a.N) ((bf16*)a.y)[(int64_t)m * a.ldy + n + r] = (bf16)v[r];
+        if (n + r < a.N) ((bf16*)a.y)[(int64_t)m * a.ldy + n + r] = (bf16)finish(a, v[r], n + r);
     }
   }
 }
