@@ -337,7 +337,7 @@ int vy_decay_attn(const void* p, int64_t ldp, int64_t oq, int64_t ok, int64_t ov
                   int64_t L, int32_t h, int32_t dk, int32_t dv, int silu, const float* rope, int32_t rope_dims, int32_t rope_len,
                   float k_scale, void* ws, int64_t ws_bytes, int dtype, void* stream);
 
-/* vy_gated_attn: linear attention with a forget gate per key channel that also decides what is written, on packed rows p (q, gate
+/* vy_gated_attn: linear attention with a forget gate f per key channel, tied to the input gate 1 - f, on packed rows p (q, gate
  * logits z and v of head a at columns oq + a*dk, of + a*dk, ov + a*dv):
  *   f = lower + (1 - lower) * sigmoid(z + bias),   S_t = diag(f_t) S_(t-1) + (1 - f_t) v_t^T,   o_t = S_t^T q_t
  * with q = silu of its projection (silu = 0: taken as it is); bias (nullable) and lower fp32 [h][dk] (lower 1 in padded channels).

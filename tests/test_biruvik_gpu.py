@@ -673,6 +673,21 @@ def test_decode_with_the_widths_of_the_straight_line_products():
     compare(run(m, ids, [6] + [1] * 6), O.forward(w, cfg, ids), torch.bfloat16)
 
 
+@pytest.mark.parametrize("batch", [6, 16, 17, 32])
+def test_decode_streams_wide_products(batch):
+    """bf16 batches whose products run in each of the weight-streaming forms: wide and narrow, long and short rows, odd ends."""
+    cfg = P.config([P.attention(2, 1, 16, 32, mlp=P.dense(8203)), P.hgrn2(2, 8, 16)], width=61, vocab=8301, cap=5.0)
+    cfg, w, m = make(cfg, torch.bfloat16)
+    seqs = [P.tokens(cfg, 6, seed=b) for b in range(batch)]
+    cache = m.new_cache(batch, 8)
+    slots = cache.allocate(batch)
+    m.prefill(torch.tensor([s[:4] for s in seqs], device="cuda"), [4] * batch, cache, slots)
+    for t in range(4, 6):
+        logits = m.decode(torch.tensor([s[t] for s in seqs], device="cuda"), cache, slots)
+    some = [0, 5, batch - 1]
+    compare(logits[some], torch.stack([O.forward(w, cfg, seqs[b])[-1] for b in some]), torch.bfloat16)
+
+
 # ---- the parts in other arrangements --------------------------------------------------------------
 @pytest.mark.parametrize("dt", DT)
 def test_parts_fit_other_layers(dt):

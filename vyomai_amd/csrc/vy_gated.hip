@@ -1,4 +1,4 @@
-// Linear attention with a forget gate per key channel that also decides what is written (HGRN2):
+// Linear attention with a forget gate per key channel, tied to the input gate 1 - f (HGRN2):
 //   f = lower + (1 - lower) sigmoid(z + bias),   S_t = diag(f_t) S_(t-1) + (1 - f_t) v_t^T ,   o_t = S_t^T q_t ,   q = silu
 //
 // Two forms, as in vy_lightning.hip: the recurrence (vy_decay.h) for decode steps, fp32 models and wide keys, and chunks of

@@ -1,4 +1,4 @@
-"""Gated linear attention whose forget gate also decides what is written (HGRN2),
+"""Gated linear attention with a forget gate per key channel, tied to the input gate 1 - f (HGRN2),
 
     f = lower + (1 - lower) sigmoid(W_f h + b) ,   S_t = diag(f_t) S_(t-1) + (1 - f_t) v_t^T ,   o_t = S_t^T q_t ,
 
